@@ -45,7 +45,7 @@ extern "C" {
 #define PA_F16 2
 #define PA_FP8_E4M3 3 /* OCP e4m3fn, KV pool only; q/out stay 16- or 32-bit */
 
-/* Library ABI version (bumped when an entry point is added or a signature or contract changes; now 6). */
+/* Library ABI version (bumped when an entry point is added or a signature or contract changes; now 7). */
 int pa_version(void);
 
 /* Text of the calling thread's most recent error; "" if none. */
@@ -381,6 +381,111 @@ int pa_rope_kv_append_e4m3(const void *q, void *q_out, const void *k_src, const 
 int pa_dequantize_blocks_e4m3(const void *cache, const float *scale, const int32_t *block_ids, int n_ids,
                               void *dst, int64_t num_blocks, int block_size, int num_kv_heads, int head_dim,
                               int dst_dtype, void *stream);
+
+/*
+ * ------------------------------------------------------------------ decoder blocks around attention
+ * The entry points below serve decoder blocks other than the reference's Llama block (none of them has a counterpart
+ * there): a 32-bit residual stream, layer norm or RMS norm, gated activations, short convolutions ahead of attention,
+ * and linear-attention layers with a carried state.  dtype is PA_F32 or PA_BF16, the type of activations and
+ * products; residual, norm weights, statistics, angles and states are float whatever the dtype.  A portion is a run of
+ * consecutive new rows of one sequence: rows [q_starts[b], q_starts[b] + q_lens[b]) at positions ctx_lens[b] -
+ * q_lens[b] ... ctx_lens[b] - 1.  With q_lens and q_starts NULL every sequence brings one row, row b (a decode
+ * step); a sequence with ctx_lens[b] = 0 is padding and is skipped.  A portion at position 0 starts from an empty
+ * state whatever its slot held before.
+ */
+#define PA_NORM_NONE 0
+#define PA_NORM_LAYER 1
+#define PA_NORM_RMS 2
+#define PA_ACT_SILU 0
+#define PA_ACT_GELU_TANH 1
+#define PA_V_PLAIN 0 /* values as they are */
+#define PA_V_FIRST 1 /* values as they are, also written to v_first */
+#define PA_V_MIX 2   /* (1 - lambda) value + lambda v_first */
+#define PA_QKV_TILE_ROWS 16 /* rows of a sequence's portion per tile of pa_qkv_conv_append */
+
+/*
+ * Residual sum and norm of one row at a time:
+ *     x = table[ids[row]]                           when ids is given, else x[row]
+ *     x += y                                        when y is given; with y_weight, y / rms(y) * y_weight
+ *     out = norm(x) * norm_weight + norm_bias       PA_NORM_LAYER or PA_NORM_RMS; PA_NORM_NONE: x in dtype
+ * where rms(v) = sqrt(mean(v^2) + eps) and the layer norm divides by sqrt(variance + eps) with the variance as the
+ * mean squared deviation.  x is written back when ids or y is given.  With row_index the call only reads: output
+ * row r comes from residual row row_index[r] (< x_rows).  Ids and indices out of range read as zero rows.
+ *   x : float[rows][width];  y, table, out : dtype;  weights and bias : float[width] or NULL;  width <= 16384
+ */
+int pa_residual_norm(float *x, const void *y, const float *y_weight, float y_eps, const int64_t *ids,
+                     const void *table, int64_t table_rows, const int64_t *row_index, int64_t x_rows,
+                     const float *norm_weight, const float *norm_bias, float eps, int norm, void *out,
+                     int64_t rows, int width, int dtype, void *stream);
+
+/* out = o / rms(o) * weight * sigmoid(gate), per row over its whole width; gate rows are gate_stride elements apart. */
+int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride, const float *weight, float eps, void *out,
+                int64_t rows, int width, int dtype, void *stream);
+
+/*
+ * out = act(gate) * up, rows of `width` elements at strides of their own.  With ids, row r's factor is row ids[r] of
+ * `up`, a table of up_rows rows (a per-token input); ids out of range give zeros.
+ */
+int pa_glu(const void *gate, int64_t gate_stride, const void *up, int64_t up_stride, const int64_t *ids,
+           int64_t up_rows, void *out, int64_t rows, int width, int act, int dtype, void *stream);
+
+/*
+ * out[row][h][0:vdim] = o[row][h][0:vdim] * sigmoid(gate[row][h]): the gate of each head behind attention, and the
+ * step from attention's padded rows (d) to packed ones (vdim).  gate NULL: the packing alone.
+ */
+int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, void *out, int64_t rows, int heads, int d,
+                 int vdim, int dtype, void *stream);
+
+/*
+ * From joint projections to attention's operands: row = [q heads | k heads | v heads | anything].
+ *   1. causal convolution over time per channel: y_t = sum_j w[j] u_(t - taps + 1 + j), the rows before a portion from
+ *      conv_state (the last taps - 1 projected rows of the sequence, updated by the call);
+ *   2. q, k: the pair (2i, 2i+1) of the first rot_dims dimensions turns by the angle whose (cos, sin) is
+ *      rope[position][i];
+ *   3. q, k: with unit_norm, divided by sqrt(mean over dim of the square + eps); q also times q_scale;
+ *   4. v: as v_mode says; v_lambda is one float on the device;
+ *   5. q to q_out, k and v to the pool at slots[row] (skipped when out of range), all in heads of pool_dim elements,
+ *      the rest of a head zeros.
+ *   conv_weight : float[taps][channels], channels = (Hq + Hkv) dim + Hkv vdim; taps <= 8 (1: no convolution)
+ *   conv_state  : [state_rows][taps - 1][channels] of dtype, sequence b's at state_slots[b] (negative: zeros, unsaved)
+ *   rope        : float[rope_rows][rot_dims / 2][2]
+ *   tiles       : int32[n_tiles][2] = (sequence, first row inside its portion), every portion covered in steps of
+ *                 PA_QKV_TILE_ROWS from row 0; NULL with n_tiles = batch: one row per sequence
+ *   v_first     : [n_rows][Hkv * vdim] of dtype
+ */
+int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_rows, const float *conv_weight, int taps,
+                       void *conv_state, int64_t state_rows, const float *rope, int64_t rope_rows, int rot_dims,
+                       const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
+                       const int32_t *state_slots, const int32_t *tiles, int n_tiles, int batch,
+                       const int64_t *slots, int64_t total_slots, void *q_out, void *k_cache, void *v_cache,
+                       void *v_first, const float *v_lambda, int v_mode, int num_q_heads, int num_kv_heads,
+                       int dim, int vdim, int pool_dim, int unit_norm, float eps, float q_scale, int dtype,
+                       void *stream);
+
+/*
+ * Lightning attention: per head S_t = decay S_(t-1) + k_t v_t^T and o_t = S_t^T q_t, with q, k and v the silu of a
+ * projection row [q heads | k heads | v heads | anything].
+ *   state        : float[state_rows][heads][pad16(dim)][pad16(vdim)], zero-filled once (pa_lightning_state_floats gives
+ *                  the floats per head); sequence b's at state_slots[b] (negative: starts empty, unsaved)
+ *   decay_powers : float[heads][65], the powers 0 .. 64 of each head's decay
+ *   out          : [n_rows][heads * vdim] of dtype
+ *   dim <= 256, any vdim
+ * pa_lightning_recurrent walks a portion token by token (decode steps; 32-bit prompts).  pa_lightning_chunked
+ * (PA_BF16) multiplies 64 rows at a time on the matrix cores, with the 32-bit factors split into two bf16 terms; given
+ * a workspace it cuts long portions of small batches into segments that run at the same time.  max_q_len: at least
+ * the longest portion.
+ */
+size_t pa_lightning_state_floats(int dim, int vdim);
+int pa_lightning_recurrent(const void *u, int64_t u_stride, int64_t n_rows, float *state, int64_t state_rows,
+                           const float *decay_powers, const int32_t *ctx_lens, const int32_t *q_lens,
+                           const int32_t *q_starts, const int32_t *state_slots, int batch, void *out,
+                           int num_heads, int dim, int vdim, int dtype, void *stream);
+size_t pa_lightning_workspace_bytes(int batch, int num_heads, int dim, int vdim, int max_q_len);
+int pa_lightning_chunked(const void *u, int64_t u_stride, int64_t n_rows, float *state, int64_t state_rows,
+                         const float *decay_powers, const int32_t *ctx_lens, const int32_t *q_lens,
+                         const int32_t *q_starts, const int32_t *state_slots, int batch, int max_q_len,
+                         void *out, int num_heads, int dim, int vdim, int dtype, void *workspace,
+                         size_t workspace_bytes, void *stream);
 
 #ifdef __cplusplus
 }

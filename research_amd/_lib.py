@@ -22,6 +22,10 @@ PA_ERR_WORKSPACE = -3
 PA_ERR_HIP = -4
 
 PA_F32, PA_BF16, PA_F16, PA_FP8_E4M3 = 0, 1, 2, 3
+PA_NORM_NONE, PA_NORM_LAYER, PA_NORM_RMS = 0, 1, 2
+PA_ACT_SILU, PA_ACT_GELU_TANH = 0, 1
+PA_V_PLAIN, PA_V_FIRST, PA_V_MIX = 0, 1, 2
+PA_QKV_TILE_ROWS = 16
 
 # name -> (restype, argtypes); mirrors include/paged_attn.h declaration by declaration
 SIGNATURES = {
@@ -82,6 +86,19 @@ SIGNATURES = {
          c_void_p],
     ),
 }
+_p, _i, _l, _f = c_void_p, c_int, c_int64, c_float
+SIGNATURES.update({
+    "pa_residual_norm": (_i, [_p, _p, _p, _f, _p, _p, _l, _p, _l, _p, _p, _f, _i, _p, _l, _i, _i, _p]),
+    "pa_rms_gate": (_i, [_p, _p, _l, _p, _f, _p, _l, _i, _i, _p]),
+    "pa_glu": (_i, [_p, _l, _p, _l, _p, _l, _p, _l, _i, _i, _i, _p]),
+    "pa_head_gate": (_i, [_p, _p, _l, _p, _l, _i, _i, _i, _i, _p]),
+    "pa_qkv_conv_append": (_i, [_p, _l, _l, _p, _i, _p, _l, _p, _l, _i, _p, _p, _p, _p, _p, _i, _i, _p, _l, _p, _p, _p,
+                                _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p]),
+    "pa_lightning_state_floats": (c_size_t, [_i, _i]),
+    "pa_lightning_recurrent": (_i, [_p, _l, _l, _p, _l, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _p]),
+    "pa_lightning_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i]),
+    "pa_lightning_chunked": (_i, [_p, _l, _l, _p, _l, _p, _p, _p, _p, _p, _i, _i, _p, _i, _i, _i, _i, _p, c_size_t, _p]),
+})
 SIGNATURES["pa_decode_split"] = SIGNATURES["pa_decode_reduce"] = SIGNATURES["pa_decode"]
 SIGNATURES["pa_prefill_paged_rowwise"] = SIGNATURES["pa_prefill_paged"]
 # pa_prefill_paged + total_q, workspace, workspace_bytes

@@ -1,0 +1,589 @@
+// Lightning attention: per head S_t = decay S_(t-1) + k_t v_t^T, o_t = S_t^T q_t, with q, k, v = silu(projections) and
+// S in 32-bit floats, kept per sequence in a pool of state slots.
+//
+// Two kernels.  The recurrent one (a decode step, and 32-bit prompts) reads the state once, walks its rows token by
+// token in registers and writes the state once: HBM-bound on the state for one token.  The chunked one (16-bit
+// prompts) multiplies 64 rows at a time on the matrix cores:
+//     O = diag(decay^(t+1)) Q S + ((Q K^T) * decay^(t-s), s <= t) V
+//     S = decay^64 S + K^T diag(decay^(63-s)) V
+// The 32-bit factors of these products (S, the decayed scores, the decayed values) enter the bf16 matrix cores as a
+// sum of two bf16 terms, which keeps 16 bits of their mantissa; q, k and v are bf16 to begin with.
+//
+// The state never leaves the registers of its wave between chunks: a wave owns a slice of the value columns, its
+// accumulator tile [16 d][16 v] of S is, in register order, the B operand of Q S when the operand Q is read with the
+// same order of d.
+#include "lightning_plan.h"
+#include "row_common.h"
+
+namespace {
+
+typedef __bf16 bf8 __attribute__((ext_vector_type(8)));
+typedef float f4 __attribute__((ext_vector_type(4)));
+
+struct LaArgs {
+    const void *u;  // [rows][ldu]: heads * dim of q, heads * dim of k, heads * vdim of v, anything
+    int64_t ldu, n_rows;
+    float *state;  // [state_rows][heads][pad16(dim)][pad16(vdim)]
+    int64_t state_rows;
+    const float *decay;  // [heads][kLaChunk + 1]: powers 0 .. 64 of a head's decay
+    const int32_t *ctx_lens, *q_lens, *q_starts, *state_slots;
+    void *out;  // [rows][heads * vdim]
+    float *ws;  // segment states
+    int heads, dim, vdim, dp, vp;
+    int segments, seg_rows;
+    int vec;  // 16-byte loads are possible
+};
+
+// The portion of sequence b: rows [row0, row0 + n), the first at position pos0.  False: nothing to do.
+struct Portion {
+    int n, pos0;
+    int64_t row0, slot;
+};
+__device__ __forceinline__ bool la_portion(const LaArgs &a, int b, Portion &p) {
+    p.n = a.q_lens ? a.q_lens[b] : 1;
+    p.row0 = a.q_starts ? a.q_starts[b] : b;
+    p.pos0 = a.ctx_lens[b] - p.n;
+    p.slot = a.state_slots[b];
+    if (p.slot >= a.state_rows) p.slot = -1;
+    return p.n > 0 && p.pos0 >= 0 && p.row0 >= 0 && p.row0 + p.n <= a.n_rows;
+}
+
+// ------------------------------------------------------------------ token by token
+constexpr int kRecCols = 64;  // value columns per workgroup: 16 lanes x float4, 16 groups of lanes over the rows of S
+
+// R: rows of S per thread (16 R >= dim)
+template <typename T, int R> __global__ __launch_bounds__(256) void lightning_recurrent_kernel(const LaArgs a) {
+    __shared__ float qs[16 * R], ks[16 * R], vs[kRecCols];
+    __shared__ float4 red[16][kRecCols / 4];
+    const int b = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kRecCols;
+    Portion p;
+    if (!la_portion(a, b, p)) return;
+    const int tid = threadIdx.x, col = tid % 16 * 4, grp = tid / 16;
+    const bool live = v0 + col < a.vp;  // (vp is a multiple of 16)
+    float *sp = p.slot >= 0 ? a.state + (p.slot * a.heads + h) * (int64_t)a.dp * a.vp + v0 + col : nullptr;
+    float4 s[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        const int d = grp + 16 * r;
+        s[r] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (sp && p.pos0 > 0 && live && d < a.dp) s[r] = *reinterpret_cast<const float4 *>(sp + (int64_t)d * a.vp);
+    }
+    const float lam = a.decay[h * (kLaChunk + 1) + 1];
+    const T *u = reinterpret_cast<const T *>(a.u);
+    for (int t = 0; t < p.n; ++t) {
+        const T *row = u + (p.row0 + t) * a.ldu;
+        for (int i = tid; i < 2 * 16 * R + kRecCols; i += 256) {
+            if (i < 16 * R) {
+                qs[i] = i < a.dim ? row_silu<T>(pa_scalar<T>::load(row + h * a.dim + i)) : 0.f;
+            } else if (i < 32 * R) {
+                const int d = i - 16 * R;
+                ks[d] = d < a.dim ? row_silu<T>(pa_scalar<T>::load(row + (a.heads + h) * a.dim + d)) : 0.f;
+            } else {
+                const int v = i - 32 * R;
+                vs[v] = v0 + v < a.vdim
+                            ? row_silu<T>(pa_scalar<T>::load(row + 2 * a.heads * a.dim + h * a.vdim + v0 + v)) : 0.f;
+            }
+        }
+        __syncthreads();
+        const float4 v = *reinterpret_cast<const float4 *>(vs + col);
+        float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const float k = ks[grp + 16 * r], q = qs[grp + 16 * r];
+            s[r].x = fmaf(lam, s[r].x, k * v.x); s[r].y = fmaf(lam, s[r].y, k * v.y);
+            s[r].z = fmaf(lam, s[r].z, k * v.z); s[r].w = fmaf(lam, s[r].w, k * v.w);
+            o.x = fmaf(q, s[r].x, o.x); o.y = fmaf(q, s[r].y, o.y);
+            o.z = fmaf(q, s[r].z, o.z); o.w = fmaf(q, s[r].w, o.w);
+        }
+        red[grp][tid % 16] = o;
+        __syncthreads();
+        if (tid < kRecCols && v0 + tid < a.vdim) {
+            float sum = 0.f;
+#pragma unroll
+            for (int g = 0; g < 16; ++g) sum += reinterpret_cast<const float *>(red[g])[tid];
+            pa_scalar<T>::store(reinterpret_cast<T *>(a.out) + (p.row0 + t) * ((int64_t)a.heads * a.vdim) + h * a.vdim + v0 + tid,
+                                sum);
+        }
+        // (the next token's writes to qs, ks, vs follow every thread's reads of them, before the barrier above; its
+        // writes to red come after its own barrier, which the threads that sum here reach afterwards)
+    }
+    if (!sp || !live) return;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        const int d = grp + 16 * r;
+        if (d < a.dp) *reinterpret_cast<float4 *>(sp + (int64_t)d * a.vp) = s[r];
+    }
+}
+
+// ------------------------------------------------------------------ chunks on the matrix cores
+// LDS layouts.  Row-major [64][KD + 8] for Q and K (the pad moves a row by 16 bytes over the banks).  Transposed
+// [rows][64 s] for K^T and V^T: eight 16-byte chunks per row, chunk c of row r at position c ^ la_hash(r), so that
+// both the transposing 8-byte writes (rows 4 apart) and the 16-byte operand reads (consecutive rows) spread over the
+// banks without a pad.
+__device__ __forceinline__ int la_hash(int r) { return (r + (r >> 2)) & 7; }
+__device__ __forceinline__ int la_tr(int r, int s) { return r * 64 + ((((s >> 3) ^ la_hash(r)) << 3) | (s & 7)); }
+
+__device__ __forceinline__ f4 la_mfma(bf8 x, bf8 y, f4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, c, 0, 0, 0); }
+
+__device__ __forceinline__ bf8 la_read8(const __bf16 *p) { return *reinterpret_cast<const bf8 *>(p); }
+__device__ __forceinline__ bf8 la_read44(const __bf16 *p, const __bf16 *q) {
+    typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+    const bf4 x = *reinterpret_cast<const bf4 *>(p), y = *reinterpret_cast<const bf4 *>(q);
+    return bf8{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+}
+// x = hi + lo, both bf16
+__device__ __forceinline__ void la_split(float x, __bf16 &hi, __bf16 &lo) {
+    hi = (__bf16)x;
+    lo = (__bf16)(x - (float)hi);
+}
+
+struct LaBlock {  // four rows of four consecutive columns, raw bf16
+    uint2 r[4];
+};
+
+// The 4 x 4 block at (row s, column c) of a tile that has `n` rows and `cols` columns; zeros elsewhere.
+__device__ __forceinline__ LaBlock la_load_block(const uint16_t *base, int64_t ld, int s, int c, int n, int cols, int vec) {
+    LaBlock b;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        b.r[i] = make_uint2(0u, 0u);
+        if (s + i < n && c < cols) {
+            const uint16_t *p = base + (int64_t)(s + i) * ld + c;
+            if (vec) {
+                b.r[i] = *reinterpret_cast<const uint2 *>(p);
+            } else {
+                uint32_t e[4];
+#pragma unroll
+                for (int j = 0; j < 4; ++j) e[j] = c + j < cols ? p[j] : 0u;
+                b.r[i] = make_uint2(e[0] | (e[1] << 16), e[2] | (e[3] << 16));
+            }
+        }
+    }
+    return b;
+}
+
+// silu of a raw pair, packed again
+__device__ __forceinline__ uint32_t la_silu2(uint32_t w) {
+    return row_pack_bf16(row_silu<pa_bf16>(__builtin_bit_cast(float, w << 16)),
+                         row_silu<pa_bf16>(__builtin_bit_cast(float, w & 0xffff0000u)));
+}
+
+// silu(block) to a row-major tile (when `rm` is given) and, transposed, to a [column][64] tile
+__device__ __forceinline__ void la_put_block(LaBlock b, int s, int c, __bf16 *rm, int ld_rm, __bf16 *tr) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) b.r[i] = make_uint2(la_silu2(b.r[i].x), la_silu2(b.r[i].y));
+    if (rm) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) *reinterpret_cast<uint2 *>(rm + (s + i) * ld_rm + c) = b.r[i];
+    }
+    if (!tr) return;
+    // columns 0/1 and 2/3 of rows 0..3 as pairs over rows (v_perm picks the low or the high halves)
+    const uint32_t lo01 = __builtin_amdgcn_perm(b.r[1].x, b.r[0].x, 0x05040100u), hi01 = __builtin_amdgcn_perm(b.r[1].x, b.r[0].x, 0x07060302u);
+    const uint32_t lo23 = __builtin_amdgcn_perm(b.r[3].x, b.r[2].x, 0x05040100u), hi23 = __builtin_amdgcn_perm(b.r[3].x, b.r[2].x, 0x07060302u);
+    const uint32_t lo01b = __builtin_amdgcn_perm(b.r[1].y, b.r[0].y, 0x05040100u), hi01b = __builtin_amdgcn_perm(b.r[1].y, b.r[0].y, 0x07060302u);
+    const uint32_t lo23b = __builtin_amdgcn_perm(b.r[3].y, b.r[2].y, 0x05040100u), hi23b = __builtin_amdgcn_perm(b.r[3].y, b.r[2].y, 0x07060302u);
+    *reinterpret_cast<uint2 *>(tr + la_tr(c, s)) = make_uint2(lo01, lo23);
+    *reinterpret_cast<uint2 *>(tr + la_tr(c + 1, s)) = make_uint2(hi01, hi23);
+    *reinterpret_cast<uint2 *>(tr + la_tr(c + 2, s)) = make_uint2(lo01b, lo23b);
+    *reinterpret_cast<uint2 *>(tr + la_tr(c + 3, s)) = make_uint2(hi01b, hi23b);
+}
+
+constexpr int kLaPitchA = 72;  // bf16 per row of the decayed scores
+
+template <int KD, int NV> constexpr int la_q_elems() {  // Q tile; later the output tile
+    return 64 * (KD + 8) > 64 * (64 * NV + 8) ? 64 * (KD + 8) : 64 * (64 * NV + 8);
+}
+template <int KD> constexpr int la_k_elems() {  // K tile; later the two terms of the decayed scores
+    return 64 * (KD + 8) > 2 * 64 * kLaPitchA ? 64 * (KD + 8) : 2 * 64 * kLaPitchA;
+}
+template <int KD, int NV> constexpr size_t la_lds_bytes() {
+    return (size_t)(la_q_elems<KD, NV>() + la_k_elems<KD>() + KD * 64 + 64 * NV * 64) * 2 + 80 * 4;
+}
+
+// KD: dim padded to 64, 128 or 256.  NV: 16-column tiles of the value slice per wave (the workgroup owns 64 NV columns).
+// STATES: only the segment's own contribution to the state, to the workspace (first pass over a portion in segments).
+template <int KD, int NV, bool STATES>
+__global__ __launch_bounds__(256) void lightning_chunk_kernel(const LaArgs a) {
+    constexpr int kCols = 64 * NV, kLdR = KD + 8, kLdO = kCols + 8;
+    constexpr int kKPass = KD / 64, kVPass = NV, kDB = KD / 4;  // 4x4 blocks: kDB per four rows of K
+    extern __shared__ __align__(16) char lds[];
+    __bf16 *q_s = reinterpret_cast<__bf16 *>(lds);
+    __bf16 *k_s = q_s + la_q_elems<KD, NV>();
+    __bf16 *kt_s = k_s + la_k_elems<KD>();
+    __bf16 *vt_s = kt_s + KD * 64;
+    float *pw = reinterpret_cast<float *>(vt_s + kCols * 64);
+    __bf16 *a_hi = k_s, *a_lo = k_s + 64 * kLaPitchA, *o_s = q_s;
+
+    const int h = blockIdx.x, seg = blockIdx.y % a.segments, vsl = blockIdx.y / a.segments, b = blockIdx.z;
+    Portion p;
+    if (!la_portion(a, b, p)) return;
+    const int r_beg = seg * a.seg_rows, r_end = r_beg + a.seg_rows < p.n ? r_beg + a.seg_rows : p.n;
+    if (r_beg >= p.n) return;
+    const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
+    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int v0 = vsl * kCols, vw = wave * 16 * NV;  // first column of the workgroup, of the wave inside it
+    if (tid <= kLaChunk) pw[tid] = a.decay[h * (kLaChunk + 1) + tid];
+
+    // The state slice of this wave: tile (dt, vt) holds d = 16 dt + 4 g + i, v = v0 + vw + 16 vt + l16
+    f4 s[KD / 16][NV];
+    const int64_t state_elems = (int64_t)a.dp * a.vp;
+    float *pool = p.slot >= 0 ? a.state + (p.slot * a.heads + h) * state_elems : nullptr;
+    float *seg_state = a.segments > 1 ? a.ws + (((int64_t)b * a.heads + h) * a.segments + seg) * state_elems : nullptr;
+    const float *from = STATES ? nullptr : (a.segments > 1 ? seg_state : (p.pos0 > 0 ? pool : nullptr));
+#pragma unroll
+    for (int dt = 0; dt < KD / 16; ++dt)
+#pragma unroll
+        for (int vt = 0; vt < NV; ++vt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int d = 16 * dt + 4 * g + i, v = v0 + vw + 16 * vt + l16;
+                s[dt][vt][i] = from && d < a.dp && v < a.vp ? from[(int64_t)d * a.vp + v] : 0.f;
+            }
+
+    const uint16_t *u = reinterpret_cast<const uint16_t *>(a.u) + p.row0 * a.ldu;
+    const uint16_t *uq = u + h * a.dim, *uk = u + (a.heads + h) * a.dim;
+    const uint16_t *uv = u + 2 * a.heads * a.dim + h * a.vdim + v0;
+    const int vcols = a.vdim - v0 < kCols ? a.vdim - v0 : kCols;
+    LaBlock kb[kKPass], vb[kVPass], qb[STATES ? 1 : kKPass];
+    auto fetch = [&](int r0) {
+#pragma unroll
+        for (int i = 0; i < kKPass; ++i) {
+            const int blk = tid + 256 * i, c = blk % kDB * 4, sr = blk / kDB * 4;
+            kb[i] = la_load_block(uk + (int64_t)r0 * a.ldu, a.ldu, sr, c, r_end - r0, a.dim, a.vec);
+            if (!STATES) qb[i] = la_load_block(uq + (int64_t)r0 * a.ldu, a.ldu, sr, c, r_end - r0, a.dim, a.vec);
+        }
+#pragma unroll
+        for (int i = 0; i < kVPass; ++i) {
+            const int blk = tid + 256 * i, c = blk % (kCols / 4) * 4, sr = blk / (kCols / 4) * 4;
+            vb[i] = la_load_block(uv + (int64_t)r0 * a.ldu, a.ldu, sr, c, r_end - r0, vcols, a.vec);
+        }
+    };
+    fetch(r_beg);
+    for (int r0 = r_beg; r0 < r_end; r0 += kLaChunk) {
+        const int nv = r_end - r0 < kLaChunk ? r_end - r0 : kLaChunk;
+#pragma unroll
+        for (int i = 0; i < kKPass; ++i) {
+            const int blk = tid + 256 * i, c = blk % kDB * 4, sr = blk / kDB * 4;
+            la_put_block(kb[i], sr, c, STATES ? nullptr : k_s, kLdR, kt_s);
+            if (!STATES) la_put_block(qb[i], sr, c, q_s, kLdR, nullptr);
+        }
+#pragma unroll
+        for (int i = 0; i < kVPass; ++i) {
+            const int blk = tid + 256 * i, c = blk % (kCols / 4) * 4, sr = blk / (kCols / 4) * 4;
+            la_put_block(vb[i], sr, c, nullptr, 0, vt_s);
+        }
+        if (r0 + kLaChunk < r_end) fetch(r0 + kLaChunk);
+        __syncthreads();
+
+        f4 o[4][NV];
+        if constexpr (!STATES) {
+            // scores of this wave's 16 rows against the columns up to them
+            f4 sc[4];
+#pragma unroll
+            for (int st = 0; st < 4; ++st) sc[st] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < KD / 32; ++kk) {
+                const bf8 aq = la_read8(q_s + (16 * wave + l16) * kLdR + 32 * kk + 8 * g);
+#pragma unroll
+                for (int st = 0; st < 4; ++st)
+                    if (st <= wave) sc[st] = la_mfma(aq, la_read8(k_s + (16 * st + l16) * kLdR + 32 * kk + 8 * g), sc[st]);
+            }
+            // the rows' part from before the chunk: Q S, then the decay of the way from the chunk's start
+#pragma unroll
+            for (int tt = 0; tt < 4; ++tt)
+#pragma unroll
+                for (int vt = 0; vt < NV; ++vt) o[tt][vt] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int dp = 0; dp < KD / 32; ++dp) {
+                bf8 hi[NV], lo[NV];
+#pragma unroll
+                for (int vt = 0; vt < NV; ++vt)
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) {
+                        __bf16 x, y;
+                        la_split(s[2 * dp + j / 4][vt][j % 4], x, y);
+                        hi[vt][j] = x;
+                        lo[vt][j] = y;
+                    }
+#pragma unroll
+                for (int tt = 0; tt < 4; ++tt) {
+                    const __bf16 *qr = q_s + (16 * tt + l16) * kLdR + 32 * dp + 4 * g;
+                    const bf8 aq = la_read44(qr, qr + 16);
+#pragma unroll
+                    for (int vt = 0; vt < NV; ++vt) {
+                        o[tt][vt] = la_mfma(aq, hi[vt], o[tt][vt]);
+                        o[tt][vt] = la_mfma(aq, lo[vt], o[tt][vt]);
+                    }
+                }
+            }
+#pragma unroll
+            for (int tt = 0; tt < 4; ++tt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float f = pw[16 * tt + 4 * g + i + 1];
+#pragma unroll
+                    for (int vt = 0; vt < NV; ++vt) o[tt][vt][i] *= f;
+                }
+            __syncthreads();  // Q and K have been read: their space takes the decayed scores (and, later, O)
+#pragma unroll
+            for (int st = 0; st < 4; ++st) {
+                if (st > wave + 1) continue;  // (tile wave + 1 is read as zeros when the last k-step covers it)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const int t = 16 * wave + 4 * g + i, c = 16 * st + l16;
+                    __bf16 x = (__bf16)0.f, y = (__bf16)0.f;
+                    if (c <= t) la_split(sc[st][i] * pw[t - c], x, y);
+                    a_hi[t * kLaPitchA + c] = x;
+                    a_lo[t * kLaPitchA + c] = y;
+                }
+            }
+            __syncthreads();
+#pragma unroll
+            for (int kk = 0; kk < 2; ++kk) {
+                bf8 bv[NV];
+#pragma unroll
+                for (int vt = 0; vt < NV; ++vt) bv[vt] = la_read8(vt_s + la_tr(vw + 16 * vt + l16, 32 * kk + 8 * g));
+#pragma unroll
+                for (int tt = 2 * kk; tt < 4; ++tt) {
+                    const bf8 ah = la_read8(a_hi + (16 * tt + l16) * kLaPitchA + 32 * kk + 8 * g);
+                    const bf8 al = la_read8(a_lo + (16 * tt + l16) * kLaPitchA + 32 * kk + 8 * g);
+#pragma unroll
+                    for (int vt = 0; vt < NV; ++vt) {
+                        o[tt][vt] = la_mfma(ah, bv[vt], o[tt][vt]);
+                        o[tt][vt] = la_mfma(al, bv[vt], o[tt][vt]);
+                    }
+                }
+            }
+        }
+        // S <- decay^nv S + K^T (decay^(nv-1-s) V)
+        const float whole = pw[nv];
+#pragma unroll
+        for (int dt = 0; dt < KD / 16; ++dt)
+#pragma unroll
+            for (int vt = 0; vt < NV; ++vt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) s[dt][vt][i] *= whole;
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            bf8 hi[NV], lo[NV];
+#pragma unroll
+            for (int vt = 0; vt < NV; ++vt) {
+                const bf8 bv = la_read8(vt_s + la_tr(vw + 16 * vt + l16, 32 * kk + 8 * g));
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    const int back = nv - 1 - (32 * kk + 8 * g + j);
+                    __bf16 x, y;
+                    la_split((float)bv[j] * pw[back < 0 ? 0 : back], x, y);  // (rows past the end hold zeros)
+                    hi[vt][j] = x;
+                    lo[vt][j] = y;
+                }
+            }
+#pragma unroll
+            for (int dt = 0; dt < KD / 16; ++dt) {
+                const bf8 ak = la_read8(kt_s + la_tr(16 * dt + l16, 32 * kk + 8 * g));
+#pragma unroll
+                for (int vt = 0; vt < NV; ++vt) {
+                    s[dt][vt] = la_mfma(ak, hi[vt], s[dt][vt]);
+                    s[dt][vt] = la_mfma(ak, lo[vt], s[dt][vt]);
+                }
+            }
+        }
+        if constexpr (!STATES) {
+            // O through LDS (where Q was), so that rows are stored 16 bytes per lane
+#pragma unroll
+            for (int tt = 0; tt < 4; ++tt)
+#pragma unroll
+                for (int vt = 0; vt < NV; ++vt)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i)
+                        o_s[(16 * tt + 4 * g + i) * kLdO + vw + 16 * vt + l16] = (__bf16)o[tt][vt][i];
+            __syncthreads();
+            uint16_t *dst = reinterpret_cast<uint16_t *>(a.out) + (p.row0 + r0) * ((int64_t)a.heads * a.vdim) + h * a.vdim + v0;
+            for (int i = tid; i < 64 * (kCols / 8); i += 256) {
+                const int t = i / (kCols / 8), c = i % (kCols / 8) * 8;
+                if (t >= nv || c >= vcols) continue;
+                const __bf16 *src = o_s + t * kLdO + c;
+                uint16_t *at = dst + (int64_t)t * ((int64_t)a.heads * a.vdim) + c;
+                if (a.vec) {
+                    *reinterpret_cast<uint4 *>(at) = *reinterpret_cast<const uint4 *>(src);
+                } else {
+                    for (int j = 0; j < 8 && c + j < vcols; ++j) at[j] = __builtin_bit_cast(uint16_t, src[j]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    float *to = STATES ? seg_state : (a.segments > 1 ? nullptr : pool);
+    if (!to) return;
+#pragma unroll
+    for (int dt = 0; dt < KD / 16; ++dt)
+#pragma unroll
+        for (int vt = 0; vt < NV; ++vt)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int d = 16 * dt + 4 * g + i, v = v0 + vw + 16 * vt + l16;
+                if (d < a.dp && v < a.vp) to[(int64_t)d * a.vp + v] = s[dt][vt][i];
+            }
+}
+
+// Segment contributions -> start states, in place; the state after the last segment goes back to the pool.
+__global__ __launch_bounds__(256) void lightning_scan_kernel(const LaArgs a) {
+    const int h = blockIdx.y, b = blockIdx.z;
+    Portion p;
+    if (!la_portion(a, b, p)) return;
+    const int64_t n4 = (int64_t)a.dp * a.vp / 4, i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n4) return;
+    float4 *pool = p.slot >= 0 ? reinterpret_cast<float4 *>(a.state) + (p.slot * a.heads + h) * n4 + i : nullptr;
+    float4 *seg = reinterpret_cast<float4 *>(a.ws) + ((int64_t)b * a.heads + h) * a.segments * n4 + i;
+    float4 cur = pool && p.pos0 > 0 ? *pool : make_float4(0.f, 0.f, 0.f, 0.f);
+    const float *pw = a.decay + h * (kLaChunk + 1);
+    float whole = 1.f;  // decay^seg_rows, seg_rows a multiple of the chunk
+    for (int c = 0; c < a.seg_rows / kLaChunk; ++c) whole *= pw[kLaChunk];
+    for (int j = 0; j * a.seg_rows < p.n; ++j) {
+        float f = whole;
+        const int left = p.n - j * a.seg_rows;
+        if (left < a.seg_rows) {
+            f = pw[left % kLaChunk];
+            for (int c = 0; c < left / kLaChunk; ++c) f *= pw[kLaChunk];
+        }
+        const float4 add = seg[j * n4];
+        seg[j * n4] = cur;
+        cur = make_float4(fmaf(f, cur.x, add.x), fmaf(f, cur.y, add.y), fmaf(f, cur.z, add.z), fmaf(f, cur.w, add.w));
+    }
+    if (pool) *pool = cur;
+}
+
+int la_cus() {
+    static int cached[64];
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return 256;
+    int n = __atomic_load_n(&cached[dev], __ATOMIC_RELAXED);
+    if (n == 0) {
+        if (hipDeviceGetAttribute(&n, hipDeviceAttributeMultiprocessorCount, dev) != hipSuccess || n <= 0) n = 256;
+        __atomic_store_n(&cached[dev], n, __ATOMIC_RELAXED);
+    }
+    return n;
+}
+
+template <typename K> int la_big_lds(K kernel, size_t bytes, const char *what) {
+    if (bytes > 64 * 1024) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(kernel),
+                                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+        if (e != hipSuccess) return pa_fail(PA_ERR_HIP, "%s: %s", what, hipGetErrorString(e));
+    }
+    return PA_OK;
+}
+
+template <int KD, int NV> int launch_chunks(const LaArgs &a, int batch, hipStream_t s) {
+    constexpr size_t lds = la_lds_bytes<KD, NV>();
+    static_assert(lds <= 160 * 1024, "LDS of one compute unit");
+    const int slices = (a.vdim + 64 * NV - 1) / (64 * NV);
+    const dim3 grid((unsigned)a.heads, (unsigned)(slices * a.segments), (unsigned)batch);
+    if (a.segments > 1) {
+        if (int rc = la_big_lds(lightning_chunk_kernel<KD, NV, true>, lds, "pa_lightning_chunked")) return rc;
+        lightning_chunk_kernel<KD, NV, true><<<grid, dim3(256), lds, s>>>(a);
+        const unsigned gx = (unsigned)(((int64_t)a.dp * a.vp / 4 + 255) / 256);
+        lightning_scan_kernel<<<dim3(gx, (unsigned)a.heads, (unsigned)batch), dim3(256), 0, s>>>(a);
+    }
+    if (int rc = la_big_lds(lightning_chunk_kernel<KD, NV, false>, lds, "pa_lightning_chunked")) return rc;
+    lightning_chunk_kernel<KD, NV, false><<<grid, dim3(256), lds, s>>>(a);
+    PA_CHECK_LAUNCH("pa_lightning_chunked");
+    return PA_OK;
+}
+
+template <typename T> void launch_recurrent(const LaArgs &a, int batch, hipStream_t s) {
+    const dim3 grid((unsigned)batch, (unsigned)a.heads, (unsigned)((a.vdim + kRecCols - 1) / kRecCols)), block(256);
+    if (a.dim <= 64) lightning_recurrent_kernel<T, 4><<<grid, block, 0, s>>>(a);
+    else if (a.dim <= 128) lightning_recurrent_kernel<T, 8><<<grid, block, 0, s>>>(a);
+    else lightning_recurrent_kernel<T, 16><<<grid, block, 0, s>>>(a);
+}
+
+int la_fill(const char *what, LaArgs &a, const void *u, int64_t u_stride, int64_t n_rows, float *state, int64_t state_rows,
+            const float *decay_powers, const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
+            const int32_t *state_slots, int batch, void *out, int num_heads, int dim, int vdim, int dtype) {
+    PA_REQUIRE(n_rows >= 0 && batch >= 0 && state_rows >= 0, "%s: a count is negative", what);
+    PA_REQUIRE(num_heads > 0 && dim > 0 && vdim > 0, "%s: heads / dim / vdim must be positive", what);
+    PA_REQUIRE(num_heads <= 65535 && batch <= 65535, "%s: heads=%d / batch=%d above 65535", what, num_heads, batch);
+    if (dtype != PA_F32 && dtype != PA_BF16) return pa_fail(PA_ERR_UNSUPPORTED, "%s: dtype=%d is not F32 or BF16", what, dtype);
+    if (dim > 256) return pa_fail(PA_ERR_UNSUPPORTED, "%s: dim=%d above 256", what, dim);
+    PA_REQUIRE(u_stride >= (int64_t)num_heads * (2 * dim + vdim), "%s: u_stride=%lld is shorter than q, k and v", what,
+               (long long)u_stride);
+    PA_REQUIRE((int64_t)num_heads * (2 * dim + vdim) <= 0x7fffffff, "%s: rows are too long", what);
+    PA_REQUIRE((q_lens == nullptr) == (q_starts == nullptr), "%s: q_lens and q_starts come together", what);
+    if (n_rows == 0 || batch == 0) return PA_OK;
+    PA_REQUIRE(u && state && decay_powers && ctx_lens && state_slots && out, "%s: NULL argument", what);
+    PA_REQUIRE(pa_aligned16(state), "%s: the state must be 16-byte aligned", what);
+    a = LaArgs{};
+    a.u = u; a.ldu = u_stride; a.n_rows = n_rows; a.state = state; a.state_rows = state_rows; a.decay = decay_powers;
+    a.ctx_lens = ctx_lens; a.q_lens = q_lens; a.q_starts = q_starts; a.state_slots = state_slots; a.out = out;
+    a.heads = num_heads; a.dim = dim; a.vdim = vdim; a.dp = la_pad16(dim); a.vp = la_pad16(vdim);
+    a.segments = 1;
+    a.vec = dim % 8 == 0 && vdim % 8 == 0 && u_stride % 8 == 0 && pa_aligned16(u) && pa_aligned16(out);
+    return PA_OK;
+}
+
+int la_plan(int64_t batch, int heads, int dim, int vdim, int max_q_len) {
+    const int cols = la_value_cols(dim, vdim);
+    return la_segments(batch * heads * ((vdim + cols - 1) / cols), la_cus(), max_q_len);
+}
+
+}  // namespace
+
+extern "C" size_t pa_lightning_state_floats(int dim, int vdim) {
+    return dim > 0 && vdim > 0 ? la_state_floats(dim, vdim) : 0;
+}
+
+extern "C" int pa_lightning_recurrent(const void *u, int64_t u_stride, int64_t n_rows, float *state, int64_t state_rows,
+                                      const float *decay_powers, const int32_t *ctx_lens, const int32_t *q_lens,
+                                      const int32_t *q_starts, const int32_t *state_slots, int batch, void *out,
+                                      int num_heads, int dim, int vdim, int dtype, void *stream) {
+    pa_clear_error();
+    LaArgs a;
+    if (int rc = la_fill("pa_lightning_recurrent", a, u, u_stride, n_rows, state, state_rows, decay_powers, ctx_lens, q_lens,
+                         q_starts, state_slots, batch, out, num_heads, dim, vdim, dtype))
+        return rc;
+    if (n_rows == 0 || batch == 0) return PA_OK;
+    PA_REQUIRE(q_lens || n_rows >= batch, "n_rows=%lld below batch=%d", (long long)n_rows, batch);
+    if (dtype == PA_F32) launch_recurrent<float>(a, batch, (hipStream_t)stream);
+    else launch_recurrent<pa_bf16>(a, batch, (hipStream_t)stream);
+    PA_CHECK_LAUNCH("pa_lightning_recurrent");
+    return PA_OK;
+}
+
+extern "C" size_t pa_lightning_workspace_bytes(int batch, int num_heads, int dim, int vdim, int max_q_len) {
+    pa_clear_error();
+    if (batch < 0 || num_heads <= 0 || dim <= 0 || vdim <= 0 || max_q_len < 0) {
+        pa_fail(PA_ERR_INVALID_ARG, "pa_lightning_workspace_bytes: sizes out of range");
+        return 0;
+    }
+    return la_workspace_bytes(batch, num_heads, dim, vdim, la_plan(batch, num_heads, dim, vdim, max_q_len));
+}
+
+extern "C" int pa_lightning_chunked(const void *u, int64_t u_stride, int64_t n_rows, float *state, int64_t state_rows,
+                                    const float *decay_powers, const int32_t *ctx_lens, const int32_t *q_lens,
+                                    const int32_t *q_starts, const int32_t *state_slots, int batch, int max_q_len,
+                                    void *out, int num_heads, int dim, int vdim, int dtype, void *workspace,
+                                    size_t workspace_bytes, void *stream) {
+    pa_clear_error();
+    LaArgs a;
+    PA_REQUIRE(max_q_len >= 0, "max_q_len=%d is negative", max_q_len);
+    if (dtype != PA_BF16)
+        return pa_fail(PA_ERR_UNSUPPORTED, "pa_lightning_chunked: dtype=%d is not BF16 (32-bit rows take pa_lightning_recurrent)",
+                       dtype);
+    if (int rc = la_fill("pa_lightning_chunked", a, u, u_stride, n_rows, state, state_rows, decay_powers, ctx_lens, q_lens,
+                         q_starts, state_slots, batch, out, num_heads, dim, vdim, dtype))
+        return rc;
+    if (n_rows == 0 || batch == 0 || max_q_len == 0) return PA_OK;
+    PA_REQUIRE(q_lens, "NULL q_lens / q_starts");
+    a.segments = la_plan(batch, num_heads, dim, vdim, max_q_len);
+    while (a.segments > 1 && (!workspace || la_workspace_bytes(batch, num_heads, dim, vdim, a.segments) > workspace_bytes))
+        --a.segments;
+    a.seg_rows = la_segment_rows(max_q_len, a.segments);
+    a.ws = (float *)workspace;
+    PA_REQUIRE(a.segments == 1 || pa_aligned16(workspace), "the workspace must be 16-byte aligned");
+    hipStream_t s = (hipStream_t)stream;
+    const bool wide = la_value_cols(dim, vdim) == 128;
+    if (dim <= 64) return wide ? launch_chunks<64, 2>(a, batch, s) : launch_chunks<64, 1>(a, batch, s);
+    if (dim <= 128) return wide ? launch_chunks<128, 2>(a, batch, s) : launch_chunks<128, 1>(a, batch, s);
+    return launch_chunks<256, 1>(a, batch, s);
+}

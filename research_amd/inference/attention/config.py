@@ -2,7 +2,8 @@
 
 Same fields, defaults, derived properties and hashing rule as the reference's
 ``CacheConfig`` (rollouts/rollouts/inference/attention/config.py:8-58), plus
-one optional field for the fp8-e4m3 pool layout this backend adds.
+optional fields: the fp8-e4m3 pool layout, layers of different shapes, and
+slots for per-sequence recurrent state.
 """
 
 from __future__ import annotations
@@ -11,6 +12,9 @@ from dataclasses import dataclass, fields
 from typing import Optional, Tuple
 
 import torch
+
+
+_EXTENSIONS = {"kv_format": None, "layer_kv": None, "num_state_slots": 0}
 
 
 @dataclass(frozen=True)
@@ -26,6 +30,15 @@ class CacheConfig:
     # Extension: "fp8_e4m3" keeps K/V as one byte per element with one fp32
     # scale per (block, kv head); ``dtype`` then names the q / output type.
     kv_format: Optional[str] = None
+    # Extension: one (kv heads, head size) per layer, None for a layer that keeps no keys; ``num_kv_heads`` and
+    # ``head_dim`` then only describe the layer the caller considers typical.
+    layer_kv: Optional[Tuple[Optional[Tuple[int, int]], ...]] = None
+    # Extension: sequences that can hold recurrent state at a time (0: the model keeps none).
+    num_state_slots: int = 0
+
+    def kv_shape(self, layer_idx: int) -> Optional[Tuple[int, int]]:
+        """(kv heads, head size) of a layer's pool, None when it has none."""
+        return (self.num_kv_heads, self.head_dim) if self.layer_kv is None else self.layer_kv[layer_idx]
 
     @property
     def total_slots(self) -> int:
@@ -39,13 +52,14 @@ class CacheConfig:
 
     def __hash__(self) -> int:
         # torch dtypes are hashed through their name, as the reference does
-        # (config.py:47-58); the extension field is appended only when set so
+        # (config.py:47-58); the extension fields are appended only when set so
         # that reference-shaped configs hash to the reference's value.
         key = tuple(
             str(getattr(self, f.name)) if f.name == "dtype" else getattr(self, f.name)
             for f in fields(self)
-            if f.name != "kv_format"
+            if f.name not in _EXTENSIONS
         )
-        if self.kv_format is not None:
-            key = key + (self.kv_format,)
+        for name, default in _EXTENSIONS.items():
+            if getattr(self, name) != default:
+                key = key + (getattr(self, name),)
         return hash(key)

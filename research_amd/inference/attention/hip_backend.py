@@ -46,7 +46,7 @@ Differences of ``HipPagedAttentionBackend`` from the reference, all deliberate:
 from __future__ import annotations
 
 from collections import OrderedDict
-from typing import List, Optional, Sequence, Tuple
+from typing import Dict, List, Optional, Sequence, Tuple
 
 import numpy as np
 import torch
@@ -64,7 +64,8 @@ class _StepTensors:
     """Device copies of one context's integer fields, built once per step."""
 
     __slots__ = ("ctx", "slots", "touched", "tables", "bt_stride", "seq_lens", "extra_zero", "ctx_lens", "q_lens",
-                 "q_starts", "max_q_len", "row_first_key", "fp8_blocks", "fp8_tables", "mask_words", "mask_keys")
+                 "q_starts", "max_q_len", "row_first_key", "fp8_blocks", "fp8_tables", "mask_words", "mask_keys",
+                 "packed")
 
     def __init__(self, ctx: InferenceContext) -> None:
         self.ctx = ctx  # keeps id(ctx) alive while the entry is cached
@@ -73,6 +74,7 @@ class _StepTensors:
         self.fp8_blocks = self.fp8_tables = None  # distinct blocks of the tables and the tables renumbered to them
         self.mask_words = None  # bits of an arbitrary mask predicate evaluated for this step, and their key count
         self.mask_keys = 0
+        self.packed = None
         self.bt_stride = self.max_q_len = 0
 
 
@@ -83,6 +85,24 @@ def _padded_tables(block_tables: Sequence[Sequence[int]]) -> np.ndarray:
         if len(row):
             out[i, : len(row)] = np.asarray(row, dtype=np.int64)
     return out
+
+
+class PackedStep:
+    """Device integers of a packed batch: the sequences that bring one token each come first (``decodes``), portions
+    of several tokens follow (``chunks``); ``rows`` describes both together."""
+
+    __slots__ = ("num_decodes", "num_rows", "slots", "tables", "rows", "decodes", "chunks")
+
+    def __init__(self, num_decodes: int, num_rows: int, slots: Optional[Tensor], tables: Tensor, rows: ops.Portions) -> None:
+        self.num_decodes, self.num_rows, self.slots, self.tables, self.rows = num_decodes, num_rows, slots, tables, rows
+        cut = lambda t, lo, hi: None if t is None else t[lo:hi]
+        batch, nd = rows.ctx_lens.numel(), num_decodes
+        self.decodes = self.chunks = None
+        if nd:
+            self.decodes = ops.Portions(rows.ctx_lens[:nd], cut(rows.state_slots, 0, nd))
+        if batch > nd:
+            self.chunks = ops.Portions(rows.ctx_lens[nd:], cut(rows.state_slots, nd, batch), rows.q_lens[nd:],
+                                       rows.q_starts[nd:], None, rows.max_q_len)
 
 
 class HipPagedAttentionBackend:
@@ -111,9 +131,20 @@ class HipPagedAttentionBackend:
             raise ValueError(f"unsupported cache dtype {config.dtype}")
         self._fp8 = config.kv_format == "fp8_e4m3"
         pool_dtype = torch.float8_e4m3fn if self._fp8 else config.dtype
-        # one allocation per tensor for all layers, zero-initialised (flex_backend.py:38-41)
-        self.k_cache = torch.zeros(config.cache_shape, dtype=pool_dtype, device=config.device)
-        self.v_cache = torch.zeros(config.cache_shape, dtype=pool_dtype, device=config.device)
+        self.state: Dict[Tuple[int, str], Tensor] = {}
+        if config.layer_kv is None:
+            # one allocation per tensor for all layers, zero-initialised (flex_backend.py:38-41)
+            self.k_cache = torch.zeros(config.cache_shape, dtype=pool_dtype, device=config.device)
+            self.v_cache = torch.zeros(config.cache_shape, dtype=pool_dtype, device=config.device)
+        else:  # layers of their own shapes: one tensor per layer that keeps keys
+            if self._fp8:
+                raise ValueError("an fp8 pool has one shape for all layers")
+            pool = lambda kv: None if kv is None else torch.zeros((config.total_slots,) + tuple(kv), dtype=pool_dtype,
+                                                                  device=config.device)
+            self.k_cache = [pool(kv) for kv in config.layer_kv]
+            self.v_cache = [pool(kv) for kv in config.layer_kv]
+        self._probe = torch.empty(0, device=config.device)
+        self._device = self._probe.device
         self.k_scale = self.v_scale = None
         if self._fp8:
             shape = (config.num_layers, config.num_blocks, config.num_kv_heads)
@@ -170,7 +201,7 @@ class HipPagedAttentionBackend:
         ``pa_attend_masked`` takes; computed once per context (all layers share it).  ``q_pos`` int ``[B, T]``:
         the q_idx of every row.  A predicate that does not look at ``h`` gives one row of bits for all heads."""
         if step.mask_words is None:
-            dev = self.k_cache.device
+            dev = self._device
             b = torch.arange(batch, device=dev)[:, None, None, None]
             h = torch.arange(heads, device=dev)[None, :, None, None]
             kv = torch.arange(n_keys, device=dev)[None, None, None, :]
@@ -211,9 +242,24 @@ class HipPagedAttentionBackend:
     def clear_mask_cache(self) -> None:
         self._mask_cache.clear()
 
+    def register_state(self, layer_idx: int, name: str, shape: Tuple[int, ...], dtype: torch.dtype) -> Tensor:
+        """A zero-filled tensor ``[num_state_slots, *shape]`` of per-sequence state, owned with the cache and
+        cleared with it.  The kernels start a sequence's first portion from an empty state whatever its slot holds."""
+        if self.config.num_state_slots <= 0:
+            raise ValueError("recurrent state needs CacheConfig.num_state_slots")
+        if (layer_idx, name) in self.state:
+            raise ValueError(f"state {name!r} of layer {layer_idx} is registered already")
+        self.state[layer_idx, name] = torch.zeros((self.config.num_state_slots,) + tuple(shape), dtype=dtype,
+                                                  device=self._device)
+        return self.state[layer_idx, name]
+
     def clear_cache(self) -> None:
-        self.k_cache.zero_()
-        self.v_cache.zero_()
+        for pool in (self.k_cache, self.v_cache):
+            for layer in [pool] if isinstance(pool, Tensor) else pool:
+                if layer is not None:
+                    layer.zero_()
+        for tensor in self.state.values():
+            tensor.zero_()
         if self._fp8:
             self.k_scale.fill_(1.0)
             self.v_scale.fill_(1.0)
@@ -233,6 +279,10 @@ class HipPagedAttentionBackend:
     __call__ = forward
 
     def _attend(self, q: Tensor, k: Tensor, v: Tensor, layer_idx: int, ctx: InferenceContext) -> Tensor:
+        if getattr(ctx, "q_lens", None) is not None:
+            rows = self.attend_packed(q.reshape(-1, q.shape[-2], q.shape[-1]).contiguous(), layer_idx,
+                                      self.packed_step(ctx), self.scale, self._window)
+            return rows.view(q.shape)
         if ctx.is_prefill:
             if getattr(ctx, "prefix_lens", None) is not None:  # absent on the reference's own context type
                 return self._prefill_paged(q, layer_idx, ctx)
@@ -253,7 +303,7 @@ class HipPagedAttentionBackend:
         cfg = self.config
         batch, seq_len, num_heads, head_dim = q.shape
         n = batch * seq_len
-        self._require_device(q, k, v, cos, sin, self.k_cache)
+        self._require_device(q, k, v, cos, sin)
         q3 = q.contiguous().view(n, num_heads, head_dim)
         k3 = k.reshape(n, cfg.num_kv_heads, head_dim).contiguous()
         v3 = v.reshape(n, cfg.num_kv_heads, head_dim).contiguous()
@@ -273,7 +323,8 @@ class HipPagedAttentionBackend:
         if ctx.slot_mapping is not None:
             step = self._step(ctx)
             slots = self._device_slots(ctx.slot_mapping, n, step)
-        dense = ctx.is_prefill and getattr(ctx, "prefix_lens", None) is None  # attends the step's own K/V
+        dense = (ctx.is_prefill and getattr(ctx, "prefix_lens", None) is None
+                 and getattr(ctx, "q_lens", None) is None)  # attends the step's own K/V
         kc, vc = self._layer(layer_idx)
         if self._fp8 and slots is not None:
             self._touched(step, slots, ctx, layer_idx)
@@ -317,7 +368,7 @@ class HipPagedAttentionBackend:
         return entry
 
     def _to_device(self, array: np.ndarray) -> Tensor:
-        return torch.from_numpy(array).to(self.k_cache.device)
+        return torch.from_numpy(array).to(self._device)
 
     def _tables(self, step: _StepTensors, block_tables) -> None:
         """Device copy of the block tables.  The reference's tuple-of-tuples costs a Python-level pass over every
@@ -333,7 +384,7 @@ class HipPagedAttentionBackend:
                         raise TypeError("a device-resident block_tables must be a contiguous int32 tensor")
                     step.tables = block_tables
                 else:
-                    step.tables = block_tables.to(device=self.k_cache.device, dtype=torch.int32).contiguous()
+                    step.tables = block_tables.to(device=self._device, dtype=torch.int32).contiguous()
             elif isinstance(block_tables, np.ndarray):
                 if block_tables.ndim != 2:
                     raise ValueError("block_tables array must be [num_seqs, width], padded with -1")
@@ -359,7 +410,7 @@ class HipPagedAttentionBackend:
                 self._retired_workspaces.append(self._workspace)
             # zero-filled: the arrival counters at the start of a workspace must read zero before its first use
             self._workspace = torch.zeros(max(nbytes, 2 * have, 1 << 20), dtype=torch.uint8,
-                                          device=self.k_cache.device)
+                                          device=self._device)
         return self._workspace
 
     def _layer(self, layer_idx: int) -> Tuple[Tensor, Tensor]:
@@ -377,7 +428,7 @@ class HipPagedAttentionBackend:
             return step.slots
         if isinstance(slot_mapping, Tensor) and slot_mapping.device.type == "cuda":
             # already on the device: used as it is (out-of-range slots are dropped by the kernel, not reported)
-            self._require_device(*tensors, self.k_cache)
+            self._require_device(*tensors, self._probe)
             if slot_mapping.dtype != torch.int64 or not slot_mapping.is_contiguous():
                 raise TypeError("a device-resident slot_mapping must be a contiguous int64 tensor")
             slots = slot_mapping
@@ -388,7 +439,7 @@ class HipPagedAttentionBackend:
             if host.size and host.max() >= cfg.total_slots:
                 raise IndexError(
                     f"index {int(host.max())} is out of bounds for dimension 0 with size {cfg.total_slots}")
-            self._require_device(*tensors, self.k_cache)
+            self._require_device(*tensors, self._probe)
             slots = self._to_device(host)
         if step is not None:
             step.slots = slots
@@ -460,7 +511,7 @@ class HipPagedAttentionBackend:
         """Zero-padded ``[num_seqs, max(seq_lens), Hkv, D]`` copies (flex_backend.py:233-279)."""
         cfg = self.config
         num_seqs, max_len = len(block_tables), max(seq_lens)
-        self._require_device(self.k_cache)
+        self._require_device(self._probe)
         tables = self._to_device(_padded_tables(block_tables))
         lens = self._to_device(np.asarray(seq_lens, dtype=np.int32)[:num_seqs])
         kc, vc = self._layer(layer_idx)
@@ -640,6 +691,77 @@ class HipPagedAttentionBackend:
         ops.prefill_paged(q3, kc, vc, tables, step.ctx_lens, step.q_lens, step.q_starts, step.max_q_len,
                           cfg.block_size, self.scale, out=out.view(batch * seq_len, num_heads, head_dim), window=window,
                           row_first_key=first, workspace=self._workspace_for(need) if need else None)
+        return out
+
+    # ------------------------------------------------------------------ packed batches
+    def packed_step(self, ctx: InferenceContext) -> PackedStep:
+        """The device side of a packed context (``q_lens`` set), or of a decode step of models that run packed rows;
+        built once per context.  The integers of a host context travel in one copy."""
+        step = self._step(ctx)
+        if step.packed is not None:
+            return step.packed
+        cfg = self.config
+        if isinstance(ctx.seq_lens, Tensor) and ctx.seq_lens.device.type == "cuda":
+            # a decode step whose fields live on the device and are rewritten in place between graph replays
+            if ctx.is_prefill or ctx.q_lens is not None:
+                raise TypeError("device-resident packed contexts are decode steps")
+            self._tables(step, ctx.block_tables)
+            n = ctx.seq_lens.numel()
+            slots = self._device_slots(ctx.slot_mapping, n, step) if ctx.slot_mapping is not None else None
+            step.packed = PackedStep(n, n, slots, step.tables, ops.Portions(ctx.seq_lens, ctx.state_slots))
+            return step.packed
+        lens = np.asarray(ctx.seq_lens, dtype=np.int64)
+        batch = len(lens)
+        q_lens = np.ones(batch, dtype=np.int64) if ctx.q_lens is None else np.asarray(ctx.q_lens, dtype=np.int64)
+        nd = batch if ctx.q_lens is None else int(ctx.num_decodes)
+        if len(q_lens) != batch or (q_lens < 1).any() or (q_lens > lens).any() or (q_lens[:nd] != 1).any():
+            raise ValueError("q_lens / num_decodes do not describe portions of the sequences")
+        rows = int(q_lens.sum())
+        starts = np.cumsum(q_lens) - q_lens
+        state = np.full(batch, -1) if ctx.state_slots is None else np.asarray(ctx.state_slots)
+        if cfg.num_state_slots and (state >= cfg.num_state_slots).any():
+            raise IndexError("a state slot past the pool")
+        ints = [lens, state]
+        tile_rows = None
+        if nd < batch:
+            per_seq = -(-q_lens // ops.QKV_TILE_ROWS)
+            seq = np.repeat(np.arange(batch), per_seq)
+            first = (np.arange(len(seq)) - np.repeat(np.cumsum(per_seq) - per_seq, per_seq)) * ops.QKV_TILE_ROWS
+            tile_rows = np.stack([seq, first], axis=1)
+            ints += [q_lens, starts, tile_rows.reshape(-1)]
+        dev = self._to_device(np.concatenate(ints).astype(np.int32))
+        parts = torch.split(dev, [len(a) for a in ints])
+        portions = ops.Portions(parts[0], parts[1])
+        if nd < batch:
+            portions = ops.Portions(parts[0], parts[1], parts[2], parts[3], parts[4].view(-1, 2), int(q_lens.max()))
+        self._tables(step, ctx.block_tables)
+        slots = None
+        if ctx.slot_mapping is not None:
+            slots = self._device_slots(ctx.slot_mapping, rows, step)
+        step.packed = PackedStep(nd, rows, slots, step.tables, portions)
+        return step.packed
+
+    def attend_packed(self, q: Tensor, layer_idx: int, step: PackedStep, scale: float, window: int) -> Tensor:
+        """Attention of packed rows ``q [rows, Hq, D]`` over the pool (their own keys appended already): the decode
+        kernel for the sequences that bring one token, the prefill kernels for the portions."""
+        if self._fp8:
+            raise NotImplementedError("packed batches run on 16- and 32-bit pools")
+        cfg = self.config
+        self._require_device(q)
+        kc, vc = self._layer(layer_idx)
+        heads, d = q.shape[1], q.shape[2]
+        nd = step.num_decodes
+        out = torch.empty_like(q)
+        if nd:
+            ws = self._workspace_for(ops.decode_workspace_bytes(nd, heads, kc.shape[1], d, kc.dtype))
+            ops.decode(q[:nd], kc, vc, step.tables[:nd], step.decodes.ctx_lens, cfg.block_size, scale, ws, window=window,
+                       out=out[:nd])
+        c = step.chunks
+        if c is not None:
+            tables = step.tables[nd:]
+            need = ops.prefill_workspace_bytes(q, tables, c.max_q_len, cfg.block_size, kc.shape[1], window)
+            ops.prefill_paged(q, kc, vc, tables, c.ctx_lens, c.q_lens, c.q_starts, c.max_q_len, cfg.block_size, scale,
+                              out=out, window=window, workspace=self._workspace_for(need) if need else None)
         return out
 
     # ------------------------------------------------------------------ fp8 pool

@@ -19,6 +19,12 @@ scheduler a made-up block count (engine.py:147) and ``flush_cache`` is empty
   to the head of the waiting queue to be prefilled again later.
 * ``cache_type="none"`` keeps the reference's behaviour of recomputing the
   whole sequence every step (dense causal prefill, nothing stored).
+* Models that run packed rows (``model.packed``) get one batch per step: the
+  decodes and the portions of prompts that the schedule admits, in one forward
+  pass (``forward_portions``).  Models with recurrent state keep it in slots that
+  the allocator hands out with the blocks (``cache/private.py``).
+* ``open_sequence`` / ``feed`` / ``close_sequence`` run given tokens through the
+  same step function without sampling (bin/trace_run).
 """
 
 from __future__ import annotations
@@ -29,11 +35,11 @@ import numpy as np
 import torch
 from torch import nn
 
-from .attention import CacheConfig, HipPagedAttentionBackend
-from .cache import CountingPagedKVCache, RadixKVCache
-from .model import ModelConfig, PagedLlama, default_num_kv_blocks
+from .cache import CountingPagedKVCache, PrivateKVCache, RadixKVCache
+from .model import PagedLlama, default_num_kv_blocks
+from .registry import DTYPES, LoadOptions, load_model
 from .sampling import sample_with_logprobs
-from .scheduler import schedule
+from .scheduler import schedule, step_tokens
 from .types import (EngineConfig, InferenceContext, SamplingParams, SchedulerConfig, Sequence, SequenceStatus,
                     TrainingSample)
 
@@ -65,14 +71,16 @@ class _DecodeGraph:
         self.slots = torch.full((batch,), -1, dtype=torch.int64, device=device)
         self.tables = torch.full((batch, table_width), -1, dtype=torch.int32, device=device)
         self.lens = torch.zeros((batch,), dtype=torch.int32, device=device)
+        self.state_slots = torch.full((batch,), -1, dtype=torch.int32, device=device)
         self.ctx = InferenceContext(is_prefill=False, slot_mapping=self.slots, block_tables=self.tables,
-                                    seq_lens=self.lens, max_seq_len=table_width)
+                                    seq_lens=self.lens, max_seq_len=table_width, state_slots=self.state_slots)
         # host staging, one copy per field and step
         self._h_ids = np.zeros((batch, 1), dtype=np.int64)
         self._h_pos = np.zeros((batch, 1), dtype=np.int64)
         self._h_slots = np.full((batch,), -1, dtype=np.int64)
         self._h_tables = np.full((batch, table_width), -1, dtype=np.int32)
         self._h_lens = np.zeros((batch,), dtype=np.int32)
+        self._h_state = np.full((batch,), -1, dtype=np.int32)
         # one eager pass on a side stream first (workspaces, rotary tables and library handles come into being
         # outside the capture); all rows are padding, so it writes nothing to the pool
         side = torch.cuda.Stream(device=device)
@@ -86,7 +94,7 @@ class _DecodeGraph:
             self.hidden = model(self.ids, self.pos, self.ctx)
 
     def run(self, ids: np.ndarray, last_pos: np.ndarray, slots: np.ndarray, tables: np.ndarray,
-            lens: np.ndarray) -> torch.Tensor:
+            lens: np.ndarray, state_slots: Optional[np.ndarray] = None) -> torch.Tensor:
         n = len(ids)
         if tables.shape[1] > self.width:
             raise ValueError(f"a block table of {tables.shape[1]} entries exceeds max_model_len / block_size = {self.width}")
@@ -100,8 +108,13 @@ class _DecodeGraph:
         self._h_tables[:n, : tables.shape[1]] = tables
         self._h_lens[:n] = lens
         self._h_lens[n:] = 0
-        for dst, src in ((self.ids, self._h_ids), (self.pos, self._h_pos), (self.slots, self._h_slots),
-                         (self.tables, self._h_tables), (self.lens, self._h_lens)):
+        fields = [(self.ids, self._h_ids), (self.pos, self._h_pos), (self.slots, self._h_slots),
+                  (self.tables, self._h_tables), (self.lens, self._h_lens)]
+        if state_slots is not None:
+            self._h_state[:n] = state_slots
+            self._h_state[n:] = -1
+            fields.append((self.state_slots, self._h_state))
+        for dst, src in fields:
             dst.copy_(torch.from_numpy(src))
         self.graph.replay()
         return self.hidden
@@ -111,7 +124,7 @@ class InferenceEngine:
     def __init__(self, config: EngineConfig, model: Optional[PagedLlama] = None, tokenizer=None) -> None:
         assert config.block_size > 0
         assert config.max_batch_size > 0
-        if config.cache_type not in ("paged", "radix", "none"):
+        if config.cache_type not in ("paged", "radix", "private", "none"):
             raise ValueError(f"unknown cache_type {config.cache_type!r}")
         self.config = config
         if not torch.cuda.is_available():
@@ -121,17 +134,23 @@ class InferenceEngine:
             config.max_batch_size, config.max_model_len, config.block_size)
         self.model = model if model is not None else self._load_model(config.model_path)
         self.backend = self.model.backend
+        self.packed = bool(getattr(self.model, "packed", False))
         limit = getattr(getattr(self.model, "cfg", None), "max_position_embeddings", None)
+        if limit is None:
+            limit = getattr(self.model, "max_positions", None)
         if limit is not None and config.max_model_len > limit:
             # the rotary tables end at max_position_embeddings; later positions would all take the last row
             raise ValueError(f"max_model_len={config.max_model_len} exceeds the model's "
-                             f"max_position_embeddings={limit}")
+                             f"{limit} positions")
         self.tokenizer = tokenizer if tokenizer is not None else self._load_tokenizer(config.model_path)
-        self.scheduler_config = SchedulerConfig(
-            max_batch_size=config.max_batch_size,
-            max_tokens_per_batch=config.max_batch_size * 512,  # as the reference (engine.py:50)
-            block_size=config.block_size,
-        )
+        budget = config.max_batch_size * 512  # as the reference (engine.py:50)
+        portion = 0
+        if self.packed:
+            portion = min(config.prefill_portion or max(1, budget // 2), budget)
+        elif config.prefill_portion:
+            raise ValueError("prefill_portion needs a model that runs packed batches")
+        self.scheduler_config = SchedulerConfig(max_batch_size=config.max_batch_size, max_tokens_per_batch=budget,
+                                                block_size=config.block_size, prefill_portion=portion)
         self.cache = self._new_cache()
         self.waiting: List[Sequence] = []
         self.running: List[Sequence] = []
@@ -142,13 +161,12 @@ class InferenceEngine:
 
     # ------------------------------------------------------------------ construction
     def _load_model(self, model_path: str) -> nn.Module:
-        """A local HuggingFace checkpoint directory of the Llama / Qwen2 family (nothing is downloaded)."""
-        def backend_for(cfg: ModelConfig):
-            return HipPagedAttentionBackend(CacheConfig(
-                num_layers=cfg.num_layers, num_kv_heads=cfg.num_kv_heads, head_dim=cfg.head_dim,
-                num_blocks=self.num_kv_blocks, block_size=self.config.block_size, device="cuda",
-                dtype=torch.bfloat16))
-        return PagedLlama.from_local(model_path, backend_for, dtype=torch.bfloat16, device="cuda")
+        """A local checkpoint directory of a registered design (nothing is downloaded)."""
+        if self.config.dtype not in DTYPES:
+            raise ValueError(f"unknown dtype {self.config.dtype!r}")
+        return load_model(model_path, LoadOptions(
+            num_blocks=self.num_kv_blocks, block_size=self.config.block_size, num_state_slots=self.config.max_batch_size,
+            max_positions=self.config.max_model_len, dtype=DTYPES[self.config.dtype]))
 
     @staticmethod
     def _load_tokenizer(model_path: str):
@@ -159,11 +177,14 @@ class InferenceEngine:
             return None
 
     def _new_cache(self):
-        if self.config.cache_type == "none":
+        recurrent = bool(getattr(getattr(self, "model", None), "recurrent", False))
+        if self.config.cache_type == "none" and not recurrent:
             return None
         if self.backend.config.block_size != self.config.block_size:
             raise ValueError("EngineConfig.block_size differs from the backend's CacheConfig.block_size")
         blocks = self.backend.config.num_blocks
+        if recurrent or self.config.cache_type == "private":
+            return PrivateKVCache(blocks, self.config.block_size, getattr(self.backend.config, "num_state_slots", 0))
         cls = RadixKVCache if self.config.cache_type == "radix" else CountingPagedKVCache
         return cls(blocks, self.config.block_size)
 
@@ -212,9 +233,7 @@ class InferenceEngine:
         if self.cache is not None:
             # Decodes run before the prefills of the same step and take a block for every sequence whose new
             # token starts one: those blocks are not there for the prompts admitted below.
-            bs = self.config.block_size
-            growth = sum(1 for s in self.running[: self.scheduler_config.max_batch_size]
-                         if (len(s.token_ids) - 1) % bs == 0)
+            growth = sum(1 for s in self.running[: self.scheduler_config.max_batch_size] if self._grows(s))
             free = max(0, self.cache.num_free_blocks() - growth)
         out = schedule(self.waiting, self.running, free, self.scheduler_config)
         if self.cache is not None and not out.prefill_seqs and not out.decode_seqs and self.waiting:
@@ -233,6 +252,8 @@ class InferenceEngine:
         with torch.no_grad():
             if self.cache is None:
                 finished += self._recompute(prefill_seqs + decode_seqs)
+            elif getattr(self, "packed", False):
+                finished += self._packed_step(self._make_room(decode_seqs), prefill_seqs)
             else:
                 if decode_seqs:
                     finished += self._decode(self._make_room(decode_seqs))
@@ -260,6 +281,7 @@ class InferenceEngine:
         for seq in reversed(self.running):
             seq.status = SequenceStatus.WAITING
             seq.block_ids = []
+            seq.num_computed = 0
             self.waiting.insert(0, seq)
         self.running = []
         self.backend.clear_cache()
@@ -272,12 +294,19 @@ class InferenceEngine:
         self.cache = self._new_cache()
 
     # ------------------------------------------------------------------ forward passes
+    def _grows(self, seq: Sequence) -> bool:
+        """Whether a running sequence's next step takes a new block: the token sampled last starts one.  (Packed
+        batches compute prompts in portions; their blocks were all taken when the sequence was admitted.)"""
+        n = len(seq.token_ids)
+        if getattr(self, "packed", False) and n <= self.cache.num_tokens(seq.seq_id):
+            return False
+        return (n - 1) % self.config.block_size == 0
+
     def _make_room(self, decode_seqs: List[Sequence]) -> List[Sequence]:
         """Preempt from the most recently admitted end until the decodes that start a new block fit."""
-        bs = self.config.block_size
         keep = list(decode_seqs)
         while keep:
-            need = sum(1 for s in keep if (len(s.token_ids) - 1) % bs == 0)
+            need = sum(1 for s in keep if self._grows(s))
             if need <= self.cache.num_free_blocks():
                 break
             self._preempt(keep.pop())
@@ -297,6 +326,7 @@ class InferenceEngine:
         self.cache.deallocate(seq.seq_id)
         seq.status = SequenceStatus.WAITING
         seq.block_ids = []
+        seq.num_computed = 0
         self.running = [s for s in self.running if s.seq_id != seq.seq_id]
         self.waiting.insert(0, seq)
         self.num_preemptions += 1
@@ -307,6 +337,100 @@ class InferenceEngine:
         for i, s in enumerate(seqs):
             tables[i, : len(s.block_ids)] = s.block_ids
         return tables
+
+    # ------------------------------------------------------------------ packed batches
+    def forward_portions(self, portions: List[Tuple[Sequence, int]]) -> Tuple[torch.Tensor, List[int]]:
+        """One forward pass over the next ``count`` tokens of every sequence, all in one packed batch; the sequences
+        own the blocks for them.  Returns the hidden rows ``[tokens, width]`` and each portion's first row.  Single
+        tokens go first: they are attended by the decode kernel."""
+        order = sorted(range(len(portions)), key=lambda i: portions[i][1] > 1)
+        first = [0] * len(portions)
+        bs, at = self.config.block_size, 0
+        ids: List[int] = []
+        pos, slots, lens, q_lens, state = [], [], [], [], []
+        for i in order:
+            seq, count = portions[i]
+            lo = seq.num_computed
+            if count < 1 or lo + count > len(seq.token_ids):
+                raise ValueError(f"sequence {seq.seq_id} has no {count} tokens after {lo}")
+            p = np.arange(lo, lo + count)
+            ids += seq.token_ids[lo: lo + count]
+            pos.append(p)
+            slots.append(np.asarray(seq.block_ids, dtype=np.int64)[p // bs] * bs + p % bs)
+            lens.append(lo + count)
+            q_lens.append(count)
+            state.append(self.cache.state_slot(seq.seq_id) if isinstance(self.cache, PrivateKVCache) else -1)
+            first[i] = at
+            at += count
+        seqs = [portions[i][0] for i in order]
+        singles = sum(1 for c in q_lens if c == 1)
+        if singles == len(seqs) and self.config.use_graphs:
+            hidden = self._decode_replay(np.asarray(ids, dtype=np.int64)[:, None], np.concatenate(pos),
+                                         np.concatenate(slots), self._tables(seqs), np.asarray(lens),
+                                         np.asarray(state, dtype=np.int32))[:, 0]
+        else:
+            ctx = InferenceContext(is_prefill=True, slot_mapping=np.concatenate(slots), block_tables=self._tables(seqs),
+                                   seq_lens=np.asarray(lens), max_seq_len=max(lens), q_lens=np.asarray(q_lens),
+                                   num_decodes=singles, state_slots=np.asarray(state))
+            to_device = lambda a: torch.from_numpy(a).to(self.device)[None]
+            hidden = self.model(to_device(np.asarray(ids, dtype=np.int64)), to_device(np.concatenate(pos)), ctx)[0]
+        for seq, count in portions:
+            seq.num_computed += count
+        return hidden, first
+
+    def _packed_step(self, running: List[Sequence], admitted: List[Sequence]) -> List[Sequence]:
+        """The step of a model that runs packed rows: the running sequences' next tokens (a decoded token, or the next
+        portion of a prompt) and the admitted prompts' first portions, together.  Sequences whose every token has been
+        computed are sampled."""
+        for s in running:
+            if len(s.token_ids) > self.cache.num_tokens(s.seq_id):  # (the token sampled last)
+                self.cache.append_token(s.seq_id, s.token_ids[-1])
+                s.block_ids = list(self.cache.get_block_ids(s.seq_id))
+        for i, s in enumerate(admitted):
+            try:
+                s.block_ids = list(self.cache.allocate(s.seq_id, s.token_ids))
+            except RuntimeError:
+                self._defer(admitted[i:])
+                admitted = admitted[:i]
+                break
+        portions = [(s, step_tokens(s, self.scheduler_config)) for s in running + admitted]
+        if not portions:
+            return []
+        hidden, first = self.forward_portions(portions)
+        done = [(s, at + count - 1) for (s, count), at in zip(portions, first) if s.num_computed == len(s.token_ids)]
+        if not done:
+            return []
+        rows = torch.tensor([row for _, row in done], device=hidden.device)
+        return self._sample([s for s, _ in done], hidden[rows])
+
+    def open_sequence(self) -> Sequence:
+        """A sequence that is fed by hand: it has no tokens yet and is not scheduled."""
+        seq = Sequence(seq_id=self.seq_counter, token_ids=[], block_ids=[], num_prompt_tokens=0,
+                       status=SequenceStatus.RUNNING, temperature=0.0, max_tokens=0, stop_token_ids=frozenset(),
+                       output_logprobs=[])
+        self.seq_counter += 1
+        return seq
+
+    def feed(self, entries: List[Tuple[Sequence, List[int]]]) -> Tuple[torch.Tensor, List[int]]:
+        """Run the next tokens of sequences from ``open_sequence`` as one batch; returns ``forward_portions``' rows.
+        Needs the private allocator: what is fed is computed, never taken from another sequence's blocks."""
+        if not isinstance(self.cache, PrivateKVCache):
+            raise ValueError('feeding tokens needs cache_type="private"')
+        for seq, tokens in entries:
+            if len(seq.token_ids) + len(tokens) > self.config.max_model_len:
+                raise ValueError(f"sequence {seq.seq_id} exceeds max_model_len={self.config.max_model_len}")
+            if seq.token_ids:
+                self.cache.extend(seq.seq_id, len(tokens))
+            else:
+                self.cache.allocate(seq.seq_id, tokens)
+            seq.token_ids.extend(tokens)
+            seq.block_ids = list(self.cache.get_block_ids(seq.seq_id))
+        with torch.no_grad():
+            return self.forward_portions([(seq, len(tokens)) for seq, tokens in entries])
+
+    def close_sequence(self, seq: Sequence) -> None:
+        seq.status = SequenceStatus.FINISHED
+        self.cache.deallocate(seq.seq_id)
 
     def _prefill(self, seqs: List[Sequence]) -> List[Sequence]:
         cached, chunks = [], []
@@ -381,7 +505,7 @@ class InferenceEngine:
         return self._sample(seqs, hidden[:, 0])
 
     def _decode_replay(self, ids: np.ndarray, last_pos: np.ndarray, slots: np.ndarray, tables: np.ndarray,
-                       lens: np.ndarray) -> torch.Tensor:
+                       lens: np.ndarray, state_slots: Optional[np.ndarray] = None) -> torch.Tensor:
         """The decode step's forward pass from a captured graph.  Batches are padded to a bucket size with
         sequences of length 0 and slot -1 (nothing is written, their rows are ignored); the graph reads token
         ids, positions, slots, block tables and lengths from buffers that are rewritten before every replay."""
@@ -394,7 +518,7 @@ class InferenceEngine:
         if g is None:
             width = -(-self.config.max_model_len // self.config.block_size)
             g = self._decode_graphs[bucket] = _DecodeGraph(self.model, bucket, width, self.device)
-        return g.run(ids, last_pos, slots, tables, lens)[:n]
+        return g.run(ids, last_pos, slots, tables, lens, state_slots)[:n]
 
     def _recompute(self, seqs: List[Sequence]) -> List[Sequence]:
         """The reference's cache-less step: every sequence's whole token list, one at a time (engine.py:218-250)."""

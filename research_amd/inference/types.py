@@ -35,6 +35,13 @@ class InferenceContext:
                       are already in the cache.  When set on a prefill context
                       the chunk's queries attend over cache[0:prefix] followed
                       by the chunk itself (bottom-right aligned causal mask).
+    ``q_lens``        packed rows: the input is one row of tokens, the sequences one
+                      after the other with ``q_lens[b]`` new tokens each (``seq_lens``
+                      counts them).  Decode steps and portions of prompts share a batch.
+    ``num_decodes``   packed rows: the first so many sequences bring one token each and
+                      are attended by the decode kernel.
+    ``state_slots``   for models with recurrent state: the slot of each sequence, ``-1`` =
+                      none (a padding row of a captured decode step).
     """
 
     is_prefill: bool
@@ -44,6 +51,9 @@ class InferenceContext:
     max_seq_len: int = 0
     block_mask: Optional[object] = None
     prefix_lens: Optional[Tuple[int, ...]] = None
+    q_lens: Optional[Tuple[int, ...]] = None
+    num_decodes: int = 0
+    state_slots: Optional[Tuple[int, ...]] = None
 
 
 # --------------------------------------------------------------------------- engine configuration (types.py:14-49)
@@ -56,10 +66,13 @@ class EngineConfig:
     ``num_kv_blocks`` (pool size; default: enough for ``max_batch_size`` sequences of ``max_model_len`` tokens,
     capped at 65 536 blocks), ``eos_token_id`` (used when there is no tokenizer), ``use_graphs`` (replay the
     decode step's forward pass from a captured HIP graph per batch-size bucket instead of launching it kernel by
-    kernel)."""
+    kernel), ``dtype`` of a model loaded from ``model_path``, ``prefill_portion`` (models that run packed batches: the
+    most tokens of one prompt that a step takes; a longer prompt is computed over several steps, beside the
+    decodes; default: half the step's token budget).  ``cache_type="private"`` shares no blocks between sequences;
+    models with recurrent state always run on it, because a shared block does not bring its state along."""
 
     model_path: str
-    cache_type: str = "none"  # "paged" | "radix" | "none"
+    cache_type: str = "none"  # "paged" | "radix" | "private" | "none"
     block_size: int = 16
     max_batch_size: int = 256
     max_model_len: int = 8192
@@ -68,6 +81,8 @@ class EngineConfig:
     num_kv_blocks: Optional[int] = None
     eos_token_id: Optional[int] = None
     use_graphs: bool = False
+    dtype: str = "bfloat16"  # | "float32"
+    prefill_portion: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -81,11 +96,13 @@ class SamplingParams:
 
 @dataclass(frozen=True)
 class SchedulerConfig:
-    """Scheduler limits (types.py:36-42)."""
+    """Scheduler limits (types.py:36-42).  Added, optional: ``prefill_portion``, the most tokens of one sequence
+    that a step computes (0: whole prompts)."""
 
     max_batch_size: int
     max_tokens_per_batch: int
     block_size: int
+    prefill_portion: int = 0
 
 
 # --------------------------------------------------------------------------- outputs (types.py:50-69)
@@ -134,6 +151,7 @@ class Sequence:
     max_tokens: int
     stop_token_ids: FrozenSet[int]
     output_logprobs: List[float]
+    num_computed: int = 0  # tokens whose keys and state the cache holds (kept by packed batches)
 
     def append_token(self, token_id: int, logprob: float) -> None:
         assert self.status == SequenceStatus.RUNNING

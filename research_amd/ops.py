@@ -18,6 +18,8 @@ from . import _lib
 PA_DTYPE = {torch.float32: _lib.PA_F32, torch.bfloat16: _lib.PA_BF16, torch.float16: _lib.PA_F16,
             torch.float8_e4m3fn: _lib.PA_FP8_E4M3, torch.uint8: _lib.PA_FP8_E4M3}
 
+QKV_TILE_ROWS = _lib.PA_QKV_TILE_ROWS
+
 
 def _ptr(t: Optional[Tensor]) -> Optional[int]:
     return None if t is None else t.data_ptr()
@@ -324,3 +326,186 @@ def dequantize_blocks_e4m3(cache: Tensor, scale: Tensor, block_ids: Tensor, bloc
     _run("pa_dequantize_blocks_e4m3", _ptr(cache), _ptr(scale), _ptr(block_ids), block_ids.numel(), _ptr(dst),
          total_slots // block_size, block_size, hkv, d, PA_DTYPE[dtype], _stream(cache))
     return dst
+
+
+# ------------------------------------------------------------------ decoder blocks around attention
+
+
+def _row_stride(t: Tensor) -> int:
+    """Elements between the rows of a 2-D tensor whose rows are contiguous (a column slice of a wider one)."""
+    if t.dim() != 2 or (t.shape[1] > 1 and t.stride(1) != 1):
+        raise ValueError("expected a 2-D tensor with contiguous rows")
+    return t.stride(0) if t.shape[0] > 1 else max(t.stride(0), t.shape[1])
+
+
+def _dense(*tensors: Optional[Tensor]) -> None:
+    for t in tensors:
+        if t is not None and not t.is_contiguous():
+            raise ValueError("expected contiguous tensors")
+
+
+def _typed(dtype: torch.dtype, *tensors: Optional[Tensor]) -> None:
+    for t in tensors:
+        if t is not None and t.dtype != dtype:
+            raise ValueError(f"expected {dtype}, got {t.dtype}")
+
+
+_NORMS = {None: _lib.PA_NORM_NONE, "layer": _lib.PA_NORM_LAYER, "rms": _lib.PA_NORM_RMS}
+_ACTS = {"silu": _lib.PA_ACT_SILU, "gelu_tanh": _lib.PA_ACT_GELU_TANH}
+_V_MODES = {None: _lib.PA_V_PLAIN, "first": _lib.PA_V_FIRST, "mix": _lib.PA_V_MIX}
+
+
+def residual_norm(x: Tensor, dtype: torch.dtype, y: Optional[Tensor] = None, y_weight: Optional[Tensor] = None,
+                  y_eps: float = 0.0, ids: Optional[Tensor] = None, table: Optional[Tensor] = None,
+                  row_index: Optional[Tensor] = None, norm: Optional[str] = None, weight: Optional[Tensor] = None,
+                  bias: Optional[Tensor] = None, eps: float = 0.0, want_out: bool = True) -> Optional[Tensor]:
+    """Residual sum and norm in one pass over the rows (``pa_residual_norm``): ``x`` float32 ``[rows, width]`` is
+    updated in place (``table[ids]`` or itself, plus ``y`` or its RMS norm times ``y_weight``), and
+    ``norm(x) * weight + bias`` (``"layer"``, ``"rms"`` or None: a cast) comes back in ``dtype``.  ``row_index``
+    picks rows of ``x`` instead of updating it."""
+    rows, width = x.shape
+    _dense(x, y, y_weight, ids, table, row_index, weight, bias)
+    _typed(torch.float32, x, y_weight, weight, bias)
+    _typed(torch.int64, ids, row_index)
+    _typed(dtype, y, table)
+    n = rows if row_index is None else row_index.numel()
+    if (y is not None and tuple(y.shape) != (rows, width)) or (ids is not None and ids.numel() != rows):
+        raise ValueError("y / ids do not fit the residual")
+    if table is not None and table.shape[1] != width:
+        raise ValueError("table rows are not as wide as the residual")
+    for w in (y_weight, weight, bias):
+        if w is not None and w.numel() != width:
+            raise ValueError("norm weights are not as wide as the residual")
+    out = torch.empty((n, width), dtype=dtype, device=x.device) if want_out else None
+    _run("pa_residual_norm", _ptr(x), _ptr(y), _ptr(y_weight), float(y_eps), _ptr(ids), _ptr(table),
+         table.shape[0] if table is not None else 0, _ptr(row_index), rows, _ptr(weight), _ptr(bias), float(eps),
+         _NORMS[norm], _ptr(out), n, width, PA_DTYPE[dtype], _stream(x))
+    return out
+
+
+def rms_gate(o: Tensor, gate: Tensor, weight: Tensor, eps: float) -> Tensor:
+    """``o / rms(o) * weight * sigmoid(gate)`` per row (``pa_rms_gate``); ``gate`` may be a column slice."""
+    rows, width = o.shape
+    _dense(o, weight)
+    _typed(o.dtype, gate)
+    _typed(torch.float32, weight)
+    if tuple(gate.shape) != (rows, width) or weight.numel() != width:
+        raise ValueError("gate / weight do not fit o")
+    out = torch.empty_like(o)
+    _run("pa_rms_gate", _ptr(o), _ptr(gate), _row_stride(gate), _ptr(weight), float(eps), _ptr(out), rows, width,
+         PA_DTYPE[o.dtype], _stream(o))
+    return out
+
+
+def glu(gate: Tensor, up: Tensor, act: str, ids: Optional[Tensor] = None) -> Tensor:
+    """``act(gate) * up`` (``pa_glu``); both may be column slices.  With ``ids`` the factor of row r is row
+    ``ids[r]`` of ``up``."""
+    rows, width = gate.shape
+    _typed(gate.dtype, up)
+    _typed(torch.int64, ids)
+    if up.shape[1] != width or (up.shape[0] if ids is None else ids.numel()) != rows:
+        raise ValueError("up / ids do not fit gate")
+    out = torch.empty((rows, width), dtype=gate.dtype, device=gate.device)
+    _run("pa_glu", _ptr(gate), _row_stride(gate), _ptr(up), _row_stride(up), _ptr(ids), up.shape[0], _ptr(out), rows,
+         width, _ACTS[act], PA_DTYPE[gate.dtype], _stream(gate))
+    return out
+
+
+def head_gate(o: Tensor, gate: Optional[Tensor], vdim: int) -> Tensor:
+    """``[rows, heads, d]`` -> ``[rows, heads * vdim]``: the leading ``vdim`` of every head times the sigmoid of its
+    gate logit (``pa_head_gate``)."""
+    rows, heads, d = o.shape
+    _dense(o)
+    if gate is not None:
+        _typed(o.dtype, gate)
+        if tuple(gate.shape) != (rows, heads):
+            raise ValueError("gate must hold one logit per row and head")
+    out = torch.empty((rows, heads * vdim), dtype=o.dtype, device=o.device)
+    _run("pa_head_gate", _ptr(o), _ptr(gate), _row_stride(gate) if gate is not None else 0, _ptr(out), rows, heads, d, vdim,
+         PA_DTYPE[o.dtype], _stream(o))
+    return out
+
+
+class Portions(NamedTuple):
+    """Runs of new rows, one per sequence, as the kernels take them (int32 on the device).  ``q_lens`` /
+    ``q_starts`` None: one row per sequence, in order."""
+
+    ctx_lens: Tensor
+    state_slots: Optional[Tensor]
+    q_lens: Optional[Tensor] = None
+    q_starts: Optional[Tensor] = None
+    tiles: Optional[Tensor] = None  # [n, 2]: (sequence, first row) of every PA_QKV_TILE_ROWS rows
+    max_q_len: int = 1
+
+
+def qkv_conv_append(u: Tensor, portions: Portions, slots: Tensor, k_cache: Tensor, v_cache: Tensor, num_q_heads: int,
+                    dim: int, vdim: int, q_scale: float, eps: float, unit_norm: bool, rope: Optional[Tensor], rot_dims: int,
+                    conv_weight: Optional[Tensor], conv_state: Optional[Tensor], v_mode: Optional[str] = None,
+                    v_first: Optional[Tensor] = None, v_lambda: Optional[Tensor] = None,
+                    q_out: Optional[Tensor] = None) -> Tensor:
+    """Projection rows to rotated, normalised q and appended k / v (``pa_qkv_conv_append``).  Returns q
+    ``[rows, Hq, D]`` with D the pool's head size; k and v go to ``k_cache`` / ``v_cache`` ``[slots, Hkv, D]``."""
+    rows = u.shape[0]
+    total_slots, hkv, d = k_cache.shape
+    taps = conv_weight.shape[0] if conv_weight is not None else 1
+    channels = (num_q_heads + hkv) * dim + hkv * vdim
+    _dense(slots, k_cache, v_cache, rope, conv_weight, conv_state, v_first, *portions[:5])
+    _typed(u.dtype, k_cache, v_cache, conv_state, v_first)
+    _typed(torch.int32, *portions[:5])
+    _typed(torch.float32, rope, conv_weight, v_lambda)
+    _typed(torch.int64, slots)
+    batch = portions.ctx_lens.numel()
+    if slots.numel() != rows or v_cache.shape != k_cache.shape or u.shape[1] < channels:
+        raise ValueError("slots / v_cache / u do not fit")
+    if conv_weight is not None and (conv_weight.shape[1] != channels or (taps > 1 and tuple(conv_state.shape[1:]) != (taps - 1, channels))):
+        raise ValueError("convolution weights or state of another size")
+    if rope is not None and tuple(rope.shape[1:]) != (rot_dims // 2, 2):
+        raise ValueError("rope must be [positions, rot_dims / 2, 2]")
+    if v_first is not None and tuple(v_first.shape) != (rows, hkv * vdim):
+        raise ValueError("v_first must be [rows, Hkv * vdim]")
+    if q_out is None:
+        q_out = torch.empty((rows, num_q_heads, d), dtype=u.dtype, device=u.device)
+    n_tiles = batch if portions.tiles is None else portions.tiles.shape[0]
+    _run("pa_qkv_conv_append", _ptr(u), _row_stride(u), rows, _ptr(conv_weight), taps, _ptr(conv_state),
+         conv_state.shape[0] if conv_state is not None else 0, _ptr(rope), rope.shape[0] if rope is not None else 0,
+         rot_dims if rope is not None else 0, _ptr(portions.ctx_lens), _ptr(portions.q_lens), _ptr(portions.q_starts),
+         _ptr(portions.state_slots), _ptr(portions.tiles), n_tiles, batch, _ptr(slots), total_slots, _ptr(q_out),
+         _ptr(k_cache), _ptr(v_cache), _ptr(v_first), _ptr(v_lambda), _V_MODES[v_mode], num_q_heads, hkv, dim, vdim, d,
+         int(unit_norm), float(eps), float(q_scale), PA_DTYPE[u.dtype], _stream(u))
+    return q_out
+
+
+def lightning_state(num_slots: int, heads: int, dim: int, vdim: int, device) -> Tensor:
+    """The zero-filled state pool of one lightning layer, float32 ``[slots, heads, pad16(dim), pad16(vdim)]``."""
+    pad = lambda n: -(-n // 16) * 16
+    return torch.zeros((num_slots, heads, pad(dim), pad(vdim)), dtype=torch.float32, device=device)
+
+
+def lightning_workspace_bytes(batch: int, heads: int, dim: int, vdim: int, max_q_len: int) -> int:
+    return int(_lib.load().pa_lightning_workspace_bytes(batch, heads, dim, vdim, max_q_len))
+
+
+def lightning(u: Tensor, portions: Portions, state: Tensor, decay_powers: Tensor, heads: int, dim: int, vdim: int,
+              out: Tensor, workspace: Optional[Tensor] = None) -> Tensor:
+    """Lightning attention over projection rows ``[q | k | v | ...]`` with the state carried in ``state`` (see
+    ``lightning_state``): portions of bf16 rows in chunks on the matrix cores (``pa_lightning_chunked``), single rows
+    and float32 rows token by token (``pa_lightning_recurrent``).  ``out`` ``[rows, heads * vdim]``."""
+    _dense(state, decay_powers, out, *portions[:4])
+    _typed(torch.int32, *portions[:4])
+    _typed(torch.float32, state, decay_powers)
+    _typed(u.dtype, out)
+    rows, batch = u.shape[0], portions.ctx_lens.numel()
+    pad = lambda n: -(-n // 16) * 16
+    if tuple(state.shape[1:]) != (heads, pad(dim), pad(vdim)) or tuple(decay_powers.shape) != (heads, 65):
+        raise ValueError("state or decay table of another size")
+    if tuple(out.shape) != (rows, heads * vdim):
+        raise ValueError("out must be [rows, heads * vdim]")
+    head = (_ptr(u), _row_stride(u), rows, _ptr(state), state.shape[0], _ptr(decay_powers), _ptr(portions.ctx_lens),
+            _ptr(portions.q_lens), _ptr(portions.q_starts), _ptr(portions.state_slots), batch)
+    tail = (_ptr(out), heads, dim, vdim, PA_DTYPE[u.dtype])
+    if portions.q_lens is None or u.dtype == torch.float32:
+        _run("pa_lightning_recurrent", *head, *tail, _stream(u))
+    else:
+        _run("pa_lightning_chunked", *head, portions.max_q_len, *tail, _ptr(workspace),
+             workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(u))
+    return out
