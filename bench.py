@@ -10,7 +10,7 @@ head_dim 256 and 64; dense prefill of 64 x 512 and 4 x 8192 tokens; one chunk
 behind 200 000 cached keys at head_dim 128 and 256) under ``secondary``.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--no-secondary]
-                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine]
+                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen]
     python bench.py --traffic-from-pmc NAME KERNEL FETCH.csv WRITE.csv   # refresh profiles/traffic.json
 """
 
@@ -101,7 +101,7 @@ def parse_args():
     ap.add_argument("--steps", type=int, default=50)
     ap.add_argument("--warmup", type=int, default=10)
     ap.add_argument("--workload", default="c4", choices=["c1", "c2", "c3", "c3-d256", "c3-d64", "c3-d96", "long-d128", "long-d256", "dense-64x512",
-                                                         "dense-4x8192", "c4", "c5", "engine"])
+                                                         "dense-4x8192", "c4", "c5", "engine", "lotozen"])
     ap.add_argument("--preheat-s", type=float, default=0.5,
                     help="seconds of untimed steps before the warmup steps: an idle GPU sits at its lowest clocks "
                          "and takes a few hundred milliseconds of work to leave them")
@@ -710,6 +710,239 @@ def bench_decode(name, args, dev) -> dict:
     return result
 
 
+HYBRID_SHAPES = {
+    # width, query heads, kv heads, dim, vdim, lightning heads (of 128 x 128), feed-forward, token-side columns
+    "w2048": (2048, 16, 4, 128, 128, 16, 5632, 128),
+    "w2048-v64": (2048, 16, 4, 128, 64, 16, 5632, 128),
+    "w4096": (4096, 32, 8, 128, 128, 32, 14336, 256),
+}
+HYBRID_LAYERS, HYBRID_WINDOW, HYBRID_VOCAB = 8, 1024, 32000
+HYBRID_PREFILL, HYBRID_DECODE = (8, 2048), (128, 2048)  # (sequences, tokens), (sequences, cached tokens)
+
+
+def hybrid_model(shape, dev, num_blocks, slots, max_positions):
+    """A Lotozen-shaped model (window attention and lightning layers in turn) with random weights."""
+    from research_amd.inference import HipPagedAttentionBackend, HybridConfig, HybridDecoder
+    from research_amd.inference.hybrid import LayerSpec
+    from research_amd.inference.mixers import AttentionSpec, LightningSpec
+
+    width, heads, kv, dim, vdim, lheads, ff, side = shape
+    att = AttentionSpec(heads=heads, kv_heads=kv, dim=dim, vdim=vdim, scale=dim ** -0.5, window=HYBRID_WINDOW, taps=4,
+                        rot_dims=dim // 2, rot_base=10000.0, rot_factor=2.0, v_mix=True)
+    lin = LightningSpec(heads=lheads, dim=128, vdim=128, decay=tuple(1.0 - 2.0 ** -(2 + 6 * h / lheads) for h in range(lheads)))
+    cfg = HybridConfig(vocab_size=HYBRID_VOCAB, width=width, norm_eps=1e-6, side_dim=side,
+                       layers=tuple(LayerSpec(att if i % 2 == 0 else lin, ff) for i in range(HYBRID_LAYERS)))
+    backend = HipPagedAttentionBackend(cfg.cache_config(num_blocks, 16, slots, torch.bfloat16, "cuda"))
+    model = HybridDecoder(cfg, backend, max_positions)
+    with torch.no_grad():
+        for p in model.parameters():
+            p.normal_(0.0, p.shape[-1] ** -0.5)
+    return model.eval()
+
+
+def llama_model(shape, dev, num_blocks, max_positions):
+    """The closest other model at equal size: the same width, heads, feed-forward and layer count."""
+    from research_amd.inference import CacheConfig, HipPagedAttentionBackend, ModelConfig, PagedLlama
+
+    width, heads, kv, dim, _, _, ff, _ = shape
+    cfg = ModelConfig(vocab_size=HYBRID_VOCAB, hidden_size=width, intermediate_size=ff, num_layers=HYBRID_LAYERS,
+                      num_heads=heads, num_kv_heads=kv, head_dim=dim, max_position_embeddings=max_positions)
+    backend = HipPagedAttentionBackend(CacheConfig(num_layers=HYBRID_LAYERS, num_kv_heads=kv, head_dim=dim,
+                                                   num_blocks=num_blocks, block_size=16, device="cuda",
+                                                   dtype=torch.bfloat16))
+    with torch.device(dev):
+        model = PagedLlama(cfg, backend).to(torch.bfloat16)
+    return model.eval()
+
+
+def hybrid_throughput(model, dev, packed, steps, warmup, preheat_s):
+    """Milliseconds of one prefill pass and of one decode step (replayed from a captured graph)."""
+    from research_amd.inference import InferenceContext
+    from research_amd.inference.engine import _DecodeGraph
+
+    g = np.random.default_rng(3)
+    n_seq, n_tok = HYBRID_PREFILL
+    per = n_tok // 16
+    tables = g.permutation(n_seq * per).reshape(n_seq, per).astype(np.int32)
+    pos = np.tile(np.arange(n_tok), (n_seq, 1))
+    slots = np.take_along_axis(tables, pos // 16, 1).astype(np.int64) * 16 + pos % 16
+    ids = torch.from_numpy(g.integers(0, HYBRID_VOCAB, (n_seq, n_tok))).to(dev)
+    lens = np.full(n_seq, n_tok)
+    extra = dict(q_lens=lens, state_slots=np.arange(n_seq)) if packed else dict(prefix_lens=np.zeros(n_seq, dtype=np.int64))
+    ctx = InferenceContext(is_prefill=True, slot_mapping=slots.reshape(-1), block_tables=tables, seq_lens=lens,
+                           max_seq_len=n_tok, **extra)
+    tpos = torch.from_numpy(pos).to(dev)
+    fn = lambda: model(ids, tpos, ctx)
+    out = {}
+    with torch.no_grad():
+        preheat(fn, preheat_s)
+        for _ in range(warmup):
+            fn()
+        out["prefill_ms"] = timed_steps(fn, steps)[1]
+        batch, ctx_len = HYBRID_DECODE
+        width = ctx_len // 16 + 1
+        graph = _DecodeGraph(model, batch, width, dev)
+        tables = g.permutation(batch * width).reshape(batch, width).astype(np.int32)
+        args = (g.integers(0, HYBRID_VOCAB, (batch, 1)), np.full(batch, ctx_len),
+                tables[:, ctx_len // 16].astype(np.int64) * 16 + ctx_len % 16, tables, np.full(batch, ctx_len + 1))
+        graph.run(*args, np.arange(batch, dtype=np.int32) if packed else None)
+        fn = graph.graph.replay
+        preheat(fn, preheat_s)
+        for _ in range(warmup):
+            fn()
+        out["decode_ms"] = timed_steps(fn, steps)[1]
+    out["prefill_tokens_per_s"] = n_seq * n_tok / out["prefill_ms"] * 1e3
+    out["decode_tokens_per_s"] = batch / out["decode_ms"] * 1e3
+    return out
+
+
+def hybrid_kernels(shape, dev, steps):
+    """Every kernel of the new blocks alone at the layer's shapes, against its roofline, with the like kernel of the
+    Llama block.  Bytes and FLOPs are the algorithmic ones (heads unpadded)."""
+    from research_amd import ops
+
+    width, heads, kv, dim, vdim, lheads, ff, side = shape
+    bf, f32 = torch.bfloat16, torch.float32
+    rnd = lambda *s, dtype=bf: torch.randn(*s, device=dev, dtype=torch.float32).to(dtype)
+    i32 = lambda a: torch.as_tensor(np.ascontiguousarray(a), dtype=torch.int32).to(dev)
+    rows_out = []
+
+    def add(phase, name, fn, like, n_bytes=0.0, flops=0.0):
+        # (a graph of several launches: what the host takes to launch a short kernel is not the kernel's time)
+        fn()
+        torch.cuda.synchronize()
+        graph = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(graph):
+            for _ in range(8):
+                fn()
+        preheat(graph.replay, 0.05)
+        ms = timed_ms(graph.replay, max(1, steps // 4)) / 8
+        bound = max(n_bytes / HBM_PEAK_GBPS / 1e6, flops / MFMA_BF16_PEAK_TFLOPS / 1e9)
+        rows_out.append({"phase": phase, "kernel": name, "like": like, "us": round(1e3 * ms, 2),
+                         "pct_of_roofline": round(100.0 * bound / ms, 1),
+                         "bound": "mfma" if flops / MFMA_BF16_PEAK_TFLOPS / 1e9 > n_bytes / HBM_PEAK_GBPS / 1e6 else "hbm"})
+
+    d = -(-max(dim, vdim) // 8) * 8
+    chans = (heads + kv) * dim + kv * vdim
+    for phase, (batch, length) in (("prefill", HYBRID_PREFILL), ("decode", HYBRID_DECODE)):
+        dec = phase == "decode"
+        n = batch if dec else batch * length
+        per = length // 16 + (1 if dec else 0)
+        tables = np.random.default_rng(5).permutation(batch * per).reshape(batch, per).astype(np.int32)
+        ctx = np.full(batch, length + 1 if dec else length)
+        pos = np.full((batch, 1), length) if dec else np.tile(np.arange(length), (batch, 1))
+        slots = torch.from_numpy((np.take_along_axis(tables, pos // 16, 1).astype(np.int64) * 16 + pos % 16).reshape(-1)).to(dev)
+        bt, lens, sslots = i32(tables), i32(ctx), i32(np.arange(batch))
+        if dec:
+            por = ops.Portions(lens, sslots)
+        else:
+            first = np.arange(0, length, ops.QKV_TILE_ROWS)
+            tiles = np.stack([np.repeat(np.arange(batch), len(first)), np.tile(first, batch)], 1)
+            por = ops.Portions(lens, sslots, i32(ctx), i32(np.arange(batch) * length), i32(tiles), length)
+        x, y = rnd(n, width, dtype=f32), rnd(n, width)
+        w = rnd(width, dtype=f32)
+        add(phase, "residual + layer norm", lambda: ops.residual_norm(x, bf, y=y, norm="layer", weight=w, bias=w, eps=1e-6),
+            "rope_kv_append", n * width * 12.0)
+        add(phase, "residual + RMS-normed branch + layer norm",
+            lambda: ops.residual_norm(x, bf, y=y, y_weight=w, y_eps=1e-6, norm="layer", weight=w, bias=w, eps=1e-6),
+            "rope_kv_append", n * width * 12.0)
+        u2 = rnd(n, 2 * ff)
+        add(phase, "silu(gate) * up", lambda: ops.glu(u2[:, :ff], u2[:, ff:], "silu"), "rope_kv_append", n * ff * 6.0)
+        del u2
+        sg, st, ids = rnd(n, side), rnd(HYBRID_VOCAB, side * HYBRID_LAYERS), torch.randint(0, HYBRID_VOCAB, (n,), device=dev)
+        add(phase, "gelu(gate) * token row", lambda: ops.glu(sg, st[:, side: 2 * side], "gelu_tanh", ids=ids), "rope_kv_append",
+            n * (side * 6.0 + 8))
+        del x, y, st
+        # attention layer
+        u = rnd(n, chans + heads)
+        total = batch * per * 16
+        kc, vc = rnd(total, kv, d), rnd(total, kv, d)
+        conv = rnd(4, chans, dtype=f32)
+        cstate = torch.zeros(batch, 3, chans, dtype=bf, device=dev)
+        rope = rnd(length + 1, dim // 4, 2, dtype=f32)
+        vf, lam = rnd(n, kv * vdim), rnd(1, dtype=f32)
+        q = torch.empty(n, heads, d, dtype=bf, device=dev)
+        conv_bytes = n * 2.0 * (2 * chans + kv * vdim) + (batch * 2.0 * 2 * 3 * chans if dec else 0.0) + chans * 16.0
+        add(phase, "conv + rotation + unit norm + append",
+            lambda: ops.qkv_conv_append(u, por, slots, kc, vc, heads, dim, vdim, 1.0, 1e-6, True, rope, dim // 2, conv, cstate,
+                                        "mix", vf, lam, q_out=q), "rope_kv_append", conv_bytes)
+        cos = rnd(length + 1, d)
+        k0, v0 = rnd(n, kv, d), rnd(n, kv, d)
+        tpos = i32(pos.reshape(-1))
+        add(phase, "like: rope_kv_append", lambda: ops.rope_kv_append(q, k0, v0, cos, cos, kc, vc, slots, positions=tpos, q_out=q),
+            "", n * 2.0 * d * (2 * heads + 4 * kv))
+        o = torch.empty_like(q)
+        seen = np.minimum(ctx, HYBRID_WINDOW)
+        if dec:
+            ws = ops.decode_workspace(q, kc)
+            att = lambda win: ops.decode(q, kc, vc, bt, lens, 16, 0.1, ws, out=o, window=win)
+            add(phase, "decode attention, window", lambda: att(HYBRID_WINDOW), "decode attention",
+                2.0 * kv * (dim + vdim) * float(seen.sum()))
+            add(phase, "like: decode attention", lambda: att(0), "", 4.0 * kv * d * float(ctx.sum()))
+        else:
+            att = lambda win: ops.prefill_paged(q, kc, vc, bt, lens, por.q_lens, por.q_starts, length, 16, 0.1, out=o, window=win)
+            vis = np.minimum(np.arange(1, length + 1), HYBRID_WINDOW).sum() * batch
+            add(phase, "prefill attention, window", lambda: att(HYBRID_WINDOW), "prefill attention",
+                flops=2.0 * (dim + vdim) * heads * float(vis))
+            add(phase, "like: prefill attention", lambda: att(0), "",
+                flops=4.0 * d * heads * batch * length * (length + 1) / 2.0)
+        add(phase, "head gate", lambda: ops.head_gate(o, u[:, chans: chans + heads], vdim), "rope_kv_append",
+            n * heads * 2.0 * (2 * vdim + 1))
+        del u, kc, vc, q, o, k0, v0, vf
+        # lightning layer
+        inner = lheads * 128
+        u = rnd(n, 4 * inner)
+        state = ops.lightning_state(batch, lheads, 128, 128, dev)
+        powers = torch.full((lheads, 65), 0.97, device=dev) ** torch.arange(65, device=dev)
+        o = torch.empty(n, inner, dtype=bf, device=dev)
+        need = 0 if dec else ops.lightning_workspace_bytes(batch, lheads, 128, 128, length)
+        ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+        add(phase, "lightning attention", lambda: ops.lightning(u, por, state, powers, lheads, 128, 128, o, workspace=ws),
+            "decode attention" if dec else "prefill attention", n * inner * 8.0 + batch * lheads * 128 * 128 * 8.0)
+        nw = rnd(inner, dtype=f32)
+        add(phase, "RMS norm + sigmoid gate", lambda: ops.rms_gate(o, u[:, 3 * inner:], nw, 1e-6), "rope_kv_append", n * inner * 6.0)
+        if not dec:  # one long portion alone, in segments
+            por1 = ops.Portions(i32([n]), i32([0]), i32([n]), i32([0]), None, n)
+            need = ops.lightning_workspace_bytes(1, lheads, 128, 128, n)
+            ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+            add(phase, f"lightning attention, one sequence of {n}",
+                lambda: ops.lightning(u, por1, state, powers, lheads, 128, 128, o, workspace=ws), "prefill attention",
+                n * inner * 8.0 + lheads * 128 * 128 * 8.0)
+        del u, state, o
+        torch.cuda.empty_cache()
+    return rows_out
+
+
+def bench_hybrid(args, dev) -> int:
+    """Prefill and decode throughput of Lotozen-shaped models with random weights beside Llama-shaped ones of equal
+    size, and the new kernels against their rooflines.  Not the headline workload."""
+    sizes = {}
+    steps, warmup = min(args.steps, 20), min(args.warmup, 3)
+    for name, shape in HYBRID_SHAPES.items():
+        batch, ctx_len = HYBRID_DECODE
+        blocks = batch * (ctx_len // 16 + 1)
+        entry = {"shape": dict(zip(("width", "heads", "kv_heads", "dim", "vdim", "lightning_heads", "ff", "side"), shape))}
+        model = hybrid_model(shape, dev, blocks, batch, ctx_len + 16)
+        entry["lotozen"] = hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)
+        del model
+        torch.cuda.empty_cache()
+        model = llama_model(shape, dev, blocks, ctx_len + 16)
+        entry["llama"] = hybrid_throughput(model, dev, False, steps, warmup, args.preheat_s)
+        del model
+        torch.cuda.empty_cache()
+        entry["kernels"] = hybrid_kernels(shape, dev, steps)
+        sizes[name] = entry
+        print(f"[{name}] done", file=sys.stderr, flush=True)
+    main_size = sizes["w4096"]["lotozen"]
+    print(json.dumps({
+        "metric": "Lotozen prefill tokens/s", "value": main_size["prefill_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+        "steps": steps, "warmup": warmup, "ms_per_step": main_size["prefill_ms"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "lotozen", "layers": HYBRID_LAYERS, "window": HYBRID_WINDOW, "prefill": HYBRID_PREFILL,
+                   "decode": HYBRID_DECODE}, "sizes": sizes}))
+    return 0
+
+
 def secondary(args, dev) -> dict:
     """Short runs of the configurations that are not the headline: what the step costs, the dominant kernel
     against its roofline and a few seconds of the CPU restatement, per workload."""
@@ -751,6 +984,8 @@ def main() -> int:
     torch.cuda.set_device(dev)
     if args.workload == "engine":
         return bench_engine(args, dev)
+    if args.workload == "lotozen":
+        return bench_hybrid(args, dev)
     if args.workload in PREFILL_HEAD_SHAPES:
         result = bench_prefill_head(args, dev, args.workload)
     elif args.workload in PREFILL_LONG_SHAPES:

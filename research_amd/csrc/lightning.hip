@@ -31,7 +31,6 @@ struct LaArgs {
     float *ws;  // segment states
     int heads, dim, vdim, dp, vp;
     int segments, seg_rows;
-    int vec;  // 16-byte loads are possible
 };
 
 // The portion of sequence b: rows [row0, row0 + n), the first at position pos0.  False: nothing to do.
@@ -50,6 +49,13 @@ __device__ __forceinline__ bool la_portion(const LaArgs &a, int b, Portion &p) {
 
 // ------------------------------------------------------------------ token by token
 constexpr int kRecCols = 64;  // value columns per workgroup: 16 lanes x float4, 16 groups of lanes over the rows of S
+
+// silu as the products of a layer see it: in the type of the activations
+template <typename T> __device__ __forceinline__ float la_act(float x) {
+    x = row_silu<T>(x);
+    if constexpr (sizeof(T) == 2) return (float)(__bf16)x;
+    return x;
+}
 
 // R: rows of S per thread (16 R >= dim)
 template <typename T, int R> __global__ __launch_bounds__(256) void lightning_recurrent_kernel(const LaArgs a) {
@@ -74,14 +80,14 @@ template <typename T, int R> __global__ __launch_bounds__(256) void lightning_re
         const T *row = u + (p.row0 + t) * a.ldu;
         for (int i = tid; i < 2 * 16 * R + kRecCols; i += 256) {
             if (i < 16 * R) {
-                qs[i] = i < a.dim ? row_silu<T>(pa_scalar<T>::load(row + h * a.dim + i)) : 0.f;
+                qs[i] = i < a.dim ? la_act<T>(pa_scalar<T>::load(row + h * a.dim + i)) : 0.f;
             } else if (i < 32 * R) {
                 const int d = i - 16 * R;
-                ks[d] = d < a.dim ? row_silu<T>(pa_scalar<T>::load(row + (a.heads + h) * a.dim + d)) : 0.f;
+                ks[d] = d < a.dim ? la_act<T>(pa_scalar<T>::load(row + (a.heads + h) * a.dim + d)) : 0.f;
             } else {
                 const int v = i - 32 * R;
                 vs[v] = v0 + v < a.vdim
-                            ? row_silu<T>(pa_scalar<T>::load(row + 2 * a.heads * a.dim + h * a.vdim + v0 + v)) : 0.f;
+                            ? la_act<T>(pa_scalar<T>::load(row + 2 * a.heads * a.dim + h * a.vdim + v0 + v)) : 0.f;
             }
         }
         __syncthreads();
@@ -141,23 +147,25 @@ struct LaBlock {  // four rows of four consecutive columns, raw bf16
     uint2 r[4];
 };
 
-// The 4 x 4 block at (row s, column c) of a tile that has `n` rows and `cols` columns; zeros elsewhere.
-__device__ __forceinline__ LaBlock la_load_block(const uint16_t *base, int64_t ld, int s, int c, int n, int cols, int vec) {
+typedef uint32_t la_u2 __attribute__((ext_vector_type(2)));
+typedef uint32_t la_u4 __attribute__((ext_vector_type(4)));
+
+// A tile of `rows` rows of `cols` columns at row stride `ld` as a buffer: loads past its end give zeros, stores past it
+// are dropped.  (Columns past `cols` inside a row are the caller's: it gives such lanes the offset kLaOutside.)
+constexpr uint32_t kLaOutside = 0x40000000u;
+__device__ __forceinline__ __amdgpu_buffer_rsrc_t la_tile(const uint16_t *base, int64_t ld, int rows, int cols) {
+    return __builtin_amdgcn_make_buffer_rsrc((void *)base, 0, (int)(((rows - 1) * ld + cols) * 2), 0x00020000);
+}
+// Byte offset of the 4 x 4 block at (row s, column c)
+__device__ __forceinline__ uint32_t la_block_off(int64_t ld, int s, int c, int cols) {
+    return c < cols ? (uint32_t)(s * ld + c) * 2u : kLaOutside;
+}
+__device__ __forceinline__ LaBlock la_load_block(__amdgpu_buffer_rsrc_t tile, uint32_t off, uint32_t row_bytes) {
     LaBlock b;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        b.r[i] = make_uint2(0u, 0u);
-        if (s + i < n && c < cols) {
-            const uint16_t *p = base + (int64_t)(s + i) * ld + c;
-            if (vec) {
-                b.r[i] = *reinterpret_cast<const uint2 *>(p);
-            } else {
-                uint32_t e[4];
-#pragma unroll
-                for (int j = 0; j < 4; ++j) e[j] = c + j < cols ? p[j] : 0u;
-                b.r[i] = make_uint2(e[0] | (e[1] << 16), e[2] | (e[3] << 16));
-            }
-        }
+        const la_u2 x = __builtin_amdgcn_raw_buffer_load_b64(tile, off + i * row_bytes, 0, 0);
+        b.r[i] = make_uint2(x[0], x[1]);
     }
     return b;
 }
@@ -190,28 +198,31 @@ __device__ __forceinline__ void la_put_block(LaBlock b, int s, int c, __bf16 *rm
 
 constexpr int kLaPitchA = 72;  // bf16 per row of the decayed scores
 
-template <int KD, int NV> constexpr int la_q_elems() {  // Q tile; later the output tile
-    return 64 * (KD + 8) > 64 * (64 * NV + 8) ? 64 * (KD + 8) : 64 * (64 * NV + 8);
+template <int KD, int NW> constexpr int la_q_elems() {  // Q tile; later the output tile
+    return 64 * (KD + 8) > 64 * (16 * NW + 8) ? 64 * (KD + 8) : 64 * (16 * NW + 8);
 }
 template <int KD> constexpr int la_k_elems() {  // K tile; later the two terms of the decayed scores
     return 64 * (KD + 8) > 2 * 64 * kLaPitchA ? 64 * (KD + 8) : 2 * 64 * kLaPitchA;
 }
-template <int KD, int NV> constexpr size_t la_lds_bytes() {
-    return (size_t)(la_q_elems<KD, NV>() + la_k_elems<KD>() + KD * 64 + 64 * NV * 64) * 2 + 80 * 4;
+template <int KD, int NW> constexpr size_t la_lds_bytes() {
+    return (size_t)(la_q_elems<KD, NW>() + la_k_elems<KD>() + KD * 64 + 16 * NW * 64) * 2 + (64 + 64 + 80) * 4;
 }
 
-// KD: dim padded to 64, 128 or 256.  NV: 16-column tiles of the value slice per wave (the workgroup owns 64 NV columns).
+// KD: dim padded to 64, 128 or 256.  NW: waves; each owns 16 value columns.  All products are taken transposed (value
+// columns, or keys, as the rows of the result), so that a lane holds four consecutive elements of one row t.
 // STATES: only the segment's own contribution to the state, to the workspace (first pass over a portion in segments).
-template <int KD, int NV, bool STATES>
-__global__ __launch_bounds__(256) void lightning_chunk_kernel(const LaArgs a) {
-    constexpr int kCols = 64 * NV, kLdR = KD + 8, kLdO = kCols + 8;
-    constexpr int kKPass = KD / 64, kVPass = NV, kDB = KD / 4;  // 4x4 blocks: kDB per four rows of K
+template <int KD, int NW, bool STATES>
+__global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) void lightning_chunk_kernel(const LaArgs a) {
+    constexpr int kCols = 16 * NW, kLdR = KD + 8, kLdO = kCols + 8, kThr = 64 * NW;
+    constexpr int kDB = KD / 4, kKBlocks = 16 * kDB, kKPass = (kKBlocks + kThr - 1) / kThr;  // 4x4 blocks of K
+    constexpr int kST = NW == 8 ? 2 : 4;  // score tiles per wave
     extern __shared__ __align__(16) char lds[];
     __bf16 *q_s = reinterpret_cast<__bf16 *>(lds);
-    __bf16 *k_s = q_s + la_q_elems<KD, NV>();
+    __bf16 *k_s = q_s + la_q_elems<KD, NW>();
     __bf16 *kt_s = k_s + la_k_elems<KD>();
     __bf16 *vt_s = kt_s + KD * 64;
-    float *pw = reinterpret_cast<float *>(vt_s + kCols * 64);
+    float *rev = reinterpret_cast<float *>(vt_s + kCols * 64);  // decay from row s to the chunk's last row
+    float *pw = rev + 128;  // powers 0 .. 64, behind 64 zeros for the keys after a row
     __bf16 *a_hi = k_s, *a_lo = k_s + 64 * kLaPitchA, *o_s = q_s;
 
     const int h = blockIdx.x, seg = blockIdx.y % a.segments, vsl = blockIdx.y / a.segments, b = blockIdx.z;
@@ -219,211 +230,208 @@ __global__ __launch_bounds__(256) void lightning_chunk_kernel(const LaArgs a) {
     if (!la_portion(a, b, p)) return;
     const int r_beg = seg * a.seg_rows, r_end = r_beg + a.seg_rows < p.n ? r_beg + a.seg_rows : p.n;
     if (r_beg >= p.n) return;
-    const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, g = lane >> 4;
-    const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int v0 = vsl * kCols, vw = wave * 16 * NV;  // first column of the workgroup, of the wave inside it
-    if (tid <= kLaChunk) pw[tid] = a.decay[h * (kLaChunk + 1) + tid];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int v0 = vsl * kCols, vw = wave * 16;  // first column of the workgroup, of the wave inside it
+    const float *powers = a.decay + h * (kLaChunk + 1);
+    if (tid <= kLaChunk) pw[tid] = powers[tid];
+    if (tid < 64) {
+        rev[tid] = powers[63 - tid];
+        pw[tid - 64] = 0.f;
+    }
+    const int lane0 = tid & 63;
+    float pt[4];  // decay from the chunk's start to row 16 tt + l16
+#pragma unroll
+    for (int tt = 0; tt < 4; ++tt) pt[tt] = powers[16 * tt + (lane0 & 15) + 1];
 
-    // The state slice of this wave: tile (dt, vt) holds d = 16 dt + 4 g + i, v = v0 + vw + 16 vt + l16
-    f4 s[KD / 16][NV];
+    // The state slice of this wave: tile dt holds d = 16 dt + 4 g + i, v = v0 + vw + l16
+    f4 s[KD / 16];
     const int64_t state_elems = (int64_t)a.dp * a.vp;
     float *pool = p.slot >= 0 ? a.state + (p.slot * a.heads + h) * state_elems : nullptr;
     float *seg_state = a.segments > 1 ? a.ws + (((int64_t)b * a.heads + h) * a.segments + seg) * state_elems : nullptr;
     const float *from = STATES ? nullptr : (a.segments > 1 ? seg_state : (p.pos0 > 0 ? pool : nullptr));
+    // (a state as a buffer: rows past dp lie past its end, columns past vp get an offset outside)
+    const int state_bytes = (int)state_elems * 4;
+    const int v = v0 + vw + (lane0 & 15);
+    const uint32_t soff = v < a.vp ? (uint32_t)(4 * (lane0 >> 4) * a.vp + v) * 4u : kLaOutside;
+    {
+        const __amdgpu_buffer_rsrc_t src = __builtin_amdgcn_make_buffer_rsrc(
+            (void *)(from ? from : a.state), 0, from ? state_bytes : 0, 0x00020000);  // (no state: every load is past the end)
 #pragma unroll
-    for (int dt = 0; dt < KD / 16; ++dt)
+        for (int dt = 0; dt < KD / 16; ++dt)
 #pragma unroll
-        for (int vt = 0; vt < NV; ++vt)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int d = 16 * dt + 4 * g + i, v = v0 + vw + 16 * vt + l16;
-                s[dt][vt][i] = from && d < a.dp && v < a.vp ? from[(int64_t)d * a.vp + v] : 0.f;
-            }
+            for (int i = 0; i < 4; ++i)
+                s[dt][i] = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(src, soff + (16 * dt + i) * a.vp * 4, 0, 0));
+    }
 
     const uint16_t *u = reinterpret_cast<const uint16_t *>(a.u) + p.row0 * a.ldu;
     const uint16_t *uq = u + h * a.dim, *uk = u + (a.heads + h) * a.dim;
     const uint16_t *uv = u + 2 * a.heads * a.dim + h * a.vdim + v0;
     const int vcols = a.vdim - v0 < kCols ? a.vdim - v0 : kCols;
-    LaBlock kb[kKPass], vb[kVPass], qb[STATES ? 1 : kKPass];
+    const uint32_t row_bytes = (uint32_t)a.ldu * 2u;
+    LaBlock kb[kKPass], qb[STATES ? 1 : kKPass], vb;
+    uint32_t koff[kKPass];
+#pragma unroll
+    for (int i = 0; i < kKPass; ++i) {
+        const int blk = tid + kThr * i;
+        koff[i] = blk < kKBlocks ? la_block_off(a.ldu, blk / kDB * 4, blk % kDB * 4, a.dim) : kLaOutside;
+    }
+    const uint32_t voff = la_block_off(a.ldu, tid / (kCols / 4) * 4, tid % (kCols / 4) * 4, vcols);
     auto fetch = [&](int r0) {
+        const int rows = r_end - r0 < kLaChunk ? r_end - r0 : kLaChunk;
+        const int64_t at = (int64_t)r0 * a.ldu;
+        const __amdgpu_buffer_rsrc_t tk = la_tile(uk + at, a.ldu, rows, a.dim), tv = la_tile(uv + at, a.ldu, rows, vcols);
+        if (!STATES) {
+            const __amdgpu_buffer_rsrc_t tq = la_tile(uq + at, a.ldu, rows, a.dim);
 #pragma unroll
-        for (int i = 0; i < kKPass; ++i) {
-            const int blk = tid + 256 * i, c = blk % kDB * 4, sr = blk / kDB * 4;
-            kb[i] = la_load_block(uk + (int64_t)r0 * a.ldu, a.ldu, sr, c, r_end - r0, a.dim, a.vec);
-            if (!STATES) qb[i] = la_load_block(uq + (int64_t)r0 * a.ldu, a.ldu, sr, c, r_end - r0, a.dim, a.vec);
+            for (int i = 0; i < kKPass; ++i) qb[i] = la_load_block(tq, koff[i], row_bytes);
         }
 #pragma unroll
-        for (int i = 0; i < kVPass; ++i) {
-            const int blk = tid + 256 * i, c = blk % (kCols / 4) * 4, sr = blk / (kCols / 4) * 4;
-            vb[i] = la_load_block(uv + (int64_t)r0 * a.ldu, a.ldu, sr, c, r_end - r0, vcols, a.vec);
-        }
+        for (int i = 0; i < kKPass; ++i) kb[i] = la_load_block(tk, koff[i], row_bytes);
+        vb = la_load_block(tv, voff, row_bytes);
     };
     fetch(r_beg);
     for (int r0 = r_beg; r0 < r_end; r0 += kLaChunk) {
         const int nv = r_end - r0 < kLaChunk ? r_end - r0 : kLaChunk;
+        int self = tid;
+        asm volatile("" : "+v"(self));  // (LDS addresses are made again per chunk: kept over the loop they would spill)
+        const int lane = self & 63, l16 = lane & 15, g = lane >> 4;
 #pragma unroll
         for (int i = 0; i < kKPass; ++i) {
-            const int blk = tid + 256 * i, c = blk % kDB * 4, sr = blk / kDB * 4;
+            const int blk = self + kThr * i, c = blk % kDB * 4, sr = blk / kDB * 4;
+            if (kKBlocks % kThr != 0 && blk >= kKBlocks) continue;
             la_put_block(kb[i], sr, c, STATES ? nullptr : k_s, kLdR, kt_s);
             if (!STATES) la_put_block(qb[i], sr, c, q_s, kLdR, nullptr);
         }
-#pragma unroll
-        for (int i = 0; i < kVPass; ++i) {
-            const int blk = tid + 256 * i, c = blk % (kCols / 4) * 4, sr = blk / (kCols / 4) * 4;
-            la_put_block(vb[i], sr, c, nullptr, 0, vt_s);
-        }
+        la_put_block(vb, self / (kCols / 4) * 4, self % (kCols / 4) * 4, nullptr, 0, vt_s);
+        if (nv < kLaChunk && tid < 64) rev[tid] = tid < nv ? powers[nv - 1 - tid] : 0.f;
         if (r0 + kLaChunk < r_end) fetch(r0 + kLaChunk);
         __syncthreads();
 
-        f4 o[4][NV];
+        f4 o[4];  // O^T: v = 4 g + i of the wave's columns, t = 16 tt + l16
         if constexpr (!STATES) {
-            // scores of this wave's 16 rows against the columns up to them
-            f4 sc[4];
+            // score tiles (st, rt): keys 16 st + 4 g + i, rows 16 rt + l16
+            const int rt = NW == 8 ? wave >> 1 : wave;
+            f4 sc[kST];
 #pragma unroll
-            for (int st = 0; st < 4; ++st) sc[st] = f4{0.f, 0.f, 0.f, 0.f};
+            for (int m = 0; m < kST; ++m) sc[m] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int kk = 0; kk < KD / 32; ++kk) {
-                const bf8 aq = la_read8(q_s + (16 * wave + l16) * kLdR + 32 * kk + 8 * g);
+                const bf8 bq = la_read8(q_s + (16 * rt + l16) * kLdR + 32 * kk + 8 * g);
 #pragma unroll
-                for (int st = 0; st < 4; ++st)
-                    if (st <= wave) sc[st] = la_mfma(aq, la_read8(k_s + (16 * st + l16) * kLdR + 32 * kk + 8 * g), sc[st]);
+                for (int m = 0; m < kST; ++m) {
+                    const int st = NW == 8 ? 2 * m + (wave & 1) : m;
+                    if (st <= rt) sc[m] = la_mfma(la_read8(k_s + (16 * st + l16) * kLdR + 32 * kk + 8 * g), bq, sc[m]);
+                }
             }
             // the rows' part from before the chunk: Q S, then the decay of the way from the chunk's start
 #pragma unroll
-            for (int tt = 0; tt < 4; ++tt)
+            for (int tt = 0; tt < 4; ++tt) o[tt] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int vt = 0; vt < NV; ++vt) o[tt][vt] = f4{0.f, 0.f, 0.f, 0.f};
+            for (int dd = 0; dd < KD / 32; ++dd) {
+                bf8 hi, lo;
 #pragma unroll
-            for (int dp = 0; dp < KD / 32; ++dp) {
-                bf8 hi[NV], lo[NV];
-#pragma unroll
-                for (int vt = 0; vt < NV; ++vt)
-#pragma unroll
-                    for (int j = 0; j < 8; ++j) {
-                        __bf16 x, y;
-                        la_split(s[2 * dp + j / 4][vt][j % 4], x, y);
-                        hi[vt][j] = x;
-                        lo[vt][j] = y;
-                    }
+                for (int j = 0; j < 8; ++j) {
+                    __bf16 x, y;
+                    la_split(s[2 * dd + j / 4][j % 4], x, y);
+                    hi[j] = x;
+                    lo[j] = y;
+                }
 #pragma unroll
                 for (int tt = 0; tt < 4; ++tt) {
-                    const __bf16 *qr = q_s + (16 * tt + l16) * kLdR + 32 * dp + 4 * g;
-                    const bf8 aq = la_read44(qr, qr + 16);
-#pragma unroll
-                    for (int vt = 0; vt < NV; ++vt) {
-                        o[tt][vt] = la_mfma(aq, hi[vt], o[tt][vt]);
-                        o[tt][vt] = la_mfma(aq, lo[vt], o[tt][vt]);
-                    }
+                    const __bf16 *qr = q_s + (16 * tt + l16) * kLdR + 32 * dd + 4 * g;
+                    const bf8 bq = la_read44(qr, qr + 16);
+                    o[tt] = la_mfma(hi, bq, o[tt]);
+                    o[tt] = la_mfma(lo, bq, o[tt]);
                 }
+                __builtin_amdgcn_sched_barrier(0);
             }
 #pragma unroll
             for (int tt = 0; tt < 4; ++tt)
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const float f = pw[16 * tt + 4 * g + i + 1];
-#pragma unroll
-                    for (int vt = 0; vt < NV; ++vt) o[tt][vt][i] *= f;
-                }
+                for (int i = 0; i < 4; ++i) o[tt][i] *= pt[tt];
             __syncthreads();  // Q and K have been read: their space takes the decayed scores (and, later, O)
 #pragma unroll
-            for (int st = 0; st < 4; ++st) {
-                if (st > wave + 1) continue;  // (tile wave + 1 is read as zeros when the last k-step covers it)
+            for (int m = 0; m < kST; ++m) {
+                const int st = NW == 8 ? 2 * m + (wave & 1) : m;
+                if (st > rt + 1) continue;  // (tile rt + 1 is read as zeros when the last k-step covers it)
+                const int t = 16 * rt + l16, c = 16 * st + 4 * g;
+                float hi[4], lo[4];
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
-                    const int t = 16 * wave + 4 * g + i, c = 16 * st + l16;
-                    __bf16 x = (__bf16)0.f, y = (__bf16)0.f;
-                    if (c <= t) la_split(sc[st][i] * pw[t - c], x, y);
-                    a_hi[t * kLaPitchA + c] = x;
-                    a_lo[t * kLaPitchA + c] = y;
+                    const float f = sc[m][i] * pw[t - c - i];
+                    const __bf16 x = (__bf16)f;
+                    hi[i] = f;
+                    lo[i] = f - (float)x;
                 }
+                *reinterpret_cast<uint2 *>(a_hi + t * kLaPitchA + c) = make_uint2(row_pack_bf16(hi[0], hi[1]), row_pack_bf16(hi[2], hi[3]));
+                *reinterpret_cast<uint2 *>(a_lo + t * kLaPitchA + c) = make_uint2(row_pack_bf16(lo[0], lo[1]), row_pack_bf16(lo[2], lo[3]));
             }
             __syncthreads();
 #pragma unroll
             for (int kk = 0; kk < 2; ++kk) {
-                bf8 bv[NV];
-#pragma unroll
-                for (int vt = 0; vt < NV; ++vt) bv[vt] = la_read8(vt_s + la_tr(vw + 16 * vt + l16, 32 * kk + 8 * g));
+                const bf8 av = la_read8(vt_s + la_tr(vw + l16, 32 * kk + 8 * g));
 #pragma unroll
                 for (int tt = 2 * kk; tt < 4; ++tt) {
-                    const bf8 ah = la_read8(a_hi + (16 * tt + l16) * kLaPitchA + 32 * kk + 8 * g);
-                    const bf8 al = la_read8(a_lo + (16 * tt + l16) * kLaPitchA + 32 * kk + 8 * g);
-#pragma unroll
-                    for (int vt = 0; vt < NV; ++vt) {
-                        o[tt][vt] = la_mfma(ah, bv[vt], o[tt][vt]);
-                        o[tt][vt] = la_mfma(al, bv[vt], o[tt][vt]);
-                    }
+                    o[tt] = la_mfma(av, la_read8(a_hi + (16 * tt + l16) * kLaPitchA + 32 * kk + 8 * g), o[tt]);
+                    o[tt] = la_mfma(av, la_read8(a_lo + (16 * tt + l16) * kLaPitchA + 32 * kk + 8 * g), o[tt]);
                 }
             }
+#pragma unroll
+            for (int tt = 0; tt < 4; ++tt)  // to LDS (where Q was), so that rows are stored 16 bytes per lane
+                *reinterpret_cast<uint2 *>(o_s + (16 * tt + l16) * kLdO + vw + 4 * g) =
+                    make_uint2(row_pack_bf16(o[tt][0], o[tt][1]), row_pack_bf16(o[tt][2], o[tt][3]));
         }
         // S <- decay^nv S + K^T (decay^(nv-1-s) V)
         const float whole = pw[nv];
 #pragma unroll
         for (int dt = 0; dt < KD / 16; ++dt)
 #pragma unroll
-            for (int vt = 0; vt < NV; ++vt)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) s[dt][vt][i] *= whole;
+            for (int i = 0; i < 4; ++i) s[dt][i] *= whole;
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
-            bf8 hi[NV], lo[NV];
+            bf8 hi, lo;
+            const bf8 bv = la_read8(vt_s + la_tr(vw + l16, 32 * kk + 8 * g));
+            const f4 w0 = *reinterpret_cast<const f4 *>(rev + 32 * kk + 8 * g), w1 = *reinterpret_cast<const f4 *>(rev + 32 * kk + 8 * g + 4);
 #pragma unroll
-            for (int vt = 0; vt < NV; ++vt) {
-                const bf8 bv = la_read8(vt_s + la_tr(vw + 16 * vt + l16, 32 * kk + 8 * g));
-#pragma unroll
-                for (int j = 0; j < 8; ++j) {
-                    const int back = nv - 1 - (32 * kk + 8 * g + j);
-                    __bf16 x, y;
-                    la_split((float)bv[j] * pw[back < 0 ? 0 : back], x, y);  // (rows past the end hold zeros)
-                    hi[vt][j] = x;
-                    lo[vt][j] = y;
-                }
+            for (int j = 0; j < 8; ++j) {
+                __bf16 x, y;
+                la_split((float)bv[j] * (j < 4 ? w0[j % 4] : w1[j % 4]), x, y);
+                hi[j] = x;
+                lo[j] = y;
             }
 #pragma unroll
             for (int dt = 0; dt < KD / 16; ++dt) {
                 const bf8 ak = la_read8(kt_s + la_tr(16 * dt + l16, 32 * kk + 8 * g));
-#pragma unroll
-                for (int vt = 0; vt < NV; ++vt) {
-                    s[dt][vt] = la_mfma(ak, hi[vt], s[dt][vt]);
-                    s[dt][vt] = la_mfma(ak, lo[vt], s[dt][vt]);
-                }
+                s[dt] = la_mfma(ak, hi, s[dt]);
+                s[dt] = la_mfma(ak, lo, s[dt]);
             }
         }
         if constexpr (!STATES) {
-            // O through LDS (where Q was), so that rows are stored 16 bytes per lane
-#pragma unroll
-            for (int tt = 0; tt < 4; ++tt)
-#pragma unroll
-                for (int vt = 0; vt < NV; ++vt)
-#pragma unroll
-                    for (int i = 0; i < 4; ++i)
-                        o_s[(16 * tt + 4 * g + i) * kLdO + vw + 16 * vt + l16] = (__bf16)o[tt][vt][i];
             __syncthreads();
-            uint16_t *dst = reinterpret_cast<uint16_t *>(a.out) + (p.row0 + r0) * ((int64_t)a.heads * a.vdim) + h * a.vdim + v0;
-            for (int i = tid; i < 64 * (kCols / 8); i += 256) {
-                const int t = i / (kCols / 8), c = i % (kCols / 8) * 8;
-                if (t >= nv || c >= vcols) continue;
-                const __bf16 *src = o_s + t * kLdO + c;
-                uint16_t *at = dst + (int64_t)t * ((int64_t)a.heads * a.vdim) + c;
-                if (a.vec) {
-                    *reinterpret_cast<uint4 *>(at) = *reinterpret_cast<const uint4 *>(src);
-                } else {
-                    for (int j = 0; j < 8 && c + j < vcols; ++j) at[j] = __builtin_bit_cast(uint16_t, src[j]);
-                }
+            const int ldo = a.heads * a.vdim;
+            const __amdgpu_buffer_rsrc_t dst = la_tile(reinterpret_cast<const uint16_t *>(a.out) + (p.row0 + r0) * (int64_t)ldo + h * a.vdim + v0,
+                                                       ldo, nv, vcols);
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {  // (64 rows of kCols columns are two 16-byte vectors per thread)
+                const int vec = self + kThr * i, t = vec / (kCols / 8), c = vec % (kCols / 8) * 8;
+                const la_u4 x = *reinterpret_cast<const la_u4 *>(o_s + t * kLdO + c);
+                __builtin_amdgcn_raw_buffer_store_b128(x, dst, c < vcols ? (uint32_t)(t * ldo + c) * 2u : kLaOutside, 0, 0);
             }
         }
         __syncthreads();
     }
     float *to = STATES ? seg_state : (a.segments > 1 ? nullptr : pool);
     if (!to) return;
+    const __amdgpu_buffer_rsrc_t dst = __builtin_amdgcn_make_buffer_rsrc((void *)to, 0, state_bytes, 0x00020000);
+    uint32_t base = soff;
+    asm volatile("" : "+v"(base));  // (offsets made again here instead of kept in registers over the loop)
 #pragma unroll
     for (int dt = 0; dt < KD / 16; ++dt)
 #pragma unroll
-        for (int vt = 0; vt < NV; ++vt)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) {
-                const int d = 16 * dt + 4 * g + i, v = v0 + vw + 16 * vt + l16;
-                if (d < a.dp && v < a.vp) to[(int64_t)d * a.vp + v] = s[dt][vt][i];
-            }
+        for (int i = 0; i < 4; ++i) {
+            const float f = s[dt][i];
+            __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(uint32_t, f), dst, base + (16 * dt + i) * a.vp * 4, 0, 0);
+        }
 }
 
 // Segment contributions -> start states, in place; the state after the last segment goes back to the pool.
@@ -474,19 +482,19 @@ template <typename K> int la_big_lds(K kernel, size_t bytes, const char *what) {
     return PA_OK;
 }
 
-template <int KD, int NV> int launch_chunks(const LaArgs &a, int batch, hipStream_t s) {
-    constexpr size_t lds = la_lds_bytes<KD, NV>();
+template <int KD, int NW> int launch_chunks(const LaArgs &a, int batch, hipStream_t s) {
+    constexpr size_t lds = la_lds_bytes<KD, NW>();
     static_assert(lds <= 160 * 1024, "LDS of one compute unit");
-    const int slices = (a.vdim + 64 * NV - 1) / (64 * NV);
-    const dim3 grid((unsigned)a.heads, (unsigned)(slices * a.segments), (unsigned)batch);
+    const int slices = (a.vdim + 16 * NW - 1) / (16 * NW);
+    const dim3 grid((unsigned)a.heads, (unsigned)(slices * a.segments), (unsigned)batch), block(64 * NW);
     if (a.segments > 1) {
-        if (int rc = la_big_lds(lightning_chunk_kernel<KD, NV, true>, lds, "pa_lightning_chunked")) return rc;
-        lightning_chunk_kernel<KD, NV, true><<<grid, dim3(256), lds, s>>>(a);
+        if (int rc = la_big_lds(lightning_chunk_kernel<KD, NW, true>, lds, "pa_lightning_chunked")) return rc;
+        lightning_chunk_kernel<KD, NW, true><<<grid, block, lds, s>>>(a);
         const unsigned gx = (unsigned)(((int64_t)a.dp * a.vp / 4 + 255) / 256);
         lightning_scan_kernel<<<dim3(gx, (unsigned)a.heads, (unsigned)batch), dim3(256), 0, s>>>(a);
     }
-    if (int rc = la_big_lds(lightning_chunk_kernel<KD, NV, false>, lds, "pa_lightning_chunked")) return rc;
-    lightning_chunk_kernel<KD, NV, false><<<grid, dim3(256), lds, s>>>(a);
+    if (int rc = la_big_lds(lightning_chunk_kernel<KD, NW, false>, lds, "pa_lightning_chunked")) return rc;
+    lightning_chunk_kernel<KD, NW, false><<<grid, block, lds, s>>>(a);
     PA_CHECK_LAUNCH("pa_lightning_chunked");
     return PA_OK;
 }
@@ -518,12 +526,12 @@ int la_fill(const char *what, LaArgs &a, const void *u, int64_t u_stride, int64_
     a.ctx_lens = ctx_lens; a.q_lens = q_lens; a.q_starts = q_starts; a.state_slots = state_slots; a.out = out;
     a.heads = num_heads; a.dim = dim; a.vdim = vdim; a.dp = la_pad16(dim); a.vp = la_pad16(vdim);
     a.segments = 1;
-    a.vec = dim % 8 == 0 && vdim % 8 == 0 && u_stride % 8 == 0 && pa_aligned16(u) && pa_aligned16(out);
     return PA_OK;
 }
 
 int la_plan(int64_t batch, int heads, int dim, int vdim, int max_q_len) {
-    const int cols = la_value_cols(dim, vdim);
+    (void)dim;
+    const int cols = la_value_cols(vdim);
     return la_segments(batch * heads * ((vdim + cols - 1) / cols), la_cus(), max_q_len);
 }
 
@@ -582,8 +590,15 @@ extern "C" int pa_lightning_chunked(const void *u, int64_t u_stride, int64_t n_r
     a.ws = (float *)workspace;
     PA_REQUIRE(a.segments == 1 || pa_aligned16(workspace), "the workspace must be 16-byte aligned");
     hipStream_t s = (hipStream_t)stream;
-    const bool wide = la_value_cols(dim, vdim) == 128;
-    if (dim <= 64) return wide ? launch_chunks<64, 2>(a, batch, s) : launch_chunks<64, 1>(a, batch, s);
-    if (dim <= 128) return wide ? launch_chunks<128, 2>(a, batch, s) : launch_chunks<128, 1>(a, batch, s);
-    return launch_chunks<256, 1>(a, batch, s);
+    // rows that are not whole 16-byte vectors, or too far apart for a tile's 32-bit offsets: token by token
+    if (dim % 8 != 0 || vdim % 8 != 0 || u_stride % 8 != 0 || !pa_aligned16(u) || !pa_aligned16(out) ||
+        u_stride > (1 << 22) || (int64_t)num_heads * vdim > (1 << 22)) {
+        launch_recurrent<pa_bf16>(a, batch, s);
+        PA_CHECK_LAUNCH("pa_lightning_chunked");
+        return PA_OK;
+    }
+    const bool wide = la_value_cols(vdim) == 128;
+    if (dim <= 64) return wide ? launch_chunks<64, 8>(a, batch, s) : launch_chunks<64, 4>(a, batch, s);
+    if (dim <= 128) return wide ? launch_chunks<128, 8>(a, batch, s) : launch_chunks<128, 4>(a, batch, s);
+    return wide ? launch_chunks<256, 8>(a, batch, s) : launch_chunks<256, 4>(a, batch, s);
 }

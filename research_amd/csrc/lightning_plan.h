@@ -10,9 +10,8 @@ constexpr int kLaMaxSegments = 64;
 
 static inline int la_pad16(int n) { return (n + 15) / 16 * 16; }
 
-// Columns of the value dimension that one workgroup of the chunked kernel owns: four waves of 16 or 32 (a wave holds
-// dim x 16 or dim x 32 of the state in registers, which bounds the wide form to dim 128).
-static inline int la_value_cols(int dim, int vdim) { return vdim <= 64 || dim > 128 ? 64 : 128; }
+// Columns of the value dimension that one workgroup of the chunked kernel owns: 16 for each of its four or eight waves.
+static inline int la_value_cols(int vdim) { return vdim <= 64 ? 64 : 128; }
 
 // Segments of a portion of up to max_len rows: enough that (sequences x heads x value slices x segments) gives every
 // compute unit two workgroups, but no shorter than kLaMinSegChunks chunks (a segment's start state costs two passes
