@@ -19,6 +19,8 @@ namespace {
 
 typedef __bf16 bf8 __attribute__((ext_vector_type(8)));
 typedef float f4 __attribute__((ext_vector_type(4)));
+typedef uint32_t la_u2 __attribute__((ext_vector_type(2)));
+typedef uint32_t la_u4 __attribute__((ext_vector_type(4)));
 
 struct LaArgs {
     const void *u;  // [rows][ldu]: heads * dim of q, heads * dim of k, heads * vdim of v, anything
@@ -126,7 +128,9 @@ template <typename T, int R> __global__ __launch_bounds__(256) void lightning_re
 // [rows][64 s] for K^T and V^T: eight 16-byte chunks per row, chunk c of row r at position c ^ la_hash(r), so that
 // both the transposing 8-byte writes (rows 4 apart) and the 16-byte operand reads (consecutive rows) spread over the
 // banks without a pad.
-__device__ __forceinline__ int la_hash(int r) { return (r + (r >> 2)) & 7; }
+// (Of the row bits that change over the lanes of an access - 0 to 3 in reads, 2 to 6 in writes - bit 0 picks half of the
+// banks, and three more have to reach all eight chunks.)
+__device__ __forceinline__ int la_hash(int r) { return ((r >> 1) & 7) ^ ((r >> 4) & 1); }
 __device__ __forceinline__ int la_tr(int r, int s) { return r * 64 + ((((s >> 3) ^ la_hash(r)) << 3) | (s & 7)); }
 
 __device__ __forceinline__ f4 la_mfma(bf8 x, bf8 y, f4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, c, 0, 0, 0); }
@@ -137,18 +141,20 @@ __device__ __forceinline__ bf8 la_read44(const __bf16 *p, const __bf16 *q) {
     const bf4 x = *reinterpret_cast<const bf4 *>(p), y = *reinterpret_cast<const bf4 *>(q);
     return bf8{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
 }
-// x = hi + lo, both bf16
-__device__ __forceinline__ void la_split(float x, __bf16 &hi, __bf16 &lo) {
-    hi = (__bf16)x;
-    lo = (__bf16)(x - (float)hi);
+// Pairs x = hi + lo, packed bf16
+__device__ __forceinline__ void la_split2(float x0, float x1, uint32_t &hi, uint32_t &lo) {
+    hi = row_pack_bf16(x0, x1);
+    lo = row_pack_bf16(x0 - __builtin_bit_cast(float, hi << 16), x1 - __builtin_bit_cast(float, hi & 0xffff0000u));
 }
+struct LaSplit {  // eight values as two operands
+    uint32_t hi[4], lo[4];
+    __device__ __forceinline__ bf8 high() const { return __builtin_bit_cast(bf8, la_u4{hi[0], hi[1], hi[2], hi[3]}); }
+    __device__ __forceinline__ bf8 low() const { return __builtin_bit_cast(bf8, la_u4{lo[0], lo[1], lo[2], lo[3]}); }
+};
 
 struct LaBlock {  // four rows of four consecutive columns, raw bf16
     uint2 r[4];
 };
-
-typedef uint32_t la_u2 __attribute__((ext_vector_type(2)));
-typedef uint32_t la_u4 __attribute__((ext_vector_type(4)));
 
 // A tile of `rows` rows of `cols` columns at row stride `ld` as a buffer: loads past its end give zeros, stores past it
 // are dropped.  (Columns past `cols` inside a row are the caller's: it gives such lanes the offset kLaOutside.)
@@ -198,32 +204,33 @@ __device__ __forceinline__ void la_put_block(LaBlock b, int s, int c, __bf16 *rm
 
 constexpr int kLaPitchA = 72;  // bf16 per row of the decayed scores
 
-template <int KD, int NW> constexpr int la_q_elems() {  // Q tile; later the output tile
-    return 64 * (KD + 8) > 64 * (16 * NW + 8) ? 64 * (KD + 8) : 64 * (16 * NW + 8);
-}
-template <int KD> constexpr int la_k_elems() {  // K tile; later the two terms of the decayed scores
-    return 64 * (KD + 8) > 2 * 64 * kLaPitchA ? 64 * (KD + 8) : 2 * 64 * kLaPitchA;
-}
-template <int KD, int NW> constexpr size_t la_lds_bytes() {
-    return (size_t)(la_q_elems<KD, NW>() + la_k_elems<KD>() + KD * 64 + 16 * NW * 64) * 2 + (64 + 64 + 80) * 4;
+// Elements of the tiles: Q and K row-major, the two terms of the decayed scores, the transposed K and V, the output.
+template <int KD> constexpr int la_r_elems() { return 64 * (KD + 8); }
+constexpr int kLaAElems = 2 * 64 * kLaPitchA;
+template <int KD, int NW> constexpr int la_t_elems() { return (KD + 16 * NW) * 64; }
+template <int NW> constexpr int la_o_elems() { return 64 * (16 * NW + 8); }
+template <int KD, int NW, bool STATES> constexpr size_t la_lds_bytes() {
+    const size_t elems = STATES ? 2 * la_t_elems<KD, NW>()  // (double-buffered: one barrier per chunk)
+                                : 2 * la_r_elems<KD>() + kLaAElems + la_t_elems<KD, NW>() + la_o_elems<NW>();
+    return elems * 2 + (64 + 64 + 64 + 80) * 4;
 }
 
 // KD: dim padded to 64, 128 or 256.  NW: waves; each owns 16 value columns.  All products are taken transposed (value
 // columns, or keys, as the rows of the result), so that a lane holds four consecutive elements of one row t.
 // STATES: only the segment's own contribution to the state, to the workspace (first pass over a portion in segments).
 template <int KD, int NW, bool STATES>
-__global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) void lightning_chunk_kernel(const LaArgs a) {
+__global__ __launch_bounds__(64 * NW, 2) void lightning_chunk_kernel(const LaArgs a) {
     constexpr int kCols = 16 * NW, kLdR = KD + 8, kLdO = kCols + 8, kThr = 64 * NW;
     constexpr int kDB = KD / 4, kKBlocks = 16 * kDB, kKPass = (kKBlocks + kThr - 1) / kThr;  // 4x4 blocks of K
     constexpr int kST = NW == 8 ? 2 : 4;  // score tiles per wave
     extern __shared__ __align__(16) char lds[];
-    __bf16 *q_s = reinterpret_cast<__bf16 *>(lds);
-    __bf16 *k_s = q_s + la_q_elems<KD, NW>();
-    __bf16 *kt_s = k_s + la_k_elems<KD>();
-    __bf16 *vt_s = kt_s + KD * 64;
-    float *rev = reinterpret_cast<float *>(vt_s + kCols * 64);  // decay from row s to the chunk's last row
-    float *pw = rev + 128;  // powers 0 .. 64, behind 64 zeros for the keys after a row
-    __bf16 *a_hi = k_s, *a_lo = k_s + 64 * kLaPitchA, *o_s = q_s;
+    float *rev = reinterpret_cast<float *>(lds);  // decay from row s to the last row of a whole chunk ...
+    float *rev_tail = rev + 64;                   // ... and of a portion's last chunk
+    float *pw = rev + 192;                        // powers 0 .. 64, behind 64 zeros for the keys after a row
+    __bf16 *tiles = reinterpret_cast<__bf16 *>(rev + 272);
+    __bf16 *kt_s = tiles, *vt_s = kt_s + KD * 64;
+    __bf16 *q_s = tiles + la_t_elems<KD, NW>(), *k_s = q_s + la_r_elems<KD>(), *a_hi = k_s + la_r_elems<KD>();
+    __bf16 *a_lo = a_hi + 64 * kLaPitchA, *o_s = a_hi + kLaAElems;
 
     const int h = blockIdx.x, seg = blockIdx.y % a.segments, vsl = blockIdx.y / a.segments, b = blockIdx.z;
     Portion p;
@@ -293,7 +300,6 @@ __global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) voi
     for (int r0 = r_beg; r0 < r_end; r0 += kLaChunk) {
         const int nv = r_end - r0 < kLaChunk ? r_end - r0 : kLaChunk;
         int self = tid;
-        asm volatile("" : "+v"(self));  // (LDS addresses are made again per chunk: kept over the loop they would spill)
         const int lane = self & 63, l16 = lane & 15, g = lane >> 4;
 #pragma unroll
         for (int i = 0; i < kKPass; ++i) {
@@ -303,7 +309,7 @@ __global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) voi
             if (!STATES) la_put_block(qb[i], sr, c, q_s, kLdR, nullptr);
         }
         la_put_block(vb, self / (kCols / 4) * 4, self % (kCols / 4) * 4, nullptr, 0, vt_s);
-        if (nv < kLaChunk && tid < 64) rev[tid] = tid < nv ? powers[nv - 1 - tid] : 0.f;
+        if (nv < kLaChunk && tid < 64) rev_tail[tid] = tid < nv ? powers[nv - 1 - tid] : 0.f;
         if (r0 + kLaChunk < r_end) fetch(r0 + kLaChunk);
         __syncthreads();
 
@@ -328,14 +334,11 @@ __global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) voi
             for (int tt = 0; tt < 4; ++tt) o[tt] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int dd = 0; dd < KD / 32; ++dd) {
-                bf8 hi, lo;
+                LaSplit sp;
 #pragma unroll
-                for (int j = 0; j < 8; ++j) {
-                    __bf16 x, y;
-                    la_split(s[2 * dd + j / 4][j % 4], x, y);
-                    hi[j] = x;
-                    lo[j] = y;
-                }
+                for (int j = 0; j < 4; ++j)
+                    la_split2(s[2 * dd + j / 2][2 * j % 4], s[2 * dd + j / 2][2 * j % 4 + 1], sp.hi[j], sp.lo[j]);
+                const bf8 hi = sp.high(), lo = sp.low();
 #pragma unroll
                 for (int tt = 0; tt < 4; ++tt) {
                     const __bf16 *qr = q_s + (16 * tt + l16) * kLdR + 32 * dd + 4 * g;
@@ -343,28 +346,22 @@ __global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) voi
                     o[tt] = la_mfma(hi, bq, o[tt]);
                     o[tt] = la_mfma(lo, bq, o[tt]);
                 }
-                __builtin_amdgcn_sched_barrier(0);
             }
 #pragma unroll
             for (int tt = 0; tt < 4; ++tt)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) o[tt][i] *= pt[tt];
-            __syncthreads();  // Q and K have been read: their space takes the decayed scores (and, later, O)
 #pragma unroll
             for (int m = 0; m < kST; ++m) {
                 const int st = NW == 8 ? 2 * m + (wave & 1) : m;
                 if (st > rt + 1) continue;  // (tile rt + 1 is read as zeros when the last k-step covers it)
                 const int t = 16 * rt + l16, c = 16 * st + 4 * g;
-                float hi[4], lo[4];
-#pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    const float f = sc[m][i] * pw[t - c - i];
-                    const __bf16 x = (__bf16)f;
-                    hi[i] = f;
-                    lo[i] = f - (float)x;
-                }
-                *reinterpret_cast<uint2 *>(a_hi + t * kLaPitchA + c) = make_uint2(row_pack_bf16(hi[0], hi[1]), row_pack_bf16(hi[2], hi[3]));
-                *reinterpret_cast<uint2 *>(a_lo + t * kLaPitchA + c) = make_uint2(row_pack_bf16(lo[0], lo[1]), row_pack_bf16(lo[2], lo[3]));
+                const float *f = pw + t - c;
+                uint2 hi, lo;
+                la_split2(sc[m][0] * f[0], sc[m][1] * f[-1], hi.x, lo.x);
+                la_split2(sc[m][2] * f[-2], sc[m][3] * f[-3], hi.y, lo.y);
+                *reinterpret_cast<uint2 *>(a_hi + t * kLaPitchA + c) = hi;
+                *reinterpret_cast<uint2 *>(a_lo + t * kLaPitchA + c) = lo;
             }
             __syncthreads();
 #pragma unroll
@@ -377,28 +374,29 @@ __global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) voi
                 }
             }
 #pragma unroll
-            for (int tt = 0; tt < 4; ++tt)  // to LDS (where Q was), so that rows are stored 16 bytes per lane
+            for (int tt = 0; tt < 4; ++tt)  // to LDS, so that rows are stored 16 bytes per lane
                 *reinterpret_cast<uint2 *>(o_s + (16 * tt + l16) * kLdO + vw + 4 * g) =
                     make_uint2(row_pack_bf16(o[tt][0], o[tt][1]), row_pack_bf16(o[tt][2], o[tt][3]));
         }
         // S <- decay^nv S + K^T (decay^(nv-1-s) V)
         const float whole = pw[nv];
+        const float *wt = nv < kLaChunk ? rev_tail : rev;
 #pragma unroll
         for (int dt = 0; dt < KD / 16; ++dt)
 #pragma unroll
             for (int i = 0; i < 4; ++i) s[dt][i] *= whole;
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
-            bf8 hi, lo;
-            const bf8 bv = la_read8(vt_s + la_tr(vw + l16, 32 * kk + 8 * g));
-            const f4 w0 = *reinterpret_cast<const f4 *>(rev + 32 * kk + 8 * g), w1 = *reinterpret_cast<const f4 *>(rev + 32 * kk + 8 * g + 4);
+            LaSplit sp;
+            const la_u4 bv = *reinterpret_cast<const la_u4 *>(vt_s + la_tr(vw + l16, 32 * kk + 8 * g));
+            const f4 w0 = *reinterpret_cast<const f4 *>(wt + 32 * kk + 8 * g), w1 = *reinterpret_cast<const f4 *>(wt + 32 * kk + 8 * g + 4);
 #pragma unroll
-            for (int j = 0; j < 8; ++j) {
-                __bf16 x, y;
-                la_split((float)bv[j] * (j < 4 ? w0[j % 4] : w1[j % 4]), x, y);
-                hi[j] = x;
-                lo[j] = y;
+            for (int j = 0; j < 4; ++j) {
+                const uint32_t pair = bv[j];
+                la_split2(__builtin_bit_cast(float, pair << 16) * (j < 2 ? w0 : w1)[2 * j % 4],
+                          __builtin_bit_cast(float, pair & 0xffff0000u) * (j < 2 ? w0 : w1)[2 * j % 4 + 1], sp.hi[j], sp.lo[j]);
             }
+            const bf8 hi = sp.high(), lo = sp.low();
 #pragma unroll
             for (int dt = 0; dt < KD / 16; ++dt) {
                 const bf8 ak = la_read8(kt_s + la_tr(16 * dt + l16, 32 * kk + 8 * g));
@@ -417,8 +415,12 @@ __global__ __launch_bounds__(64 * NW, KD * (NW == 8 ? 1 : 2) <= 128 ? 4 : 2) voi
                 const la_u4 x = *reinterpret_cast<const la_u4 *>(o_s + t * kLdO + c);
                 __builtin_amdgcn_raw_buffer_store_b128(x, dst, c < vcols ? (uint32_t)(t * ldo + c) * 2u : kLaOutside, 0, 0);
             }
+            // (the next chunk's tiles may be written now: their readers are past the barrier above, and its scores and
+            // output come behind barriers of its own)
+        } else {  // the other half of the tiles
+            kt_s = kt_s == tiles ? tiles + la_t_elems<KD, NW>() : tiles;
+            vt_s = kt_s + KD * 64;
         }
-        __syncthreads();
     }
     float *to = STATES ? seg_state : (a.segments > 1 ? nullptr : pool);
     if (!to) return;
@@ -483,13 +485,13 @@ template <typename K> int la_big_lds(K kernel, size_t bytes, const char *what) {
 }
 
 template <int KD, int NW> int launch_chunks(const LaArgs &a, int batch, hipStream_t s) {
-    constexpr size_t lds = la_lds_bytes<KD, NW>();
-    static_assert(lds <= 160 * 1024, "LDS of one compute unit");
+    constexpr size_t lds = la_lds_bytes<KD, NW, false>(), lds_states = la_lds_bytes<KD, NW, true>();
+    static_assert(lds <= 160 * 1024 && lds_states <= 160 * 1024, "LDS of one compute unit");
     const int slices = (a.vdim + 16 * NW - 1) / (16 * NW);
     const dim3 grid((unsigned)a.heads, (unsigned)(slices * a.segments), (unsigned)batch), block(64 * NW);
     if (a.segments > 1) {
-        if (int rc = la_big_lds(lightning_chunk_kernel<KD, NW, true>, lds, "pa_lightning_chunked")) return rc;
-        lightning_chunk_kernel<KD, NW, true><<<grid, block, lds, s>>>(a);
+        if (int rc = la_big_lds(lightning_chunk_kernel<KD, NW, true>, lds_states, "pa_lightning_chunked")) return rc;
+        lightning_chunk_kernel<KD, NW, true><<<grid, block, lds_states, s>>>(a);
         const unsigned gx = (unsigned)(((int64_t)a.dp * a.vp / 4 + 255) / 256);
         lightning_scan_kernel<<<dim3(gx, (unsigned)a.heads, (unsigned)batch), dim3(256), 0, s>>>(a);
     }

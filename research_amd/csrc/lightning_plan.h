@@ -13,14 +13,13 @@ static inline int la_pad16(int n) { return (n + 15) / 16 * 16; }
 // Columns of the value dimension that one workgroup of the chunked kernel owns: 16 for each of its four or eight waves.
 static inline int la_value_cols(int vdim) { return vdim <= 64 ? 64 : 128; }
 
-// Segments of a portion of up to max_len rows: enough that (sequences x heads x value slices x segments) gives every
-// compute unit two workgroups, but no shorter than kLaMinSegChunks chunks (a segment's start state costs two passes
-// over a state's bytes and a second reading of its keys and values).
+// Segments of a portion of up to max_len rows: as many as (sequences x heads x value slices) leave compute units for,
+// one workgroup each, but no shorter than kLaMinSegChunks chunks (a segment's start state costs a second reading of
+// its keys and values and two passes over a state's bytes).
 static inline int la_segments(int64_t workgroups, int cus, int max_len) {
     if (workgroups <= 0 || max_len <= 0) return 1;
     const int64_t chunks = (max_len + kLaChunk - 1) / kLaChunk;
-    int64_t want = (2 * (int64_t)cus + workgroups - 1) / workgroups;
-    if (workgroups >= cus) want = 1;
+    int64_t want = cus / workgroups;
     const int64_t most = chunks / kLaMinSegChunks;
     if (want > most) want = most;
     if (want > kLaMaxSegments) want = kLaMaxSegments;
