@@ -29,6 +29,7 @@ scheduler a made-up block count (engine.py:147) and ``flush_cache`` is empty
 
 from __future__ import annotations
 
+import os
 from typing import Dict, List, Optional, Tuple
 
 import numpy as np
@@ -170,10 +171,13 @@ class InferenceEngine:
 
     @staticmethod
     def _load_tokenizer(model_path: str):
+        names = os.listdir(model_path) if os.path.isdir(model_path) else []
+        if not any(n.startswith("tokenizer") or n in ("vocab.json", "spiece.model") for n in names):
+            return None  # token-id prompts still work
         try:
             from transformers import AutoTokenizer
             return AutoTokenizer.from_pretrained(model_path, local_files_only=True)
-        except Exception:  # no tokenizer files: token-id prompts still work
+        except Exception:  # files that are no tokenizer
             return None
 
     def _new_cache(self):

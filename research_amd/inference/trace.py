@@ -49,7 +49,7 @@ def replay(engine, lines, out_dir: str, report: TextIO) -> None:
         if not line.strip():
             continue
         step = json.loads(line)
-        entries = step["entries"]
+        entries = [e for e in step["entries"] if e["tokens"]]
         batch = []
         for e in entries:
             if e["id"] not in live:

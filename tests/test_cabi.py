@@ -224,3 +224,54 @@ def test_generated_prefill_loop_is_current(tmp_path, script, generated):
     out = tmp_path / "loop.inc"
     subprocess.run([sys.executable, os.path.join(csrc, script), str(out)], check=True, stdout=subprocess.DEVNULL)
     assert out.read_text() == open(os.path.join(csrc, generated)).read()
+
+
+def test_block_entry_points_check_their_arguments():
+    """The kernels around attention in hybrid blocks: rejected before any device call."""
+    f32, bf16 = _lib.PA_F32, _lib.PA_BF16
+    residual = lambda **kw: [{**dict(x=FAKE, y=FAKE, yw=None, ye=0.0, ids=None, table=None, tr=0, ri=None, xr=4, w=FAKE, b=FAKE,
+                                     eps=1e-6, norm=_lib.PA_NORM_LAYER, out=FAKE, rows=4, width=64, dt=bf16, s=None), **kw}[k]
+                             for k in ("x", "y", "yw", "ye", "ids", "table", "tr", "ri", "xr", "w", "b", "eps", "norm", "out",
+                                       "rows", "width", "dt", "s")]
+    for kw, status, text in ((dict(x=None), -1, "neither"), (dict(norm=7), -1, "norm=7"), (dict(width=20000), -2, "above"),
+                             (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(ids=FAKE), -1, "table"), (dict(ri=FAKE), -1, "row_index"),
+                             (dict(y=None, out=None), -1, "nothing"), (dict(y=None, yw=FAKE), -1, "y_weight"),
+                             (dict(norm=_lib.PA_NORM_NONE), -1, "without a norm")):
+        rc, msg = _status("pa_residual_norm", *residual(**kw))
+        assert rc == status and text in msg, (kw, msg)
+    assert _status("pa_residual_norm", *residual(rows=0, x=None))[0] == 0
+    rc, msg = _status("pa_rms_gate", FAKE, FAKE, 60, FAKE, 1e-6, FAKE, 4, 64, f32, None)
+    assert rc == -1 and "gate_stride" in msg
+    rc, msg = _status("pa_glu", FAKE, 64, FAKE, 64, None, 0, FAKE, 4, 64, 9, f32, None)
+    assert rc == -1 and "act" in msg
+    rc, msg = _status("pa_head_gate", FAKE, FAKE, 4, FAKE, 4, 4, 16, 24, f32, None)
+    assert rc == -1 and "sizes" in msg
+
+    qkv = lambda **kw: [{**dict(u=FAKE, ld=200, n=4, cw=FAKE, taps=3, cs=FAKE, sr=2, rope=FAKE, rr=9, rot=8, cl=FAKE, ql=None,
+                                qs=None, ss=FAKE, tiles=None, nt=4, batch=4, slots=FAKE, ts=64, q=FAKE, k=FAKE, v=FAKE, vf=None,
+                                lam=None, vm=0, hq=4, hkv=2, dim=16, vdim=24, d=24, un=1, eps=1e-6, qsc=1.0, dt=bf16, s=None),
+                           **kw}[k] for k in ("u", "ld", "n", "cw", "taps", "cs", "sr", "rope", "rr", "rot", "cl", "ql", "qs", "ss",
+                                              "tiles", "nt", "batch", "slots", "ts", "q", "k", "v", "vf", "lam", "vm", "hq", "hkv",
+                                              "dim", "vdim", "d", "un", "eps", "qsc", "dt", "s")]
+    for kw, status, text in ((dict(hkv=3), -1, "multiple"), (dict(d=20), -1, "pool_dim"), (dict(rot=9), -1, "rot_dims"),
+                             (dict(taps=9), -2, "taps"), (dict(cw=None), -1, "convolution"), (dict(cs=None), -1, "carried"),
+                             (dict(rope=None), -1, "table"), (dict(vm=2, vf=FAKE), -1, "v_lambda"), (dict(vm=1), -1, "v_first"),
+                             (dict(nt=3), -1, "one row"), (dict(ld=100), -1, "u_stride"), (dict(tiles=FAKE), -1, "tiles"),
+                             (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(d=264), -2, "above 256")):
+        rc, msg = _status("pa_qkv_conv_append", *qkv(**kw))
+        assert rc == status and text in msg, (kw, msg)
+    assert _status("pa_qkv_conv_append", *qkv(n=0, u=None, batch=0, nt=0))[0] == 0
+
+    lib = _lib.load()
+    assert lib.pa_lightning_state_floats(20, 40) == 32 * 48
+    chunked = lambda **kw: [{**dict(u=FAKE, ld=200, n=4, st=FAKE, sr=2, dp=FAKE, cl=FAKE, ql=FAKE, qs=FAKE, ss=FAKE, batch=2, mq=4,
+                                    out=FAKE, h=2, dim=16, vdim=24, dt=bf16, ws=None, wb=0, s=None), **kw}[k]
+                            for k in ("u", "ld", "n", "st", "sr", "dp", "cl", "ql", "qs", "ss", "batch", "mq", "out", "h", "dim",
+                                      "vdim", "dt", "ws", "wb", "s")]
+    for kw, status, text in ((dict(dt=f32), -2, "BF16"), (dict(dim=300, ld=2000), -2, "above 256"), (dict(ld=100), -1, "u_stride"),
+                             (dict(qs=None), -1, "together"), (dict(st=None), -1, "NULL"), (dict(mq=-1), -1, "max_q_len")):
+        rc, msg = _status("pa_lightning_chunked", *chunked(**kw))
+        assert rc == status and text in msg, (kw, msg)
+    rc, msg = _status("pa_lightning_recurrent", FAKE, 200, 1, FAKE, 2, FAKE, FAKE, None, None, FAKE, 2, FAKE, 2, 16, 24, f32, None)
+    assert rc == -1 and "below batch" in msg
+    assert lib.pa_lightning_workspace_bytes(-1, 2, 16, 24, 8) == 0 and "pa_lightning_workspace_bytes" in _lib.last_error()
