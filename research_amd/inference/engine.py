@@ -142,7 +142,7 @@ class InferenceEngine:
         if limit is not None and config.max_model_len > limit:
             # the rotary tables end at max_position_embeddings; later positions would all take the last row
             raise ValueError(f"max_model_len={config.max_model_len} exceeds the model's "
-                             f"{limit} positions")
+                             f"max_position_embeddings={limit}")
         self.tokenizer = tokenizer if tokenizer is not None else self._load_tokenizer(config.model_path)
         budget = config.max_batch_size * 512  # as the reference (engine.py:50)
         portion = 0
