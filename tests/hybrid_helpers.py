@@ -116,7 +116,7 @@ def logit_error(got, want):
 
 def bf16_tolerance(forward, cfg, w, tokens, want, runs=3):
     """Per position, what rounding to bf16 may do to the logits: four times what noise of bf16's size on every weight does
-    to the checker's, and never less than 0.03 (some positions are ill-conditioned: a normed sum that nearly cancels, two
+    to the oracle's, and never less than 0.03 (some positions are ill-conditioned: a normed sum that nearly cancels, two
     keys that nearly tie)."""
     g = torch.Generator().manual_seed(5)
     worst = torch.full((len(tokens),), 0.0075, dtype=torch.float64)

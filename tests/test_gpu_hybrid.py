@@ -1,4 +1,4 @@
-"""Hybrid decoders on the GPU, loaded from a checkpoint folder and run by the engine, against the checker's forward:
+"""Hybrid decoders on the GPU, loaded from a checkpoint folder and run by the engine, against the oracle's forward:
 whole prompts, portions, single tokens, mixed batches with blocks and slots used again, and generation."""
 
 import io
@@ -38,7 +38,7 @@ def _engine(path, dtype, blocks=40, slots=4, max_len=640, **kw):
 
 
 class Wanted:
-    """The checker's logits of one sequence, and how far from them each position may be."""
+    """The oracle's logits of one sequence, and how far from them each position may be."""
 
     def __init__(self, cfg, w, tokens, dtype):
         with torch.no_grad():
@@ -155,7 +155,7 @@ def _by_prompt(samples):
 @pytest.mark.parametrize("name,kw", [("plain", {}), ("plain", {"use_graphs": True}), ("odd", {"prefill_portion": 7}),
                                      ("no-mixing", {"use_graphs": True, "prefill_portion": 20})])
 def test_greedy_generation_through_the_scheduler(folders, name, kw):
-    """Long greedy decoding of ragged prompts by ``generate``: the tokens are the checker's argmax at every position,
+    """Long greedy decoding of ragged prompts by ``generate``: the tokens are the oracle's argmax at every position,
     the log probabilities its own; graphs are replayed between eager prefills."""
     announce(f"hybrid generate {name} {kw}")
     path, cfg, w = folders(name)

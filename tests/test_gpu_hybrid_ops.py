@@ -1,4 +1,4 @@
-"""The kernels around attention in hybrid blocks, each against a plain float32 statement or the checker: residual sums
+"""The kernels around attention in hybrid blocks, each against a plain float32 statement or the oracle: residual sums
 and norms, gates, the joint q/k/v step with its carried rows, and packed attention at the edges of windows and pages."""
 
 import numpy as np

@@ -1,4 +1,4 @@
-"""Lightning attention on the GPU against the checker's token-by-token recurrence: outputs and carried states, whole
+"""Lightning attention on the GPU against the oracle's token-by-token recurrence: outputs and carried states, whole
 sequences, portions of any length, unequal batches, slots used again, and long portions cut into segments."""
 
 import numpy as np
@@ -24,7 +24,7 @@ def _powers(decay):
 
 
 class Case:
-    """Random projection rows ``[q | k | v | gate]`` of some sequences and the checker's outputs and states."""
+    """Random projection rows ``[q | k | v | gate]`` of some sequences and the oracle's outputs and states."""
 
     def __init__(self, lens, heads, dim, vdim, decay, dtype, seed=0):
         g = torch.Generator().manual_seed(seed)

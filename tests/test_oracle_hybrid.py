@@ -1,4 +1,4 @@
-"""The checker's statement of the hybrid mechanisms against independent routes (CPU only), and what a planted mistake
+"""The oracle's statement of the hybrid mechanisms against independent routes (CPU only), and what a planted mistake
 does to its logits: more than the tolerance of the tests that compare the GPU with it."""
 
 import copy
