@@ -192,14 +192,12 @@ __device__ __forceinline__ void la_put_block(LaBlock b, int s, int c, __bf16 *rm
     }
     if (!tr) return;
     // columns 0/1 and 2/3 of rows 0..3 as pairs over rows (v_perm picks the low or the high halves)
-    const uint32_t lo01 = __builtin_amdgcn_perm(b.r[1].x, b.r[0].x, 0x05040100u), hi01 = __builtin_amdgcn_perm(b.r[1].x, b.r[0].x, 0x07060302u);
-    const uint32_t lo23 = __builtin_amdgcn_perm(b.r[3].x, b.r[2].x, 0x05040100u), hi23 = __builtin_amdgcn_perm(b.r[3].x, b.r[2].x, 0x07060302u);
-    const uint32_t lo01b = __builtin_amdgcn_perm(b.r[1].y, b.r[0].y, 0x05040100u), hi01b = __builtin_amdgcn_perm(b.r[1].y, b.r[0].y, 0x07060302u);
-    const uint32_t lo23b = __builtin_amdgcn_perm(b.r[3].y, b.r[2].y, 0x05040100u), hi23b = __builtin_amdgcn_perm(b.r[3].y, b.r[2].y, 0x07060302u);
-    *reinterpret_cast<uint2 *>(tr + la_tr(c, s)) = make_uint2(lo01, lo23);
-    *reinterpret_cast<uint2 *>(tr + la_tr(c + 1, s)) = make_uint2(hi01, hi23);
-    *reinterpret_cast<uint2 *>(tr + la_tr(c + 2, s)) = make_uint2(lo01b, lo23b);
-    *reinterpret_cast<uint2 *>(tr + la_tr(c + 3, s)) = make_uint2(hi01b, hi23b);
+    auto low = [](uint32_t x, uint32_t y) { return __builtin_amdgcn_perm(y, x, 0x05040100u); };
+    auto high = [](uint32_t x, uint32_t y) { return __builtin_amdgcn_perm(y, x, 0x07060302u); };
+    *reinterpret_cast<uint2 *>(tr + la_tr(c, s)) = make_uint2(low(b.r[0].x, b.r[1].x), low(b.r[2].x, b.r[3].x));
+    *reinterpret_cast<uint2 *>(tr + la_tr(c + 1, s)) = make_uint2(high(b.r[0].x, b.r[1].x), high(b.r[2].x, b.r[3].x));
+    *reinterpret_cast<uint2 *>(tr + la_tr(c + 2, s)) = make_uint2(low(b.r[0].y, b.r[1].y), low(b.r[2].y, b.r[3].y));
+    *reinterpret_cast<uint2 *>(tr + la_tr(c + 3, s)) = make_uint2(high(b.r[0].y, b.r[1].y), high(b.r[2].y, b.r[3].y));
 }
 
 constexpr int kLaPitchA = 72;  // bf16 per row of the decayed scores
@@ -245,10 +243,10 @@ __global__ __launch_bounds__(64 * NW, 2) void lightning_chunk_kernel(const LaArg
         rev[tid] = powers[63 - tid];
         pw[tid - 64] = 0.f;
     }
-    const int lane0 = tid & 63;
+    const int l16 = tid & 15, g = (tid & 63) >> 4;
     float pt[4];  // decay from the chunk's start to row 16 tt + l16
 #pragma unroll
-    for (int tt = 0; tt < 4; ++tt) pt[tt] = powers[16 * tt + (lane0 & 15) + 1];
+    for (int tt = 0; tt < 4; ++tt) pt[tt] = powers[16 * tt + l16 + 1];
 
     // The state slice of this wave: tile dt holds d = 16 dt + 4 g + i, v = v0 + vw + l16
     f4 s[KD / 16];
@@ -258,8 +256,8 @@ __global__ __launch_bounds__(64 * NW, 2) void lightning_chunk_kernel(const LaArg
     const float *from = STATES ? nullptr : (a.segments > 1 ? seg_state : (p.pos0 > 0 ? pool : nullptr));
     // (a state as a buffer: rows past dp lie past its end, columns past vp get an offset outside)
     const int state_bytes = (int)state_elems * 4;
-    const int v = v0 + vw + (lane0 & 15);
-    const uint32_t soff = v < a.vp ? (uint32_t)(4 * (lane0 >> 4) * a.vp + v) * 4u : kLaOutside;
+    const int v = v0 + vw + l16;
+    const uint32_t soff = v < a.vp ? (uint32_t)(4 * g * a.vp + v) * 4u : kLaOutside;
     {
         const __amdgpu_buffer_rsrc_t src = __builtin_amdgcn_make_buffer_rsrc(
             (void *)(from ? from : a.state), 0, from ? state_bytes : 0, 0x00020000);  // (no state: every load is past the end)
@@ -299,16 +297,14 @@ __global__ __launch_bounds__(64 * NW, 2) void lightning_chunk_kernel(const LaArg
     fetch(r_beg);
     for (int r0 = r_beg; r0 < r_end; r0 += kLaChunk) {
         const int nv = r_end - r0 < kLaChunk ? r_end - r0 : kLaChunk;
-        int self = tid;
-        const int lane = self & 63, l16 = lane & 15, g = lane >> 4;
 #pragma unroll
         for (int i = 0; i < kKPass; ++i) {
-            const int blk = self + kThr * i, c = blk % kDB * 4, sr = blk / kDB * 4;
+            const int blk = tid + kThr * i, c = blk % kDB * 4, sr = blk / kDB * 4;
             if (kKBlocks % kThr != 0 && blk >= kKBlocks) continue;
             la_put_block(kb[i], sr, c, STATES ? nullptr : k_s, kLdR, kt_s);
             if (!STATES) la_put_block(qb[i], sr, c, q_s, kLdR, nullptr);
         }
-        la_put_block(vb, self / (kCols / 4) * 4, self % (kCols / 4) * 4, nullptr, 0, vt_s);
+        la_put_block(vb, tid / (kCols / 4) * 4, tid % (kCols / 4) * 4, nullptr, 0, vt_s);
         if (nv < kLaChunk && tid < 64) rev_tail[tid] = tid < nv ? powers[nv - 1 - tid] : 0.f;
         if (r0 + kLaChunk < r_end) fetch(r0 + kLaChunk);
         __syncthreads();
@@ -389,7 +385,8 @@ __global__ __launch_bounds__(64 * NW, 2) void lightning_chunk_kernel(const LaArg
         for (int kk = 0; kk < 2; ++kk) {
             LaSplit sp;
             const la_u4 bv = *reinterpret_cast<const la_u4 *>(vt_s + la_tr(vw + l16, 32 * kk + 8 * g));
-            const f4 w0 = *reinterpret_cast<const f4 *>(wt + 32 * kk + 8 * g), w1 = *reinterpret_cast<const f4 *>(wt + 32 * kk + 8 * g + 4);
+            const f4 w0 = *reinterpret_cast<const f4 *>(wt + 32 * kk + 8 * g);
+            const f4 w1 = *reinterpret_cast<const f4 *>(wt + 32 * kk + 8 * g + 4);
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 const uint32_t pair = bv[j];
@@ -407,11 +404,11 @@ __global__ __launch_bounds__(64 * NW, 2) void lightning_chunk_kernel(const LaArg
         if constexpr (!STATES) {
             __syncthreads();
             const int ldo = a.heads * a.vdim;
-            const __amdgpu_buffer_rsrc_t dst = la_tile(reinterpret_cast<const uint16_t *>(a.out) + (p.row0 + r0) * (int64_t)ldo + h * a.vdim + v0,
-                                                       ldo, nv, vcols);
+            const uint16_t *first = reinterpret_cast<const uint16_t *>(a.out) + (p.row0 + r0) * (int64_t)ldo + h * a.vdim + v0;
+            const __amdgpu_buffer_rsrc_t dst = la_tile(first, ldo, nv, vcols);
 #pragma unroll
             for (int i = 0; i < 2; ++i) {  // (64 rows of kCols columns are two 16-byte vectors per thread)
-                const int vec = self + kThr * i, t = vec / (kCols / 8), c = vec % (kCols / 8) * 8;
+                const int vec = tid + kThr * i, t = vec / (kCols / 8), c = vec % (kCols / 8) * 8;
                 const la_u4 x = *reinterpret_cast<const la_u4 *>(o_s + t * kLdO + c);
                 __builtin_amdgcn_raw_buffer_store_b128(x, dst, c < vcols ? (uint32_t)(t * ldo + c) * 2u : kLaOutside, 0, 0);
             }
