@@ -45,7 +45,7 @@ extern "C" {
 #define PA_F16 2
 #define PA_FP8_E4M3 3 /* OCP e4m3fn, KV pool only; q/out stay 16- or 32-bit */
 
-/* Library ABI version (bumped when an entry point is added or a signature or contract changes; now 7). */
+/* Library ABI version (bumped when an entry point is added or a signature or contract changes; now 8). */
 int pa_version(void);
 
 /* Text of the calling thread's most recent error; "" if none. */
@@ -133,7 +133,9 @@ int pa_decode_passes(int batch, int num_q_heads, int num_kv_heads, int head_dim,
  *                   zero-pads ragged batches to the longest sequence without a
  *                   mask (:253-264, :227-229); passing max_len - seq_lens[b]
  *                   reproduces it.
- *   window        : 0, or a sliding window: only the last `window` keys of each sequence are attended
+ *   window        : 0; negative: chunks of -window positions counted from the sequence's start, of which a query sees
+ *                   its own (keys j <= p of the same chunk; no counterpart in the reference); or positive, a
+ *                   sliding window: only the last `window` keys of each sequence are attended
  *                   (j >= seq_lens[b] - window), the rule of the reference's causal_sliding_window_mask
  *                   (attention/mask.py:83-89: q_idx - kv_idx < window_size) for the query at position
  *                   seq_lens[b]-1; blocks wholly before the window are never read.  The reference's own
@@ -212,7 +214,7 @@ int pa_decode_static(const void *q, const void *k_cache, const void *v_cache, vo
  *              memory keep their length); PA_F32 runs on the vector kernel
  *   ctx_lens, q_lens, q_starts : int32[batch]
  *   max_q_len: upper bound of q_lens (grid sizing)
- *   window   : 0, or the sliding window of CacheConfig.sliding_window (attention/config.py:31): row i at
+ *   window   : 0; negative: chunks of -window positions, as in pa_decode; or the sliding window of CacheConfig.sliding_window (attention/config.py:31): row i at
  *              position p = ctx_lens[b] - q_lens[b] + i attends keys p - window < j <= p
  *              (attention/mask.py:83-89); tiles wholly before the window of a workgroup's rows are not loaded.
  *   row_first_key : NULL, or int32[total_q] indexed like the rows of q: the first key position (in the
@@ -398,29 +400,47 @@ int pa_dequantize_blocks_e4m3(const void *cache, const float *scale, const int32
 #define PA_NORM_RMS 2
 #define PA_ACT_SILU 0
 #define PA_ACT_GELU_TANH 1
+#define PA_ACT_NONE 2
+#define PA_GATE_SIGMOID_LAST 0 /* norm, then sigmoid(gate) */
+#define PA_GATE_SILU_FIRST 1   /* silu(gate), then norm */
+#define PA_GL_SSD 0            /* recurrences of pa_gated_linear */
+#define PA_GL_MLSTM 1
 #define PA_V_PLAIN 0 /* values as they are */
 #define PA_V_FIRST 1 /* values as they are, also written to v_first */
 #define PA_V_MIX 2   /* (1 - lambda) value + lambda v_first */
-#define PA_QKV_TILE_ROWS 16 /* rows of a sequence's portion per tile of pa_qkv_conv_append */
+#define PA_QKV_TILE_ROWS 16 /* rows of a sequence's portion per tile of pa_qkv_conv_append and pa_short_conv */
 
 /*
  * Residual sum and norm of one row at a time:
- *     x = table[ids[row]]                           when ids is given, else x[row]
+ *     x = table[ids[row]] * table_scale             when ids is given, else x[row]
+ *     x += pos_table[positions[row]]                when positions is given (with ids)
  *     x += y                                        when y is given; with y_weight, y / rms(y) * y_weight
  *     out = norm(x) * norm_weight + norm_bias       PA_NORM_LAYER or PA_NORM_RMS; PA_NORM_NONE: x in dtype
  * where rms(v) = sqrt(mean(v^2) + eps) and the layer norm divides by sqrt(variance + eps) with the variance as the
  * mean squared deviation.  x is written back when ids or y is given.  With row_index the call only reads: output
  * row r comes from residual row row_index[r] (< x_rows).  Ids and indices out of range read as zero rows.
- *   x : float[rows][width];  y, table, out : dtype;  weights and bias : float[width] or NULL;  width <= 16384
+ * With mix_weight (float[rows][mix + 1]) y is a weighted sum of rows, taken in 32-bit: sum over i < mix of
+ * mix_weight[row][i] y[row * mix + i], plus mix_weight[row][mix] y_extra[row] when y_extra is given.
+ *   x : float[rows][width];  y, y_extra, table, pos_table, out : dtype;  weights and bias : float[width] or NULL;  width <= 16384
  */
-int pa_residual_norm(float *x, const void *y, const float *y_weight, float y_eps, const int64_t *ids,
-                     const void *table, int64_t table_rows, const int64_t *row_index, int64_t x_rows,
+int pa_residual_norm(float *x, const void *y, const float *mix_weight, int mix, const void *y_extra,
+                     const float *y_weight, float y_eps, const int64_t *ids, const void *table, int64_t table_rows,
+                     float table_scale, const int64_t *positions, const void *pos_table, int64_t pos_rows,
+                     const int64_t *row_index, int64_t x_rows,
                      const float *norm_weight, const float *norm_bias, float eps, int norm, void *out,
                      int64_t rows, int width, int dtype, void *stream);
 
-/* out = o / rms(o) * weight * sigmoid(gate), per row over its whole width; gate rows are gate_stride elements apart. */
+/*
+ * A gated RMS norm of each of `groups` equal parts of a row:
+ *     PA_GATE_SIGMOID_LAST   out = o / rms(o) * weight * sigmoid(gate)
+ *     PA_GATE_SILU_FIRST     z = o * silu(gate), out = z / rms(z) * weight
+ * gate and out rows are gate_stride and out_stride elements apart; weight : float[width].
+ */
 int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride, const float *weight, float eps, void *out,
-                int64_t rows, int width, int dtype, void *stream);
+                int64_t out_stride, int64_t rows, int width, int groups, int gate_mode, int dtype, void *stream);
+
+/* out = cap * tanh(x / cap), n elements of dtype to float. */
+int pa_softcap(const void *x, float *out, int64_t n, float cap, int dtype, void *stream);
 
 /*
  * out = act(gate) * up, rows of `width` elements at strides of their own.  With ids, row r's factor is row ids[r] of
@@ -430,16 +450,18 @@ int pa_glu(const void *gate, int64_t gate_stride, const void *up, int64_t up_str
            int64_t up_rows, void *out, int64_t rows, int width, int act, int dtype, void *stream);
 
 /*
- * out[row][h][0:vdim] = o[row][h][0:vdim] * sigmoid(gate[row][h]): the gate of each head behind attention, and the
- * step from attention's padded rows (d) to packed ones (vdim).  gate NULL: the packing alone.
+ * out[row][h][0:vdim] = scale * o[row][h][0:vdim] * sigmoid(gate[row][h]): the gate of each head behind attention, and the
+ * step from attention's padded rows (d) to packed ones (vdim), out_stride elements apart.  gate NULL: without it.
  */
-int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, void *out, int64_t rows, int heads, int d,
-                 int vdim, int dtype, void *stream);
+int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, float scale, void *out, int64_t out_stride,
+                 int64_t rows, int heads, int d, int vdim, int dtype, void *stream);
 
 /*
  * From joint projections to attention's operands: row = [q heads | k heads | v heads | anything].
  *   1. causal convolution over time per channel: y_t = sum_j w[j] u_(t - taps + 1 + j), the rows before a portion from
  *      conv_state (the last taps - 1 projected rows of the sequence, updated by the call);
+ *      then, with q_norm and k_norm (float[dim]), q and k divided by sqrt(mean over dim of the square + eps) and times
+ *      these weights;
  *   2. q, k: the pair (2i, 2i+1) of the first rot_dims dimensions turns by the angle whose (cos, sin) is
  *      rope[position][i];
  *   3. q, k: with unit_norm, divided by sqrt(mean over dim of the square + eps); q also times q_scale;
@@ -458,9 +480,9 @@ int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_rows, const fl
                        const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
                        const int32_t *state_slots, const int32_t *tiles, int n_tiles, int batch,
                        const int64_t *slots, int64_t total_slots, void *q_out, void *k_cache, void *v_cache,
-                       void *v_first, const float *v_lambda, int v_mode, int num_q_heads, int num_kv_heads,
-                       int dim, int vdim, int pool_dim, int unit_norm, float eps, float q_scale, int dtype,
-                       void *stream);
+                       void *v_first, const float *v_lambda, int v_mode, const float *q_norm, const float *k_norm,
+                       int num_q_heads, int num_kv_heads, int dim, int vdim, int pool_dim, int unit_norm, float eps,
+                       float q_scale, int dtype, void *stream);
 
 /*
  * Lightning attention: per head S_t = decay S_(t-1) + k_t v_t^T and o_t = S_t^T q_t, with q, k and v the silu of a
@@ -486,6 +508,66 @@ int pa_lightning_chunked(const void *u, int64_t u_stride, int64_t n_rows, float 
                          const int32_t *q_starts, const int32_t *state_slots, int batch, int max_q_len,
                          void *out, int num_heads, int dim, int vdim, int dtype, void *workspace,
                          size_t workspace_bytes, void *stream);
+
+/*
+ * A causal convolution over time per channel, y_t = act(bias + sum_j w[j] u_(t - taps + 1 + j)), with the rows before a
+ * portion from conv_state (the last taps - 1 input rows of the sequence, updated by the call).
+ *   weight : float[taps][channels], bias : float[channels] or NULL;  taps <= 8;  act : PA_ACT_NONE or PA_ACT_SILU
+ *   conv_state, tiles, n_tiles : as in pa_qkv_conv_append;  out : [n_rows][channels]
+ */
+int pa_short_conv(const void *u, int64_t u_stride, int64_t n_rows, const float *weight, const float *bias, int taps,
+                  int act, void *conv_state, int64_t state_rows, const int32_t *ctx_lens, const int32_t *q_lens,
+                  const int32_t *q_starts, const int32_t *state_slots, const int32_t *tiles, int n_tiles, int batch,
+                  void *out, int channels, int dtype, void *stream);
+
+/*
+ * Linear recurrences with a decay and an input weight per token and head.  Per head (q and k of head h are those of
+ * group h / heads_per_group):
+ *   PA_GL_SSD    dt = softplus(gate_a + head_a);  S_t = exp(-head_b dt) S_(t-1) + dt k_t v_t^T;
+ *                o_t = S_t^T q_t + head_c v_t                          (Mamba-2: q = C, k = B, v = x, head_b = exp(A_log))
+ *   PA_GL_MLSTM  i = cap tanh((gate_a + head_a) / cap);  f = logsigmoid(cap tanh((gate_b + head_b) / cap));
+ *                m_t = max(f + m_(t-1), i), m_0 = 0;  S_t = exp(f + m_(t-1) - m_t) S_(t-1) + exp(i - m_t) k_t v_t^T;
+ *                n_t likewise with k alone;  o_t = q_scale S_t^T q_t / (max(|q_scale n_t . q_t|, exp(-m_t)) + den_eps)
+ *   q, k, v       : rows of dtype at strides of their own (column slices of a projection)
+ *   gate_a, gate_b: gate logits [row][head] of dtype, gate_stride elements between rows
+ *   state         : float[state_rows][heads][pa_gated_linear_state_floats(kind, dim, vdim)], zero-filled once; sequence
+ *                   b's at state_slots[b] (negative: starts empty, unsaved)
+ *   out           : [n_rows][heads * vdim] of dtype;  dim <= 256, any vdim
+ * Single rows (q_lens NULL), PA_F32 and rows that are not whole 8-byte vectors run token by token; PA_BF16 portions in
+ * chunks of 64 rows on the matrix cores, with the 32-bit factors split into two bf16 terms, and, given a workspace, in
+ * segments that run at the same time when there are few sequences.  max_q_len: at least the longest portion.
+ */
+size_t pa_gated_linear_state_floats(int kind, int dim, int vdim);
+size_t pa_gated_linear_workspace_bytes(int batch, int num_heads, int dim, int vdim, int max_q_len);
+int pa_gated_linear(int kind, const void *q, int64_t q_stride, const void *k, int64_t k_stride, const void *v,
+                    int64_t v_stride, int heads_per_group, const void *gate_a, const void *gate_b, int64_t gate_stride,
+                    const float *head_a, const float *head_b, const float *head_c, float cap, float q_scale,
+                    float den_eps, int64_t n_rows, float *state, int64_t state_rows, const int32_t *ctx_lens,
+                    const int32_t *q_lens, const int32_t *q_starts, const int32_t *state_slots, int batch,
+                    int max_q_len, void *out, int num_heads, int dim, int vdim, int dtype, void *workspace,
+                    size_t workspace_bytes, void *stream);
+
+/* out = x w^T with 32-bit sums and results, for few outputs: x [rows] at x_stride, w [n][k], out float[rows][n]. */
+int pa_narrow_linear(const void *x, int64_t x_stride, const void *w, float *out, int64_t rows, int n, int k, int dtype,
+                     void *stream);
+
+/*
+ * Mixture of experts.  pa_moe_select, per row: scores s = sigmoid(logits); of `groups` equal groups of neighbours the
+ * `keep` with the largest sums of their two largest scores stay; of their experts the `top` with the largest scores are
+ * chosen (the lowest number first on ties).  ids int32[rows][top]; weights float[rows][top + 1]: the chosen scores over
+ * (their sum + 1e-20), then sigmoid(logits[experts]) when `shared`, else 0.  top <= 64, experts <= 1024.
+ * pa_moe_lists: counts int32[experts] and lists int32[experts][rows], expert e's items (row * top + place) in order.
+ * pa_moe_product: for every listed item, out[item] = W_e x[item / items_per_row], or with glu
+ * silu(G_e x) * (U_e x) where an expert's weight rows are the n rows of G followed by the n rows of U.
+ *   w : [experts][w_rows][w_stride] of dtype, rows zero past k.  The matrix-core kernels want w_stride % 64 == 0,
+ *   k % 8 == 0, n % 4 == 0 and 16-byte aligned tensors; anything else runs on the vector units.
+ */
+int pa_moe_select(const float *logits, int64_t logits_stride, int64_t rows, int experts, int top, int groups, int keep,
+                  int shared, int32_t *ids, float *weights, void *stream);
+int pa_moe_lists(const int32_t *ids, int64_t rows, int top, int experts, int32_t *counts, int32_t *lists, void *stream);
+int pa_moe_product(const void *x, int64_t x_stride, int items_per_row, const void *w, int64_t w_rows, int w_stride, int k,
+                   const int32_t *counts, const int32_t *lists, int64_t rows, int top, int experts, int glu, void *out,
+                   int n, int dtype, void *stream);
 
 #ifdef __cplusplus
 }

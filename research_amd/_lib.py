@@ -23,7 +23,9 @@ PA_ERR_HIP = -4
 
 PA_F32, PA_BF16, PA_F16, PA_FP8_E4M3 = 0, 1, 2, 3
 PA_NORM_NONE, PA_NORM_LAYER, PA_NORM_RMS = 0, 1, 2
-PA_ACT_SILU, PA_ACT_GELU_TANH = 0, 1
+PA_ACT_SILU, PA_ACT_GELU_TANH, PA_ACT_NONE = 0, 1, 2
+PA_GATE_SIGMOID_LAST, PA_GATE_SILU_FIRST = 0, 1
+PA_GL_SSD, PA_GL_MLSTM = 0, 1
 PA_V_PLAIN, PA_V_FIRST, PA_V_MIX = 0, 1, 2
 PA_QKV_TILE_ROWS = 16
 
@@ -88,16 +90,26 @@ SIGNATURES = {
 }
 _p, _i, _l, _f = c_void_p, c_int, c_int64, c_float
 SIGNATURES.update({
-    "pa_residual_norm": (_i, [_p, _p, _p, _f, _p, _p, _l, _p, _l, _p, _p, _f, _i, _p, _l, _i, _i, _p]),
-    "pa_rms_gate": (_i, [_p, _p, _l, _p, _f, _p, _l, _i, _i, _p]),
+    "pa_residual_norm": (_i, [_p, _p, _p, _i, _p, _p, _f, _p, _p, _l, _f, _p, _p, _l, _p, _l, _p, _p, _f, _i, _p, _l, _i, _i, _p]),
+    "pa_rms_gate": (_i, [_p, _p, _l, _p, _f, _p, _l, _l, _i, _i, _i, _i, _p]),
+    "pa_softcap": (_i, [_p, _p, _l, _f, _i, _p]),
     "pa_glu": (_i, [_p, _l, _p, _l, _p, _l, _p, _l, _i, _i, _i, _p]),
-    "pa_head_gate": (_i, [_p, _p, _l, _p, _l, _i, _i, _i, _i, _p]),
+    "pa_head_gate": (_i, [_p, _p, _l, _f, _p, _l, _l, _i, _i, _i, _i, _p]),
     "pa_qkv_conv_append": (_i, [_p, _l, _l, _p, _i, _p, _l, _p, _l, _i, _p, _p, _p, _p, _p, _i, _i, _p, _l, _p, _p, _p,
-                                _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p]),
+                                _p, _p, _i, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p]),
     "pa_lightning_state_floats": (c_size_t, [_i, _i]),
     "pa_lightning_recurrent": (_i, [_p, _l, _l, _p, _l, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _p]),
     "pa_lightning_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i]),
     "pa_lightning_chunked": (_i, [_p, _l, _l, _p, _l, _p, _p, _p, _p, _p, _i, _i, _p, _i, _i, _i, _i, _p, c_size_t, _p]),
+    "pa_short_conv": (_i, [_p, _l, _l, _p, _p, _i, _i, _p, _l, _p, _p, _p, _p, _p, _i, _i, _p, _i, _i, _p]),
+    "pa_gated_linear_state_floats": (c_size_t, [_i, _i, _i]),
+    "pa_gated_linear_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i]),
+    "pa_gated_linear": (_i, [_i, _p, _l, _p, _l, _p, _l, _i, _p, _p, _l, _p, _p, _p, _f, _f, _f, _l, _p, _l, _p, _p, _p, _p,
+                             _i, _i, _p, _i, _i, _i, _i, _p, c_size_t, _p]),
+    "pa_narrow_linear": (_i, [_p, _l, _p, _p, _l, _i, _i, _i, _p]),
+    "pa_moe_select": (_i, [_p, _l, _l, _i, _i, _i, _i, _i, _p, _p, _p]),
+    "pa_moe_lists": (_i, [_p, _l, _i, _i, _p, _p, _p]),
+    "pa_moe_product": (_i, [_p, _l, _i, _p, _l, _i, _i, _p, _p, _l, _i, _i, _i, _p, _i, _i, _p]),
 })
 SIGNATURES["pa_decode_split"] = SIGNATURES["pa_decode_reduce"] = SIGNATURES["pa_decode"]
 SIGNATURES["pa_prefill_paged_rowwise"] = SIGNATURES["pa_prefill_paged"]

@@ -109,8 +109,8 @@ int decode_launch(int phases, const void *q, const void *k_cache, const void *v_
     PA_REQUIRE(num_q_heads % num_kv_heads == 0, "num_q_heads=%d is not a multiple of num_kv_heads=%d",
                num_q_heads, num_kv_heads);
     PA_REQUIRE(block_size > 0, "block_size=%d must be positive", block_size);
-    PA_REQUIRE(window >= 0, "window=%d is negative (0 = no sliding window)", window);
-    PA_REQUIRE(window == 0 || !extra_zero_keys, "a sliding window cannot be combined with extra_zero_keys");
+    PA_REQUIRE(window >= -0x7fffffff, "window=%d is out of range", window);
+    PA_REQUIRE(window == 0 || !extra_zero_keys, "a window cannot be combined with extra_zero_keys");
     PA_REQUIRE(num_blocks >= 0 && bt_stride >= 0, "num_blocks / bt_stride must be non-negative");
     PA_REQUIRE(num_blocks * (int64_t)block_size < (1ll << 40), "pool of %lld blocks is too large", (long long)num_blocks);
     PA_REQUIRE((int64_t)block_size * num_kv_heads * head_dim * 4 < (1ll << 31),

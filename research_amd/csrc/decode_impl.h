@@ -53,7 +53,8 @@ struct PoolArgs {
             // (and d indices) at or past d hold zeros and store nothing
     int64_t num_blocks;
     float scale_log2;  // softmax scale * log2(e)
-    int window;        // sliding window: a query at position i sees keys j with i - j < window (0 = all keys)
+    int window;        // > 0 sliding window: a query at position i sees keys j with i - j < window; < 0 chunks of -window
+                       // positions: it sees keys of its own chunk; 0 all keys
     int hpw, tpw, n_hgroups, n_rgroups;
 };
 
@@ -94,7 +95,7 @@ struct RowwiseArgs {
 
 __device__ __forceinline__ uint4 ld16(const void *p) { return *reinterpret_cast<const uint4 *>(p); }
 
-// First key a query at position n_keys-1 sees under the sliding window (0 without one).
+// First key a query at position n_keys-1 sees under the window or chunk mask (0 without one).
 __device__ __forceinline__ int window_first_key(const PoolArgs &p, int n_keys) {
     return plan_first_key(n_keys, p.window);
 }

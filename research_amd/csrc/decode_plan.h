@@ -68,9 +68,15 @@ PA_PLAN_FN HeadPlan plan_heads(int num_q_heads, int num_kv_heads, int head_dim_r
     return h;
 }
 
-// Blocks of a sequence of `len` keys that hold visible keys under a sliding window (0 = none): the query sits at
-// position len-1 and sees keys j >= len - window, so blocks [first_key / bs, ceil(len / bs)) take part.
-PA_PLAN_FN int plan_first_key(int len, int window) { return window > 0 && len > window ? len - window : 0; }
+// First key that the query at position len-1 sees.  window > 0: a sliding window, keys j >= len - window; window < 0:
+// chunks of -window positions counted from the sequence's start, keys of the query's own chunk; 0: all keys.
+PA_PLAN_FN int plan_first_key(int len, int window) {
+    if (window > 0) return len > window ? len - window : 0;
+    return window < 0 && len > 0 ? (len - 1) - (len - 1) % -window : 0;
+}
+// Keys that a window or chunk lets a query see at most (0: no bound).
+PA_PLAN_FN int64_t plan_window_span(int window) { return window < 0 ? -(int64_t)window : window; }
+// Blocks of a sequence of `len` keys that hold visible keys: [first_key / bs, ceil(len / bs)).
 PA_PLAN_FN int plan_blocks_of(int len, int block_size, int window) {
     if (len <= 0) return 0;
     return (len + block_size - 1) / block_size - plan_first_key(len, window) / block_size;

@@ -36,3 +36,12 @@ static inline size_t la_state_floats(int dim, int vdim) { return (size_t)la_pad1
 static inline size_t la_workspace_bytes(int64_t batch, int heads, int dim, int vdim, int segments) {
     return segments <= 1 ? 0 : (size_t)batch * heads * segments * la_state_floats(dim, vdim) * sizeof(float);
 }
+
+// Gated recurrences: a head's floats in the pool (with a normaliser: S, and n and the running maximum once per 64 value
+// columns) and the segments' states (S, n, and three scalars).
+static inline size_t gl_state_floats(bool normaliser, int dim, int vdim) {
+    return la_state_floats(dim, vdim) + (normaliser ? (size_t)((vdim + 63) / 64) * (la_pad16(dim) + 16) : 0);
+}
+static inline size_t gl_workspace_bytes(int64_t batch, int heads, int dim, int vdim, int segments) {
+    return segments <= 1 ? 0 : (size_t)batch * heads * segments * (la_state_floats(dim, vdim) + la_pad16(dim) + 16) * sizeof(float);
+}

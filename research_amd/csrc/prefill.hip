@@ -79,7 +79,8 @@ int prefill_launch(bool force_rowwise, const void *q, const void *k_cache, const
     PA_REQUIRE(num_q_heads % num_kv_heads == 0, "num_q_heads=%d is not a multiple of num_kv_heads=%d",
                num_q_heads, num_kv_heads);
     PA_REQUIRE(block_size > 0, "block_size=%d must be positive", block_size);
-    PA_REQUIRE(window >= 0, "window=%d is negative (0 = no sliding window)", window);
+    PA_REQUIRE(window >= -0x7fffffff, "window=%d is out of range", window);
+    const int64_t span = plan_window_span(window);  // 0: every earlier key
     PA_REQUIRE(num_blocks >= 0 && bt_stride >= 0, "num_blocks / bt_stride must be non-negative");
     PA_REQUIRE(num_blocks * (int64_t)block_size < (1ll << 40), "pool of %lld blocks is too large", (long long)num_blocks);
     PA_REQUIRE(dtype == PA_F32 || dtype == PA_BF16 || dtype == PA_F16, "dtype=%d is not F32, BF16 or F16", dtype);
@@ -131,18 +132,18 @@ int prefill_launch(bool force_rowwise, const void *q, const void *k_cache, const
         (int64_t)max_q_len * num_q_heads * head_dim * 2 < (1ll << 31)) {
         const int64_t cap_keys = (int64_t)pa_asm_cap_tiles(d_pad) * kPfKeys;
         const bool fits = bt_stride * (int64_t)block_size <= cap_keys ||
-                          (window > 0 && (int64_t)window + kPfTasks * kPfRows + 3 * kPfKeys <= cap_keys);
+                          (span > 0 && span + kPfTasks * kPfRows + 3 * kPfKeys <= cap_keys);
         // With a workspace, a launch that cannot fill the chip has every workgroup's tiles cut into pieces (the
         // instance with lower bounds runs them: a piece is a later first tile and an earlier last key).
         if (workspace) {
             const int row_blocks = (max_q_len + kPfRows - 1) / kPfRows;
             const int64_t groups = (row_blocks * (int64_t)a.p.n_rep + kPfTasks - 1) / kPfTasks;
             int want = prefill_splits((int64_t)num_kv_heads * groups * batch, prefill_cus(),
-                                      window > 0 ? (int64_t)window + kPfTasks * kPfRows : bt_stride * (int64_t)block_size);
+                                      span > 0 ? span + kPfTasks * kPfRows : bt_stride * (int64_t)block_size);
             while (want > 1 && prefill_ws_bytes(total_q, num_q_heads, d_pad, want) > workspace_bytes) --want;
             split = want;
         }
-        const bool lower_bounds = split > 1 || window > 0 || row_first_key != nullptr;
+        const bool lower_bounds = split > 1 || span > 0 || row_first_key != nullptr;
         mfma = pa_prefill_asm_kernel(dtype, d_pad, lower_bounds, !fits);
         if (!lower_bounds && fits) {
             // The plain instance runs several groups of one (sequence, kv head) per workgroup, which share the
@@ -164,16 +165,16 @@ int prefill_launch(bool force_rowwise, const void *q, const void *k_cache, const
         // (the tables hold kWdCapGroups groups of 16 keys from the workgroup's first tile on; under a sliding window
         // a workgroup's kWdTasks blocks of kPfRows rows, and the tiles its loads run ahead, bound what it needs)
         const bool fits = bt_stride * (int64_t)block_size <= (int64_t)kWdCapGroups * 16 ||
-                          (window > 0 && (int64_t)window + kWdTasks * kPfRows + 10 * 32 <= (int64_t)kWdCapGroups * 16);
+                          (span > 0 && span + kWdTasks * kPfRows + 10 * 32 <= (int64_t)kWdCapGroups * 16);
         if (workspace) {  // (as above; a workgroup of this kernel holds kWdTasks tasks)
             const int row_blocks = (max_q_len + kPfRows - 1) / kPfRows;
             const int64_t groups = (row_blocks * (int64_t)a.p.n_rep + kWdTasks - 1) / kWdTasks;
             int want = prefill_splits((int64_t)num_kv_heads * groups * batch, prefill_cus(),
-                                      window > 0 ? (int64_t)window + kWdTasks * kPfRows : bt_stride * (int64_t)block_size);
+                                      span > 0 ? span + kWdTasks * kPfRows : bt_stride * (int64_t)block_size);
             while (want > 1 && prefill_ws_bytes(total_q, num_q_heads, d_pad, want) > workspace_bytes) --want;
             split = want;
         }
-        mfma = pa_prefill_d256_kernel(dtype, split > 1 || window > 0 || row_first_key != nullptr, !fits);
+        mfma = pa_prefill_d256_kernel(dtype, split > 1 || span > 0 || row_first_key != nullptr, !fits);
         tasks_per_wg = kWdTasks;
     }
     if (mfma) {
@@ -226,7 +227,7 @@ extern "C" size_t pa_prefill_workspace_bytes(int batch, int max_q_len, int64_t t
                                              int block_size, int window, int num_q_heads, int num_kv_heads,
                                              int head_dim, int dtype) {
     pa_clear_error();
-    if (batch < 0 || max_q_len < 0 || total_q < 0 || bt_stride < 0 || block_size <= 0 || window < 0 ||
+    if (batch < 0 || max_q_len < 0 || total_q < 0 || bt_stride < 0 || block_size <= 0 || window < -0x7fffffff ||
         num_q_heads <= 0 || num_kv_heads <= 0 || num_q_heads % num_kv_heads != 0 || head_dim <= 0) {
         pa_fail(PA_ERR_INVALID_ARG, "pa_prefill_workspace_bytes: negative size or inconsistent head counts");
         return 0;
@@ -240,8 +241,9 @@ extern "C" size_t pa_prefill_workspace_bytes(int batch, int max_q_len, int64_t t
     const int row_blocks = (max_q_len + kPfRows - 1) / kPfRows;
     const int tasks = d_pad == 256 ? kWdTasks : kPfTasks;
     const int64_t groups = (row_blocks * (int64_t)n_rep + tasks - 1) / tasks;
+    const int64_t span = plan_window_span(window);
     const int split = prefill_splits((int64_t)num_kv_heads * groups * batch, prefill_cus(),
-                                     window > 0 ? (int64_t)window + tasks * kPfRows : bt_stride * (int64_t)block_size);
+                                     span > 0 ? span + tasks * kPfRows : bt_stride * (int64_t)block_size);
     return prefill_ws_bytes(total_q, num_q_heads, d_pad, split);
 }
 

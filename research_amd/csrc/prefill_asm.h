@@ -172,7 +172,7 @@ __global__ __launch_bounds__(kPfThreads) void prefill_asm_kernel(const RowwiseAr
         const int32_t *rlo = a.row_lo ? a.row_lo + q_start : nullptr;
         auto row_first = [&](int row) PF_INLINE {
             const int pos = prefix + row;
-            int first = win > 0 ? pos - win + 1 : 0;
+            int first = win > 0 ? pos - win + 1 : win < 0 && pos > 0 ? pos - pos % -win : 0;
             if (rlo) first = max(first, rlo[min(row, q_len - 1)]);
             return min(max(first, 0), min(pos, ctx_len - 1));
         };

@@ -96,10 +96,10 @@ __global__ __launch_bounds__(kPfThreads) void prefill_d256_kernel(const RowwiseA
     // lower bounds (sliding window, per-row first keys): see prefill_mfma_kernel
     const int win = p.window;
     const int32_t *rlo = a.row_lo ? a.row_lo + a.q_starts[b] : nullptr;
-    const bool bounded = win > 0 || rlo != nullptr;  // uniform
+    const bool bounded = win != 0 || rlo != nullptr;  // uniform
     auto row_first = [&](int row) PF_INLINE {
         const int pos = prefix + row;
-        int lo = win > 0 ? pos - win + 1 : 0;
+        int lo = win > 0 ? pos - win + 1 : win < 0 && pos > 0 ? pos - pos % -win : 0;
         if (rlo) lo = max(lo, rlo[min(row, q_len - 1)]);
         return min(max(lo, 0), min(pos, ctx_len - 1));
     };

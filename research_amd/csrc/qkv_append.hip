@@ -1,5 +1,5 @@
 // From the joint q/k/v projection to attention's operands in one pass: a short causal convolution over time with its
-// carried state, interleaved rotary positions on the leading dimensions, unit-RMS q and k, value mixing, and the
+// carried state, RMS norms of q and k, interleaved rotary positions on the leading dimensions, value mixing, and the
 // append of k and v to the paged pool.  HBM-bound: every projected value is read once, everything between is in
 // 32-bit registers.
 //
@@ -29,6 +29,7 @@ struct QkvArgs {
     void *k_cache, *v_cache;  // [total_slots][hkv][d]
     void *v_first;            // [rows][hkv * vdim]
     const float *lambda;
+    const float *q_norm, *k_norm;  // [dim]: weights of RMS norms ahead of the rotation, or NULL
     int v_mode, batch, hq, hkv, dim, vdim, d, taps, rot, unit_norm;
     float eps, q_scale;
 };
@@ -129,6 +130,10 @@ __global__ __launch_bounds__(kThreadsQkv) void qkv_append_kernel(const QkvArgs a
     }
 
     const float lam = is_v && a.v_mode == PA_V_MIX ? *a.lambda : 0.f;
+    const float *norm_w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
+    float nw[8];
+    row_zero<8>(nw);
+    if (norm_w) load8<float, VEC>(norm_w + c0, left, nw);
     const int half = a.rot / 2;
     for (int i = i0; i < i1; ++i) {
         const int64_t row = row0 + i;
@@ -161,6 +166,14 @@ __global__ __launch_bounds__(kThreadsQkv) void qkv_append_kernel(const QkvArgs a
                 }
             }
         } else {
+            if (norm_w) {
+                float ss = 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) ss = fmaf(y[e], y[e], ss);
+                const float inv = 1.f / sqrtf(pa_group_sum<LPH>(ss) / (float)a.dim + a.eps);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) y[e] *= inv * nw[e];
+            }
             if (c0 < a.rot) {
                 int64_t pos = pos0 + i;
                 if (pos >= a.rope_rows) pos = a.rope_rows - 1;  // (the caller sizes the table; never read past it)
@@ -220,9 +233,9 @@ extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_row
                                   const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
                                   const int32_t *state_slots, const int32_t *tiles, int n_tiles, int batch,
                                   const int64_t *slots, int64_t total_slots, void *q_out, void *k_cache, void *v_cache,
-                                  void *v_first, const float *v_lambda, int v_mode, int num_q_heads, int num_kv_heads,
-                                  int dim, int vdim, int pool_dim, int unit_norm, float eps, float q_scale, int dtype,
-                                  void *stream) {
+                                  void *v_first, const float *v_lambda, int v_mode, const float *q_norm,
+                                  const float *k_norm, int num_q_heads, int num_kv_heads, int dim, int vdim, int pool_dim,
+                                  int unit_norm, float eps, float q_scale, int dtype, void *stream) {
     pa_clear_error();
     PA_REQUIRE(n_rows >= 0 && batch >= 0 && n_tiles >= 0 && total_slots >= 0 && state_rows >= 0 && rope_rows >= 0,
                "a count is negative");
@@ -248,6 +261,7 @@ extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_row
     PA_REQUIRE(taps == 1 || (conv_state && state_slots), "a convolution needs its carried state");
     PA_REQUIRE(v_mode == PA_V_PLAIN || v_first, "v_mode without v_first");
     PA_REQUIRE(v_mode != PA_V_MIX || v_lambda, "value mixing without v_lambda");
+    PA_REQUIRE((q_norm == nullptr) == (k_norm == nullptr), "q_norm and k_norm come together");
     PA_REQUIRE(pa_aligned16(q_out) && pa_aligned16(k_cache) && pa_aligned16(v_cache), "pointers must be 16-byte aligned");
     QkvArgs a{};
     a.u = u; a.ldu = u_stride; a.conv_w = conv_weight; a.conv_state = taps > 1 ? conv_state : nullptr;
@@ -256,9 +270,9 @@ extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_row
     a.slots = slots; a.total_slots = total_slots; a.n_rows = n_rows; a.q_out = q_out; a.k_cache = k_cache;
     a.v_cache = v_cache; a.v_first = v_first; a.lambda = v_lambda; a.v_mode = v_mode; a.batch = batch;
     a.hq = num_q_heads; a.hkv = num_kv_heads; a.dim = dim; a.vdim = vdim; a.d = pool_dim; a.taps = taps; a.rot = rot_dims;
-    a.unit_norm = unit_norm; a.eps = eps; a.q_scale = q_scale;
+    a.q_norm = q_norm; a.k_norm = k_norm; a.unit_norm = unit_norm; a.eps = eps; a.q_scale = q_scale;
     const bool vec = dim % 8 == 0 && vdim % 8 == 0 && u_stride % 8 == 0 && pa_aligned16(u) && pa_aligned16(conv_weight) &&
-                     pa_aligned16(conv_state) && pa_aligned16(v_first);
+                     pa_aligned16(conv_state) && pa_aligned16(v_first) && pa_aligned16(q_norm) && pa_aligned16(k_norm);
     hipStream_t s = (hipStream_t)stream;
     if (dtype == PA_F32) launch_qkv_typed<float>(a, n_tiles, vec, s);
     else launch_qkv_typed<pa_bf16>(a, n_tiles, vec, s);

@@ -49,9 +49,9 @@ template <typename T, int V> __device__ __forceinline__ void row_store(T *p, con
     }
 }
 
-// Sum over the TPR threads of a row (a wave, or the whole workgroup of 256 through `red`, 8 floats of LDS).
+// Sum over the TPR threads of a row (part of a wave, a wave, or the whole workgroup of 256 through `red`, 8 floats of LDS).
 template <int TPR> __device__ __forceinline__ float row_sum(float x, float *red) {
-    x = pa_group_sum<64>(x);
+    x = pa_group_sum<(TPR < 64 ? TPR : 64)>(x);
     if constexpr (TPR > 64) {
         __syncthreads();  // the previous sum has been read
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = x;

@@ -8,11 +8,18 @@ namespace {
 // ------------------------------------------------------------------ residual sum + norm
 struct ResidualArgs {
     float *x;               // [rows][width], the residual stream (read and, with y or ids, written)
-    const void *y;          // branch output [rows][width] of T, or NULL
+    const void *y;          // branch output [rows][width] of T (with mix_w: [rows * mix][width]), or NULL
+    const float *mix_w;     // [rows][mix + 1]: y = sum of mix_w[i] y[row * mix + i], i < mix, + mix_w[mix] y_extra[row]
+    const void *y_extra;    // [rows][width] of T, or NULL: without the last term
+    int mix;
     const float *y_weight;  // RMS norm applied to y before the sum, or NULL
     const int64_t *ids;     // x starts as table[ids[row]], or NULL
     const void *table;
     int64_t table_rows;
+    float table_scale;           // on the table's rows
+    const int64_t *positions;    // row positions[row] of pos_table is added, or NULL
+    const void *pos_table;
+    int64_t pos_rows;
     const int64_t *row_index;  // output row r reads residual row row_index[r] (x is not written), or NULL
     int64_t x_rows;
     const float *w, *b;  // norm weight and bias
@@ -45,6 +52,18 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualArgs a
             row_zero<V>(x[i]);
             if (ok && c < a.width) row_load<T, V>(src + c, x[i]);
         }
+        const int64_t pos = a.positions ? a.positions[row] : -1;
+        const bool placed = pos >= 0 && pos < a.pos_rows;
+        const T *psrc = reinterpret_cast<const T *>(a.pos_table) + (placed ? pos : 0) * a.width;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int c = (i * TPR + lane) * V;
+            float p[V];
+            row_zero<V>(p);
+            if (placed && c < a.width) row_load<T, V>(psrc + c, p);
+#pragma unroll
+            for (int j = 0; j < V; ++j) x[i][j] = fmaf(x[i][j], a.table_scale, p[j]);
+        }
     } else {
         const float *src = a.x + (have_x ? xrow : 0) * a.width;
 #pragma unroll
@@ -55,13 +74,33 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualArgs a
         }
     }
     if (a.y) {
-        const T *src = reinterpret_cast<const T *>(a.y) + row * a.width;
         float y[NV][V];
+        if (a.mix_w) {
+            const float *w = a.mix_w + row * (a.mix + 1);
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
-            const int c = (i * TPR + lane) * V;
-            row_zero<V>(y[i]);
-            if (c < a.width) row_load<T, V>(src + c, y[i]);
+            for (int i = 0; i < NV; ++i) row_zero<V>(y[i]);
+            for (int m = 0; m < a.mix + (a.y_extra ? 1 : 0); ++m) {
+                const T *src = m < a.mix ? reinterpret_cast<const T *>(a.y) + (row * a.mix + m) * a.width
+                                         : reinterpret_cast<const T *>(a.y_extra) + row * a.width;
+                const float f = w[m];
+#pragma unroll
+                for (int i = 0; i < NV; ++i) {
+                    const int c = (i * TPR + lane) * V;
+                    float t[V];
+                    row_zero<V>(t);
+                    if (c < a.width) row_load<T, V>(src + c, t);
+#pragma unroll
+                    for (int j = 0; j < V; ++j) y[i][j] = fmaf(f, t[j], y[i][j]);
+                }
+            }
+        } else {
+            const T *src = reinterpret_cast<const T *>(a.y) + row * a.width;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                const int c = (i * TPR + lane) * V;
+                row_zero<V>(y[i]);
+                if (c < a.width) row_load<T, V>(src + c, y[i]);
+            }
         }
         if (a.y_weight) {
             float ss = 0.f;
@@ -132,15 +171,15 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualArgs a
     }
 }
 
-// ------------------------------------------------------------------ RMS norm + sigmoid gate
+// ------------------------------------------------------------------ RMS norm + gate
 struct RmsGateArgs {
-    const void *o;  // [rows][width] of T
+    const void *o;  // [rows][groups * width] of T
     const void *g;  // gate logits, row stride ldg
-    int64_t ldg;
+    int64_t ldg, ldo;
     const float *w;
-    void *out;  // [rows][width]
-    int64_t rows;
-    int width;
+    void *out;  // row stride ldo
+    int64_t rows;  // of one group each: row * groups + group
+    int width, groups, gate;
     float eps;
 };
 
@@ -150,8 +189,10 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(const RmsGateArgs a) {
     const int64_t row = (int64_t)blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
     if (row >= a.rows) return;
     const int lane = threadIdx.x % TPR;
+    const int64_t trow = a.groups == 1 ? row : row / a.groups;
+    const int first = a.groups == 1 ? 0 : (int)(row - trow * a.groups) * a.width;  // column of the group
     const T *src = reinterpret_cast<const T *>(a.o) + row * a.width;
-    const T *gate = reinterpret_cast<const T *>(a.g) + row * a.ldg;
+    const T *gate = reinterpret_cast<const T *>(a.g) + trow * a.ldg + first;
     float x[NV][V], g[NV][V];
     float ss = 0.f;
 #pragma unroll
@@ -167,17 +208,23 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(const RmsGateArgs a) {
 #pragma unroll
     for (int i = 0; i < NV; ++i)
 #pragma unroll
-        for (int j = 0; j < V; ++j) ss = fmaf(x[i][j], x[i][j], ss);
+        for (int j = 0; j < V; ++j) {
+            if (a.gate == PA_GATE_SILU_FIRST) x[i][j] *= row_silu<T>(g[i][j]);
+            ss = fmaf(x[i][j], x[i][j], ss);
+        }
     const float inv = 1.f / sqrtf(row_sum<TPR>(ss, red) / (float)a.width + a.eps);
-    T *dst = reinterpret_cast<T *>(a.out) + row * a.width;
+    T *dst = reinterpret_cast<T *>(a.out) + trow * a.ldo + first;
 #pragma unroll
     for (int i = 0; i < NV; ++i) {
         const int c = (i * TPR + lane) * V;
         if (c >= a.width) continue;
         float w[V], o[V];
-        row_load<float, V>(a.w + c, w);
+        row_load<float, V>(a.w + first + c, w);
 #pragma unroll
-        for (int j = 0; j < V; ++j) o[j] = x[i][j] * inv * w[j] * row_sigmoid<T>(g[i][j]);
+        for (int j = 0; j < V; ++j) {
+            o[j] = x[i][j] * inv * w[j];
+            if (a.gate == PA_GATE_SIGMOID_LAST) o[j] *= row_sigmoid<T>(g[i][j]);
+        }
         row_store<T, V>(dst + c, o);
     }
 }
@@ -220,12 +267,14 @@ struct HeadGateArgs {
     const void *o;  // [rows][heads][d]
     const void *g;  // one logit per head, row stride ldg
     int64_t ldg;
-    void *out;  // [rows][heads][vdim]
+    void *out;  // rows of heads * vdim, row stride ldo
+    int64_t ldo;
     int64_t rows;
     int heads, d, vdim;
+    float scale;
 };
 
-// out = o * sigmoid(gate of the head), the first vdim of every head's d values, packed
+// out = scale * o * sigmoid(gate of the head), the first vdim of every head's d values, packed
 template <typename T, int V> __global__ __launch_bounds__(256) void head_gate_kernel(const HeadGateArgs a) {
     const int per_head = a.vdim / V, per_row = a.heads * per_head;
     const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
@@ -234,19 +283,36 @@ template <typename T, int V> __global__ __launch_bounds__(256) void head_gate_ke
     const int r = (int)(i - row * per_row), h = r / per_head, c = (r - h * per_head) * V;
     float o[V];
     row_load<T, V>(reinterpret_cast<const T *>(a.o) + (row * a.heads + h) * a.d + c, o);
-    if (a.g) {
-        const float s = row_sigmoid<T>(pa_scalar<T>::load(reinterpret_cast<const T *>(a.g) + row * a.ldg + h));
+    if (a.g || a.scale != 1.f) {
+        float s = a.scale;
+        if (a.g) s *= row_sigmoid<T>(pa_scalar<T>::load(reinterpret_cast<const T *>(a.g) + row * a.ldg + h));
 #pragma unroll
         for (int j = 0; j < V; ++j) o[j] *= s;
     }
-    row_store<T, V>(reinterpret_cast<T *>(a.out) + (row * a.heads + h) * a.vdim + c, o);
+    row_store<T, V>(reinterpret_cast<T *>(a.out) + row * a.ldo + h * a.vdim + c, o);
 }
 
-// Threads per row and registers per thread by row width: one wave up to 1024 columns, a workgroup above.
+// out = cap * tanh(x / cap)
+template <typename T, int V> __global__ __launch_bounds__(256) void softcap_kernel(const void *x, float *out, int64_t n, float cap) {
+    const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * V;
+    if (i >= n) return;
+    float f[V];
+    row_load<T, V>(reinterpret_cast<const T *>(x) + i, f);
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+        const float z = f[j] / cap;
+        f[j] = cap * (sizeof(T) == 4 ? tanhf(z) : 2.f * row_sigmoid<T>(2.f * z) - 1.f);
+    }
+    row_store<float, V>(out + i, f);
+}
+
+// Threads per row and registers per thread by row width: part of a wave, a wave (256 columns), a workgroup.
 #define ROW_DISPATCH(KERNEL, T, vec4, width, rows, args, s)                                                \
     do {                                                                                                   \
         const unsigned grid64_ = (unsigned)(((rows) + 3) / 4), grid256_ = (unsigned)(rows);                \
         if (!(vec4)) KERNEL<T, 256, 1, 64><<<dim3(grid256_), dim3(256), 0, s>>>(args);                     \
+        else if ((width) <= 64) KERNEL<T, 16, 4, 1><<<dim3((unsigned)(((rows) + 15) / 16)), dim3(256), 0, s>>>(args); \
+        else if ((width) <= 128) KERNEL<T, 32, 4, 1><<<dim3((unsigned)(((rows) + 7) / 8)), dim3(256), 0, s>>>(args); \
         else if ((width) <= 256) KERNEL<T, 64, 4, 1><<<dim3(grid64_), dim3(256), 0, s>>>(args);            \
         else if ((width) <= 512) KERNEL<T, 64, 4, 2><<<dim3(grid64_), dim3(256), 0, s>>>(args);            \
         else if ((width) <= 1024) KERNEL<T, 256, 4, 1><<<dim3(grid256_), dim3(256), 0, s>>>(args);         \
@@ -268,8 +334,10 @@ int check_rows(const char *what, int64_t rows, int width, int dtype) {
 
 }  // namespace
 
-extern "C" int pa_residual_norm(float *x, const void *y, const float *y_weight, float y_eps, const int64_t *ids,
-                                const void *table, int64_t table_rows, const int64_t *row_index, int64_t x_rows,
+extern "C" int pa_residual_norm(float *x, const void *y, const float *mix_weight, int mix, const void *y_extra,
+                                const float *y_weight, float y_eps, const int64_t *ids, const void *table,
+                                int64_t table_rows, float table_scale, const int64_t *positions, const void *pos_table,
+                                int64_t pos_rows, const int64_t *row_index, int64_t x_rows,
                                 const float *norm_weight, const float *norm_bias, float eps, int norm, void *out,
                                 int64_t rows, int width, int dtype, void *stream) {
     pa_clear_error();
@@ -280,11 +348,18 @@ extern "C" int pa_residual_norm(float *x, const void *y, const float *y_weight, 
     PA_REQUIRE(!ids || table, "ids without a table");
     PA_REQUIRE(!row_index || (x && !y && !ids), "row_index only reads the residual");
     PA_REQUIRE(!y_weight || y, "y_weight without y");
+    PA_REQUIRE(!positions || (ids && pos_table), "positions without ids or a table");
+    PA_REQUIRE(!mix_weight || (y && mix > 0), "mix_weight without y");
+    PA_REQUIRE(!y_extra || mix_weight, "y_extra without mix_weight");
     PA_REQUIRE(out || (x && (y || ids)), "nothing to write");
     PA_REQUIRE(norm != PA_NORM_NONE || (!norm_weight && !norm_bias), "norm weights without a norm");
-    ResidualArgs a{x, y, y_weight, ids, table, table_rows, row_index, x_rows, norm_weight, norm_bias, out, rows, width,
-                   norm, y_eps, eps};
+    ResidualArgs a{};
+    a.x = x; a.y = y; a.mix_w = mix_weight; a.y_extra = y_extra; a.mix = mix; a.y_weight = y_weight; a.ids = ids;
+    a.table = table; a.table_rows = table_rows; a.table_scale = table_scale; a.positions = positions;
+    a.pos_table = pos_table; a.pos_rows = pos_rows; a.row_index = row_index; a.x_rows = x_rows; a.w = norm_weight;
+    a.b = norm_bias; a.out = out; a.rows = rows; a.width = width; a.norm = norm; a.y_eps = y_eps; a.eps = eps;
     const bool vec4 = width % 4 == 0 && pa_aligned16(x) && pa_aligned16(y) && pa_aligned16(table) && pa_aligned16(out) &&
+                      pa_aligned16(y_extra) && pa_aligned16(pos_table) &&
                       pa_aligned16(y_weight) && pa_aligned16(norm_weight) && pa_aligned16(norm_bias);
     hipStream_t s = (hipStream_t)stream;
     if (dtype == PA_F32) ROW_DISPATCH(residual_norm_kernel, float, vec4, width, rows, a, s);
@@ -294,19 +369,25 @@ extern "C" int pa_residual_norm(float *x, const void *y, const float *y_weight, 
 }
 
 extern "C" int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride, const float *weight, float eps, void *out,
-                           int64_t rows, int width, int dtype, void *stream) {
+                           int64_t out_stride, int64_t rows, int width, int groups, int gate_mode, int dtype,
+                           void *stream) {
     pa_clear_error();
-    if (int rc = check_rows("pa_rms_gate", rows, width, dtype)) return rc;
+    PA_REQUIRE(groups > 0 && width % groups == 0, "pa_rms_gate: width=%d is not %d equal groups", width, groups);
+    const int per = width / groups;
+    const int64_t parts = rows * groups;
+    if (int rc = check_rows("pa_rms_gate", rows < 0 ? rows : parts, per, dtype)) return rc;
+    PA_REQUIRE(gate_mode == PA_GATE_SIGMOID_LAST || gate_mode == PA_GATE_SILU_FIRST, "gate_mode=%d is unknown", gate_mode);
     if (rows == 0) return PA_OK;
     PA_REQUIRE(o && gate && weight && out, "NULL argument");
     PA_REQUIRE(gate_stride >= width, "gate_stride=%lld is shorter than a row", (long long)gate_stride);
-    RmsGateArgs a{o, gate, gate_stride, weight, out, rows, width, eps};
-    const uintptr_t gmask = dtype == PA_F32 ? 15u : 7u;  // four elements
-    const bool vec4 = width % 4 == 0 && gate_stride % 4 == 0 && ((uintptr_t)gate & gmask) == 0 && pa_aligned16(o) &&
-                      pa_aligned16(weight) && pa_aligned16(out);
+    PA_REQUIRE(out_stride >= width, "out_stride=%lld is shorter than a row", (long long)out_stride);
+    RmsGateArgs a{o, gate, gate_stride, out_stride, weight, out, parts, per, groups, gate_mode, eps};
+    const uintptr_t four = dtype == PA_F32 ? 15u : 7u;  // four elements
+    const bool vec4 = per % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && ((uintptr_t)gate & four) == 0 &&
+                      ((uintptr_t)out & four) == 0 && pa_aligned16(o) && pa_aligned16(weight);
     hipStream_t s = (hipStream_t)stream;
-    if (dtype == PA_F32) ROW_DISPATCH(rms_gate_kernel, float, vec4, width, rows, a, s);
-    else ROW_DISPATCH(rms_gate_kernel, pa_bf16, vec4, width, rows, a, s);
+    if (dtype == PA_F32) ROW_DISPATCH(rms_gate_kernel, float, vec4, per, parts, a, s);
+    else ROW_DISPATCH(rms_gate_kernel, pa_bf16, vec4, per, parts, a, s);
     PA_CHECK_LAUNCH("pa_rms_gate");
     return PA_OK;
 }
@@ -339,17 +420,18 @@ extern "C" int pa_glu(const void *gate, int64_t gate_stride, const void *up, int
     return PA_OK;
 }
 
-extern "C" int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, void *out, int64_t rows, int heads, int d,
-                            int vdim, int dtype, void *stream) {
+extern "C" int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, float scale, void *out,
+                            int64_t out_stride, int64_t rows, int heads, int d, int vdim, int dtype, void *stream) {
     pa_clear_error();
     PA_REQUIRE(rows >= 0 && heads > 0 && d > 0 && vdim > 0 && vdim <= d, "pa_head_gate: sizes out of range");
     if (dtype != PA_F32 && dtype != PA_BF16) return pa_fail(PA_ERR_UNSUPPORTED, "pa_head_gate: dtype=%d is not F32 or BF16", dtype);
     if (rows == 0) return PA_OK;
     PA_REQUIRE(o && out, "NULL argument");
     PA_REQUIRE(!gate || gate_stride >= heads, "gate_stride=%lld is shorter than a row", (long long)gate_stride);
-    HeadGateArgs a{o, gate, gate_stride, out, rows, heads, d, vdim};
+    PA_REQUIRE(out_stride >= (int64_t)heads * vdim, "out_stride=%lld is shorter than a row", (long long)out_stride);
+    HeadGateArgs a{o, gate, gate_stride, out, out_stride, rows, heads, d, vdim, scale};
     const int n = dtype == PA_F32 ? 4 : 8;
-    const bool vec = d % n == 0 && vdim % n == 0 && pa_aligned16(o) && pa_aligned16(out);
+    const bool vec = d % n == 0 && vdim % n == 0 && out_stride % n == 0 && pa_aligned16(o) && pa_aligned16(out);
     const int64_t items = rows * heads * (vec ? vdim / n : vdim), grid = (items + 255) / 256;
     PA_REQUIRE(grid <= 0x7fffffff, "pa_head_gate: rows=%lld is too large for one launch", (long long)rows);
     const dim3 g((unsigned)grid), blk(256);
@@ -362,5 +444,27 @@ extern "C" int pa_head_gate(const void *o, const void *gate, int64_t gate_stride
         else head_gate_kernel<pa_bf16, 1><<<g, blk, 0, s>>>(a);
     }
     PA_CHECK_LAUNCH("pa_head_gate");
+    return PA_OK;
+}
+
+extern "C" int pa_softcap(const void *x, float *out, int64_t n, float cap, int dtype, void *stream) {
+    pa_clear_error();
+    PA_REQUIRE(n >= 0 && cap > 0.f, "pa_softcap: n / cap out of range");
+    if (dtype != PA_F32 && dtype != PA_BF16) return pa_fail(PA_ERR_UNSUPPORTED, "pa_softcap: dtype=%d is not F32 or BF16", dtype);
+    if (n == 0) return PA_OK;
+    PA_REQUIRE(x && out, "NULL argument");
+    const bool vec = n % 4 == 0 && pa_aligned16(x) && pa_aligned16(out);
+    const int64_t grid = ((vec ? n / 4 : n) + 255) / 256;
+    PA_REQUIRE(grid <= 0x7fffffff, "pa_softcap: n=%lld is too large for one launch", (long long)n);
+    const dim3 g((unsigned)grid), blk(256);
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == PA_F32) {
+        if (vec) softcap_kernel<float, 4><<<g, blk, 0, s>>>(x, out, n, cap);
+        else softcap_kernel<float, 1><<<g, blk, 0, s>>>(x, out, n, cap);
+    } else {
+        if (vec) softcap_kernel<pa_bf16, 4><<<g, blk, 0, s>>>(x, out, n, cap);
+        else softcap_kernel<pa_bf16, 1><<<g, blk, 0, s>>>(x, out, n, cap);
+    }
+    PA_CHECK_LAUNCH("pa_softcap");
     return PA_OK;
 }

@@ -29,11 +29,12 @@ def generate(argv) -> int:
     ap.add_argument("--graphs", action="store_true", help="replay decode steps from captured graphs")
     args = ap.parse_args(argv)
     from .engine import InferenceEngine
+    from .registry import model_len
     from .types import EngineConfig, SamplingParams
 
     engine = InferenceEngine(EngineConfig(
         model_path=args.model, cache_type=args.cache_type, max_batch_size=args.max_batch_size,
-        max_model_len=args.max_model_len, use_graphs=args.graphs, dtype=args.dtype,
+        max_model_len=model_len(args.model, args.max_model_len), use_graphs=args.graphs, dtype=args.dtype,
         prefill_portion=args.prefill_portion))
     prompts = [[int(t) for t in p.split(",")] for p in args.prompt_ids]
     for sample in engine.generate(prompts, SamplingParams(temperature=args.temperature, max_tokens=args.max_tokens),

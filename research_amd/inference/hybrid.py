@@ -1,8 +1,9 @@
-"""Hybrid decoder: window attention and linear-attention layers in any order over one packed batch.
+"""Hybrid decoder: attention and recurrent layers in any order over one packed batch.
 
-``HybridDecoder`` is the block structure: a 32-bit residual, pre-norm mixer and
-feed-forward, optionally a per-layer token input.  The residual sums are fused
-with the norms that read them (``pa_residual_norm``).  It runs packed rows: a
+``HybridDecoder`` is the block structure: a 32-bit residual, mixer and
+feed-forward with norms ahead of or behind them, optionally a per-layer token
+input and learned positions.  The residual sums are fused with the norms around
+them (``pa_residual_norm``).  It runs packed rows: a
 batch is one run of tokens, sequences one after the other, single decoded
 tokens beside portions of prompts, and the context says which rows belong to
 whom (``InferenceContext.q_lens``).
@@ -10,7 +11,9 @@ whom (``InferenceContext.q_lens``).
 Designs on top of it are a function from their ``config.json`` to a
 ``HybridConfig`` and a table of checkpoint names.  Lotozen is one: layer norms
 with biases, unit-RMS q and k behind three-way short convolutions, value mixing,
-per-head output gates, lightning attention, per-layer token inputs.
+per-head output gates, lightning attention, per-layer token inputs.  Tevirax is
+another: RMS norms on the sublayers' outputs, chunk attention beside a matrix
+memory in one layer, Mamba-2 layers, mixtures of experts, capped logits.
 """
 
 from __future__ import annotations
@@ -24,15 +27,25 @@ from torch import Tensor, nn
 
 from .. import ops
 from .attention import CacheConfig, HipPagedAttentionBackend
-from .mixers import (AttentionSpec, ConvAttention, GatedMLP, LightningMixer, LightningSpec, RotaryTables, StepRows,
-                     TokenSide, _param, fill)
+from .mixers import (AttentionSpec, ConvAttention, GatedMLP, LightningMixer, LightningSpec, Mamba2Mixer, Mamba2Spec,
+                     MlstmSpec, ParallelMixer, ParallelSpec, RotaryTables, StepRows, TokenSide, YarnScaling, _param, fill)
+from .moe import MoE, MoESpec
 from .types import InferenceContext
+
+
+MixerSpec = Union[AttentionSpec, LightningSpec, Mamba2Spec, ParallelSpec]
 
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[AttentionSpec, LightningSpec]
-    ff: Optional[int]  # inner width of the feed-forward, None: the layer has none
+    mixer: MixerSpec
+    ff: Union[int, MoESpec, None]  # inner width of a dense feed-forward, experts, None: the layer has none
+
+    @property
+    def attention(self) -> Optional[AttentionSpec]:
+        """The part of the layer that keeps keys, if any."""
+        mixer = self.mixer.left if isinstance(self.mixer, ParallelSpec) else self.mixer
+        return mixer if isinstance(mixer, AttentionSpec) else None
 
 
 @dataclass(frozen=True)
@@ -42,8 +55,15 @@ class HybridConfig:
     layers: Tuple[LayerSpec, ...]
     norm_eps: float
     side_dim: int = 0  # columns per layer of the second embedding, 0: no per-layer token input
+    norm: str = "layer"  # "layer" (with biases) | "rms"
+    post_norm: bool = False  # the norms are on the sublayers' outputs ("rms"), which read the residual itself
+    embed_scale: float = 1.0
+    positions: int = 0  # rows of a learned position table that the embedding adds, 0: none
+    logit_softcap: Optional[float] = None
 
     def __post_init__(self) -> None:
+        if self.post_norm and (self.norm != "rms" or self.side_dim):
+            raise ValueError("norms behind the sublayers are RMS norms, without a per-layer token input")
         mixed = {(l.mixer.kv_heads, l.mixer.vdim) for l in self.layers if isinstance(l.mixer, AttentionSpec) and l.mixer.v_mix}
         if len(mixed) > 1:
             raise ValueError(f"layers that mix values differ in their value heads: {sorted(mixed)}")
@@ -58,21 +78,23 @@ class HybridConfig:
 
     def cache_config(self, num_blocks: int, block_size: int, num_state_slots: int, dtype: torch.dtype,
                      device: str) -> CacheConfig:
-        shapes = tuple((l.mixer.kv_heads, l.mixer.pool_dim) if isinstance(l.mixer, AttentionSpec) else None
-                       for l in self.layers)
+        keys = [l.attention for l in self.layers]
+        shapes = tuple((a.kv_heads, a.pool_dim) if a is not None else None for a in keys)
         typical = next((s for s in shapes if s is not None), (1, 8))
         return CacheConfig(num_layers=len(shapes), num_kv_heads=typical[0], head_dim=typical[1], num_blocks=num_blocks,
                            block_size=block_size, dtype=dtype, device=device, layer_kv=shapes,
                            num_state_slots=num_state_slots)
 
 
+def _only(what: str, got: dict, *keys: str) -> None:
+    extra = sorted(set(got) - set(keys))
+    if extra:
+        raise ValueError(f"{what}: unknown fields {extra}")
+
+
 def lotozen_config(d: dict) -> HybridConfig:
     """From the fields of a Lotozen ``config.json``.  Anything it does not know it refuses."""
-    def only(what: str, got: dict, *keys: str) -> None:
-        extra = sorted(set(got) - set(keys))
-        if extra:
-            raise ValueError(f"{what}: unknown fields {extra}")
-
+    only = _only
     layers = []
     for i, layer in enumerate(d["layers"]):
         m, mlp = layer["mixer"], layer.get("mlp")
@@ -107,17 +129,79 @@ def lotozen_config(d: dict) -> HybridConfig:
                         norm_eps=float(d["norm"]["eps"]), side_dim=int(side.get("dim", 0)))
 
 
-class _Norm(nn.Module):
-    """Weights of a layer norm; the arithmetic is fused into the residual sums."""
+def _tevirax_ff(where: str, mlp: Optional[dict]) -> Union[int, MoESpec, None]:
+    if mlp is None:
+        return None
+    if mlp["kind"] == "dense":
+        _only(where, mlp, "kind", "ff")
+        return int(mlp["ff"])
+    if mlp["kind"] != "moe":
+        raise ValueError(f"{where}: unknown feed-forward {mlp['kind']!r}")
+    _only(where, mlp, "kind", "expert", "router", "shared")
+    expert, router, shared = mlp["expert"], mlp["router"], mlp.get("shared")
+    groups = router.get("groups") or {"count": 1, "keep": 1}
+    _only(f"{where} expert", expert, "ff")
+    _only(f"{where} router", router, "experts", "top", "groups")
+    _only(f"{where} router.groups", groups, "count", "keep")
+    if shared is not None:
+        _only(f"{where} shared", shared, "ff")
+    return MoESpec(experts=int(router["experts"]), ff=int(expert["ff"]), top=int(router["top"]), groups=int(groups["count"]),
+                   keep=int(groups["keep"]), shared=int(shared["ff"]) if shared is not None else None)
 
-    def __init__(self, width: int, device) -> None:
+
+def tevirax_config(d: dict) -> HybridConfig:
+    """From the fields of a Tevirax ``config.json``.  Anything it does not know it refuses."""
+    layers = []
+    for i, layer in enumerate(d["layers"]):
+        m, at = layer["mixer"], f"layer {i} mixer"
+        _only(f"layer {i}", layer, "type", "mixer", "mlp")
+        if layer["type"] == "mamba2":
+            _only(at, m, "heads", "vdim", "state", "groups", "conv", "norm_groups")
+            mixer: MixerSpec = Mamba2Spec(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
+                                          taps=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+        elif layer["type"] == "parallel":
+            _only(at, m, "left", "right", "left_scale", "right_scale")
+            left, right = m["left"], m["right"]
+            _only(at + ".left", left, "heads", "kv_heads", "dim", "vdim", "rot", "scale", "mask")
+            _only(at + ".right", right, "heads", "dim", "vdim", "gate_cap")
+            rot, mask = left.get("rot") or {}, left.get("mask") or {}
+            _only(at + ".left.rot", rot, "base", "dims", "scaling")
+            _only(at + ".left.mask", mask, "size")
+            scaling = rot.get("scaling")
+            if scaling is not None:
+                _only(at + ".left.rot.scaling", scaling, "factor", "original", "fast", "slow")
+                scaling = YarnScaling(**{key: float(scaling[key]) for key in ("factor", "original", "fast", "slow")})
+            mixer = ParallelSpec(
+                left=AttentionSpec(heads=int(left["heads"]), kv_heads=int(left["kv_heads"]), dim=int(left["dim"]), vdim=int(left["vdim"]),
+                                   scale=float(left["scale"]), window=None, taps=0, rot_dims=int(rot.get("dims", 0)),
+                                   rot_base=float(rot.get("base", 1.0)), chunk=int(mask["size"]) if mask.get("size") is not None else None,
+                                   rot_yarn=scaling, rot_halves=True, qk_weights=True, gates=False),
+                right=MlstmSpec(heads=int(right["heads"]), dim=int(right["dim"]), vdim=int(right["vdim"]), gate_cap=float(right["gate_cap"])),
+                left_scale=float(m["left_scale"]), right_scale=float(m["right_scale"]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}")
+        layers.append(LayerSpec(mixer, _tevirax_ff(f"layer {i} mlp", layer.get("mlp"))))
+    _only("norm", d["norm"], "eps")
+    _only("embedding", d["embedding"], "scale")
+    cap = d.get("logit_softcap")
+    return HybridConfig(vocab_size=int(d["vocab"]), width=int(d["width"]), layers=tuple(layers), norm_eps=float(d["norm"]["eps"]),
+                        norm="rms", post_norm=True, embed_scale=float(d["embedding"]["scale"]), positions=int(d["max_positions"]),
+                        logit_softcap=float(cap) if cap else None)
+
+
+class _Norm(nn.Module):
+    """Weights of a norm; the arithmetic is fused into the residual sums.  ``args`` as ``pa_residual_norm`` takes them."""
+
+    def __init__(self, cfg: HybridConfig, device) -> None:
         super().__init__()
-        self.w = _param(width, dtype=torch.float32, device=device)
-        self.b = _param(width, dtype=torch.float32, device=device)
+        self.w = _param(cfg.width, dtype=torch.float32, device=device)
+        self.b = _param(cfg.width, dtype=torch.float32, device=device) if cfg.norm == "layer" else None
+        self.args = dict(norm=cfg.norm, weight=self.w, bias=self.b, eps=cfg.norm_eps)
 
     def load(self, get, name: str) -> None:
         fill(self.w, get(name), name)
-        fill(self.b, get(name + ".b"), name + ".b")
+        if self.b is not None:
+            fill(self.b, get(name + ".b"), name + ".b")
 
 
 class _HybridLayer(nn.Module):
@@ -125,15 +209,20 @@ class _HybridLayer(nn.Module):
                  v_role: Optional[str], dtype: torch.dtype, device) -> None:
         super().__init__()
         spec = cfg.layers[i]
-        self.norm1 = _Norm(cfg.width, device)
+        self.norm1 = _Norm(cfg, device)
         if isinstance(spec.mixer, AttentionSpec):
             self.mixer = ConvAttention(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, v_role, dtype, device)
+        elif isinstance(spec.mixer, ParallelSpec):
+            self.mixer = ParallelMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, dtype, device)
+        elif isinstance(spec.mixer, Mamba2Spec):
+            self.mixer = Mamba2Mixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
         else:
             self.mixer = LightningMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
         self.norm2 = self.mlp = self.side = None
         if spec.ff is not None:
-            self.norm2 = _Norm(cfg.width, device)
-            self.mlp = GatedMLP(cfg.width, spec.ff, dtype, device)
+            self.norm2 = _Norm(cfg, device)
+            self.mlp = (MoE(spec.ff, cfg.width, dtype, device) if isinstance(spec.ff, MoESpec)
+                        else GatedMLP(cfg.width, spec.ff, dtype, device))
         if cfg.side_dim:
             self.side = TokenSide(cfg.width, cfg.side_dim, i, dtype, device)
 
@@ -159,15 +248,16 @@ class HybridDecoder(nn.Module):
         super().__init__()
         device = backend.config.device
         self.cfg, self.backend, self.dtype = cfg, backend, dtype
-        self.max_positions = max_positions
+        self.max_positions = min(max_positions, cfg.positions) if cfg.positions else max_positions
         self.rotary = RotaryTables(max_positions, device)
         self.embed = _param(cfg.vocab_size, cfg.width, dtype=dtype, device=device)
+        self.pos_embed = _param(cfg.positions, cfg.width, dtype=dtype, device=device) if cfg.positions else None
         self.side_embed = None
         if cfg.side_dim:
             self.side_embed = _param(cfg.vocab_size, cfg.side_dim * len(cfg.layers), dtype=dtype, device=device)
         self.layers = nn.ModuleList(_HybridLayer(cfg, i, backend, self.rotary, role, dtype, device)
                                     for i, role in enumerate(cfg.v_roles()))
-        self.norm = _Norm(cfg.width, device)
+        self.norm = _Norm(cfg, device)
         self.head = _param(cfg.vocab_size, cfg.width, dtype=dtype, device=device)
 
     # ------------------------------------------------------------------ weights
@@ -184,6 +274,8 @@ class HybridDecoder(nn.Module):
 
         with torch.no_grad():
             fill(self.embed, get("embed"), "embed")
+            if self.pos_embed is not None:
+                fill(self.pos_embed, get("pos"), "pos")
             if self.side_embed is not None:
                 fill(self.side_embed, get("side.embed"), "side.embed")
             for i, layer in enumerate(self.layers):
@@ -204,16 +296,23 @@ class HybridDecoder(nn.Module):
         if packed.num_rows != ids.numel():
             raise ValueError(f"{ids.numel()} tokens for a context of {packed.num_rows} rows")
         step = StepRows(packed, ids)
-        eps, dtype = self.cfg.norm_eps, self.dtype
+        cfg, eps, dtype = self.cfg, self.cfg.norm_eps, self.dtype
         x = torch.empty((ids.numel(), self.cfg.width), dtype=torch.float32, device=ids.device)
         # what the next residual sum adds: nothing but the embedding at first, then the last branch's output
-        pending: dict = {"ids": ids, "table": self.embed}
+        pending: dict = {"ids": ids, "table": self.embed, "table_scale": cfg.embed_scale}
+        if self.pos_embed is not None:
+            if positions is None:
+                raise ValueError("learned positions need the rows' positions")
+            pending.update(positions=positions.reshape(-1), pos_table=self.pos_embed)
+        # a norm's weights either with the sum that a sublayer reads, or with the sublayer's output as it is added
+        ahead = (lambda norm: {}) if cfg.post_norm else (lambda norm: norm.args)
+        behind = (lambda norm: {"y_weight": norm.w, "y_eps": eps}) if cfg.post_norm else (lambda norm: {})
         for layer in self.layers:
-            h = ops.residual_norm(x, dtype, **pending, norm="layer", weight=layer.norm1.w, bias=layer.norm1.b, eps=eps)
-            pending = {"y": layer.mixer(h, step)}
+            h = ops.residual_norm(x, dtype, **pending, **ahead(layer.norm1))
+            pending = {"y": layer.mixer(h, step), **behind(layer.norm1)}
             if layer.mlp is not None:
-                h = ops.residual_norm(x, dtype, **pending, norm="layer", weight=layer.norm2.w, bias=layer.norm2.b, eps=eps)
-                pending = {"y": layer.mlp(h)}
+                h = ops.residual_norm(x, dtype, **pending, **ahead(layer.norm2))
+                pending = {**layer.mlp.branch(h), **behind(layer.norm2)}
             if layer.side is not None:
                 h = ops.residual_norm(x, dtype, **pending)
                 pending = {"y": layer.side(h, ids, self.side_embed), "y_weight": layer.side.norm, "y_eps": eps}
@@ -226,6 +325,6 @@ class HybridDecoder(nn.Module):
         return x.view(*input_ids.shape, self.cfg.width)
 
     def logits(self, hidden_rows: Tensor) -> Tensor:
-        h = ops.residual_norm(hidden_rows.contiguous(), self.dtype, norm="layer", weight=self.norm.w, bias=self.norm.b,
-                              eps=self.cfg.norm_eps)
-        return F.linear(h, self.head)
+        h = ops.residual_norm(hidden_rows.contiguous(), self.dtype, **self.norm.args)
+        y = F.linear(h, self.head)
+        return y if self.cfg.logit_softcap is None else ops.softcap(y, self.cfg.logit_softcap)

@@ -10,7 +10,13 @@ product and everything between the products into one or two kernels:
   convolution with its carried rows, rotation, unit norms, value mixing, append)
   -> paged attention -> ``pa_head_gate`` -> output projection;
 * ``LightningMixer``: joint projection -> ``pa_lightning_*`` (silu, recurrence)
-  -> ``pa_rms_gate`` -> output projection.
+  -> ``pa_rms_gate`` -> output projection;
+* ``MlstmMixer``: joint projection -> ``pa_gated_linear`` (gates, recurrence,
+  normaliser) -> ``pa_rms_gate`` per head -> output projection;
+* ``Mamba2Mixer``: joint projection -> ``pa_short_conv`` -> ``pa_gated_linear``
+  -> ``pa_rms_gate`` (gate first) -> output projection;
+* ``ParallelMixer``: two of them side by side with one joint input and one joint
+  output projection; their scales ride on the steps before the latter.
 """
 
 from __future__ import annotations
@@ -33,9 +39,22 @@ Getter = Callable[[str], Tensor]  # checkpoint tensor by name
 
 
 @dataclass(frozen=True)
+class YarnScaling:
+    """Rotary frequencies interpolated by parts: pairs that turn more than ``fast`` times over ``original`` positions keep
+    theirs, those that turn less than ``slow`` times are divided by ``factor``, with a ramp over the pairs between."""
+
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
 class AttentionSpec:
-    """Softmax attention over a sliding window behind short convolutions.  ``window`` None: plain causal; ``taps`` 0:
-    no convolution; ``v_mix``: the layer takes part in value mixing."""
+    """Softmax attention over a sliding window behind short convolutions.  ``window`` and ``chunk`` None: plain causal;
+    ``chunk``: keys of the query's own chunk of positions; ``taps`` 0: no convolution; ``v_mix``: the layer takes part in
+    value mixing; ``rot_halves``: dimension i turns with i + rot_dims / 2, else 2i with 2i + 1; ``qk_weights``: RMS norms of
+    q and k with weights ahead of the rotation, else norms without weights behind it; ``gates``: a gate per head."""
 
     heads: int
     kv_heads: int
@@ -48,6 +67,11 @@ class AttentionSpec:
     rot_base: float
     rot_factor: float = 1.0
     v_mix: bool = False
+    chunk: Optional[int] = None
+    rot_yarn: Optional[YarnScaling] = None
+    rot_halves: bool = False
+    qk_weights: bool = False
+    gates: bool = True
 
     def __post_init__(self) -> None:
         if self.heads % self.kv_heads != 0:
@@ -56,6 +80,8 @@ class AttentionSpec:
             raise ValueError(f"rot_dims={self.rot_dims} must be even and at most dim={self.dim}")
         if self.window is not None and self.window < 1:
             raise ValueError(f"window={self.window} must be positive")
+        if self.chunk is not None and (self.chunk < 1 or self.window is not None):
+            raise ValueError(f"chunk={self.chunk} must be positive, and no window beside it")
         if self.pool_dim > 256:
             raise ValueError(f"head sizes {self.dim} / {self.vdim} above 256")
 
@@ -67,6 +93,18 @@ class AttentionSpec:
     @property
     def channels(self) -> int:
         return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+    @property
+    def mask_window(self) -> int:
+        """The kernels' ``window``: positive a sliding window, negative chunks, 0 neither."""
+        return self.window or -(self.chunk or 0)
+
+    def head_order(self) -> Tensor:
+        """The order in which the dimensions of q and k heads are stored: pairs that turn together side by side."""
+        order = torch.arange(self.dim)
+        if self.rot_halves:
+            order[: self.rot_dims] = order[: self.rot_dims].view(2, -1).t().reshape(-1)
+        return order
 
 
 @dataclass(frozen=True)
@@ -85,23 +123,87 @@ class LightningSpec:
             raise ValueError(f"dim={self.dim} above 256")
 
 
+@dataclass(frozen=True)
+class MlstmSpec:
+    """Matrix memory with exponential gates under a soft cap."""
+
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+    def __post_init__(self) -> None:
+        if self.dim > 256:
+            raise ValueError(f"dim={self.dim} above 256")
+
+
+@dataclass(frozen=True)
+class Mamba2Spec:
+    """Mamba-2: a state of ``state`` x ``vdim`` per head, input and output vectors shared by the heads of a group."""
+
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    taps: int
+    norm_groups: int
+
+    def __post_init__(self) -> None:
+        if self.heads % self.groups or (self.heads * self.vdim) % self.norm_groups:
+            raise ValueError(f"{self.heads} heads of {self.vdim} do not divide into groups={self.groups} / norm_groups={self.norm_groups}")
+        if self.state > 256 or not 1 <= self.taps <= 8:
+            raise ValueError(f"state={self.state} above 256 or taps={self.taps} not in 1 .. 8")
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+
+@dataclass(frozen=True)
+class ParallelSpec:
+    """Attention and a recurrent mixer on the same input, their outputs added under two scales."""
+
+    left: AttentionSpec
+    right: MlstmSpec
+    left_scale: float = 1.0
+    right_scale: float = 1.0
+
+
+def yarn_frequencies(base: float, dims: int, yarn: YarnScaling) -> Tuple[Tensor, float]:
+    """float64 frequencies of the ``dims / 2`` pairs, and the factor on cosine and sine."""
+    def pair_of(turns: float) -> float:
+        return dims * math.log(yarn.original / (2 * math.pi * turns)) / (2 * math.log(base))
+
+    first, last = max(math.floor(pair_of(yarn.fast)), 0), min(math.ceil(pair_of(yarn.slow)), dims - 1)
+    pairs = torch.arange(dims // 2, dtype=torch.float64)
+    ramp = ((pairs - first) / max(last - first, 0.001)).clamp(0.0, 1.0)
+    freq = base ** (-2.0 * pairs / dims)
+    return freq / yarn.factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(yarn.factor) + 1.0
+
+
 class RotaryTables:
-    """(cos, sin) per position and pair, float32 from float64 angles; one table per (base, dims, factor), shared by the
-    layers that name it.  The position limit is fixed once a captured graph may hold a table's address."""
+    """(cos, sin) per position and pair, float32 from float64 angles; one table per (base, dims, factor, scaling), shared by
+    the layers that name it.  The position limit is fixed once a captured graph may hold a table's address."""
 
     def __init__(self, max_positions: int, device) -> None:
         self.max_positions = max_positions
         self.device = device
-        self._tables: Dict[Tuple[float, int, float], Tensor] = {}
+        self._tables: Dict[tuple, Tensor] = {}
 
-    def get(self, base: float, dims: int, factor: float) -> Optional[Tensor]:
+    def get(self, base: float, dims: int, factor: float, yarn: Optional[YarnScaling] = None) -> Optional[Tensor]:
         if dims == 0:
             return None
-        key = (base, dims, factor)
+        key = (base, dims, factor, yarn)
         if key not in self._tables:
-            freq = base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims) / factor
-            angle = torch.arange(self.max_positions, dtype=torch.float64)[:, None] * freq[None, :]
-            table = torch.stack([angle.cos(), angle.sin()], dim=-1).float()
+            freq, size = base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims), 1.0
+            if yarn is not None:
+                freq, size = yarn_frequencies(base, dims, yarn)
+            angle = torch.arange(self.max_positions, dtype=torch.float64)[:, None] * (freq / factor)[None, :]
+            table = (torch.stack([angle.cos(), angle.sin()], dim=-1) * size).float()
             self._tables[key] = table.contiguous().to(self.device)
         return self._tables[key]
 
@@ -125,16 +227,50 @@ def fill(dst: Tensor, src: Tensor, name: str) -> None:
     dst.copy_(src)
 
 
-class ConvAttention(nn.Module):
-    def __init__(self, spec: AttentionSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 rotary: RotaryTables, v_role: Optional[str], dtype: torch.dtype, device) -> None:
-        """``v_role``: None, "first" (the layer whose values the others mix in) or "mix"."""
+def _pad8(n: int) -> int:
+    return -(-n // 8) * 8
+
+
+Slices = Optional[Tuple[Tensor, Tensor]]
+
+
+class Mixer(nn.Module):
+    """A joint input product, ``mix`` between the products, an output product.  ``in_rows`` and ``out_cols`` are the sizes of
+    the two weights; a mixer that is part of another is handed its slices of that one's weights.  ``out_scale`` multiplies
+    what ``mix`` returns."""
+
+    def __init__(self, in_rows: int, out_cols: int, width: int, dtype: torch.dtype, device, slices: Slices = None,
+                 out_scale: float = 1.0) -> None:
         super().__init__()
+        self.out_scale = out_scale
+        if slices is None:
+            slices = _param(in_rows, width, dtype=dtype, device=device), _param(width, out_cols, dtype=dtype, device=device)
+        self.w_in, self.w_out = slices
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        raise NotImplementedError
+
+    def forward(self, h: Tensor, step: StepRows) -> Tensor:
+        return F.linear(self.mix(F.linear(h, self.w_in), step), self.w_out)
+
+
+class ConvAttention(Mixer):
+    @staticmethod
+    def sizes(spec: AttentionSpec) -> Tuple[int, int]:
+        return _pad8(spec.channels + (spec.heads if spec.gates else 0)), spec.heads * spec.vdim
+
+    def __init__(self, spec: AttentionSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
+                 rotary: RotaryTables, v_role: Optional[str], dtype: torch.dtype, device, slices: Slices = None,
+                 out_scale: float = 1.0) -> None:
+        """``v_role``: None, "first" (the layer whose values the others mix in) or "mix".  Rows of ``w_in``: q, k, v, head
+        gates, padding."""
+        super().__init__(*self.sizes(spec), width, dtype, device, slices, out_scale)
         self.spec, self.eps, self.layer_idx, self.backend, self.v_role = spec, eps, layer_idx, backend, v_role
         self.rotary = rotary
-        rows = spec.channels + spec.heads
-        self.w_in = _param(-(-rows // 8) * 8, width, dtype=dtype, device=device)  # q, k, v, head gates, padding
-        self.w_out = _param(width, spec.heads * spec.vdim, dtype=dtype, device=device)
+        self.q_norm = self.k_norm = None
+        if spec.qk_weights:
+            self.q_norm = _param(spec.dim, dtype=torch.float32, device=device)
+            self.k_norm = _param(spec.dim, dtype=torch.float32, device=device)
         self.conv = _param(spec.taps, spec.channels, dtype=torch.float32, device=device) if spec.taps else None
         self.v_lambda = _param(1, dtype=torch.float32, device=device)
         self.conv_state = None
@@ -143,41 +279,46 @@ class ConvAttention(nn.Module):
 
     def load(self, get: Getter, prefix: str) -> None:
         s, at = self.spec, 0
+        order = s.head_order()
         for name, n in (("q", s.heads * s.dim), ("k", s.kv_heads * s.dim), ("v", s.kv_heads * s.vdim)):
-            fill(self.w_in[at: at + n], get(prefix + name), prefix + name)
+            pick = slice(None)
+            if s.rot_halves and name != "v":  # (the scores do not change when q and k heads are stored in another order)
+                pick = (torch.arange(0, n, s.dim)[:, None] + order).reshape(-1)
+            fill(self.w_in[at: at + n], get(prefix + name)[pick], prefix + name)
             if self.conv is not None:
-                fill(self.conv[:, at: at + n], get(f"{prefix}{name}.conv").t(), f"{prefix}{name}.conv")
+                fill(self.conv[:, at: at + n], get(f"{prefix}{name}.conv")[pick].t(), f"{prefix}{name}.conv")
             at += n
-        fill(self.w_in[at: at + s.heads], get(prefix + "g"), prefix + "g")
+        if s.gates:
+            fill(self.w_in[at: at + s.heads], get(prefix + "g"), prefix + "g")
+        if s.qk_weights:
+            fill(self.q_norm, get(prefix + "q.norm")[order], prefix + "q.norm")
+            fill(self.k_norm, get(prefix + "k.norm")[order], prefix + "k.norm")
         fill(self.w_out, get(prefix + "o"), prefix + "o")
         if self.v_role == "mix":
             fill(self.v_lambda, get(prefix + "vmix").reshape(1), prefix + "vmix")
 
-    def forward(self, h: Tensor, step: StepRows) -> Tensor:
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s, packed = self.spec, step.packed
-        u = F.linear(h, self.w_in)
         if self.v_role == "first":
-            step.v_first = torch.empty((h.shape[0], s.kv_heads * s.vdim), dtype=h.dtype, device=h.device)
+            step.v_first = torch.empty((u.shape[0], s.kv_heads * s.vdim), dtype=u.dtype, device=u.device)
         kc, vc = self.backend._layer(self.layer_idx)
         # q carries scale * log2(e) from its 32-bit registers, so that the attention kernels' own factor is one
-        q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, s.scale / _LN2, self.eps, True,
-                                self.rotary.get(s.rot_base, s.rot_dims, s.rot_factor), s.rot_dims, self.conv, self.conv_state,
-                                self.v_role, step.v_first if self.v_role else None,
-                                self.v_lambda if self.v_role == "mix" else None)
-        o = self.backend.attend_packed(q, self.layer_idx, packed, _LN2, s.window or 0)
-        o = ops.head_gate(o, u[:, s.channels: s.channels + s.heads], s.vdim)
-        return F.linear(o, self.w_out)
+        q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, s.scale / _LN2, self.eps,
+                                not s.qk_weights, self.rotary.get(s.rot_base, s.rot_dims, s.rot_factor, s.rot_yarn), s.rot_dims,
+                                self.conv, self.conv_state, self.v_role, step.v_first if self.v_role else None,
+                                self.v_lambda if self.v_role == "mix" else None, q_norm=self.q_norm, k_norm=self.k_norm)
+        o = self.backend.attend_packed(q, self.layer_idx, packed, _LN2, s.mask_window)
+        gate = u[:, s.channels: s.channels + s.heads] if s.gates else None
+        return ops.head_gate(o, gate, s.vdim, self.out_scale, out)
 
 
-class LightningMixer(nn.Module):
+class LightningMixer(Mixer):
     def __init__(self, spec: LightningSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
                  dtype: torch.dtype, device) -> None:
-        super().__init__()
-        self.spec, self.eps, self.backend = spec, eps, backend
         inner = spec.heads * spec.vdim
-        rows = spec.heads * 2 * spec.dim + 2 * inner
-        self.w_in = _param(-(-rows // 8) * 8, width, dtype=dtype, device=device)  # q, k, v, output gate, padding
-        self.w_out = _param(width, inner, dtype=dtype, device=device)
+        # (rows of w_in: q, k, v, output gate, padding)
+        super().__init__(_pad8(spec.heads * 2 * spec.dim + 2 * inner), inner, width, dtype, device)
+        self.spec, self.eps, self.backend = spec, eps, backend
         self.norm = _param(inner, dtype=torch.float32, device=device)
         pad = lambda n: -(-n // 16) * 16
         self.state = backend.register_state(layer_idx, "lightning", (spec.heads, pad(spec.dim), pad(spec.vdim)), torch.float32)
@@ -192,11 +333,10 @@ class LightningMixer(nn.Module):
         fill(self.w_out, get(prefix + "o"), prefix + "o")
         fill(self.norm, get(prefix + "norm"), prefix + "norm")
 
-    def forward(self, h: Tensor, step: StepRows) -> Tensor:
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s, packed = self.spec, step.packed
-        u = F.linear(h, self.w_in)
         inner = s.heads * s.vdim
-        o = torch.empty((h.shape[0], inner), dtype=h.dtype, device=h.device)
+        o = torch.empty((u.shape[0], inner), dtype=u.dtype, device=u.device)
         nd = packed.num_decodes
         if packed.decodes is not None:
             ops.lightning(u[:nd], packed.decodes, self.state, self.decay_powers, s.heads, s.dim, s.vdim, o[:nd])
@@ -206,12 +346,135 @@ class LightningMixer(nn.Module):
             ops.lightning(u, c, self.state, self.decay_powers, s.heads, s.dim, s.vdim, o,
                           workspace=self.backend._workspace_for(need) if need else None)
         g = 2 * s.heads * s.dim + inner
-        o = ops.rms_gate(o, u[:, g: g + inner], self.norm, self.eps)
-        return F.linear(o, self.w_out)
+        return ops.rms_gate(o, u[:, g: g + inner], self.norm, self.eps, out=out)
+
+
+def _gated_rows(kind: str, q: Tensor, k: Tensor, v: Tensor, gates, constants, step: StepRows, state: Tensor, heads: int, dim: int,
+                vdim: int, backend: HipPagedAttentionBackend, **kw) -> Tensor:
+    """A gated recurrence over a step's rows: single tokens, then portions."""
+    packed = step.packed
+    out = torch.empty((v.shape[0], heads * vdim), dtype=v.dtype, device=v.device)
+    if packed.decodes is not None:
+        cut = lambda t: None if t is None else t[: packed.num_decodes]
+        ops.gated_linear(kind, cut(q), cut(k), cut(v), tuple(cut(g) for g in gates), constants, packed.decodes, state, heads, dim,
+                         vdim, cut(out), **kw)
+    if packed.chunks is not None:
+        c = packed.chunks
+        need = ops.gated_linear_workspace_bytes(c.ctx_lens.numel(), heads, dim, vdim, c.max_q_len)
+        ops.gated_linear(kind, q, k, v, gates, constants, c, state, heads, dim, vdim, out,
+                         workspace=backend._workspace_for(need) if need else None, **kw)
+    return out
+
+
+class MlstmMixer(Mixer):
+    DEN_EPS = 1e-6
+
+    @staticmethod
+    def sizes(spec: MlstmSpec) -> Tuple[int, int]:
+        inner = spec.heads * spec.vdim
+        return _pad8(2 * spec.heads * spec.dim + 2 * inner + 2 * spec.heads), inner
+
+    def __init__(self, spec: MlstmSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
+                 dtype: torch.dtype, device, slices: Slices = None, out_scale: float = 1.0) -> None:
+        """Rows of ``w_in``: q, k, v, output gate, input gates, forget gates, padding."""
+        super().__init__(*self.sizes(spec), width, dtype, device, slices, out_scale)
+        self.spec, self.eps, self.backend = spec, eps, backend
+        self.norm = _param(spec.heads * spec.vdim, dtype=torch.float32, device=device)  # times out_scale
+        self.i_bias = _param(spec.heads, dtype=torch.float32, device=device)
+        self.f_bias = _param(spec.heads, dtype=torch.float32, device=device)
+        floats = ops.gated_linear_state_floats("mlstm", spec.dim, spec.vdim)
+        self.state = backend.register_state(layer_idx, "mlstm", (spec.heads, floats), torch.float32)
+
+    def _parts(self) -> Tuple[Tuple[str, int], ...]:
+        s = self.spec
+        return (("q", s.heads * s.dim), ("k", s.heads * s.dim), ("v", s.heads * s.vdim), ("g", s.heads * s.vdim), ("i", s.heads),
+                ("f", s.heads))
+
+    def load(self, get: Getter, prefix: str) -> None:
+        at = 0
+        for name, n in self._parts():
+            fill(self.w_in[at: at + n], get(prefix + name), prefix + name)
+            at += n
+        fill(self.i_bias, get(prefix + "i.b"), prefix + "i.b")
+        fill(self.f_bias, get(prefix + "f.b"), prefix + "f.b")
+        fill(self.norm, get(prefix + "norm"), prefix + "norm")
+        self.norm.mul_(self.out_scale)
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s = self.spec
+        sizes = [n for _, n in self._parts()]
+        q, k, v, g, i, f = u[:, : sum(sizes)].split(sizes, dim=1)
+        o = _gated_rows("mlstm", q, k, v, (i, f), (self.i_bias, self.f_bias, None), step, self.state, s.heads, s.dim, s.vdim,
+                        self.backend, cap=s.gate_cap, q_scale=s.dim ** -0.5, den_eps=self.DEN_EPS)
+        return ops.rms_gate(o, g, self.norm, self.eps, groups=s.heads, out=out)
+
+
+class Mamba2Mixer(Mixer):
+    def __init__(self, spec: Mamba2Spec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
+                 dtype: torch.dtype, device) -> None:
+        """Rows of ``w_in``: gate, x, B, C, step sizes, padding."""
+        super().__init__(_pad8(spec.inner + spec.channels + spec.heads), spec.inner, width, dtype, device)
+        self.spec, self.eps, self.backend = spec, eps, backend
+        f32 = dict(dtype=torch.float32, device=device)
+        self.conv = _param(spec.taps, spec.channels, **f32)
+        self.conv_bias = _param(spec.channels, **f32)
+        self.dt_bias, self.rate, self.skip = (_param(spec.heads, **f32) for _ in range(3))
+        self.norm = _param(spec.inner, **f32)
+        self.conv_state = None
+        if spec.taps > 1:
+            self.conv_state = backend.register_state(layer_idx, "conv", (spec.taps - 1, spec.channels), dtype)
+        floats = ops.gated_linear_state_floats("ssd", spec.state, spec.vdim)
+        self.state = backend.register_state(layer_idx, "ssd", (spec.heads, floats), torch.float32)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        s = self.spec
+        fill(self.w_in[: s.inner + s.channels + s.heads], get(prefix + "in"), prefix + "in")
+        fill(self.conv, get(prefix + "conv").t(), prefix + "conv")
+        fill(self.conv_bias, get(prefix + "conv.b"), prefix + "conv.b")
+        fill(self.dt_bias, get(prefix + "dt_bias"), prefix + "dt_bias")
+        fill(self.rate, get(prefix + "A_log").float().exp(), prefix + "A_log")
+        fill(self.skip, get(prefix + "D"), prefix + "D")
+        fill(self.norm, get(prefix + "norm"), prefix + "norm")
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s = self.spec
+        z, x, dt = u[:, : s.inner + s.channels + s.heads].split([s.inner, s.channels, s.heads], dim=1)
+        x = ops.short_conv(x, step.packed.rows, self.conv, self.conv_bias, self.conv_state, "silu")
+        n = s.groups * s.state
+        x, b, c = x.split([s.inner, n, n], dim=1)
+        y = _gated_rows("ssd", c, b, x, (dt, None), (self.dt_bias, self.rate, self.skip), step, self.state, s.heads, s.state,
+                        s.vdim, self.backend, heads_per_group=s.heads // s.groups)
+        return ops.rms_gate(y, z, self.norm, self.eps, groups=s.norm_groups, order="silu_first", out=out)
+
+
+class ParallelMixer(Mixer):
+    def __init__(self, spec: ParallelSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
+                 rotary: RotaryTables, dtype: torch.dtype, device) -> None:
+        (in_l, in_r), (out_l, out_r) = zip(ConvAttention.sizes(spec.left), MlstmMixer.sizes(spec.right))
+        super().__init__(in_l + in_r, out_l + out_r, width, dtype, device)
+        self._in, self._out = in_l, out_l
+        self.left = ConvAttention(spec.left, width, eps, layer_idx, backend, rotary, None, dtype, device,
+                                  (self.w_in[: self._in], self.w_out[:, : self._out]), spec.left_scale)
+        self.right = MlstmMixer(spec.right, width, eps, layer_idx, backend, dtype, device,
+                                (self.w_in[self._in:], self.w_out[:, self._out:]), spec.right_scale)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        self.left.load(get, prefix + "left.")
+        self.right.load(get, prefix + "right.")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        if out is None:
+            out = torch.empty((u.shape[0], self.w_out.shape[1]), dtype=u.dtype, device=u.device)
+        self.left.mix(u[:, : self._in], step, out[:, : self._out])
+        self.right.mix(u[:, self._in:], step, out[:, self._out:])
+        return out
 
 
 class GatedMLP(nn.Module):
-    """``down(silu(gate h) * up h)`` with gate and up in one product."""
+    """``down(silu(gate h) * up h)`` with gate and up in one product.  ``branch`` returns what the residual sum adds, as
+    ``pa_residual_norm`` takes it."""
 
     def __init__(self, width: int, inner: int, dtype: torch.dtype, device) -> None:
         super().__init__()
@@ -227,6 +490,9 @@ class GatedMLP(nn.Module):
     def forward(self, h: Tensor) -> Tensor:
         u = F.linear(h, self.w_in)
         return F.linear(ops.glu(u[:, : self.inner], u[:, self.inner:], "silu"), self.w_out)
+
+    def branch(self, h: Tensor) -> Dict[str, Tensor]:
+        return {"y": self(h)}
 
 
 class TokenSide(nn.Module):

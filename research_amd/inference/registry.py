@@ -11,13 +11,13 @@ from __future__ import annotations
 import json
 import os
 from dataclasses import dataclass
-from typing import Callable, Dict, List
+from typing import Callable, Dict, List, Optional
 
 import torch
 from torch import Tensor, nn
 
 from .attention import CacheConfig, HipPagedAttentionBackend
-from .hybrid import HybridDecoder, lotozen_config
+from .hybrid import HybridConfig, HybridDecoder, lotozen_config, tevirax_config
 from .model import ModelConfig, PagedLlama
 
 DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
@@ -40,6 +40,7 @@ class ModelEntry:
     name: str
     matches: Callable[[dict], bool]
     build: Callable[[str, dict, LoadOptions], nn.Module]
+    positions: Callable[[dict], Optional[int]] = lambda config: None  # positions the design ends at, None: any
 
 
 _ENTRIES: List[ModelEntry] = []
@@ -80,15 +81,24 @@ def load_model(path: str, options: LoadOptions) -> nn.Module:
     return find(config).build(path, config, options)
 
 
+def model_len(path: str, wanted: int) -> int:
+    """``wanted``, or what the design of the folder has positions for."""
+    config = read_config(path)
+    limit = find(config).positions(config)
+    return wanted if limit is None else min(wanted, limit)
+
+
 # ------------------------------------------------------------------ entries
 
 
-def _build_lotozen(path: str, config: dict, o: LoadOptions) -> nn.Module:
-    cfg = lotozen_config(config)
-    backend = HipPagedAttentionBackend(cfg.cache_config(o.num_blocks, o.block_size, o.num_state_slots, o.dtype, o.device))
-    model = HybridDecoder(cfg, backend, o.max_positions, o.dtype)
-    model.load_state_dict(read_weights(path), strict=False)
-    return model.eval()
+def _hybrid(reader: Callable[[dict], HybridConfig]) -> Callable[[str, dict, LoadOptions], nn.Module]:
+    def build(path: str, config: dict, o: LoadOptions) -> nn.Module:
+        cfg = reader(config)
+        backend = HipPagedAttentionBackend(cfg.cache_config(o.num_blocks, o.block_size, o.num_state_slots, o.dtype, o.device))
+        model = HybridDecoder(cfg, backend, o.max_positions, o.dtype)
+        model.load_state_dict(read_weights(path), strict=False)
+        return model.eval()
+    return build
 
 
 def _build_llama(path: str, config: dict, o: LoadOptions) -> nn.Module:
@@ -99,5 +109,8 @@ def _build_llama(path: str, config: dict, o: LoadOptions) -> nn.Module:
     return PagedLlama.from_local(path, backend_for, dtype=o.dtype, device=o.device)
 
 
-register(ModelEntry("lotozen", lambda c: c.get("architecture") == "Lotozen", _build_lotozen))
-register(ModelEntry("llama", lambda c: "num_attention_heads" in c, _build_llama))
+register(ModelEntry("lotozen", lambda c: c.get("architecture") == "Lotozen", _hybrid(lotozen_config)))
+register(ModelEntry("tevirax", lambda c: c.get("architecture") == "Tevirax", _hybrid(tevirax_config),
+                    lambda c: int(c["max_positions"])))
+register(ModelEntry("llama", lambda c: "num_attention_heads" in c, _build_llama,
+                    lambda c: c.get("max_position_embeddings")))

@@ -75,11 +75,12 @@ def main(argv: Optional[List[str]] = None) -> int:
     if not os.path.exists(_lib.LIB_PATH):
         build.build(jobs=min(16, os.cpu_count() or 1))
     from .engine import InferenceEngine
+    from .registry import model_len
 
     torch.backends.cuda.matmul.allow_tf32 = False  # float32 means float32
     blocks = max(1, -(-args.max_tokens // BLOCK_SIZE))
     engine = InferenceEngine(EngineConfig(
         model_path=args.model, cache_type="private", block_size=BLOCK_SIZE, max_batch_size=args.max_sequences,
-        max_model_len=args.max_tokens, num_kv_blocks=blocks, dtype=args.dtype))
+        max_model_len=model_len(args.model, args.max_tokens), num_kv_blocks=blocks, dtype=args.dtype))
     replay(engine, sys.stdin, args.out, sys.stdout)
     return 0

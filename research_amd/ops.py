@@ -86,7 +86,7 @@ def decode(q: Tensor, k_cache: Tensor, v_cache: Tensor, block_tables: Tensor, se
     """Paged decode attention; q ``[B, Hq, D]`` -> out ``[B, Hq, D]`` (same dtype).
 
     ``entry`` may name ``pa_decode_split`` or ``pa_decode_reduce`` to run one pass only; ``window`` > 0
-    restricts every sequence to its last ``window`` keys.
+    restricts every sequence to its last ``window`` keys, < 0 to its last chunk of ``-window`` positions.
     """
     batch, hq, d = q.shape
     total_slots, hkv, _ = k_cache.shape
@@ -134,7 +134,8 @@ def prefill_paged(q: Tensor, k_cache: Tensor, v_cache: Tensor, block_tables: Ten
                   out: Optional[Tensor] = None, window: int = 0, row_first_key: Optional[Tensor] = None,
                   rowwise: bool = False, workspace: Optional[Tensor] = None) -> Tensor:
     """Causal prefill over a paged context; q ``[total_q, Hq, D]`` packed rows; ``window`` > 0 adds the
-    sliding window (a row at position p sees keys p - window < j <= p); ``row_first_key`` (int32 per q row,
+    sliding window (a row at position p sees keys p - window < j <= p), < 0 chunks of ``-window`` positions (it sees
+    keys of its own chunk); ``row_first_key`` (int32 per q row,
     non-decreasing along a sequence) adds a per-row first key, e.g. the start of the row's document;
     ``rowwise`` selects the vector kernel (``pa_prefill_paged_rowwise``) also where a matrix-core kernel exists;
     ``workspace`` (uint8, ``prefill_workspace_bytes`` or more) lets a launch of few rows split its keys over
@@ -351,49 +352,68 @@ def _typed(dtype: torch.dtype, *tensors: Optional[Tensor]) -> None:
 
 
 _NORMS = {None: _lib.PA_NORM_NONE, "layer": _lib.PA_NORM_LAYER, "rms": _lib.PA_NORM_RMS}
-_ACTS = {"silu": _lib.PA_ACT_SILU, "gelu_tanh": _lib.PA_ACT_GELU_TANH}
+_ACTS = {"silu": _lib.PA_ACT_SILU, "gelu_tanh": _lib.PA_ACT_GELU_TANH, None: _lib.PA_ACT_NONE}
+_GATES = {"sigmoid_last": _lib.PA_GATE_SIGMOID_LAST, "silu_first": _lib.PA_GATE_SILU_FIRST}
+_GATED = {"ssd": _lib.PA_GL_SSD, "mlstm": _lib.PA_GL_MLSTM}
 _V_MODES = {None: _lib.PA_V_PLAIN, "first": _lib.PA_V_FIRST, "mix": _lib.PA_V_MIX}
 
 
 def residual_norm(x: Tensor, dtype: torch.dtype, y: Optional[Tensor] = None, y_weight: Optional[Tensor] = None,
                   y_eps: float = 0.0, ids: Optional[Tensor] = None, table: Optional[Tensor] = None,
                   row_index: Optional[Tensor] = None, norm: Optional[str] = None, weight: Optional[Tensor] = None,
-                  bias: Optional[Tensor] = None, eps: float = 0.0, want_out: bool = True) -> Optional[Tensor]:
+                  bias: Optional[Tensor] = None, eps: float = 0.0, want_out: bool = True, table_scale: float = 1.0,
+                  positions: Optional[Tensor] = None, pos_table: Optional[Tensor] = None, mix: Optional[Tensor] = None,
+                  y_extra: Optional[Tensor] = None) -> Optional[Tensor]:
     """Residual sum and norm in one pass over the rows (``pa_residual_norm``): ``x`` float32 ``[rows, width]`` is
-    updated in place (``table[ids]`` or itself, plus ``y`` or its RMS norm times ``y_weight``), and
-    ``norm(x) * weight + bias`` (``"layer"``, ``"rms"`` or None: a cast) comes back in ``dtype``.  ``row_index``
-    picks rows of ``x`` instead of updating it."""
+    updated in place (``table[ids] * table_scale``, with ``positions`` also their rows of ``pos_table``, or itself,
+    plus ``y`` or its RMS norm times ``y_weight``), and ``norm(x) * weight + bias`` (``"layer"``, ``"rms"`` or None: a
+    cast) comes back in ``dtype``.  With ``mix`` float32 ``[rows, m + 1]`` the branch is a weighted sum: of ``y``
+    ``[rows * m, width]``, m rows each, and of ``y_extra``.  ``row_index`` picks rows of ``x`` instead of updating it."""
     rows, width = x.shape
-    _dense(x, y, y_weight, ids, table, row_index, weight, bias)
-    _typed(torch.float32, x, y_weight, weight, bias)
-    _typed(torch.int64, ids, row_index)
-    _typed(dtype, y, table)
+    _dense(x, y, y_weight, ids, table, row_index, weight, bias, positions, pos_table, mix, y_extra)
+    _typed(torch.float32, x, y_weight, weight, bias, mix)
+    _typed(torch.int64, ids, row_index, positions)
+    _typed(dtype, y, table, pos_table, y_extra)
     n = rows if row_index is None else row_index.numel()
-    if (y is not None and tuple(y.shape) != (rows, width)) or (ids is not None and ids.numel() != rows):
+    m = mix.shape[1] - 1 if mix is not None else 0
+    if (y is not None and tuple(y.shape) != (rows * (m or 1), width)) or (ids is not None and ids.numel() != rows):
         raise ValueError("y / ids do not fit the residual")
-    if table is not None and table.shape[1] != width:
-        raise ValueError("table rows are not as wide as the residual")
+    if (mix is not None and mix.shape[0] != rows) or (y_extra is not None and tuple(y_extra.shape) != (rows, width)):
+        raise ValueError("mix / y_extra do not fit the residual")
+    if positions is not None and positions.numel() != rows:
+        raise ValueError("positions do not fit the residual")
+    for t in (table, pos_table):
+        if t is not None and t.shape[1] != width:
+            raise ValueError("table rows are not as wide as the residual")
     for w in (y_weight, weight, bias):
         if w is not None and w.numel() != width:
             raise ValueError("norm weights are not as wide as the residual")
     out = torch.empty((n, width), dtype=dtype, device=x.device) if want_out else None
-    _run("pa_residual_norm", _ptr(x), _ptr(y), _ptr(y_weight), float(y_eps), _ptr(ids), _ptr(table),
-         table.shape[0] if table is not None else 0, _ptr(row_index), rows, _ptr(weight), _ptr(bias), float(eps),
+    _run("pa_residual_norm", _ptr(x), _ptr(y), _ptr(mix), m, _ptr(y_extra), _ptr(y_weight), float(y_eps), _ptr(ids), _ptr(table),
+         table.shape[0] if table is not None else 0, float(table_scale), _ptr(positions), _ptr(pos_table),
+         pos_table.shape[0] if pos_table is not None else 0, _ptr(row_index), rows, _ptr(weight), _ptr(bias), float(eps),
          _NORMS[norm], _ptr(out), n, width, PA_DTYPE[dtype], _stream(x))
     return out
 
 
-def rms_gate(o: Tensor, gate: Tensor, weight: Tensor, eps: float) -> Tensor:
-    """``o / rms(o) * weight * sigmoid(gate)`` per row (``pa_rms_gate``); ``gate`` may be a column slice."""
+def rms_gate(o: Tensor, gate: Tensor, weight: Tensor, eps: float, groups: int = 1, order: str = "sigmoid_last",
+             out: Optional[Tensor] = None) -> Tensor:
+    """The gated RMS norm of every one of ``groups`` equal parts of a row (``pa_rms_gate``): ``"sigmoid_last"``:
+    ``o / rms(o) * weight * sigmoid(gate)``; ``"silu_first"``: ``z / rms(z) * weight`` of ``z = o * silu(gate)``.
+    ``gate`` and ``out`` may be column slices."""
     rows, width = o.shape
     _dense(o, weight)
     _typed(o.dtype, gate)
     _typed(torch.float32, weight)
     if tuple(gate.shape) != (rows, width) or weight.numel() != width:
         raise ValueError("gate / weight do not fit o")
-    out = torch.empty_like(o)
-    _run("pa_rms_gate", _ptr(o), _ptr(gate), _row_stride(gate), _ptr(weight), float(eps), _ptr(out), rows, width,
-         PA_DTYPE[o.dtype], _stream(o))
+    if out is None:
+        out = torch.empty_like(o)
+    _typed(o.dtype, out)
+    if tuple(out.shape) != (rows, width):
+        raise ValueError("out does not fit o")
+    _run("pa_rms_gate", _ptr(o), _ptr(gate), _row_stride(gate), _ptr(weight), float(eps), _ptr(out), _row_stride(out), rows,
+         width, groups, _GATES[order], PA_DTYPE[o.dtype], _stream(o))
     return out
 
 
@@ -411,18 +431,22 @@ def glu(gate: Tensor, up: Tensor, act: str, ids: Optional[Tensor] = None) -> Ten
     return out
 
 
-def head_gate(o: Tensor, gate: Optional[Tensor], vdim: int) -> Tensor:
-    """``[rows, heads, d]`` -> ``[rows, heads * vdim]``: the leading ``vdim`` of every head times the sigmoid of its
-    gate logit (``pa_head_gate``)."""
+def head_gate(o: Tensor, gate: Optional[Tensor], vdim: int, scale: float = 1.0, out: Optional[Tensor] = None) -> Tensor:
+    """``[rows, heads, d]`` -> ``[rows, heads * vdim]``: the leading ``vdim`` of every head times ``scale`` and the
+    sigmoid of its gate logit (``pa_head_gate``); ``out`` may be a column slice."""
     rows, heads, d = o.shape
     _dense(o)
     if gate is not None:
         _typed(o.dtype, gate)
         if tuple(gate.shape) != (rows, heads):
             raise ValueError("gate must hold one logit per row and head")
-    out = torch.empty((rows, heads * vdim), dtype=o.dtype, device=o.device)
-    _run("pa_head_gate", _ptr(o), _ptr(gate), _row_stride(gate) if gate is not None else 0, _ptr(out), rows, heads, d, vdim,
-         PA_DTYPE[o.dtype], _stream(o))
+    if out is None:
+        out = torch.empty((rows, heads * vdim), dtype=o.dtype, device=o.device)
+    _typed(o.dtype, out)
+    if tuple(out.shape) != (rows, heads * vdim):
+        raise ValueError("out does not fit o")
+    _run("pa_head_gate", _ptr(o), _ptr(gate), _row_stride(gate) if gate is not None else 0, float(scale), _ptr(out),
+         _row_stride(out), rows, heads, d, vdim, PA_DTYPE[o.dtype], _stream(o))
     return out
 
 
@@ -442,17 +466,22 @@ def qkv_conv_append(u: Tensor, portions: Portions, slots: Tensor, k_cache: Tenso
                     dim: int, vdim: int, q_scale: float, eps: float, unit_norm: bool, rope: Optional[Tensor], rot_dims: int,
                     conv_weight: Optional[Tensor], conv_state: Optional[Tensor], v_mode: Optional[str] = None,
                     v_first: Optional[Tensor] = None, v_lambda: Optional[Tensor] = None,
-                    q_out: Optional[Tensor] = None) -> Tensor:
+                    q_out: Optional[Tensor] = None, q_norm: Optional[Tensor] = None,
+                    k_norm: Optional[Tensor] = None) -> Tensor:
     """Projection rows to rotated, normalised q and appended k / v (``pa_qkv_conv_append``).  Returns q
-    ``[rows, Hq, D]`` with D the pool's head size; k and v go to ``k_cache`` / ``v_cache`` ``[slots, Hkv, D]``."""
+    ``[rows, Hq, D]`` with D the pool's head size; k and v go to ``k_cache`` / ``v_cache`` ``[slots, Hkv, D]``.
+    ``q_norm`` / ``k_norm`` float32 ``[dim]``: weights of RMS norms ahead of the rotation."""
     rows = u.shape[0]
     total_slots, hkv, d = k_cache.shape
     taps = conv_weight.shape[0] if conv_weight is not None else 1
     channels = (num_q_heads + hkv) * dim + hkv * vdim
-    _dense(slots, k_cache, v_cache, rope, conv_weight, conv_state, v_first, *portions[:5])
+    _dense(slots, k_cache, v_cache, rope, conv_weight, conv_state, v_first, q_norm, k_norm, *portions[:5])
     _typed(u.dtype, k_cache, v_cache, conv_state, v_first)
     _typed(torch.int32, *portions[:5])
-    _typed(torch.float32, rope, conv_weight, v_lambda)
+    _typed(torch.float32, rope, conv_weight, v_lambda, q_norm, k_norm)
+    for t in (q_norm, k_norm):
+        if t is not None and t.numel() != dim:
+            raise ValueError("q_norm / k_norm must hold one weight per dimension")
     _typed(torch.int64, slots)
     batch = portions.ctx_lens.numel()
     if slots.numel() != rows or v_cache.shape != k_cache.shape or u.shape[1] < channels:
@@ -470,8 +499,8 @@ def qkv_conv_append(u: Tensor, portions: Portions, slots: Tensor, k_cache: Tenso
          conv_state.shape[0] if conv_state is not None else 0, _ptr(rope), rope.shape[0] if rope is not None else 0,
          rot_dims if rope is not None else 0, _ptr(portions.ctx_lens), _ptr(portions.q_lens), _ptr(portions.q_starts),
          _ptr(portions.state_slots), _ptr(portions.tiles), n_tiles, batch, _ptr(slots), total_slots, _ptr(q_out),
-         _ptr(k_cache), _ptr(v_cache), _ptr(v_first), _ptr(v_lambda), _V_MODES[v_mode], num_q_heads, hkv, dim, vdim, d,
-         int(unit_norm), float(eps), float(q_scale), PA_DTYPE[u.dtype], _stream(u))
+         _ptr(k_cache), _ptr(v_cache), _ptr(v_first), _ptr(v_lambda), _V_MODES[v_mode], _ptr(q_norm), _ptr(k_norm),
+         num_q_heads, hkv, dim, vdim, d, int(unit_norm), float(eps), float(q_scale), PA_DTYPE[u.dtype], _stream(u))
     return q_out
 
 
@@ -508,4 +537,132 @@ def lightning(u: Tensor, portions: Portions, state: Tensor, decay_powers: Tensor
     else:
         _run("pa_lightning_chunked", *head, portions.max_q_len, *tail, _ptr(workspace),
              workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(u))
+    return out
+
+
+def softcap(x: Tensor, cap: float) -> Tensor:
+    """``cap * tanh(x / cap)`` as float32 (``pa_softcap``)."""
+    _dense(x)
+    out = torch.empty(x.shape, dtype=torch.float32, device=x.device)
+    _run("pa_softcap", _ptr(x), _ptr(out), x.numel(), float(cap), PA_DTYPE[x.dtype], _stream(x))
+    return out
+
+
+def short_conv(u: Tensor, portions: Portions, weight: Tensor, bias: Optional[Tensor], conv_state: Optional[Tensor],
+               act: Optional[str]) -> Tensor:
+    """Causal convolution over time with its carried rows (``pa_short_conv``): ``u`` ``[rows, channels]`` (may be a column
+    slice), ``weight`` float32 ``[taps, channels]``, ``conv_state`` ``[slots, taps - 1, channels]``."""
+    rows, channels = u.shape
+    taps = weight.shape[0]
+    _dense(weight, bias, conv_state, *portions[:5])
+    _typed(torch.float32, weight, bias)
+    _typed(torch.int32, *portions[:5])
+    _typed(u.dtype, conv_state)
+    if weight.shape[1] != channels or (bias is not None and bias.numel() != channels):
+        raise ValueError("weight / bias do not fit u")
+    if taps > 1 and (conv_state is None or tuple(conv_state.shape[1:]) != (taps - 1, channels)):
+        raise ValueError("carried rows of another size")
+    batch = portions.ctx_lens.numel()
+    out = torch.empty((rows, channels), dtype=u.dtype, device=u.device)
+    _run("pa_short_conv", _ptr(u), _row_stride(u), rows, _ptr(weight), _ptr(bias), taps, _ACTS[act], _ptr(conv_state),
+         conv_state.shape[0] if conv_state is not None else 0, _ptr(portions.ctx_lens), _ptr(portions.q_lens),
+         _ptr(portions.q_starts), _ptr(portions.state_slots), _ptr(portions.tiles),
+         batch if portions.tiles is None else portions.tiles.shape[0], batch, _ptr(out), channels, PA_DTYPE[u.dtype], _stream(u))
+    return out
+
+
+def gated_linear_state_floats(kind: str, dim: int, vdim: int) -> int:
+    """Floats per head of a gated recurrence's state."""
+    return int(_lib.load().pa_gated_linear_state_floats(_GATED[kind], dim, vdim))
+
+
+def gated_linear_workspace_bytes(batch: int, heads: int, dim: int, vdim: int, max_q_len: int) -> int:
+    return int(_lib.load().pa_gated_linear_workspace_bytes(batch, heads, dim, vdim, max_q_len))
+
+
+def gated_linear(kind: str, q: Tensor, k: Tensor, v: Tensor, gates: Tuple[Tensor, Optional[Tensor]],
+                 constants: Tuple[Tensor, Tensor, Optional[Tensor]], portions: Portions, state: Tensor, heads: int, dim: int,
+                 vdim: int, out: Tensor, heads_per_group: int = 1, cap: float = 1.0, q_scale: float = 1.0, den_eps: float = 0.0,
+                 workspace: Optional[Tensor] = None) -> Tensor:
+    """A linear recurrence with gates per token and head (``pa_gated_linear``), ``kind`` ``"ssd"`` or ``"mlstm"``.  q, k, v
+    and the gates ``[rows, heads]`` may be column slices; ``constants`` float32 ``[heads]`` each: dt bias, decay rate and
+    skip, or the biases of the two gates; ``state`` float32 ``[slots, heads, gated_linear_state_floats]``."""
+    rows, batch = v.shape[0], portions.ctx_lens.numel()
+    ga, gb = gates
+    _dense(state, out, *constants, *portions[:4])
+    _typed(torch.int32, *portions[:4])
+    _typed(torch.float32, state, *constants)
+    _typed(v.dtype, q, k, ga, gb, out)
+    qk = (rows, heads // heads_per_group * dim)
+    if tuple(q.shape) != qk or tuple(k.shape) != qk or tuple(v.shape) != (rows, heads * vdim) or out.shape != v.shape:
+        raise ValueError("q / k / v / out do not fit each other")
+    if any(c is not None and c.numel() != heads for c in constants) or tuple(ga.shape) != (rows, heads):
+        raise ValueError("gates / constants do not fit the heads")
+    if gb is not None and (tuple(gb.shape) != (rows, heads) or _row_stride(gb) != _row_stride(ga)):
+        raise ValueError("the two gates differ in their rows")
+    if tuple(state.shape[1:]) != (heads, gated_linear_state_floats(kind, dim, vdim)):
+        raise ValueError("state of another size")
+    _run("pa_gated_linear", _GATED[kind], _ptr(q), _row_stride(q), _ptr(k), _row_stride(k), _ptr(v), _row_stride(v),
+         heads_per_group, _ptr(ga), _ptr(gb), _row_stride(ga), *(_ptr(c) for c in constants), float(cap), float(q_scale),
+         float(den_eps), rows, _ptr(state), state.shape[0], _ptr(portions.ctx_lens), _ptr(portions.q_lens),
+         _ptr(portions.q_starts), _ptr(portions.state_slots), batch, portions.max_q_len, _ptr(out), heads, dim, vdim,
+         PA_DTYPE[v.dtype], _ptr(workspace), workspace.numel() * workspace.element_size() if workspace is not None else 0,
+         _stream(v))
+    return out
+
+
+def narrow_linear(x: Tensor, w: Tensor) -> Tensor:
+    """``x w^T`` summed and returned in float32 (``pa_narrow_linear``), for a few outputs."""
+    _dense(w)
+    _typed(x.dtype, w)
+    if w.shape[1] != x.shape[1]:
+        raise ValueError("w does not fit x")
+    out = torch.empty((x.shape[0], w.shape[0]), dtype=torch.float32, device=x.device)
+    _run("pa_narrow_linear", _ptr(x), _row_stride(x), _ptr(w), _ptr(out), x.shape[0], w.shape[0], w.shape[1],
+         PA_DTYPE[x.dtype], _stream(x))
+    return out
+
+
+class ExpertChoice(NamedTuple):
+    """Which experts every row uses: ``ids`` int32 ``[rows, top]``, ``weights`` float32 ``[rows, top + 1]`` (the last one the
+    shared expert's) and, per expert, how many and which items (row * top + place)."""
+
+    ids: Tensor
+    weights: Tensor
+    counts: Tensor
+    lists: Tensor
+
+
+def moe_choose(logits: Tensor, experts: int, top: int, groups: int, keep: int) -> ExpertChoice:
+    """``pa_moe_select`` and ``pa_moe_lists`` over float32 ``logits`` ``[rows, experts]``, or one column more for the gate of a
+    shared expert."""
+    rows = logits.shape[0]
+    _dense(logits)
+    _typed(torch.float32, logits)
+    if logits.shape[1] not in (experts, experts + 1):
+        raise ValueError("logits must hold one column per expert, and one for a shared expert")
+    dev = logits.device
+    ids = torch.empty((rows, top), dtype=torch.int32, device=dev)
+    weights = torch.empty((rows, top + 1), dtype=torch.float32, device=dev)
+    counts = torch.empty(experts, dtype=torch.int32, device=dev)
+    lists = torch.empty((experts, rows), dtype=torch.int32, device=dev)
+    _run("pa_moe_select", _ptr(logits), logits.shape[1], rows, experts, top, groups, keep, int(logits.shape[1] > experts),
+         _ptr(ids), _ptr(weights), _stream(logits))
+    _run("pa_moe_lists", _ptr(ids), rows, top, experts, _ptr(counts), _ptr(lists), _stream(logits))
+    return ExpertChoice(ids, weights, counts, lists)
+
+
+def moe_product(x: Tensor, choice: ExpertChoice, w: Tensor, n: int, k: int, glu: bool) -> Tensor:
+    """Every item's product with its expert's weights (``pa_moe_product``): ``x`` ``[rows, k]`` or one row per item,
+    ``w`` ``[experts, n (glu: 2n), stride]`` zero past k -> ``[rows * top, n]``."""
+    rows, top = choice.ids.shape
+    _dense(w, *choice)
+    _typed(x.dtype, w)
+    if x.shape[0] not in (rows, rows * top) or x.shape[1] != k:
+        raise ValueError("x does not fit the choice")
+    if w.shape[0] != choice.counts.numel() or w.shape[1] < n * (2 if glu else 1) or w.shape[2] < k:
+        raise ValueError("w does not fit the choice")
+    out = torch.empty((rows * top, n), dtype=x.dtype, device=x.device)
+    _run("pa_moe_product", _ptr(x), _row_stride(x), rows * top // x.shape[0] if x.shape[0] else 1, _ptr(w), w.shape[1], w.shape[2], k,
+         _ptr(choice.counts), _ptr(choice.lists), rows, top, w.shape[0], int(glu), _ptr(out), n, PA_DTYPE[x.dtype], _stream(x))
     return out

@@ -33,7 +33,7 @@ def test_binding_table_matches_header():
 
 def test_version_and_dtype_sizes():
     lib = _lib.load()
-    assert lib.pa_version() == 7
+    assert lib.pa_version() == 8
     assert [lib.pa_dtype_bytes(c) for c in (0, 1, 2, 3, 4, -1)] == [4, 2, 2, 1, 0, 0]
 
 
@@ -229,35 +229,43 @@ def test_generated_prefill_loop_is_current(tmp_path, script, generated):
 def test_block_entry_points_check_their_arguments():
     """The kernels around attention in hybrid blocks: rejected before any device call."""
     f32, bf16 = _lib.PA_F32, _lib.PA_BF16
-    residual = lambda **kw: [{**dict(x=FAKE, y=FAKE, yw=None, ye=0.0, ids=None, table=None, tr=0, ri=None, xr=4, w=FAKE, b=FAKE,
-                                     eps=1e-6, norm=_lib.PA_NORM_LAYER, out=FAKE, rows=4, width=64, dt=bf16, s=None), **kw}[k]
-                             for k in ("x", "y", "yw", "ye", "ids", "table", "tr", "ri", "xr", "w", "b", "eps", "norm", "out",
-                                       "rows", "width", "dt", "s")]
+    residual = lambda **kw: [{**dict(x=FAKE, y=FAKE, mw=None, mix=0, yx=None, yw=None, ye=0.0, ids=None, table=None, tr=0,
+                                     ts=1.0, pos=None, pt=None, pr=0, ri=None, xr=4, w=FAKE, b=FAKE, eps=1e-6,
+                                     norm=_lib.PA_NORM_LAYER, out=FAKE, rows=4, width=64, dt=bf16, s=None), **kw}[k]
+                             for k in ("x", "y", "mw", "mix", "yx", "yw", "ye", "ids", "table", "tr", "ts", "pos", "pt", "pr", "ri",
+                                       "xr", "w", "b", "eps", "norm", "out", "rows", "width", "dt", "s")]
     for kw, status, text in ((dict(x=None), -1, "neither"), (dict(norm=7), -1, "norm=7"), (dict(width=20000), -2, "above"),
                              (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(ids=FAKE), -1, "table"), (dict(ri=FAKE), -1, "row_index"),
                              (dict(y=None, out=None), -1, "nothing"), (dict(y=None, yw=FAKE), -1, "y_weight"),
-                             (dict(norm=_lib.PA_NORM_NONE), -1, "without a norm")):
+                             (dict(norm=_lib.PA_NORM_NONE), -1, "without a norm"), (dict(pos=FAKE, pt=FAKE), -1, "positions"),
+                             (dict(mw=FAKE), -1, "mix_weight"), (dict(yx=FAKE), -1, "y_extra")):
         rc, msg = _status("pa_residual_norm", *residual(**kw))
         assert rc == status and text in msg, (kw, msg)
     assert _status("pa_residual_norm", *residual(rows=0, x=None))[0] == 0
-    rc, msg = _status("pa_rms_gate", FAKE, FAKE, 60, FAKE, 1e-6, FAKE, 4, 64, f32, None)
+    rc, msg = _status("pa_rms_gate", FAKE, FAKE, 60, FAKE, 1e-6, FAKE, 64, 4, 64, 1, 0, f32, None)
     assert rc == -1 and "gate_stride" in msg
+    rc, msg = _status("pa_rms_gate", FAKE, FAKE, 64, FAKE, 1e-6, FAKE, 60, 4, 64, 1, 0, f32, None)
+    assert rc == -1 and "out_stride" in msg
+    rc, msg = _status("pa_rms_gate", FAKE, FAKE, 64, FAKE, 1e-6, FAKE, 64, 4, 64, 3, 0, f32, None)
+    assert rc == -1 and "equal groups" in msg
+    rc, msg = _status("pa_softcap", FAKE, FAKE, 4, 0.0, f32, None)
+    assert rc == -1 and "cap" in msg
     rc, msg = _status("pa_glu", FAKE, 64, FAKE, 64, None, 0, FAKE, 4, 64, 9, f32, None)
     assert rc == -1 and "act" in msg
-    rc, msg = _status("pa_head_gate", FAKE, FAKE, 4, FAKE, 4, 4, 16, 24, f32, None)
+    rc, msg = _status("pa_head_gate", FAKE, FAKE, 4, 1.0, FAKE, 96, 4, 4, 16, 24, f32, None)
     assert rc == -1 and "sizes" in msg
 
     qkv = lambda **kw: [{**dict(u=FAKE, ld=200, n=4, cw=FAKE, taps=3, cs=FAKE, sr=2, rope=FAKE, rr=9, rot=8, cl=FAKE, ql=None,
                                 qs=None, ss=FAKE, tiles=None, nt=4, batch=4, slots=FAKE, ts=64, q=FAKE, k=FAKE, v=FAKE, vf=None,
-                                lam=None, vm=0, hq=4, hkv=2, dim=16, vdim=24, d=24, un=1, eps=1e-6, qsc=1.0, dt=bf16, s=None),
+                                lam=None, vm=0, qn=None, kn=None, hq=4, hkv=2, dim=16, vdim=24, d=24, un=1, eps=1e-6, qsc=1.0, dt=bf16, s=None),
                            **kw}[k] for k in ("u", "ld", "n", "cw", "taps", "cs", "sr", "rope", "rr", "rot", "cl", "ql", "qs", "ss",
-                                              "tiles", "nt", "batch", "slots", "ts", "q", "k", "v", "vf", "lam", "vm", "hq", "hkv",
+                                              "tiles", "nt", "batch", "slots", "ts", "q", "k", "v", "vf", "lam", "vm", "qn", "kn", "hq", "hkv",
                                               "dim", "vdim", "d", "un", "eps", "qsc", "dt", "s")]
     for kw, status, text in ((dict(hkv=3), -1, "multiple"), (dict(d=20), -1, "pool_dim"), (dict(rot=9), -1, "rot_dims"),
                              (dict(taps=9), -2, "taps"), (dict(cw=None), -1, "convolution"), (dict(cs=None), -1, "carried"),
                              (dict(rope=None), -1, "table"), (dict(vm=2, vf=FAKE), -1, "v_lambda"), (dict(vm=1), -1, "v_first"),
                              (dict(nt=3), -1, "one row"), (dict(ld=100), -1, "u_stride"), (dict(tiles=FAKE), -1, "tiles"),
-                             (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(d=264), -2, "above 256")):
+                             (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(d=264), -2, "above 256"), (dict(qn=FAKE), -1, "together")):
         rc, msg = _status("pa_qkv_conv_append", *qkv(**kw))
         assert rc == status and text in msg, (kw, msg)
     assert _status("pa_qkv_conv_append", *qkv(n=0, u=None, batch=0, nt=0))[0] == 0
@@ -275,3 +283,50 @@ def test_block_entry_points_check_their_arguments():
     rc, msg = _status("pa_lightning_recurrent", FAKE, 200, 1, FAKE, 2, FAKE, FAKE, None, None, FAKE, 2, FAKE, 2, 16, 24, f32, None)
     assert rc == -1 and "below batch" in msg
     assert lib.pa_lightning_workspace_bytes(-1, 2, 16, 24, 8) == 0 and "pa_lightning_workspace_bytes" in _lib.last_error()
+
+
+def test_recurrence_and_expert_entry_points_check_their_arguments():
+    f32, bf16 = _lib.PA_F32, _lib.PA_BF16
+    conv = lambda **kw: [{**dict(u=FAKE, ld=64, n=4, w=FAKE, b=None, taps=3, act=_lib.PA_ACT_SILU, cs=FAKE, sr=2, cl=FAKE, ql=None,
+                                 qs=None, ss=FAKE, tiles=None, nt=4, batch=4, out=FAKE, ch=48, dt=bf16, s=None), **kw}[k]
+                         for k in ("u", "ld", "n", "w", "b", "taps", "act", "cs", "sr", "cl", "ql", "qs", "ss", "tiles", "nt", "batch",
+                                   "out", "ch", "dt", "s")]
+    for kw, status, text in ((dict(ld=40), -1, "u_stride"), (dict(taps=9), -2, "taps"), (dict(act=1), -1, "act"), (dict(cs=None), -1, "carried"),
+                             (dict(nt=3), -1, "one row"), (dict(tiles=FAKE), -1, "tiles"), (dict(dt=_lib.PA_F16), -2, "dtype")):
+        rc, msg = _status("pa_short_conv", *conv(**kw))
+        assert rc == status and text in msg, (kw, msg)
+
+    lib = _lib.load()
+    assert lib.pa_gated_linear_state_floats(_lib.PA_GL_SSD, 20, 130) == 32 * 144
+    assert lib.pa_gated_linear_state_floats(_lib.PA_GL_MLSTM, 20, 130) == 32 * 144 + 3 * (32 + 16)
+    assert lib.pa_gated_linear_state_floats(5, 20, 130) == 0
+    names = ("kind", "q", "lq", "k", "lk", "v", "lv", "hpg", "ga", "gb", "lg", "ha", "hb", "hc", "cap", "qsc", "eps", "n", "st", "sr", "cl",
+             "ql", "qs", "ss", "batch", "mq", "out", "h", "dim", "vdim", "dt", "ws", "wb", "s")
+    gated = lambda **kw: [{**dict(kind=_lib.PA_GL_MLSTM, q=FAKE, lq=64, k=FAKE, lk=64, v=FAKE, lv=96, hpg=1, ga=FAKE, gb=FAKE, lg=4, ha=FAKE,
+                                  hb=FAKE, hc=None, cap=2.0, qsc=1.0, eps=1e-6, n=4, st=FAKE, sr=2, cl=FAKE, ql=FAKE, qs=FAKE, ss=FAKE, batch=2,
+                                  mq=2, out=FAKE, h=4, dim=16, vdim=24, dt=bf16, ws=None, wb=0, s=None), **kw}[k] for k in names]
+    for kw, status, text in ((dict(kind=3), -1, "kind"), (dict(hpg=3), -1, "heads_per_group"), (dict(dim=264, lq=2000, lk=2000), -2, "above 256"),
+                             (dict(lv=90), -1, "stride"), (dict(lg=3), -1, "stride"), (dict(cap=0.0), -1, "cap"), (dict(gb=None), -1, "NULL"),
+                             (dict(kind=_lib.PA_GL_SSD), -1, "NULL"), (dict(ql=None), -1, "together"),
+                             (dict(ql=None, qs=None, batch=5), -1, "below batch"), (dict(dt=_lib.PA_F16), -2, "dtype")):
+        rc, msg = _status("pa_gated_linear", *gated(**kw))
+        assert rc == status and text in msg, (kw, msg)
+    assert lib.pa_gated_linear_workspace_bytes(2, 0, 16, 24, 8) == 0 and "workspace_bytes" in _lib.last_error()
+
+    rc, msg = _status("pa_narrow_linear", FAKE, 30, FAKE, FAKE, 4, 8, 32, f32, None)
+    assert rc == -1 and "x_stride" in msg
+    for args, status, text in (((9, 2, 2, 1), -1, "equal groups"), ((8, 5, 2, 1), -1, "cannot be chosen"), ((8, 2, 2, 3), -1, "cannot be chosen"),
+                               ((2048, 2, 1, 1), -2, "above")):
+        rc, msg = _status("pa_moe_select", FAKE, 4096, 4, *args, 0, FAKE, FAKE, None)
+        assert rc == status and text in msg, (args, msg)
+    rc, msg = _status("pa_moe_select", FAKE, 8, 4, 8, 2, 1, 1, 1, FAKE, FAKE, None)
+    assert rc == -1 and "logits_stride" in msg
+    rc, msg = _status("pa_moe_lists", FAKE, 4, 2, 8, None, FAKE, None)
+    assert rc == -1 and "NULL" in msg
+    product = lambda **kw: [{**dict(x=FAKE, lx=64, ipr=2, w=FAKE, wr=96, lw=64, k=64, c=FAKE, l=FAKE, rows=4, top=2, e=8, glu=1, out=FAKE, n=48,
+                                    dt=bf16, s=None), **kw}[k] for k in ("x", "lx", "ipr", "w", "wr", "lw", "k", "c", "l", "rows", "top", "e",
+                                                                         "glu", "out", "n", "dt", "s")]
+    for kw, status, text in ((dict(wr=90), -1, "w_rows"), (dict(lx=60), -1, "stride"), (dict(c=None), -1, "NULL"), (dict(dt=_lib.PA_F16), -2, "dtype"),
+                             (dict(ipr=0), -1, "out of range")):
+        rc, msg = _status("pa_moe_product", *product(**kw))
+        assert rc == status and text in msg, (kw, msg)
