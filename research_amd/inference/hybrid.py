@@ -79,7 +79,7 @@ class HybridConfig:
     def cache_config(self, num_blocks: int, block_size: int, num_state_slots: int, dtype: torch.dtype,
                      device: str) -> CacheConfig:
         keys = [l.attention for l in self.layers]
-        shapes = tuple((a.kv_heads, a.pool_dim) if a is not None else None for a in keys)
+        shapes = tuple((a.pool_heads, a.pool_dim) if a is not None else None for a in keys)
         typical = next((s for s in shapes if s is not None), (1, 8))
         return CacheConfig(num_layers=len(shapes), num_kv_heads=typical[0], head_dim=typical[1], num_blocks=num_blocks,
                            block_size=block_size, dtype=dtype, device=device, layer_kv=shapes,

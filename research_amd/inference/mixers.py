@@ -82,17 +82,33 @@ class AttentionSpec:
             raise ValueError(f"window={self.window} must be positive")
         if self.chunk is not None and (self.chunk < 1 or self.window is not None):
             raise ValueError(f"chunk={self.chunk} must be positive, and no window beside it")
-        if self.pool_dim > 256:
-            raise ValueError(f"head sizes {self.dim} / {self.vdim} above 256")
+        if self.dim > 256:
+            raise ValueError(f"dim={self.dim} above 256")
+        if self.v_slices > 1 and (self.v_mix or self.gates or self.taps):
+            raise ValueError(f"vdim={self.vdim} above 256 with value mixing, head gates or convolutions")
+
+    @property
+    def v_slices(self) -> int:
+        """Equal slices of a value head that keep it within 256.  Each is stored and attended as a head of its own beside a
+        copy of the key, with a copy of its query heads (in the order key head, slice, query head)."""
+        return -(-self.vdim // 256)
+
+    @property
+    def slice_dim(self) -> int:
+        return -(-self.vdim // self.v_slices)
+
+    @property
+    def pool_heads(self) -> int:
+        return self.kv_heads * self.v_slices
 
     @property
     def pool_dim(self) -> int:
         """Head size of the layer's pool: holds a key or a value, in whole 8-element vectors."""
-        return -(-max(self.dim, self.vdim) // 8) * 8
+        return -(-max(self.dim, self.slice_dim) // 8) * 8
 
     @property
     def channels(self) -> int:
-        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+        return self.v_slices * ((self.heads + self.kv_heads) * self.dim + self.kv_heads * self.slice_dim)
 
     @property
     def mask_window(self) -> int:
@@ -257,7 +273,7 @@ class Mixer(nn.Module):
 class ConvAttention(Mixer):
     @staticmethod
     def sizes(spec: AttentionSpec) -> Tuple[int, int]:
-        return _pad8(spec.channels + (spec.heads if spec.gates else 0)), spec.heads * spec.vdim
+        return _pad8(spec.channels + (spec.heads if spec.gates else 0)), spec.heads * spec.v_slices * spec.slice_dim
 
     def __init__(self, spec: AttentionSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
                  rotary: RotaryTables, v_role: Optional[str], dtype: torch.dtype, device, slices: Slices = None,
@@ -280,6 +296,9 @@ class ConvAttention(Mixer):
     def load(self, get: Getter, prefix: str) -> None:
         s, at = self.spec, 0
         order = s.head_order()
+        if s.v_slices > 1:
+            self._load_slices(get, prefix, order)
+            return
         for name, n in (("q", s.heads * s.dim), ("k", s.kv_heads * s.dim), ("v", s.kv_heads * s.vdim)):
             pick = slice(None)
             if s.rot_halves and name != "v":  # (the scores do not change when q and k heads are stored in another order)
@@ -290,12 +309,43 @@ class ConvAttention(Mixer):
             at += n
         if s.gates:
             fill(self.w_in[at: at + s.heads], get(prefix + "g"), prefix + "g")
-        if s.qk_weights:
-            fill(self.q_norm, get(prefix + "q.norm")[order], prefix + "q.norm")
-            fill(self.k_norm, get(prefix + "k.norm")[order], prefix + "k.norm")
+        self._load_qk_norms(get, prefix, order)
         fill(self.w_out, get(prefix + "o"), prefix + "o")
         if self.v_role == "mix":
             fill(self.v_lambda, get(prefix + "vmix").reshape(1), prefix + "vmix")
+
+    def _load_qk_norms(self, get: Getter, prefix: str, order: Tensor) -> None:
+        if self.spec.qk_weights:
+            fill(self.q_norm, get(prefix + "q.norm")[order], prefix + "q.norm")
+            fill(self.k_norm, get(prefix + "k.norm")[order], prefix + "k.norm")
+
+    def _load_slices(self, get: Getter, prefix: str, order: Tensor) -> None:
+        """The layout of ``v_slices``: copies of the key heads and their query heads for every slice of the value head; the
+        part of the last slice past the head's end is zeros."""
+        s = self.spec
+        n, rep, width = s.v_slices, s.heads // s.kv_heads, self.w_in.shape[1]
+
+        def heads(name: str, count: int, dim: int) -> Tensor:
+            w = get(prefix + name)
+            if tuple(w.shape) != (count * dim, width):
+                raise ValueError(f"{prefix}{name}: checkpoint shape {tuple(w.shape)}, expected {(count * dim, width)}")
+            return w.view(s.kv_heads, -1, dim, width)
+
+        q = heads("q", s.heads, s.dim)[:, None, :, order].expand(-1, n, -1, -1, -1)
+        k = heads("k", s.kv_heads, s.dim)[:, :, order].expand(-1, n, -1, -1)
+        pad = n * s.slice_dim - s.vdim
+        v = F.pad(heads("v", s.kv_heads, s.vdim)[:, 0], (0, 0, 0, pad))
+        at = 0
+        for name, w in (("q", q), ("k", k), ("v", v)):
+            w = w.reshape(-1, width)
+            fill(self.w_in[at: at + w.shape[0]], w, prefix + name)
+            at += w.shape[0]
+        self._load_qk_norms(get, prefix, order)
+        o = get(prefix + "o")
+        if tuple(o.shape) != (self.w_out.shape[0], s.heads * s.vdim):
+            raise ValueError(f"{prefix}o: checkpoint shape {tuple(o.shape)}")
+        o = F.pad(o.view(-1, s.kv_heads, rep, s.vdim), (0, pad)).view(-1, s.kv_heads, rep, n, s.slice_dim).transpose(2, 3)
+        fill(self.w_out, o.reshape(self.w_out.shape), prefix + "o")
 
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s, packed = self.spec, step.packed
@@ -303,13 +353,13 @@ class ConvAttention(Mixer):
             step.v_first = torch.empty((u.shape[0], s.kv_heads * s.vdim), dtype=u.dtype, device=u.device)
         kc, vc = self.backend._layer(self.layer_idx)
         # q carries scale * log2(e) from its 32-bit registers, so that the attention kernels' own factor is one
-        q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, s.scale / _LN2, self.eps,
+        q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads * s.v_slices, s.dim, s.slice_dim, s.scale / _LN2, self.eps,
                                 not s.qk_weights, self.rotary.get(s.rot_base, s.rot_dims, s.rot_factor, s.rot_yarn), s.rot_dims,
                                 self.conv, self.conv_state, self.v_role, step.v_first if self.v_role else None,
                                 self.v_lambda if self.v_role == "mix" else None, q_norm=self.q_norm, k_norm=self.k_norm)
         o = self.backend.attend_packed(q, self.layer_idx, packed, _LN2, s.mask_window)
         gate = u[:, s.channels: s.channels + s.heads] if s.gates else None
-        return ops.head_gate(o, gate, s.vdim, self.out_scale, out)
+        return ops.head_gate(o, gate, s.slice_dim, self.out_scale, out)
 
 
 class LightningMixer(Mixer):

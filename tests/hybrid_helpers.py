@@ -1,11 +1,14 @@
-"""Small random hybrid models for the tests: a ``config.json`` dictionary, weights under their checkpoint names, and a
-checkpoint folder of both."""
+"""Small random hybrid models for the tests: a ``config.json`` dictionary, weights under their checkpoint names, a
+checkpoint folder of both, and the oracle of the design (Lotozen here, Tevirax in tevirax_helpers.py)."""
 
 import json
 import os
 
 import numpy as np
 import torch
+
+from oracle import hybrid_oracle, tevirax_oracle
+from tests import tevirax_helpers as tv
 
 
 def attention(heads, kv_heads, dim, vdim, window, conv, rot_dims, base=1000.0, factor=1.0, scale=None, v_mix=True, ff=40):
@@ -42,8 +45,19 @@ CONFIGS = {
 }
 
 
+CONFIGS.update(tv.CONFIGS)
+
+
+def forward(w, cfg, tokens, **kw):
+    """The oracle's logits of a whole sequence."""
+    oracle = tevirax_oracle if cfg["architecture"] == "Tevirax" else hybrid_oracle
+    return oracle.decoder_forward(w, cfg, tokens, **kw)
+
+
 def weights(cfg, seed=0):
     """bfloat16 tensors (as stored in a checkpoint) scaled so that every mechanism moves the logits."""
+    if cfg["architecture"] == "Tevirax":
+        return tv.weights(cfg, seed)
     g = torch.Generator().manual_seed(seed)
     w = {}
 

@@ -70,7 +70,7 @@ def test_ragged_batches(replay, seed):
             lens = rng.integers(0, 3000, batch) * (rng.random(batch) < 0.5)
         shape = SHAPES[int(rng.integers(len(SHAPES)))]
         grid = int(rng.choice([1, 2, 3, 17, 64, 512, 608, 4096]))
-        window = int(rng.choice([0, 0, 1, 17, 512, 100000]))
+        window = int(rng.choice([0, 0, 1, 17, 512, 100000, -1, -17, -512, -100000]))
         bs = int(rng.choice([16, 16, 1, 8, 64, 256]))
         s = replay(lens, shape, block_size=bs, window=window, grid=grid, grid_cap=max(grid, 4096) if rng.random() < 0.5 else grid)
         assert s["max_slot"] < s["slot_cap"]

@@ -9,7 +9,6 @@ import numpy as np
 import pytest
 import torch
 
-from oracle import hybrid_oracle as ho
 from research_amd.inference import EngineConfig, InferenceEngine, SamplingParams
 from tests import hybrid_helpers as hh
 from tests.gpu_helpers import announce
@@ -42,10 +41,10 @@ class Wanted:
 
     def __init__(self, cfg, w, tokens, dtype):
         with torch.no_grad():
-            self.logits = ho.decoder_forward(w, cfg, tokens)
+            self.logits = hh.forward(w, cfg, tokens)
             self.tol = torch.full((len(tokens),), F32_TOL, dtype=torch.float64)
             if dtype == "bfloat16":
-                self.tol = hh.bf16_tolerance(ho.decoder_forward, cfg, w, tokens, self.logits)
+                self.tol = hh.bf16_tolerance(hh.forward, cfg, w, tokens, self.logits)
         self.scale = self.logits.pow(2).mean().sqrt()
 
     def check(self, got, places, what):
@@ -81,12 +80,13 @@ def test_whole_prompts_of_unequal_length_in_one_batch(folders, name, dtype):
     assert engine.cache.num_free_blocks() == 40 and len(engine.cache.free_state_slots) == 4
 
 
-def test_residual_after_every_layer(folders):
-    announce("hybrid layers")
-    path, cfg, w = folders("odd")
+@pytest.mark.parametrize("name", ["odd", "tvx-odd", "tvx-wide"])
+def test_residual_after_every_layer(folders, name):
+    announce(f"hybrid layers {name}")
+    path, cfg, w = folders(name)
     (prompt,) = hh.prompts(cfg, [37])
     want = []
-    ho.decoder_forward(w, cfg, prompt, trace=want)
+    hh.forward(w, cfg, prompt, trace=want)
     engine = _engine(path, "float32")
     forward, got = engine.model.forward, []
     engine.model.forward = lambda ids, pos, ctx: forward(ids, pos, ctx, got)
@@ -116,7 +116,7 @@ def test_portions_and_token_by_token(folders, name, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["plain", "odd"])
+@pytest.mark.parametrize("name", ["plain", "odd", "tvx-plain", "tvx-odd"])
 def test_mixed_batches_use_blocks_and_slots_again(folders, name, dtype):
     """Up to three live sequences in a pool that barely holds them: portions of some beside single tokens of others,
     sequences that pause, and successors in the blocks and state slots of the ones that ended."""
@@ -153,7 +153,9 @@ def _by_prompt(samples):
 
 
 @pytest.mark.parametrize("name,kw", [("plain", {}), ("plain", {"use_graphs": True}), ("odd", {"prefill_portion": 7}),
-                                     ("no-mixing", {"use_graphs": True, "prefill_portion": 20})])
+                                     ("no-mixing", {"use_graphs": True, "prefill_portion": 20}),
+                                     ("tvx-plain", {"use_graphs": True}), ("tvx-odd", {"prefill_portion": 7}),
+                                     ("tvx-wide", {"use_graphs": True, "prefill_portion": 20})])
 def test_greedy_generation_through_the_scheduler(folders, name, kw):
     """Long greedy decoding of ragged prompts by ``generate``: the tokens are the oracle's argmax at every position,
     the log probabilities its own; graphs are replayed between eager prefills."""
@@ -167,16 +169,17 @@ def test_greedy_generation_through_the_scheduler(folders, name, kw):
             s = samples[tuple(p)]
             tokens = list(p) + list(s.completion_tokens)
             with torch.no_grad():
-                lp = torch.log_softmax(ho.decoder_forward(w, cfg, tokens[:-1])[len(p) - 1:], -1)
+                lp = torch.log_softmax(hh.forward(w, cfg, tokens[:-1])[len(p) - 1:], -1)
             assert len(s.completion_tokens) == 40 + 60 * round_
             assert lp.argmax(-1).tolist() == list(s.completion_tokens)
             assert s.logprobs == pytest.approx(lp.max(-1).values.tolist(), abs=2e-4)
     assert engine.cache.num_free_blocks() == 80
 
 
-def test_preemption_starts_the_state_over(folders):
-    announce("hybrid preemption")
-    path, cfg, w = folders("plain")
+@pytest.mark.parametrize("name", ["plain", "tvx-plain"])
+def test_preemption_starts_the_state_over(folders, name):
+    announce(f"hybrid preemption {name}")
+    path, cfg, w = folders(name)
     engine = _engine(path, "float32", blocks=9, slots=4, max_len=120, prefill_portion=10)
     prompts = hh.prompts(cfg, [30, 25, 28], seed=5)
     samples = _by_prompt(engine.generate(prompts, SamplingParams(temperature=0.0, max_tokens=40)))
@@ -184,12 +187,13 @@ def test_preemption_starts_the_state_over(folders):
     for p in prompts:
         tokens = list(p) + list(samples[tuple(p)].completion_tokens)
         with torch.no_grad():
-            assert ho.decoder_forward(w, cfg, tokens[:-1])[len(p) - 1:].argmax(-1).tolist() == tokens[len(p):]
+            assert hh.forward(w, cfg, tokens[:-1])[len(p) - 1:].argmax(-1).tolist() == tokens[len(p):]
 
 
-def test_weight_updates_keep_graphs_and_restart_sequences(folders):
-    announce("hybrid update")
-    path, cfg, _ = folders("plain")
+@pytest.mark.parametrize("name,tensor", [("plain", "l0.mix.o"), ("tvx-plain", "l1.mix.left.o")])
+def test_weight_updates_keep_graphs_and_restart_sequences(folders, name, tensor):
+    announce(f"hybrid update {name}")
+    path, cfg, _ = folders(name)
     engine = _engine(path, "float32", use_graphs=True)
     prompts = hh.prompts(cfg, [9, 20])
     engine.generate(prompts, SamplingParams(temperature=0.0, max_tokens=5))
@@ -200,16 +204,17 @@ def test_weight_updates_keep_graphs_and_restart_sequences(folders):
     for p in prompts:
         tokens = list(p) + list(samples[tuple(p)].completion_tokens)
         with torch.no_grad():
-            assert ho.decoder_forward(w, cfg, tokens[:-1])[len(p) - 1:].argmax(-1).tolist() == tokens[len(p):]
+            assert hh.forward(w, cfg, tokens[:-1])[len(p) - 1:].argmax(-1).tolist() == tokens[len(p):]
     with pytest.raises(KeyError, match="checkpoint lacks"):
-        engine.update_weights({k: v for k, v in w.items() if k != "l0.mix.o"})
+        engine.update_weights({k: v for k, v in w.items() if k != tensor})
 
 
-def test_trace_replay(folders, tmp_path):
-    announce("hybrid trace")
+@pytest.mark.parametrize("name", ["plain", "tvx-plain"])
+def test_trace_replay(folders, tmp_path, name):
+    announce(f"hybrid trace {name}")
     from research_amd.inference.trace import replay
 
-    path, cfg, w = folders("plain")
+    path, cfg, w = folders(name)
     a, b, c = hh.prompts(cfg, [40, 21, 30], seed=9)
     steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:38], "want": [0, 37]}], "end": []},
              {"step": 1, "entries": [{"id": "a", "tokens": a[38:39], "want": []}, {"id": "b", "tokens": b, "want": [20, 5]}], "end": ["b"]},

@@ -85,8 +85,8 @@ def test_forward_is_causal(name):
     cfg = hh.CONFIGS[name]
     w = hh.weights(cfg)
     (tokens,) = hh.prompts(cfg, [14])
-    whole = ho.decoder_forward(w, cfg, tokens)
-    assert torch.allclose(whole[:9], ho.decoder_forward(w, cfg, tokens[:9]))
+    whole = hh.forward(w, cfg, tokens)
+    assert torch.allclose(whole[:9], hh.forward(w, cfg, tokens[:9]))
 
 
 PLANTED = {
@@ -109,8 +109,8 @@ def test_planted_mistakes_show(what):
     cfg = hh.CONFIGS["plain"]
     w = hh.weights(cfg)
     (tokens,) = hh.prompts(cfg, [60])
-    right = ho.decoder_forward(w, cfg, tokens)
+    right = hh.forward(w, cfg, tokens)
     bad_cfg, bad_w = copy.deepcopy(cfg), {k: v.clone() for k, v in w.items()}
     PLANTED[what](bad_cfg, bad_w)
-    wrong = ho.decoder_forward(bad_w, bad_cfg, tokens)
+    wrong = hh.forward(bad_w, bad_cfg, tokens)
     assert hh.logit_error(wrong, right).max() > 2 * BF16_TOL
