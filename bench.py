@@ -10,7 +10,7 @@ head_dim 256 and 64; dense prefill of 64 x 512 and 4 x 8192 tokens; one chunk
 behind 200 000 cached keys at head_dim 128 and 256) under ``secondary``.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--no-secondary]
-                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen]
+                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen|tevirax]
     python bench.py --traffic-from-pmc NAME KERNEL FETCH.csv WRITE.csv   # refresh profiles/traffic.json
 """
 
@@ -101,7 +101,8 @@ def parse_args():
     ap.add_argument("--steps", type=int, default=50)
     ap.add_argument("--warmup", type=int, default=10)
     ap.add_argument("--workload", default="c4", choices=["c1", "c2", "c3", "c3-d256", "c3-d64", "c3-d96", "long-d128", "long-d256", "dense-64x512",
-                                                         "dense-4x8192", "c4", "c5", "engine", "lotozen"])
+                                                         "dense-4x8192", "c4", "c5", "engine", "lotozen",
+                                                         "tevirax"])
     ap.add_argument("--preheat-s", type=float, default=0.5,
                     help="seconds of untimed steps before the warmup steps: an idle GPU sits at its lowest clocks "
                          "and takes a few hundred milliseconds of work to leave them")
@@ -796,15 +797,8 @@ def hybrid_throughput(model, dev, packed, steps, warmup, preheat_s):
     return out
 
 
-def hybrid_kernels(shape, dev, steps):
-    """Every kernel of the new blocks alone at the layer's shapes, against its roofline, with the like kernel of the
-    Llama block.  Bytes and FLOPs are the algorithmic ones (heads unpadded)."""
-    from research_amd import ops
-
-    width, heads, kv, dim, vdim, lheads, ff, side = shape
-    bf, f32 = torch.bfloat16, torch.float32
-    rnd = lambda *s, dtype=bf: torch.randn(*s, device=dev, dtype=torch.float32).to(dtype)
-    i32 = lambda a: torch.as_tensor(np.ascontiguousarray(a), dtype=torch.int32).to(dev)
+def kernel_table(steps):
+    """A list of kernels with their times and rooflines, and the function that adds one."""
     rows_out = []
 
     def add(phase, name, fn, like, n_bytes=0.0, flops=0.0):
@@ -822,6 +816,19 @@ def hybrid_kernels(shape, dev, steps):
                          "pct_of_roofline": round(100.0 * bound / ms, 1),
                          "bound": "mfma" if flops / MFMA_BF16_PEAK_TFLOPS / 1e9 > n_bytes / HBM_PEAK_GBPS / 1e6 else "hbm"})
 
+    return rows_out, add
+
+
+def hybrid_kernels(shape, dev, steps):
+    """Every kernel of the new blocks alone at the layer's shapes, against its roofline, with the like kernel of the
+    Llama block.  Bytes and FLOPs are the algorithmic ones (heads unpadded)."""
+    from research_amd import ops
+
+    width, heads, kv, dim, vdim, lheads, ff, side = shape
+    bf, f32 = torch.bfloat16, torch.float32
+    rnd = lambda *s, dtype=bf: torch.randn(*s, device=dev, dtype=torch.float32).to(dtype)
+    i32 = lambda a: torch.as_tensor(np.ascontiguousarray(a), dtype=torch.int32).to(dev)
+    rows_out, add = kernel_table(steps)
     d = -(-max(dim, vdim) // 8) * 8
     chans = (heads + kv) * dim + kv * vdim
     for phase, (batch, length) in (("prefill", HYBRID_PREFILL), ("decode", HYBRID_DECODE)):
@@ -943,6 +950,226 @@ def bench_hybrid(args, dev) -> int:
     return 0
 
 
+# width; attention query heads, kv heads (of 128 x 128), chunk; mLSTM heads, dim, vdim; Mamba-2 heads, vdim, state, groups;
+# experts, chosen, groups, kept, inner width, shared inner width; dense feed-forward of the first layer
+TEVIRAX_SHAPES = {
+    "w2048": dict(width=2048, heads=16, kv_heads=4, chunk=1024, m_heads=4, m_dim=256, m_vdim=512, s_heads=64, s_vdim=64, s_state=128, s_groups=8,
+                  experts=64, top=6, groups=8, keep=4, ff=768, shared=1024, dense=5632),
+    "w4096": dict(width=4096, heads=32, kv_heads=8, chunk=1024, m_heads=8, m_dim=256, m_vdim=512, s_heads=128, s_vdim=64, s_state=128, s_groups=8,
+                  experts=64, top=8, groups=8, keep=4, ff=1408, shared=2816, dense=14336),
+}
+
+
+def tevirax_model(p, dev, num_blocks, slots, max_positions):
+    """Mamba-2 layers with a parallel layer (chunk attention and matrix memory) in every fourth place, a dense feed-forward in
+    the first layer and experts in the others; random weights."""
+    from research_amd.inference import HipPagedAttentionBackend, HybridConfig, HybridDecoder
+    from research_amd.inference.hybrid import LayerSpec
+    from research_amd.inference.mixers import AttentionSpec, Mamba2Mixer, Mamba2Spec, MlstmMixer, MlstmSpec, ParallelSpec, YarnScaling
+    from research_amd.inference.moe import MoESpec
+
+    att = AttentionSpec(heads=p["heads"], kv_heads=p["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, window=None, taps=0, rot_dims=128,
+                        rot_base=500000.0, chunk=p["chunk"], rot_yarn=YarnScaling(4.0, 8192, 32.0, 1.0), rot_halves=True, qk_weights=True, gates=False)
+    par = ParallelSpec(att, MlstmSpec(p["m_heads"], p["m_dim"], p["m_vdim"], 15.0), 1.0, 1.0)
+    ssd = Mamba2Spec(p["s_heads"], p["s_vdim"], p["s_state"], p["s_groups"], 4, p["s_groups"])
+    moe = MoESpec(p["experts"], p["ff"], p["top"], p["groups"], p["keep"], p["shared"])
+    cfg = HybridConfig(vocab_size=HYBRID_VOCAB, width=p["width"], norm_eps=1e-6, norm="rms", post_norm=True, embed_scale=p["width"] ** 0.5,
+                       positions=max_positions, logit_softcap=30.0,
+                       layers=tuple(LayerSpec(par if i % 4 == 3 else ssd, moe if i else p["dense"]) for i in range(HYBRID_LAYERS)))
+    backend = HipPagedAttentionBackend(cfg.cache_config(num_blocks, 16, slots, torch.bfloat16, "cuda"))
+    model = HybridDecoder(cfg, backend, max_positions)
+    with torch.no_grad():
+        for q in model.parameters():
+            q.normal_(0.0, q.shape[-1] ** -0.5)
+        for m in model.modules():
+            if isinstance(m, Mamba2Mixer):
+                m.rate.uniform_(1.0, 16.0)
+                m.dt_bias.fill_(-4.0)
+            if isinstance(m, MlstmMixer):
+                m.f_bias.fill_(4.0)
+    return model.eval()
+
+
+def tevirax_kernels(p, dev, steps):
+    """Every kernel of the design's blocks at the layer's shapes, against its roofline, with the like kernel of the Lotozen or
+    Llama block.  Bytes and FLOPs are the algorithmic ones."""
+    import torch.nn.functional as F
+    from research_amd import ops
+
+    bf, f32 = torch.bfloat16, torch.float32
+    rnd = lambda *s, dtype=bf: torch.randn(*s, device=dev, dtype=torch.float32).to(dtype)
+    i32 = lambda a: torch.as_tensor(np.ascontiguousarray(a), dtype=torch.int32).to(dev)
+    rows_out, add = kernel_table(steps)
+    width, heads, kv, d = p["width"], p["heads"], p["kv_heads"], 128
+    for phase, (batch, length) in (("prefill", HYBRID_PREFILL), ("decode", HYBRID_DECODE)):
+        dec = phase == "decode"
+        n = batch if dec else batch * length
+        per = length // 16 + (1 if dec else 0)
+        tables = np.random.default_rng(5).permutation(batch * per).reshape(batch, per).astype(np.int32)
+        ctx = np.full(batch, length + 1 if dec else length)
+        pos = np.full((batch, 1), length) if dec else np.tile(np.arange(length), (batch, 1))
+        slots = torch.from_numpy((np.take_along_axis(tables, pos // 16, 1).astype(np.int64) * 16 + pos % 16).reshape(-1)).to(dev)
+        bt, lens, sslots = i32(tables), i32(ctx), i32(np.arange(batch))
+        if dec:
+            por = ops.Portions(lens, sslots)
+        else:
+            first = np.arange(0, length, ops.QKV_TILE_ROWS)
+            tiles = np.stack([np.repeat(np.arange(batch), len(first)), np.tile(first, batch)], 1)
+            por = ops.Portions(lens, sslots, i32(ctx), i32(np.arange(batch) * length), i32(tiles), length)
+        x, y, w = rnd(n, width, dtype=f32), rnd(n, width), rnd(width, dtype=f32)
+        add(phase, "residual + RMS-normed branch", lambda: ops.residual_norm(x, bf, y=y, y_weight=w, y_eps=1e-6), "residual + layer norm", n * width * 12.0)
+        add(phase, "like: residual + layer norm", lambda: ops.residual_norm(x, bf, y=y, norm="layer", weight=w, bias=w, eps=1e-6), "", n * width * 12.0)
+        # experts
+        e, top, ff, inner = p["experts"], p["top"], p["ff"], -(-p["ff"] // 64) * 64
+        h, router = rnd(n, width), rnd(e + 1, width)
+        router *= width ** -0.5
+        add(phase, "router logits", lambda: ops.narrow_linear(h, router), "bf16 product of equal size", (n * width + e * width) * 2.0 + n * (e + 1) * 4.0,
+            2.0 * n * width * (e + 1))
+        add(phase, "like: bf16 product of equal size", lambda: F.linear(h, router), "", (n * width + e * width) * 2.0 + n * (e + 1) * 2.0, 2.0 * n * width * (e + 1))
+        logits = ops.narrow_linear(h, router)
+        choice = ops.moe_choose(logits, e, top, p["groups"], p["keep"])
+        add(phase, "choice of experts and lists", lambda: ops.moe_choose(logits, e, top, p["groups"], p["keep"]), "silu(gate) * up",
+            n * (e + 1) * 4.0 + n * top * 20.0)
+        w_in, w_out = rnd(e, 2 * inner, width), rnd(e, width, inner)
+        act, items = rnd(n * top, inner), n * top
+        used = int((choice.counts > 0).sum())
+        add(phase, "experts: gate, up, silu", lambda: ops.moe_product(h, choice, w_in, inner, width, True), "dense product of equal flops",
+            used * 2.0 * inner * width * 2 + n * width * 2.0 + items * inner * 2.0, 4.0 * items * inner * width)
+        add(phase, "experts: down", lambda: ops.moe_product(act, choice, w_out, width, inner, False), "dense product of equal flops",
+            used * 2.0 * inner * width + items * (inner + width) * 2.0, 2.0 * items * inner * width)
+        if not dec:
+            dw, dw2 = rnd(2 * top * inner, width), rnd(width, top * inner)
+            dact = rnd(n, top * inner)
+            add(phase, "like: dense gate and up of equal flops", lambda: F.linear(h, dw), "", 0.0, 4.0 * items * inner * width)
+            add(phase, "like: dense down of equal flops", lambda: F.linear(dact, dw2), "", 0.0, 2.0 * items * inner * width)
+            del dw, dw2, dact
+        else:  # (the same bytes of weights)
+            dw, dw2 = rnd(used * 2 * inner, width), rnd(used * width, inner)
+            dh = rnd(n * top // used or 1, inner)
+            add(phase, "like: dense gate and up of equal bytes", lambda: F.linear(h[: n * top // used or 1], dw), "", used * 2.0 * inner * width * 2)
+            add(phase, "like: dense down of equal bytes", lambda: F.linear(dh, dw2), "", used * 2.0 * inner * width)
+            del dw, dw2, dh
+        del w_in, w_out, act
+        eo, shared = rnd(items, width), rnd(n, width)
+        add(phase, "residual + RMS-normed sum over experts",
+            lambda: ops.residual_norm(x, bf, y=eo, mix=choice.weights, y_extra=shared, y_weight=w, y_eps=1e-6), "residual + layer norm",
+            n * width * (10.0 + 2.0 * (top + 1)))
+        del eo, shared, x, y
+        # attention
+        u = rnd(n, (heads + 2 * kv) * d)
+        kc, vc = rnd(batch * per * 16, kv, d), rnd(batch * per * 16, kv, d)
+        rope, qn = rnd(length + 1, d // 2, 2, dtype=f32), rnd(d, dtype=f32)
+        q = torch.empty(n, heads, d, dtype=bf, device=dev)
+        add(phase, "q/k norm + rotation + append", lambda: ops.qkv_conv_append(u, por, slots, kc, vc, heads, d, d, 1.0, 1e-6, False, rope, d, None, None,
+                                                                               q_out=q, q_norm=qn, k_norm=qn), "rope_kv_append", n * 4.0 * d * (heads + 2 * kv))
+        cos, k0, v0, tpos = rnd(length + 1, d), rnd(n, kv, d), rnd(n, kv, d), i32(pos.reshape(-1))
+        add(phase, "like: rope_kv_append", lambda: ops.rope_kv_append(q, k0, v0, cos, cos, kc, vc, slots, positions=tpos, q_out=q), "",
+            n * 2.0 * d * (2 * heads + 4 * kv))
+        o = torch.empty_like(q)
+        if dec:
+            ws = ops.decode_workspace(q, kc)
+            half = i32(np.full(batch, length - p["chunk"] // 2))  # (half a chunk is visible)
+            att = lambda win, ln: ops.decode(q, kc, vc, bt, ln, 16, 0.1, ws, out=o, window=win)
+            add(phase, "decode attention, half a chunk", lambda: att(-p["chunk"], half), "decode attention, window", 4.0 * kv * d * batch * p["chunk"] / 2)
+            add(phase, "like: decode attention, window", lambda: att(p["chunk"] // 2, lens), "", 4.0 * kv * d * batch * p["chunk"] / 2)
+        else:
+            att = lambda win: ops.prefill_paged(q, kc, vc, bt, lens, por.q_lens, por.q_starts, length, 16, 0.1, out=o, window=win)
+            i = np.arange(length)
+            add(phase, "prefill attention, chunks", lambda: att(-p["chunk"]), "prefill attention, window", flops=4.0 * d * heads * batch * float((i % p["chunk"] + 1).sum()))
+            add(phase, "like: prefill attention, window", lambda: att(p["chunk"]), "",
+                flops=4.0 * d * heads * batch * float(np.minimum(i + 1, p["chunk"]).sum()))
+        joint = torch.empty(n, heads * d + p["m_heads"] * p["m_vdim"], dtype=bf, device=dev)
+        add(phase, "head packing", lambda: ops.head_gate(o, None, d, 1.2, joint[:, : heads * d]), "silu(gate) * up", n * heads * d * 4.0)
+        del u, kc, vc, q, o, k0, v0
+        # recurrences
+        shapes = {"matrix memory": ("mlstm", p["m_heads"], p["m_dim"], p["m_vdim"], p["m_heads"]),
+                  "state space": ("ssd", p["s_heads"], p["s_state"], p["s_vdim"], p["s_groups"])}
+        for name, (kind, hs, dim, vdim, groups) in shapes.items():
+            qk = groups * dim
+            u = rnd(n, 2 * qk + hs * vdim + 2 * hs)
+            uq, uk, uv, ga, gb = u.split([qk, qk, hs * vdim, hs, hs], 1)
+            state = torch.zeros(batch, hs, ops.gated_linear_state_floats(kind, dim, vdim), device=dev)
+            out = torch.empty(n, hs * vdim, dtype=bf, device=dev)
+            const = (torch.full((hs,), -4.0, device=dev), torch.full((hs,), 4.0, device=dev), torch.ones(hs, device=dev) if kind == "ssd" else None)
+            need = 0 if dec else ops.gated_linear_workspace_bytes(batch, hs, dim, vdim, length)
+            ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+            run = lambda por, ws: ops.gated_linear(kind, uq, uk, uv, (ga, gb if kind == "mlstm" else None), const, por, state, hs, dim, vdim, out,
+                                                   heads_per_group=hs // groups, cap=15.0, q_scale=dim ** -0.5, den_eps=1e-6, workspace=ws)
+            n_bytes = n * 2.0 * (2 * qk + 2 * hs * vdim + 2 * hs) + (batch * state[0].numel() * 8.0 if dec else 0.0)
+            chunked = n * hs * (4.0 * dim * vdim + 64.0 * (dim + vdim))  # the products of 64-row chunks, one bf16 term each
+            add(phase, name, lambda: run(por, ws), "lightning attention", n_bytes, 0.0 if dec else chunked)
+            if not dec:
+                por1 = ops.Portions(i32([n]), i32([0]), i32([n]), i32([0]), None, n)
+                need = ops.gated_linear_workspace_bytes(1, hs, dim, vdim, n)
+                ws1 = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+                add(phase, f"{name}, one sequence of {n}", lambda: run(por1, ws1), "lightning attention, one sequence", n_bytes, chunked)
+            nw, z = rnd(hs * vdim, dtype=f32), rnd(n, hs * vdim)
+            if kind == "mlstm":
+                add(phase, "RMS norm per head + sigmoid gate", lambda: ops.rms_gate(out, z, nw, 1e-6, groups=hs, out=joint[:, heads * d:]), "RMS norm + sigmoid gate",
+                    n * hs * vdim * 6.0)
+            else:
+                add(phase, "silu gate + RMS norm of groups", lambda: ops.rms_gate(out, z, nw, 1e-6, groups=groups, order="silu_first"), "RMS norm + sigmoid gate",
+                    n * hs * vdim * 6.0)
+                add(phase, "like: RMS norm + sigmoid gate", lambda: ops.rms_gate(out, z, nw, 1e-6), "", n * hs * vdim * 6.0)
+                ch = hs * vdim + 2 * qk
+                cu, cw, cb = rnd(n, ch), rnd(4, ch, dtype=f32), rnd(ch, dtype=f32)
+                cs = torch.zeros(batch, 3, ch, dtype=bf, device=dev)
+                add(phase, "short convolution", lambda: ops.short_conv(cu, por, cw, cb, cs, "silu"), "rope_kv_append",
+                    n * ch * 4.0 + (batch * 12.0 * ch if dec else 0.0) + ch * 20.0)
+                del cu
+            del u, state, out, z
+        lheads = width // 128
+        u = rnd(n, 4 * width)
+        state = ops.lightning_state(batch, lheads, 128, 128, dev)
+        powers = torch.full((lheads, 65), 0.97, device=dev) ** torch.arange(65, device=dev)
+        o = torch.empty(n, width, dtype=bf, device=dev)
+        need = 0 if dec else ops.lightning_workspace_bytes(batch, lheads, 128, 128, length)
+        ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+        n_bytes, chunked = n * width * 8.0 + (batch * lheads * 128 * 128 * 8.0 if dec else 0.0), n * lheads * (4.0 * 128 * 128 + 64.0 * 256)
+        add(phase, "like: lightning attention", lambda: ops.lightning(u, por, state, powers, lheads, 128, 128, o, workspace=ws), "", n_bytes, 0.0 if dec else chunked)
+        if not dec:
+            need = ops.lightning_workspace_bytes(1, lheads, 128, 128, n)
+            ws1 = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+            add(phase, "like: lightning attention, one sequence", lambda: ops.lightning(u, por1, state, powers, lheads, 128, 128, o, workspace=ws1), "", n_bytes, chunked)
+        add(phase, "like: silu(gate) * up", lambda: ops.glu(u[:, :width], u[:, width: 2 * width], "silu"), "", n * width * 6.0)
+        del u, state, o, joint
+        if dec:
+            lg = rnd(n, HYBRID_VOCAB)
+            add(phase, "capped logits", lambda: ops.softcap(lg, 30.0), "silu(gate) * up", n * HYBRID_VOCAB * 6.0)
+        torch.cuda.empty_cache()
+    return rows_out
+
+
+def bench_tevirax(args, dev) -> int:
+    """Prefill and decode throughput of Tevirax-shaped models with random weights beside Lotozen-shaped ones of the same width,
+    heads, depth and feed-forward work per token, and the design's kernels against their rooflines.  Not the headline
+    workload."""
+    sizes = {}
+    steps, warmup = min(args.steps, 20), min(args.warmup, 3)
+    for name, p in TEVIRAX_SHAPES.items():
+        batch, ctx_len = HYBRID_DECODE
+        blocks = batch * (ctx_len // 16 + 1)
+        model = tevirax_model(p, dev, blocks, batch, ctx_len + 16)
+        entry = {"shape": p, "tevirax": hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)}
+        del model
+        torch.cuda.empty_cache()
+        shape = (p["width"], p["heads"], p["kv_heads"], 128, 128, p["width"] // 128, p["top"] * p["ff"] + p["shared"], 128)
+        model = hybrid_model(shape, dev, blocks, batch, ctx_len + 16)
+        entry["lotozen"] = hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)
+        del model
+        torch.cuda.empty_cache()
+        entry["kernels"] = tevirax_kernels(p, dev, steps)
+        sizes[name] = entry
+        print(f"[{name}] done", file=sys.stderr, flush=True)
+    main_size = sizes["w4096"]["tevirax"]
+    print(json.dumps({
+        "metric": "Tevirax prefill tokens/s", "value": main_size["prefill_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+        "steps": steps, "warmup": warmup, "ms_per_step": main_size["prefill_ms"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "tevirax", "layers": HYBRID_LAYERS, "prefill": HYBRID_PREFILL, "decode": HYBRID_DECODE}, "sizes": sizes}))
+    return 0
+
+
 def secondary(args, dev) -> dict:
     """Short runs of the configurations that are not the headline: what the step costs, the dominant kernel
     against its roofline and a few seconds of the CPU restatement, per workload."""
@@ -986,6 +1213,8 @@ def main() -> int:
         return bench_engine(args, dev)
     if args.workload == "lotozen":
         return bench_hybrid(args, dev)
+    if args.workload == "tevirax":
+        return bench_tevirax(args, dev)
     if args.workload in PREFILL_HEAD_SHAPES:
         result = bench_prefill_head(args, dev, args.workload)
     elif args.workload in PREFILL_LONG_SHAPES:
