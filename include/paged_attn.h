@@ -552,19 +552,21 @@ int pa_narrow_linear(const void *x, int64_t x_stride, const void *w, float *out,
                      void *stream);
 
 /*
- * Mixture of experts.  pa_moe_select, per row: scores s = sigmoid(logits); of `groups` equal groups of neighbours the
+ * Mixture of experts.  pa_moe_choose, per row: scores s = sigmoid(logits); of `groups` equal groups of neighbours the
  * `keep` with the largest sums of their two largest scores stay; of their experts the `top` with the largest scores are
  * chosen (the lowest number first on ties).  ids int32[rows][top]; weights float[rows][top + 1]: the chosen scores over
- * (their sum + 1e-20), then sigmoid(logits[experts]) when `shared`, else 0.  top <= 64, experts <= 1024.
- * pa_moe_lists: counts int32[experts] and lists int32[experts][rows], expert e's items (row * top + place) in order.
+ * (their sum + 1e-20), then sigmoid(logits[experts]) when `shared`, else 0.  top <= 64, experts <= 1024.  And per
+ * expert counts int32[experts] and lists int32[experts][rows]: its items (row * top + place) in order.  (Scores that are
+ * NaN are not chosen: id -1.)  The workspace needs no initial contents.
  * pa_moe_product: for every listed item, out[item] = W_e x[item / items_per_row], or with glu
  * silu(G_e x) * (U_e x) where an expert's weight rows are the n rows of G followed by the n rows of U.
  *   w : [experts][w_rows][w_stride] of dtype, rows zero past k.  The matrix-core kernels want w_stride % 64 == 0,
  *   k % 8 == 0, n % 4 == 0 and 16-byte aligned tensors; anything else runs on the vector units.
  */
-int pa_moe_select(const float *logits, int64_t logits_stride, int64_t rows, int experts, int top, int groups, int keep,
-                  int shared, int32_t *ids, float *weights, void *stream);
-int pa_moe_lists(const int32_t *ids, int64_t rows, int top, int experts, int32_t *counts, int32_t *lists, void *stream);
+size_t pa_moe_workspace_bytes(int64_t rows, int experts, int top);
+int pa_moe_choose(const float *logits, int64_t logits_stride, int64_t rows, int experts, int top, int groups, int keep,
+                  int shared, int32_t *ids, float *weights, int32_t *counts, int32_t *lists, void *workspace,
+                  size_t workspace_bytes, void *stream);
 int pa_moe_product(const void *x, int64_t x_stride, int items_per_row, const void *w, int64_t w_rows, int w_stride, int k,
                    const int32_t *counts, const int32_t *lists, int64_t rows, int top, int experts, int glu, void *out,
                    int n, int dtype, void *stream);

@@ -107,8 +107,8 @@ SIGNATURES.update({
     "pa_gated_linear": (_i, [_i, _p, _l, _p, _l, _p, _l, _i, _p, _p, _l, _p, _p, _p, _f, _f, _f, _l, _p, _l, _p, _p, _p, _p,
                              _i, _i, _p, _i, _i, _i, _i, _p, c_size_t, _p]),
     "pa_narrow_linear": (_i, [_p, _l, _p, _p, _l, _i, _i, _i, _p]),
-    "pa_moe_select": (_i, [_p, _l, _l, _i, _i, _i, _i, _i, _p, _p, _p]),
-    "pa_moe_lists": (_i, [_p, _l, _i, _i, _p, _p, _p]),
+    "pa_moe_workspace_bytes": (c_size_t, [_l, _i, _i]),
+    "pa_moe_choose": (_i, [_p, _l, _l, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, c_size_t, _p]),
     "pa_moe_product": (_i, [_p, _l, _i, _p, _l, _i, _i, _p, _p, _l, _i, _i, _i, _p, _i, _i, _p]),
 })
 SIGNATURES["pa_decode_split"] = SIGNATURES["pa_decode_reduce"] = SIGNATURES["pa_decode"]

@@ -75,31 +75,32 @@ template <int KIND> __device__ __forceinline__ void gl_gate(const GlArgs &a, con
 // ------------------------------------------------------------------ token by token
 constexpr int kRecCols = 64;  // value columns per workgroup: 16 lanes x float4, 16 groups of lanes over the rows of S
 
-// R: rows of S per thread (16 R >= dim)
-template <typename T, int R, int KIND> __global__ __launch_bounds__(256) void gated_recurrent_kernel(const GlArgs a) {
+// R: rows of S per thread (16 R >= dim).  kMlstm: thread d follows n[d].
+template <typename T, int R, int KIND> __global__ __launch_bounds__(256, 4) void gated_recurrent_kernel(const GlArgs a) {
     __shared__ float qs[16 * R], ks[16 * R], vs[kRecCols];
     __shared__ float4 red[16][kRecCols / 4];
-    __shared__ float redn[16];
-    const int b = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kRecCols;
+    __shared__ float redn[4];
+    const int h = blockIdx.y, b = blockIdx.z, v0 = blockIdx.x * kRecCols;
     GlPortion p;
     if (!gl_portion(a, b, p)) return;
     const int tid = threadIdx.x, col = tid % 16 * 4, grp = tid / 16;
     const bool live = v0 + col < a.vp;  // (vp is a multiple of 16)
     float *head = p.slot >= 0 ? a.state + (p.slot * a.heads + h) * a.head_floats : nullptr;
     float *sp = head ? head + v0 + col : nullptr;
-    float *np = head ? head + (int64_t)a.dp * a.vp + blockIdx.z * (int64_t)(a.dp + 16) : nullptr;  // this workgroup's copy
+    float *np = head ? head + (int64_t)a.dp * a.vp + blockIdx.x * (int64_t)(a.dp + 16) : nullptr;  // this workgroup's copy
     const bool resume = head && p.pos0 > 0;
     float4 s[R];
-    float n[R], m = 0.f;
+    float n = 0.f, m = 0.f;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
         const int d = grp + 16 * r;
         s[r] = make_float4(0.f, 0.f, 0.f, 0.f);
-        n[r] = 0.f;
         if (resume && live && d < a.dp) s[r] = *reinterpret_cast<const float4 *>(sp + (int64_t)d * a.vp);
-        if (KIND == kMlstm && resume && d < a.dp) n[r] = np[d];
     }
-    if (KIND == kMlstm && resume) m = np[a.dp];
+    if (KIND == kMlstm && resume) {
+        if (tid < a.dp && tid < 16 * R) n = np[tid];
+        m = np[a.dp];
+    }
     const GlHead hd = gl_head(a, h);
     const int g = h / a.per_group;
     const T *q = reinterpret_cast<const T *>(a.q) + g * a.dim, *k = reinterpret_cast<const T *>(a.k) + g * a.dim;
@@ -133,7 +134,6 @@ template <typename T, int R, int KIND> __global__ __launch_bounds__(256) void ga
         float4 x = *reinterpret_cast<const float4 *>(vs + col);
         x = make_float4(in * x.x, in * x.y, in * x.z, in * x.w);
         float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
-        float nq = 0.f;
 #pragma unroll
         for (int r = 0; r < R; ++r) {
             const float kd = ks[grp + 16 * r], qd = qs[grp + 16 * r];
@@ -141,41 +141,44 @@ template <typename T, int R, int KIND> __global__ __launch_bounds__(256) void ga
             s[r].z = fmaf(keep, s[r].z, kd * x.z); s[r].w = fmaf(keep, s[r].w, kd * x.w);
             o.x = fmaf(qd, s[r].x, o.x); o.y = fmaf(qd, s[r].y, o.y);
             o.z = fmaf(qd, s[r].z, o.z); o.w = fmaf(qd, s[r].w, o.w);
-            if (KIND == kMlstm) {
-                n[r] = fmaf(keep, n[r], in * kd);
-                nq = fmaf(qd, n[r], nq);
-            }
         }
         red[grp][tid % 16] = o;
-        if (KIND == kMlstm && tid % 16 == 0) redn[grp] = nq;
+        if (KIND == kMlstm) {
+            float nq = 0.f;
+            if (tid < 16 * R) {
+                n = fmaf(keep, n, in * ks[tid]);
+                nq = qs[tid] * n;
+            }
+            nq = pa_group_sum<64>(nq);
+            if (tid % 64 == 0) redn[tid / 64] = nq;
+        }
         __syncthreads();
         if (tid < kRecCols && v0 + tid < a.vdim) {
             float sum = 0.f;
 #pragma unroll
             for (int i = 0; i < 16; ++i) sum += reinterpret_cast<const float *>(red[i])[tid];
             if (KIND == kMlstm) {
-                float den = 0.f;
-#pragma unroll
-                for (int i = 0; i < 16; ++i) den += redn[i];
+                const float den = (redn[0] + redn[1]) + (redn[2] + redn[3]);
                 sum = a.q_scale * sum / (fmaxf(fabsf(a.q_scale * den), exp2f(-m)) + a.den_eps);
             } else {
-                sum = fmaf(hd.c, vs[tid], a.q_scale * sum);
+                sum = fmaf(hd.c, vs[tid], sum);
             }
             pa_scalar<T>::store(reinterpret_cast<T *>(a.out) + row * ((int64_t)a.heads * a.vdim) + h * a.vdim + v0 + tid, sum);
         }
         if (KIND == kSsd) __syncthreads();  // (vs is read above)
         // (otherwise: the next token's writes to qs, ks, vs follow every thread's reads of them, before the barrier above;
-        // its writes to red come after its own barrier, which the threads that sum here reach afterwards)
+        // its writes to red and redn come after its own barrier, which the threads that sum here reach afterwards)
     }
     if (!head) return;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
         const int d = grp + 16 * r;
-        if (d >= a.dp) continue;
-        if (live) *reinterpret_cast<float4 *>(sp + (int64_t)d * a.vp) = s[r];
-        if (KIND == kMlstm && tid % 16 == 0) np[d] = n[r];
+        if (live && d < a.dp) *reinterpret_cast<float4 *>(sp + (int64_t)d * a.vp) = s[r];
     }
-    if (KIND == kMlstm && tid == 0) np[a.dp] = m;
+    if (KIND == kMlstm) {
+        if (tid < a.dp && tid < 16 * R) np[tid] = n;
+        if (tid == 0) np[a.dp] = m;
+    }
 }
 
 // ------------------------------------------------------------------ chunks on the matrix cores
@@ -197,28 +200,35 @@ template <int KD, int NW, int KIND, bool STATES> constexpr size_t gl_lds_bytes()
     return elems * 2 + (STATES ? 2 : 1) * sizeof(GlRows) + (KIND == kMlstm && !STATES ? (3 * 64 + KD) * 4 : 0);
 }
 
+// Inclusive scans over the wave: rows of 16 lanes by shifts inside the row, then the rows before.
+template <int CTRL> __device__ __forceinline__ float gl_shift(float x, float outside) {
+    return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(__builtin_bit_cast(int, outside), __builtin_bit_cast(int, x), CTRL, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float gl_lane(float x, int lane) {
+    return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, x), lane));
+}
 __device__ __forceinline__ float gl_scan_add(float x, int lane) {
-#pragma unroll
-    for (int d = 1; d < 64; d *= 2) {
-        const float y = __shfl_up(x, d, 64);
-        if (lane >= d) x += y;
-    }
-    return x;
+    x += gl_shift<0x111>(x, 0.f);
+    x += gl_shift<0x112>(x, 0.f);
+    x += gl_shift<0x114>(x, 0.f);
+    x += gl_shift<0x118>(x, 0.f);
+    const float r0 = gl_lane(x, 15), r1 = r0 + gl_lane(x, 31), r2 = r1 + gl_lane(x, 47);
+    return x + (lane < 16 ? 0.f : lane < 32 ? r0 : lane < 48 ? r1 : r2);
 }
 __device__ __forceinline__ float gl_scan_max(float x, int lane) {
-#pragma unroll
-    for (int d = 1; d < 64; d *= 2) {
-        const float y = __shfl_up(x, d, 64);
-        if (lane >= d) x = fmaxf(x, y);
-    }
-    return x;
+    x = fmaxf(x, gl_shift<0x111>(x, kGlNone));
+    x = fmaxf(x, gl_shift<0x112>(x, kGlNone));
+    x = fmaxf(x, gl_shift<0x114>(x, kGlNone));
+    x = fmaxf(x, gl_shift<0x118>(x, kGlNone));
+    const float r0 = gl_lane(x, 15), r1 = fmaxf(r0, gl_lane(x, 31)), r2 = fmaxf(r1, gl_lane(x, 47));
+    return fmaxf(x, lane < 16 ? kGlNone : lane < 32 ? r0 : lane < 48 ? r1 : r2);
 }
 
 // KD: dim padded to 64, 128 or 256.  NW: waves; each owns 16 value columns.  All products are taken transposed (value
 // columns, or keys, as the rows of the result), so that a lane holds four consecutive elements of one row t.
 // STATES: only the segment's own contribution to the state, to the workspace (first pass over a portion in segments).
 template <int KD, int NW, int KIND, bool STATES>
-__global__ __launch_bounds__(64 * NW, 2) void gated_chunk_kernel(const GlArgs a) {
+__global__ __launch_bounds__(64 * NW, NW == 4 && KD == 256 ? 1 : 2) void gated_chunk_kernel(const GlArgs a) {
     constexpr int kCols = 16 * NW, kLdR = KD + 8, kThr = 64 * NW;
     constexpr int kDB = KD / 4, kKBlocks = 16 * kDB, kKPass = (kKBlocks + kThr - 1) / kThr;  // 4x4 blocks of K
     constexpr int kST = NW == 8 ? 2 : 4;  // score tiles per wave
@@ -321,7 +331,7 @@ __global__ __launch_bounds__(64 * NW, 2) void gated_chunk_kernel(const GlArgs a)
             float decay, in;
             gl_gate<KIND>(a, hd, raw_a, raw_b, decay, in);
             if (tid >= nv) decay = 0.f;
-            const float f = gl_scan_add(decay, tid), f_last = __shfl(f, 63, 64);
+            const float f = gl_scan_add(decay, tid), f_last = gl_lane(f, 63);
             if constexpr (KIND == kSsd) {
                 const float mul = tid < nv ? in : 0.f;
                 rows->row[tid] = f;
@@ -332,7 +342,7 @@ __global__ __launch_bounds__(64 * NW, 2) void gated_chunk_kernel(const GlArgs a)
                 if (tid == 0) rows->whole = exp2f(f_last);
             } else {
                 const float col = tid < nv ? in - f : kGlNone;
-                const float top = fmaxf(m_prev, gl_scan_max(col, tid)), top_last = __shfl(top, 63, 64);
+                const float top = fmaxf(m_prev, gl_scan_max(col, tid)), top_last = gl_lane(top, 63);
                 rows->row[tid] = -top;
                 rows->col[tid] = col;
                 rows->inter[tid] = exp2f(m_prev - top);
@@ -605,15 +615,17 @@ template <int KIND> int launch_chunks_kind(const GlArgs &a, int batch, hipStream
 }
 
 template <typename T, int KIND> void launch_recurrent(const GlArgs &a, int batch, hipStream_t s) {
-    const dim3 grid((unsigned)batch, (unsigned)a.heads, (unsigned)((a.vdim + kRecCols - 1) / kRecCols)), block(256);
+    // (a head's slices, whose rows lie side by side in memory, run at the same time)
+    const dim3 grid((unsigned)((a.vdim + kRecCols - 1) / kRecCols), (unsigned)a.heads, (unsigned)batch), block(256);
     if (a.dim <= 64) gated_recurrent_kernel<T, 4, KIND><<<grid, block, 0, s>>>(a);
     else if (a.dim <= 128) gated_recurrent_kernel<T, 8, KIND><<<grid, block, 0, s>>>(a);
     else gated_recurrent_kernel<T, 16, KIND><<<grid, block, 0, s>>>(a);
 }
 
-int gl_plan(int64_t batch, int heads, int vdim, int max_q_len) {
+int gl_plan(int64_t batch, int heads, int dim, int vdim, int max_q_len) {
     const int cols = la_value_cols(vdim);
-    return la_segments(batch * heads * ((vdim + cols - 1) / cols), la_cus(), max_q_len);
+    const int at_once = cols == 64 && dim <= 128 ? 2 * la_cus() : la_cus();  // workgroups: two of four waves fit a compute unit
+    return la_segments(batch * heads * ((vdim + cols - 1) / cols), at_once, max_q_len);
 }
 
 }  // namespace
@@ -628,7 +640,7 @@ extern "C" size_t pa_gated_linear_workspace_bytes(int batch, int num_heads, int 
         pa_fail(PA_ERR_INVALID_ARG, "pa_gated_linear_workspace_bytes: sizes out of range");
         return 0;
     }
-    return gl_workspace_bytes(batch, num_heads, dim, vdim, gl_plan(batch, num_heads, vdim, max_q_len));
+    return gl_workspace_bytes(batch, num_heads, dim, vdim, gl_plan(batch, num_heads, dim, vdim, max_q_len));
 }
 
 extern "C" int pa_gated_linear(int kind, const void *q, int64_t q_stride, const void *k, int64_t k_stride, const void *v,
@@ -683,7 +695,7 @@ extern "C" int pa_gated_linear(int kind, const void *q, int64_t q_stride, const 
         PA_CHECK_LAUNCH("pa_gated_linear");
         return PA_OK;
     }
-    a.segments = gl_plan(batch, num_heads, vdim, max_q_len);
+    a.segments = gl_plan(batch, num_heads, dim, vdim, max_q_len);
     while (a.segments > 1 && (!workspace || gl_workspace_bytes(batch, num_heads, dim, vdim, a.segments) > workspace_bytes))
         --a.segments;
     a.seg_rows = la_segment_rows(max_q_len, a.segments);

@@ -9,10 +9,20 @@ static inline int64_t moe_max_tiles(int64_t items, int experts, int bm) {
     return lists + (items - lists) / bm;
 }
 
-enum MoeShape { kMoeStream16, kMoeStream32, kMoeStream64, kMoeTile64, kMoeTile256 };
+enum MoeShape { kMoeStream, kMoeTile64, kMoeTile256 };
 
 // By the items an expert has on average (lists of unequal length fill the next tile up).
 static inline MoeShape moe_shape(int64_t items, int experts) {
     const int64_t mean = items / experts;
-    return mean <= 8 ? kMoeStream16 : mean <= 20 ? kMoeStream32 : mean <= 48 ? kMoeStream64 : mean <= 160 ? kMoeTile64 : kMoeTile256;
+    return mean <= 4 ? kMoeStream : mean <= 160 ? kMoeTile64 : kMoeTile256;
 }
+
+// Rows of a part of the choice of experts (one workgroup): few parts, so that a part's place behind the others is quickly
+// summed, but one row per wave (sixteen per workgroup) while there are few rows; a part's items fit LDS.
+static inline int moe_part_rows(int64_t rows, int top) {
+    int64_t n = (rows + 255) / 256;
+    if (n < 16) n = 16;
+    const int64_t most = 8192 / top;
+    return (int)(n < most ? n : most);
+}
+static inline int64_t moe_parts(int64_t rows, int top) { return (rows + moe_part_rows(rows, top) - 1) / moe_part_rows(rows, top); }

@@ -5,7 +5,7 @@ among the best groups of experts; a shared expert may run for every token.  The
 step stays on the device from the router to the weighted sum:
 
 ``pa_narrow_linear`` (router logits and the shared expert's gate, 32-bit) ->
-``pa_moe_select`` -> ``pa_moe_lists`` -> ``pa_moe_product`` with the gated
+``pa_moe_choose`` -> ``pa_moe_product`` with the gated
 activation in its epilogue -> ``pa_moe_product``; the weighted sum over a token's
 experts is part of the residual sum that follows (``pa_residual_norm``).
 """

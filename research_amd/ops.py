@@ -634,7 +634,7 @@ class ExpertChoice(NamedTuple):
 
 
 def moe_choose(logits: Tensor, experts: int, top: int, groups: int, keep: int) -> ExpertChoice:
-    """``pa_moe_select`` and ``pa_moe_lists`` over float32 ``logits`` ``[rows, experts]``, or one column more for the gate of a
+    """``pa_moe_choose`` over float32 ``logits`` ``[rows, experts]``, or one column more for the gate of a
     shared expert."""
     rows = logits.shape[0]
     _dense(logits)
@@ -646,9 +646,9 @@ def moe_choose(logits: Tensor, experts: int, top: int, groups: int, keep: int) -
     weights = torch.empty((rows, top + 1), dtype=torch.float32, device=dev)
     counts = torch.empty(experts, dtype=torch.int32, device=dev)
     lists = torch.empty((experts, rows), dtype=torch.int32, device=dev)
-    _run("pa_moe_select", _ptr(logits), logits.shape[1], rows, experts, top, groups, keep, int(logits.shape[1] > experts),
-         _ptr(ids), _ptr(weights), _stream(logits))
-    _run("pa_moe_lists", _ptr(ids), rows, top, experts, _ptr(counts), _ptr(lists), _stream(logits))
+    workspace = torch.empty(int(_lib.load().pa_moe_workspace_bytes(rows, experts, top)), dtype=torch.uint8, device=dev)
+    _run("pa_moe_choose", _ptr(logits), logits.shape[1], rows, experts, top, groups, keep, int(logits.shape[1] > experts),
+         _ptr(ids), _ptr(weights), _ptr(counts), _ptr(lists), _ptr(workspace), workspace.numel(), _stream(logits))
     return ExpertChoice(ids, weights, counts, lists)
 
 

@@ -317,12 +317,15 @@ def test_recurrence_and_expert_entry_points_check_their_arguments():
     assert rc == -1 and "x_stride" in msg
     for args, status, text in (((9, 2, 2, 1), -1, "equal groups"), ((8, 5, 2, 1), -1, "cannot be chosen"), ((8, 2, 2, 3), -1, "cannot be chosen"),
                                ((2048, 2, 1, 1), -2, "above")):
-        rc, msg = _status("pa_moe_select", FAKE, 4096, 4, *args, 0, FAKE, FAKE, None)
+        rc, msg = _status("pa_moe_choose", FAKE, 4096, 4, *args, 0, FAKE, FAKE, FAKE, FAKE, FAKE, 1 << 20, None)
         assert rc == status and text in msg, (args, msg)
-    rc, msg = _status("pa_moe_select", FAKE, 8, 4, 8, 2, 1, 1, 1, FAKE, FAKE, None)
+    rc, msg = _status("pa_moe_choose", FAKE, 8, 4, 8, 2, 1, 1, 1, FAKE, FAKE, FAKE, FAKE, FAKE, 1 << 20, None)
     assert rc == -1 and "logits_stride" in msg
-    rc, msg = _status("pa_moe_lists", FAKE, 4, 2, 8, None, FAKE, None)
+    rc, msg = _status("pa_moe_choose", FAKE, 8, 4, 8, 2, 1, 1, 0, FAKE, FAKE, None, FAKE, FAKE, 1 << 20, None)
     assert rc == -1 and "NULL" in msg
+    rc, msg = _status("pa_moe_choose", FAKE, 8, 4, 8, 2, 1, 1, 0, FAKE, FAKE, FAKE, FAKE, FAKE, 8, None)
+    assert rc == -3 and "needed" in msg
+    assert lib.pa_moe_workspace_bytes(16384, 64, 8) == 256 * 64 * 4
     product = lambda **kw: [{**dict(x=FAKE, lx=64, ipr=2, w=FAKE, wr=96, lw=64, k=64, c=FAKE, l=FAKE, rows=4, top=2, e=8, glu=1, out=FAKE, n=48,
                                     dt=bf16, s=None), **kw}[k] for k in ("x", "lx", "ipr", "w", "wr", "lw", "k", "c", "l", "rows", "top", "e",
                                                                          "glu", "out", "n", "dt", "s")]

@@ -432,7 +432,8 @@ def test_narrow_products_are_32_bit(rows, n, k, dtype):
 
 
 @pytest.mark.parametrize("rows,experts,top,groups,keep,shared", [(1, 6, 2, 3, 2, True), (37, 8, 3, 2, 1, False), (130, 5, 4, 1, 1, True), (64, 256, 8, 8, 4, True),
-                                                                (9, 100, 20, 100, 40, False), (2000, 16, 4, 4, 2, True), (3, 1, 1, 1, 1, False)])
+                                                                (9, 100, 20, 100, 40, False), (2000, 16, 4, 4, 2, True), (3, 1, 1, 1, 1, False),
+                                                                (50, 1000, 10, 20, 5, True), (5000, 120, 6, 12, 12, True)])
 def test_choice_of_experts(rows, experts, top, groups, keep, shared):
     announce(f"choose {rows} {experts} {top} {groups} {keep}")
     logits = _rand(rows, experts + shared, seed=rows)

@@ -198,7 +198,12 @@ int main() {
         }
         if (tiles > moe_max_tiles(items, experts, bm)) return 4;
     }
-    if (moe_shape(7, 8) != kMoeStream16 || moe_shape(1 << 20, 8) != kMoeTile256) return 5;
+    for (long long rows = 1; rows < 3000000; rows = rows * 3 / 2 + 1)
+        for (int top : {1, 3, 8, 64}) {
+            const long long part = moe_part_rows(rows, top), parts = moe_parts(rows, top);
+            if (part < 1 || part * top > 8192 || part * parts < rows || part * (parts - 1) >= rows) return 7;
+        }
+    if (moe_shape(7, 8) != kMoeStream || moe_shape(1 << 20, 8) != kMoeTile256) return 5;
     if (gl_state_floats(true, 20, 130) != 32 * 144 + 3 * 48 || gl_workspace_bytes(2, 3, 20, 40, 4) != 2ull * 3 * 4 * (32 * 48 + 48) * 4) return 6;
     std::puts("ok");
 }
