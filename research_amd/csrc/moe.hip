@@ -5,11 +5,11 @@
 // at the item's number, so nothing is sorted in memory: the lists say which rows an expert reads and writes, and the
 // weighted sum over a token's items happens where the result is used (pa_residual_norm).  No counts go through the host.
 //
-// Product kernels, by how many tokens an expert has on average: tiles through LDS (the loads go straight to LDS, a
-// ring of steps, one barrier per step), or, for a few tokens per expert, weights streamed from
-// memory into registers.  The weights' rows are zero-padded to whole 64-element steps; token rows are not read past
-// their end.  All products are taken transposed (weight rows as the rows of the result), so that a lane holds four
-// consecutive outputs of one item.
+// Product kernels, by how many tokens an expert has on average (moe_plan.h): weights streamed from memory into registers
+// for a few; 64 x 128 tiles through a ring of LDS buffers; 256 x 256 tiles by workgroups that stay on their compute unit.
+// 32-bit operands have a plain kernel.  The weights' rows are zero-padded to whole 64-element steps; token rows are not
+// read past their end.  All products are taken transposed (weight rows as the rows of the result), so that a lane holds
+// four consecutive outputs of one item.
 #include "moe_plan.h"
 #include "row_common.h"
 
