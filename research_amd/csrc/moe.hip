@@ -141,24 +141,33 @@ template <typename T> __global__ __launch_bounds__(256) void narrow_dot_kernel(c
 struct ChooseArgs {
     const float *logits;  // [rows][ld]: the experts', then (shared) one for the shared expert's gate
     int64_t ld, rows;
+    const float *correction;  // [experts]: added to the scores where they choose, or NULL
     int32_t *ids;    // [rows][top]
-    float *weights;  // [rows][top + 1], the last one the shared expert's
+    float *weights;  // [rows][top + 1], the last one the shared expert's; with identity experts one more, the sum of theirs
     int32_t *partial;  // [parts][experts]: how many items of each expert the rows of a part have
     int32_t *counts, *lists;
     int experts, top, groups, keep, shared, part_rows;
+    int real;  // experts from here on are identity experts
+    int softmax, group_top, renormalize;
 };
+
+constexpr float kMoeNone = -3.0e38f;  // stands for minus infinity
+
+__device__ __forceinline__ float moe_wave_max(float top) {
+    top = fmaxf(top, pa_dpp<0xB1>(top));   // (the patterns of pa_group_sum)
+    top = fmaxf(top, pa_dpp<0x4E>(top));
+    top = fmaxf(top, pa_dpp<0x141>(top));
+    top = fmaxf(top, pa_dpp<0x140>(top));
+    auto lane_of = [&](int l) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, top), l)); };
+    return fmaxf(fmaxf(lane_of(0), lane_of(16)), fmaxf(lane_of(32), lane_of(48)));
+}
 
 // The largest of NPL values per lane, value i * 64 + lane: its number, the lowest on ties, or -1 when none is above `floor`.
 template <int NPL> __device__ __forceinline__ int moe_argmax(const float (&v)[NPL], float floor, float &best) {
     float top = v[0];
 #pragma unroll
     for (int i = 1; i < NPL; ++i) top = fmaxf(top, v[i]);
-    top = fmaxf(top, pa_dpp<0xB1>(top));   // (the patterns of pa_group_sum)
-    top = fmaxf(top, pa_dpp<0x4E>(top));
-    top = fmaxf(top, pa_dpp<0x141>(top));
-    top = fmaxf(top, pa_dpp<0x140>(top));
-    auto lane_of = [&](int l) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, top), l)); };
-    best = fmaxf(fmaxf(lane_of(0), lane_of(16)), fmaxf(lane_of(32), lane_of(48)));
+    best = moe_wave_max(top);
     if (!(best > floor)) return -1;
 #pragma unroll
     for (int i = 0; i < NPL; ++i) {
@@ -180,12 +189,34 @@ template <int NPL, int NW> __global__ __launch_bounds__(64 * NW) void moe_choose
     const int64_t first = (int64_t)blockIdx.x * a.part_rows, end = first + a.part_rows < a.rows ? first + a.part_rows : a.rows;
     for (int64_t row = first + wave; row < end; row += NW) {
         const float *logit = a.logits + row * a.ld;
-        float s[NPL];  // (scores are positive: a value that is not, or is NaN, cannot be chosen)
+        float s[NPL], weight[NPL];  // what chooses, and what weighs  (a value that is NaN, or not above kMoeNone, cannot be chosen)
+        if (a.softmax) {
+            float most = kMoeNone, sum = 0.f;
+#pragma unroll
+            for (int i = 0; i < NPL; ++i) {
+                const int e = i * 64 + lane;
+                s[i] = e < a.experts ? logit[e] : kMoeNone;
+                most = fmaxf(most, s[i]);
+            }
+            most = moe_wave_max(most);
+#pragma unroll
+            for (int i = 0; i < NPL; ++i) {
+                weight[i] = i * 64 + lane < a.experts ? expf(s[i] - most) : 0.f;
+                sum += weight[i];
+            }
+            sum = pa_group_sum<64>(sum);
+#pragma unroll
+            for (int i = 0; i < NPL; ++i) weight[i] /= sum;
+        } else {
+#pragma unroll
+            for (int i = 0; i < NPL; ++i) weight[i] = i * 64 + lane < a.experts ? 1.f / (1.f + expf(-logit[i * 64 + lane])) : 0.f;
+        }
 #pragma unroll
         for (int i = 0; i < NPL; ++i) {
             const int e = i * 64 + lane;
-            s[i] = e < a.experts ? 1.f / (1.f + expf(-logit[e])) : -1.f;
-            if (!(s[i] >= 0.f)) s[i] = -1.f;
+            s[i] = kMoeNone;
+            if (e < a.experts) s[i] = weight[i] + (a.correction ? a.correction[e] : 0.f);
+            if (!(s[i] > kMoeNone)) s[i] = kMoeNone;
         }
         if (a.keep < a.groups) {
             // (a wave's own part of LDS: its accesses are in order, the compiler must keep them so)
@@ -195,56 +226,67 @@ template <int NPL, int NW> __global__ __launch_bounds__(64 * NW) void moe_choose
                 if (i * 64 + lane < a.experts) row_s[i * 64 + lane] = s[i];
             __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
             __builtin_amdgcn_wave_barrier();
-            float value[NPL];  // a group's value: its two largest scores
+            float value[NPL];  // a group's value: its largest score, or its two largest
             bool able[NPL];
 #pragma unroll
             for (int i = 0; i < NPL; ++i) {
                 const int g = i * 64 + lane;
-                value[i] = -1.f;
+                value[i] = kMoeNone;
                 able[i] = false;
                 if (g >= a.groups) continue;
-                float one = -1.f, two = 0.f;
+                float one = kMoeNone, two = kMoeNone;
                 for (int e = g * size; e < (g + 1) * size; ++e) {
                     const float x = row_s[e];
                     two = fmaxf(two, fminf(one, x));
                     one = fmaxf(one, x);
                 }
-                value[i] = one + two;
+                value[i] = a.group_top == 1 || two == kMoeNone ? one : one + two;
             }
             for (int k = 0; k < a.keep; ++k) {
                 float best;
-                const int g = moe_argmax<NPL>(value, -1.f, best);
+                const int g = moe_argmax<NPL>(value, kMoeNone, best);
 #pragma unroll
                 for (int i = 0; i < NPL; ++i) {
-                    if (i * 64 + lane == g) value[i] = -1.f;
-                    able[i] |= (i * 64 + lane) / size == g;
+                    if (i * 64 + lane == g) value[i] = kMoeNone;
+                    able[i] |= g >= 0 && (i * 64 + lane) / size == g;
                 }
             }
 #pragma unroll
             for (int i = 0; i < NPL; ++i)
-                if (!able[i]) s[i] = -1.f;
+                if (!able[i]) s[i] = kMoeNone;
         }
         float sum = 0.f, mine = 0.f;
         int my_id = -1;
         for (int k = 0; k < a.top; ++k) {
-            float best;
-            const int at = moe_argmax<NPL>(s, -1.f, best);
+            float best, took = 0.f;
+            const int at = moe_argmax<NPL>(s, kMoeNone, best);
             if (at < 0) break;
 #pragma unroll
             for (int i = 0; i < NPL; ++i)
-                if (i * 64 + lane == at) s[i] = -1.f;
-            sum += best;
+                if (i == at / 64) {  // (uniform)
+                    took = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, weight[i]), at % 64));
+                    if (lane == at % 64) s[i] = kMoeNone;
+                }
+            sum += took;
             if (lane == k) {
-                mine = best;
+                mine = took;
                 my_id = at;
             }
         }
+        if (a.renormalize) mine /= sum + 1e-20f;
+        // an identity expert's item is in no list: its weight goes to the row's own input
+        const bool same = my_id >= a.real;
+        const int ld_w = a.top + (a.real < a.experts ? 2 : 1);
+        const float own = a.real < a.experts ? pa_group_sum<64>(lane < a.top && same ? mine : 0.f) : 0.f;
         if (lane < a.top) {
-            a.ids[row * a.top + lane] = my_id;
-            a.weights[row * (a.top + 1) + lane] = mine / (sum + 1e-20f);
-            if (my_id >= 0) atomicAdd(hist + my_id, 1);
+            a.ids[row * a.top + lane] = same ? -1 : my_id;
+            a.weights[row * ld_w + lane] = same ? 0.f : mine;
+            if (my_id >= 0 && !same) atomicAdd(hist + my_id, 1);
         }
-        if (lane == 0) a.weights[row * (a.top + 1) + a.top] = a.shared ? 1.f / (1.f + expf(-logit[a.experts])) : 0.f;
+        if (lane == 0) {
+            a.weights[row * ld_w + a.top] = a.shared == PA_MOE_SHARED_GATED ? 1.f / (1.f + expf(-logit[a.experts])) : a.shared ? 1.f : 0.f;
+            if (a.real < a.experts) a.weights[row * ld_w + a.top + 1] = own;
+        }
     }
     __syncthreads();
     for (int e = tid; e < a.experts; e += 64 * NW) a.partial[(int64_t)blockIdx.x * a.experts + e] = hist[e];
@@ -871,30 +913,35 @@ extern "C" size_t pa_moe_workspace_bytes(int64_t rows, int experts, int top) {
     return (size_t)moe_parts(rows, top) * experts * sizeof(int32_t);
 }
 
-extern "C" int pa_moe_choose(const float *logits, int64_t logits_stride, int64_t rows, int experts, int top, int groups, int keep,
-                             int shared, int32_t *ids, float *weights, int32_t *counts, int32_t *lists, void *workspace,
-                             size_t workspace_bytes, void *stream) {
+extern "C" int pa_moe_choose(const float *logits, int64_t logits_stride, int64_t rows, int experts, int identity, int top, int groups,
+                             int keep, int shared, int scores, int group_top, int renormalize, const float *correction, int32_t *ids,
+                             float *weights, int32_t *counts, int32_t *lists, void *workspace, size_t workspace_bytes, void *stream) {
     pa_clear_error();
-    PA_REQUIRE(rows >= 0 && experts > 0 && top > 0 && groups > 0, "pa_moe_choose: sizes out of range");
-    PA_REQUIRE(experts % groups == 0, "experts=%d are not %d equal groups", experts, groups);
-    PA_REQUIRE(keep > 0 && keep <= groups && top <= keep * (experts / groups), "%d experts cannot be chosen from %d of %d groups of %d", top,
-               keep, groups, experts / groups);
-    if (top > 64 || experts > 1024) return pa_fail(PA_ERR_UNSUPPORTED, "pa_moe_choose: top=%d above 64 or experts=%d above 1024", top, experts);
-    PA_REQUIRE(logits_stride >= experts + (shared ? 1 : 0), "logits_stride=%lld is shorter than a row", (long long)logits_stride);
+    PA_REQUIRE(rows >= 0 && experts > 0 && identity >= 0 && top > 0 && groups > 0, "pa_moe_choose: sizes out of range");
+    const int all = experts + identity;
+    PA_REQUIRE(all % groups == 0, "experts=%d are not %d equal groups", all, groups);
+    PA_REQUIRE(keep > 0 && keep <= groups && top <= keep * (all / groups), "%d experts cannot be chosen from %d of %d groups of %d", top,
+               keep, groups, all / groups);
+    if (top > 64 || all > 1024) return pa_fail(PA_ERR_UNSUPPORTED, "pa_moe_choose: top=%d above 64 or experts=%d above 1024", top, all);
+    PA_REQUIRE(scores == PA_MOE_SIGMOID || scores == PA_MOE_SOFTMAX, "scores=%d is unknown", scores);
+    PA_REQUIRE(group_top == 1 || group_top == 2, "group_top=%d is not 1 or 2", group_top);
+    PA_REQUIRE(shared >= PA_MOE_NO_SHARED && shared <= PA_MOE_SHARED, "shared=%d is unknown", shared);
+    PA_REQUIRE(logits_stride >= all + (shared == PA_MOE_SHARED_GATED ? 1 : 0), "logits_stride=%lld is shorter than a row", (long long)logits_stride);
     PA_REQUIRE(rows * top <= 0x7fffffff, "pa_moe_choose: rows=%lld is too large for one launch", (long long)rows);
     if (rows == 0) return PA_OK;
     PA_REQUIRE(logits && ids && weights && counts && lists, "NULL argument");
-    if (!workspace || workspace_bytes < pa_moe_workspace_bytes(rows, experts, top))
+    if (!workspace || workspace_bytes < pa_moe_workspace_bytes(rows, all, top))
         return pa_fail(PA_ERR_WORKSPACE, "pa_moe_choose: workspace of %zu bytes, %zu needed", workspace_bytes,
-                       pa_moe_workspace_bytes(rows, experts, top));
+                       pa_moe_workspace_bytes(rows, all, top));
     const int part_rows = moe_part_rows(rows, top);
-    ChooseArgs a{logits, logits_stride, rows, ids, weights, (int32_t *)workspace, counts, lists, experts, top, groups, keep, shared, part_rows};
+    ChooseArgs a{logits, logits_stride, rows, correction, ids, weights, (int32_t *)workspace, counts, lists, all, top, groups, keep, shared,
+                 part_rows, experts, scores == PA_MOE_SOFTMAX, group_top, renormalize};
     const dim3 grid((unsigned)moe_parts(rows, top));
-    auto lds = [&](int waves) { return (size_t)(1 + waves) * experts * sizeof(float); };
+    auto lds = [&](int waves) { return (size_t)(1 + waves) * all * sizeof(float); };
     hipStream_t s = (hipStream_t)stream;
-    if (experts <= 64) moe_choose_kernel<1, 16><<<grid, dim3(1024), lds(16), s>>>(a);
-    else if (experts <= 128) moe_choose_kernel<2, 16><<<grid, dim3(1024), lds(16), s>>>(a);
-    else if (experts <= 256) moe_choose_kernel<4, 16><<<grid, dim3(1024), lds(16), s>>>(a);
+    if (all <= 64) moe_choose_kernel<1, 16><<<grid, dim3(1024), lds(16), s>>>(a);
+    else if (all <= 128) moe_choose_kernel<2, 16><<<grid, dim3(1024), lds(16), s>>>(a);
+    else if (all <= 256) moe_choose_kernel<4, 16><<<grid, dim3(1024), lds(16), s>>>(a);
     else moe_choose_kernel<16, 4><<<grid, dim3(256), lds(4), s>>>(a);
     PA_CHECK_LAUNCH("pa_moe_choose");
     moe_lists_kernel<<<grid, dim3(kListThreads), (size_t)part_rows * top * sizeof(int32_t), s>>>(a);

@@ -224,6 +224,7 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(const RmsGateArgs a) {
         for (int j = 0; j < V; ++j) {
             o[j] = x[i][j] * inv * w[j];
             if (a.gate == PA_GATE_SIGMOID_LAST) o[j] *= row_sigmoid<T>(g[i][j]);
+            if (a.gate == PA_GATE_SILU_LAST) o[j] *= row_silu<T>(g[i][j]);
         }
         row_store<T, V>(dst + c, o);
     }
@@ -376,7 +377,7 @@ extern "C" int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride,
     const int per = width / groups;
     const int64_t parts = rows * groups;
     if (int rc = check_rows("pa_rms_gate", rows < 0 ? rows : parts, per, dtype)) return rc;
-    PA_REQUIRE(gate_mode == PA_GATE_SIGMOID_LAST || gate_mode == PA_GATE_SILU_FIRST, "gate_mode=%d is unknown", gate_mode);
+    PA_REQUIRE(gate_mode >= PA_GATE_SIGMOID_LAST && gate_mode <= PA_GATE_SILU_LAST, "gate_mode=%d is unknown", gate_mode);
     if (rows == 0) return PA_OK;
     PA_REQUIRE(o && gate && weight && out, "NULL argument");
     PA_REQUIRE(gate_stride >= width, "gate_stride=%lld is shorter than a row", (long long)gate_stride);
