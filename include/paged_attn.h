@@ -45,7 +45,7 @@ extern "C" {
 #define PA_F16 2
 #define PA_FP8_E4M3 3 /* OCP e4m3fn, KV pool only; q/out stay 16- or 32-bit */
 
-/* Library ABI version (bumped when an entry point is added or a signature or contract changes; now 8). */
+/* Library ABI version (bumped when an entry point is added or a signature or contract changes; now 9). */
 int pa_version(void);
 
 /* Text of the calling thread's most recent error; "" if none. */
@@ -403,8 +403,14 @@ int pa_dequantize_blocks_e4m3(const void *cache, const float *scale, const int32
 #define PA_ACT_NONE 2
 #define PA_GATE_SIGMOID_LAST 0 /* norm, then sigmoid(gate) */
 #define PA_GATE_SILU_FIRST 1   /* silu(gate), then norm */
+#define PA_GATE_SILU_LAST 2    /* norm, then silu(gate) */
 #define PA_GL_SSD 0            /* recurrences of pa_gated_linear */
 #define PA_GL_MLSTM 1
+#define PA_MOE_SIGMOID 0 /* scores of pa_moe_choose */
+#define PA_MOE_SOFTMAX 1
+#define PA_MOE_NO_SHARED 0
+#define PA_MOE_SHARED_GATED 1 /* weight sigmoid(its logit) */
+#define PA_MOE_SHARED 2       /* weight 1 */
 #define PA_V_PLAIN 0 /* values as they are */
 #define PA_V_FIRST 1 /* values as they are, also written to v_first */
 #define PA_V_MIX 2   /* (1 - lambda) value + lambda v_first */
@@ -434,6 +440,7 @@ int pa_residual_norm(float *x, const void *y, const float *mix_weight, int mix, 
  * A gated RMS norm of each of `groups` equal parts of a row:
  *     PA_GATE_SIGMOID_LAST   out = o / rms(o) * weight * sigmoid(gate)
  *     PA_GATE_SILU_FIRST     z = o * silu(gate), out = z / rms(z) * weight
+ *     PA_GATE_SILU_LAST      out = o / rms(o) * weight * silu(gate)
  * gate and out rows are gate_stride and out_stride elements apart; weight : float[width].
  */
 int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride, const float *weight, float eps, void *out,
@@ -552,21 +559,88 @@ int pa_narrow_linear(const void *x, int64_t x_stride, const void *w, float *out,
                      void *stream);
 
 /*
- * Mixture of experts.  pa_moe_choose, per row: scores s = sigmoid(logits); of `groups` equal groups of neighbours the
- * `keep` with the largest sums of their two largest scores stay; of their experts the `top` with the largest scores are
- * chosen (the lowest number first on ties).  ids int32[rows][top]; weights float[rows][top + 1]: the chosen scores over
- * (their sum + 1e-20), then sigmoid(logits[experts]) when `shared`, else 0.  top <= 64, experts <= 1024.  And per
- * expert counts int32[experts] and lists int32[experts][rows]: its items (row * top + place) in order.  (Scores that are
- * NaN are not chosen: id -1.)  The workspace needs no initial contents.
+ * The gated delta rule.  Per head, with q and k of group h / heads_per_group divided by sqrt(sum of squares + 1e-6) and q also
+ * times q_scale:
+ *     g_t = exp(-decay_rate softplus(decay_logit + decay_bias));  beta_t = sigmoid(beta_logit);
+ *     S <- g_t S_(t-1);  u = beta_t (v_t - S^T k_t);  S_t = S + k_t u^T;  o_t = S_t^T q_t
+ * Tensors, state (float[state_rows][heads][pad16(dim)][pad16(vdim)]) and kernels as in pa_gated_linear; 16-bit portions are
+ * multiplied in chunks of 64 rows when the workspace holds pa_delta_workspace_bytes, else they run token by token.
+ */
+size_t pa_delta_workspace_bytes(int batch, int num_heads, int dim, int vdim, int max_q_len);
+int pa_delta(const void *q, int64_t q_stride, const void *k, int64_t k_stride, const void *v, int64_t v_stride,
+             int heads_per_group, const void *decay_logits, const void *beta_logits, int64_t gate_stride,
+             const float *decay_bias, const float *decay_rate, float q_scale, int64_t n_rows, float *state,
+             int64_t state_rows, const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
+             const int32_t *state_slots, int batch, int max_q_len, void *out, int num_heads, int dim, int vdim, int dtype,
+             void *workspace, size_t workspace_bytes, void *stream);
+
+/*
+ * Residual streams (hyper-connections), one row at a time: x[row][s], s < streams <= 16.
+ *     x_t = table[ids[row]] for every t             when ids is given; else, when y is given,
+ *     x_t = sum_s between[s][t] x_s + into[t] y     (all from the old streams; written back unless `sum` is given)
+ *     z = sum_t sum_weight[t] x_t                   (NULL: ones)
+ *     out = z / rms(z) * norm_weight;  sum = z      whichever is given
+ * With mix_weight (float[rows][mix_stride]) y is the weighted sum over i < mix of y[row * mix + i], plus y_extra[row] under
+ * weight mix and y_self[row] under weight mix + 1 where given; rows under a weight of exactly 0 are not read.
+ *   x : float[rows][streams][width];  y, y_extra, y_self, table, out : dtype;  sum : float[rows][width];  width <= 16384
+ */
+int pa_hyper_norm(float *x, const void *y, const float *mix_weight, int mix, int mix_stride, const void *y_extra,
+                  const void *y_self, const float *between, const float *into, const int64_t *ids, const void *table,
+                  int64_t table_rows, const float *sum_weight, const float *norm_weight, float eps, void *out, float *sum,
+                  int64_t rows, int streams, int width, int dtype, void *stream);
+
+/*
+ * Latent attention's operands from rows [heads of dim + rot_dim | rank | rot_dim]: q_out gets every head times q_scale with
+ * its last rot_dim elements turned (pairs 2i, 2i + 1 by rope[position][i]), zeros up to q_dim; the pool's row of the token
+ * is [rank elements / rms * norm_weight | last rot_dim elements turned | zeros] of pool_row elements.  Portions, tiles and
+ * slots as in pa_qkv_conv_append.
+ * pa_latent_gather: out[r] = pool row slots[r], zeros for slots out of range.
+ */
+int pa_latent_append(const void *u, int64_t u_stride, int64_t n_rows, const float *norm_weight, float eps, const float *rope,
+                     int64_t rope_rows, const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
+                     const int32_t *tiles, int n_tiles, int batch, const int64_t *slots, int64_t total_slots, void *q_out,
+                     void *pool, int num_heads, int dim, int rot_dim, int rank, int q_dim, int pool_row, float q_scale,
+                     int dtype, void *stream);
+int pa_latent_gather(const void *pool, const int64_t *slots, int64_t total_slots, void *out, int64_t rows, int pool_row,
+                     int dtype, void *stream);
+
+/*
+ * Paged attention with score terms.  For the row at position i, over the visible keys j <= i (window > 0: i - j < window):
+ *     score_j = softcap tanh(scale q . k_j / softcap) + bias[h][min(i - j, bias_n - 1)]     (softcap 0, bias NULL: without)
+ *     out = sum_j e^score_j v_j / (sum_j e^score_j + e^sink[h])                              (sink NULL: without)
+ * A query is n1 elements of q1 followed by n2 of q2, head h of row r at r * q_row + h * q_head.  k_cache, v_cache: pool
+ * rows [slot][kv head][k_dim], [slot][kv head][v_dim], of which the first n1 + n2 and vdim count; v_cache may point into
+ * k_cache's rows.  out : [n_rows][heads][vdim].  Missing blocks read as zero rows.  16-bit decode steps (q_lens NULL) with
+ * a workspace spread a sequence's keys over the device.
+ */
+size_t pa_scored_workspace_bytes(int batch, int num_q_heads, int num_kv_heads, int key_size, int vdim, int64_t max_keys, int window);
+int pa_scored_attention(const void *q1, int64_t q1_row, int64_t q1_head, int n1, const void *q2, int64_t q2_row,
+                        int64_t q2_head, int n2, const void *k_cache, int k_dim, const void *v_cache, int v_dim, int vdim,
+                        const int32_t *block_tables, int64_t bt_stride, int block_size, int64_t num_blocks,
+                        const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts, int64_t n_rows, int batch,
+                        int max_q_len, int num_q_heads, int num_kv_heads, float scale, int window, float softcap,
+                        const float *bias, int bias_n, const float *sink, void *out, int dtype, void *workspace,
+                        size_t workspace_bytes, void *stream);
+
+/*
+ * Mixture of experts.  pa_moe_choose, per row over the experts and, behind them, `identity` identity experts (which hand on the
+ * row's own input): scores s = sigmoid(logits) or their softmax; choice scores s + correction (NULL: s).  Of `groups`
+ * equal groups of neighbours the `keep` with the largest sums of their group_top (1 or 2) largest choice scores stay; of
+ * their experts the `top` with the largest choice scores are chosen (the lowest number first on ties).  ids int32[rows][top],
+ * -1 for an identity expert; weights float[rows][top + 1], with identity experts [top + 2]: the chosen s (renormalize: over
+ * their sum + 1e-20; 0 in the place of an identity expert), the shared expert's sigmoid(logits[experts]), 1 or 0 as
+ * `shared` says, and the sum of the chosen identity experts' s.  top <= 64, experts + identity <= 1024.  And per expert
+ * (identity ones included) counts int32[] and lists int32[][rows]: its items (row * top + place) in order.  (Scores that
+ * are NaN are not chosen: id -1.)  The workspace is for experts + identity and needs no initial contents.
  * pa_moe_product: for every listed item, out[item] = W_e x[item / items_per_row], or with glu
  * silu(G_e x) * (U_e x) where an expert's weight rows are the n rows of G followed by the n rows of U.
  *   w : [experts][w_rows][w_stride] of dtype, rows zero past k.  The matrix-core kernels want w_stride % 64 == 0,
  *   k % 8 == 0, n % 4 == 0 and 16-byte aligned tensors; anything else runs on the vector units.
  */
 size_t pa_moe_workspace_bytes(int64_t rows, int experts, int top);
-int pa_moe_choose(const float *logits, int64_t logits_stride, int64_t rows, int experts, int top, int groups, int keep,
-                  int shared, int32_t *ids, float *weights, int32_t *counts, int32_t *lists, void *workspace,
-                  size_t workspace_bytes, void *stream);
+int pa_moe_choose(const float *logits, int64_t logits_stride, int64_t rows, int experts, int identity, int top, int groups,
+                  int keep, int shared, int scores, int group_top, int renormalize, const float *correction, int32_t *ids,
+                  float *weights, int32_t *counts, int32_t *lists, void *workspace, size_t workspace_bytes, void *stream);
 int pa_moe_product(const void *x, int64_t x_stride, int items_per_row, const void *w, int64_t w_rows, int w_stride, int k,
                    const int32_t *counts, const int32_t *lists, int64_t rows, int top, int experts, int glu, void *out,
                    int n, int dtype, void *stream);

@@ -24,8 +24,10 @@ PA_ERR_HIP = -4
 PA_F32, PA_BF16, PA_F16, PA_FP8_E4M3 = 0, 1, 2, 3
 PA_NORM_NONE, PA_NORM_LAYER, PA_NORM_RMS = 0, 1, 2
 PA_ACT_SILU, PA_ACT_GELU_TANH, PA_ACT_NONE = 0, 1, 2
-PA_GATE_SIGMOID_LAST, PA_GATE_SILU_FIRST = 0, 1
+PA_GATE_SIGMOID_LAST, PA_GATE_SILU_FIRST, PA_GATE_SILU_LAST = 0, 1, 2
 PA_GL_SSD, PA_GL_MLSTM = 0, 1
+PA_MOE_SIGMOID, PA_MOE_SOFTMAX = 0, 1
+PA_MOE_NO_SHARED, PA_MOE_SHARED_GATED, PA_MOE_SHARED = 0, 1, 2
 PA_V_PLAIN, PA_V_FIRST, PA_V_MIX = 0, 1, 2
 PA_QKV_TILE_ROWS = 16
 
@@ -108,7 +110,16 @@ SIGNATURES.update({
                              _i, _i, _p, _i, _i, _i, _i, _p, c_size_t, _p]),
     "pa_narrow_linear": (_i, [_p, _l, _p, _p, _l, _i, _i, _i, _p]),
     "pa_moe_workspace_bytes": (c_size_t, [_l, _i, _i]),
-    "pa_moe_choose": (_i, [_p, _l, _l, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, c_size_t, _p]),
+    "pa_moe_choose": (_i, [_p, _l, _l, _i, _i, _i, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, c_size_t, _p]),
+    "pa_delta_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i]),
+    "pa_delta": (_i, [_p, _l, _p, _l, _p, _l, _i, _p, _p, _l, _p, _p, _f, _l, _p, _l, _p, _p, _p, _p, _i, _i, _p, _i, _i, _i, _i,
+                      _p, c_size_t, _p]),
+    "pa_hyper_norm": (_i, [_p, _p, _p, _i, _i, _p, _p, _p, _p, _p, _p, _l, _p, _p, _f, _p, _p, _l, _i, _i, _i, _p]),
+    "pa_latent_append": (_i, [_p, _l, _l, _p, _f, _p, _l, _p, _p, _p, _p, _i, _i, _p, _l, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
+    "pa_latent_gather": (_i, [_p, _p, _l, _p, _l, _i, _i, _p]),
+    "pa_scored_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i, _l, _i]),
+    "pa_scored_attention": (_i, [_p, _l, _l, _i, _p, _l, _l, _i, _p, _i, _p, _i, _i, _p, _l, _i, _l, _p, _p, _p, _l, _i, _i, _i, _i,
+                                 _f, _i, _f, _p, _i, _p, _p, _i, _p, c_size_t, _p]),
     "pa_moe_product": (_i, [_p, _l, _i, _p, _l, _i, _i, _p, _p, _l, _i, _i, _i, _p, _i, _i, _p]),
 })
 SIGNATURES["pa_decode_split"] = SIGNATURES["pa_decode_reduce"] = SIGNATURES["pa_decode"]

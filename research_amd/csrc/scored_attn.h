@@ -1,0 +1,55 @@
+// Attention over a paged context whose scores are more than q . k, and whose keys and values may have sizes of their own or
+// be one tensor:
+//     score(i, j) = cap tanh(scale q_i . k_j / cap) + bias[h][min(i - j, bias_n - 1)]       (cap 0: without it)
+//     out_i = sum over visible j of e^score(i, j) v_j / (sum over visible j of e^score(i, j) + e^sink[h])
+// A query row is two pieces side by side (a latent part and a rotated part), or one.
+#pragma once
+#include "row_common.h"
+
+struct ScoredArgs {
+    const void *q1, *q2;  // pieces of n1 and n2 elements, head h of row r at r * q*_row + h * q*_head
+    int64_t q1_row, q1_head, q2_row, q2_head;
+    int n1, n2;
+    const void *k, *v;  // pool rows of a token: [hkv][k_dim], [hkv][v_dim]; v may lie inside k
+    int k_dim, v_dim, vdim;
+    const int32_t *bt;
+    int64_t bt_stride, num_blocks;
+    int bs;
+    const int32_t *ctx_lens, *q_lens, *q_starts;  // (q_lens NULL: one row per sequence)
+    int64_t n_rows;
+    int batch, max_q_len, heads, hkv, n_rep, window;
+    float scale, cap;
+    const float *bias;  // [heads][bias_n], or NULL
+    int bias_n;
+    const float *sink;  // [heads], or NULL
+    void *out;          // [rows][heads][vdim]
+    int splits;         // decode: pieces of a sequence's keys
+    float *part_o, *part_ml;
+};
+
+struct ScoredPortion {
+    int n, pos0;
+    int64_t row0;
+};
+__device__ __forceinline__ bool scored_portion(const ScoredArgs &a, int b, ScoredPortion &p) {
+    p.n = a.q_lens ? a.q_lens[b] : 1;
+    p.row0 = a.q_starts ? a.q_starts[b] : b;
+    p.pos0 = a.ctx_lens[b] - p.n;
+    return p.n > 0 && p.pos0 >= 0 && p.row0 >= 0 && p.row0 + p.n <= a.n_rows;
+}
+__device__ __forceinline__ int scored_first_key(const ScoredArgs &a, int pos) {
+    return a.window > 0 && pos >= a.window ? pos - a.window + 1 : 0;
+}
+// Pool row of a key, -1 when its block is missing
+__device__ __forceinline__ int64_t scored_slot(const ScoredArgs &a, const int32_t *table, int key) {
+    const int blk = key / a.bs;
+    const int64_t id = blk < a.bt_stride ? table[blk] : -1;
+    return id >= 0 && id < a.num_blocks ? id * a.bs + key % a.bs : -1;
+}
+
+constexpr float kScoredLog2e = 1.4426950408889634f;
+constexpr float kScoredNone = -1.0e30f;  // finite stand-in for minus infinity
+
+// false: no matrix-core kernel for these sizes
+bool pa_scored_decode_launch(const ScoredArgs &a, int dtype, hipStream_t s, int &rc);
+bool pa_scored_prefill_launch(const ScoredArgs &a, int dtype, hipStream_t s, int &rc);

@@ -30,14 +30,15 @@ class CacheConfig:
     # Extension: "fp8_e4m3" keeps K/V as one byte per element with one fp32
     # scale per (block, kv head); ``dtype`` then names the q / output type.
     kv_format: Optional[str] = None
-    # Extension: one (kv heads, head size) per layer, None for a layer that keeps no keys; ``num_kv_heads`` and
-    # ``head_dim`` then only describe the layer the caller considers typical.
-    layer_kv: Optional[Tuple[Optional[Tuple[int, int]], ...]] = None
+    # Extension: one (kv heads, head size) per layer, or (kv heads, key size, value size), where value size 0 stands for a
+    # layer without a value pool; None for a layer that keeps no keys.  ``num_kv_heads`` and ``head_dim`` then only
+    # describe the layer the caller considers typical.
+    layer_kv: Optional[Tuple[Optional[Tuple[int, ...]], ...]] = None
     # Extension: sequences that can hold recurrent state at a time (0: the model keeps none).
     num_state_slots: int = 0
 
-    def kv_shape(self, layer_idx: int) -> Optional[Tuple[int, int]]:
-        """(kv heads, head size) of a layer's pool, None when it has none."""
+    def kv_shape(self, layer_idx: int) -> Optional[Tuple[int, ...]]:
+        """(kv heads, head size), or (kv heads, key size, value size), of a layer's pool, None when it has none."""
         return (self.num_kv_heads, self.head_dim) if self.layer_kv is None else self.layer_kv[layer_idx]
 
     @property

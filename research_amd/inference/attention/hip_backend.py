@@ -46,7 +46,7 @@ Differences of ``HipPagedAttentionBackend`` from the reference, all deliberate:
 from __future__ import annotations
 
 from collections import OrderedDict
-from typing import Dict, List, Optional, Sequence, Tuple
+from typing import Dict, List, NamedTuple, Optional, Sequence, Tuple
 
 import numpy as np
 import torch
@@ -91,9 +91,12 @@ class PackedStep:
     """Device integers of a packed batch: the sequences that bring one token each come first (``decodes``), portions
     of several tokens follow (``chunks``); ``rows`` describes both together."""
 
-    __slots__ = ("num_decodes", "num_rows", "slots", "tables", "rows", "decodes", "chunks")
+    __slots__ = ("num_decodes", "num_rows", "slots", "tables", "rows", "decodes", "chunks", "host", "stretches")
 
-    def __init__(self, num_decodes: int, num_rows: int, slots: Optional[Tensor], tables: Tensor, rows: ops.Portions) -> None:
+    def __init__(self, num_decodes: int, num_rows: int, slots: Optional[Tensor], tables: Tensor, rows: ops.Portions,
+                 host: Optional[Tuple[np.ndarray, np.ndarray, np.ndarray]] = None) -> None:
+        self.host = host  # lengths, new rows and block tables of the sequences, on the host (where there are portions)
+        self.stretches: Dict[int, Stretch] = {}
         self.num_decodes, self.num_rows, self.slots, self.tables, self.rows = num_decodes, num_rows, slots, tables, rows
         cut = lambda t, lo, hi: None if t is None else t[lo:hi]
         batch, nd = rows.ctx_lens.numel(), num_decodes
@@ -103,6 +106,38 @@ class PackedStep:
         if batch > nd:
             self.chunks = ops.Portions(rows.ctx_lens[nd:], cut(rows.state_slots, nd, batch), rows.q_lens[nd:],
                                        rows.q_starts[nd:], None, rows.max_q_len)
+
+
+class Stretch(NamedTuple):
+    """The keys that the portions of a step can see, as a pool of their own in blocks of ``STRETCH_BLOCK`` rows: ``slots``
+    (int64, -1: a zero row) says where the rows are in the cache, ``tables`` and ``portions`` address the new pool."""
+
+    slots: Tensor
+    tables: Tensor
+    portions: ops.Portions
+
+
+STRETCH_BLOCK = 16
+
+
+def plan_stretch(lens: np.ndarray, q_lens: np.ndarray, tables: np.ndarray, block_size: int,
+                 window: int) -> Tuple[np.ndarray, np.ndarray, np.ndarray]:
+    """Cache slots of the visible keys of every sequence, each sequence padded to whole blocks with -1; their block tables
+    in the new pool; how many keys each has.  Positions count from the first visible key, which neither causality nor a
+    sliding window notices."""
+    first = np.maximum(lens - q_lens - window + 1, 0) if window else np.zeros_like(lens)
+    count = lens - first
+    blocks = -(-count // STRETCH_BLOCK)
+    slots = np.full(int(blocks.sum()) * STRETCH_BLOCK, -1, dtype=np.int64)
+    out = np.full((len(lens), max(int(blocks.max(initial=0)), 1)), -1, dtype=np.int32)
+    at = 0
+    for i in range(len(lens)):
+        pos = np.arange(first[i], lens[i])
+        ids = tables[i, pos // block_size].astype(np.int64)
+        slots[at * STRETCH_BLOCK: at * STRETCH_BLOCK + len(pos)] = np.where(ids >= 0, ids * block_size + pos % block_size, -1)
+        out[i, : blocks[i]] = np.arange(at, at + blocks[i])
+        at += int(blocks[i])
+    return slots, out, count
 
 
 class HipPagedAttentionBackend:
@@ -139,10 +174,12 @@ class HipPagedAttentionBackend:
         else:  # layers of their own shapes: one tensor per layer that keeps keys
             if self._fp8:
                 raise ValueError("an fp8 pool has one shape for all layers")
-            pool = lambda kv: None if kv is None else torch.zeros((config.total_slots,) + tuple(kv), dtype=pool_dtype,
-                                                                  device=config.device)
-            self.k_cache = [pool(kv) for kv in config.layer_kv]
-            self.v_cache = [pool(kv) for kv in config.layer_kv]
+            def pool(kv, which: int) -> Optional[Tensor]:  # 1: keys, -1: values
+                if kv is None or kv[which] == 0:
+                    return None
+                return torch.zeros((config.total_slots, kv[0], kv[which]), dtype=pool_dtype, device=config.device)
+            self.k_cache = [pool(kv, 1) for kv in config.layer_kv]
+            self.v_cache = [pool(kv, -1) for kv in config.layer_kv]
         self._probe = torch.empty(0, device=config.device)
         self._device = self._probe.device
         self.k_scale = self.v_scale = None
@@ -738,8 +775,50 @@ class HipPagedAttentionBackend:
         slots = None
         if ctx.slot_mapping is not None:
             slots = self._device_slots(ctx.slot_mapping, rows, step)
-        step.packed = PackedStep(nd, rows, slots, step.tables, portions)
+        host = None
+        if nd < batch and isinstance(ctx.block_tables, np.ndarray):
+            host = lens[nd:], q_lens[nd:], ctx.block_tables[nd:]
+        step.packed = PackedStep(nd, rows, slots, step.tables, portions, host)
         return step.packed
+
+    def stretch(self, step: PackedStep, window: int) -> Stretch:
+        """What the step's portions see under a sliding window (0: everything before them); built once per step."""
+        if window not in step.stretches:
+            if step.host is None:
+                raise TypeError("portions with keys made again need host block tables as an array")
+            lens, q_lens, tables = step.host
+            slots, new_tables, count = plan_stretch(lens, q_lens, tables, self.config.block_size, window)
+            dev = self._to_device(np.concatenate([count, new_tables.reshape(-1)]).astype(np.int32))
+            n = len(count)
+            step.stretches[window] = Stretch(self._to_device(slots), dev[n:].view(n, -1), step.chunks._replace(ctx_lens=dev[:n]))
+        return step.stretches[window]
+
+    def attend_stretch(self, q: Tensor, k: Tensor, v: Tensor, stretch: Stretch, scale: float, window: int, out: Tensor) -> Tensor:
+        """Attention of a step's portions over the keys and values ``[rows, Hkv, D]`` of their stretch."""
+        c = stretch.portions
+        need = ops.prefill_workspace_bytes(q, stretch.tables, c.max_q_len, STRETCH_BLOCK, k.shape[1], window)
+        return ops.prefill_paged(q, k, v, stretch.tables, c.ctx_lens, c.q_lens, c.q_starts, c.max_q_len, STRETCH_BLOCK, scale, out=out,
+                                 window=window, workspace=self._workspace_for(need) if need else None)
+
+    def attend_scored(self, q: Tuple[Tensor, ...], layer_idx: int, step: PackedStep, vdim: int, scale: float, window: int,
+                      part: Optional[str] = None, **terms) -> Tensor:
+        """Attention with score terms (``ops.scored_attention``) of packed rows over the pool; a layer without a value pool
+        attends to the leading elements of its keys.  ``part`` ``"decodes"`` or ``"chunks"``: q holds only these rows'
+        sequences' (decodes), or only these are computed (chunks)."""
+        self._require_device(*q)
+        kc, vc = self._layer(layer_idx)
+        vc = kc if vc is None else vc
+        nd = step.num_decodes
+        out = torch.empty((q[0].shape[0], q[0].shape[1], vdim), dtype=q[0].dtype, device=q[0].device)
+        kw = dict(block_size=self.config.block_size, scale=scale, window=window, **terms)
+        if step.decodes is not None and part != "chunks":
+            need = ops.scored_workspace_bytes(nd, q[0].shape[1], kc.shape[1], sum(t.shape[2] for t in q), vdim,
+                                              step.tables.shape[1] * self.config.block_size, window)
+            ops.scored_attention(tuple(t[:nd] for t in q), kc, vc, vdim, step.decodes, step.tables[:nd], out=out[:nd],
+                                 workspace=self._workspace_for(need) if need else None, **kw)
+        if step.chunks is not None and part != "decodes":
+            ops.scored_attention(q, kc, vc, vdim, step.chunks, step.tables[nd:], out=out, **kw)
+        return out
 
     def attend_packed(self, q: Tensor, layer_idx: int, step: PackedStep, scale: float, window: int) -> Tensor:
         """Attention of packed rows ``q [rows, Hq, D]`` over the pool (their own keys appended already): the decode

@@ -13,13 +13,15 @@ Designs on top of it are a function from their ``config.json`` to a
 with biases, unit-RMS q and k behind three-way short convolutions, value mixing,
 per-head output gates, lightning attention, per-layer token inputs.  Tevirax is
 another: RMS norms on the sublayers' outputs, chunk attention beside a matrix
-memory in one layer, Mamba-2 layers, mixtures of experts, capped logits.
+memory in one layer, Mamba-2 layers, mixtures of experts, capped logits.  Vusalix:
+several residual streams with learned mixing, latent attention, attention with
+distance biases and sinks, the gated delta rule, experts beside identity experts.
 """
 
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Dict, Iterable, List, Optional, Tuple, Union
+from typing import Callable, Dict, Iterable, List, Optional, Tuple, Union
 
 import torch
 import torch.nn.functional as F
@@ -27,13 +29,14 @@ from torch import Tensor, nn
 
 from .. import ops
 from .attention import CacheConfig, HipPagedAttentionBackend
-from .mixers import (AttentionSpec, ConvAttention, GatedMLP, LightningMixer, LightningSpec, Mamba2Mixer, Mamba2Spec,
-                     MlstmSpec, ParallelMixer, ParallelSpec, RotaryTables, StepRows, TokenSide, YarnScaling, _param, fill)
+from .mixers import (AttentionSpec, BiasedAttention, BiasedAttentionSpec, ConvAttention, DeltaMixer, DeltaSpec, GatedMLP,
+                     LatentAttention, LatentSpec, LightningMixer, LightningSpec, Mamba2Mixer, Mamba2Spec, MlstmSpec,
+                     ParallelMixer, ParallelSpec, RotaryTables, StepRows, TokenSide, YarnScaling, _param, fill)
 from .moe import MoE, MoESpec
 from .types import InferenceContext
 
 
-MixerSpec = Union[AttentionSpec, LightningSpec, Mamba2Spec, ParallelSpec]
+MixerSpec = Union[AttentionSpec, BiasedAttentionSpec, LatentSpec, LightningSpec, Mamba2Spec, DeltaSpec, ParallelSpec]
 
 
 @dataclass(frozen=True)
@@ -42,10 +45,10 @@ class LayerSpec:
     ff: Union[int, MoESpec, None]  # inner width of a dense feed-forward, experts, None: the layer has none
 
     @property
-    def attention(self) -> Optional[AttentionSpec]:
-        """The part of the layer that keeps keys, if any."""
+    def kv_pool(self) -> Optional[Tuple[int, ...]]:
+        """What the layer keeps per token (an entry of ``CacheConfig.layer_kv``), None for a layer without keys."""
         mixer = self.mixer.left if isinstance(self.mixer, ParallelSpec) else self.mixer
-        return mixer if isinstance(mixer, AttentionSpec) else None
+        return getattr(mixer, "kv_pool", None)
 
 
 @dataclass(frozen=True)
@@ -60,8 +63,15 @@ class HybridConfig:
     embed_scale: float = 1.0
     positions: int = 0  # rows of a learned position table that the embedding adds, 0: none
     logit_softcap: Optional[float] = None
+    streams: int = 0  # residual streams with learned mixing around every sublayer, 0: one plain residual
 
     def __post_init__(self) -> None:
+        if self.streams and (self.norm != "rms" or self.post_norm or self.side_dim or self.positions or self.embed_scale != 1.0):
+            raise ValueError("residual streams are for RMS norms ahead of the sublayers and a plain embedding")
+        if not 0 <= self.streams <= 16:
+            raise ValueError(f"streams={self.streams} not in 1 .. 16")
+        if not self.streams and any(isinstance(l.ff, MoESpec) and l.ff.identity for l in self.layers):
+            raise ValueError("identity experts are for residual streams")
         if self.post_norm and (self.norm != "rms" or self.side_dim):
             raise ValueError("norms behind the sublayers are RMS norms, without a per-layer token input")
         mixed = {(l.mixer.kv_heads, l.mixer.vdim) for l in self.layers if isinstance(l.mixer, AttentionSpec) and l.mixer.v_mix}
@@ -78,8 +88,7 @@ class HybridConfig:
 
     def cache_config(self, num_blocks: int, block_size: int, num_state_slots: int, dtype: torch.dtype,
                      device: str) -> CacheConfig:
-        keys = [l.attention for l in self.layers]
-        shapes = tuple((a.pool_heads, a.pool_dim) if a is not None else None for a in keys)
+        shapes = tuple(l.kv_pool for l in self.layers)
         typical = next((s for s in shapes if s is not None), (1, 8))
         return CacheConfig(num_layers=len(shapes), num_kv_heads=typical[0], head_dim=typical[1], num_blocks=num_blocks,
                            block_size=block_size, dtype=dtype, device=device, layer_kv=shapes,
@@ -90,6 +99,13 @@ def _only(what: str, got: dict, *keys: str) -> None:
     extra = sorted(set(got) - set(keys))
     if extra:
         raise ValueError(f"{what}: unknown fields {extra}")
+
+
+def _yarn(where: str, scaling: Optional[dict]) -> Optional[YarnScaling]:
+    if scaling is None:
+        return None
+    _only(where, scaling, "factor", "original", "fast", "slow")
+    return YarnScaling(**{key: float(scaling[key]) for key in ("factor", "original", "fast", "slow")})
 
 
 def lotozen_config(d: dict) -> HybridConfig:
@@ -167,10 +183,7 @@ def tevirax_config(d: dict) -> HybridConfig:
             rot, mask = left.get("rot") or {}, left.get("mask") or {}
             _only(at + ".left.rot", rot, "base", "dims", "scaling")
             _only(at + ".left.mask", mask, "size")
-            scaling = rot.get("scaling")
-            if scaling is not None:
-                _only(at + ".left.rot.scaling", scaling, "factor", "original", "fast", "slow")
-                scaling = YarnScaling(**{key: float(scaling[key]) for key in ("factor", "original", "fast", "slow")})
+            scaling = _yarn(at + ".left.rot.scaling", rot.get("scaling"))
             mixer = ParallelSpec(
                 left=AttentionSpec(heads=int(left["heads"]), kv_heads=int(left["kv_heads"]), dim=int(left["dim"]), vdim=int(left["vdim"]),
                                    scale=float(left["scale"]), window=None, taps=0, rot_dims=int(rot.get("dims", 0)),
@@ -189,6 +202,64 @@ def tevirax_config(d: dict) -> HybridConfig:
                         logit_softcap=float(cap) if cap else None)
 
 
+def _window(where: str, m: dict) -> Optional[int]:
+    mask = m.get("mask") or {}
+    _only(f"{where}.mask", mask, "size")
+    return int(mask["size"]) if mask.get("size") is not None else None
+
+
+def vusalix_config(d: dict, buckets: Callable[[int], int]) -> HybridConfig:
+    """From the fields of a Vusalix ``config.json``; ``buckets``: how many distance buckets layer i's table has (the length of
+    a checkpoint tensor).  Anything it does not know it refuses."""
+    layers = []
+    for i, layer in enumerate(d["layers"]):
+        m, mlp, at = layer["mixer"], layer.get("mlp"), f"layer {i} mixer"
+        _only(f"layer {i}", layer, "type", "mixer", "mlp")
+        if layer["type"] == "delta":
+            _only(at, m, "heads", "kv_heads", "dim", "vdim", "conv")
+            mixer: MixerSpec = DeltaSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                         taps=int(m["conv"]))
+        elif layer["type"] == "latent_attention":
+            _only(at, m, "heads", "dim", "rot_dim", "vdim", "kv_rank", "rot", "scale", "mask")
+            rot = m.get("rot") or {}
+            _only(at + ".rot", rot, "base", "dims", "scaling")
+            if int(rot.get("dims", m["rot_dim"])) != int(m["rot_dim"]):
+                raise ValueError(f"{at}: rot.dims={rot['dims']} is not rot_dim={m['rot_dim']}")
+            mixer = LatentSpec(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                               kv_rank=int(m["kv_rank"]), scale=float(m["scale"]), window=_window(at, m),
+                               rot_base=float(rot.get("base", 1.0)), rot_yarn=_yarn(at + ".rot.scaling", rot.get("scaling")))
+        elif layer["type"] == "attention":
+            _only(at, m, "heads", "kv_heads", "dim", "vdim", "scale", "softcap", "bias_max", "mask")
+            cap = m.get("softcap")
+            mixer = BiasedAttentionSpec(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]),
+                                        scale=float(m["scale"]), window=_window(at, m), softcap=float(cap) if cap else None,
+                                        buckets=buckets(i), bias_max=int(m["bias_max"]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}")
+        layers.append(LayerSpec(mixer, _vusalix_ff(f"layer {i} mlp", mlp)))
+    _only("norm", d["norm"], "eps")
+    return HybridConfig(vocab_size=int(d["vocab"]), width=int(d["width"]), layers=tuple(layers), norm_eps=float(d["norm"]["eps"]),
+                        norm="rms", streams=int(d["streams"]))
+
+
+def _vusalix_ff(where: str, mlp: Optional[dict]) -> Optional[MoESpec]:
+    if mlp is None:
+        return None
+    if mlp["kind"] != "moe":
+        raise ValueError(f"{where}: unknown feed-forward {mlp['kind']!r}")
+    _only(where, mlp, "kind", "expert", "router", "shared")
+    router, shared = mlp["router"], mlp.get("shared")
+    groups = router.get("groups") or {"count": 1, "keep": 1}
+    _only(f"{where} expert", mlp["expert"], "ff")
+    _only(f"{where} router", router, "experts", "identity", "top", "groups")
+    _only(f"{where} router.groups", groups, "count", "keep")
+    if shared is not None:
+        _only(f"{where} shared", shared, "ff")
+    return MoESpec(experts=int(router["experts"]), ff=int(mlp["expert"]["ff"]), top=int(router["top"]), groups=int(groups["count"]),
+                   keep=int(groups["keep"]), shared=int(shared["ff"]) if shared is not None else None, shared_gate=False,
+                   identity=int(router.get("identity") or 0), scores="softmax", group_top=1, correction=True, renormalize=False)
+
+
 class _Norm(nn.Module):
     """Weights of a norm; the arithmetic is fused into the residual sums.  ``args`` as ``pa_residual_norm`` takes them."""
 
@@ -204,6 +275,22 @@ class _Norm(nn.Module):
             fill(self.b, get(name + ".b"), name + ".b")
 
 
+class _Streams(nn.Module):
+    """Weights of the residual streams around one sublayer; the arithmetic is one kernel (``pa_hyper_norm``)."""
+
+    def __init__(self, streams: int, device) -> None:
+        super().__init__()
+        kw = dict(dtype=torch.float32, device=device)
+        self.weights = _param(streams, **kw)
+        self.between = _param(streams, streams, **kw)
+        self.into = _param(streams, **kw)
+
+    def load(self, get, prefix: str) -> None:
+        fill(self.weights, get(prefix + "in"), prefix + "in")
+        fill(self.between, get(prefix + "mix"), prefix + "mix")
+        fill(self.into, get(prefix + "out"), prefix + "out")
+
+
 class _HybridLayer(nn.Module):
     def __init__(self, cfg: HybridConfig, i: int, backend: HipPagedAttentionBackend, rotary: RotaryTables,
                  v_role: Optional[str], dtype: torch.dtype, device) -> None:
@@ -214,11 +301,20 @@ class _HybridLayer(nn.Module):
             self.mixer = ConvAttention(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, v_role, dtype, device)
         elif isinstance(spec.mixer, ParallelSpec):
             self.mixer = ParallelMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, dtype, device)
+        elif isinstance(spec.mixer, BiasedAttentionSpec):
+            self.mixer = BiasedAttention(spec.mixer, cfg.width, i, backend, dtype, device)
+        elif isinstance(spec.mixer, LatentSpec):
+            self.mixer = LatentAttention(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, dtype, device)
+        elif isinstance(spec.mixer, DeltaSpec):
+            self.mixer = DeltaMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
         elif isinstance(spec.mixer, Mamba2Spec):
             self.mixer = Mamba2Mixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
         else:
             self.mixer = LightningMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
-        self.norm2 = self.mlp = self.side = None
+        self.norm2 = self.mlp = self.side = self.streams1 = self.streams2 = None
+        if cfg.streams:
+            self.streams1 = _Streams(cfg.streams, device)
+            self.streams2 = _Streams(cfg.streams, device) if spec.ff is not None else None
         if spec.ff is not None:
             self.norm2 = _Norm(cfg, device)
             self.mlp = (MoE(spec.ff, cfg.width, dtype, device) if isinstance(spec.ff, MoESpec)
@@ -234,6 +330,9 @@ class _HybridLayer(nn.Module):
             self.mlp.load(get, prefix + "mlp.")
         if self.side is not None:
             self.side.load(get, prefix + "side.")
+        for streams, name in ((self.streams1, "hc1."), (self.streams2, "hc2.")):
+            if streams is not None:
+                streams.load(get, prefix + name)
 
 
 class HybridDecoder(nn.Module):
@@ -296,6 +395,8 @@ class HybridDecoder(nn.Module):
         if packed.num_rows != ids.numel():
             raise ValueError(f"{ids.numel()} tokens for a context of {packed.num_rows} rows")
         step = StepRows(packed, ids)
+        if self.cfg.streams:
+            return self._forward_streams(step, trace).view(*input_ids.shape, self.cfg.width)
         cfg, eps, dtype = self.cfg, self.cfg.norm_eps, self.dtype
         x = torch.empty((ids.numel(), self.cfg.width), dtype=torch.float32, device=ids.device)
         # what the next residual sum adds: nothing but the embedding at first, then the last branch's output
@@ -323,6 +424,23 @@ class HybridDecoder(nn.Module):
         if pending:
             ops.residual_norm(x, dtype, **pending, want_out=False)
         return x.view(*input_ids.shape, self.cfg.width)
+
+    def _forward_streams(self, step: StepRows, trace: Optional[List[Tensor]]) -> Tensor:
+        """The sum of the streams ``[rows, width]`` after the last layer."""
+        cfg, dtype = self.cfg, self.dtype
+        x = torch.empty((step.ids.numel(), cfg.streams, cfg.width), dtype=torch.float32, device=step.ids.device)
+        # what the next pass over the streams takes in: the embedding at first, then the last branch's output
+        pending: dict = {"ids": step.ids, "table": self.embed}
+        for layer in self.layers:
+            for norm, streams, branch in ((layer.norm1, layer.streams1, lambda h: {"y": layer.mixer(h, step)}),
+                                          (layer.norm2, layer.streams2, lambda h: layer.mlp.branch(h))):
+                if norm is None:
+                    continue
+                h = ops.hyper_norm(x, dtype, **pending, sum_weight=streams.weights, weight=norm.w, eps=cfg.norm_eps)
+                pending = {**branch(h), "between": streams.between, "into": streams.into}
+            if trace is not None:
+                trace.append(ops.hyper_norm(x, dtype, **pending, want="sum"))
+        return ops.hyper_norm(x, dtype, **pending, want="sum")
 
     def logits(self, hidden_rows: Tensor) -> Tensor:
         h = ops.residual_norm(hidden_rows.contiguous(), self.dtype, **self.norm.args)

@@ -15,6 +15,13 @@ product and everything between the products into one or two kernels:
   normaliser) -> ``pa_rms_gate`` per head -> output projection;
 * ``Mamba2Mixer``: joint projection -> ``pa_short_conv`` -> ``pa_gated_linear``
   -> ``pa_rms_gate`` (gate first) -> output projection;
+* ``DeltaMixer``: joint projection -> ``pa_short_conv`` -> ``pa_delta`` (unit
+  norms, gates, delta rule) -> ``pa_rms_gate`` per head -> output projection;
+* ``BiasedAttention``: joint projection -> ``pa_qkv_conv_append`` (append) ->
+  ``pa_scored_attention`` (cap, distance biases, sinks) -> output projection;
+* ``LatentAttention``: joint projection -> ``pa_latent_append``; decoded tokens
+  attend to the cached latents themselves (``pa_scored_attention`` between two
+  products per head), portions to keys and values made again from them;
 * ``ParallelMixer``: two of them side by side with one joint input and one joint
   output projection; their scales ride on the steps before the latter.
 """
@@ -23,7 +30,7 @@ from __future__ import annotations
 
 import math
 from dataclasses import dataclass
-from typing import Callable, Dict, Optional, Tuple
+from typing import Callable, Dict, List, Optional, Tuple
 
 import torch
 import torch.nn.functional as F
@@ -121,6 +128,112 @@ class AttentionSpec:
         if self.rot_halves:
             order[: self.rot_dims] = order[: self.rot_dims].view(2, -1).t().reshape(-1)
         return order
+
+
+    @property
+    def kv_pool(self) -> Tuple[int, ...]:
+        """The layer's pool, as an entry of ``CacheConfig.layer_kv``."""
+        return self.pool_heads, self.pool_dim
+
+
+@dataclass(frozen=True)
+class BiasedAttentionSpec:
+    """Softmax attention without rotation: scores under a soft cap, a learned bias per distance bucket and head, a sink per
+    head in the denominator.  ``bias_max``: the distance from which on all share the last bucket."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    window: Optional[int]
+    softcap: Optional[float]
+    buckets: int
+    bias_max: int
+
+    def __post_init__(self) -> None:
+        if self.heads % self.kv_heads != 0:
+            raise ValueError(f"heads={self.heads} is not a multiple of kv_heads={self.kv_heads}")
+        if self.window is not None and self.window < 1:
+            raise ValueError(f"window={self.window} must be positive")
+        if self.buckets < 2 or self.bias_max <= self.buckets // 2:
+            raise ValueError(f"bias_max={self.bias_max} must be above half of buckets={self.buckets}")
+        if max(self.dim, self.vdim) > 256:
+            raise ValueError(f"dim={self.dim} or vdim={self.vdim} above 256")
+
+    @property
+    def kv_pool(self) -> Tuple[int, ...]:
+        return self.kv_heads, _pad8(max(self.dim, self.vdim))
+
+    def bucket_of(self) -> List[int]:
+        """The bucket of every distance 0 .. bias_max: single distances up to half of the buckets, then equal ratios.  Bucket
+        half + k starts where (n / half)^rest reaches (bias_max / half)^k, in whole numbers."""
+        half, most = self.buckets // 2, self.bias_max
+        rest, out = self.buckets - half, list(range(half))
+        k = 0
+        for n in range(half, most + 1):
+            while k + 1 < rest and n ** rest * half ** (k + 1) >= most ** (k + 1) * half ** rest:
+                k += 1
+            out.append(half + k)
+        return out
+
+
+@dataclass(frozen=True)
+class LatentSpec:
+    """Attention whose keys and values per head are linear in one latent of ``kv_rank`` per token; beside them a rotated key
+    part of ``rot_dim`` shared by all heads.  The cache keeps the latent and the rotated part."""
+
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: Optional[int]
+    rot_base: float
+    rot_yarn: Optional[YarnScaling] = None
+
+    def __post_init__(self) -> None:
+        if self.rot_dim % 2:
+            raise ValueError(f"rot_dim={self.rot_dim} must be even")
+        if self.window is not None and self.window < 1:
+            raise ValueError(f"window={self.window} must be positive")
+        if self.kv_rank > 1024 or self.kv_rank + self.rot_dim > 2048:
+            raise ValueError(f"kv_rank={self.kv_rank} above 1024")
+
+    @property
+    def pool_row(self) -> int:
+        return _pad8(self.kv_rank + self.rot_dim)
+
+    @property
+    def kv_pool(self) -> Tuple[int, ...]:
+        return 1, self.pool_row, 0
+
+    @property
+    def head_dim(self) -> int:
+        """Size of a head's key or value made again from the latents."""
+        return _pad8(max(self.dim + self.rot_dim, self.vdim))
+
+
+@dataclass(frozen=True)
+class DeltaSpec:
+    """The gated delta rule behind short convolutions; ``heads`` value heads share ``kv_heads`` q/k heads."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+
+    def __post_init__(self) -> None:
+        if self.heads % self.kv_heads != 0:
+            raise ValueError(f"heads={self.heads} is not a multiple of kv_heads={self.kv_heads}")
+        if self.dim > 256 or not 1 <= self.taps <= 8:
+            raise ValueError(f"dim={self.dim} above 256 or taps={self.taps} not in 1 .. 8")
+
+    @property
+    def channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
 
 
 @dataclass(frozen=True)
@@ -497,6 +610,174 @@ class Mamba2Mixer(Mixer):
         y = _gated_rows("ssd", c, b, x, (dt, None), (self.dt_bias, self.rate, self.skip), step, self.state, s.heads, s.state,
                         s.vdim, self.backend, heads_per_group=s.heads // s.groups)
         return ops.rms_gate(y, z, self.norm, self.eps, groups=s.norm_groups, order="silu_first", out=out)
+
+
+class DeltaMixer(Mixer):
+    def __init__(self, spec: DeltaSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
+                 dtype: torch.dtype, device) -> None:
+        """Rows of ``w_in``: q, k, v, output gate, decay logits, beta logits, padding."""
+        inner = spec.heads * spec.vdim
+        super().__init__(_pad8(spec.channels + inner + 2 * spec.heads), inner, width, dtype, device)
+        self.spec, self.eps, self.backend = spec, eps, backend
+        f32 = dict(dtype=torch.float32, device=device)
+        self.conv = _param(spec.taps, spec.channels, **f32)
+        self.dt_bias, self.rate = (_param(spec.heads, **f32) for _ in range(2))
+        self.norm = _param(inner, **f32)  # one head's weights, for every head
+        self.conv_state = None
+        if spec.taps > 1:
+            self.conv_state = backend.register_state(layer_idx, "conv", (spec.taps - 1, spec.channels), dtype)
+        pad = lambda n: -(-n // 16) * 16
+        self.state = backend.register_state(layer_idx, "delta", (spec.heads, pad(spec.dim), pad(spec.vdim)), torch.float32)
+
+    def _parts(self) -> Tuple[Tuple[str, int], ...]:
+        s = self.spec
+        qk, inner = s.kv_heads * s.dim, s.heads * s.vdim
+        return ("q", qk), ("k", qk), ("v", inner), ("g", inner), ("a", s.heads), ("b", s.heads)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        s, at = self.spec, 0
+        for name, n in self._parts():
+            fill(self.w_in[at: at + n], get(prefix + name), prefix + name)
+            if name in "qkv":
+                fill(self.conv[:, at: at + n], get(f"{prefix}{name}.conv").t(), f"{prefix}{name}.conv")
+            at += n
+        fill(self.dt_bias, get(prefix + "dt_bias"), prefix + "dt_bias")
+        fill(self.rate, get(prefix + "A_log").float().exp(), prefix + "A_log")
+        fill(self.norm, get(prefix + "norm").repeat(s.heads), prefix + "norm")
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s, packed = self.spec, step.packed
+        x, g, a, b = u[:, : s.channels + s.heads * (s.vdim + 2)].split([s.channels, s.heads * s.vdim, s.heads, s.heads], dim=1)
+        x = ops.short_conv(x, packed.rows, self.conv, None, self.conv_state, "silu")
+        q, k, v = x.split([s.kv_heads * s.dim, s.kv_heads * s.dim, s.heads * s.vdim], dim=1)
+        o = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
+        sizes = (self.dt_bias, self.rate)
+        tail = (self.state, s.heads, s.dim, s.vdim, s.dim ** -0.5)
+        kw = dict(heads_per_group=s.heads // s.kv_heads)
+        if packed.decodes is not None:
+            n = packed.num_decodes
+            ops.delta_rule(*(t[:n] for t in (q, k, v, a, b)), *sizes, packed.decodes, *tail, o[:n], **kw)
+        if packed.chunks is not None:
+            c = packed.chunks
+            need = ops.delta_workspace_bytes(c.ctx_lens.numel(), s.heads, s.dim, s.vdim, c.max_q_len) if u.dtype == torch.bfloat16 else 0
+            ops.delta_rule(q, k, v, a, b, *sizes, c, *tail, o, workspace=self.backend._workspace_for(need) if need else None, **kw)
+        return ops.rms_gate(o, g, self.norm, self.eps, groups=s.heads, order="silu_last", out=out)
+
+
+class BiasedAttention(Mixer):
+    def __init__(self, spec: BiasedAttentionSpec, width: int, layer_idx: int, backend: HipPagedAttentionBackend, dtype: torch.dtype,
+                 device) -> None:
+        """Rows of ``w_in``: q, k, v, padding."""
+        super().__init__(_pad8((spec.heads + spec.kv_heads) * spec.dim + spec.kv_heads * spec.vdim), spec.heads * spec.vdim, width,
+                         dtype, device)
+        self.spec, self.layer_idx, self.backend = spec, layer_idx, backend
+        self.buckets = torch.tensor(spec.bucket_of())
+        self.bias = _param(spec.heads, len(self.buckets), dtype=torch.float32, device=device)  # by distance
+        self.sink = _param(spec.heads, dtype=torch.float32, device=device)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        s, at = self.spec, 0
+        for name, n in (("q", s.heads * s.dim), ("k", s.kv_heads * s.dim), ("v", s.kv_heads * s.vdim)):
+            fill(self.w_in[at: at + n], get(prefix + name), prefix + name)
+            at += n
+        rel = get(prefix + "rel")
+        if tuple(rel.shape) != (s.buckets, s.heads):
+            raise ValueError(f"{prefix}rel: checkpoint shape {tuple(rel.shape)}, expected {(s.buckets, s.heads)}")
+        fill(self.bias, rel[self.buckets.to(rel.device)].t(), prefix + "rel")
+        fill(self.sink, get(prefix + "sink"), prefix + "sink")
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s, packed = self.spec, step.packed
+        kc, vc = self.backend._layer(self.layer_idx)
+        q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, 1.0, 0.0, False, None, 0, None, None)
+        o = self.backend.attend_scored((q[..., : s.dim],), self.layer_idx, packed, s.vdim, s.scale, s.window or 0,
+                                       softcap=s.softcap or 0.0, bias=self.bias, sink=self.sink)
+        o = o.view(u.shape[0], -1)
+        return o if out is None else out.copy_(o)
+
+
+class LatentAttention(Mixer):
+    def __init__(self, spec: LatentSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
+                 rotary: RotaryTables, dtype: torch.dtype, device) -> None:
+        """Rows of ``w_in``: q, latent, rotated key part, padding.  The two weights on the latent are kept in two forms: per
+        head, for products before and behind attention over the latents (``w_key`` transposed), and over whole pool rows,
+        for keys and values made again (the rotated part passes through an identity)."""
+        s = spec
+        super().__init__(_pad8(s.heads * (s.dim + s.rot_dim) + s.kv_rank + s.rot_dim), s.heads * s.vdim, width, dtype, device)
+        self.spec, self.eps, self.layer_idx, self.backend, self.rotary = spec, eps, layer_idx, backend, rotary
+        pad = lambda n: -(-n // 64) * 64
+        kw = dict(dtype=dtype, device=device)
+        self.norm = _param(s.kv_rank, dtype=torch.float32, device=device)
+        self.w_key = _param(s.heads, s.kv_rank, pad(s.dim), **kw)
+        self.w_value = _param(s.heads, s.vdim, pad(s.kv_rank), **kw)
+        self.remake = dtype == torch.bfloat16 and s.head_dim <= 256
+        if self.remake:
+            self.k_made = _param(s.heads, s.head_dim, s.pool_row, **kw)
+            self.v_made = _param(s.heads, s.head_dim, s.pool_row, **kw)
+        self._lists: Dict[int, ops.ExpertChoice] = {}
+
+    def load(self, get: Getter, prefix: str) -> None:
+        s = self.spec
+        n = s.heads * (s.dim + s.rot_dim)
+        fill(self.w_in[:n], get(prefix + "q"), prefix + "q")
+        fill(self.w_in[n: n + s.kv_rank + s.rot_dim], get(prefix + "dkv"), prefix + "dkv")
+        fill(self.norm, get(prefix + "dkv.norm"), prefix + "dkv.norm")
+        key, value = (get(prefix + name).view(s.heads, -1, s.kv_rank) for name in ("uk", "uv"))
+        fill(self.w_key[:, :, : s.dim], key.transpose(1, 2), prefix + "uk")
+        fill(self.w_value[:, :, : s.kv_rank], value, prefix + "uv")
+        if self.remake:
+            fill(self.k_made[:, : s.dim, : s.kv_rank], key, prefix + "uk")
+            self.k_made[:, s.dim: s.dim + s.rot_dim, s.kv_rank: s.kv_rank + s.rot_dim] = torch.eye(s.rot_dim).to(self.k_made)
+            fill(self.v_made[:, : s.vdim, : s.kv_rank], value, prefix + "uv")
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def _per_head(self, rows: int, device, keep: bool) -> ops.ExpertChoice:
+        """Products per head as products per expert: every row uses every head.  (``keep``: a captured graph may hold them.)"""
+        if rows in self._lists:
+            return self._lists[rows]
+        h = self.spec.heads
+        lists = (torch.arange(rows, dtype=torch.int32, device=device)[None] * h +
+                 torch.arange(h, dtype=torch.int32, device=device)[:, None]).contiguous()
+        choice = ops.ExpertChoice(lists.view(rows, h), torch.empty(0, device=device),
+                                  torch.full((h,), rows, dtype=torch.int32, device=device), lists)
+        if keep:
+            self._lists[rows] = choice
+        return choice
+
+    def _over_latents(self, q: Tensor, packed: PackedStep, part: str) -> Tensor:
+        s, rows = self.spec, q.shape[0]
+        choice = self._per_head(rows, q.device, part == "decodes")
+        over = ops.moe_product(q.view(rows * s.heads, -1)[:, : s.dim], choice, self.w_key, s.kv_rank, s.dim, glu=False)
+        o = self.backend.attend_scored((over.view(rows, s.heads, s.kv_rank), q[..., s.dim: s.dim + s.rot_dim]), self.layer_idx, packed,
+                                       s.kv_rank, _LN2, s.window or 0, part=part)
+        return ops.moe_product(o.view(rows * s.heads, s.kv_rank), choice, self.w_value, s.vdim, s.kv_rank, glu=False).view(rows, -1)
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s, packed = self.spec, step.packed
+        pool, _ = self.backend._layer(self.layer_idx)
+        # (q carries scale * log2(e) from its 32-bit registers)
+        q = ops.latent_append(u, packed.rows, packed.slots, pool, self.norm, self.eps, self.rotary.get(s.rot_base, s.rot_dim, 1.0, s.rot_yarn),
+                              s.heads, s.dim, s.rot_dim, s.kv_rank, s.head_dim, s.scale / _LN2)
+        nd = packed.num_decodes
+        if packed.chunks is None:
+            o = self._over_latents(q, packed, "decodes")
+            return o if out is None else out.copy_(o)
+        if self.remake:
+            stretch = self.backend.stretch(packed, s.window or 0)
+            rows = ops.latent_gather(pool, stretch.slots)
+            k, v = (F.linear(rows, w.view(-1, s.pool_row)).view(-1, s.heads, s.head_dim) for w in (self.k_made, self.v_made))
+            o = self.backend.attend_stretch(q, k, v, stretch, _LN2, s.window or 0, torch.empty_like(q))
+            if out is None:
+                out = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
+            ops.head_gate(o[nd:], None, s.vdim, out=out[nd:])
+        else:
+            o = self._over_latents(q, packed, "chunks")
+            out = o if out is None else out.copy_(o)
+        if nd:
+            out[:nd] = self._over_latents(q[:nd], packed, "decodes")
+        return out
 
 
 class ParallelMixer(Mixer):

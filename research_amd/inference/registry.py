@@ -17,7 +17,7 @@ import torch
 from torch import Tensor, nn
 
 from .attention import CacheConfig, HipPagedAttentionBackend
-from .hybrid import HybridConfig, HybridDecoder, lotozen_config, tevirax_config
+from .hybrid import HybridConfig, HybridDecoder, lotozen_config, tevirax_config, vusalix_config
 from .model import ModelConfig, PagedLlama
 
 DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
@@ -91,14 +91,22 @@ def model_len(path: str, wanted: int) -> int:
 # ------------------------------------------------------------------ entries
 
 
-def _hybrid(reader: Callable[[dict], HybridConfig]) -> Callable[[str, dict, LoadOptions], nn.Module]:
+Weights = Dict[str, Tensor]
+
+
+def _hybrid(reader: Callable[[dict, Weights], HybridConfig]) -> Callable[[str, dict, LoadOptions], nn.Module]:
     def build(path: str, config: dict, o: LoadOptions) -> nn.Module:
-        cfg = reader(config)
+        weights = read_weights(path)
+        cfg = reader(config, weights)
         backend = HipPagedAttentionBackend(cfg.cache_config(o.num_blocks, o.block_size, o.num_state_slots, o.dtype, o.device))
         model = HybridDecoder(cfg, backend, o.max_positions, o.dtype)
-        model.load_state_dict(read_weights(path), strict=False)
+        model.load_state_dict(weights, strict=False)
         return model.eval()
     return build
+
+
+def _vusalix(config: dict, weights: Weights) -> HybridConfig:
+    return vusalix_config(config, lambda i: weights[f"l{i}.mix.rel"].shape[0])
 
 
 def _build_llama(path: str, config: dict, o: LoadOptions) -> nn.Module:
@@ -109,8 +117,9 @@ def _build_llama(path: str, config: dict, o: LoadOptions) -> nn.Module:
     return PagedLlama.from_local(path, backend_for, dtype=o.dtype, device=o.device)
 
 
-register(ModelEntry("lotozen", lambda c: c.get("architecture") == "Lotozen", _hybrid(lotozen_config)))
-register(ModelEntry("tevirax", lambda c: c.get("architecture") == "Tevirax", _hybrid(tevirax_config),
+register(ModelEntry("lotozen", lambda c: c.get("architecture") == "Lotozen", _hybrid(lambda c, w: lotozen_config(c))))
+register(ModelEntry("tevirax", lambda c: c.get("architecture") == "Tevirax", _hybrid(lambda c, w: tevirax_config(c)),
                     lambda c: int(c["max_positions"])))
+register(ModelEntry("vusalix", lambda c: c.get("architecture") == "Vusalix", _hybrid(_vusalix)))
 register(ModelEntry("llama", lambda c: "num_attention_heads" in c, _build_llama,
                     lambda c: c.get("max_position_embeddings")))

@@ -353,7 +353,10 @@ def _typed(dtype: torch.dtype, *tensors: Optional[Tensor]) -> None:
 
 _NORMS = {None: _lib.PA_NORM_NONE, "layer": _lib.PA_NORM_LAYER, "rms": _lib.PA_NORM_RMS}
 _ACTS = {"silu": _lib.PA_ACT_SILU, "gelu_tanh": _lib.PA_ACT_GELU_TANH, None: _lib.PA_ACT_NONE}
-_GATES = {"sigmoid_last": _lib.PA_GATE_SIGMOID_LAST, "silu_first": _lib.PA_GATE_SILU_FIRST}
+_GATES = {"sigmoid_last": _lib.PA_GATE_SIGMOID_LAST, "silu_first": _lib.PA_GATE_SILU_FIRST,
+          "silu_last": _lib.PA_GATE_SILU_LAST}
+_SCORES = {"sigmoid": _lib.PA_MOE_SIGMOID, "softmax": _lib.PA_MOE_SOFTMAX}
+_SHARED = {None: _lib.PA_MOE_NO_SHARED, "gated": _lib.PA_MOE_SHARED_GATED, "plain": _lib.PA_MOE_SHARED}
 _GATED = {"ssd": _lib.PA_GL_SSD, "mlstm": _lib.PA_GL_MLSTM}
 _V_MODES = {None: _lib.PA_V_PLAIN, "first": _lib.PA_V_FIRST, "mix": _lib.PA_V_MIX}
 
@@ -399,7 +402,7 @@ def residual_norm(x: Tensor, dtype: torch.dtype, y: Optional[Tensor] = None, y_w
 def rms_gate(o: Tensor, gate: Tensor, weight: Tensor, eps: float, groups: int = 1, order: str = "sigmoid_last",
              out: Optional[Tensor] = None) -> Tensor:
     """The gated RMS norm of every one of ``groups`` equal parts of a row (``pa_rms_gate``): ``"sigmoid_last"``:
-    ``o / rms(o) * weight * sigmoid(gate)``; ``"silu_first"``: ``z / rms(z) * weight`` of ``z = o * silu(gate)``.
+    ``o / rms(o) * weight * sigmoid(gate)``; ``"silu_last"`` likewise with the silu; ``"silu_first"``: ``z / rms(z) * weight`` of ``z = o * silu(gate)``.
     ``gate`` and ``out`` may be column slices."""
     rows, width = o.shape
     _dense(o, weight)
@@ -625,7 +628,8 @@ def narrow_linear(x: Tensor, w: Tensor) -> Tensor:
 
 class ExpertChoice(NamedTuple):
     """Which experts every row uses: ``ids`` int32 ``[rows, top]``, ``weights`` float32 ``[rows, top + 1]`` (the last one the
-    shared expert's) and, per expert, how many and which items (row * top + place)."""
+    shared expert's; with identity experts one more, the sum of theirs) and, per expert, how many and which items (row * top
+    + place)."""
 
     ids: Tensor
     weights: Tensor
@@ -633,23 +637,26 @@ class ExpertChoice(NamedTuple):
     lists: Tensor
 
 
-def moe_choose(logits: Tensor, experts: int, top: int, groups: int, keep: int) -> ExpertChoice:
-    """``pa_moe_choose`` over float32 ``logits`` ``[rows, experts]``, or one column more for the gate of a
-    shared expert."""
-    rows = logits.shape[0]
-    _dense(logits)
-    _typed(torch.float32, logits)
-    if logits.shape[1] not in (experts, experts + 1):
-        raise ValueError("logits must hold one column per expert, and one for a shared expert")
+def moe_choose(logits: Tensor, experts: int, top: int, groups: int, keep: int, shared: Optional[str] = None, identity: int = 0,
+               scores: str = "sigmoid", group_top: int = 2, renormalize: bool = True,
+               correction: Optional[Tensor] = None) -> ExpertChoice:
+    """``pa_moe_choose`` over float32 ``logits`` ``[rows, experts + identity]``; ``shared`` ``"gated"`` (one column more, its
+    gate), ``"plain"`` or None."""
+    rows, every = logits.shape[0], experts + identity
+    _dense(logits, correction)
+    _typed(torch.float32, logits, correction)
+    if logits.shape[1] != every + (shared == "gated") or (correction is not None and correction.numel() != every):
+        raise ValueError("logits must hold one column per expert, and one for a gated shared expert; correction likewise")
     dev = logits.device
     ids = torch.empty((rows, top), dtype=torch.int32, device=dev)
-    weights = torch.empty((rows, top + 1), dtype=torch.float32, device=dev)
-    counts = torch.empty(experts, dtype=torch.int32, device=dev)
-    lists = torch.empty((experts, rows), dtype=torch.int32, device=dev)
-    workspace = torch.empty(int(_lib.load().pa_moe_workspace_bytes(rows, experts, top)), dtype=torch.uint8, device=dev)
-    _run("pa_moe_choose", _ptr(logits), logits.shape[1], rows, experts, top, groups, keep, int(logits.shape[1] > experts),
-         _ptr(ids), _ptr(weights), _ptr(counts), _ptr(lists), _ptr(workspace), workspace.numel(), _stream(logits))
-    return ExpertChoice(ids, weights, counts, lists)
+    weights = torch.empty((rows, top + (2 if identity else 1)), dtype=torch.float32, device=dev)
+    counts = torch.empty(every, dtype=torch.int32, device=dev)
+    lists = torch.empty((every, rows), dtype=torch.int32, device=dev)
+    workspace = torch.empty(int(_lib.load().pa_moe_workspace_bytes(rows, every, top)), dtype=torch.uint8, device=dev)
+    _run("pa_moe_choose", _ptr(logits), logits.shape[1], rows, experts, identity, top, groups, keep, _SHARED[shared], _SCORES[scores],
+         group_top, int(renormalize), _ptr(correction), _ptr(ids), _ptr(weights), _ptr(counts), _ptr(lists), _ptr(workspace),
+         workspace.numel(), _stream(logits))
+    return ExpertChoice(ids, weights, counts[:experts], lists[:experts])
 
 
 def moe_product(x: Tensor, choice: ExpertChoice, w: Tensor, n: int, k: int, glu: bool) -> Tensor:
@@ -665,4 +672,134 @@ def moe_product(x: Tensor, choice: ExpertChoice, w: Tensor, n: int, k: int, glu:
     out = torch.empty((rows * top, n), dtype=x.dtype, device=x.device)
     _run("pa_moe_product", _ptr(x), _row_stride(x), rows * top // x.shape[0] if x.shape[0] else 1, _ptr(w), w.shape[1], w.shape[2], k,
          _ptr(choice.counts), _ptr(choice.lists), rows, top, w.shape[0], int(glu), _ptr(out), n, PA_DTYPE[x.dtype], _stream(x))
+    return out
+
+
+def delta_workspace_bytes(batch: int, heads: int, dim: int, vdim: int, max_q_len: int) -> int:
+    return int(_lib.load().pa_delta_workspace_bytes(batch, heads, dim, vdim, max_q_len))
+
+
+def delta_rule(q: Tensor, k: Tensor, v: Tensor, decay_logits: Tensor, beta_logits: Tensor, decay_bias: Tensor, decay_rate: Tensor,
+               portions: Portions, state: Tensor, heads: int, dim: int, vdim: int, q_scale: float, out: Tensor,
+               heads_per_group: int = 1, workspace: Optional[Tensor] = None) -> Tensor:
+    """The gated delta rule (``pa_delta``).  q, k, v and the logits ``[rows, heads]`` may be column slices; ``state`` float32
+    ``[slots, heads, pad16(dim), pad16(vdim)]``."""
+    rows, batch = v.shape[0], portions.ctx_lens.numel()
+    pad = lambda n: -(-n // 16) * 16
+    _dense(state, out, decay_bias, decay_rate, *portions[:4])
+    _typed(torch.int32, *portions[:4])
+    _typed(torch.float32, state, decay_bias, decay_rate)
+    _typed(v.dtype, q, k, decay_logits, beta_logits, out)
+    qk = (rows, heads // heads_per_group * dim)
+    if tuple(q.shape) != qk or tuple(k.shape) != qk or tuple(v.shape) != (rows, heads * vdim) or out.shape != v.shape:
+        raise ValueError("q / k / v / out do not fit each other")
+    if any(tuple(g.shape) != (rows, heads) for g in (decay_logits, beta_logits)) or _row_stride(decay_logits) != _row_stride(beta_logits):
+        raise ValueError("the two logits do not fit the heads, or differ in their rows")
+    if decay_bias.numel() != heads or decay_rate.numel() != heads or tuple(state.shape[1:]) != (heads, pad(dim), pad(vdim)):
+        raise ValueError("constants or state of another size")
+    _run("pa_delta", _ptr(q), _row_stride(q), _ptr(k), _row_stride(k), _ptr(v), _row_stride(v), heads_per_group, _ptr(decay_logits),
+         _ptr(beta_logits), _row_stride(decay_logits), _ptr(decay_bias), _ptr(decay_rate), float(q_scale), rows, _ptr(state),
+         state.shape[0], _ptr(portions.ctx_lens), _ptr(portions.q_lens), _ptr(portions.q_starts), _ptr(portions.state_slots), batch,
+         portions.max_q_len, _ptr(out), heads, dim, vdim, PA_DTYPE[v.dtype], _ptr(workspace),
+         workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(v))
+    return out
+
+
+def hyper_norm(x: Tensor, dtype: torch.dtype, y: Optional[Tensor] = None, between: Optional[Tensor] = None,
+               into: Optional[Tensor] = None, mix: Optional[Tensor] = None, y_extra: Optional[Tensor] = None,
+               y_self: Optional[Tensor] = None, ids: Optional[Tensor] = None, table: Optional[Tensor] = None,
+               sum_weight: Optional[Tensor] = None, weight: Optional[Tensor] = None, eps: float = 0.0, want: str = "out") -> Tensor:
+    """One step of residual streams ``x`` float32 ``[rows, streams, width]`` (``pa_hyper_norm``): they start as
+    ``table[ids]``, or are mixed by ``between`` and take ``y`` by ``into``.  ``want`` ``"out"``: updates x and returns the
+    RMS norm of their weighted sum in ``dtype``; ``"sum"``: returns the float32 sum and leaves x.  ``mix`` float32
+    ``[rows, m + 1]`` or, with ``y_self``, ``[rows, m + 2]``: y is a weighted sum of ``y`` ``[rows * m, width]``, ``y_extra``
+    and ``y_self``."""
+    rows, streams, width = x.shape
+    _dense(x, y, between, into, mix, y_extra, y_self, ids, table, sum_weight, weight)
+    _typed(torch.float32, x, between, into, mix, sum_weight, weight)
+    _typed(torch.int64, ids)
+    _typed(dtype, y, y_extra, y_self, table)
+    m = mix.shape[1] - (1 if y_self is None else 2) if mix is not None else 0
+    if y is not None and tuple(y.shape) != (rows * (m or 1), width):
+        raise ValueError("y does not fit the streams")
+    if (mix is not None and mix.shape[0] != rows) or any(t is not None and tuple(t.shape) != (rows, width) for t in (y_extra, y_self)):
+        raise ValueError("mix / y_extra / y_self do not fit the streams")
+    if ids is not None and (ids.numel() != rows or table.shape[1] != width):
+        raise ValueError("ids / table do not fit the streams")
+    if (between is not None and tuple(between.shape) != (streams, streams)) or \
+            any(t is not None and t.numel() != streams for t in (into, sum_weight)) or (weight is not None and weight.numel() != width):
+        raise ValueError("weights do not fit the streams")
+    if want == "out":
+        out, sum_ = torch.empty((rows, width), dtype=dtype, device=x.device), None
+    else:
+        out, sum_ = None, torch.empty((rows, width), dtype=torch.float32, device=x.device)
+    _run("pa_hyper_norm", _ptr(x), _ptr(y), _ptr(mix), m, mix.shape[1] if mix is not None else 0, _ptr(y_extra), _ptr(y_self),
+         _ptr(between), _ptr(into), _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, _ptr(sum_weight), _ptr(weight),
+         float(eps), _ptr(out), _ptr(sum_), rows, streams, width, PA_DTYPE[dtype], _stream(x))
+    return out if sum_ is None else sum_
+
+
+def latent_append(u: Tensor, portions: Portions, slots: Tensor, pool: Tensor, norm: Tensor, eps: float, rope: Optional[Tensor],
+                  heads: int, dim: int, rot_dim: int, rank: int, q_dim: int, q_scale: float) -> Tensor:
+    """Projection rows to rotated queries ``[rows, heads, q_dim]`` and the appended pool rows ``[slots, 1, row]``
+    (``pa_latent_append``)."""
+    rows, batch = u.shape[0], portions.ctx_lens.numel()
+    total_slots, one, pool_row = pool.shape
+    _dense(slots, pool, norm, rope, *portions[:5])
+    _typed(torch.int32, *portions[:5])
+    _typed(torch.float32, norm, rope)
+    _typed(u.dtype, pool)
+    _typed(torch.int64, slots)
+    if one != 1 or slots.numel() != rows or norm.numel() != rank or u.shape[1] < heads * (dim + rot_dim) + rank + rot_dim:
+        raise ValueError("slots / pool / norm / u do not fit")
+    if rot_dim and tuple(rope.shape[1:]) != (rot_dim // 2, 2):
+        raise ValueError("rope must be [positions, rot_dim / 2, 2]")
+    q = torch.empty((rows, heads, q_dim), dtype=u.dtype, device=u.device)
+    n_tiles = batch if portions.tiles is None else portions.tiles.shape[0]
+    _run("pa_latent_append", _ptr(u), _row_stride(u), rows, _ptr(norm), float(eps), _ptr(rope), rope.shape[0] if rope is not None else 0,
+         _ptr(portions.ctx_lens), _ptr(portions.q_lens), _ptr(portions.q_starts), _ptr(portions.tiles), n_tiles, batch, _ptr(slots),
+         total_slots, _ptr(q), _ptr(pool), heads, dim, rot_dim, rank, q_dim, pool_row, float(q_scale), PA_DTYPE[u.dtype], _stream(u))
+    return q
+
+
+def latent_gather(pool: Tensor, slots: Tensor) -> Tensor:
+    """Rows ``[n, row]`` of a latent pool, zeros for slots out of range (``pa_latent_gather``)."""
+    _dense(pool, slots)
+    _typed(torch.int64, slots)
+    total_slots, _, row = pool.shape
+    out = torch.empty((slots.numel(), row), dtype=pool.dtype, device=pool.device)
+    _run("pa_latent_gather", _ptr(pool), _ptr(slots), total_slots, _ptr(out), slots.numel(), row, PA_DTYPE[pool.dtype], _stream(pool))
+    return out
+
+
+def scored_workspace_bytes(batch: int, heads: int, kv_heads: int, key_size: int, vdim: int, max_keys: int, window: int) -> int:
+    return int(_lib.load().pa_scored_workspace_bytes(batch, heads, kv_heads, key_size, vdim, max_keys, window))
+
+
+def scored_attention(q: Tuple[Tensor, ...], k_cache: Tensor, v_cache: Tensor, vdim: int, portions: Portions, block_tables: Tensor,
+                     block_size: int, scale: float, window: int, out: Tensor, softcap: float = 0.0, bias: Optional[Tensor] = None,
+                     sink: Optional[Tensor] = None, workspace: Optional[Tensor] = None) -> Tensor:
+    """Paged attention with score terms (``pa_scored_attention``): ``q`` one or two pieces ``[rows, heads, n]`` whose last
+    dimension is contiguous, ``bias`` float32 ``[heads, distances]``, ``sink`` float32 ``[heads]``; ``out`` ``[rows, heads,
+    vdim]``.  ``v_cache`` may be ``k_cache``: the values are its first ``vdim`` elements."""
+    rows, heads = q[0].shape[:2]
+    total_slots, kv_heads, k_dim = k_cache.shape
+    _dense(k_cache, v_cache, block_tables, bias, sink, out, *portions[:4])
+    _typed(torch.int32, block_tables, *portions[:4])
+    _typed(torch.float32, bias, sink)
+    _typed(out.dtype, k_cache, v_cache, *q)
+    if any(tuple(t.shape[:2]) != (rows, heads) or t.stride(2) != 1 for t in q) or not 1 <= len(q) <= 2:
+        raise ValueError("q pieces do not fit each other")
+    if tuple(v_cache.shape[:2]) != (total_slots, kv_heads) or tuple(out.shape) != (rows, heads, vdim):
+        raise ValueError("v_cache / out do not fit")
+    if (bias is not None and bias.shape[0] != heads) or (sink is not None and sink.numel() != heads):
+        raise ValueError("bias / sink must have a row per head")
+    piece = lambda t: (_ptr(t), t.stride(0), t.stride(1), t.shape[2])
+    second = piece(q[1]) if len(q) == 2 else (None, 0, 0, 0)
+    batch = portions.ctx_lens.numel()
+    _run("pa_scored_attention", *piece(q[0]), *second, _ptr(k_cache), k_dim, _ptr(v_cache), v_cache.shape[2], vdim, _ptr(block_tables),
+         block_tables.shape[1], block_size, total_slots // block_size, _ptr(portions.ctx_lens), _ptr(portions.q_lens),
+         _ptr(portions.q_starts), rows, batch, portions.max_q_len, heads, kv_heads, float(scale), int(window), float(softcap), _ptr(bias),
+         bias.shape[1] if bias is not None else 0, _ptr(sink), _ptr(out), PA_DTYPE[out.dtype], _ptr(workspace),
+         workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(out))
     return out
