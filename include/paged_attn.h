@@ -613,7 +613,8 @@ int pa_latent_gather(const void *pool, const int64_t *slots, int64_t total_slots
  * k_cache's rows.  out : [n_rows][heads][vdim].  Missing blocks read as zero rows.  16-bit decode steps (q_lens NULL) with
  * a workspace spread a sequence's keys over the device.
  */
-size_t pa_scored_workspace_bytes(int batch, int num_q_heads, int num_kv_heads, int key_size, int vdim, int64_t max_keys, int window);
+size_t pa_scored_workspace_bytes(int batch, int num_q_heads, int num_kv_heads, int key_size, int vdim, int one_tensor,
+                                 int64_t max_keys, int window);
 int pa_scored_attention(const void *q1, int64_t q1_row, int64_t q1_head, int n1, const void *q2, int64_t q2_row,
                         int64_t q2_head, int n2, const void *k_cache, int k_dim, const void *v_cache, int v_dim, int vdim,
                         const int32_t *block_tables, int64_t bt_stride, int block_size, int64_t num_blocks,

@@ -30,6 +30,7 @@ PA_MOE_SIGMOID, PA_MOE_SOFTMAX = 0, 1
 PA_MOE_NO_SHARED, PA_MOE_SHARED_GATED, PA_MOE_SHARED = 0, 1, 2
 PA_V_PLAIN, PA_V_FIRST, PA_V_MIX = 0, 1, 2
 PA_QKV_TILE_ROWS = 16
+PA_DECODE_TICKET_BYTES = 640 << 10
 
 # name -> (restype, argtypes); mirrors include/paged_attn.h declaration by declaration
 SIGNATURES = {
@@ -117,7 +118,7 @@ SIGNATURES.update({
     "pa_hyper_norm": (_i, [_p, _p, _p, _i, _i, _p, _p, _p, _p, _p, _p, _l, _p, _p, _f, _p, _p, _l, _i, _i, _i, _p]),
     "pa_latent_append": (_i, [_p, _l, _l, _p, _f, _p, _l, _p, _p, _p, _p, _i, _i, _p, _l, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
     "pa_latent_gather": (_i, [_p, _p, _l, _p, _l, _i, _i, _p]),
-    "pa_scored_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i, _l, _i]),
+    "pa_scored_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i, _i, _l, _i]),
     "pa_scored_attention": (_i, [_p, _l, _l, _i, _p, _l, _l, _i, _p, _i, _p, _i, _i, _p, _l, _i, _l, _p, _p, _p, _l, _i, _i, _i, _i,
                                  _f, _i, _f, _p, _i, _p, _p, _i, _p, c_size_t, _p]),
     "pa_moe_product": (_i, [_p, _l, _i, _p, _l, _i, _i, _p, _p, _l, _i, _i, _i, _p, _i, _i, _p]),

@@ -50,6 +50,20 @@ __device__ __forceinline__ int64_t scored_slot(const ScoredArgs &a, const int32_
 constexpr float kScoredLog2e = 1.4426950408889634f;
 constexpr float kScoredNone = -1.0e30f;  // finite stand-in for minus infinity
 
+// Value columns that the decode kernel for these sizes holds, 0: there is none.
+inline int scored_value_cols(int keys, int vdim, bool one) {
+    if (one) return keys <= 160 && vdim <= 128 ? 128 : keys <= 320 && vdim <= 256 ? 256 : keys <= 576 && vdim <= 512 ? 512 : 0;
+    const int most = keys > vdim ? keys : vdim;
+    return most <= 64 ? 64 : most <= 128 ? 128 : most <= 256 ? 256 : 0;
+}
+
+// Pieces that a decode step's sequences are cut into: enough for two workgroups per compute unit, of at least 256 keys each.
+inline int scored_splits(int64_t workgroups, int cus, int64_t span) {
+    int64_t n = (2 * (int64_t)cus + workgroups - 1) / workgroups;
+    if (n > span / 256) n = span / 256;
+    return n < 1 ? 1 : n > 16 ? 16 : (int)n;
+}
+
 // false: no matrix-core kernel for these sizes
 bool pa_scored_decode_launch(const ScoredArgs &a, int dtype, hipStream_t s, int &rc);
 bool pa_scored_prefill_launch(const ScoredArgs &a, int dtype, hipStream_t s, int &rc);

@@ -69,10 +69,32 @@ template <typename T> void launch_vector(const ScoredArgs &a, hipStream_t s) {
     else scored_vector_kernel<T, 16><<<grid, block, lds, s>>>(a);
 }
 
+int scored_cus() {
+    static int cached[64];
+    int dev = 0;
+    if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 64) return 256;
+    int n = __atomic_load_n(&cached[dev], __ATOMIC_RELAXED);
+    if (n == 0) {
+        if (hipDeviceGetAttribute(&n, hipDeviceAttributeMultiprocessorCount, dev) != hipSuccess || n <= 0) n = 256;
+        __atomic_store_n(&cached[dev], n, __ATOMIC_RELAXED);
+    }
+    return n;
+}
+
+int plan_splits(int batch, int heads, int hkv, bool one, int64_t max_keys, int window) {
+    const int rep = heads / hkv, tile = one && rep > 32 ? 64 : one && rep > 16 ? 32 : 16;
+    const int64_t workgroups = (int64_t)batch * hkv * ((rep + tile - 1) / tile);
+    return scored_splits(workgroups, scored_cus(), window > 0 && window < max_keys ? window : max_keys);
+}
+
 }  // namespace
 
-extern "C" size_t pa_scored_workspace_bytes(int batch, int num_q_heads, int num_kv_heads, int key_size, int vdim, int64_t max_keys, int window) {
-    return 0;
+extern "C" size_t pa_scored_workspace_bytes(int batch, int num_q_heads, int num_kv_heads, int key_size, int vdim, int one_tensor,
+                                            int64_t max_keys, int window) {
+    if (batch <= 0 || num_kv_heads <= 0 || num_q_heads <= 0) return 0;
+    const int splits = plan_splits(batch, num_q_heads, num_kv_heads, one_tensor != 0, max_keys, window);
+    const int vc = scored_value_cols(key_size, vdim, one_tensor != 0);
+    return splits > 1 && vc ? (size_t)batch * num_q_heads * splits * (vc + 2) * sizeof(float) : 0;
 }
 
 extern "C" int pa_scored_attention(const void *q1, int64_t q1_row, int64_t q1_head, int n1, const void *q2, int64_t q2_row,
@@ -108,6 +130,18 @@ extern "C" int pa_scored_attention(const void *q1, int64_t q1_row, int64_t q1_he
     a.window = window; a.scale = scale; a.cap = softcap; a.bias = bias; a.bias_n = bias_n; a.sink = sink; a.out = out;
     a.splits = 1;
     hipStream_t s = (hipStream_t)stream;
+    const bool one = k_cache == v_cache;
+    if (!q_lens && workspace) {
+        const int vc = scored_value_cols(n1 + n2, vdim, one);
+        a.splits = plan_splits(batch, num_q_heads, num_kv_heads, one, bt_stride * block_size, window);
+        const size_t per = (size_t)batch * num_q_heads * (vc + 2) * sizeof(float);
+        while (a.splits > 1 && per * a.splits > workspace_bytes) --a.splits;
+        a.part_o = (float *)workspace;
+        a.part_ml = a.part_o + (size_t)batch * num_q_heads * a.splits * vc;
+        PA_REQUIRE(a.splits == 1 || pa_aligned16(workspace), "the workspace must be 16-byte aligned");
+    }
+    int rc = PA_OK;
+    if (pa_scored_decode_launch(a, dtype, s, rc) || pa_scored_prefill_launch(a, dtype, s, rc)) return rc;
     if (dtype == PA_F32) launch_vector<float>(a, s);
     else launch_vector<pa_bf16>(a, s);
     PA_CHECK_LAUNCH("pa_scored_attention");

@@ -450,6 +450,10 @@ class HipPagedAttentionBackend:
                                           device=self._device)
         return self._workspace
 
+    def _scratch_for(self, nbytes: int) -> Tensor:
+        """Workspace of calls that keep nothing in it: behind the decode kernels' arrival counters."""
+        return self._workspace_for(nbytes + _lib.PA_DECODE_TICKET_BYTES)[_lib.PA_DECODE_TICKET_BYTES:]
+
     def _layer(self, layer_idx: int) -> Tuple[Tensor, Tensor]:
         return self.k_cache[layer_idx], self.v_cache[layer_idx]
 
@@ -727,7 +731,7 @@ class HipPagedAttentionBackend:
         need = ops.prefill_workspace_bytes(q3, tables, step.max_q_len, cfg.block_size, cfg.num_kv_heads, window)
         ops.prefill_paged(q3, kc, vc, tables, step.ctx_lens, step.q_lens, step.q_starts, step.max_q_len,
                           cfg.block_size, self.scale, out=out.view(batch * seq_len, num_heads, head_dim), window=window,
-                          row_first_key=first, workspace=self._workspace_for(need) if need else None)
+                          row_first_key=first, workspace=self._scratch_for(need) if need else None)
         return out
 
     # ------------------------------------------------------------------ packed batches
@@ -798,7 +802,7 @@ class HipPagedAttentionBackend:
         c = stretch.portions
         need = ops.prefill_workspace_bytes(q, stretch.tables, c.max_q_len, STRETCH_BLOCK, k.shape[1], window)
         return ops.prefill_paged(q, k, v, stretch.tables, c.ctx_lens, c.q_lens, c.q_starts, c.max_q_len, STRETCH_BLOCK, scale, out=out,
-                                 window=window, workspace=self._workspace_for(need) if need else None)
+                                 window=window, workspace=self._scratch_for(need) if need else None)
 
     def attend_scored(self, q: Tuple[Tensor, ...], layer_idx: int, step: PackedStep, vdim: int, scale: float, window: int,
                       part: Optional[str] = None, **terms) -> Tensor:
@@ -813,9 +817,9 @@ class HipPagedAttentionBackend:
         kw = dict(block_size=self.config.block_size, scale=scale, window=window, **terms)
         if step.decodes is not None and part != "chunks":
             need = ops.scored_workspace_bytes(nd, q[0].shape[1], kc.shape[1], sum(t.shape[2] for t in q), vdim,
-                                              step.tables.shape[1] * self.config.block_size, window)
+                                              vc is kc, step.tables.shape[1] * self.config.block_size, window)
             ops.scored_attention(tuple(t[:nd] for t in q), kc, vc, vdim, step.decodes, step.tables[:nd], out=out[:nd],
-                                 workspace=self._workspace_for(need) if need else None, **kw)
+                                 workspace=self._scratch_for(need) if need else None, **kw)
         if step.chunks is not None and part != "decodes":
             ops.scored_attention(q, kc, vc, vdim, step.chunks, step.tables[nd:], out=out, **kw)
         return out
@@ -840,7 +844,7 @@ class HipPagedAttentionBackend:
             tables = step.tables[nd:]
             need = ops.prefill_workspace_bytes(q, tables, c.max_q_len, cfg.block_size, kc.shape[1], window)
             ops.prefill_paged(q, kc, vc, tables, c.ctx_lens, c.q_lens, c.q_starts, c.max_q_len, cfg.block_size, scale,
-                              out=out, window=window, workspace=self._workspace_for(need) if need else None)
+                              out=out, window=window, workspace=self._scratch_for(need) if need else None)
         return out
 
     # ------------------------------------------------------------------ fp8 pool

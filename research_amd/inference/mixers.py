@@ -507,7 +507,7 @@ class LightningMixer(Mixer):
             c = packed.chunks
             need = ops.lightning_workspace_bytes(c.ctx_lens.numel(), s.heads, s.dim, s.vdim, c.max_q_len)
             ops.lightning(u, c, self.state, self.decay_powers, s.heads, s.dim, s.vdim, o,
-                          workspace=self.backend._workspace_for(need) if need else None)
+                          workspace=self.backend._scratch_for(need) if need else None)
         g = 2 * s.heads * s.dim + inner
         return ops.rms_gate(o, u[:, g: g + inner], self.norm, self.eps, out=out)
 
@@ -525,7 +525,7 @@ def _gated_rows(kind: str, q: Tensor, k: Tensor, v: Tensor, gates, constants, st
         c = packed.chunks
         need = ops.gated_linear_workspace_bytes(c.ctx_lens.numel(), heads, dim, vdim, c.max_q_len)
         ops.gated_linear(kind, q, k, v, gates, constants, c, state, heads, dim, vdim, out,
-                         workspace=backend._workspace_for(need) if need else None, **kw)
+                         workspace=backend._scratch_for(need) if need else None, **kw)
     return out
 
 
@@ -661,7 +661,7 @@ class DeltaMixer(Mixer):
         if packed.chunks is not None:
             c = packed.chunks
             need = ops.delta_workspace_bytes(c.ctx_lens.numel(), s.heads, s.dim, s.vdim, c.max_q_len) if u.dtype == torch.bfloat16 else 0
-            ops.delta_rule(q, k, v, a, b, *sizes, c, *tail, o, workspace=self.backend._workspace_for(need) if need else None, **kw)
+            ops.delta_rule(q, k, v, a, b, *sizes, c, *tail, o, workspace=self.backend._scratch_for(need) if need else None, **kw)
         return ops.rms_gate(o, g, self.norm, self.eps, groups=s.heads, order="silu_last", out=out)
 
 
@@ -692,7 +692,8 @@ class BiasedAttention(Mixer):
         s, packed = self.spec, step.packed
         kc, vc = self.backend._layer(self.layer_idx)
         q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, 1.0, 0.0, False, None, 0, None, None)
-        o = self.backend.attend_scored((q[..., : s.dim],), self.layer_idx, packed, s.vdim, s.scale, s.window or 0,
+        # (q and the pool hold zeros between dim and its next multiple of 8)
+        o = self.backend.attend_scored((q[..., : _pad8(s.dim)],), self.layer_idx, packed, s.vdim, s.scale, s.window or 0,
                                        softcap=s.softcap or 0.0, bias=self.bias, sink=self.sink)
         o = o.view(u.shape[0], -1)
         return o if out is None else out.copy_(o)

@@ -772,8 +772,10 @@ def latent_gather(pool: Tensor, slots: Tensor) -> Tensor:
     return out
 
 
-def scored_workspace_bytes(batch: int, heads: int, kv_heads: int, key_size: int, vdim: int, max_keys: int, window: int) -> int:
-    return int(_lib.load().pa_scored_workspace_bytes(batch, heads, kv_heads, key_size, vdim, max_keys, window))
+def scored_workspace_bytes(batch: int, heads: int, kv_heads: int, key_size: int, vdim: int, one_tensor: bool, max_keys: int,
+                           window: int) -> int:
+    """Bytes with which a decode step spreads its sequences' keys over the device; ``one_tensor``: values are part of the keys."""
+    return int(_lib.load().pa_scored_workspace_bytes(batch, heads, kv_heads, key_size, vdim, int(one_tensor), max_keys, window))
 
 
 def scored_attention(q: Tuple[Tensor, ...], k_cache: Tensor, v_cache: Tensor, vdim: int, portions: Portions, block_tables: Tensor,
