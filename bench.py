@@ -1027,8 +1027,8 @@ def tevirax_kernels(p, dev, steps):
             2.0 * n * width * (e + 1))
         add(phase, "like: bf16 product of equal size", lambda: F.linear(h, router), "", (n * width + e * width) * 2.0 + n * (e + 1) * 2.0, 2.0 * n * width * (e + 1))
         logits = ops.narrow_linear(h, router)
-        choice = ops.moe_choose(logits, e, top, p["groups"], p["keep"])
-        add(phase, "choice of experts and lists", lambda: ops.moe_choose(logits, e, top, p["groups"], p["keep"]), "silu(gate) * up",
+        choice = ops.moe_choose(logits, e, top, p["groups"], p["keep"], "gated" if logits.shape[1] > e else None)
+        add(phase, "choice of experts and lists", lambda: ops.moe_choose(logits, e, top, p["groups"], p["keep"], "gated" if logits.shape[1] > e else None), "silu(gate) * up",
             n * (e + 1) * 4.0 + n * top * 20.0)
         w_in, w_out = rnd(e, 2 * inner, width), rnd(e, width, inner)
         act, items = rnd(n * top, inner), n * top

@@ -315,16 +315,17 @@ def test_recurrence_and_expert_entry_points_check_their_arguments():
 
     rc, msg = _status("pa_narrow_linear", FAKE, 30, FAKE, FAKE, 4, 8, 32, f32, None)
     assert rc == -1 and "x_stride" in msg
-    for args, status, text in (((9, 2, 2, 1), -1, "equal groups"), ((8, 5, 2, 1), -1, "cannot be chosen"), ((8, 2, 2, 3), -1, "cannot be chosen"),
-                               ((2048, 2, 1, 1), -2, "above")):
-        rc, msg = _status("pa_moe_choose", FAKE, 4096, 4, *args, 0, FAKE, FAKE, FAKE, FAKE, FAKE, 1 << 20, None)
-        assert rc == status and text in msg, (args, msg)
-    rc, msg = _status("pa_moe_choose", FAKE, 8, 4, 8, 2, 1, 1, 1, FAKE, FAKE, FAKE, FAKE, FAKE, 1 << 20, None)
-    assert rc == -1 and "logits_stride" in msg
-    rc, msg = _status("pa_moe_choose", FAKE, 8, 4, 8, 2, 1, 1, 0, FAKE, FAKE, None, FAKE, FAKE, 1 << 20, None)
-    assert rc == -1 and "NULL" in msg
-    rc, msg = _status("pa_moe_choose", FAKE, 8, 4, 8, 2, 1, 1, 0, FAKE, FAKE, FAKE, FAKE, FAKE, 8, None)
-    assert rc == -3 and "needed" in msg
+    names = ("logits", "ld", "rows", "e", "ident", "top", "groups", "keep", "shared", "scores", "gtop", "renorm", "corr", "ids", "w", "c", "l", "ws",
+             "wb", "s")
+    choose = lambda **kw: [{**dict(logits=FAKE, ld=4096, rows=4, e=8, ident=0, top=2, groups=1, keep=1, shared=0, scores=0, gtop=2, renorm=1,
+                                   corr=None, ids=FAKE, w=FAKE, c=FAKE, l=FAKE, ws=FAKE, wb=1 << 20, s=None), **kw}[k] for k in names]
+    for kw, status, text in ((dict(e=9, groups=2), -1, "equal groups"), (dict(e=8, ident=1, groups=2), -1, "equal groups"),
+                             (dict(top=5, groups=2), -1, "cannot be chosen"), (dict(groups=2, keep=3), -1, "cannot be chosen"),
+                             (dict(e=2048), -2, "above"), (dict(e=1024, ident=2), -2, "above"), (dict(scores=2), -1, "scores"),
+                             (dict(gtop=3), -1, "group_top"), (dict(shared=3), -1, "shared"), (dict(ld=8, shared=1), -1, "logits_stride"),
+                             (dict(ld=9, ident=2), -1, "logits_stride"), (dict(c=None), -1, "NULL"), (dict(wb=8), -3, "needed")):
+        rc, msg = _status("pa_moe_choose", *choose(**kw))
+        assert rc == status and text in msg, (kw, msg)
     assert lib.pa_moe_workspace_bytes(16384, 64, 8) == 256 * 64 * 4
     product = lambda **kw: [{**dict(x=FAKE, lx=64, ipr=2, w=FAKE, wr=96, lw=64, k=64, c=FAKE, l=FAKE, rows=4, top=2, e=8, glu=1, out=FAKE, n=48,
                                     dt=bf16, s=None), **kw}[k] for k in ("x", "lx", "ipr", "w", "wr", "lw", "k", "c", "l", "rows", "top", "e",
@@ -333,3 +334,45 @@ def test_recurrence_and_expert_entry_points_check_their_arguments():
                              (dict(ipr=0), -1, "out of range")):
         rc, msg = _status("pa_moe_product", *product(**kw))
         assert rc == status and text in msg, (kw, msg)
+
+
+def test_argument_checks_of_the_latent_scored_delta_and_stream_kernels():
+    lib = _lib.load()
+    def cases(name, names, good, bad):
+        for kw, status, text in bad:
+            rc, msg = _status(name, *[{**good, **kw}[k] for k in names])
+            assert rc == status and text in msg, (name, kw, msg)
+
+    bf16 = _lib.PA_BF16
+    cases("pa_hyper_norm", ("x", "y", "mw", "mix", "ml", "ye", "ys", "bt", "into", "ids", "tab", "tr", "sw", "nw", "eps", "out", "sum", "rows",
+                            "n", "width", "dt", "s"),
+          dict(x=FAKE, y=FAKE, mw=None, mix=0, ml=0, ye=None, ys=None, bt=FAKE, into=FAKE, ids=None, tab=None, tr=0, sw=None, nw=FAKE, eps=1e-5,
+               out=FAKE, sum=None, rows=2, n=3, width=64, dt=bf16, s=None),
+          [(dict(n=17), -2, "streams"), (dict(width=20000), -2, "width"), (dict(n=0), -1, "out of range"), (dict(x=None), -1, "NULL"),
+           (dict(bt=None), -1, "without its weights"), (dict(ids=FAKE), -1, "ids"), (dict(mw=FAKE, mix=2, ml=2, ye=FAKE), -1, "does not fit"),
+           (dict(ye=FAKE), -1, "without mix_weight"), (dict(nw=None), -1, "norm_weight"), (dict(y=None, out=None), -1, "nothing"),
+           (dict(dt=_lib.PA_F16), -2, "dtype")])
+    cases("pa_latent_append", ("u", "lu", "n", "nw", "eps", "rope", "rr", "cl", "ql", "qs", "t", "nt", "batch", "slots", "ts", "q", "pool", "h",
+                               "dim", "rot", "rank", "qd", "row", "sc", "dt", "s"),
+          dict(u=FAKE, lu=200, n=2, nw=FAKE, eps=1e-5, rope=FAKE, rr=8, cl=FAKE, ql=None, qs=None, t=None, nt=2, batch=2, slots=FAKE, ts=32,
+               q=FAKE, pool=FAKE, h=4, dim=24, rot=8, rank=40, qd=32, row=48, sc=1.0, dt=bf16, s=None),
+          [(dict(rot=7), -1, "out of range"), (dict(qd=24), -1, "multiples of 8"), (dict(row=50), -1, "multiples of 8"), (dict(lu=100), -1, "u_stride"),
+           (dict(nt=3), -1, "one row"), (dict(t=FAKE), -1, "tiles"), (dict(rope=None), -1, "table"), (dict(dt=_lib.PA_F16), -2, "dtype"),
+           (dict(pool=None), -1, "NULL")])
+    cases("pa_scored_attention", ("q1", "r1", "h1", "n1", "q2", "r2", "h2", "n2", "k", "kd", "v", "vd", "vdim", "bt", "bs_", "bs", "nb", "cl", "ql",
+                                  "qs", "n", "batch", "mq", "hq", "hkv", "sc", "win", "cap", "bias", "bn", "sink", "out", "dt", "ws", "wb", "s"),
+          dict(q1=FAKE, r1=128, h1=32, n1=32, q2=None, r2=0, h2=0, n2=0, k=FAKE, kd=32, v=FAKE, vd=32, vdim=24, bt=FAKE, bs_=4, bs=16, nb=8,
+               cl=FAKE, ql=None, qs=None, n=2, batch=2, mq=1, hq=4, hkv=2, sc=1.0, win=0, cap=0.0, bias=None, bn=0, sink=None, out=FAKE, dt=bf16,
+               ws=None, wb=0, s=None),
+          [(dict(n1=40), -1, "fit the pool"), (dict(vdim=40), -1, "fit the pool"), (dict(hq=3), -1, "multiple"), (dict(win=-1), -1, "window"),
+           (dict(bias=FAKE), -1, "bias_n"), (dict(ql=FAKE), -1, "together"), (dict(n2=8, kd=48), -1, "NULL"), (dict(batch=3), -1, "below batch"),
+           (dict(vdim=1032, vd=1032), -2, "above 1024"), (dict(dt=_lib.PA_F16), -2, "dtype")])
+    cases("pa_delta", ("q", "lq", "k", "lk", "v", "lv", "hpg", "ga", "gb", "lg", "bias", "rate", "sc", "n", "st", "sr", "cl", "ql", "qs", "ss", "batch",
+                       "mq", "out", "h", "dim", "vdim", "dt", "ws", "wb", "s"),
+          dict(q=FAKE, lq=64, k=FAKE, lk=64, v=FAKE, lv=96, hpg=1, ga=FAKE, gb=FAKE, lg=4, bias=FAKE, rate=FAKE, sc=0.25, n=4, st=FAKE, sr=2,
+               cl=FAKE, ql=FAKE, qs=FAKE, ss=FAKE, batch=2, mq=2, out=FAKE, h=4, dim=16, vdim=24, dt=bf16, ws=None, wb=0, s=None),
+          [(dict(hpg=3), -1, "heads_per_group"), (dict(dim=264, lq=2000, lk=2000), -2, "above 256"), (dict(lv=90), -1, "stride"),
+           (dict(lg=3), -1, "stride"), (dict(gb=None), -1, "NULL"), (dict(ql=None), -1, "together"), (dict(ql=None, qs=None, batch=5), -1, "below batch"),
+           (dict(dt=_lib.PA_F16), -2, "dtype")])
+    assert lib.pa_scored_workspace_bytes(0, 4, 2, 32, 32, 0, 100, 0) == 0
+    assert lib.pa_delta_workspace_bytes(2, 3, 64, 64, 65) == 2 * 3 * 2 * (4 * 64 * 64 * 2 + 1024)

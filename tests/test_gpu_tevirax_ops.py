@@ -437,7 +437,7 @@ def test_narrow_products_are_32_bit(rows, n, k, dtype):
 def test_choice_of_experts(rows, experts, top, groups, keep, shared):
     announce(f"choose {rows} {experts} {top} {groups} {keep}")
     logits = _rand(rows, experts + shared, seed=rows)
-    c = ops.moe_choose(logits.to(DEV), experts, top, groups, keep)
+    c = ops.moe_choose(logits.to(DEV), experts, top, groups, keep, "gated" if shared else None)
     ids, weights, counts, lists = (t.cpu() for t in c)
     for r in range(min(rows, 60)):
         want, ww = to.route(torch.sigmoid(logits[r, :experts].double()), top, groups, keep)
