@@ -1,5 +1,6 @@
 """Small random hybrid models for the tests: a ``config.json`` dictionary, weights under their checkpoint names, a
-checkpoint folder of both, and the oracle of the design (Lotozen here, Tevirax in tevirax_helpers.py)."""
+checkpoint folder of both, and the oracle of the design (Lotozen here, Tevirax in tevirax_helpers.py, Vusalix in
+vusalix_helpers.py)."""
 
 import json
 import os
@@ -7,8 +8,8 @@ import os
 import numpy as np
 import torch
 
-from oracle import hybrid_oracle, tevirax_oracle
-from tests import tevirax_helpers as tv
+from oracle import hybrid_oracle, tevirax_oracle, vusalix_oracle
+from tests import tevirax_helpers as tv, vusalix_helpers as vx
 
 
 def attention(heads, kv_heads, dim, vdim, window, conv, rot_dims, base=1000.0, factor=1.0, scale=None, v_mix=True, ff=40):
@@ -46,11 +47,12 @@ CONFIGS = {
 
 
 CONFIGS.update(tv.CONFIGS)
+CONFIGS.update(vx.CONFIGS)
 
 
 def forward(w, cfg, tokens, **kw):
     """The oracle's logits of a whole sequence."""
-    oracle = tevirax_oracle if cfg["architecture"] == "Tevirax" else hybrid_oracle
+    oracle = {"Lotozen": hybrid_oracle, "Tevirax": tevirax_oracle, "Vusalix": vusalix_oracle}[cfg["architecture"]]
     return oracle.decoder_forward(w, cfg, tokens, **kw)
 
 
@@ -58,6 +60,8 @@ def weights(cfg, seed=0):
     """bfloat16 tensors (as stored in a checkpoint) scaled so that every mechanism moves the logits."""
     if cfg["architecture"] == "Tevirax":
         return tv.weights(cfg, seed)
+    if cfg["architecture"] == "Vusalix":
+        return vx.weights(cfg, seed)
     g = torch.Generator().manual_seed(seed)
     w = {}
 
