@@ -10,7 +10,7 @@ head_dim 256 and 64; dense prefill of 64 x 512 and 4 x 8192 tokens; one chunk
 behind 200 000 cached keys at head_dim 128 and 256) under ``secondary``.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--no-secondary]
-                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen|tevirax]
+                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen|tevirax|vusalix]
     python bench.py --traffic-from-pmc NAME KERNEL FETCH.csv WRITE.csv   # refresh profiles/traffic.json
 """
 
@@ -102,7 +102,7 @@ def parse_args():
     ap.add_argument("--warmup", type=int, default=10)
     ap.add_argument("--workload", default="c4", choices=["c1", "c2", "c3", "c3-d256", "c3-d64", "c3-d96", "long-d128", "long-d256", "dense-64x512",
                                                          "dense-4x8192", "c4", "c5", "engine", "lotozen",
-                                                         "tevirax"])
+                                                         "tevirax", "vusalix"])
     ap.add_argument("--preheat-s", type=float, default=0.5,
                     help="seconds of untimed steps before the warmup steps: an idle GPU sits at its lowest clocks "
                          "and takes a few hundred milliseconds of work to leave them")
@@ -1170,6 +1170,235 @@ def bench_tevirax(args, dev) -> int:
     return 0
 
 
+# width; streams; attention query heads, kv heads (of 128 x 128), distance buckets, last distance; latent heads (128 + 64 rotated, values of
+# 128), rank; window of both; delta value heads, q/k heads (of 128); experts, identity experts, chosen, groups, kept, inner
+# width, shared inner width
+VUSALIX_SHAPES = {
+    "w2048": dict(width=2048, streams=4, heads=16, kv_heads=4, buckets=32, bias_max=128, l_heads=16, rank=512, window=1024, d_heads=16, d_groups=8,
+                  experts=64, identity=8, top=6, groups=8, keep=4, ff=768, shared=1024),
+    "w4096": dict(width=4096, streams=4, heads=32, kv_heads=8, buckets=32, bias_max=128, l_heads=32, rank=512, window=1024, d_heads=32, d_groups=16,
+                  experts=64, identity=8, top=8, groups=8, keep=4, ff=1408, shared=2816),
+}
+
+
+def vusalix_model(p, dev, num_blocks, slots, max_positions):
+    """Two delta layers, a latent-attention layer and a biased-attention layer in turn, experts in every layer; random weights."""
+    from research_amd.inference import HipPagedAttentionBackend, HybridConfig, HybridDecoder
+    from research_amd.inference.hybrid import LayerSpec, _Streams
+    from research_amd.inference.mixers import BiasedAttention, BiasedAttentionSpec, DeltaMixer, DeltaSpec, LatentAttention, LatentSpec, YarnScaling
+    from research_amd.inference.moe import MoE, MoESpec
+
+    delta = DeltaSpec(p["d_heads"], p["d_groups"], 128, 128, 4)
+    latent = LatentSpec(p["l_heads"], 128, 64, 128, p["rank"], 192 ** -0.5, p["window"], 10000.0, YarnScaling(4.0, 8192, 32.0, 1.0))
+    att = BiasedAttentionSpec(p["heads"], p["kv_heads"], 128, 128, 128 ** -0.5, p["window"], 30.0, p["buckets"], p["bias_max"])
+    moe = MoESpec(p["experts"], p["ff"], p["top"], p["groups"], p["keep"], p["shared"], shared_gate=False, identity=p["identity"], scores="softmax",
+                  group_top=1, correction=True, renormalize=False)
+    cfg = HybridConfig(vocab_size=HYBRID_VOCAB, width=p["width"], norm_eps=1e-6, norm="rms", streams=p["streams"],
+                       layers=tuple(LayerSpec((delta, delta, latent, att)[i % 4], moe) for i in range(HYBRID_LAYERS)))
+    backend = HipPagedAttentionBackend(cfg.cache_config(num_blocks, 16, slots, torch.bfloat16, "cuda"))
+    model = HybridDecoder(cfg, backend, max_positions)
+    with torch.no_grad():
+        for q in model.parameters():
+            q.normal_(0.0, q.shape[-1] ** -0.5)
+        for m in model.modules():
+            if isinstance(m, DeltaMixer):
+                m.rate.uniform_(1.0, 16.0)
+                m.dt_bias.fill_(-4.0)
+            if isinstance(m, LatentAttention):  # (the rotated part passes through)
+                m.k_made[:, 128:].zero_()
+                m.k_made[:, 128:, p["rank"]:] = torch.eye(64)
+            if isinstance(m, _Streams):
+                m.between.copy_(torch.eye(p["streams"]))
+            if isinstance(m, MoE):
+                m.correction.normal_(0.0, 0.01)
+    return model.eval()
+
+
+def vusalix_kernels(p, dev, steps):
+    """Every kernel of the design's blocks at the layer's shapes, against its roofline, with the like kernel of the Tevirax
+    block.  Bytes and FLOPs are the algorithmic ones (heads unpadded)."""
+    import torch.nn.functional as F
+    from research_amd import ops
+
+    bf, f32 = torch.bfloat16, torch.float32
+    rnd = lambda *s, dtype=bf: torch.randn(*s, device=dev, dtype=torch.float32).to(dtype)
+    i32 = lambda a: torch.as_tensor(np.ascontiguousarray(a), dtype=torch.int32).to(dev)
+    rows_out, add = kernel_table(steps)
+    width, streams, window, d = p["width"], p["streams"], p["window"], 128
+    for phase, (batch, length) in (("prefill", HYBRID_PREFILL), ("decode", HYBRID_DECODE)):
+        dec = phase == "decode"
+        n = batch if dec else batch * length
+        per = length // 16 + (1 if dec else 0)
+        tables = np.random.default_rng(5).permutation(batch * per).reshape(batch, per).astype(np.int32)
+        ctx = np.full(batch, length + 1 if dec else length)
+        pos = np.full((batch, 1), length) if dec else np.tile(np.arange(length), (batch, 1))
+        slots = torch.from_numpy((np.take_along_axis(tables, pos // 16, 1).astype(np.int64) * 16 + pos % 16).reshape(-1)).to(dev)
+        bt, lens, sslots = i32(tables), i32(ctx), i32(np.arange(batch))
+        if dec:
+            por = ops.Portions(lens, sslots)
+        else:
+            first = np.arange(0, length, ops.QKV_TILE_ROWS)
+            tiles = np.stack([np.repeat(np.arange(batch), len(first)), np.tile(first, batch)], 1)
+            por = ops.Portions(lens, sslots, i32(ctx), i32(np.arange(batch) * length), i32(tiles), length)
+        seen = np.minimum(np.full(batch, length + 1) if dec else np.tile(np.arange(1, length + 1), batch), window).astype(float).sum()
+        # streams
+        x, y, w = rnd(n, streams, width, dtype=f32), rnd(n, width), rnd(width, dtype=f32)
+        hc = dict(between=torch.eye(streams, device=dev), into=rnd(streams, dtype=f32), sum_weight=rnd(streams, dtype=f32), weight=w, eps=1e-6)
+        add(phase, "streams mixed, summed, normed", lambda: ops.hyper_norm(x, bf, y=y, **hc), "residual + RMS-normed branch", n * width * (8.0 * streams + 4))
+        x1 = rnd(n, width, dtype=f32)
+        add(phase, "like: residual + RMS-normed branch", lambda: ops.residual_norm(x1, bf, y=y, y_weight=w, y_eps=1e-6), "", n * width * 12.0)
+        # experts
+        e, top, ident = p["experts"], p["top"], p["identity"]
+        h, router, corr = rnd(n, width), rnd(e + ident, width), rnd(e + ident, dtype=f32)
+        router *= width ** -0.5
+        corr *= 0.01
+        logits = ops.narrow_linear(h, router)
+        add(phase, "router logits", lambda: ops.narrow_linear(h, router), "router logits (65 columns)", (n * width + (e + ident) * width) * 2.0 + n * (e + ident) * 4.0)
+        r65 = router[: e + 1].contiguous()
+        add(phase, "like: router logits (65 columns)", lambda: ops.narrow_linear(h, r65), "", (n * width + (e + 1) * width) * 2.0 + n * (e + 1) * 4.0)
+        pick = lambda: ops.moe_choose(logits, e, top, p["groups"], p["keep"], "plain", ident, "softmax", 1, False, corr)
+        add(phase, "choice of experts and lists", pick, "choice by sigmoid scores", n * (e + ident) * 4.0 + n * top * 20.0)
+        l65 = logits[:, : e + 1].contiguous()
+        add(phase, "like: choice by sigmoid scores", lambda: ops.moe_choose(l65, e, top, p["groups"], p["keep"], "gated"), "", n * (e + 1) * 4.0 + n * top * 20.0)
+        choice = pick()
+        eo, shared = rnd(n * top, width), rnd(n, width)
+        add(phase, "streams + sum over experts", lambda: ops.hyper_norm(x, bf, y=eo, mix=choice.weights, y_extra=shared, y_self=h, **hc),
+            "residual + RMS-normed sum over experts", n * width * (8.0 * streams + 2) + (float((choice.weights[:, :top] != 0).sum()) + 2 * n) * width * 2.0)
+        mix65 = choice.weights[:, : top + 1].contiguous()
+        add(phase, "like: residual + RMS-normed sum over experts", lambda: ops.residual_norm(x1, bf, y=eo, mix=mix65, y_extra=shared, y_weight=w, y_eps=1e-6), "",
+            n * width * (10.0 + 2.0 * (top + 1)))
+        del eo, shared, x, x1, y
+        # attention with distance biases
+        heads, kv = p["heads"], p["kv_heads"]
+        u = rnd(n, (heads + 2 * kv) * d)
+        kc, vc = rnd(batch * per * 16, kv, d), rnd(batch * per * 16, kv, d)
+        rope = rnd(length + 1, d // 2, 2, dtype=f32)
+        app = lambda rp, rot, norm: ops.qkv_conv_append(u, por, slots, kc, vc, heads, d, d, 1.0, 1e-6, False, rp, rot, None, None, q_norm=norm, k_norm=norm)
+        qn = rnd(d, dtype=f32)
+        add(phase, "append", lambda: app(None, 0, None), "q/k norm + rotation + append", n * 4.0 * d * (heads + 2 * kv))
+        add(phase, "like: q/k norm + rotation + append", lambda: app(rope, d, qn), "", n * 4.0 * d * (heads + 2 * kv))
+        q, o = app(None, 0, None), torch.empty(n, heads, d, dtype=bf, device=dev)
+        bias, sink = rnd(heads, p["bias_max"] + 1, dtype=f32), rnd(heads, dtype=f32)
+        terms = dict(softcap=30.0, bias=bias, sink=sink)
+        need = ops.scored_workspace_bytes(batch, heads, kv, d, d, False, per * 16, window) if dec else 0
+        ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+        scored = lambda **kw: ops.scored_attention((q,), kc, vc, d, por, bt, 16, d ** -0.5, window, o, workspace=ws, **kw)
+        if dec:
+            add(phase, "decode attention, cap, biases, sinks", lambda: scored(**terms), "decode attention, window", 4.0 * kv * d * seen)
+            dws = ops.decode_workspace(q, kc)
+            add(phase, "like: decode attention, window", lambda: ops.decode(q, kc, vc, bt, lens, 16, 0.1, dws, out=o, window=window), "", 4.0 * kv * d * seen)
+        else:
+            add(phase, "prefill attention, cap, biases, sinks", lambda: scored(**terms), "prefill attention, window", flops=4.0 * d * heads * seen)
+            add(phase, "(the same without a cap)", lambda: scored(bias=bias, sink=sink), "prefill attention, window", flops=4.0 * d * heads * seen)
+            add(phase, "like: prefill attention, window",
+                lambda: ops.prefill_paged(q, kc, vc, bt, lens, por.q_lens, por.q_starts, length, 16, 0.1, out=o, window=window), "", flops=4.0 * d * heads * seen)
+        del u, kc, vc, q, o
+        # latent attention
+        lh, rank, rot = p["l_heads"], p["rank"], 64
+        row, size = rank + rot, d + rot
+        u, pool, norm = rnd(n, lh * size + row), rnd(batch * per * 16, 1, row), rnd(rank, dtype=f32)
+        rope = rnd(length + 1, rot // 2, 2, dtype=f32)
+        app = lambda: ops.latent_append(u, por, slots, pool, norm, 1e-6, rope, lh, d, rot, rank, size, 0.1)
+        add(phase, "latent norm + rotation + append", app, "q/k norm + rotation + append", n * 4.0 * (lh * size + row))
+        q = app()
+        if dec:
+            over, o = rnd(n, lh, rank), torch.empty(n, lh, rank, dtype=bf, device=dev)
+            need = ops.scored_workspace_bytes(batch, lh, 1, row, rank, True, per * 16, window)
+            ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+            add(phase, "decode attention over latents", lambda: ops.scored_attention((over, q[..., d:]), pool, pool, rank, por, bt, 16, 0.1, window, o, workspace=ws),
+                "decode attention, window", 2.0 * row * seen, 2.0 * (row + rank) * lh * seen)
+            lists = (torch.arange(n, dtype=torch.int32, device=dev)[None] * lh + torch.arange(lh, dtype=torch.int32, device=dev)[:, None]).contiguous()
+            every = ops.ExpertChoice(lists.view(n, lh), torch.empty(0, device=dev), torch.full((lh,), n, dtype=torch.int32, device=dev), lists)
+            wk, wv = rnd(lh, rank, d), rnd(lh, d, rank)
+            q2 = q.view(n * lh, size)[:, :d]
+            add(phase, "product per head, keys' side", lambda: ops.moe_product(q2, every, wk, rank, d, False), "experts: down of equal flops",
+                lh * (rank * d * 2.0 + n * 2.0 * (rank + d)), 2.0 * n * lh * rank * d)
+            add(phase, "product per head, values' side", lambda: ops.moe_product(o.view(n * lh, rank), every, wv, d, rank, False), "experts: down of equal flops",
+                lh * (rank * d * 2.0 + n * 2.0 * (rank + d)), 2.0 * n * lh * rank * d)
+            dw, dx = rnd(lh * d, rank), rnd(n, rank)
+            add(phase, "like: dense product of equal flops", lambda: F.linear(dx, dw), "", lh * rank * d * 2.0 + n * 2.0 * (rank + lh * d), 2.0 * n * lh * rank * d)
+            del over, o, wk, wv
+        else:
+            add(phase, "latent rows gathered", lambda: ops.latent_gather(pool, slots), "rope_kv_append", n * row * 4.0)
+            wk = rnd(lh * size, row)
+            lat = ops.latent_gather(pool, slots)
+            add(phase, "keys made again (library product)", lambda: F.linear(lat, wk), "dense product of equal flops", flops=2.0 * n * lh * d * rank)
+            k, v = (F.linear(lat, wk).view(n, lh, size) for _ in range(2))
+            at = i32(np.arange(n // 16).reshape(batch, -1))
+            o = torch.empty_like(q)
+            add(phase, "prefill attention over made keys",
+                lambda: ops.prefill_paged(q, k, v, at, lens, por.q_lens, por.q_starts, length, 16, 0.1, out=o, window=window), "prefill attention, window",
+                flops=2.0 * (size + d) * lh * seen)
+            add(phase, "head packing", lambda: ops.head_gate(o, None, d), "silu(gate) * up", n * lh * d * 4.0)
+            del k, v, o, lat
+        del u, pool, q
+        # delta rule
+        hs, groups = p["d_heads"], p["d_groups"]
+        qk, inner = groups * d, hs * d
+        u = rnd(n, 2 * qk + inner + 2 * hs)
+        uq, uk, uv, ga, gb = u.split([qk, qk, inner, hs, hs], 1)
+        state, out = torch.zeros(batch, hs, d, d, device=dev), torch.empty(n, inner, dtype=bf, device=dev)
+        bias, rate = torch.full((hs,), -4.0, device=dev), torch.full((hs,), 4.0, device=dev)
+
+        def run(por, ws):
+            return ops.delta_rule(uq, uk, uv, ga, gb, bias, rate, por, state, hs, d, d, d ** -0.5, out, heads_per_group=hs // groups, workspace=ws)
+        need = 0 if dec else ops.delta_workspace_bytes(batch, hs, d, d, length)
+        ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+        n_bytes = n * 2.0 * (2 * qk + 2 * inner + 2 * hs) + (batch * state[0].numel() * 8.0 if dec else 0.0)
+        # (per row and head: K K^T, Q K^T, T R, C U over 64 columns, half of them; K S, Q S, K^T U; one bf16 term each)
+        chunked = n * hs * (6.0 * d * d + 128.0 * 2 * d)
+        add(phase, "delta rule", lambda: run(por, ws), "state space", n_bytes, 0.0 if dec else chunked)
+        gstate = torch.zeros(batch, hs, ops.gated_linear_state_floats("ssd", d, d), device=dev)
+        need = 0 if dec else ops.gated_linear_workspace_bytes(batch, hs, d, d, length)
+        gws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+        ssd = lambda por, gws: ops.gated_linear("ssd", uq, uk, uv, (ga, None), (bias, rate, rate), por, gstate, hs, d, d, out, heads_per_group=hs // groups, workspace=gws)
+        add(phase, "like: state space", lambda: ssd(por, gws), "", n_bytes, 0.0 if dec else n * hs * (4.0 * d * d + 64.0 * 2 * d))
+        if not dec:
+            por1 = ops.Portions(i32([n]), i32([0]), i32([n]), i32([0]), None, n)
+            ws1 = torch.empty(ops.delta_workspace_bytes(1, hs, d, d, n), dtype=torch.uint8, device=dev)
+            add(phase, f"delta rule, one sequence of {n}", lambda: run(por1, ws1), "state space, one sequence", n_bytes, chunked)
+            gws1 = torch.empty(max(ops.gated_linear_workspace_bytes(1, hs, d, d, n), 16), dtype=torch.uint8, device=dev)
+            add(phase, "like: state space, one sequence", lambda: ssd(por1, gws1), "", n_bytes, n * hs * (4.0 * d * d + 64.0 * 2 * d))
+        nw, z = rnd(inner, dtype=f32), rnd(n, inner)
+        add(phase, "RMS norm per head + silu gate", lambda: ops.rms_gate(out, z, nw, 1e-6, groups=hs, order="silu_last"), "RMS norm per head + sigmoid gate", n * inner * 6.0)
+        add(phase, "like: RMS norm per head + sigmoid gate", lambda: ops.rms_gate(out, z, nw, 1e-6, groups=hs), "", n * inner * 6.0)
+        ch = 2 * qk + inner
+        cw, cs = rnd(4, ch, dtype=f32), torch.zeros(batch, 3, ch, dtype=bf, device=dev)
+        add(phase, "short convolution", lambda: ops.short_conv(u[:, :ch], por, cw, None, cs, "silu"), "short convolution (the same kernel)",
+            n * ch * 4.0 + (batch * 12.0 * ch if dec else 0.0) + ch * 16.0)
+        del u, state, gstate, out, z
+        torch.cuda.empty_cache()
+    return rows_out
+
+
+def bench_vusalix(args, dev) -> int:
+    """Prefill and decode throughput of Vusalix-shaped models with random weights beside Tevirax-shaped ones of the same width,
+    heads, depth and experts, and the design's kernels against their rooflines.  Not the headline workload."""
+    sizes = {}
+    steps, warmup = min(args.steps, 20), min(args.warmup, 3)
+    for name, p in VUSALIX_SHAPES.items():
+        batch, ctx_len = HYBRID_DECODE
+        blocks = batch * (ctx_len // 16 + 1)
+        model = vusalix_model(p, dev, blocks, batch, ctx_len + 16)
+        entry = {"shape": p, "vusalix": hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)}
+        del model
+        torch.cuda.empty_cache()
+        model = tevirax_model(TEVIRAX_SHAPES[name], dev, blocks, batch, ctx_len + 16)
+        entry["tevirax"] = hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)
+        del model
+        torch.cuda.empty_cache()
+        entry["kernels"] = vusalix_kernels(p, dev, steps)
+        sizes[name] = entry
+        print(f"[{name}] done", file=sys.stderr, flush=True)
+    main_size = sizes["w4096"]["vusalix"]
+    print(json.dumps({
+        "metric": "Vusalix prefill tokens/s", "value": main_size["prefill_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+        "steps": steps, "warmup": warmup, "ms_per_step": main_size["prefill_ms"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "vusalix", "layers": HYBRID_LAYERS, "prefill": HYBRID_PREFILL, "decode": HYBRID_DECODE}, "sizes": sizes}))
+    return 0
+
+
 def secondary(args, dev) -> dict:
     """Short runs of the configurations that are not the headline: what the step costs, the dominant kernel
     against its roofline and a few seconds of the CPU restatement, per workload."""
@@ -1215,6 +1444,8 @@ def main() -> int:
         return bench_hybrid(args, dev)
     if args.workload == "tevirax":
         return bench_tevirax(args, dev)
+    if args.workload == "vusalix":
+        return bench_vusalix(args, dev)
     if args.workload in PREFILL_HEAD_SHAPES:
         result = bench_prefill_head(args, dev, args.workload)
     elif args.workload in PREFILL_LONG_SHAPES:
