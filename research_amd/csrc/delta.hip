@@ -376,8 +376,8 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
     const int vcols = a.vdim - v0 < kCols ? a.vdim - v0 : kCols;
     const DeltaChunk *mats = reinterpret_cast<const DeltaChunk *>(a.ws) + (int64_t)b * a.chunks * a.heads + h;
     LaBlock qb[kKB], kb[kKB], vb[kVB];
-    uint4 mb[kMB];
-    float keep_next = 0.f, row_g[3];
+    la_u4 mb[kMB];
+    float keep_next = 0.f, row_g0 = 0.f, row_g1 = 0.f, row_g2 = 0.f;
     auto fetch = [&](int r0) {
         const int nr = p.n - r0 < 64 ? p.n - r0 : 64;
         const __amdgpu_buffer_rsrc_t tq = la_tile(uq + r0 * a.ldq, a.ldq, nr, a.dim), tk = la_tile(uk + r0 * a.ldk, a.ldk, nr, a.dim);
@@ -395,9 +395,10 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
         }
         const DeltaChunk *m = mats + (int64_t)(r0 / 64) * a.heads;
 #pragma unroll
-        for (int i = 0; i < kMB; ++i) mb[i] = reinterpret_cast<const uint4 *>(m)[tid + kThr * i];
-#pragma unroll
-        for (int i = 0; i < 3; ++i) row_g[i] = tid < 64 ? m->k_in[64 * i + tid] : 0.f;  // (k_in, q_in, k_out lie side by side)
+        for (int i = 0; i < kMB; ++i) mb[i] = reinterpret_cast<const la_u4 *>(m)[tid + kThr * i];
+        row_g0 = m->k_in[tid & 63];
+        row_g1 = m->q_in[tid & 63];
+        row_g2 = m->k_out[tid & 63];
         keep_next = m->keep;
     };
     fetch(0);
@@ -418,11 +419,12 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
 #pragma unroll
         for (int i = 0; i < kMB; ++i) {
             const int at = tid + kThr * i;  // 16-byte piece: row at / 8 over the four matrices
-            *reinterpret_cast<uint4 *>(m_s + at / 8 * kDcPitch + at % 8 * 8) = mb[i];
+            *reinterpret_cast<la_u4 *>(m_s + at / 8 * kDcPitch + at % 8 * 8) = mb[i];
         }
         if (tid < 64) {
-#pragma unroll
-            for (int i = 0; i < 3; ++i) rows[64 * i + tid] = row_g[i];
+            rows[tid] = row_g0;
+            rows[64 + tid] = row_g1;
+            rows[128 + tid] = row_g2;
         }
         const float keep = keep_next;
         if (r0 + 64 < p.n) fetch(r0 + 64);
@@ -544,10 +546,13 @@ template <int KD> int launch_delta_chunks(const DeltaArgs &a, int batch, hipStre
     // the widest slices of the value columns that leave no compute unit without one
     const int64_t heads = (int64_t)batch * a.heads;
     // (at dim 256 four waves' registers hold the state and the next chunk)
-    if constexpr (KD == 256) return launch_walk<KD, 4>(a, batch, s);
-    if (a.vdim > 64 && heads * ((a.vdim + 127) / 128) >= la_cus()) return launch_walk<KD, 8>(a, batch, s);
-    if (a.vdim > 32 && heads * ((a.vdim + 63) / 64) >= la_cus()) return launch_walk<KD, 4>(a, batch, s);
-    return launch_walk<KD, 2>(a, batch, s);
+    if constexpr (KD == 256) {
+        return launch_walk<KD, 4>(a, batch, s);
+    } else {
+        if (a.vdim > 64 && heads * ((a.vdim + 127) / 128) >= la_cus()) return launch_walk<KD, 8>(a, batch, s);
+        if (a.vdim > 32 && heads * ((a.vdim + 63) / 64) >= la_cus()) return launch_walk<KD, 4>(a, batch, s);
+        return launch_walk<KD, 2>(a, batch, s);
+    }
 }
 
 size_t delta_ws_bytes(int batch, int heads, int max_q_len) { return (size_t)batch * heads * ((max_q_len + 63) / 64) * sizeof(DeltaChunk); }

@@ -6,6 +6,8 @@
 #pragma once
 #include "row_common.h"
 
+typedef uint32_t scored_u4 __attribute__((ext_vector_type(4)));
+
 struct ScoredArgs {
     const void *q1, *q2;  // pieces of n1 and n2 elements, head h of row r at r * q*_row + h * q*_head
     int64_t q1_row, q1_head, q2_row, q2_head;
@@ -47,6 +49,20 @@ __device__ __forceinline__ int64_t scored_slot(const ScoredArgs &a, const int32_
     return id >= 0 && id < a.num_blocks ? id * a.bs + key % a.bs : -1;
 }
 
+// For loops that fetch a tile ahead: the block id of a key, loaded without a branch, and, when the tile is fetched, the key's
+// pool row.  (bt_stride > 0.)
+__device__ __forceinline__ int scored_block_id(const ScoredArgs &a, const int32_t *table, int key) {
+    return table[min((int64_t)(key / a.bs), a.bt_stride - 1)];
+}
+__device__ __forceinline__ int scored_slot_of(const ScoredArgs &a, int id, int key, int end) {
+    return key < end && key / a.bs < a.bt_stride && (uint32_t)id < (uint64_t)a.num_blocks ? id * a.bs + key % a.bs : -1;
+}
+// 16 bytes of a row, zeros where there is none: always one load, so that nothing waits for it before it is used.
+static __device__ const uint32_t kScoredZeros[4] __attribute__((aligned(16))) = {0, 0, 0, 0};
+__device__ __forceinline__ scored_u4 scored_load16(const uint16_t *p, bool there) {
+    return *reinterpret_cast<const scored_u4 *>(there ? p : reinterpret_cast<const uint16_t *>(kScoredZeros));
+}
+
 constexpr float kScoredLog2e = 1.4426950408889634f;
 constexpr float kScoredNone = -1.0e30f;  // finite stand-in for minus infinity
 
@@ -57,9 +73,10 @@ inline int scored_value_cols(int keys, int vdim, bool one) {
     return most <= 64 ? 64 : most <= 128 ? 128 : most <= 256 ? 256 : 0;
 }
 
-// Pieces that a decode step's sequences are cut into: enough for two workgroups per compute unit, of at least 256 keys each.
-inline int scored_splits(int64_t workgroups, int cus, int64_t span) {
-    int64_t n = (2 * (int64_t)cus + workgroups - 1) / workgroups;
+// Pieces that a decode step's sequences are cut into: two workgroups per compute unit (`full`: one, which has its LDS to
+// itself, and none of which waits for another's end), of at least 256 keys each.
+inline int scored_splits(int64_t workgroups, int cus, int64_t span, bool full) {
+    int64_t n = full ? cus / workgroups : (2 * (int64_t)cus + workgroups - 1) / workgroups;
     if (n > span / 256) n = span / 256;
     return n < 1 ? 1 : n > 16 ? 16 : (int)n;
 }

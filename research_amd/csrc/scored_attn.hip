@@ -81,10 +81,10 @@ int scored_cus() {
     return n;
 }
 
-int plan_splits(int batch, int heads, int hkv, bool one, int64_t max_keys, int window) {
+int plan_splits(int batch, int heads, int hkv, bool one, int vc, int64_t max_keys, int window) {
     const int rep = heads / hkv, tile = one && rep > 32 ? 64 : one && rep > 16 ? 32 : 16;
     const int64_t workgroups = (int64_t)batch * hkv * ((rep + tile - 1) / tile);
-    return scored_splits(workgroups, scored_cus(), window > 0 && window < max_keys ? window : max_keys);
+    return scored_splits(workgroups, scored_cus(), window > 0 && window < max_keys ? window : max_keys, vc > 256);
 }
 
 }  // namespace
@@ -92,8 +92,8 @@ int plan_splits(int batch, int heads, int hkv, bool one, int64_t max_keys, int w
 extern "C" size_t pa_scored_workspace_bytes(int batch, int num_q_heads, int num_kv_heads, int key_size, int vdim, int one_tensor,
                                             int64_t max_keys, int window) {
     if (batch <= 0 || num_kv_heads <= 0 || num_q_heads <= 0) return 0;
-    const int splits = plan_splits(batch, num_q_heads, num_kv_heads, one_tensor != 0, max_keys, window);
     const int vc = scored_value_cols(key_size, vdim, one_tensor != 0);
+    const int splits = plan_splits(batch, num_q_heads, num_kv_heads, one_tensor != 0, vc, max_keys, window);
     return splits > 1 && vc ? (size_t)batch * num_q_heads * splits * (vc + 2) * sizeof(float) : 0;
 }
 
@@ -133,7 +133,7 @@ extern "C" int pa_scored_attention(const void *q1, int64_t q1_row, int64_t q1_he
     const bool one = k_cache == v_cache;
     if (!q_lens && workspace) {
         const int vc = scored_value_cols(n1 + n2, vdim, one);
-        a.splits = plan_splits(batch, num_q_heads, num_kv_heads, one, bt_stride * block_size, window);
+        a.splits = plan_splits(batch, num_q_heads, num_kv_heads, one, vc, bt_stride * block_size, window);
         const size_t per = (size_t)batch * num_q_heads * (vc + 2) * sizeof(float);
         while (a.splits > 1 && per * a.splits > workspace_bytes) --a.splits;
         a.part_o = (float *)workspace;

@@ -68,19 +68,20 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
     const int kreal = (a.n1 + a.n2 + 7) / 8 * 8, vreal = (a.vdim + 7) / 8 * 8;
     const uint16_t *kp = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)kvh * a.k_dim, *vp = reinterpret_cast<const uint16_t *>(a.v) + (int64_t)kvh * a.v_dim;
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim, v_tok = (int64_t)a.hkv * a.v_dim;
-    auto slots_of = [&](int k0) { return k0 + lane < end ? (int)scored_slot(a, table, k0 + lane) : -1; };
-    uint4 kr[kKL], vr[kVL ? kVL : 1];
-    auto fetch = [&](int slots) {
+    auto id_of = [&](int k0) { return scored_block_id(a, table, min(k0 + lane, end - 1)); };
+    scored_u4 kr[kKL], vr[kVL ? kVL : 1];
+    auto fetch = [&](int id, int k0) {
+        const int slots = scored_slot_of(a, id, k0 + lane, end);
 #pragma unroll
         for (int n = 0; n < kKL; ++n) {
             const int c = tid + 256 * n, s = __shfl(slots, c / (KC / 8), 64), e = c % (KC / 8) * 8;
-            kr[n] = s >= 0 && e < kreal ? *reinterpret_cast<const uint4 *>(kp + s * k_tok + e) : make_uint4(0, 0, 0, 0);
+            kr[n] = scored_load16(kp + s * k_tok + e, s >= 0 && e < kreal);
         }
         if constexpr (!ONE) {
 #pragma unroll
             for (int n = 0; n < kVL; ++n) {
                 const int c = tid + 256 * n, s = __shfl(slots, c / (VC / 8), 64), e = c % (VC / 8) * 8;
-                vr[n] = s >= 0 && e < vreal ? *reinterpret_cast<const uint4 *>(vp + s * v_tok + e) : make_uint4(0, 0, 0, 0);
+                vr[n] = scored_load16(vp + s * v_tok + e, s >= 0 && e < vreal);
             }
         }
     };
@@ -94,25 +95,36 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
         for (int c = 0; c < kVT; ++c) o[t][c] = sd_f4{0.f, 0.f, 0.f, 0.f};
     }
     const float to2 = kScoredLog2e, plain = a.scale * kScoredLog2e, cap_in = a.cap > 0.f ? 2.f * plain / a.cap : 0.f  /* tanh(z) = 1 - 2 / (1 + e^(2z)) */, cap_out = a.cap * kScoredLog2e;
-    fetch(slots_of(lo));
-    int slots = slots_of(lo + kSdKeys);
+    const float *bias[QT];  // of this lane's heads
+#pragma unroll
+    for (int t = 0; t < QT; ++t) bias[t] = a.bias + (int64_t)(h0 + min(16 * t + l16, n_heads - 1)) * a.bias_n;
+    fetch(id_of(lo), lo);
+    int id = id_of(lo + kSdKeys);
     for (int k0 = lo; k0 < end; k0 += kSdKeys) {
 #pragma unroll
         for (int n = 0; n < kKL; ++n) {
             const int c = tid + 256 * n;
-            *reinterpret_cast<uint4 *>(ks + c / (KC / 8) * L::kPitch + c % (KC / 8) * 8) = kr[n];
+            *reinterpret_cast<scored_u4 *>(ks + c / (KC / 8) * L::kPitch + c % (KC / 8) * 8) = kr[n];
         }
         if constexpr (!ONE) {
 #pragma unroll
             for (int n = 0; n < kVL; ++n) {
                 const int c = tid + 256 * n;
-                *reinterpret_cast<uint4 *>(vs + c / (VC / 8) * L::vPitch + c % (VC / 8) * 8) = vr[n];
+                *reinterpret_cast<scored_u4 *>(vs + c / (VC / 8) * L::vPitch + c % (VC / 8) * 8) = vr[n];
             }
         }
         __syncthreads();
+        const int key = k0 + 16 * wave + 4 * g;
+        float near[QT][4];  // biases: ahead of the next tile's loads, which they do not wait for
+        if (a.bias) {
+#pragma unroll
+            for (int t = 0; t < QT; ++t)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) near[t][i] = bias[t][min(max(pos - key - i, 0), a.bias_n - 1)];
+        }
         if (k0 + kSdKeys < end) {
-            fetch(slots);
-            slots = slots_of(k0 + 2 * kSdKeys);
+            fetch(id, k0 + kSdKeys);
+            id = id_of(k0 + 2 * kSdKeys);
         }
         // scores: keys k0 + 16 wave + 4 g + i, head l16 of each query tile
         sd_f4 s[QT];
@@ -125,18 +137,30 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
 #pragma unroll
             for (int t = 0; t < QT; ++t) s[t] = sd_mfma(x, sd_read8(qa + 16 * t * L::kPitch + 32 * kk), s[t]);
         }
-        const int key = k0 + 16 * wave + 4 * g;
+        if (a.cap > 0.f) {  // (in units of the base-2 exponential)
+#pragma unroll
+            for (int t = 0; t < QT; ++t)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) s[t][i] = cap_out - 2.f * cap_out * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s[t][i] * cap_in));
+        } else {
+#pragma unroll
+            for (int t = 0; t < QT; ++t)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) s[t][i] *= plain;
+        }
+        if (a.bias) {
+#pragma unroll
+            for (int t = 0; t < QT; ++t)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) s[t][i] = fmaf(near[t][i], to2, s[t][i]);
+        }
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
             const int r = 16 * t + l16;
             float top = kScoredNone;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                float x;  // in units of the base-2 exponential
-                if (a.cap > 0.f) x = cap_out - 2.f * cap_out * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s[t][i] * cap_in));
-                else x = s[t][i] * plain;
-                if (a.bias && r < n_heads && key + i < end) x = fmaf(a.bias[(int64_t)(h0 + r) * a.bias_n + min(pos - key - i, a.bias_n - 1)], to2, x);
-                s[t][i] = key + i < end ? x : kScoredNone;
+                s[t][i] = key + i < end ? s[t][i] : kScoredNone;
                 top = fmaxf(top, s[t][i]);
             }
             top = fmaxf(top, __shfl_xor(top, 16, 64));
@@ -281,7 +305,7 @@ bool pa_scored_decode_launch(const ScoredArgs &a, int dtype, hipStream_t s, int 
     const uintptr_t at = (uintptr_t)a.q1 | (uintptr_t)a.q2 | (uintptr_t)a.k | (uintptr_t)a.v | (uintptr_t)a.out;
     if (dtype != PA_BF16 || a.q_lens || vc == 0 || (at & 15u) != 0 || a.n1 % 8 != 0 || a.n2 % 8 != 0 || a.k_dim % 8 != 0 ||
         a.v_dim % 8 != 0 || a.q1_row % 8 != 0 || a.q1_head % 8 != 0 || a.q2_row % 8 != 0 || a.q2_head % 8 != 0 ||
-        a.num_blocks * a.bs >= 0x7fffffff || !(a.scale > 0.f))
+        a.num_blocks * a.bs >= 0x7fffffff || a.bt_stride == 0 || !(a.scale > 0.f))
         return false;
     if (a.v == a.k) rc = vc == 128 ? launch_one<160, 128>(a, s) : vc == 256 ? launch_one<320, 256>(a, s) : launch_one<576, 512>(a, s);
     else rc = vc == 64 ? launch_decode<64, 64, false, 1>(a, s) : vc == 128 ? launch_decode<128, 128, false, 1>(a, s) : launch_decode<256, 256, false, 1>(a, s);

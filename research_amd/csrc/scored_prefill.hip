@@ -74,32 +74,33 @@ template <int D, bool CAP> __global__ __launch_bounds__(256, D == 256 ? 1 : 2) v
     const uint16_t *kp = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)kvh * a.k_dim, *vp = reinterpret_cast<const uint16_t *>(a.v) + (int64_t)kvh * a.v_dim;
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim, v_tok = (int64_t)a.hkv * a.v_dim;
     const int kreal = (a.n1 + 7) / 8 * 8, vreal = (a.vdim + 7) / 8 * 8;
-    auto slots_of = [&](int k0) { return k0 + lane < wg_hi ? (int)scored_slot(a, table, k0 + lane) : -1; };
-    uint4 kr[NL], vr[NL];
-    auto fetch = [&](int slots) {
+    auto id_of = [&](int k0) { return scored_block_id(a, table, min(k0 + lane, wg_hi - 1)); };
+    scored_u4 kr[NL], vr[NL];
+    auto fetch = [&](int id, int k0) {
+        const int slots = scored_slot_of(a, id, k0 + lane, wg_hi);
 #pragma unroll
         for (int n = 0; n < NL; ++n) {
             const int c = tid + 256 * n, s = __shfl(slots, c / (D / 8), 64), e = c % (D / 8) * 8;
-            kr[n] = s >= 0 && e < kreal ? *reinterpret_cast<const uint4 *>(kp + s * k_tok + e) : make_uint4(0, 0, 0, 0);
-            vr[n] = s >= 0 && e < vreal ? *reinterpret_cast<const uint4 *>(vp + s * v_tok + e) : make_uint4(0, 0, 0, 0);
+            kr[n] = scored_load16(kp + s * k_tok + e, s >= 0 && e < kreal);
+            vr[n] = scored_load16(vp + s * v_tok + e, s >= 0 && e < vreal);
         }
     };
     const int g16 = lane >> 4, s16 = lane & 15;
     const uint16_t *v_at = vs + (4 * (g16 >> 1) + (s16 >> 2)) * L::pitch + 16 * (g16 & 1) + 4 * (s16 & 3);
     const int k_start = wg_lo / kSpKeys * kSpKeys;
-    fetch(slots_of(k_start));
-    int slots = slots_of(k_start + kSpKeys);
+    fetch(id_of(k_start), k_start);
+    int id = id_of(k_start + kSpKeys);
     for (int k0 = k_start; k0 < wg_hi; k0 += kSpKeys) {
 #pragma unroll
         for (int n = 0; n < NL; ++n) {
             const int c = tid + 256 * n, at = c / (D / 8) * L::pitch + c % (D / 8) * 8;
-            *reinterpret_cast<uint4 *>(ks + at) = kr[n];
-            *reinterpret_cast<uint4 *>(vs + at) = vr[n];
+            *reinterpret_cast<scored_u4 *>(ks + at) = kr[n];
+            *reinterpret_cast<scored_u4 *>(vs + at) = vr[n];
         }
         __syncthreads();
         if (k0 + kSpKeys < wg_hi) {
-            fetch(slots);
-            slots = slots_of(k0 + 2 * kSpKeys);
+            fetch(id, k0 + kSpKeys);
+            id = id_of(k0 + 2 * kSpKeys);
         }
 #pragma unroll
         for (int sub = 0; sub < 2; ++sub) {
@@ -211,7 +212,7 @@ bool pa_scored_prefill_launch(const ScoredArgs &a, int dtype, hipStream_t s, int
     if (a.window > 0 && bias_n > a.window) bias_n = a.window;  // (no distance reaches the window)
     if (dtype != PA_BF16 || !a.q_lens || a.n2 != 0 || most > 256 || bias_n > kSpMaxBias || (at & 15u) != 0 || a.n1 % 8 != 0 ||
         a.k_dim % 8 != 0 || a.v_dim % 8 != 0 || a.q1_row % 8 != 0 || a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff ||
-        !(a.scale > 0.f))
+        a.bt_stride == 0 || !(a.scale > 0.f))
         return false;
     rc = most <= 64 ? launch_prefill_cap<64>(a, bias_n, s) : most <= 128 ? launch_prefill_cap<128>(a, bias_n, s) : launch_prefill_cap<256>(a, bias_n, s);
     return true;
