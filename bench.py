@@ -1320,16 +1320,16 @@ def vusalix_kernels(p, dev, steps):
             del over, o, wk, wv
         else:
             add(phase, "latent rows gathered", lambda: ops.latent_gather(pool, slots), "rope_kv_append", n * row * 4.0)
-            wk = rnd(lh * size, row)
+            wk, wv = rnd(lh * size, row), rnd(lh * d, row)
             lat = ops.latent_gather(pool, slots)
             add(phase, "keys made again (library product)", lambda: F.linear(lat, wk), "dense product of equal flops", flops=2.0 * n * lh * d * rank)
-            k, v = (F.linear(lat, wk).view(n, lh, size) for _ in range(2))
+            add(phase, "values made again (library product)", lambda: F.linear(lat, wv), "dense product of equal flops", flops=2.0 * n * lh * d * rank)
+            k, v = (F.linear(lat, w).view(n, lh, -1) for w in (wk, wv))
             at = i32(np.arange(n // 16).reshape(batch, -1))
-            o = torch.empty_like(q)
-            add(phase, "prefill attention over made keys",
-                lambda: ops.prefill_paged(q, k, v, at, lens, por.q_lens, por.q_starts, length, 16, 0.1, out=o, window=window), "prefill attention, window",
+            o = torch.empty(n, lh, d, dtype=bf, device=dev)
+            made = ops.Portions(lens, lens, por.q_lens, por.q_starts, None, length)
+            add(phase, "prefill attention over made keys", lambda: ops.scored_attention((q,), k, v, d, made, at, 16, 0.1, window, o), "prefill attention, window",
                 flops=2.0 * (size + d) * lh * seen)
-            add(phase, "head packing", lambda: ops.head_gate(o, None, d), "silu(gate) * up", n * lh * d * 4.0)
             del k, v, o, lat
         del u, pool, q
         # delta rule

@@ -1,4 +1,4 @@
-// Portions of prompts of attention with score terms on the matrix cores (16-bit pools of one head size up to 256).
+// Portions of prompts of attention with score terms on the matrix cores (16-bit pools, keys and values of up to 256).
 //
 // A wave owns 32 rows of one query head, a workgroup four (row block, head) pairs of one kv head in turn, which share tiles of
 // 64 keys and values in LDS; the next tile is on its way in registers.  As in prefill_mfma.h everything is transposed:
@@ -15,19 +15,19 @@ using namespace pa_decode_detail;
 constexpr int kSpKeys = 64, kSpMargin = 64, kSpMaxBias = 4096;
 constexpr float kSpSlack = 8.f;  // log2 of the factor by which a row's reference maximum may lag
 
-template <int D> struct SpTile {
-    static constexpr int pitch = D + 8;
-    static constexpr size_t tiles = (size_t)2 * kSpKeys * pitch * 2;
+template <int DK, int DV> struct SpTile {
+    static constexpr int k_pitch = DK + 8, v_pitch = DV + 8;
+    static constexpr size_t tiles = (size_t)kSpKeys * (k_pitch + v_pitch) * 2;
 };
 
-template <int D, bool CAP> __global__ __launch_bounds__(256, D == 256 ? 1 : 2) void scored_prefill_kernel(const ScoredArgs a, int bias_n) {
+template <int DK, int DV, bool CAP> __global__ __launch_bounds__(256, DV == 256 ? 1 : 2) void scored_prefill_kernel(const ScoredArgs a, int bias_n) {
     using M = Mfma16<pa_bf16>;
     using X8 = M::x8;
     using X4 = M::x4;
-    using L = SpTile<D>;
-    constexpr int KS = D / 16, DT = D / 32, NL = kSpKeys * D / 8 / 256;
+    using L = SpTile<DK, DV>;
+    constexpr int KS = DK / 16, DT = DV / 32, NK = kSpKeys * DK / 8 / 256, NV = kSpKeys * DV / 8 / 256;
     extern __shared__ __align__(16) char sp_lds[];
-    uint16_t *ks = reinterpret_cast<uint16_t *>(sp_lds), *vs = ks + kSpKeys * L::pitch;
+    uint16_t *ks = reinterpret_cast<uint16_t *>(sp_lds), *vs = ks + kSpKeys * L::k_pitch;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), half = lane >> 5, col = lane & 31;
     const int table_n = bias_n + 2 * kSpMargin;
     float *bias = reinterpret_cast<float *>(sp_lds + L::tiles) + wave * table_n;
@@ -75,27 +75,35 @@ template <int D, bool CAP> __global__ __launch_bounds__(256, D == 256 ? 1 : 2) v
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim, v_tok = (int64_t)a.hkv * a.v_dim;
     const int kreal = (a.n1 + 7) / 8 * 8, vreal = (a.vdim + 7) / 8 * 8;
     auto id_of = [&](int k0) { return scored_block_id(a, table, min(k0 + lane, wg_hi - 1)); };
-    scored_u4 kr[NL], vr[NL];
+    scored_u4 kr[NK], vr[NV];
     auto fetch = [&](int id, int k0) {
         const int slots = scored_slot_of(a, id, k0 + lane, wg_hi);
 #pragma unroll
-        for (int n = 0; n < NL; ++n) {
-            const int c = tid + 256 * n, s = __shfl(slots, c / (D / 8), 64), e = c % (D / 8) * 8;
+        for (int n = 0; n < NK; ++n) {
+            const int c = tid + 256 * n, s = __shfl(slots, c / (DK / 8), 64), e = c % (DK / 8) * 8;
             kr[n] = scored_load16(kp + s * k_tok + e, s >= 0 && e < kreal);
+        }
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const int c = tid + 256 * n, s = __shfl(slots, c / (DV / 8), 64), e = c % (DV / 8) * 8;
             vr[n] = scored_load16(vp + s * v_tok + e, s >= 0 && e < vreal);
         }
     };
     const int g16 = lane >> 4, s16 = lane & 15;
-    const uint16_t *v_at = vs + (4 * (g16 >> 1) + (s16 >> 2)) * L::pitch + 16 * (g16 & 1) + 4 * (s16 & 3);
+    const uint16_t *v_at = vs + (4 * (g16 >> 1) + (s16 >> 2)) * L::v_pitch + 16 * (g16 & 1) + 4 * (s16 & 3);
     const int k_start = wg_lo / kSpKeys * kSpKeys;
     fetch(id_of(k_start), k_start);
     int id = id_of(k_start + kSpKeys);
     for (int k0 = k_start; k0 < wg_hi; k0 += kSpKeys) {
 #pragma unroll
-        for (int n = 0; n < NL; ++n) {
-            const int c = tid + 256 * n, at = c / (D / 8) * L::pitch + c % (D / 8) * 8;
-            *reinterpret_cast<scored_u4 *>(ks + at) = kr[n];
-            *reinterpret_cast<scored_u4 *>(vs + at) = vr[n];
+        for (int n = 0; n < NK; ++n) {
+            const int c = tid + 256 * n;
+            *reinterpret_cast<scored_u4 *>(ks + c / (DK / 8) * L::k_pitch + c % (DK / 8) * 8) = kr[n];
+        }
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const int c = tid + 256 * n;
+            *reinterpret_cast<scored_u4 *>(vs + c / (DV / 8) * L::v_pitch + c % (DV / 8) * 8) = vr[n];
         }
         __syncthreads();
         if (k0 + kSpKeys < wg_hi) {
@@ -111,7 +119,7 @@ template <int D, bool CAP> __global__ __launch_bounds__(256, D == 256 ? 1 : 2) v
             for (int i = 0; i < 16; ++i) s[i] = 0.f;
 #pragma unroll
             for (int k = 0; k < KS; ++k)
-                s = M::mma(__builtin_bit_cast(X8, *reinterpret_cast<const uint4 *>(ks + (32 * sub + col) * L::pitch + 16 * k + 8 * half)), q[k], s);
+                s = M::mma(__builtin_bit_cast(X8, *reinterpret_cast<const uint4 *>(ks + (32 * sub + col) * L::k_pitch + 16 * k + 8 * half)), q[k], s);
             // element i: key kb + 8 (i / 4) + 4 half + i % 4
             const bool is_far = p.pos0 + row0 - (kb + 31) >= bias_n - 1;  // every distance shares the last bias
             const float *bp = bias + kSpMargin - 1 + bias_n - (p.pos0 + row) + kb + 4 * half;
@@ -154,8 +162,8 @@ template <int D, bool CAP> __global__ __launch_bounds__(256, D == 256 ? 1 : 2) v
                 const X8 pb = __builtin_bit_cast(X8, make_uint4(w[4 * k2], w[4 * k2 + 1], w[4 * k2 + 2], w[4 * k2 + 3]));
 #pragma unroll
                 for (int t = 0; t < DT; ++t) {
-                    const uint16_t *at = v_at + (32 * sub + 16 * k2) * L::pitch + 32 * t;
-                    const X4 x = M::tr_read(at), y = M::tr_read(at + 8 * L::pitch);
+                    const uint16_t *at = v_at + (32 * sub + 16 * k2) * L::v_pitch + 32 * t;
+                    const X4 x = M::tr_read(at), y = M::tr_read(at + 8 * L::v_pitch);
                     X8 va;
 #pragma unroll
                     for (int e = 0; e < 4; ++e) { va[e] = x[e]; va[4 + e] = y[e]; }
@@ -185,22 +193,22 @@ template <int D, bool CAP> __global__ __launch_bounds__(256, D == 256 ? 1 : 2) v
         }
 }
 
-template <int D, bool CAP> int launch_prefill(const ScoredArgs &a, int bias_n, hipStream_t s) {
-    const size_t lds = SpTile<D>::tiles + (size_t)4 * (bias_n + 2 * kSpMargin) * sizeof(float);
+template <int DK, int DV, bool CAP> int launch_prefill(const ScoredArgs &a, int bias_n, hipStream_t s) {
+    const size_t lds = SpTile<DK, DV>::tiles + (size_t)4 * (bias_n + 2 * kSpMargin) * sizeof(float);
     if (lds > 64 * 1024) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(scored_prefill_kernel<D, CAP>),
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(scored_prefill_kernel<DK, DV, CAP>),
                                                  hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return pa_fail(PA_ERR_HIP, "pa_scored_attention: %s", hipGetErrorString(e));
     }
     const int groups = ((a.max_q_len + 31) / 32 * a.n_rep + 3) / 4;
     PA_REQUIRE(groups <= 65535, "pa_scored_attention: max_q_len=%d is too long for one launch", a.max_q_len);
-    scored_prefill_kernel<D, CAP><<<dim3((unsigned)a.hkv, (unsigned)groups, (unsigned)a.batch), dim3(256), lds, s>>>(a, bias_n);
+    scored_prefill_kernel<DK, DV, CAP><<<dim3((unsigned)a.hkv, (unsigned)groups, (unsigned)a.batch), dim3(256), lds, s>>>(a, bias_n);
     PA_CHECK_LAUNCH("pa_scored_attention (portions)");
     return PA_OK;
 }
 
-template <int D> int launch_prefill_cap(const ScoredArgs &a, int bias_n, hipStream_t s) {
-    return a.cap > 0.f ? launch_prefill<D, true>(a, bias_n, s) : launch_prefill<D, false>(a, bias_n, s);
+template <int DK, int DV> int launch_prefill_cap(const ScoredArgs &a, int bias_n, hipStream_t s) {
+    return a.cap > 0.f ? launch_prefill<DK, DV, true>(a, bias_n, s) : launch_prefill<DK, DV, false>(a, bias_n, s);
 }
 
 }  // namespace
@@ -214,6 +222,9 @@ bool pa_scored_prefill_launch(const ScoredArgs &a, int dtype, hipStream_t s, int
         a.k_dim % 8 != 0 || a.v_dim % 8 != 0 || a.q1_row % 8 != 0 || a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff ||
         a.bt_stride == 0 || !(a.scale > 0.f))
         return false;
-    rc = most <= 64 ? launch_prefill_cap<64>(a, bias_n, s) : most <= 128 ? launch_prefill_cap<128>(a, bias_n, s) : launch_prefill_cap<256>(a, bias_n, s);
+    rc = most <= 64                        ? launch_prefill_cap<64, 64>(a, bias_n, s)
+         : most <= 128                     ? launch_prefill_cap<128, 128>(a, bias_n, s)
+         : a.n1 <= 192 && a.vdim <= 128    ? launch_prefill_cap<192, 128>(a, bias_n, s)
+                                           : launch_prefill_cap<256, 256>(a, bias_n, s);
     return true;
 }

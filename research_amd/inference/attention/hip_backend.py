@@ -798,8 +798,11 @@ class HipPagedAttentionBackend:
         return step.stretches[window]
 
     def attend_stretch(self, q: Tensor, k: Tensor, v: Tensor, stretch: Stretch, scale: float, window: int, out: Tensor) -> Tensor:
-        """Attention of a step's portions over the keys and values ``[rows, Hkv, D]`` of their stretch."""
+        """Attention of a step's portions over the keys and values ``[rows, Hkv, size]`` of their stretch; values of another
+        size than keys go to the kernel that holds two sizes."""
         c = stretch.portions
+        if k.shape[2] != v.shape[2]:
+            return ops.scored_attention((q,), k, v, v.shape[2], c, stretch.tables, STRETCH_BLOCK, scale, window, out)
         need = ops.prefill_workspace_bytes(q, stretch.tables, c.max_q_len, STRETCH_BLOCK, k.shape[1], window)
         return ops.prefill_paged(q, k, v, stretch.tables, c.ctx_lens, c.q_lens, c.q_starts, c.max_q_len, STRETCH_BLOCK, scale, out=out,
                                  window=window, workspace=self._scratch_for(need) if need else None)

@@ -210,9 +210,11 @@ class LatentSpec:
         return 1, self.pool_row, 0
 
     @property
-    def head_dim(self) -> int:
-        """Size of a head's key or value made again from the latents."""
-        return _pad8(max(self.dim + self.rot_dim, self.vdim))
+    def made(self) -> Tuple[int, int]:
+        """Sizes of a head's key and value made again from the latents: one size, as the kernels for plain attention have it,
+        except where that would carry values of at most 128 in rows of 256."""
+        key, value = _pad8(self.dim + self.rot_dim), _pad8(self.vdim)
+        return (key, value) if 128 < key <= 192 and value <= 128 else (max(key, value),) * 2
 
 
 @dataclass(frozen=True)
@@ -713,10 +715,9 @@ class LatentAttention(Mixer):
         self.norm = _param(s.kv_rank, dtype=torch.float32, device=device)
         self.w_key = _param(s.heads, s.kv_rank, pad(s.dim), **kw)
         self.w_value = _param(s.heads, s.vdim, pad(s.kv_rank), **kw)
-        self.remake = dtype == torch.bfloat16 and s.head_dim <= 256
+        self.remake = dtype == torch.bfloat16 and max(s.made) <= 256
         if self.remake:
-            self.k_made = _param(s.heads, s.head_dim, s.pool_row, **kw)
-            self.v_made = _param(s.heads, s.head_dim, s.pool_row, **kw)
+            self.k_made, self.v_made = (_param(s.heads, size, s.pool_row, **kw) for size in s.made)
         self._lists: Dict[int, ops.ExpertChoice] = {}
 
     def load(self, get: Getter, prefix: str) -> None:
@@ -760,7 +761,7 @@ class LatentAttention(Mixer):
         pool, _ = self.backend._layer(self.layer_idx)
         # (q carries scale * log2(e) from its 32-bit registers)
         q = ops.latent_append(u, packed.rows, packed.slots, pool, self.norm, self.eps, self.rotary.get(s.rot_base, s.rot_dim, 1.0, s.rot_yarn),
-                              s.heads, s.dim, s.rot_dim, s.kv_rank, s.head_dim, s.scale / _LN2)
+                              s.heads, s.dim, s.rot_dim, s.kv_rank, s.made[0], s.scale / _LN2)
         nd = packed.num_decodes
         if packed.chunks is None:
             o = self._over_latents(q, packed, "decodes")
@@ -768,11 +769,14 @@ class LatentAttention(Mixer):
         if self.remake:
             stretch = self.backend.stretch(packed, s.window or 0)
             rows = ops.latent_gather(pool, stretch.slots)
-            k, v = (F.linear(rows, w.view(-1, s.pool_row)).view(-1, s.heads, s.head_dim) for w in (self.k_made, self.v_made))
-            o = self.backend.attend_stretch(q, k, v, stretch, _LN2, s.window or 0, torch.empty_like(q))
-            if out is None:
-                out = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
-            ops.head_gate(o[nd:], None, s.vdim, out=out[nd:])
+            k, v = (F.linear(rows, w.view(-1, s.pool_row)).view(-1, s.heads, w.shape[1]) for w in (self.k_made, self.v_made))
+            o = self.backend.attend_stretch(q, k, v, stretch, _LN2, s.window or 0, q.new_empty(u.shape[0], s.heads, v.shape[2]))
+            if out is None and v.shape[2] == s.vdim:
+                out = o.view(u.shape[0], -1)
+            else:
+                if out is None:
+                    out = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
+                ops.head_gate(o[nd:], None, s.vdim, out=out[nd:])
         else:
             o = self._over_latents(q, packed, "chunks")
             out = o if out is None else out.copy_(o)

@@ -246,7 +246,8 @@ def _whole(paged, i, q, vdim, scale, window, cap, rel, most, sink):
 
 
 SCORED = [  # heads, kv heads, dim, vdim, window, cap, buckets, bias_max
-    (6, 3, 48, 48, 70, 20.0, 16, 90), (4, 1, 64, 32, 33, 5.0, 8, 20), (8, 2, 128, 96, 100, 30.0, 32, 128), (3, 3, 20, 36, 17, None, 4, 9),
+    (6, 2, 40, 56, 70, 18.0, 16, 90), (4, 1, 64, 32, 33, 5.0, 8, 20), (4, 2, 184, 120, 80, 12.0, 14, 50), (3, 3, 160, 72, 45, None, 10, 60),
+    (8, 2, 128, 96, 100, 30.0, 32, 128), (3, 3, 20, 36, 17, None, 4, 9),
     (20, 1, 40, 40, None, 8.0, 12, 300), (2, 1, 136, 200, 64, 15.0, 6, 64), (5, 5, 24, 16, 1, 4.0, 2, 3), (9, 3, 33, 21, 50, 12.0, 10, 40)]
 
 
@@ -361,7 +362,7 @@ def test_decode_pieces_with_sinks_and_padding_rows():
 
 
 @pytest.mark.parametrize("dtype", [F32, BF])
-@pytest.mark.parametrize("heads,dim,rot,rank", [(3, 24, 8, 40), (2, 64, 16, 128), (5, 20, 10, 30), (1, 0, 6, 17), (16, 128, 64, 512)])
+@pytest.mark.parametrize("heads,dim,rot,rank", [(3, 24, 8, 40), (2, 72, 16, 120), (5, 20, 10, 30), (1, 0, 6, 17), (16, 128, 64, 512)])
 def test_latent_rows_are_normed_turned_and_appended(heads, dim, rot, rank, dtype):
     announce(f"latent append {heads} {dim} {rot} {rank} {dtype}")
     pad = lambda n: -(-n // 8) * 8
