@@ -151,7 +151,10 @@ template <typename T, int R> __global__ __launch_bounds__(256, 4) void delta_rec
 
 // ------------------------------------------------------------------ chunks: T and C
 constexpr int kDcPitch = 72;  // bf16 per row of T and C in LDS
-struct DeltaChunk {           // what the first pass leaves per chunk and head
+// Operands that meet a result as their partner have the inner order 4 g + 0 .. 3, 16 + 4 g + 0 .. 3 within 32: stored in that
+// order, a lane's eight elements are one 16-byte chunk.  Position of element c:
+__host__ __device__ constexpr int delta_paired(int c) { return (c & ~31) | (c & 12) << 1 | (c & 16) >> 2 | (c & 3); }
+struct DeltaChunk {           // what the first pass leaves per chunk and head (columns of T and C paired)
     uint16_t t_hi[64][64], t_lo[64][64], c_hi[64][64], c_lo[64][64];
     float k_in[64];   // e^F times k's unit factor (on K S)
     float q_in[64];   // e^F times q's unit factor and scale (on Q S)
@@ -173,10 +176,12 @@ __device__ __forceinline__ float delta_scan(float x, int lane) {
 }
 
 // Workgroup: one chunk of one head.  Wave w: rows 16 w .. of the products.
-template <int KD> __global__ __launch_bounds__(256) void delta_prepare_kernel(const DeltaArgs a) {
-    constexpr int kLd = KD + 8, kMat = 68;
-    __shared__ __align__(16) __bf16 q_s[64 * kLd], k_s[64 * kLd];
-    __shared__ float mat[64][kMat], inv[64][kMat];  // A below the diagonal, then (I + A)^-1
+template <int KD> __global__ __launch_bounds__(256, KD == 256 ? 2 : 4) void delta_prepare_kernel(const DeltaArgs a) {
+    constexpr int kLd = KD + 8, kMat = 68, kRowBytes = 2 * 64 * kLd * 2, kMatBytes = 2 * 64 * kMat * 4;
+    __shared__ __align__(16) char room[kRowBytes > kMatBytes ? kRowBytes : kMatBytes];
+    __bf16 *q_s = reinterpret_cast<__bf16 *>(room), *k_s = q_s + 64 * kLd;
+    // in their place once the products are made: A below the diagonal, (I + A)^-1
+    float(*mat)[kMat] = reinterpret_cast<float(*)[kMat]>(room), (*inv)[kMat] = mat + 64;
     __shared__ float part[4][16][17];
     __shared__ float f_s[64], beta_s[64], kn_s[64], qn_s[64];
     const int h = blockIdx.x, chunk = blockIdx.y, b = blockIdx.z;
@@ -255,6 +260,7 @@ template <int KD> __global__ __launch_bounds__(256) void delta_prepare_kernel(co
             qk[st] = la_mfma(x, bq, qk[st]);
         }
     }
+    __syncthreads();
     const int t = 16 * wave + l16;
     const float ft = f_s[t], bt = beta_s[t] * kn_s[t], qt = qn_s[t];
 #pragma unroll
@@ -270,8 +276,8 @@ template <int KD> __global__ __launch_bounds__(256) void delta_prepare_kernel(co
         uint2 hi, lo;
         la_split2(c[0], c[1], hi.x, lo.x);
         la_split2(c[2], c[3], hi.y, lo.y);
-        *reinterpret_cast<uint2 *>(&out->c_hi[t][16 * st + 4 * g]) = hi;
-        *reinterpret_cast<uint2 *>(&out->c_lo[t][16 * st + 4 * g]) = lo;
+        *reinterpret_cast<uint2 *>(&out->c_hi[t][delta_paired(16 * st + 4 * g)]) = hi;
+        *reinterpret_cast<uint2 *>(&out->c_lo[t][delta_paired(16 * st + 4 * g)]) = lo;
     }
     // (the wave's own 16 rows of mat: its accesses are in order, the compiler must keep them so)
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
@@ -318,14 +324,23 @@ template <int KD> __global__ __launch_bounds__(256) void delta_prepare_kernel(co
         uint2 hi, lo;
         la_split2(x[0], x[1], hi.x, lo.x);
         la_split2(x[2], x[3], hi.y, lo.y);
-        *reinterpret_cast<uint2 *>(&out->t_hi[r][c]) = hi;
-        *reinterpret_cast<uint2 *>(&out->t_lo[r][c]) = lo;
+        *reinterpret_cast<uint2 *>(&out->t_hi[r][delta_paired(c)]) = hi;
+        *reinterpret_cast<uint2 *>(&out->t_lo[r][delta_paired(c)]) = lo;
     }
 }
 
 // ------------------------------------------------------------------ chunks: the walk
+// Tiles of Q and K: paired columns, chunk c of row r at position c ^ delta_hash(r).  Operand reads (16 rows, one chunk) and
+// transposing reads (four rows, four chunks) both spread over the banks.
+template <int KD> __device__ __forceinline__ int delta_hash(int r) { return (KD == 64 ? (r & 2) << 1 : (r & 3) << 2) | (r >> 2 & 3); }
+template <int KD> __device__ __forceinline__ void delta_put(const LaBlock &b, int r, int c, __bf16 *tile) {
+    const int e = delta_paired(c);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) *reinterpret_cast<uint2 *>(tile + (r + i) * KD + (((e >> 3) ^ delta_hash<KD>(r + i)) << 3) + (e & 4)) = b.r[i];
+}
+
 template <int KD, int COLS> constexpr size_t delta_walk_lds() {
-    return (size_t)(2 * 64 * (KD + 8) + KD * 64 + COLS * 64 + 4 * 64 * kDcPitch) * 2 + 3 * 64 * 4 + 64;
+    return (size_t)(2 * 64 * KD + 64 * (COLS + 8) + 4 * 64 * kDcPitch) * 2 + 3 * 64 * 4 + 64;
 }
 
 // Two bf16 terms of eight values of a result tile pair, as an operand whose inner index runs 4 g + 0 .. 3, then 16 more
@@ -340,14 +355,14 @@ __device__ __forceinline__ LaSplit delta_split(const f4 &x, const f4 &y) {
 
 // KD: dim padded to 64, 128 or 256.  A workgroup of NW waves owns 16 NW value columns of a head and all chunks of a portion.
 template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_walk_kernel(const DeltaArgs a) {
-    constexpr int kCols = 16 * NW, kThr = 64 * NW, kLd = KD + 8;
+    constexpr int kCols = 16 * NW, kThr = 64 * NW, kLv = kCols + 8;
     constexpr int kBlocks = 16 * (KD / 4), kKB = (kBlocks + kThr - 1) / kThr;  // 4 x 4 blocks of K, of V; 16-byte pieces of T and C
     constexpr int kVB = 16 * (kCols / 4) / kThr, kMB = 4 * 64 * 8 / kThr;
     static_assert(16 * (kCols / 4) % kThr == 0 && (kBlocks % kThr == 0 || kKB == 1), "whole passes");
     const bool k_live = kBlocks >= kThr || (int)threadIdx.x < kBlocks;
     extern __shared__ __align__(16) char lds[];
-    __bf16 *q_s = reinterpret_cast<__bf16 *>(lds), *k_s = q_s + 64 * kLd, *kt_s = k_s + 64 * kLd, *vt_s = kt_s + KD * 64;
-    __bf16 *m_s = vt_s + kCols * 64;  // T's two terms, C's two terms
+    __bf16 *q_s = reinterpret_cast<__bf16 *>(lds), *k_s = q_s + 64 * KD, *v_s = k_s + 64 * KD;
+    __bf16 *m_s = v_s + 64 * kLv;  // T's two terms, C's two terms
     float *rows = reinterpret_cast<float *>(m_s + 4 * 64 * kDcPitch);  // k_in, q_in, k_out
     const __bf16 *t_hi = m_s, *t_lo = m_s + 64 * kDcPitch, *c_hi = m_s + 2 * 64 * kDcPitch, *c_lo = m_s + 3 * 64 * kDcPitch;
     const int h = blockIdx.x, v0 = blockIdx.y * kCols, b = blockIdx.z;
@@ -408,13 +423,13 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
         for (int i = 0; i < kKB; ++i) {
             const int blk = tid + kThr * i, r = blk / (KD / 4) * 4, c = blk % (KD / 4) * 4;
             if (!k_live) continue;
-            la_put_block<false>(qb[i], r, c, q_s, kLd, nullptr);
-            la_put_block<false>(kb[i], r, c, k_s, kLd, kt_s);
+            delta_put<KD>(qb[i], r, c, q_s);
+            delta_put<KD>(kb[i], r, c, k_s);
         }
 #pragma unroll
         for (int i = 0; i < kVB; ++i) {
             const int blk = tid + kThr * i, r = blk / (kCols / 4) * 4, c = blk % (kCols / 4) * 4;
-            la_put_block<false>(vb[i], r, c, nullptr, 0, vt_s);
+            la_put_block<false>(vb[i], r, c, v_s, kLv, nullptr);
         }
 #pragma unroll
         for (int i = 0; i < kMB; ++i) {
@@ -439,19 +454,18 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
             const bf8 hi = sp.high(), lo = sp.low();
 #pragma unroll
             for (int tt = 0; tt < 4; ++tt) {
-                const int at = (16 * tt + l16) * kLd + 32 * dd + 4 * g;
-                const bf8 xk = la_read44(k_s + at, k_s + at + 16), xq = la_read44(q_s + at, q_s + at + 16);
+                const int at = (16 * tt + l16) * KD + ((4 * dd + g) ^ delta_hash<KD>(l16)) * 8;
+                const bf8 xk = la_read8(k_s + at), xq = la_read8(q_s + at);
                 u[tt] = la_mfma(xk, hi, u[tt]);
                 u[tt] = la_mfma(xk, lo, u[tt]);
                 o[tt] = la_mfma(hi, xq, o[tt]);
                 o[tt] = la_mfma(lo, xq, o[tt]);
             }
         }
-        typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
 #pragma unroll
         for (int tt = 0; tt < 4; ++tt) {
             const f4 ki = *reinterpret_cast<const f4 *>(rows + 16 * tt + 4 * g);
-            const bf4 vv = *reinterpret_cast<const bf4 *>(vt_s + la_tr(vw + l16, 16 * tt + 4 * g));
+            const la_bf4 vv = la_read_tr(v_s + (16 * tt + 4 * g + l16 / 4) * kLv + vw + l16 % 4 * 4);
             const float qi = rows[64 + 16 * tt + l16];
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
@@ -469,8 +483,8 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
             const bf8 hi = sp.high(), lo = sp.low();
 #pragma unroll
             for (int tt = 2 * kk; tt < 4; ++tt) {
-                const int at = (16 * tt + l16) * kDcPitch + 32 * kk + 4 * g;
-                const bf8 th = la_read44(t_hi + at, t_hi + at + 16), tl = la_read44(t_lo + at, t_lo + at + 16);
+                const int at = (16 * tt + l16) * kDcPitch + 32 * kk + 8 * g;
+                const bf8 th = la_read8(t_hi + at), tl = la_read8(t_lo + at);
                 w[tt] = la_mfma(th, hi, w[tt]);
                 w[tt] = la_mfma(th, lo, w[tt]);
                 w[tt] = la_mfma(tl, hi, w[tt]);
@@ -488,8 +502,8 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
                 const bf8 hi = sp.high(), lo = sp.low();
 #pragma unroll
                 for (int tt = 2 * kk; tt < 4; ++tt) {
-                    const int at = (16 * tt + l16) * kDcPitch + 32 * kk + 4 * g;
-                    const bf8 ch = la_read44(c_hi + at, c_hi + at + 16), cl = la_read44(c_lo + at, c_lo + at + 16);
+                    const int at = (16 * tt + l16) * kDcPitch + 32 * kk + 8 * g;
+                    const bf8 ch = la_read8(c_hi + at), cl = la_read8(c_lo + at);
                     o[tt] = la_mfma(hi, ch, o[tt]);
                     o[tt] = la_mfma(lo, ch, o[tt]);
                     o[tt] = la_mfma(hi, cl, o[tt]);
@@ -505,7 +519,9 @@ template <int KD, int NW> __global__ __launch_bounds__(64 * NW, 1) void delta_wa
             const bf8 hi = sp.high(), lo = sp.low();
 #pragma unroll
             for (int dt = 0; dt < KD / 16; ++dt) {
-                const bf8 xk = la_read44(kt_s + la_tr(16 * dt + l16, 32 * kk + 4 * g), kt_s + la_tr(16 * dt + l16, 32 * kk + 4 * g + 16));
+                const int row = 4 * g + l16 / 4;
+                const __bf16 *at = k_s + (32 * kk + row) * KD + ((dt / 2 * 4 + l16 % 4) ^ delta_hash<KD>(row)) * 8 + dt % 2 * 4;
+                const bf8 xk = la_join(la_read_tr(at), la_read_tr(at + 16 * KD));
                 s[dt] = la_mfma(xk, hi, s[dt]);
                 s[dt] = la_mfma(xk, lo, s[dt]);
             }

@@ -7,6 +7,7 @@
 namespace {
 
 typedef __bf16 bf8 __attribute__((ext_vector_type(8)));
+typedef __bf16 la_bf4 __attribute__((ext_vector_type(4)));
 typedef float f4 __attribute__((ext_vector_type(4)));
 typedef uint32_t la_u2 __attribute__((ext_vector_type(2)));
 typedef uint32_t la_u4 __attribute__((ext_vector_type(4)));
@@ -23,10 +24,14 @@ __device__ __forceinline__ int la_tr(int r, int s) { return r * 64 + ((((s >> 3)
 __device__ __forceinline__ f4 la_mfma(bf8 x, bf8 y, f4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, c, 0, 0, 0); }
 
 __device__ __forceinline__ bf8 la_read8(const __bf16 *p) { return *reinterpret_cast<const bf8 *>(p); }
+__device__ __forceinline__ bf8 la_join(la_bf4 x, la_bf4 y) { return bf8{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]}; }
 __device__ __forceinline__ bf8 la_read44(const __bf16 *p, const __bf16 *q) {
-    typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
-    const bf4 x = *reinterpret_cast<const bf4 *>(p), y = *reinterpret_cast<const bf4 *>(q);
-    return bf8{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+    return la_join(*reinterpret_cast<const la_bf4 *>(p), *reinterpret_cast<const la_bf4 *>(q));
+}
+// Lane i of 16 gets column i of four rows from a 4 x 16 block in LDS whose lane s points at row s / 4, columns 4 (s % 4) ..
+__device__ __forceinline__ la_bf4 la_read_tr(const __bf16 *p) {
+    typedef short s4 __attribute__((ext_vector_type(4)));
+    return __builtin_bit_cast(la_bf4, __builtin_amdgcn_ds_read_tr16_b64_v4i16((s4 __attribute__((address_space(3))) *)p));
 }
 // Pairs x = hi + lo, packed bf16
 __device__ __forceinline__ void la_split2(float x0, float x1, uint32_t &hi, uint32_t &lo) {

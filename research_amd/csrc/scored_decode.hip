@@ -1,9 +1,10 @@
 // Decode steps of attention with score terms on the matrix cores (16-bit pools): one row per sequence, a workgroup per
 // (kv head, 16 QT of its query heads, piece of the sequence's keys).
 //
-// A tile of 64 keys goes from memory through registers into LDS while the tile before it is multiplied.  Each of the four
-// waves scores 16 of its keys for all query heads (S^T = K Q^T), the probabilities go through LDS, then each wave multiplies
-// all 64 keys into its share of the value columns (O^T += V^T P^T, V^T by transposing LDS reads).  With one tensor for keys
+// A tile of 64 keys goes from memory through registers into LDS while the tile before it is multiplied.  Each of four
+// waves scores 16 of its keys for all query heads (S^T = K Q^T; with eight waves, for half of them), the probabilities go
+// through LDS, then each wave multiplies all 64 keys into its share of the value columns (O^T += V^T P^T, V^T by transposing
+// LDS reads).  With one tensor for keys
 // and values (latent attention) the tile is read from memory once for both.
 #include "scored_attn.h"
 
@@ -22,26 +23,31 @@ __device__ __forceinline__ sd_s4 sd_tr(const __bf16 *p) {
     return __builtin_amdgcn_ds_read_tr16_b64_v4i16((sd_s4 __attribute__((address_space(3))) *)p);
 }
 
-// KC, VC: key and value elements held (multiples of 32 and 64).  ONE: values are the keys' first columns.
+// KC, VC: key and value elements held (multiples of 32 and 64).  ONE: values are the keys' first columns.  A workgroup whose
+// tile fills the LDS of a compute unit has eight waves where its queries fill them.
 template <int KC, int VC, bool ONE, int QT> struct SdTile {
+    static constexpr int waves = KC >= 512 && QT > 1 ? 8 : 4, threads = 64 * waves;
     static constexpr int kPitch = KC + 8, vPitch = ONE ? KC + 8 : VC + 8;
     static constexpr int kElems = kSdKeys * kPitch, vElems = ONE ? 0 : kSdKeys * vPitch, qElems = 16 * QT * kPitch;
     static constexpr int pPitch = kSdKeys + 8, pElems = 16 * QT * pPitch;
     static constexpr size_t bytes = (size_t)(kElems + vElems + qElems + pElems) * 2 + 4 * 16 * QT * 4;
 };
 
-template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) void scored_decode_kernel(const ScoredArgs a) {
+template <int KC, int VC, bool ONE, int QT>
+__global__ __launch_bounds__((SdTile<KC, VC, ONE, QT>::threads)) void scored_decode_kernel(const ScoredArgs a) {
     using L = SdTile<KC, VC, ONE, QT>;
-    constexpr int kVT = VC / 64;                                     // value column tiles per wave
-    constexpr int kKL = kSdKeys * KC / 8 / 256, kVL = ONE ? 0 : kSdKeys * VC / 8 / 256;  // 16-byte loads per thread and tile
-    static_assert(kSdKeys * KC / 8 % 256 == 0 && VC % 64 == 0, "whole loads");
+    constexpr int kThr = L::threads, kVT = VC / 16 / L::waves;       // value column tiles per wave
+    constexpr int kTQ = QT * 4 / L::waves;                           // query tiles that a wave scores
+    constexpr int kKL = kSdKeys * KC / 8 / kThr, kVL = ONE ? 0 : kSdKeys * VC / 8 / kThr;  // 16-byte loads per thread and tile
+    static_assert(kSdKeys * KC / 8 % kThr == 0 && VC % (16 * L::waves) == 0 && kTQ > 0, "whole loads");
     extern __shared__ __align__(16) char sd_lds[];
     __bf16 *ks = reinterpret_cast<__bf16 *>(sd_lds), *vs = ONE ? ks : ks + L::kElems;
     __bf16 *qs = ks + L::kElems + L::vElems, *ps = qs + L::qElems;
-    float *tops = reinterpret_cast<float *>(ps + L::pElems);  // [4 waves][16 QT]
+    float *tops = reinterpret_cast<float *>(ps + L::pElems);  // [4 key groups][16 QT]
     const int groups = (a.n_rep + 16 * QT - 1) / (16 * QT);
     const int kvh = blockIdx.x / groups, rep0 = blockIdx.x % groups * 16 * QT, piece = blockIdx.y, b = blockIdx.z;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
+    const int kg = wave & 3, t0 = wave / 4 * kTQ;  // the wave's keys of a tile, its first query tile
     const int pos = a.ctx_lens[b] - 1, h0 = kvh * a.n_rep + rep0, n_heads = min(16 * QT, a.n_rep - rep0);
     if (pos < 0) return;  // padding
     const int first = scored_first_key(a, pos), per = ((pos + 1 - first + a.splits - 1) / a.splits + kSdKeys - 1) / kSdKeys * kSdKeys;
@@ -54,7 +60,7 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
     // ---- queries ----
     const uint16_t *q1 = reinterpret_cast<const uint16_t *>(a.q1) + b * a.q1_row, *q2 = reinterpret_cast<const uint16_t *>(a.q2) + b * a.q2_row;
     uint16_t *qw = reinterpret_cast<uint16_t *>(qs);
-    for (int i = tid; i < 16 * QT * (KC / 8); i += 256) {
+    for (int i = tid; i < 16 * QT * (KC / 8); i += kThr) {
         const int r = i / (KC / 8), e = i % (KC / 8) * 8;
         uint4 x = make_uint4(0, 0, 0, 0);
         if (r < n_heads) {
@@ -74,51 +80,52 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
         const int slots = scored_slot_of(a, id, k0 + lane, end);
 #pragma unroll
         for (int n = 0; n < kKL; ++n) {
-            const int c = tid + 256 * n, s = __shfl(slots, c / (KC / 8), 64), e = c % (KC / 8) * 8;
+            const int c = tid + kThr * n, s = __shfl(slots, c / (KC / 8), 64), e = c % (KC / 8) * 8;
             kr[n] = scored_load16(kp + s * k_tok + e, s >= 0 && e < kreal);
         }
         if constexpr (!ONE) {
 #pragma unroll
             for (int n = 0; n < kVL; ++n) {
-                const int c = tid + 256 * n, s = __shfl(slots, c / (VC / 8), 64), e = c % (VC / 8) * 8;
+                const int c = tid + kThr * n, s = __shfl(slots, c / (VC / 8), 64), e = c % (VC / 8) * 8;
                 vr[n] = scored_load16(vp + s * v_tok + e, s >= 0 && e < vreal);
             }
         }
     };
     sd_f4 o[QT][kVT];
-    float m[QT], l[QT];
+    float m[QT], l[kTQ];
+#pragma unroll
+    for (int t = 0; t < kTQ; ++t) l[t] = 0.f;
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
         m[t] = kScoredNone;
-        l[t] = 0.f;
 #pragma unroll
         for (int c = 0; c < kVT; ++c) o[t][c] = sd_f4{0.f, 0.f, 0.f, 0.f};
     }
     const float to2 = kScoredLog2e, plain = a.scale * kScoredLog2e, cap_in = a.cap > 0.f ? 2.f * plain / a.cap : 0.f  /* tanh(z) = 1 - 2 / (1 + e^(2z)) */, cap_out = a.cap * kScoredLog2e;
-    const float *bias[QT];  // of this lane's heads
+    const float *bias[kTQ];  // of this lane's heads
 #pragma unroll
-    for (int t = 0; t < QT; ++t) bias[t] = a.bias + (int64_t)(h0 + min(16 * t + l16, n_heads - 1)) * a.bias_n;
+    for (int t = 0; t < kTQ; ++t) bias[t] = a.bias + (int64_t)(h0 + min(16 * (t0 + t) + l16, n_heads - 1)) * a.bias_n;
     fetch(id_of(lo), lo);
     int id = id_of(lo + kSdKeys);
     for (int k0 = lo; k0 < end; k0 += kSdKeys) {
 #pragma unroll
         for (int n = 0; n < kKL; ++n) {
-            const int c = tid + 256 * n;
+            const int c = tid + kThr * n;
             *reinterpret_cast<scored_u4 *>(ks + c / (KC / 8) * L::kPitch + c % (KC / 8) * 8) = kr[n];
         }
         if constexpr (!ONE) {
 #pragma unroll
             for (int n = 0; n < kVL; ++n) {
-                const int c = tid + 256 * n;
+                const int c = tid + kThr * n;
                 *reinterpret_cast<scored_u4 *>(vs + c / (VC / 8) * L::vPitch + c % (VC / 8) * 8) = vr[n];
             }
         }
         __syncthreads();
-        const int key = k0 + 16 * wave + 4 * g;
-        float near[QT][4];  // biases: ahead of the next tile's loads, which they do not wait for
+        const int key = k0 + 16 * kg + 4 * g;
+        float near[kTQ][4];  // biases: ahead of the next tile's loads, which they do not wait for
         if (a.bias) {
 #pragma unroll
-            for (int t = 0; t < QT; ++t)
+            for (int t = 0; t < kTQ; ++t)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) near[t][i] = bias[t][min(max(pos - key - i, 0), a.bias_n - 1)];
         }
@@ -126,37 +133,37 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
             fetch(id, k0 + kSdKeys);
             id = id_of(k0 + 2 * kSdKeys);
         }
-        // scores: keys k0 + 16 wave + 4 g + i, head l16 of each query tile
-        sd_f4 s[QT];
+        // scores: keys k0 + 16 wave + 4 g + i, head l16 of its query tiles
+        sd_f4 s[kTQ];
 #pragma unroll
-        for (int t = 0; t < QT; ++t) s[t] = sd_f4{0.f, 0.f, 0.f, 0.f};
-        const __bf16 *ka = ks + (16 * wave + l16) * L::kPitch + 8 * g, *qa = qs + l16 * L::kPitch + 8 * g;
+        for (int t = 0; t < kTQ; ++t) s[t] = sd_f4{0.f, 0.f, 0.f, 0.f};
+        const __bf16 *ka = ks + (16 * kg + l16) * L::kPitch + 8 * g, *qa = qs + (16 * t0 + l16) * L::kPitch + 8 * g;
 #pragma unroll
         for (int kk = 0; kk < KC / 32; ++kk) {
             const sd_bf8 x = sd_read8(ka + 32 * kk);
 #pragma unroll
-            for (int t = 0; t < QT; ++t) s[t] = sd_mfma(x, sd_read8(qa + 16 * t * L::kPitch + 32 * kk), s[t]);
+            for (int t = 0; t < kTQ; ++t) s[t] = sd_mfma(x, sd_read8(qa + 16 * t * L::kPitch + 32 * kk), s[t]);
         }
         if (a.cap > 0.f) {  // (in units of the base-2 exponential)
 #pragma unroll
-            for (int t = 0; t < QT; ++t)
+            for (int t = 0; t < kTQ; ++t)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) s[t][i] = cap_out - 2.f * cap_out * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s[t][i] * cap_in));
         } else {
 #pragma unroll
-            for (int t = 0; t < QT; ++t)
+            for (int t = 0; t < kTQ; ++t)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) s[t][i] *= plain;
         }
         if (a.bias) {
 #pragma unroll
-            for (int t = 0; t < QT; ++t)
+            for (int t = 0; t < kTQ; ++t)
 #pragma unroll
                 for (int i = 0; i < 4; ++i) s[t][i] = fmaf(near[t][i], to2, s[t][i]);
         }
 #pragma unroll
-        for (int t = 0; t < QT; ++t) {
-            const int r = 16 * t + l16;
+        for (int t = 0; t < kTQ; ++t) {
+            const int r = 16 * (t0 + t) + l16;
             float top = kScoredNone;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
@@ -165,7 +172,7 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
             }
             top = fmaxf(top, __shfl_xor(top, 16, 64));
             top = fmaxf(top, __shfl_xor(top, 32, 64));
-            if (g == 0) tops[wave * 16 * QT + r] = top;
+            if (g == 0) tops[kg * 16 * QT + r] = top;
         }
         __syncthreads();
 #pragma unroll
@@ -176,11 +183,14 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
             for (int w = 0; w < 4; ++w) next = fmaxf(next, tops[w * 16 * QT + r]);
             const float keep = __builtin_amdgcn_exp2f(m[t] - next);
             m[t] = next;
-            float p[4];
+            if (kTQ == QT || t / kTQ == wave / 4) {
+                const int own = t % kTQ;
+                float p[4];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) p[i] = __builtin_amdgcn_exp2f(s[t][i] - next);
-            l[t] = fmaf(l[t], keep, (p[0] + p[1]) + (p[2] + p[3]));
-            *reinterpret_cast<uint2 *>(ps + r * L::pPitch + 16 * wave + 4 * g) = make_uint2(row_pack_bf16(p[0], p[1]), row_pack_bf16(p[2], p[3]));
+                for (int i = 0; i < 4; ++i) p[i] = __builtin_amdgcn_exp2f(s[own][i] - next);
+                l[own] = fmaf(l[own], keep, (p[0] + p[1]) + (p[2] + p[3]));
+                *reinterpret_cast<uint2 *>(ps + r * L::pPitch + 16 * kg + 4 * g) = make_uint2(row_pack_bf16(p[0], p[1]), row_pack_bf16(p[2], p[3]));
+            }
 #pragma unroll
             for (int c = 0; c < kVT; ++c)
 #pragma unroll
@@ -206,10 +216,10 @@ template <int KC, int VC, bool ONE, int QT> __global__ __launch_bounds__(256) vo
     }
     // ---- sums over the waves, then out ----
 #pragma unroll
-    for (int t = 0; t < QT; ++t) {
+    for (int t = 0; t < kTQ; ++t) {
         l[t] += __shfl_xor(l[t], 16, 64);
         l[t] += __shfl_xor(l[t], 32, 64);
-        if (g == 0) tops[wave * 16 * QT + 16 * t + l16] = l[t];
+        if (g == 0) tops[kg * 16 * QT + 16 * (t0 + t) + l16] = l[t];
     }
     __syncthreads();
 #pragma unroll
@@ -282,7 +292,7 @@ template <int KC, int VC, bool ONE, int QT> int launch_decode(const ScoredArgs &
         if (e != hipSuccess) return pa_fail(PA_ERR_HIP, "pa_scored_attention: %s", hipGetErrorString(e));
     }
     const int groups = (a.n_rep + 16 * QT - 1) / (16 * QT);
-    scored_decode_kernel<KC, VC, ONE, QT><<<dim3((unsigned)(a.hkv * groups), (unsigned)a.splits, (unsigned)a.batch), dim3(256), lds, s>>>(a);
+    scored_decode_kernel<KC, VC, ONE, QT><<<dim3((unsigned)(a.hkv * groups), (unsigned)a.splits, (unsigned)a.batch), dim3(SdTile<KC, VC, ONE, QT>::threads), lds, s>>>(a);
     PA_CHECK_LAUNCH("pa_scored_attention (decode)");
     if (a.splits > 1) {
         const int64_t grid = ((int64_t)a.batch * a.heads * a.vdim + 255) / 256;
