@@ -262,25 +262,37 @@ __global__ __launch_bounds__((SdTile<KC, VC, ONE, QT>::threads)) void scored_dec
     }
 }
 
-// Pieces of a sequence's keys joined: a thread per (row, head, value column)
-__global__ __launch_bounds__(256) void scored_merge_kernel(const ScoredArgs a, int vc) {
-    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-    const int64_t rh = i / a.vdim;
-    if (rh >= (int64_t)a.batch * a.heads) return;
-    const int d = (int)(i - rh * a.vdim), h = (int)(rh % a.heads);
+// Pieces of a sequence's keys joined: a wave per (row, head), four value columns per lane and turn
+__global__ __launch_bounds__(64) void scored_merge_kernel(const ScoredArgs a, int vc) {
+    const int64_t rh = blockIdx.x;
+    const int h = (int)(rh % a.heads);
     if (a.ctx_lens[rh / a.heads] < 1) return;
-    const float *ml = a.part_ml + rh * a.splits * 2, *po = a.part_o + rh * a.splits * vc + d;
+    const float *ml = a.part_ml + rh * a.splits * 2;
     float m = a.sink ? a.sink[h] * kScoredLog2e : kScoredNone;
     for (int s = 0; s < a.splits; ++s)
         if (ml[2 * s + 1] > 0.f) m = fmaxf(m, ml[2 * s]);
-    float den = a.sink ? __builtin_amdgcn_exp2f(a.sink[h] * kScoredLog2e - m) : 0.f, num = 0.f;
-    for (int s = 0; s < a.splits; ++s) {
-        if (!(ml[2 * s + 1] > 0.f)) continue;  // (a piece without keys wrote no values)
-        const float w = __builtin_amdgcn_exp2f(ml[2 * s] - m);
-        den = fmaf(w, ml[2 * s + 1], den);
-        num = fmaf(w, po[(int64_t)s * vc], num);
+    for (int d = threadIdx.x * 4; d < a.vdim; d += 256) {
+        const float *po = a.part_o + rh * a.splits * vc + d;
+        float den = a.sink ? __builtin_amdgcn_exp2f(a.sink[h] * kScoredLog2e - m) : 0.f;
+        sd_f4 num = sd_f4{0.f, 0.f, 0.f, 0.f};
+        for (int s = 0; s < a.splits; ++s) {
+            if (!(ml[2 * s + 1] > 0.f)) continue;  // (a piece without keys wrote no values)
+            const float w = __builtin_amdgcn_exp2f(ml[2 * s] - m);
+            const sd_f4 x = *reinterpret_cast<const sd_f4 *>(po + (int64_t)s * vc);
+            den = fmaf(w, ml[2 * s + 1], den);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) num[i] = fmaf(w, x[i], num[i]);
+        }
+        pa_bf16 *out = reinterpret_cast<pa_bf16 *>(a.out) + rh * a.vdim + d;
+        const float f = 1.f / den;
+        if (a.vdim % 4 == 0) {
+            *reinterpret_cast<uint2 *>(out) = make_uint2(row_pack_bf16(num[0] * f, num[1] * f), row_pack_bf16(num[2] * f, num[3] * f));
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (d + i < a.vdim) pa_scalar<pa_bf16>::store(out + i, num[i] * f);
+        }
     }
-    pa_scalar<pa_bf16>::store(reinterpret_cast<pa_bf16 *>(a.out) + i, num / den);
 }
 
 template <int KC, int VC, bool ONE, int QT> int launch_decode(const ScoredArgs &a, hipStream_t s) {
@@ -295,8 +307,7 @@ template <int KC, int VC, bool ONE, int QT> int launch_decode(const ScoredArgs &
     scored_decode_kernel<KC, VC, ONE, QT><<<dim3((unsigned)(a.hkv * groups), (unsigned)a.splits, (unsigned)a.batch), dim3(SdTile<KC, VC, ONE, QT>::threads), lds, s>>>(a);
     PA_CHECK_LAUNCH("pa_scored_attention (decode)");
     if (a.splits > 1) {
-        const int64_t grid = ((int64_t)a.batch * a.heads * a.vdim + 255) / 256;
-        scored_merge_kernel<<<dim3((unsigned)grid), dim3(256), 0, s>>>(a, VC);
+        scored_merge_kernel<<<dim3((unsigned)(a.batch * a.heads)), dim3(64), 0, s>>>(a, VC);
         PA_CHECK_LAUNCH("pa_scored_attention (merge)");
     }
     return PA_OK;
