@@ -160,3 +160,9 @@ def test_stretches_hold_the_visible_keys(window):
         assert got == want
     used = new[new >= 0]
     assert sorted(used.tolist()) == list(range(len(slots) // STRETCH_BLOCK))
+
+
+@pytest.mark.parametrize("dim,rot,vdim,made", [(128, 64, 128, (192, 128)), (136, 24, 72, (160, 72)), (24, 8, 40, (40, 40)),
+                                               (64, 16, 128, (128, 128)), (112, 32, 136, (144, 144)), (180, 32, 64, (216, 216))])
+def test_sizes_of_made_keys_and_values(dim, rot, vdim, made):
+    assert LatentSpec(2, dim, rot, vdim, 48, 0.1, None, 100.0).made == made
