@@ -401,9 +401,11 @@ int pa_dequantize_blocks_e4m3(const void *cache, const float *scale, const int32
 #define PA_ACT_SILU 0
 #define PA_ACT_GELU_TANH 1
 #define PA_ACT_NONE 2
+#define PA_ACT_RELU2 3 /* max(z, 0)^2 (pa_bias_act) */
 #define PA_GATE_SIGMOID_LAST 0 /* norm, then sigmoid(gate) */
 #define PA_GATE_SILU_FIRST 1   /* silu(gate), then norm */
 #define PA_GATE_SILU_LAST 2    /* norm, then silu(gate) */
+#define PA_GATE_NONE 3         /* norm only */
 #define PA_GL_SSD 0            /* recurrences of pa_gated_linear */
 #define PA_GL_MLSTM 1
 #define PA_MOE_SIGMOID 0 /* scores of pa_moe_choose */
@@ -418,7 +420,7 @@ int pa_dequantize_blocks_e4m3(const void *cache, const float *scale, const int32
 
 /*
  * Residual sum and norm of one row at a time:
- *     x = table[ids[row]] * table_scale             when ids is given, else x[row]
+ *     x = table[ids[row]] * table_scale             when ids is given (with ids_add, plus x[row]), else x[row]
  *     x += pos_table[positions[row]]                when positions is given (with ids)
  *     x += y                                        when y is given; with y_weight, y / rms(y) * y_weight
  *     out = norm(x) * norm_weight + norm_bias       PA_NORM_LAYER or PA_NORM_RMS; PA_NORM_NONE: x in dtype
@@ -427,11 +429,14 @@ int pa_dequantize_blocks_e4m3(const void *cache, const float *scale, const int32
  * row r comes from residual row row_index[r] (< x_rows).  Ids and indices out of range read as zero rows.
  * With mix_weight (float[rows][mix + 1]) y is a weighted sum of rows, taken in 32-bit: sum over i < mix of
  * mix_weight[row][i] y[row * mix + i], plus mix_weight[row][mix] y_extra[row] when y_extra is given.
- *   x : float[rows][width];  y, y_extra, table, pos_table, out : dtype;  weights and bias : float[width] or NULL;  width <= 16384
+ * Without mix_weight y may have a y_bias, and with y2 it is the sum of two branches, each normed (with y_eps) on its own:
+ * y = y / rms(y) * y_part + y2 / rms(y2) * y2_part, ahead of y_weight's norm.
+ *   x : float[rows][width];  y, y2, y_extra, table, pos_table, out : dtype;  weights and bias : float[width] or NULL;  width <= 16384
  */
 int pa_residual_norm(float *x, const void *y, const float *mix_weight, int mix, const void *y_extra,
-                     const float *y_weight, float y_eps, const int64_t *ids, const void *table, int64_t table_rows,
-                     float table_scale, const int64_t *positions, const void *pos_table, int64_t pos_rows,
+                     const float *y_bias, const void *y2, const float *y_part, const float *y2_part,
+                     const float *y_weight, float y_eps, const int64_t *ids, int ids_add, const void *table,
+                     int64_t table_rows, float table_scale, const int64_t *positions, const void *pos_table, int64_t pos_rows,
                      const int64_t *row_index, int64_t x_rows,
                      const float *norm_weight, const float *norm_bias, float eps, int norm, void *out,
                      int64_t rows, int width, int dtype, void *stream);
@@ -441,6 +446,7 @@ int pa_residual_norm(float *x, const void *y, const float *mix_weight, int mix, 
  *     PA_GATE_SIGMOID_LAST   out = o / rms(o) * weight * sigmoid(gate)
  *     PA_GATE_SILU_FIRST     z = o * silu(gate), out = z / rms(z) * weight
  *     PA_GATE_SILU_LAST      out = o / rms(o) * weight * silu(gate)
+ *     PA_GATE_NONE           out = o / rms(o) * weight                (gate NULL)
  * gate and out rows are gate_stride and out_stride elements apart; weight : float[width].
  */
 int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride, const float *weight, float eps, void *out,
@@ -456,6 +462,10 @@ int pa_softcap(const void *x, float *out, int64_t n, float cap, int dtype, void 
 int pa_glu(const void *gate, int64_t gate_stride, const void *up, int64_t up_stride, const int64_t *ids,
            int64_t up_rows, void *out, int64_t rows, int width, int act, int dtype, void *stream);
 
+/* out = act(x + bias), rows of `width` elements at x_stride; bias : float[width] or NULL. */
+int pa_bias_act(const void *x, int64_t x_stride, const float *bias, void *out, int64_t rows, int width, int act, int dtype,
+                void *stream);
+
 /*
  * out[row][h][0:vdim] = scale * o[row][h][0:vdim] * sigmoid(gate[row][h]): the gate of each head behind attention, and the
  * step from attention's padded rows (d) to packed ones (vdim), out_stride elements apart.  gate NULL: without it.
@@ -465,6 +475,7 @@ int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, float sca
 
 /*
  * From joint projections to attention's operands: row = [q heads | k heads | v heads | anything].
+ *   0. plus bias (float[channels], only without a convolution), when given;
  *   1. causal convolution over time per channel: y_t = sum_j w[j] u_(t - taps + 1 + j), the rows before a portion from
  *      conv_state (the last taps - 1 projected rows of the sequence, updated by the call);
  *      then, with q_norm and k_norm (float[dim]), q and k divided by sqrt(mean over dim of the square + eps) and times
@@ -482,7 +493,7 @@ int pa_head_gate(const void *o, const void *gate, int64_t gate_stride, float sca
  *                 PA_QKV_TILE_ROWS from row 0; NULL with n_tiles = batch: one row per sequence
  *   v_first     : [n_rows][Hkv * vdim] of dtype
  */
-int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_rows, const float *conv_weight, int taps,
+int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_rows, const float *bias, const float *conv_weight, int taps,
                        void *conv_state, int64_t state_rows, const float *rope, int64_t rope_rows, int rot_dims,
                        const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
                        const int32_t *state_slots, const int32_t *tiles, int n_tiles, int batch,
@@ -622,6 +633,40 @@ int pa_scored_attention(const void *q1, int64_t q1_row, int64_t q1_head, int n1,
                         int max_q_len, int num_q_heads, int num_kv_heads, float scale, int window, float softcap,
                         const float *bias, int bias_n, const float *sink, void *out, int dtype, void *workspace,
                         size_t workspace_bytes, void *stream);
+
+/*
+ * Paged attention whose heads' weights are mixed before they meet the values.  For the row at position i, over the visible
+ * keys j <= i:
+ *     s_h(j) = scale q_h . k_j - bias_size[h] ln(1 + bias_rate[h] (i - j))        (bias_size, bias_rate NULL: without)
+ *     p_h = softmax of s_h;  w_h(j) = sum_g talk[h][g] p_g(j);  out_h = sum_j w_h(j) v_j      (v of h's own kv head)
+ * q: head h of row r at r * q_row + h * q_head, dim elements; pools as in pa_scored_attention.  bias_size, bias_rate :
+ * float[Hq]; talk : float[Hq][Hq]; out : [n_rows][Hq][vdim].  Hq <= 128, dim and vdim <= 256.  The workspace
+ * (pa_talking_workspace_bytes, decode: q_lens NULL; max_keys = bt_stride * block_size) holds the sums of every row and head and,
+ * for 16-bit decode steps, the scores and the parts of the output that a sequence's pieces leave; less than that but enough
+ * for the sums runs on the vector units.
+ */
+size_t pa_talking_workspace_bytes(int64_t n_rows, int batch, int num_q_heads, int num_kv_heads, int vdim, int64_t max_keys, int decode);
+int pa_talking_attention(const void *q, int64_t q_row, int64_t q_head, int dim, const void *k_cache, int k_dim, const void *v_cache,
+                         int v_dim, int vdim, const int32_t *block_tables, int64_t bt_stride, int block_size, int64_t num_blocks,
+                         const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts, int64_t n_rows, int batch,
+                         int max_q_len, int num_q_heads, int num_kv_heads, float scale, const float *bias_size,
+                         const float *bias_rate, const float *talk, void *out, int dtype, void *workspace,
+                         size_t workspace_bytes, void *stream);
+
+/*
+ * Linear attention with a forget gate per channel that also decides what is written.  Per head and channel, with act one of
+ * PA_ACT_NONE and PA_ACT_SILU:
+ *     f_t = lower + (1 - lower) sigmoid(forget_t + f_bias);  S_t = diag(f_t) S_(t-1) + (1 - f_t) v_t^T;  o_t = S_t^T act(q_t)
+ *   q, forget, v : rows of dtype at strides of their own;  f_bias (or NULL), lower : float[heads * dim]
+ *   state        : float[state_rows][heads][pad16(dim)][pad16(vdim)]; slots, portions and kernels as in pa_gated_linear
+ *   out          : [n_rows][heads * vdim] of dtype;  dim <= 256, any vdim
+ */
+size_t pa_channel_linear_workspace_bytes(int batch, int num_heads, int dim, int vdim, int max_q_len);
+int pa_channel_linear(const void *q, int64_t q_stride, int q_act, const void *forget, int64_t f_stride, const float *f_bias,
+                      const float *lower, const void *v, int64_t v_stride, int64_t n_rows, float *state, int64_t state_rows,
+                      const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts, const int32_t *state_slots,
+                      int batch, int max_q_len, void *out, int num_heads, int dim, int vdim, int dtype, void *workspace,
+                      size_t workspace_bytes, void *stream);
 
 /*
  * Mixture of experts.  pa_moe_choose, per row over the experts and, behind them, `identity` identity experts (which hand on the

@@ -23,8 +23,8 @@ PA_ERR_HIP = -4
 
 PA_F32, PA_BF16, PA_F16, PA_FP8_E4M3 = 0, 1, 2, 3
 PA_NORM_NONE, PA_NORM_LAYER, PA_NORM_RMS = 0, 1, 2
-PA_ACT_SILU, PA_ACT_GELU_TANH, PA_ACT_NONE = 0, 1, 2
-PA_GATE_SIGMOID_LAST, PA_GATE_SILU_FIRST, PA_GATE_SILU_LAST = 0, 1, 2
+PA_ACT_SILU, PA_ACT_GELU_TANH, PA_ACT_NONE, PA_ACT_RELU2 = 0, 1, 2, 3
+PA_GATE_SIGMOID_LAST, PA_GATE_SILU_FIRST, PA_GATE_SILU_LAST, PA_GATE_NONE = 0, 1, 2, 3
 PA_GL_SSD, PA_GL_MLSTM = 0, 1
 PA_MOE_SIGMOID, PA_MOE_SOFTMAX = 0, 1
 PA_MOE_NO_SHARED, PA_MOE_SHARED_GATED, PA_MOE_SHARED = 0, 1, 2
@@ -93,12 +93,14 @@ SIGNATURES = {
 }
 _p, _i, _l, _f = c_void_p, c_int, c_int64, c_float
 SIGNATURES.update({
-    "pa_residual_norm": (_i, [_p, _p, _p, _i, _p, _p, _f, _p, _p, _l, _f, _p, _p, _l, _p, _l, _p, _p, _f, _i, _p, _l, _i, _i, _p]),
+    "pa_residual_norm": (_i, [_p, _p, _p, _i, _p, _p, _p, _p, _p, _p, _f, _p, _i, _p, _l, _f, _p, _p, _l, _p, _l, _p, _p, _f, _i, _p, _l, _i, _i,
+                              _p]),
+    "pa_bias_act": (_i, [_p, _l, _p, _p, _l, _i, _i, _i, _p]),
     "pa_rms_gate": (_i, [_p, _p, _l, _p, _f, _p, _l, _l, _i, _i, _i, _i, _p]),
     "pa_softcap": (_i, [_p, _p, _l, _f, _i, _p]),
     "pa_glu": (_i, [_p, _l, _p, _l, _p, _l, _p, _l, _i, _i, _i, _p]),
     "pa_head_gate": (_i, [_p, _p, _l, _f, _p, _l, _l, _i, _i, _i, _i, _p]),
-    "pa_qkv_conv_append": (_i, [_p, _l, _l, _p, _i, _p, _l, _p, _l, _i, _p, _p, _p, _p, _p, _i, _i, _p, _l, _p, _p, _p,
+    "pa_qkv_conv_append": (_i, [_p, _l, _l, _p, _p, _i, _p, _l, _p, _l, _i, _p, _p, _p, _p, _p, _i, _i, _p, _l, _p, _p, _p,
                                 _p, _p, _i, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p]),
     "pa_lightning_state_floats": (c_size_t, [_i, _i]),
     "pa_lightning_recurrent": (_i, [_p, _l, _l, _p, _l, _p, _p, _p, _p, _p, _i, _p, _i, _i, _i, _i, _p]),
@@ -121,6 +123,11 @@ SIGNATURES.update({
     "pa_scored_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i, _i, _l, _i]),
     "pa_scored_attention": (_i, [_p, _l, _l, _i, _p, _l, _l, _i, _p, _i, _p, _i, _i, _p, _l, _i, _l, _p, _p, _p, _l, _i, _i, _i, _i,
                                  _f, _i, _f, _p, _i, _p, _p, _i, _p, c_size_t, _p]),
+    "pa_channel_linear_workspace_bytes": (c_size_t, [_i, _i, _i, _i, _i]),
+    "pa_channel_linear": (_i, [_p, _l, _i, _p, _l, _p, _p, _p, _l, _l, _p, _l, _p, _p, _p, _p, _i, _i, _p, _i, _i, _i, _i, _p, c_size_t, _p]),
+    "pa_talking_workspace_bytes": (c_size_t, [_l, _i, _i, _i, _i, _l, _i]),
+    "pa_talking_attention": (_i, [_p, _l, _l, _i, _p, _i, _p, _i, _i, _p, _l, _i, _l, _p, _p, _p, _l, _i, _i, _i, _i, _f, _p, _p, _p, _p, _i,
+                                  _p, c_size_t, _p]),
     "pa_moe_product": (_i, [_p, _l, _i, _p, _l, _i, _i, _p, _p, _l, _i, _i, _i, _p, _i, _i, _p]),
 })
 SIGNATURES["pa_decode_split"] = SIGNATURES["pa_decode_reduce"] = SIGNATURES["pa_decode"]

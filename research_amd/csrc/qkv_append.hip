@@ -17,6 +17,7 @@ constexpr int kThreadsQkv = 256;
 struct QkvArgs {
     const void *u;  // [rows][ldu]: hq * dim of q, hkv * dim of k, hkv * vdim of v, anything
     int64_t ldu;
+    const float *bias;    // [channels], or NULL (only without a convolution)
     const float *conv_w;  // [taps][channels], or NULL (taps == 1)
     void *conv_state;     // [state_rows][taps - 1][channels] of T
     int64_t state_rows;
@@ -134,6 +135,9 @@ __global__ __launch_bounds__(kThreadsQkv) void qkv_append_kernel(const QkvArgs a
     float nw[8];
     row_zero<8>(nw);
     if (norm_w) load8<float, VEC>(norm_w + c0, left, nw);
+    float bias[8];
+    row_zero<8>(bias);
+    if (a.bias) load8<float, VEC>(a.bias + chan, left, bias);
     const int half = a.rot / 2;
     for (int i = i0; i < i1; ++i) {
         const int64_t row = row0 + i;
@@ -144,7 +148,7 @@ __global__ __launch_bounds__(kThreadsQkv) void qkv_append_kernel(const QkvArgs a
             float acc = 0.f;
 #pragma unroll
             for (int j = 0; j < HT; ++j) acc = fmaf(w[j][e], hist[j][e], acc);
-            y[e] = fmaf(w[HT][e], cur[e], acc);
+            y[e] = fmaf(w[HT][e], cur[e], acc + bias[e]);
         }
 #pragma unroll
         for (int j = 0; j + 1 < HT; ++j)
@@ -228,7 +232,7 @@ template <typename T> void launch_qkv_typed(const QkvArgs &a, int n_tiles, bool 
 
 }  // namespace
 
-extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_rows, const float *conv_weight, int taps,
+extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_rows, const float *bias, const float *conv_weight, int taps,
                                   void *conv_state, int64_t state_rows, const float *rope, int64_t rope_rows, int rot_dims,
                                   const int32_t *ctx_lens, const int32_t *q_lens, const int32_t *q_starts,
                                   const int32_t *state_slots, const int32_t *tiles, int n_tiles, int batch,
@@ -245,6 +249,7 @@ extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_row
                "pool_dim=%d must be a multiple of 8 that holds dim=%d and vdim=%d", pool_dim, dim, vdim);
     PA_REQUIRE(rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0, "rot_dims=%d must be even and at most dim=%d", rot_dims, dim);
     PA_REQUIRE(taps >= 1 && (taps == 1 || conv_weight), "taps=%d without convolution weights", taps);
+    PA_REQUIRE(!bias || taps == 1, "a bias ahead of a convolution");
     PA_REQUIRE(v_mode == PA_V_PLAIN || v_mode == PA_V_FIRST || v_mode == PA_V_MIX, "v_mode=%d is unknown", v_mode);
     if (dtype != PA_F32 && dtype != PA_BF16)
         return pa_fail(PA_ERR_UNSUPPORTED, "pa_qkv_conv_append: dtype=%d is not F32 or BF16", dtype);
@@ -264,14 +269,14 @@ extern "C" int pa_qkv_conv_append(const void *u, int64_t u_stride, int64_t n_row
     PA_REQUIRE((q_norm == nullptr) == (k_norm == nullptr), "q_norm and k_norm come together");
     PA_REQUIRE(pa_aligned16(q_out) && pa_aligned16(k_cache) && pa_aligned16(v_cache), "pointers must be 16-byte aligned");
     QkvArgs a{};
-    a.u = u; a.ldu = u_stride; a.conv_w = conv_weight; a.conv_state = taps > 1 ? conv_state : nullptr;
+    a.u = u; a.ldu = u_stride; a.bias = bias; a.conv_w = conv_weight; a.conv_state = taps > 1 ? conv_state : nullptr;
     a.state_rows = state_rows; a.rope = (const float2 *)rope; a.rope_rows = rope_rows;
     a.ctx_lens = ctx_lens; a.q_lens = q_lens; a.q_starts = q_starts; a.state_slots = state_slots; a.tiles = tiles;
     a.slots = slots; a.total_slots = total_slots; a.n_rows = n_rows; a.q_out = q_out; a.k_cache = k_cache;
     a.v_cache = v_cache; a.v_first = v_first; a.lambda = v_lambda; a.v_mode = v_mode; a.batch = batch;
     a.hq = num_q_heads; a.hkv = num_kv_heads; a.dim = dim; a.vdim = vdim; a.d = pool_dim; a.taps = taps; a.rot = rot_dims;
     a.q_norm = q_norm; a.k_norm = k_norm; a.unit_norm = unit_norm; a.eps = eps; a.q_scale = q_scale;
-    const bool vec = dim % 8 == 0 && vdim % 8 == 0 && u_stride % 8 == 0 && pa_aligned16(u) && pa_aligned16(conv_weight) &&
+    const bool vec = dim % 8 == 0 && vdim % 8 == 0 && u_stride % 8 == 0 && pa_aligned16(u) && pa_aligned16(bias) && pa_aligned16(conv_weight) &&
                      pa_aligned16(conv_state) && pa_aligned16(v_first) && pa_aligned16(q_norm) && pa_aligned16(k_norm);
     hipStream_t s = (hipStream_t)stream;
     if (dtype == PA_F32) launch_qkv_typed<float>(a, n_tiles, vec, s);

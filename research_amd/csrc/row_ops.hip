@@ -12,8 +12,12 @@ struct ResidualArgs {
     const float *mix_w;     // [rows][mix + 1]: y = sum of mix_w[i] y[row * mix + i], i < mix, + mix_w[mix] y_extra[row]
     const void *y_extra;    // [rows][width] of T, or NULL: without the last term
     int mix;
+    const float *y_bias;    // added to y, or NULL
+    const void *y2;         // a second branch, [rows][width] of T: y = y / rms(y) y_part + y2 / rms(y2) y2_part, or NULL
+    const float *y_part, *y2_part;
     const float *y_weight;  // RMS norm applied to y before the sum, or NULL
-    const int64_t *ids;     // x starts as table[ids[row]], or NULL
+    const int64_t *ids;     // x starts as table[ids[row]] (ids_add: gets it added), or NULL
+    int ids_add;
     const void *table;
     int64_t table_rows;
     float table_scale;           // on the table's rows
@@ -64,7 +68,19 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualArgs a
 #pragma unroll
             for (int j = 0; j < V; ++j) x[i][j] = fmaf(x[i][j], a.table_scale, p[j]);
         }
-    } else {
+    }
+    if (a.ids && a.ids_add) {
+        const float *src = a.x + row * a.width;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+            const int c = (i * TPR + lane) * V;
+            float old[V];
+            row_zero<V>(old);
+            if (c < a.width) row_load<float, V>(src + c, old);
+#pragma unroll
+            for (int j = 0; j < V; ++j) x[i][j] += old[j];
+        }
+    } else if (!a.ids) {
         const float *src = a.x + (have_x ? xrow : 0) * a.width;
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
@@ -100,6 +116,43 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResidualArgs a
                 const int c = (i * TPR + lane) * V;
                 row_zero<V>(y[i]);
                 if (c < a.width) row_load<T, V>(src + c, y[i]);
+                if (a.y_bias) {
+                    float b[V];
+                    row_zero<V>(b);
+                    if (c < a.width) row_load<float, V>(a.y_bias + c, b);
+#pragma unroll
+                    for (int j = 0; j < V; ++j) y[i][j] += b[j];
+                }
+            }
+        }
+        if (a.y2) {
+            const T *src = reinterpret_cast<const T *>(a.y2) + row * a.width;
+            float z[NV][V], sy = 0.f, sz = 0.f;
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                const int c = (i * TPR + lane) * V;
+                row_zero<V>(z[i]);
+                if (c < a.width) row_load<T, V>(src + c, z[i]);
+#pragma unroll
+                for (int j = 0; j < V; ++j) {
+                    sy = fmaf(y[i][j], y[i][j], sy);
+                    sz = fmaf(z[i][j], z[i][j], sz);
+                }
+            }
+            const float fy = 1.f / sqrtf(row_sum<TPR>(sy, red) / (float)a.width + a.y_eps);
+            const float fz = 1.f / sqrtf(row_sum<TPR>(sz, red) / (float)a.width + a.y_eps);
+#pragma unroll
+            for (int i = 0; i < NV; ++i) {
+                const int c = (i * TPR + lane) * V;
+                float wy[V], wz[V];
+                row_zero<V>(wy);
+                row_zero<V>(wz);
+                if (c < a.width) {
+                    row_load<float, V>(a.y_part + c, wy);
+                    row_load<float, V>(a.y2_part + c, wz);
+                }
+#pragma unroll
+                for (int j = 0; j < V; ++j) y[i][j] = fmaf(y[i][j] * fy, wy[j], z[i][j] * fz * wz[j]);
             }
         }
         if (a.y_weight) {
@@ -192,7 +245,7 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(const RmsGateArgs a) {
     const int64_t trow = a.groups == 1 ? row : row / a.groups;
     const int first = a.groups == 1 ? 0 : (int)(row - trow * a.groups) * a.width;  // column of the group
     const T *src = reinterpret_cast<const T *>(a.o) + row * a.width;
-    const T *gate = reinterpret_cast<const T *>(a.g) + trow * a.ldg + first;
+    const T *gate = a.gate == PA_GATE_NONE ? nullptr : reinterpret_cast<const T *>(a.g) + trow * a.ldg + first;
     float x[NV][V], g[NV][V];
     float ss = 0.f;
 #pragma unroll
@@ -202,7 +255,7 @@ __global__ __launch_bounds__(256) void rms_gate_kernel(const RmsGateArgs a) {
         row_zero<V>(g[i]);
         if (c < a.width) {
             row_load<T, V>(src + c, x[i]);
-            row_load<T, V>(gate + c, g[i]);
+            if (a.gate != PA_GATE_NONE) row_load<T, V>(gate + c, g[i]);
         }
     }
 #pragma unroll
@@ -293,6 +346,40 @@ template <typename T, int V> __global__ __launch_bounds__(256) void head_gate_ke
     row_store<T, V>(reinterpret_cast<T *>(a.out) + row * a.ldo + h * a.vdim + c, o);
 }
 
+struct BiasActArgs {
+    const void *x;  // row stride ldx
+    int64_t ldx;
+    const float *bias;  // [width], or NULL
+    void *out;          // [rows][width]
+    int64_t rows;
+    int width, act;
+};
+
+// out = act(x + bias)
+template <typename T, int V> __global__ __launch_bounds__(256) void bias_act_kernel(const BiasActArgs a) {
+    const int per_row = (a.width + V - 1) / V;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x, row = i / per_row;
+    if (row >= a.rows) return;
+    const int c = (int)(i - row * per_row) * V;
+    float x[V], b[V];
+    row_load<T, V>(reinterpret_cast<const T *>(a.x) + row * a.ldx + c, x);
+    row_zero<V>(b);
+    if (a.bias) {
+        if constexpr (V == 8) {
+            row_load<float, 4>(a.bias + c, b);
+            row_load<float, 4>(a.bias + c + 4, b + 4);
+        } else {
+            row_load<float, V>(a.bias + c, b);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+        const float z = x[j] + b[j], r = fmaxf(z, 0.f);
+        x[j] = a.act == PA_ACT_RELU2 ? r * r : a.act == PA_ACT_SILU ? row_silu<T>(z) : a.act == PA_ACT_GELU_TANH ? row_gelu_tanh<T>(z) : z;
+    }
+    row_store<T, V>(reinterpret_cast<T *>(a.out) + row * a.width + c, x);
+}
+
 // out = cap * tanh(x / cap)
 template <typename T, int V> __global__ __launch_bounds__(256) void softcap_kernel(const void *x, float *out, int64_t n, float cap) {
     const int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * V;
@@ -336,7 +423,8 @@ int check_rows(const char *what, int64_t rows, int width, int dtype) {
 }  // namespace
 
 extern "C" int pa_residual_norm(float *x, const void *y, const float *mix_weight, int mix, const void *y_extra,
-                                const float *y_weight, float y_eps, const int64_t *ids, const void *table,
+                                const float *y_bias, const void *y2, const float *y_part, const float *y2_part,
+                                const float *y_weight, float y_eps, const int64_t *ids, int ids_add, const void *table,
                                 int64_t table_rows, float table_scale, const int64_t *positions, const void *pos_table,
                                 int64_t pos_rows, const int64_t *row_index, int64_t x_rows,
                                 const float *norm_weight, const float *norm_bias, float eps, int norm, void *out,
@@ -348,6 +436,10 @@ extern "C" int pa_residual_norm(float *x, const void *y, const float *mix_weight
     PA_REQUIRE(x || ids, "neither a residual nor an embedding to start from");
     PA_REQUIRE(!ids || table, "ids without a table");
     PA_REQUIRE(!row_index || (x && !y && !ids), "row_index only reads the residual");
+    PA_REQUIRE(!ids_add || (x && ids), "ids_add without a residual or ids");
+    PA_REQUIRE(!y_bias || (y && !mix_weight), "y_bias without a plain y");
+    PA_REQUIRE(!y2 || (y && !mix_weight), "y2 without a plain y");
+    PA_REQUIRE((y2 != nullptr) == (y_part != nullptr) && (y2 != nullptr) == (y2_part != nullptr), "y2, y_part and y2_part come together");
     PA_REQUIRE(!y_weight || y, "y_weight without y");
     PA_REQUIRE(!positions || (ids && pos_table), "positions without ids or a table");
     PA_REQUIRE(!mix_weight || (y && mix > 0), "mix_weight without y");
@@ -356,11 +448,13 @@ extern "C" int pa_residual_norm(float *x, const void *y, const float *mix_weight
     PA_REQUIRE(norm != PA_NORM_NONE || (!norm_weight && !norm_bias), "norm weights without a norm");
     ResidualArgs a{};
     a.x = x; a.y = y; a.mix_w = mix_weight; a.y_extra = y_extra; a.mix = mix; a.y_weight = y_weight; a.ids = ids;
+    a.y_bias = y_bias; a.y2 = y2; a.y_part = y_part; a.y2_part = y2_part; a.ids_add = ids_add;
     a.table = table; a.table_rows = table_rows; a.table_scale = table_scale; a.positions = positions;
     a.pos_table = pos_table; a.pos_rows = pos_rows; a.row_index = row_index; a.x_rows = x_rows; a.w = norm_weight;
     a.b = norm_bias; a.out = out; a.rows = rows; a.width = width; a.norm = norm; a.y_eps = y_eps; a.eps = eps;
     const bool vec4 = width % 4 == 0 && pa_aligned16(x) && pa_aligned16(y) && pa_aligned16(table) && pa_aligned16(out) &&
-                      pa_aligned16(y_extra) && pa_aligned16(pos_table) &&
+                      pa_aligned16(y_extra) && pa_aligned16(pos_table) && pa_aligned16(y_bias) && pa_aligned16(y2) &&
+                      pa_aligned16(y_part) && pa_aligned16(y2_part) &&
                       pa_aligned16(y_weight) && pa_aligned16(norm_weight) && pa_aligned16(norm_bias);
     hipStream_t s = (hipStream_t)stream;
     if (dtype == PA_F32) ROW_DISPATCH(residual_norm_kernel, float, vec4, width, rows, a, s);
@@ -377,14 +471,15 @@ extern "C" int pa_rms_gate(const void *o, const void *gate, int64_t gate_stride,
     const int per = width / groups;
     const int64_t parts = rows * groups;
     if (int rc = check_rows("pa_rms_gate", rows < 0 ? rows : parts, per, dtype)) return rc;
-    PA_REQUIRE(gate_mode >= PA_GATE_SIGMOID_LAST && gate_mode <= PA_GATE_SILU_LAST, "gate_mode=%d is unknown", gate_mode);
+    PA_REQUIRE(gate_mode >= PA_GATE_SIGMOID_LAST && gate_mode <= PA_GATE_NONE, "gate_mode=%d is unknown", gate_mode);
     if (rows == 0) return PA_OK;
-    PA_REQUIRE(o && gate && weight && out, "NULL argument");
+    PA_REQUIRE(o && (gate || gate_mode == PA_GATE_NONE) && weight && out, "NULL argument");
+    if (gate_mode == PA_GATE_NONE) { gate = nullptr; gate_stride = width; }
     PA_REQUIRE(gate_stride >= width, "gate_stride=%lld is shorter than a row", (long long)gate_stride);
     PA_REQUIRE(out_stride >= width, "out_stride=%lld is shorter than a row", (long long)out_stride);
     RmsGateArgs a{o, gate, gate_stride, out_stride, weight, out, parts, per, groups, gate_mode, eps};
     const uintptr_t four = dtype == PA_F32 ? 15u : 7u;  // four elements
-    const bool vec4 = per % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && ((uintptr_t)gate & four) == 0 &&
+    const bool vec4 = per % 4 == 0 && (gate_mode == PA_GATE_NONE || gate_stride % 4 == 0) && out_stride % 4 == 0 && ((uintptr_t)gate & four) == 0 &&
                       ((uintptr_t)out & four) == 0 && pa_aligned16(o) && pa_aligned16(weight);
     hipStream_t s = (hipStream_t)stream;
     if (dtype == PA_F32) ROW_DISPATCH(rms_gate_kernel, float, vec4, per, parts, a, s);
@@ -418,6 +513,33 @@ extern "C" int pa_glu(const void *gate, int64_t gate_stride, const void *up, int
         else glu_kernel<pa_bf16, 1><<<g, blk, 0, s>>>(a);
     }
     PA_CHECK_LAUNCH("pa_glu");
+    return PA_OK;
+}
+
+extern "C" int pa_bias_act(const void *x, int64_t x_stride, const float *bias, void *out, int64_t rows, int width, int act,
+                           int dtype, void *stream) {
+    pa_clear_error();
+    PA_REQUIRE(rows >= 0 && width > 0, "pa_bias_act: rows=%lld / width=%d out of range", (long long)rows, width);
+    PA_REQUIRE(act >= PA_ACT_SILU && act <= PA_ACT_RELU2, "act=%d is unknown", act);
+    if (dtype != PA_F32 && dtype != PA_BF16) return pa_fail(PA_ERR_UNSUPPORTED, "pa_bias_act: dtype=%d is not F32 or BF16", dtype);
+    if (rows == 0) return PA_OK;
+    PA_REQUIRE(x && out, "NULL argument");
+    PA_REQUIRE(x_stride >= width, "x_stride=%lld is shorter than a row", (long long)x_stride);
+    BiasActArgs a{x, x_stride, bias, out, rows, width, act};
+    const int n = dtype == PA_F32 ? 4 : 8;
+    const bool vec = width % n == 0 && x_stride % n == 0 && pa_aligned16(x) && pa_aligned16(bias) && pa_aligned16(out);
+    const int64_t items = rows * (vec ? width / n : width), grid = (items + 255) / 256;
+    PA_REQUIRE(grid <= 0x7fffffff, "pa_bias_act: rows=%lld is too large for one launch", (long long)rows);
+    const dim3 g((unsigned)grid), blk(256);
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == PA_F32) {
+        if (vec) bias_act_kernel<float, 4><<<g, blk, 0, s>>>(a);
+        else bias_act_kernel<float, 1><<<g, blk, 0, s>>>(a);
+    } else {
+        if (vec) bias_act_kernel<pa_bf16, 8><<<g, blk, 0, s>>>(a);
+        else bias_act_kernel<pa_bf16, 1><<<g, blk, 0, s>>>(a);
+    }
+    PA_CHECK_LAUNCH("pa_bias_act");
     return PA_OK;
 }
 

@@ -827,6 +827,24 @@ class HipPagedAttentionBackend:
             ops.scored_attention(q, kc, vc, vdim, step.chunks, step.tables[nd:], out=out, **kw)
         return out
 
+    def attend_talking(self, q: Tensor, layer_idx: int, step: PackedStep, vdim: int, scale: float, talk: Tensor, bias_size: Optional[Tensor],
+                       bias_rate: Optional[Tensor]) -> Tensor:
+        """Attention with mixed heads (``ops.talking_attention``) of packed rows over the pool."""
+        self._require_device(q)
+        kc, vc = self._layer(layer_idx)
+        nd, rows = step.num_decodes, q.shape[0]
+        out = torch.empty((rows, q.shape[1], vdim), dtype=q.dtype, device=q.device)
+        bs = self.config.block_size
+        for part, lo, hi in ((step.decodes, 0, nd), (step.chunks, nd, None)):
+            if part is None:
+                continue
+            r = slice(0, nd) if part is step.decodes else slice(None)
+            tables = step.tables[lo:hi]
+            need = ops.talking_workspace_bytes(q[r].shape[0], part, q.shape[1], kc.shape[1], vdim, tables.shape[1] * bs)
+            ops.talking_attention(q[r], kc, vc, vdim, part, tables, bs, scale, talk, out[r], bias_size, bias_rate,
+                                  workspace=self._scratch_for(need))
+        return out
+
     def attend_packed(self, q: Tensor, layer_idx: int, step: PackedStep, scale: float, window: int) -> Tensor:
         """Attention of packed rows ``q [rows, Hq, D]`` over the pool (their own keys appended already): the decode
         kernel for the sequences that bring one token, the prefill kernels for the portions."""

@@ -16,12 +16,15 @@ another: RMS norms on the sublayers' outputs, chunk attention beside a matrix
 memory in one layer, Mamba-2 layers, mixtures of experts, capped logits.  Vusalix:
 several residual streams with learned mixing, latent attention, attention with
 distance biases and sinks, the gated delta rule, experts beside identity experts.
+Loluzen: norms ahead of and behind every sublayer, a stretch of layers that runs
+several times, attention with mixed heads beside HGRN2, convolved and rotated
+attention, feed-forwards without gates.
 """
 
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import Callable, Dict, Iterable, List, Optional, Tuple, Union
+from typing import Callable, Dict, List, NamedTuple, Optional, Tuple, Union
 
 import torch
 import torch.nn.functional as F
@@ -29,26 +32,45 @@ from torch import Tensor, nn
 
 from .. import ops
 from .attention import CacheConfig, HipPagedAttentionBackend
-from .mixers import (AttentionSpec, BiasedAttention, BiasedAttentionSpec, ConvAttention, DeltaMixer, DeltaSpec, GatedMLP,
-                     LatentAttention, LatentSpec, LightningMixer, LightningSpec, Mamba2Mixer, Mamba2Spec, MlstmSpec,
-                     ParallelMixer, ParallelSpec, RotaryTables, StepRows, TokenSide, YarnScaling, _param, fill)
+from .mixers import (MIXERS, AttentionSpec, BiasedAttentionSpec, DeltaSpec, GatedMLP, Hgrn2Spec, LatentSpec, LightningSpec,
+                     LlamaScaling, Mamba2Spec, MLPSpec, MlstmSpec, ParallelSpec, PlainMLP, RotaryTables, Site, StepRows, TalkingSpec,
+                     TokenSide, YarnScaling, _param, fill)
 from .moe import MoE, MoESpec
 from .types import InferenceContext
 
 
-MixerSpec = Union[AttentionSpec, BiasedAttentionSpec, LatentSpec, LightningSpec, Mamba2Spec, DeltaSpec, ParallelSpec]
+MixerSpec = Union[AttentionSpec, BiasedAttentionSpec, LatentSpec, LightningSpec, Mamba2Spec, DeltaSpec, TalkingSpec, Hgrn2Spec,
+                  ParallelSpec]
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: MixerSpec
-    ff: Union[int, MoESpec, None]  # inner width of a dense feed-forward, experts, None: the layer has none
+    ff: Union[int, MLPSpec, MoESpec, None]  # inner width of a gated feed-forward, one without gates, experts, None: none
 
     @property
     def kv_pool(self) -> Optional[Tuple[int, ...]]:
         """What the layer keeps per token (an entry of ``CacheConfig.layer_kv``), None for a layer without keys."""
         mixer = self.mixer.left if isinstance(self.mixer, ParallelSpec) else self.mixer
         return getattr(mixer, "kv_pool", None)
+
+
+@dataclass(frozen=True)
+class Loop:
+    """Layers ``start .. stop - 1`` run ``times`` times in a row with the same weights, each turn with keys and state of its
+    own; the embedding is added to the residual ahead of every turn but the first."""
+
+    start: int
+    stop: int
+    times: int
+
+
+class Run(NamedTuple):
+    """One pass through a layer."""
+
+    layer: int
+    turn: int
+    again: bool  # the embedding is added ahead of it
 
 
 @dataclass(frozen=True)
@@ -60,6 +82,10 @@ class HybridConfig:
     side_dim: int = 0  # columns per layer of the second embedding, 0: no per-layer token input
     norm: str = "layer"  # "layer" (with biases) | "rms"
     post_norm: bool = False  # the norms are on the sublayers' outputs ("rms"), which read the residual itself
+    both_norms: bool = False  # norms ahead of the sublayers and on their outputs ("rms")
+    norm_offset: float = 0.0  # added to the weights of these norms as they are loaded
+    residual_mult: float = 1.0  # on the normed outputs of sublayers
+    loop: Optional[Loop] = None
     embed_scale: float = 1.0
     positions: int = 0  # rows of a learned position table that the embedding adds, 0: none
     logit_softcap: Optional[float] = None
@@ -74,9 +100,26 @@ class HybridConfig:
             raise ValueError("identity experts are for residual streams")
         if self.post_norm and (self.norm != "rms" or self.side_dim):
             raise ValueError("norms behind the sublayers are RMS norms, without a per-layer token input")
+        if self.both_norms and (self.norm != "rms" or self.post_norm or self.side_dim or self.streams):
+            raise ValueError("norms on both sides of the sublayers are RMS norms of one plain residual")
+        if self.residual_mult != 1.0 and not (self.both_norms or self.post_norm):
+            raise ValueError(f"residual_mult={self.residual_mult} without norms on the sublayers' outputs")
+        if self.loop is not None:
+            if not 0 <= self.loop.start < self.loop.stop <= len(self.layers) or self.loop.times < 1:
+                raise ValueError(f"{self.loop} of {len(self.layers)} layers")
+            if self.streams or self.positions or any(isinstance(l.mixer, AttentionSpec) and l.mixer.v_mix for l in self.layers):
+                raise ValueError("layers that run again are for one plain residual, without learned positions and value mixing")
         mixed = {(l.mixer.kv_heads, l.mixer.vdim) for l in self.layers if isinstance(l.mixer, AttentionSpec) and l.mixer.v_mix}
         if len(mixed) > 1:
             raise ValueError(f"layers that mix values differ in their value heads: {sorted(mixed)}")
+
+    def runs(self) -> List[Run]:
+        """The layers in the order in which they run; each run has its own place in the cache."""
+        loop, n = self.loop or Loop(0, len(self.layers), 1), len(self.layers)
+        runs = [Run(i, 0, False) for i in range(loop.start)]
+        for turn in range(loop.times):
+            runs += [Run(i, turn, turn > 0 and i == loop.start) for i in range(loop.start, loop.stop)]
+        return runs + [Run(i, 0, False) for i in range(loop.stop, n)]
 
     def v_roles(self) -> List[Optional[str]]:
         """Per layer: "first" for the first that mixes values, "mix" for the others that do."""
@@ -88,7 +131,7 @@ class HybridConfig:
 
     def cache_config(self, num_blocks: int, block_size: int, num_state_slots: int, dtype: torch.dtype,
                      device: str) -> CacheConfig:
-        shapes = tuple(l.kv_pool for l in self.layers)
+        shapes = tuple(self.layers[run.layer].kv_pool for run in self.runs())
         typical = next((s for s in shapes if s is not None), (1, 8))
         return CacheConfig(num_layers=len(shapes), num_kv_heads=typical[0], head_dim=typical[1], num_blocks=num_blocks,
                            block_size=block_size, dtype=dtype, device=device, layer_kv=shapes,
@@ -260,17 +303,69 @@ def _vusalix_ff(where: str, mlp: Optional[dict]) -> Optional[MoESpec]:
                    identity=int(router.get("identity") or 0), scores="softmax", group_top=1, correction=True, renormalize=False)
 
 
-class _Norm(nn.Module):
-    """Weights of a norm; the arithmetic is fused into the residual sums.  ``args`` as ``pa_residual_norm`` takes them."""
+def _llama_scaling(where: str, scaling: Optional[dict]) -> Optional[LlamaScaling]:
+    if scaling is None:
+        return None
+    _only(where, scaling, "factor", "original", "low", "high")
+    return LlamaScaling(**{key: float(scaling[key]) for key in ("factor", "original", "low", "high")})
 
-    def __init__(self, cfg: HybridConfig, device) -> None:
+
+def loluzen_config(d: dict) -> HybridConfig:
+    """From the fields of a Loluzen ``config.json``.  Anything it does not know it refuses."""
+    layers = []
+    for i, layer in enumerate(d["layers"]):
+        m, mlp, at = layer["mixer"], layer.get("mlp"), f"layer {i} mixer"
+        _only(f"layer {i}", layer, "type", "mixer", "mlp")
+        if layer["type"] == "attention":
+            _only(at, m, "heads", "kv_heads", "dim", "vdim", "conv", "rot", "scale")
+            rot = m.get("rot") or {}
+            _only(at + ".rot", rot, "base", "dims", "scaling")
+            mixer: MixerSpec = AttentionSpec(
+                heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), scale=float(m["scale"]),
+                window=None, taps=int(m.get("conv") or 0), rot_dims=int(rot.get("dims", 0)), rot_base=float(rot.get("base", 1.0)),
+                rot_llama=_llama_scaling(at + ".rot.scaling", rot.get("scaling")), qk_weights=True)
+        elif layer["type"] == "parallel":
+            _only(at, m, "left", "right")
+            left, right = m["left"], m["right"]
+            _only(at + ".left", left, "heads", "kv_heads", "dim", "vdim", "scale")
+            _only(at + ".right", right, "heads", "dim", "vdim")
+            mixer = ParallelSpec(
+                left=TalkingSpec(heads=int(left["heads"]), kv_heads=int(left["kv_heads"]), dim=int(left["dim"]), vdim=int(left["vdim"]),
+                                 scale=float(left["scale"])),
+                right=Hgrn2Spec(heads=int(right["heads"]), dim=int(right["dim"]), vdim=int(right["vdim"])),
+                left_scale=0.5, right_scale=0.5, norms=True)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}")
+        if mlp is not None:
+            _only(f"layer {i} mlp", mlp, "kind", "ff")
+            if mlp["kind"] != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+        layers.append(LayerSpec(mixer, MLPSpec(int(mlp["ff"]), "relu2") if mlp is not None else None))
+    _only("norm", d["norm"], "eps")
+    embedding, loop = d.get("embedding") or {}, d.get("loop")
+    _only("embedding", embedding, "scale")
+    if loop is not None:
+        _only("loop", loop, "start", "stop", "times")
+        loop = Loop(*(int(loop[key]) for key in ("start", "stop", "times")))
+    return HybridConfig(vocab_size=int(d["vocab"]), width=int(d["width"]), layers=tuple(layers), norm_eps=float(d["norm"]["eps"]),
+                        norm="rms", both_norms=True, norm_offset=1.0, residual_mult=float(d.get("residual_mult", 1.0)),
+                        embed_scale=float(embedding.get("scale", 1.0)), loop=loop)
+
+
+class _Norm(nn.Module):
+    """Weights of a norm, ``scale`` times what is loaded plus the config's offset; the arithmetic is fused into the residual
+    sums.  ``args`` as ``pa_residual_norm`` takes them."""
+
+    def __init__(self, cfg: HybridConfig, device, scale: float = 1.0) -> None:
         super().__init__()
+        self.offset, self.scale = cfg.norm_offset, scale
         self.w = _param(cfg.width, dtype=torch.float32, device=device)
         self.b = _param(cfg.width, dtype=torch.float32, device=device) if cfg.norm == "layer" else None
         self.args = dict(norm=cfg.norm, weight=self.w, bias=self.b, eps=cfg.norm_eps)
 
     def load(self, get, name: str) -> None:
         fill(self.w, get(name), name)
+        self.w.add_(self.offset).mul_(self.scale)
         if self.b is not None:
             fill(self.b, get(name + ".b"), name + ".b")
 
@@ -292,33 +387,23 @@ class _Streams(nn.Module):
 
 
 class _HybridLayer(nn.Module):
-    def __init__(self, cfg: HybridConfig, i: int, backend: HipPagedAttentionBackend, rotary: RotaryTables,
-                 v_role: Optional[str], dtype: torch.dtype, device) -> None:
+    def __init__(self, cfg: HybridConfig, i: int, site: Site) -> None:
         super().__init__()
-        spec = cfg.layers[i]
-        self.norm1 = _Norm(cfg, device)
-        if isinstance(spec.mixer, AttentionSpec):
-            self.mixer = ConvAttention(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, v_role, dtype, device)
-        elif isinstance(spec.mixer, ParallelSpec):
-            self.mixer = ParallelMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, dtype, device)
-        elif isinstance(spec.mixer, BiasedAttentionSpec):
-            self.mixer = BiasedAttention(spec.mixer, cfg.width, i, backend, dtype, device)
-        elif isinstance(spec.mixer, LatentSpec):
-            self.mixer = LatentAttention(spec.mixer, cfg.width, cfg.norm_eps, i, backend, rotary, dtype, device)
-        elif isinstance(spec.mixer, DeltaSpec):
-            self.mixer = DeltaMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
-        elif isinstance(spec.mixer, Mamba2Spec):
-            self.mixer = Mamba2Mixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
-        else:
-            self.mixer = LightningMixer(spec.mixer, cfg.width, cfg.norm_eps, i, backend, dtype, device)
-        self.norm2 = self.mlp = self.side = self.streams1 = self.streams2 = None
+        spec, dtype, device = cfg.layers[i], site.dtype, site.device
+        behind = lambda: _Norm(cfg, device, cfg.residual_mult)
+        norm = behind if cfg.post_norm else lambda: _Norm(cfg, device)
+        self.norm1, self.norm1b = norm(), behind() if cfg.both_norms else None
+        self.mixer = MIXERS[type(spec.mixer)](spec.mixer, site)
+        self.norm2 = self.norm2b = self.mlp = self.side = self.streams1 = self.streams2 = None
         if cfg.streams:
             self.streams1 = _Streams(cfg.streams, device)
             self.streams2 = _Streams(cfg.streams, device) if spec.ff is not None else None
         if spec.ff is not None:
-            self.norm2 = _Norm(cfg, device)
-            self.mlp = (MoE(spec.ff, cfg.width, dtype, device) if isinstance(spec.ff, MoESpec)
-                        else GatedMLP(cfg.width, spec.ff, dtype, device))
+            self.norm2, self.norm2b = norm(), behind() if cfg.both_norms else None
+            if isinstance(spec.ff, MoESpec):
+                self.mlp = MoE(spec.ff, cfg.width, dtype, device)
+            else:
+                self.mlp = (PlainMLP if isinstance(spec.ff, MLPSpec) else GatedMLP)(cfg.width, spec.ff, dtype, device)
         if cfg.side_dim:
             self.side = TokenSide(cfg.width, cfg.side_dim, i, dtype, device)
 
@@ -328,6 +413,9 @@ class _HybridLayer(nn.Module):
         if self.mlp is not None:
             self.norm2.load(get, prefix + "norm2")
             self.mlp.load(get, prefix + "mlp.")
+        for behind, name in ((self.norm1b, "norm1b"), (self.norm2b, "norm2b")):
+            if behind is not None:
+                behind.load(get, prefix + name)
         if self.side is not None:
             self.side.load(get, prefix + "side.")
         for streams, name in ((self.streams1, "hc1."), (self.streams2, "hc2.")):
@@ -354,7 +442,9 @@ class HybridDecoder(nn.Module):
         self.side_embed = None
         if cfg.side_dim:
             self.side_embed = _param(cfg.vocab_size, cfg.side_dim * len(cfg.layers), dtype=dtype, device=device)
-        self.layers = nn.ModuleList(_HybridLayer(cfg, i, backend, self.rotary, role, dtype, device)
+        self.runs = cfg.runs()
+        places = lambda i: tuple(at for at, run in enumerate(self.runs) if run.layer == i)
+        self.layers = nn.ModuleList(_HybridLayer(cfg, i, Site(cfg.width, cfg.norm_eps, places(i), backend, self.rotary, dtype, device, role))
                                     for i, role in enumerate(cfg.v_roles()))
         self.norm = _Norm(cfg, device)
         self.head = _param(cfg.vocab_size, cfg.width, dtype=dtype, device=device)
@@ -389,7 +479,7 @@ class HybridDecoder(nn.Module):
     # ------------------------------------------------------------------ forward
     def forward(self, input_ids: Tensor, positions: Optional[Tensor], ctx: InferenceContext,
                 trace: Optional[List[Tensor]] = None) -> Tensor:
-        """``trace`` collects a copy of the residual after every layer."""
+        """``trace`` collects a copy of the residual after every run of a layer."""
         ids = input_ids.reshape(-1)
         packed = self.backend.packed_step(ctx)
         if packed.num_rows != ids.numel():
@@ -407,13 +497,16 @@ class HybridDecoder(nn.Module):
             pending.update(positions=positions.reshape(-1), pos_table=self.pos_embed)
         # a norm's weights either with the sum that a sublayer reads, or with the sublayer's output as it is added
         ahead = (lambda norm: {}) if cfg.post_norm else (lambda norm: norm.args)
-        behind = (lambda norm: {"y_weight": norm.w, "y_eps": eps}) if cfg.post_norm else (lambda norm: {})
-        for layer in self.layers:
+        behind = lambda norm: {} if norm is None else {"y_weight": norm.w, "y_eps": eps}
+        for i, step.turn, again in self.runs:
+            layer = self.layers[i]
+            if again:
+                pending = {**pending, "ids": ids, "table": self.embed, "table_scale": cfg.embed_scale, "ids_add": True}
             h = ops.residual_norm(x, dtype, **pending, **ahead(layer.norm1))
-            pending = {"y": layer.mixer(h, step), **behind(layer.norm1)}
+            pending = {**layer.mixer.branch(h, step), **behind(layer.norm1 if cfg.post_norm else layer.norm1b)}
             if layer.mlp is not None:
                 h = ops.residual_norm(x, dtype, **pending, **ahead(layer.norm2))
-                pending = {**layer.mlp.branch(h), **behind(layer.norm2)}
+                pending = {**layer.mlp.branch(h), **behind(layer.norm2 if cfg.post_norm else layer.norm2b)}
             if layer.side is not None:
                 h = ops.residual_norm(x, dtype, **pending)
                 pending = {"y": layer.side(h, ids, self.side_embed), "y_weight": layer.side.norm, "y_eps": eps}

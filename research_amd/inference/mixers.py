@@ -22,15 +22,24 @@ product and everything between the products into one or two kernels:
 * ``LatentAttention``: joint projection -> ``pa_latent_append``; decoded tokens
   attend to the cached latents themselves (``pa_scored_attention`` between two
   products per head), portions to keys and values made again from them;
-* ``ParallelMixer``: two of them side by side with one joint input and one joint
-  output projection; their scales ride on the steps before the latter.
+* ``TalkingAttention``: joint projection -> ``pa_qkv_conv_append`` (biases, append)
+  -> ``pa_talking_attention`` (distance bias, heads' weights mixed) ->
+  ``pa_head_gate`` -> output projection;
+* ``Hgrn2Mixer``: joint projection -> ``pa_channel_linear`` (gates, recurrence) ->
+  ``pa_rms_gate`` per head without a gate -> output projection;
+* ``ParallelMixer``: two of them side by side with one joint input projection and
+  one joint output projection (their scales ride on the steps before the latter)
+  or, where each side's output is normed on its own, one of each side's.
+
+A layer that runs several times with the same weights keeps keys and state per
+turn: a mixer's ``Site`` names one place in the cache for each of its turns.
 """
 
 from __future__ import annotations
 
 import math
 from dataclasses import dataclass
-from typing import Callable, Dict, List, Optional, Tuple
+from typing import Callable, Dict, List, Optional, Tuple, Union
 
 import torch
 import torch.nn.functional as F
@@ -57,6 +66,20 @@ class YarnScaling:
 
 
 @dataclass(frozen=True)
+class LlamaScaling:
+    """Rotary frequencies by their wavelength: those shorter than ``original / high`` positions keep theirs, those longer than
+    ``original / low`` are divided by ``factor``, with a ramp in the number of waves between."""
+
+    factor: float
+    original: float
+    low: float
+    high: float
+
+
+RotaryScaling = Union[YarnScaling, LlamaScaling]
+
+
+@dataclass(frozen=True)
 class AttentionSpec:
     """Softmax attention over a sliding window behind short convolutions.  ``window`` and ``chunk`` None: plain causal;
     ``chunk``: keys of the query's own chunk of positions; ``taps`` 0: no convolution; ``v_mix``: the layer takes part in
@@ -79,6 +102,7 @@ class AttentionSpec:
     rot_halves: bool = False
     qk_weights: bool = False
     gates: bool = True
+    rot_llama: Optional[LlamaScaling] = None
 
     def __post_init__(self) -> None:
         if self.heads % self.kv_heads != 0:
@@ -295,13 +319,54 @@ class Mamba2Spec:
 
 
 @dataclass(frozen=True)
-class ParallelSpec:
-    """Attention and a recurrent mixer on the same input, their outputs added under two scales."""
+class TalkingSpec:
+    """Softmax attention without rotation whose scores lose ``r1 ln(1 + r2 distance)`` per head and whose heads' weights are
+    mixed by a matrix before they meet the values; biases in the projections, a gate per head."""
 
-    left: AttentionSpec
-    right: MlstmSpec
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+
+    def __post_init__(self) -> None:
+        if self.heads % self.kv_heads != 0:
+            raise ValueError(f"heads={self.heads} is not a multiple of kv_heads={self.kv_heads}")
+        if max(self.dim, self.vdim) > 256 or self.heads > 128:
+            raise ValueError(f"dim={self.dim} or vdim={self.vdim} above 256, or heads={self.heads} above 128")
+
+    @property
+    def kv_pool(self) -> Tuple[int, ...]:
+        return self.kv_heads, _pad8(max(self.dim, self.vdim))
+
+    @property
+    def channels(self) -> int:
+        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+
+@dataclass(frozen=True)
+class Hgrn2Spec:
+    """Linear attention with a forget gate per channel, bounded from below, whose complement is the key."""
+
+    heads: int
+    dim: int
+    vdim: int
+
+    def __post_init__(self) -> None:
+        if self.dim > 256:
+            raise ValueError(f"dim={self.dim} above 256")
+
+
+@dataclass(frozen=True)
+class ParallelSpec:
+    """Attention and a recurrent mixer on the same input.  Their outputs are added under two scales; ``norms``: each first
+    RMS-normed with a weight of its own."""
+
+    left: Union[AttentionSpec, TalkingSpec]
+    right: Union[MlstmSpec, Hgrn2Spec]
     left_scale: float = 1.0
     right_scale: float = 1.0
+    norms: bool = False
 
 
 def yarn_frequencies(base: float, dims: int, yarn: YarnScaling) -> Tuple[Tensor, float]:
@@ -316,6 +381,15 @@ def yarn_frequencies(base: float, dims: int, yarn: YarnScaling) -> Tuple[Tensor,
     return freq / yarn.factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(yarn.factor) + 1.0
 
 
+def llama_frequencies(base: float, dims: int, s: LlamaScaling) -> Tensor:
+    """float64 frequencies of the ``dims / 2`` pairs."""
+    freq = base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims)
+    length = 2 * math.pi / freq
+    part = (s.original / length - s.low) / (s.high - s.low) if s.high != s.low else torch.zeros_like(freq)
+    between = (1 - part) * freq / s.factor + part * freq
+    return torch.where(length < s.original / s.high, freq, torch.where(length > s.original / s.low, freq / s.factor, between))
+
+
 class RotaryTables:
     """(cos, sin) per position and pair, float32 from float64 angles; one table per (base, dims, factor, scaling), shared by
     the layers that name it.  The position limit is fixed once a captured graph may hold a table's address."""
@@ -325,14 +399,16 @@ class RotaryTables:
         self.device = device
         self._tables: Dict[tuple, Tensor] = {}
 
-    def get(self, base: float, dims: int, factor: float, yarn: Optional[YarnScaling] = None) -> Optional[Tensor]:
+    def get(self, base: float, dims: int, factor: float, scaling: Optional[RotaryScaling] = None) -> Optional[Tensor]:
         if dims == 0:
             return None
-        key = (base, dims, factor, yarn)
+        key = (base, dims, factor, scaling)
         if key not in self._tables:
             freq, size = base ** (-torch.arange(0, dims, 2, dtype=torch.float64) / dims), 1.0
-            if yarn is not None:
-                freq, size = yarn_frequencies(base, dims, yarn)
+            if isinstance(scaling, YarnScaling):
+                freq, size = yarn_frequencies(base, dims, scaling)
+            elif scaling is not None:
+                freq = llama_frequencies(base, dims, scaling)
             angle = torch.arange(self.max_positions, dtype=torch.float64)[:, None] * (freq / factor)[None, :]
             table = (torch.stack([angle.cos(), angle.sin()], dim=-1) * size).float()
             self._tables[key] = table.contiguous().to(self.device)
@@ -346,6 +422,31 @@ class StepRows:
     packed: PackedStep
     ids: Tensor
     v_first: Optional[Tensor] = None
+    turn: int = 0  # how often the layer has run already
+
+
+@dataclass(frozen=True)
+class Site:
+    """Where a mixer lives: the model's width, norm constant and types, and the layer's place in the cache for each turn."""
+
+    width: int
+    eps: float
+    places: Tuple[int, ...]
+    backend: HipPagedAttentionBackend
+    rotary: RotaryTables
+    dtype: torch.dtype
+    device: Union[str, torch.device]
+    v_role: Optional[str] = None  # None, "first" (the layer whose values the others mix in) or "mix"
+
+    def weight(self, *shape: int) -> nn.Parameter:
+        return _param(*shape, dtype=self.dtype, device=self.device)
+
+    def constant(self, *shape: int) -> nn.Parameter:
+        return _param(*shape, dtype=torch.float32, device=self.device)
+
+    def keep(self, name: str, shape: Tuple[int, ...], dtype: torch.dtype, when: bool = True) -> List[Optional[Tensor]]:
+        """State per sequence: a tensor for each turn, or, without one, None for each."""
+        return [self.backend.register_state(at, name, shape, dtype) if when else None for at in self.places]
 
 
 def _param(*shape: int, dtype: torch.dtype, device) -> nn.Parameter:
@@ -362,6 +463,10 @@ def _pad8(n: int) -> int:
     return -(-n // 8) * 8
 
 
+def _pad16(n: int) -> int:
+    return -(-n // 16) * 16
+
+
 Slices = Optional[Tuple[Tensor, Tensor]]
 
 
@@ -370,12 +475,11 @@ class Mixer(nn.Module):
     the two weights; a mixer that is part of another is handed its slices of that one's weights.  ``out_scale`` multiplies
     what ``mix`` returns."""
 
-    def __init__(self, in_rows: int, out_cols: int, width: int, dtype: torch.dtype, device, slices: Slices = None,
-                 out_scale: float = 1.0) -> None:
+    def __init__(self, in_rows: int, out_cols: int, site: Site, slices: Slices = None, out_scale: float = 1.0) -> None:
         super().__init__()
-        self.out_scale = out_scale
+        self.site, self.backend, self.eps, self.out_scale = site, site.backend, site.eps, out_scale
         if slices is None:
-            slices = _param(in_rows, width, dtype=dtype, device=device), _param(width, out_cols, dtype=dtype, device=device)
+            slices = site.weight(in_rows, site.width), site.weight(site.width, out_cols)
         self.w_in, self.w_out = slices
 
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
@@ -384,29 +488,26 @@ class Mixer(nn.Module):
     def forward(self, h: Tensor, step: StepRows) -> Tensor:
         return F.linear(self.mix(F.linear(h, self.w_in), step), self.w_out)
 
+    def branch(self, h: Tensor, step: StepRows) -> Dict[str, object]:
+        """What the residual sum adds, as ``ops.residual_norm`` takes it."""
+        return {"y": self(h, step)}
+
 
 class ConvAttention(Mixer):
     @staticmethod
     def sizes(spec: AttentionSpec) -> Tuple[int, int]:
         return _pad8(spec.channels + (spec.heads if spec.gates else 0)), spec.heads * spec.v_slices * spec.slice_dim
 
-    def __init__(self, spec: AttentionSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 rotary: RotaryTables, v_role: Optional[str], dtype: torch.dtype, device, slices: Slices = None,
-                 out_scale: float = 1.0) -> None:
-        """``v_role``: None, "first" (the layer whose values the others mix in) or "mix".  Rows of ``w_in``: q, k, v, head
-        gates, padding."""
-        super().__init__(*self.sizes(spec), width, dtype, device, slices, out_scale)
-        self.spec, self.eps, self.layer_idx, self.backend, self.v_role = spec, eps, layer_idx, backend, v_role
-        self.rotary = rotary
+    def __init__(self, spec: AttentionSpec, site: Site, slices: Slices = None, out_scale: float = 1.0) -> None:
+        """Rows of ``w_in``: q, k, v, head gates, padding."""
+        super().__init__(*self.sizes(spec), site, slices, out_scale)
+        self.spec, self.v_role = spec, site.v_role
         self.q_norm = self.k_norm = None
         if spec.qk_weights:
-            self.q_norm = _param(spec.dim, dtype=torch.float32, device=device)
-            self.k_norm = _param(spec.dim, dtype=torch.float32, device=device)
-        self.conv = _param(spec.taps, spec.channels, dtype=torch.float32, device=device) if spec.taps else None
-        self.v_lambda = _param(1, dtype=torch.float32, device=device)
-        self.conv_state = None
-        if spec.taps > 1:
-            self.conv_state = backend.register_state(layer_idx, "conv", (spec.taps - 1, spec.channels), dtype)
+            self.q_norm, self.k_norm = site.constant(spec.dim), site.constant(spec.dim)
+        self.conv = site.constant(spec.taps, spec.channels) if spec.taps else None
+        self.v_lambda = site.constant(1)
+        self.conv_state = site.keep("conv", (spec.taps - 1, spec.channels), site.dtype, spec.taps > 1)
 
     def load(self, get: Getter, prefix: str) -> None:
         s, at = self.spec, 0
@@ -466,29 +567,28 @@ class ConvAttention(Mixer):
         s, packed = self.spec, step.packed
         if self.v_role == "first":
             step.v_first = torch.empty((u.shape[0], s.kv_heads * s.vdim), dtype=u.dtype, device=u.device)
-        kc, vc = self.backend._layer(self.layer_idx)
+        place = self.site.places[step.turn]
+        kc, vc = self.backend._layer(place)
         # q carries scale * log2(e) from its 32-bit registers, so that the attention kernels' own factor is one
         q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads * s.v_slices, s.dim, s.slice_dim, s.scale / _LN2, self.eps,
-                                not s.qk_weights, self.rotary.get(s.rot_base, s.rot_dims, s.rot_factor, s.rot_yarn), s.rot_dims,
-                                self.conv, self.conv_state, self.v_role, step.v_first if self.v_role else None,
+                                not s.qk_weights, self.site.rotary.get(s.rot_base, s.rot_dims, s.rot_factor, s.rot_yarn or s.rot_llama),
+                                s.rot_dims, self.conv, self.conv_state[step.turn], self.v_role, step.v_first if self.v_role else None,
                                 self.v_lambda if self.v_role == "mix" else None, q_norm=self.q_norm, k_norm=self.k_norm)
-        o = self.backend.attend_packed(q, self.layer_idx, packed, _LN2, s.mask_window)
+        o = self.backend.attend_packed(q, place, packed, _LN2, s.mask_window)
         gate = u[:, s.channels: s.channels + s.heads] if s.gates else None
         return ops.head_gate(o, gate, s.slice_dim, self.out_scale, out)
 
 
 class LightningMixer(Mixer):
-    def __init__(self, spec: LightningSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 dtype: torch.dtype, device) -> None:
+    def __init__(self, spec: LightningSpec, site: Site) -> None:
+        """Rows of ``w_in``: q, k, v, output gate, padding."""
         inner = spec.heads * spec.vdim
-        # (rows of w_in: q, k, v, output gate, padding)
-        super().__init__(_pad8(spec.heads * 2 * spec.dim + 2 * inner), inner, width, dtype, device)
-        self.spec, self.eps, self.backend = spec, eps, backend
-        self.norm = _param(inner, dtype=torch.float32, device=device)
-        pad = lambda n: -(-n // 16) * 16
-        self.state = backend.register_state(layer_idx, "lightning", (spec.heads, pad(spec.dim), pad(spec.vdim)), torch.float32)
+        super().__init__(_pad8(spec.heads * 2 * spec.dim + 2 * inner), inner, site)
+        self.spec = spec
+        self.norm = site.constant(inner)
+        self.state = site.keep("lightning", (spec.heads, _pad16(spec.dim), _pad16(spec.vdim)), torch.float32)
         powers = torch.tensor(spec.decay, dtype=torch.float64)[:, None] ** torch.arange(DECAY_POWERS, dtype=torch.float64)
-        self.register_buffer("decay_powers", powers.float().to(device).contiguous(), persistent=False)
+        self.register_buffer("decay_powers", powers.float().to(site.device).contiguous(), persistent=False)
 
     def load(self, get: Getter, prefix: str) -> None:
         s, at = self.spec, 0
@@ -499,16 +599,16 @@ class LightningMixer(Mixer):
         fill(self.norm, get(prefix + "norm"), prefix + "norm")
 
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
-        s, packed = self.spec, step.packed
+        s, packed, state = self.spec, step.packed, self.state[step.turn]
         inner = s.heads * s.vdim
         o = torch.empty((u.shape[0], inner), dtype=u.dtype, device=u.device)
         nd = packed.num_decodes
         if packed.decodes is not None:
-            ops.lightning(u[:nd], packed.decodes, self.state, self.decay_powers, s.heads, s.dim, s.vdim, o[:nd])
+            ops.lightning(u[:nd], packed.decodes, state, self.decay_powers, s.heads, s.dim, s.vdim, o[:nd])
         if packed.chunks is not None:
             c = packed.chunks
             need = ops.lightning_workspace_bytes(c.ctx_lens.numel(), s.heads, s.dim, s.vdim, c.max_q_len)
-            ops.lightning(u, c, self.state, self.decay_powers, s.heads, s.dim, s.vdim, o,
+            ops.lightning(u, c, state, self.decay_powers, s.heads, s.dim, s.vdim, o,
                           workspace=self.backend._scratch_for(need) if need else None)
         g = 2 * s.heads * s.dim + inner
         return ops.rms_gate(o, u[:, g: g + inner], self.norm, self.eps, out=out)
@@ -539,16 +639,14 @@ class MlstmMixer(Mixer):
         inner = spec.heads * spec.vdim
         return _pad8(2 * spec.heads * spec.dim + 2 * inner + 2 * spec.heads), inner
 
-    def __init__(self, spec: MlstmSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 dtype: torch.dtype, device, slices: Slices = None, out_scale: float = 1.0) -> None:
+    def __init__(self, spec: MlstmSpec, site: Site, slices: Slices = None, out_scale: float = 1.0) -> None:
         """Rows of ``w_in``: q, k, v, output gate, input gates, forget gates, padding."""
-        super().__init__(*self.sizes(spec), width, dtype, device, slices, out_scale)
-        self.spec, self.eps, self.backend = spec, eps, backend
-        self.norm = _param(spec.heads * spec.vdim, dtype=torch.float32, device=device)  # times out_scale
-        self.i_bias = _param(spec.heads, dtype=torch.float32, device=device)
-        self.f_bias = _param(spec.heads, dtype=torch.float32, device=device)
+        super().__init__(*self.sizes(spec), site, slices, out_scale)
+        self.spec = spec
+        self.norm = site.constant(spec.heads * spec.vdim)  # times out_scale
+        self.i_bias, self.f_bias = site.constant(spec.heads), site.constant(spec.heads)
         floats = ops.gated_linear_state_floats("mlstm", spec.dim, spec.vdim)
-        self.state = backend.register_state(layer_idx, "mlstm", (spec.heads, floats), torch.float32)
+        self.state = site.keep("mlstm", (spec.heads, floats), torch.float32)
 
     def _parts(self) -> Tuple[Tuple[str, int], ...]:
         s = self.spec
@@ -570,27 +668,22 @@ class MlstmMixer(Mixer):
         s = self.spec
         sizes = [n for _, n in self._parts()]
         q, k, v, g, i, f = u[:, : sum(sizes)].split(sizes, dim=1)
-        o = _gated_rows("mlstm", q, k, v, (i, f), (self.i_bias, self.f_bias, None), step, self.state, s.heads, s.dim, s.vdim,
+        o = _gated_rows("mlstm", q, k, v, (i, f), (self.i_bias, self.f_bias, None), step, self.state[step.turn], s.heads, s.dim, s.vdim,
                         self.backend, cap=s.gate_cap, q_scale=s.dim ** -0.5, den_eps=self.DEN_EPS)
         return ops.rms_gate(o, g, self.norm, self.eps, groups=s.heads, out=out)
 
 
 class Mamba2Mixer(Mixer):
-    def __init__(self, spec: Mamba2Spec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 dtype: torch.dtype, device) -> None:
+    def __init__(self, spec: Mamba2Spec, site: Site) -> None:
         """Rows of ``w_in``: gate, x, B, C, step sizes, padding."""
-        super().__init__(_pad8(spec.inner + spec.channels + spec.heads), spec.inner, width, dtype, device)
-        self.spec, self.eps, self.backend = spec, eps, backend
-        f32 = dict(dtype=torch.float32, device=device)
-        self.conv = _param(spec.taps, spec.channels, **f32)
-        self.conv_bias = _param(spec.channels, **f32)
-        self.dt_bias, self.rate, self.skip = (_param(spec.heads, **f32) for _ in range(3))
-        self.norm = _param(spec.inner, **f32)
-        self.conv_state = None
-        if spec.taps > 1:
-            self.conv_state = backend.register_state(layer_idx, "conv", (spec.taps - 1, spec.channels), dtype)
+        super().__init__(_pad8(spec.inner + spec.channels + spec.heads), spec.inner, site)
+        self.spec = spec
+        self.conv, self.conv_bias = site.constant(spec.taps, spec.channels), site.constant(spec.channels)
+        self.dt_bias, self.rate, self.skip = (site.constant(spec.heads) for _ in range(3))
+        self.norm = site.constant(spec.inner)
+        self.conv_state = site.keep("conv", (spec.taps - 1, spec.channels), site.dtype, spec.taps > 1)
         floats = ops.gated_linear_state_floats("ssd", spec.state, spec.vdim)
-        self.state = backend.register_state(layer_idx, "ssd", (spec.heads, floats), torch.float32)
+        self.state = site.keep("ssd", (spec.heads, floats), torch.float32)
 
     def load(self, get: Getter, prefix: str) -> None:
         s = self.spec
@@ -606,30 +699,25 @@ class Mamba2Mixer(Mixer):
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s = self.spec
         z, x, dt = u[:, : s.inner + s.channels + s.heads].split([s.inner, s.channels, s.heads], dim=1)
-        x = ops.short_conv(x, step.packed.rows, self.conv, self.conv_bias, self.conv_state, "silu")
+        x = ops.short_conv(x, step.packed.rows, self.conv, self.conv_bias, self.conv_state[step.turn], "silu")
         n = s.groups * s.state
         x, b, c = x.split([s.inner, n, n], dim=1)
-        y = _gated_rows("ssd", c, b, x, (dt, None), (self.dt_bias, self.rate, self.skip), step, self.state, s.heads, s.state,
-                        s.vdim, self.backend, heads_per_group=s.heads // s.groups)
+        y = _gated_rows("ssd", c, b, x, (dt, None), (self.dt_bias, self.rate, self.skip), step, self.state[step.turn], s.heads,
+                        s.state, s.vdim, self.backend, heads_per_group=s.heads // s.groups)
         return ops.rms_gate(y, z, self.norm, self.eps, groups=s.norm_groups, order="silu_first", out=out)
 
 
 class DeltaMixer(Mixer):
-    def __init__(self, spec: DeltaSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 dtype: torch.dtype, device) -> None:
+    def __init__(self, spec: DeltaSpec, site: Site) -> None:
         """Rows of ``w_in``: q, k, v, output gate, decay logits, beta logits, padding."""
         inner = spec.heads * spec.vdim
-        super().__init__(_pad8(spec.channels + inner + 2 * spec.heads), inner, width, dtype, device)
-        self.spec, self.eps, self.backend = spec, eps, backend
-        f32 = dict(dtype=torch.float32, device=device)
-        self.conv = _param(spec.taps, spec.channels, **f32)
-        self.dt_bias, self.rate = (_param(spec.heads, **f32) for _ in range(2))
-        self.norm = _param(inner, **f32)  # one head's weights, for every head
-        self.conv_state = None
-        if spec.taps > 1:
-            self.conv_state = backend.register_state(layer_idx, "conv", (spec.taps - 1, spec.channels), dtype)
-        pad = lambda n: -(-n // 16) * 16
-        self.state = backend.register_state(layer_idx, "delta", (spec.heads, pad(spec.dim), pad(spec.vdim)), torch.float32)
+        super().__init__(_pad8(spec.channels + inner + 2 * spec.heads), inner, site)
+        self.spec = spec
+        self.conv = site.constant(spec.taps, spec.channels)
+        self.dt_bias, self.rate = (site.constant(spec.heads) for _ in range(2))
+        self.norm = site.constant(inner)  # one head's weights, for every head
+        self.conv_state = site.keep("conv", (spec.taps - 1, spec.channels), site.dtype, spec.taps > 1)
+        self.state = site.keep("delta", (spec.heads, _pad16(spec.dim), _pad16(spec.vdim)), torch.float32)
 
     def _parts(self) -> Tuple[Tuple[str, int], ...]:
         s = self.spec
@@ -651,11 +739,11 @@ class DeltaMixer(Mixer):
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s, packed = self.spec, step.packed
         x, g, a, b = u[:, : s.channels + s.heads * (s.vdim + 2)].split([s.channels, s.heads * s.vdim, s.heads, s.heads], dim=1)
-        x = ops.short_conv(x, packed.rows, self.conv, None, self.conv_state, "silu")
+        x = ops.short_conv(x, packed.rows, self.conv, None, self.conv_state[step.turn], "silu")
         q, k, v = x.split([s.kv_heads * s.dim, s.kv_heads * s.dim, s.heads * s.vdim], dim=1)
         o = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
         sizes = (self.dt_bias, self.rate)
-        tail = (self.state, s.heads, s.dim, s.vdim, s.dim ** -0.5)
+        tail = (self.state[step.turn], s.heads, s.dim, s.vdim, s.dim ** -0.5)
         kw = dict(heads_per_group=s.heads // s.kv_heads)
         if packed.decodes is not None:
             n = packed.num_decodes
@@ -668,15 +756,13 @@ class DeltaMixer(Mixer):
 
 
 class BiasedAttention(Mixer):
-    def __init__(self, spec: BiasedAttentionSpec, width: int, layer_idx: int, backend: HipPagedAttentionBackend, dtype: torch.dtype,
-                 device) -> None:
+    def __init__(self, spec: BiasedAttentionSpec, site: Site) -> None:
         """Rows of ``w_in``: q, k, v, padding."""
-        super().__init__(_pad8((spec.heads + spec.kv_heads) * spec.dim + spec.kv_heads * spec.vdim), spec.heads * spec.vdim, width,
-                         dtype, device)
-        self.spec, self.layer_idx, self.backend = spec, layer_idx, backend
+        super().__init__(_pad8((spec.heads + spec.kv_heads) * spec.dim + spec.kv_heads * spec.vdim), spec.heads * spec.vdim, site)
+        self.spec = spec
         self.buckets = torch.tensor(spec.bucket_of())
-        self.bias = _param(spec.heads, len(self.buckets), dtype=torch.float32, device=device)  # by distance
-        self.sink = _param(spec.heads, dtype=torch.float32, device=device)
+        self.bias = site.constant(spec.heads, len(self.buckets))  # by distance
+        self.sink = site.constant(spec.heads)
 
     def load(self, get: Getter, prefix: str) -> None:
         s, at = self.spec, 0
@@ -692,32 +778,31 @@ class BiasedAttention(Mixer):
 
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s, packed = self.spec, step.packed
-        kc, vc = self.backend._layer(self.layer_idx)
+        place = self.site.places[step.turn]
+        kc, vc = self.backend._layer(place)
         q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, 1.0, 0.0, False, None, 0, None, None)
         # (q and the pool hold zeros between dim and its next multiple of 8)
-        o = self.backend.attend_scored((q[..., : _pad8(s.dim)],), self.layer_idx, packed, s.vdim, s.scale, s.window or 0,
+        o = self.backend.attend_scored((q[..., : _pad8(s.dim)],), place, packed, s.vdim, s.scale, s.window or 0,
                                        softcap=s.softcap or 0.0, bias=self.bias, sink=self.sink)
         o = o.view(u.shape[0], -1)
         return o if out is None else out.copy_(o)
 
 
 class LatentAttention(Mixer):
-    def __init__(self, spec: LatentSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 rotary: RotaryTables, dtype: torch.dtype, device) -> None:
+    def __init__(self, spec: LatentSpec, site: Site) -> None:
         """Rows of ``w_in``: q, latent, rotated key part, padding.  The two weights on the latent are kept in two forms: per
         head, for products before and behind attention over the latents (``w_key`` transposed), and over whole pool rows,
         for keys and values made again (the rotated part passes through an identity)."""
         s = spec
-        super().__init__(_pad8(s.heads * (s.dim + s.rot_dim) + s.kv_rank + s.rot_dim), s.heads * s.vdim, width, dtype, device)
-        self.spec, self.eps, self.layer_idx, self.backend, self.rotary = spec, eps, layer_idx, backend, rotary
+        super().__init__(_pad8(s.heads * (s.dim + s.rot_dim) + s.kv_rank + s.rot_dim), s.heads * s.vdim, site)
+        self.spec = spec
         pad = lambda n: -(-n // 64) * 64
-        kw = dict(dtype=dtype, device=device)
-        self.norm = _param(s.kv_rank, dtype=torch.float32, device=device)
-        self.w_key = _param(s.heads, s.kv_rank, pad(s.dim), **kw)
-        self.w_value = _param(s.heads, s.vdim, pad(s.kv_rank), **kw)
-        self.remake = dtype == torch.bfloat16 and max(s.made) <= 256
+        self.norm = site.constant(s.kv_rank)
+        self.w_key = site.weight(s.heads, s.kv_rank, pad(s.dim))
+        self.w_value = site.weight(s.heads, s.vdim, pad(s.kv_rank))
+        self.remake = site.dtype == torch.bfloat16 and max(s.made) <= 256
         if self.remake:
-            self.k_made, self.v_made = (_param(s.heads, size, s.pool_row, **kw) for size in s.made)
+            self.k_made, self.v_made = (site.weight(s.heads, size, s.pool_row) for size in s.made)
         self._lists: Dict[int, ops.ExpertChoice] = {}
 
     def load(self, get: Getter, prefix: str) -> None:
@@ -748,23 +833,23 @@ class LatentAttention(Mixer):
             self._lists[rows] = choice
         return choice
 
-    def _over_latents(self, q: Tensor, packed: PackedStep, part: str) -> Tensor:
-        s, rows = self.spec, q.shape[0]
+    def _over_latents(self, q: Tensor, step: StepRows, part: str) -> Tensor:
+        s, rows, packed = self.spec, q.shape[0], step.packed
         choice = self._per_head(rows, q.device, part == "decodes")
         over = ops.moe_product(q.view(rows * s.heads, -1)[:, : s.dim], choice, self.w_key, s.kv_rank, s.dim, glu=False)
-        o = self.backend.attend_scored((over.view(rows, s.heads, s.kv_rank), q[..., s.dim: s.dim + s.rot_dim]), self.layer_idx, packed,
-                                       s.kv_rank, _LN2, s.window or 0, part=part)
+        o = self.backend.attend_scored((over.view(rows, s.heads, s.kv_rank), q[..., s.dim: s.dim + s.rot_dim]),
+                                       self.site.places[step.turn], packed, s.kv_rank, _LN2, s.window or 0, part=part)
         return ops.moe_product(o.view(rows * s.heads, s.kv_rank), choice, self.w_value, s.vdim, s.kv_rank, glu=False).view(rows, -1)
 
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         s, packed = self.spec, step.packed
-        pool, _ = self.backend._layer(self.layer_idx)
+        pool, _ = self.backend._layer(self.site.places[step.turn])
         # (q carries scale * log2(e) from its 32-bit registers)
-        q = ops.latent_append(u, packed.rows, packed.slots, pool, self.norm, self.eps, self.rotary.get(s.rot_base, s.rot_dim, 1.0, s.rot_yarn),
-                              s.heads, s.dim, s.rot_dim, s.kv_rank, s.made[0], s.scale / _LN2)
+        q = ops.latent_append(u, packed.rows, packed.slots, pool, self.norm, self.eps,
+                              self.site.rotary.get(s.rot_base, s.rot_dim, 1.0, s.rot_yarn), s.heads, s.dim, s.rot_dim, s.kv_rank, s.made[0], s.scale / _LN2)
         nd = packed.num_decodes
         if packed.chunks is None:
-            o = self._over_latents(q, packed, "decodes")
+            o = self._over_latents(q, step, "decodes")
             return o if out is None else out.copy_(o)
         if self.remake:
             stretch = self.backend.stretch(packed, s.window or 0)
@@ -778,27 +863,122 @@ class LatentAttention(Mixer):
                     out = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
                 ops.head_gate(o[nd:], None, s.vdim, out=out[nd:])
         else:
-            o = self._over_latents(q, packed, "chunks")
+            o = self._over_latents(q, step, "chunks")
             out = o if out is None else out.copy_(o)
         if nd:
-            out[:nd] = self._over_latents(q[:nd], packed, "decodes")
+            out[:nd] = self._over_latents(q[:nd], step, "decodes")
         return out
 
 
+class TalkingAttention(Mixer):
+    @staticmethod
+    def sizes(spec: TalkingSpec) -> Tuple[int, int]:
+        return _pad8(spec.channels + spec.heads), spec.heads * spec.vdim
+
+    def __init__(self, spec: TalkingSpec, site: Site, slices: Slices = None, out_scale: float = 1.0) -> None:
+        """Rows of ``w_in``: q, k, v, head gates, padding."""
+        super().__init__(*self.sizes(spec), site, slices, out_scale)
+        self.spec = spec
+        self.bias = site.constant(spec.channels)
+        self.bias_size, self.bias_rate = site.constant(spec.heads), site.constant(spec.heads)
+        self.talk = site.constant(spec.heads, spec.heads)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        s, at = self.spec, 0
+        for name, n in (("q", s.heads * s.dim), ("k", s.kv_heads * s.dim), ("v", s.kv_heads * s.vdim)):
+            fill(self.w_in[at: at + n], get(prefix + name), prefix + name)
+            fill(self.bias[at: at + n], get(f"{prefix}{name}.b"), f"{prefix}{name}.b")
+            at += n
+        fill(self.w_in[at: at + s.heads], get(prefix + "g"), prefix + "g")
+        fill(self.bias_size, get(prefix + "r1"), prefix + "r1")
+        fill(self.bias_rate, get(prefix + "r2"), prefix + "r2")
+        fill(self.talk, get(prefix + "talk"), prefix + "talk")
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s, packed, place = self.spec, step.packed, self.site.places[step.turn]
+        kc, vc = self.backend._layer(place)
+        q = ops.qkv_conv_append(u, packed.rows, packed.slots, kc, vc, s.heads, s.dim, s.vdim, 1.0, 0.0, False, None, 0, None, None,
+                                bias=self.bias)
+        # (q and the pool hold zeros between dim and its next multiple of 8)
+        o = self.backend.attend_talking(q[..., : _pad8(s.dim)], place, packed, s.vdim, s.scale, self.talk, self.bias_size, self.bias_rate)
+        return ops.head_gate(o, u[:, s.channels: s.channels + s.heads], s.vdim, self.out_scale, out)
+
+
+class Hgrn2Mixer(Mixer):
+    @staticmethod
+    def sizes(spec: Hgrn2Spec) -> Tuple[int, int]:
+        inner = spec.heads * spec.vdim
+        return _pad8(2 * spec.heads * spec.dim + inner), inner
+
+    def __init__(self, spec: Hgrn2Spec, site: Site, slices: Slices = None, out_scale: float = 1.0) -> None:
+        """Rows of ``w_in``: q, forget logits, v, padding."""
+        super().__init__(*self.sizes(spec), site, slices, out_scale)
+        self.spec = spec
+        self.f_bias, self.lower = (site.constant(spec.heads * spec.dim) for _ in range(2))
+        self.norm = site.constant(spec.heads * spec.vdim)  # one head's weights, for every head, times out_scale
+        self.state = site.keep("hgrn2", (spec.heads, _pad16(spec.dim), _pad16(spec.vdim)), torch.float32)
+
+    def _parts(self) -> Tuple[Tuple[str, int], ...]:
+        s = self.spec
+        return ("q", s.heads * s.dim), ("f", s.heads * s.dim), ("v", s.heads * s.vdim)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        at = 0
+        for name, n in self._parts():
+            fill(self.w_in[at: at + n], get(prefix + name), prefix + name)
+            at += n
+        fill(self.f_bias, get(prefix + "f.b"), prefix + "f.b")
+        fill(self.lower, get(prefix + "lower"), prefix + "lower")
+        fill(self.norm, get(prefix + "norm").repeat(self.spec.heads), prefix + "norm")
+        self.norm.mul_(self.out_scale)
+        fill(self.w_out, get(prefix + "o"), prefix + "o")
+
+    def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
+        s, packed = self.spec, step.packed
+        sizes = [n for _, n in self._parts()]
+        q, f, v = u[:, : sum(sizes)].split(sizes, dim=1)
+        o = torch.empty((u.shape[0], s.heads * s.vdim), dtype=u.dtype, device=u.device)
+        tail = (self.state[step.turn], s.heads, s.dim, s.vdim)
+        if packed.decodes is not None:
+            n = packed.num_decodes
+            ops.channel_linear(q[:n], f[:n], v[:n], self.f_bias, self.lower, packed.decodes, *tail, o[:n], q_act="silu")
+        if packed.chunks is not None:
+            c = packed.chunks
+            need = ops.channel_linear_workspace_bytes(c.ctx_lens.numel(), s.heads, s.dim, s.vdim, c.max_q_len)
+            ops.channel_linear(q, f, v, self.f_bias, self.lower, c, *tail, o, q_act="silu",
+                               workspace=self.backend._scratch_for(need) if need else None)
+        return ops.rms_gate(o, None, self.norm, self.eps, groups=s.heads, order=None, out=out)
+
+
 class ParallelMixer(Mixer):
-    def __init__(self, spec: ParallelSpec, width: int, eps: float, layer_idx: int, backend: HipPagedAttentionBackend,
-                 rotary: RotaryTables, dtype: torch.dtype, device) -> None:
-        (in_l, in_r), (out_l, out_r) = zip(ConvAttention.sizes(spec.left), MlstmMixer.sizes(spec.right))
-        super().__init__(in_l + in_r, out_l + out_r, width, dtype, device)
-        self._in, self._out = in_l, out_l
-        self.left = ConvAttention(spec.left, width, eps, layer_idx, backend, rotary, None, dtype, device,
-                                  (self.w_in[: self._in], self.w_out[:, : self._out]), spec.left_scale)
-        self.right = MlstmMixer(spec.right, width, eps, layer_idx, backend, dtype, device,
-                                (self.w_in[self._in:], self.w_out[:, self._out:]), spec.right_scale)
+    SIDES = {AttentionSpec: ConvAttention, TalkingSpec: TalkingAttention, MlstmSpec: MlstmMixer, Hgrn2Spec: Hgrn2Mixer}
+
+    def __init__(self, spec: ParallelSpec, site: Site) -> None:
+        left, right = (self.SIDES[type(s)] for s in (spec.left, spec.right))
+        (in_l, out_l), (in_r, out_r) = left.sizes(spec.left), right.sizes(spec.right)
+        slices = None
+        if spec.norms:  # (each output is normed on its own: two output products)
+            slices = site.weight(in_l + in_r, site.width), None
+        super().__init__(in_l + in_r, out_l + out_r, site, slices)
+        self.spec, self._in, self._out = spec, in_l, out_l
+        scales, outs = (spec.left_scale, spec.right_scale), (None, None)
+        self.left_norm = self.right_norm = None
+        if spec.norms:
+            scales, outs = (1.0, 1.0), (site.weight(site.width, out_l), site.weight(site.width, out_r))
+            self.left_norm, self.right_norm = site.constant(site.width), site.constant(site.width)  # times the scales
+        else:
+            outs = self.w_out[:, :out_l], self.w_out[:, out_l:]
+        self.left = left(spec.left, site, (self.w_in[:in_l], outs[0]), scales[0])
+        self.right = right(spec.right, site, (self.w_in[in_l:], outs[1]), scales[1])
 
     def load(self, get: Getter, prefix: str) -> None:
         self.left.load(get, prefix + "left.")
         self.right.load(get, prefix + "right.")
+        if self.spec.norms:
+            for norm, scale, name in ((self.left_norm, self.spec.left_scale, "left.out"), (self.right_norm, self.spec.right_scale, "right.out")):
+                fill(norm, get(prefix + name), prefix + name)
+                norm.mul_(scale)
 
     def mix(self, u: Tensor, step: StepRows, out: Optional[Tensor] = None) -> Tensor:
         if out is None:
@@ -806,6 +986,18 @@ class ParallelMixer(Mixer):
         self.left.mix(u[:, : self._in], step, out[:, : self._out])
         self.right.mix(u[:, self._in:], step, out[:, self._out:])
         return out
+
+    def branch(self, h: Tensor, step: StepRows) -> Dict[str, object]:
+        if not self.spec.norms:
+            return super().branch(h, step)
+        u = F.linear(h, self.w_in)
+        left = F.linear(self.left.mix(u[:, : self._in], step), self.left.w_out)
+        right = F.linear(self.right.mix(u[:, self._in:], step), self.right.w_out)
+        return {"y": left, "y2": (right, self.left_norm, self.right_norm), "y_eps": self.eps}
+
+
+MIXERS = {AttentionSpec: ConvAttention, BiasedAttentionSpec: BiasedAttention, LatentSpec: LatentAttention, LightningSpec: LightningMixer,
+          Mamba2Spec: Mamba2Mixer, DeltaSpec: DeltaMixer, TalkingSpec: TalkingAttention, Hgrn2Spec: Hgrn2Mixer, ParallelSpec: ParallelMixer}
 
 
 class GatedMLP(nn.Module):
@@ -829,6 +1021,35 @@ class GatedMLP(nn.Module):
 
     def branch(self, h: Tensor) -> Dict[str, Tensor]:
         return {"y": self(h)}
+
+
+@dataclass(frozen=True)
+class MLPSpec:
+    """A feed-forward without a gate: ``down(act(up h))``, both products with biases."""
+
+    inner: int
+    act: str
+
+
+class PlainMLP(nn.Module):
+    """The biases ride on the steps behind the products: the activation's, and the residual sum."""
+
+    def __init__(self, width: int, spec: MLPSpec, dtype: torch.dtype, device) -> None:
+        super().__init__()
+        self.spec = spec
+        self.w_in = _param(spec.inner, width, dtype=dtype, device=device)
+        self.w_out = _param(width, spec.inner, dtype=dtype, device=device)
+        self.in_bias = _param(spec.inner, dtype=torch.float32, device=device)
+        self.out_bias = _param(width, dtype=torch.float32, device=device)
+
+    def load(self, get: Getter, prefix: str) -> None:
+        for w, bias, name in ((self.w_in, self.in_bias, "up"), (self.w_out, self.out_bias, "down")):
+            fill(w, get(prefix + name), prefix + name)
+            fill(bias, get(f"{prefix}{name}.b"), f"{prefix}{name}.b")
+
+    def branch(self, h: Tensor) -> Dict[str, Tensor]:
+        act = ops.bias_act(F.linear(h, self.w_in), self.in_bias, self.spec.act)
+        return {"y": F.linear(act, self.w_out), "y_bias": self.out_bias}
 
 
 class TokenSide(nn.Module):

@@ -17,7 +17,7 @@ import torch
 from torch import Tensor, nn
 
 from .attention import CacheConfig, HipPagedAttentionBackend
-from .hybrid import HybridConfig, HybridDecoder, lotozen_config, tevirax_config, vusalix_config
+from .hybrid import HybridConfig, HybridDecoder, loluzen_config, lotozen_config, tevirax_config, vusalix_config
 from .model import ModelConfig, PagedLlama
 
 DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
@@ -121,5 +121,6 @@ register(ModelEntry("lotozen", lambda c: c.get("architecture") == "Lotozen", _hy
 register(ModelEntry("tevirax", lambda c: c.get("architecture") == "Tevirax", _hybrid(lambda c, w: tevirax_config(c)),
                     lambda c: int(c["max_positions"])))
 register(ModelEntry("vusalix", lambda c: c.get("architecture") == "Vusalix", _hybrid(_vusalix)))
+register(ModelEntry("loluzen", lambda c: c.get("architecture") == "Loluzen", _hybrid(lambda c, w: loluzen_config(c))))
 register(ModelEntry("llama", lambda c: "num_attention_heads" in c, _build_llama,
                     lambda c: c.get("max_position_embeddings")))

@@ -352,9 +352,9 @@ def _typed(dtype: torch.dtype, *tensors: Optional[Tensor]) -> None:
 
 
 _NORMS = {None: _lib.PA_NORM_NONE, "layer": _lib.PA_NORM_LAYER, "rms": _lib.PA_NORM_RMS}
-_ACTS = {"silu": _lib.PA_ACT_SILU, "gelu_tanh": _lib.PA_ACT_GELU_TANH, None: _lib.PA_ACT_NONE}
+_ACTS = {"silu": _lib.PA_ACT_SILU, "gelu_tanh": _lib.PA_ACT_GELU_TANH, None: _lib.PA_ACT_NONE, "relu2": _lib.PA_ACT_RELU2}
 _GATES = {"sigmoid_last": _lib.PA_GATE_SIGMOID_LAST, "silu_first": _lib.PA_GATE_SILU_FIRST,
-          "silu_last": _lib.PA_GATE_SILU_LAST}
+          "silu_last": _lib.PA_GATE_SILU_LAST, None: _lib.PA_GATE_NONE}
 _SCORES = {"sigmoid": _lib.PA_MOE_SIGMOID, "softmax": _lib.PA_MOE_SOFTMAX}
 _SHARED = {None: _lib.PA_MOE_NO_SHARED, "gated": _lib.PA_MOE_SHARED_GATED, "plain": _lib.PA_MOE_SHARED}
 _GATED = {"ssd": _lib.PA_GL_SSD, "mlstm": _lib.PA_GL_MLSTM}
@@ -366,17 +366,21 @@ def residual_norm(x: Tensor, dtype: torch.dtype, y: Optional[Tensor] = None, y_w
                   row_index: Optional[Tensor] = None, norm: Optional[str] = None, weight: Optional[Tensor] = None,
                   bias: Optional[Tensor] = None, eps: float = 0.0, want_out: bool = True, table_scale: float = 1.0,
                   positions: Optional[Tensor] = None, pos_table: Optional[Tensor] = None, mix: Optional[Tensor] = None,
-                  y_extra: Optional[Tensor] = None) -> Optional[Tensor]:
+                  y_extra: Optional[Tensor] = None, y_bias: Optional[Tensor] = None,
+                  y2: Optional[Tuple[Tensor, Tensor, Tensor]] = None, ids_add: bool = False) -> Optional[Tensor]:
     """Residual sum and norm in one pass over the rows (``pa_residual_norm``): ``x`` float32 ``[rows, width]`` is
     updated in place (``table[ids] * table_scale``, with ``positions`` also their rows of ``pos_table``, or itself,
     plus ``y`` or its RMS norm times ``y_weight``), and ``norm(x) * weight + bias`` (``"layer"``, ``"rms"`` or None: a
     cast) comes back in ``dtype``.  With ``mix`` float32 ``[rows, m + 1]`` the branch is a weighted sum: of ``y``
-    ``[rows * m, width]``, m rows each, and of ``y_extra``.  ``row_index`` picks rows of ``x`` instead of updating it."""
+    ``[rows * m, width]``, m rows each, and of ``y_extra``.  ``y_bias`` is added to ``y``; ``y2`` ``(branch, weight of y's
+    own norm, weight of the branch's)``: y is the sum of two normed branches.  ``ids_add``: the table's rows are added to
+    ``x``.  ``row_index`` picks rows of ``x`` instead of updating it."""
     rows, width = x.shape
-    _dense(x, y, y_weight, ids, table, row_index, weight, bias, positions, pos_table, mix, y_extra)
-    _typed(torch.float32, x, y_weight, weight, bias, mix)
+    other, own_part, other_part = y2 if y2 is not None else (None, None, None)
+    _dense(x, y, y_weight, ids, table, row_index, weight, bias, positions, pos_table, mix, y_extra, y_bias, other, own_part, other_part)
+    _typed(torch.float32, x, y_weight, weight, bias, mix, y_bias, own_part, other_part)
     _typed(torch.int64, ids, row_index, positions)
-    _typed(dtype, y, table, pos_table, y_extra)
+    _typed(dtype, y, table, pos_table, y_extra, other)
     n = rows if row_index is None else row_index.numel()
     m = mix.shape[1] - 1 if mix is not None else 0
     if (y is not None and tuple(y.shape) != (rows * (m or 1), width)) or (ids is not None and ids.numel() != rows):
@@ -388,34 +392,37 @@ def residual_norm(x: Tensor, dtype: torch.dtype, y: Optional[Tensor] = None, y_w
     for t in (table, pos_table):
         if t is not None and t.shape[1] != width:
             raise ValueError("table rows are not as wide as the residual")
-    for w in (y_weight, weight, bias):
+    if other is not None and tuple(other.shape) != (rows, width):
+        raise ValueError("y2 does not fit the residual")
+    for w in (y_weight, weight, bias, y_bias, own_part, other_part):
         if w is not None and w.numel() != width:
             raise ValueError("norm weights are not as wide as the residual")
     out = torch.empty((n, width), dtype=dtype, device=x.device) if want_out else None
-    _run("pa_residual_norm", _ptr(x), _ptr(y), _ptr(mix), m, _ptr(y_extra), _ptr(y_weight), float(y_eps), _ptr(ids), _ptr(table),
+    _run("pa_residual_norm", _ptr(x), _ptr(y), _ptr(mix), m, _ptr(y_extra), _ptr(y_bias), _ptr(other), _ptr(own_part),
+         _ptr(other_part), _ptr(y_weight), float(y_eps), _ptr(ids), int(ids_add), _ptr(table),
          table.shape[0] if table is not None else 0, float(table_scale), _ptr(positions), _ptr(pos_table),
          pos_table.shape[0] if pos_table is not None else 0, _ptr(row_index), rows, _ptr(weight), _ptr(bias), float(eps),
          _NORMS[norm], _ptr(out), n, width, PA_DTYPE[dtype], _stream(x))
     return out
 
 
-def rms_gate(o: Tensor, gate: Tensor, weight: Tensor, eps: float, groups: int = 1, order: str = "sigmoid_last",
+def rms_gate(o: Tensor, gate: Optional[Tensor], weight: Tensor, eps: float, groups: int = 1, order: Optional[str] = "sigmoid_last",
              out: Optional[Tensor] = None) -> Tensor:
     """The gated RMS norm of every one of ``groups`` equal parts of a row (``pa_rms_gate``): ``"sigmoid_last"``:
-    ``o / rms(o) * weight * sigmoid(gate)``; ``"silu_last"`` likewise with the silu; ``"silu_first"``: ``z / rms(z) * weight`` of ``z = o * silu(gate)``.
+    ``o / rms(o) * weight * sigmoid(gate)``; ``"silu_last"`` likewise with the silu; ``"silu_first"``: ``z / rms(z) * weight`` of ``z = o * silu(gate)``; None: the norm alone.
     ``gate`` and ``out`` may be column slices."""
     rows, width = o.shape
     _dense(o, weight)
     _typed(o.dtype, gate)
     _typed(torch.float32, weight)
-    if tuple(gate.shape) != (rows, width) or weight.numel() != width:
+    if (gate is None) != (order is None) or (gate is not None and tuple(gate.shape) != (rows, width)) or weight.numel() != width:
         raise ValueError("gate / weight do not fit o")
     if out is None:
         out = torch.empty_like(o)
     _typed(o.dtype, out)
     if tuple(out.shape) != (rows, width):
         raise ValueError("out does not fit o")
-    _run("pa_rms_gate", _ptr(o), _ptr(gate), _row_stride(gate), _ptr(weight), float(eps), _ptr(out), _row_stride(out), rows,
+    _run("pa_rms_gate", _ptr(o), _ptr(gate), _row_stride(gate) if gate is not None else 0, _ptr(weight), float(eps), _ptr(out), _row_stride(out), rows,
          width, groups, _GATES[order], PA_DTYPE[o.dtype], _stream(o))
     return out
 
@@ -431,6 +438,18 @@ def glu(gate: Tensor, up: Tensor, act: str, ids: Optional[Tensor] = None) -> Ten
     out = torch.empty((rows, width), dtype=gate.dtype, device=gate.device)
     _run("pa_glu", _ptr(gate), _row_stride(gate), _ptr(up), _row_stride(up), _ptr(ids), up.shape[0], _ptr(out), rows,
          width, _ACTS[act], PA_DTYPE[gate.dtype], _stream(gate))
+    return out
+
+
+def bias_act(x: Tensor, bias: Optional[Tensor], act: Optional[str]) -> Tensor:
+    """``act(x + bias)`` (``pa_bias_act``), ``"relu2"`` the square of the positive part; ``x`` may be a column slice."""
+    rows, width = x.shape
+    _dense(bias)
+    _typed(torch.float32, bias)
+    if bias is not None and bias.numel() != width:
+        raise ValueError("bias does not fit x")
+    out = torch.empty((rows, width), dtype=x.dtype, device=x.device)
+    _run("pa_bias_act", _ptr(x), _row_stride(x), _ptr(bias), _ptr(out), rows, width, _ACTS[act], PA_DTYPE[x.dtype], _stream(x))
     return out
 
 
@@ -470,18 +489,20 @@ def qkv_conv_append(u: Tensor, portions: Portions, slots: Tensor, k_cache: Tenso
                     conv_weight: Optional[Tensor], conv_state: Optional[Tensor], v_mode: Optional[str] = None,
                     v_first: Optional[Tensor] = None, v_lambda: Optional[Tensor] = None,
                     q_out: Optional[Tensor] = None, q_norm: Optional[Tensor] = None,
-                    k_norm: Optional[Tensor] = None) -> Tensor:
+                    k_norm: Optional[Tensor] = None, bias: Optional[Tensor] = None) -> Tensor:
     """Projection rows to rotated, normalised q and appended k / v (``pa_qkv_conv_append``).  Returns q
     ``[rows, Hq, D]`` with D the pool's head size; k and v go to ``k_cache`` / ``v_cache`` ``[slots, Hkv, D]``.
-    ``q_norm`` / ``k_norm`` float32 ``[dim]``: weights of RMS norms ahead of the rotation."""
+    ``q_norm`` / ``k_norm`` float32 ``[dim]``: weights of RMS norms ahead of the rotation; ``bias`` float32 ``[channels]``."""
     rows = u.shape[0]
     total_slots, hkv, d = k_cache.shape
     taps = conv_weight.shape[0] if conv_weight is not None else 1
     channels = (num_q_heads + hkv) * dim + hkv * vdim
-    _dense(slots, k_cache, v_cache, rope, conv_weight, conv_state, v_first, q_norm, k_norm, *portions[:5])
+    _dense(slots, k_cache, v_cache, rope, conv_weight, conv_state, v_first, q_norm, k_norm, bias, *portions[:5])
     _typed(u.dtype, k_cache, v_cache, conv_state, v_first)
     _typed(torch.int32, *portions[:5])
-    _typed(torch.float32, rope, conv_weight, v_lambda, q_norm, k_norm)
+    _typed(torch.float32, rope, conv_weight, v_lambda, q_norm, k_norm, bias)
+    if bias is not None and bias.numel() != channels:
+        raise ValueError("bias must hold one number per channel")
     for t in (q_norm, k_norm):
         if t is not None and t.numel() != dim:
             raise ValueError("q_norm / k_norm must hold one weight per dimension")
@@ -498,7 +519,7 @@ def qkv_conv_append(u: Tensor, portions: Portions, slots: Tensor, k_cache: Tenso
     if q_out is None:
         q_out = torch.empty((rows, num_q_heads, d), dtype=u.dtype, device=u.device)
     n_tiles = batch if portions.tiles is None else portions.tiles.shape[0]
-    _run("pa_qkv_conv_append", _ptr(u), _row_stride(u), rows, _ptr(conv_weight), taps, _ptr(conv_state),
+    _run("pa_qkv_conv_append", _ptr(u), _row_stride(u), rows, _ptr(bias), _ptr(conv_weight), taps, _ptr(conv_state),
          conv_state.shape[0] if conv_state is not None else 0, _ptr(rope), rope.shape[0] if rope is not None else 0,
          rot_dims if rope is not None else 0, _ptr(portions.ctx_lens), _ptr(portions.q_lens), _ptr(portions.q_starts),
          _ptr(portions.state_slots), _ptr(portions.tiles), n_tiles, batch, _ptr(slots), total_slots, _ptr(q_out),
@@ -804,4 +825,57 @@ def scored_attention(q: Tuple[Tensor, ...], k_cache: Tensor, v_cache: Tensor, vd
          _ptr(portions.q_starts), rows, batch, portions.max_q_len, heads, kv_heads, float(scale), int(window), float(softcap), _ptr(bias),
          bias.shape[1] if bias is not None else 0, _ptr(sink), _ptr(out), PA_DTYPE[out.dtype], _ptr(workspace),
          workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(out))
+    return out
+
+
+def talking_workspace_bytes(rows: int, portions: Portions, heads: int, kv_heads: int, vdim: int, max_keys: int) -> int:
+    return int(_lib.load().pa_talking_workspace_bytes(rows, portions.ctx_lens.numel(), heads, kv_heads, vdim, max_keys, int(portions.q_lens is None)))
+
+
+def talking_attention(q: Tensor, k_cache: Tensor, v_cache: Tensor, vdim: int, portions: Portions, block_tables: Tensor, block_size: int,
+                      scale: float, talk: Tensor, out: Tensor, bias_size: Optional[Tensor] = None, bias_rate: Optional[Tensor] = None,
+                      workspace: Optional[Tensor] = None) -> Tensor:
+    """Paged attention whose heads' weights are mixed by ``talk`` float32 ``[heads, heads]`` (``pa_talking_attention``): ``q``
+    ``[rows, heads, dim]`` whose last dimension is contiguous, ``bias_size`` and ``bias_rate`` float32 ``[heads]``; ``out``
+    ``[rows, heads, vdim]``.  The workspace (``talking_workspace_bytes``) is needed."""
+    rows, heads, dim = q.shape
+    total_slots, kv_heads, k_dim = k_cache.shape
+    _dense(k_cache, v_cache, block_tables, talk, bias_size, bias_rate, out, *portions[:4])
+    _typed(torch.int32, block_tables, *portions[:4])
+    _typed(torch.float32, talk, bias_size, bias_rate)
+    _typed(out.dtype, k_cache, v_cache, q)
+    if q.stride(2) != 1 or tuple(v_cache.shape[:2]) != (total_slots, kv_heads) or tuple(out.shape) != (rows, heads, vdim):
+        raise ValueError("q / v_cache / out do not fit")
+    if tuple(talk.shape) != (heads, heads) or any(t is not None and t.numel() != heads for t in (bias_size, bias_rate)):
+        raise ValueError("talk / bias_size / bias_rate do not fit the heads")
+    _run("pa_talking_attention", _ptr(q), q.stride(0), q.stride(1), dim, _ptr(k_cache), k_dim, _ptr(v_cache), v_cache.shape[2], vdim,
+         _ptr(block_tables), block_tables.shape[1], block_size, total_slots // block_size, _ptr(portions.ctx_lens), _ptr(portions.q_lens),
+         _ptr(portions.q_starts), rows, portions.ctx_lens.numel(), portions.max_q_len, heads, kv_heads, float(scale), _ptr(bias_size),
+         _ptr(bias_rate), _ptr(talk), _ptr(out), PA_DTYPE[out.dtype], _ptr(workspace),
+         workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(out))
+    return out
+
+
+def channel_linear_workspace_bytes(batch: int, heads: int, dim: int, vdim: int, max_q_len: int) -> int:
+    return int(_lib.load().pa_channel_linear_workspace_bytes(batch, heads, dim, vdim, max_q_len))
+
+
+def channel_linear(q: Tensor, forget: Tensor, v: Tensor, f_bias: Optional[Tensor], lower: Tensor, portions: Portions, state: Tensor,
+                   heads: int, dim: int, vdim: int, out: Tensor, q_act: Optional[str] = None, workspace: Optional[Tensor] = None) -> Tensor:
+    """Linear attention with a forget gate per channel (``pa_channel_linear``).  q, the gate's logits and v may be column slices;
+    ``f_bias`` and ``lower`` float32 ``[heads * dim]``, ``state`` float32 ``[slots, heads, pad16(dim), pad16(vdim)]``."""
+    rows, batch = v.shape[0], portions.ctx_lens.numel()
+    pad = lambda n: -(-n // 16) * 16
+    _dense(state, out, f_bias, lower, *portions[:4])
+    _typed(torch.int32, *portions[:4])
+    _typed(torch.float32, state, f_bias, lower)
+    _typed(v.dtype, q, forget, out)
+    if any(tuple(t.shape) != (rows, heads * dim) for t in (q, forget)) or tuple(v.shape) != (rows, heads * vdim) or out.shape != v.shape:
+        raise ValueError("q / forget / v / out do not fit each other")
+    if any(t is not None and t.numel() != heads * dim for t in (f_bias, lower)) or tuple(state.shape[1:]) != (heads, pad(dim), pad(vdim)):
+        raise ValueError("constants or state of another size")
+    _run("pa_channel_linear", _ptr(q), _row_stride(q), _ACTS[q_act], _ptr(forget), _row_stride(forget), _ptr(f_bias), _ptr(lower), _ptr(v),
+         _row_stride(v), rows, _ptr(state), state.shape[0], _ptr(portions.ctx_lens), _ptr(portions.q_lens), _ptr(portions.q_starts),
+         _ptr(portions.state_slots), batch, portions.max_q_len, _ptr(out), heads, dim, vdim, PA_DTYPE[v.dtype], _ptr(workspace),
+         workspace.numel() * workspace.element_size() if workspace is not None else 0, _stream(v))
     return out

@@ -33,7 +33,7 @@ def test_binding_table_matches_header():
 
 def test_version_and_dtype_sizes():
     lib = _lib.load()
-    assert lib.pa_version() == 9
+    assert lib.pa_version() == 10
     assert [lib.pa_dtype_bytes(c) for c in (0, 1, 2, 3, 4, -1)] == [4, 2, 2, 1, 0, 0]
 
 
@@ -229,16 +229,18 @@ def test_generated_prefill_loop_is_current(tmp_path, script, generated):
 def test_block_entry_points_check_their_arguments():
     """The kernels around attention in hybrid blocks: rejected before any device call."""
     f32, bf16 = _lib.PA_F32, _lib.PA_BF16
-    residual = lambda **kw: [{**dict(x=FAKE, y=FAKE, mw=None, mix=0, yx=None, yw=None, ye=0.0, ids=None, table=None, tr=0,
+    residual = lambda **kw: [{**dict(x=FAKE, y=FAKE, mw=None, mix=0, yx=None, yb=None, y2=None, yp=None, y2p=None, yw=None, ye=0.0, ids=None, ia=0, table=None, tr=0,
                                      ts=1.0, pos=None, pt=None, pr=0, ri=None, xr=4, w=FAKE, b=FAKE, eps=1e-6,
                                      norm=_lib.PA_NORM_LAYER, out=FAKE, rows=4, width=64, dt=bf16, s=None), **kw}[k]
-                             for k in ("x", "y", "mw", "mix", "yx", "yw", "ye", "ids", "table", "tr", "ts", "pos", "pt", "pr", "ri",
+                             for k in ("x", "y", "mw", "mix", "yx", "yb", "y2", "yp", "y2p", "yw", "ye", "ids", "ia", "table", "tr", "ts", "pos", "pt", "pr", "ri",
                                        "xr", "w", "b", "eps", "norm", "out", "rows", "width", "dt", "s")]
     for kw, status, text in ((dict(x=None), -1, "neither"), (dict(norm=7), -1, "norm=7"), (dict(width=20000), -2, "above"),
                              (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(ids=FAKE), -1, "table"), (dict(ri=FAKE), -1, "row_index"),
                              (dict(y=None, out=None), -1, "nothing"), (dict(y=None, yw=FAKE), -1, "y_weight"),
                              (dict(norm=_lib.PA_NORM_NONE), -1, "without a norm"), (dict(pos=FAKE, pt=FAKE), -1, "positions"),
-                             (dict(mw=FAKE), -1, "mix_weight"), (dict(yx=FAKE), -1, "y_extra")):
+                             (dict(mw=FAKE), -1, "mix_weight"), (dict(yx=FAKE), -1, "y_extra"), (dict(ia=1), -1, "ids_add"),
+                             (dict(y=None, yb=FAKE), -1, "y_bias"), (dict(mw=FAKE, mix=2, y2=FAKE, yp=FAKE, y2p=FAKE), -1, "y2"),
+                             (dict(y2=FAKE, yp=FAKE), -1, "together"), (dict(yp=FAKE), -1, "together")):
         rc, msg = _status("pa_residual_norm", *residual(**kw))
         assert rc == status and text in msg, (kw, msg)
     assert _status("pa_residual_norm", *residual(rows=0, x=None))[0] == 0
@@ -255,17 +257,18 @@ def test_block_entry_points_check_their_arguments():
     rc, msg = _status("pa_head_gate", FAKE, FAKE, 4, 1.0, FAKE, 96, 4, 4, 16, 24, f32, None)
     assert rc == -1 and "sizes" in msg
 
-    qkv = lambda **kw: [{**dict(u=FAKE, ld=200, n=4, cw=FAKE, taps=3, cs=FAKE, sr=2, rope=FAKE, rr=9, rot=8, cl=FAKE, ql=None,
+    qkv = lambda **kw: [{**dict(u=FAKE, ld=200, n=4, ub=None, cw=FAKE, taps=3, cs=FAKE, sr=2, rope=FAKE, rr=9, rot=8, cl=FAKE, ql=None,
                                 qs=None, ss=FAKE, tiles=None, nt=4, batch=4, slots=FAKE, ts=64, q=FAKE, k=FAKE, v=FAKE, vf=None,
                                 lam=None, vm=0, qn=None, kn=None, hq=4, hkv=2, dim=16, vdim=24, d=24, un=1, eps=1e-6, qsc=1.0, dt=bf16, s=None),
-                           **kw}[k] for k in ("u", "ld", "n", "cw", "taps", "cs", "sr", "rope", "rr", "rot", "cl", "ql", "qs", "ss",
+                           **kw}[k] for k in ("u", "ld", "n", "ub", "cw", "taps", "cs", "sr", "rope", "rr", "rot", "cl", "ql", "qs", "ss",
                                               "tiles", "nt", "batch", "slots", "ts", "q", "k", "v", "vf", "lam", "vm", "qn", "kn", "hq", "hkv",
                                               "dim", "vdim", "d", "un", "eps", "qsc", "dt", "s")]
     for kw, status, text in ((dict(hkv=3), -1, "multiple"), (dict(d=20), -1, "pool_dim"), (dict(rot=9), -1, "rot_dims"),
                              (dict(taps=9), -2, "taps"), (dict(cw=None), -1, "convolution"), (dict(cs=None), -1, "carried"),
                              (dict(rope=None), -1, "table"), (dict(vm=2, vf=FAKE), -1, "v_lambda"), (dict(vm=1), -1, "v_first"),
                              (dict(nt=3), -1, "one row"), (dict(ld=100), -1, "u_stride"), (dict(tiles=FAKE), -1, "tiles"),
-                             (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(d=264), -2, "above 256"), (dict(qn=FAKE), -1, "together")):
+                             (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(d=264), -2, "above 256"), (dict(qn=FAKE), -1, "together"),
+                             (dict(ub=FAKE), -1, "bias")):
         rc, msg = _status("pa_qkv_conv_append", *qkv(**kw))
         assert rc == status and text in msg, (kw, msg)
     assert _status("pa_qkv_conv_append", *qkv(n=0, u=None, batch=0, nt=0))[0] == 0

@@ -101,7 +101,7 @@ def test_checkpoint_folder_is_loaded_into_joint_projections(loaded):
     assert torch.equal(l.mixer.w_in[48:96], w["l1.mix.k"].float()) and torch.equal(l.mlp.w_in[40:], w["l1.mlp.up"].float())
     assert torch.equal(l.mixer.decay_powers[:, 64], torch.tensor([0.7, 0.98, 0.9995], dtype=torch.float64).pow(64).float())
     assert torch.equal(l.norm2.b, w["l1.norm2.b"].float()) and torch.equal(model.side_embed, w["side.embed"].float())
-    rope = a.rotary.get(1000.0, 12, 2.0)
+    rope = a.site.rotary.get(1000.0, 12, 2.0)
     assert tuple(rope.shape) == (50, 6, 2)
     angle = torch.tensor(49 * 1000.0 ** (-4 / 12) / 2.0, dtype=torch.float64)
     assert torch.allclose(rope[49, 2].double(), torch.stack([angle.cos(), angle.sin()]), atol=1e-7)

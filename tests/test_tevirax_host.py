@@ -11,7 +11,7 @@ import torch
 from oracle import tevirax_oracle as to
 from research_amd.inference import HybridDecoder, registry
 from research_amd.inference.hybrid import tevirax_config
-from research_amd.inference.mixers import AttentionSpec, Mamba2Spec, MlstmSpec, ParallelSpec, RotaryTables, YarnScaling, yarn_frequencies
+from research_amd.inference.mixers import AttentionSpec, Mamba2Spec, MlstmSpec, ParallelSpec, RotaryTables, Site, YarnScaling, yarn_frequencies
 from research_amd.inference.moe import MoESpec
 from tests import hybrid_helpers as hh
 
@@ -140,7 +140,7 @@ def test_value_heads_in_slices():
     from research_amd.inference.attention import CacheConfig, HipPagedAttentionBackend
 
     backend = HipPagedAttentionBackend(CacheConfig(1, 4, 152, num_blocks=1, device="cpu", dtype=torch.float32))
-    att = ConvAttention(spec, 10, 1e-5, 0, backend, RotaryTables(4, "cpu"), None, torch.float32, "cpu")
+    att = ConvAttention(spec, Site(10, 1e-5, (0,), backend, RotaryTables(4, "cpu"), torch.float32, "cpu"))
     w = {"q": torch.randn(24, 10, generator=g), "k": torch.randn(12, 10, generator=g), "v": torch.randn(600, 10, generator=g),
          "o": torch.randn(10, 1200, generator=g), "q.norm": torch.ones(6), "k.norm": torch.ones(6)}
     att.load(lambda n: w[n], "")
