@@ -1,2 +1,418 @@
+// Portions of prompts of attention with mixed heads on the matrix cores (16-bit pools, keys and values of up to 128, up to 32
+// heads).
+//
+// The first kernel leaves every row's and head's sum: a wave owns 32 rows of one head, a workgroup four (row block, head) pairs
+// of one kv head, which share tiles of 64 keys in LDS (as in scored_prefill.hip, without values).  The second one makes the
+// scores again, for all heads at once: a workgroup owns 16 rows, its eight waves have their own heads, queries and value
+// accumulators in registers.  Per tile of 32 keys
+//   1. S^T = K Q^T leaves a lane four keys of one row per head; the weights go to LDS, all heads of a (key, row) pair side by
+//      side, as two bf16 terms;
+//   2. T times these, the pairs of four keys per wave, and back to LDS as weights of (head, row), keys side by side;
+//   3. O^T += V^T W^T per head, V by transposing reads from the wave's own part of LDS (which is the weights' of step 1).
+// Distance biases of a head are one logarithm per lane and tile, spread by LDS.
+#include "linear_tiles.h"
+#include "prefill_mfma.h"
 #include "talking.h"
-bool pa_talking_prefill_launch(const TalkArgs &, int, hipStream_t, int &) { return false; }
+
+namespace {
+
+using namespace pa_decode_detail;
+
+constexpr float kTpSlack = 8.f;  // log2 of the factor by which a row's reference maximum may lag
+
+__device__ __forceinline__ void tp_own_lds() {  // a wave's own part of LDS: its writes before its reads
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+}
+
+// ------------------------------------------------------------------ sums
+constexpr int kTsKeys = 64;
+template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(const TalkArgs a) {
+    using M = Mfma16<pa_bf16>;
+    using X8 = M::x8;
+    constexpr int KS = DK / 16, NK = kTsKeys * DK / 8 / 256, kPitch = DK + 8;
+    __shared__ __align__(16) uint16_t ks[kTsKeys * kPitch];
+    __shared__ float biases[4][2][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), half = lane >> 5, col = lane & 31;
+    const int kvh = blockIdx.y, b = blockIdx.x;
+    ScoredPortion p;
+    if (!scored_portion(a, b, p)) return;
+    const int n_tasks = (p.n + 31) / 32 * a.n_rep;
+    const int group = gridDim.z - 1 - blockIdx.z;  // (the rows with the most keys first)
+    if (group * 4 >= n_tasks) return;
+    const int task = group * 4 + wave, last_task = min(n_tasks, group * 4 + 4) - 1;
+    const bool live = task < n_tasks;
+    const int row0 = (live ? task / a.n_rep : 0) * 32, h = kvh * a.n_rep + (live ? task % a.n_rep : 0);
+    const int row = row0 + col, pos = p.pos0 + min(row, p.n - 1), wave_hi = p.pos0 + min(row0 + 32, p.n);
+    const int wg_hi = p.pos0 + min(last_task / a.n_rep * 32 + 32, p.n);
+    const float plain = a.scale * kScoredLog2e, size = a.size ? a.size[h] : 0.f, rate = a.rate ? a.rate[h] : 0.f;
+    X8 q[KS];
+    {
+        const uint16_t *src = reinterpret_cast<const uint16_t *>(a.q1) + (p.row0 + min(row, p.n - 1)) * a.q1_row + h * a.q1_head;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) {
+            const int d = 16 * k + 8 * half;
+            q[k] = __builtin_bit_cast(X8, d < a.n1 ? *reinterpret_cast<const uint4 *>(src + d) : make_uint4(0, 0, 0, 0));
+        }
+    }
+    float m = kScoredNone, l = 0.f;
+    const int32_t *table = a.bt + b * a.bt_stride;
+    const uint16_t *kp = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)kvh * a.k_dim;
+    const int64_t k_tok = (int64_t)a.hkv * a.k_dim;
+    auto id_of = [&](int k0) { return scored_block_id(a, table, min(k0 + lane, wg_hi - 1)); };
+    scored_u4 kr[NK];
+    auto fetch = [&](int id, int k0) {
+        const int slots = scored_slot_of(a, id, k0 + lane, wg_hi);
+#pragma unroll
+        for (int n = 0; n < NK; ++n) {
+            const int c = tid + 256 * n, s = __shfl(slots, c / (DK / 8), 64), e = c % (DK / 8) * 8;
+            kr[n] = scored_load16(kp + s * k_tok + e, s >= 0 && e < a.n1);
+        }
+    };
+    fetch(id_of(0), 0);
+    int id = id_of(kTsKeys);
+    for (int k0 = 0; k0 < wg_hi; k0 += kTsKeys) {
+#pragma unroll
+        for (int n = 0; n < NK; ++n) {
+            const int c = tid + 256 * n;
+            *reinterpret_cast<scored_u4 *>(ks + c / (DK / 8) * kPitch + c % (DK / 8) * 8) = kr[n];
+        }
+        __syncthreads();
+        if (k0 + kTsKeys < wg_hi) {
+            fetch(id, k0 + kTsKeys);
+            id = id_of(k0 + 2 * kTsKeys);
+        }
+        if (live && k0 < wave_hi && a.size) {  // distances p.pos0 + row0 + i - k of i < 32 and each half's 32 keys, from their smallest
+#pragma unroll
+            for (int sub = 0; sub < 2; ++sub)
+                biases[wave][sub][lane] = talk_bias(size, rate, max(p.pos0 + row0 - (k0 + 32 * sub + 31) + lane, 0));
+            tp_own_lds();
+        }
+#pragma unroll
+        for (int sub = 0; sub < 2; ++sub) {
+            const int kb = k0 + 32 * sub;  // (uniform per wave)
+            if (!live || kb >= wave_hi) continue;
+            f32x16 s;
+#pragma unroll
+            for (int i = 0; i < 16; ++i) s[i] = 0.f;
+#pragma unroll
+            for (int k = 0; k < KS; ++k)
+                s = M::mma(__builtin_bit_cast(X8, *reinterpret_cast<const uint4 *>(ks + (32 * sub + col) * kPitch + 16 * k + 8 * half)), q[k], s);
+            // element i: key kb + 8 (i / 4) + 4 half + i % 4
+            if (a.size) {
+                const float *bp = biases[wave][sub] + col + 31 - 4 * half;
+#pragma unroll
+                for (int i = 0; i < 16; ++i) s[i] = fmaf(s[i], plain, bp[-(8 * (i >> 2) + (i & 3))]);
+            } else {
+#pragma unroll
+                for (int i = 0; i < 16; ++i) s[i] *= plain;
+            }
+            if (kb + 31 > p.pos0 + row0) {
+                const int hi = pos - kb - 4 * half;
+#pragma unroll
+                for (int i = 0; i < 16; ++i) s[i] = 8 * (i >> 2) + (i & 3) <= hi ? s[i] : kScoredNone;
+            }
+            float top = fmaxf(s[0], s[1]);
+#pragma unroll
+            for (int i = 2; i < 16; ++i) top = fmaxf(top, s[i]);
+            if (__ballot(top > m + kTpSlack) != 0) {  // (every lane has a maximum of its own)
+                const float next = fmaxf(m, top);
+                l *= __builtin_amdgcn_exp2f(m - next);
+                m = next;
+            }
+#pragma unroll
+            for (int i = 0; i < 16; i += 2) l += __builtin_amdgcn_exp2f(s[i] - m) + __builtin_amdgcn_exp2f(s[i + 1] - m);
+        }
+        __syncthreads();
+    }
+    // (a lane that saw no key has m = kScoredNone and counted its masked ones as 1: they vanish here)
+    const float other = __shfl_xor(m, 32, 64), top = fmaxf(m, other);
+    l *= __builtin_amdgcn_exp2f(m - top);
+    l += __shfl_xor(l, 32, 64);
+    if (live && row < p.n && half == 0) a.lse[(p.row0 + row) * a.heads + h] = top + __builtin_amdgcn_logf(l);
+}
+
+// ------------------------------------------------------------------ mixed weights times values
+constexpr int kTmRows = 16, kTmKeys = 32, kTmWaves = 8, kTmThreads = 64 * kTmWaves;
+
+// D: keys and values padded to 64 or 128; HW: heads per wave, 2 or 4.
+template <int D, int HW> struct TmTile {
+    static constexpr int heads = kTmWaves * HW, vPitch = D + 8;
+    static constexpr int pair = 4 * heads;                                      // bytes of a (key, row) pair: both terms of all heads
+    static constexpr int pBytes = kTmKeys * kTmRows * pair, vBytes = kTmKeys * vPitch * 2;
+    static constexpr int first = pBytes > kTmWaves * vBytes ? pBytes : kTmWaves * vBytes, wBytes = heads * kTmRows * kTmKeys * 2;
+    static constexpr size_t bytes = (size_t)first + wBytes + kTmWaves * HW * 64 * 4;
+};
+
+template <int D, int HW> __global__ __launch_bounds__(kTmThreads, 1) void talk_mix_kernel(const TalkArgs a) {
+    using L = TmTile<D, HW>;
+    constexpr int HP = L::heads, KS = D / 32, ET = D / 16, NV = kTmKeys * D / 8 / 64, MT = HP / 16;
+    extern __shared__ __align__(16) char tm_lds[];
+    char *w_s = tm_lds + L::first;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
+    float *biases = reinterpret_cast<float *>(w_s + L::wBytes) + wave * HW * 64;
+    __bf16 *v_s = reinterpret_cast<__bf16 *>(tm_lds + wave * L::vBytes);
+    const int b = blockIdx.x;
+    ScoredPortion p;
+    if (!scored_portion(a, b, p)) return;
+    const int row0 = (int)(gridDim.y - 1 - blockIdx.y) * kTmRows;  // (the rows with the most keys first)
+    if (row0 >= p.n) return;
+    const int row = row0 + l16, pos = row < p.n ? p.pos0 + row : -1, first_pos = p.pos0 + row0, end = p.pos0 + min(row0 + kTmRows, p.n);
+    const int64_t mem_row = p.row0 + min(row, p.n - 1);
+    const float plain = a.scale * kScoredLog2e;
+    const int head0 = wave * HW, n_heads = max(0, min(HW, a.heads - head0));  // of this wave
+    bf8 q[HW][KS];
+    float lse[HW];
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        const int h = min(head0 + i, a.heads - 1);
+        const uint16_t *src = reinterpret_cast<const uint16_t *>(a.q1) + mem_row * a.q1_row + h * a.q1_head;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) q[i][k] = __builtin_bit_cast(bf8, scored_load16(src + 32 * k + 8 * g, 32 * k + 8 * g < a.n1));
+        lse[i] = a.lse[mem_row * a.heads + h];
+    }
+    // T: out head 16 mt + l16, in heads as the pairs' k order: first and second terms of 32 (or twice 16) heads
+    bf8 t_hi[MT], t_lo[MT];
+    bool exact = true;
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt) {
+        LaSplit sp;
+        const int out = 16 * mt + l16;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            float x[2];
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                const int in = (8 * g + 2 * j + e) % HP;
+                x[e] = out < a.heads && in < a.heads ? a.talk[(int64_t)out * a.heads + in] : 0.f;
+            }
+            la_split2(x[0], x[1], sp.hi[j], sp.lo[j]);
+            exact = exact && sp.lo[j] == 0;
+            if (HP == 16 && g >= 2) sp.lo[j] = 0;  // (the second term of T meets the first of the weights only)
+        }
+        t_hi[mt] = sp.high();
+        t_lo[mt] = sp.low();
+    }
+    const bool t_rest = __ballot(!exact) != 0;
+    f4 o[HW][ET];
+#pragma unroll
+    for (int i = 0; i < HW; ++i)
+#pragma unroll
+        for (int t = 0; t < ET; ++t) o[i][t] = f4{0.f, 0.f, 0.f, 0.f};
+
+    const int32_t *table = a.bt + b * a.bt_stride;
+    const int64_t k_tok = (int64_t)a.hkv * a.k_dim, v_tok = (int64_t)a.hkv * a.v_dim;
+    const int vreal = (a.vdim + 7) / 8 * 8;
+    auto slots_of = [&](int k0) { return scored_slot_of(a, scored_block_id(a, table, min(k0 + (lane & 31), end - 1)), k0 + (lane & 31), end); };
+    scored_u4 kr[2][KS], vr[NV];
+    auto fetch_k = [&](int kb, int kv, int slots) {  // keys 16 kb + l16
+        const int s = __shfl(slots, 16 * kb + l16, 64);
+        const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)max(s, 0) * k_tok + kv * a.k_dim + 8 * g;
+#pragma unroll
+        for (int k = 0; k < KS; ++k) kr[kb][k] = scored_load16(src + 32 * k, s >= 0 && 32 * k + 8 * g < a.n1);
+    };
+    auto fetch_v = [&](int kv, int slots) {
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const int c = lane + 64 * n, s = __shfl(slots, c / (D / 8), 64), e = c % (D / 8) * 8;
+            vr[n] = scored_load16(reinterpret_cast<const uint16_t *>(a.v) + (int64_t)max(s, 0) * v_tok + kv * a.v_dim + e, s >= 0 && e < vreal);
+        }
+    };
+    auto put_v = [&]() {
+#pragma unroll
+        for (int n = 0; n < NV; ++n) {
+            const int c = lane + 64 * n;
+            *reinterpret_cast<scored_u4 *>(v_s + c / (D / 8) * L::vPitch + c % (D / 8) * 8) = vr[n];
+        }
+    };
+    // 16-byte pieces of a pair's row and of a (head, row)'s keys at places that spread over the banks
+    auto pair_at = [&](int key, int piece) {
+        const int at = HP == 32 ? piece ^ ((l16 >> 1) & 7) : piece ^ ((l16 >> 2) & 3);
+        return tm_lds + (key * kTmRows + l16) * L::pair + 16 * at;
+    };
+    auto weights_at = [&](int head, int piece) { return w_s + (head * kTmRows + l16) * (kTmKeys * 2) + 16 * (piece ^ ((l16 >> 2) & 3)); };
+
+    const int kv0 = min(head0, a.heads - 1) / a.n_rep;
+    int slots = slots_of(0);
+    if (n_heads > 0) {
+        fetch_k(0, kv0, slots);
+        fetch_k(1, kv0, slots);
+    }
+    for (int k0 = 0; k0 < end; k0 += kTmKeys) {
+        // ---- scores and weights ----
+        if (n_heads > 0) {
+            if (a.size) {  // distances first_pos + r - k of 16 rows and 32 keys, from their smallest
+#pragma unroll
+                for (int i = 0; i < HW; ++i) {
+                    const int h = min(head0 + i, a.heads - 1);
+                    biases[i * 64 + lane] = talk_bias(a.size[h], a.rate[h], max(first_pos - (k0 + 31) + lane, 0));
+                }
+                tp_own_lds();
+            }
+            float w[2][HW][4];  // keys 16 kb + 4 g + j of row l16
+            int kv = kv0;
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if (i < n_heads) {
+                    const int own = (head0 + i) / a.n_rep;
+                    if (own != kv) {
+                        kv = own;
+                        fetch_k(0, kv, slots);
+                        fetch_k(1, kv, slots);
+                    }
+                }
+#pragma unroll
+                for (int kb = 0; kb < 2; ++kb) {
+                    f4 s = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int k = 0; k < KS; ++k) s = la_mfma(__builtin_bit_cast(bf8, kr[kb][k]), q[i][k], s);
+                    const float *bp = biases + i * 64 + l16 + 31 - 16 * kb - 4 * g;
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        const float x = a.size ? fmaf(s[j], plain, bp[-j]) : s[j] * plain;
+                        w[kb][i][j] = i < n_heads && k0 + 16 * kb + 4 * g + j <= pos ? __builtin_amdgcn_exp2f(x - lse[i]) : 0.f;
+                    }
+                }
+            }
+            fetch_v(kv0, slots);
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const int key = 16 * kb + 4 * g + j;
+                    if constexpr (HW == 4) {
+                        uint2 hi, lo;
+                        la_split2(w[kb][0][j], w[kb][1][j], hi.x, lo.x);
+                        la_split2(w[kb][2][j], w[kb][3][j], hi.y, lo.y);
+                        *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * (wave & 1)) = hi;
+                        *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * (wave & 1)) = lo;
+                    } else {
+                        uint32_t hi, lo;
+                        la_split2(w[kb][0][j], w[kb][1][j], hi, lo);
+                        *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * (wave & 3)) = hi;
+                        *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * (wave & 3)) = lo;
+                    }
+                }
+        } else {  // (no heads: zeros in their place)
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const int key = 16 * kb + 4 * g + j;
+                    if constexpr (HW == 4) {
+                        *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * (wave & 1)) = make_uint2(0, 0);
+                        *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * (wave & 1)) = make_uint2(0, 0);
+                    } else {
+                        *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * (wave & 3)) = 0;
+                        *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * (wave & 3)) = 0;
+                    }
+                }
+        }
+        __syncthreads();
+        // ---- mixed: keys 4 wave .. 4 wave + 3 of row l16, out heads 16 mt + 4 g + i ----
+        {
+            f4 x[4][MT];
+#pragma unroll
+            for (int k = 0; k < 4; ++k) {
+                const bf8 one = la_read8(reinterpret_cast<const __bf16 *>(pair_at(4 * wave + k, g)));
+#pragma unroll
+                for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(t_hi[mt], one, f4{0.f, 0.f, 0.f, 0.f});
+                if constexpr (HP == 32) {
+                    const bf8 two = la_read8(reinterpret_cast<const __bf16 *>(pair_at(4 * wave + k, 4 + g)));
+#pragma unroll
+                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(t_hi[mt], two, x[k][mt]);
+                }
+                if (t_rest) {
+#pragma unroll
+                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(t_lo[mt], one, x[k][mt]);
+                }
+            }
+#pragma unroll
+            for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    *reinterpret_cast<uint2 *>(weights_at(16 * mt + 4 * g + i, wave >> 1) + 8 * (wave & 1)) =
+                        make_uint2(row_pack_bf16(x[0][mt][i], x[1][mt][i]), row_pack_bf16(x[2][mt][i], x[3][mt][i]));
+        }
+        __syncthreads();
+        // ---- values ----
+        if (n_heads > 0) {
+            put_v();
+            const int old = slots;
+            if (k0 + kTmKeys < end) {
+                slots = slots_of(k0 + kTmKeys);
+                fetch_k(0, kv0, slots);
+                fetch_k(1, kv0, slots);
+            }
+            tp_own_lds();
+            int kv = kv0;
+#pragma unroll
+            for (int i = 0; i < HW; ++i) {
+                if (i >= n_heads) continue;
+                const int own = (head0 + i) / a.n_rep;
+                if (own != kv) {
+                    kv = own;
+                    fetch_v(kv, old);
+                    tp_own_lds();
+                    put_v();
+                    tp_own_lds();
+                }
+                const bf8 x = la_read8(reinterpret_cast<const __bf16 *>(weights_at(head0 + i, g)));
+#pragma unroll
+                for (int t = 0; t < ET; ++t) {
+                    const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::vPitch + 16 * t + 4 * (l16 & 3);
+                    o[i][t] = la_mfma(la_join(la_read_tr(va), la_read_tr(va + 4 * L::vPitch)), x, o[i][t]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    if (row >= p.n) return;
+#pragma unroll
+    for (int i = 0; i < HW; ++i) {
+        if (i >= n_heads) continue;
+        pa_bf16 *out = reinterpret_cast<pa_bf16 *>(a.out) + ((p.row0 + row) * a.heads + head0 + i) * a.vdim;
+#pragma unroll
+        for (int t = 0; t < ET; ++t) {
+            const int d = 16 * t + 4 * g;
+            if (d >= a.vdim) continue;
+            if (a.vdim % 4 == 0) {
+                *reinterpret_cast<uint2 *>(out + d) = make_uint2(row_pack_bf16(o[i][t][0], o[i][t][1]), row_pack_bf16(o[i][t][2], o[i][t][3]));
+            } else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (d + e < a.vdim) pa_scalar<pa_bf16>::store(out + d + e, o[i][t][e]);
+            }
+        }
+    }
+}
+
+template <int D, int HW> int launch_mix(const TalkArgs &a, hipStream_t s) {
+    constexpr size_t lds = TmTile<D, HW>::bytes;
+    static_assert(lds <= 160 * 1024, "LDS of one compute unit");
+    if (int rc = la_big_lds(talk_mix_kernel<D, HW>, lds, "pa_talking_attention")) return rc;
+    talk_mix_kernel<D, HW><<<dim3((unsigned)a.batch, (unsigned)((a.max_q_len + kTmRows - 1) / kTmRows)), dim3(kTmThreads), lds, s>>>(a);
+    PA_CHECK_LAUNCH("pa_talking_attention (portions)");
+    return PA_OK;
+}
+
+}  // namespace
+
+bool pa_talking_prefill_launch(const TalkArgs &a, int dtype, hipStream_t s, int &rc) {
+    const int most = a.n1 > a.vdim ? a.n1 : a.vdim;
+    const uintptr_t at = (uintptr_t)a.q1 | (uintptr_t)a.k | (uintptr_t)a.v | (uintptr_t)a.out;
+    if (dtype != PA_BF16 || !a.q_lens || most > 128 || a.heads > 32 || (at & 15u) != 0 || a.n1 % 8 != 0 || a.k_dim % 8 != 0 ||
+        a.v_dim % 8 != 0 || a.q1_row % 8 != 0 || a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff || a.bt_stride == 0)
+        return false;
+    rc = [&]() -> int {
+        const int groups = ((a.max_q_len + 31) / 32 * a.n_rep + 3) / 4;
+        PA_REQUIRE(groups <= 65535, "pa_talking_attention: max_q_len=%d is too long for one launch", a.max_q_len);
+        const dim3 grid((unsigned)a.batch, (unsigned)a.hkv, (unsigned)groups);
+        if (a.n1 <= 64) talk_sums_kernel<64><<<grid, dim3(256), 0, s>>>(a);
+        else talk_sums_kernel<128><<<grid, dim3(256), 0, s>>>(a);
+        PA_CHECK_LAUNCH("pa_talking_attention (sums)");
+        if (a.heads <= 16) return most <= 64 ? launch_mix<64, 2>(a, s) : launch_mix<128, 2>(a, s);
+        return most <= 64 ? launch_mix<64, 4>(a, s) : launch_mix<128, 4>(a, s);
+    }();
+    return true;
+}

@@ -1,6 +1,6 @@
 """Small random hybrid models for the tests: a ``config.json`` dictionary, weights under their checkpoint names, a
 checkpoint folder of both, and the oracle of the design (Lotozen here, Tevirax in tevirax_helpers.py, Vusalix in
-vusalix_helpers.py)."""
+vusalix_helpers.py, Loluzen in loluzen_helpers.py)."""
 
 import json
 import os
@@ -8,8 +8,8 @@ import os
 import numpy as np
 import torch
 
-from oracle import hybrid_oracle, tevirax_oracle, vusalix_oracle
-from tests import tevirax_helpers as tv, vusalix_helpers as vx
+from oracle import hybrid_oracle, loluzen_oracle, tevirax_oracle, vusalix_oracle
+from tests import loluzen_helpers as lz, tevirax_helpers as tv, vusalix_helpers as vx
 
 
 def attention(heads, kv_heads, dim, vdim, window, conv, rot_dims, base=1000.0, factor=1.0, scale=None, v_mix=True, ff=40):
@@ -48,11 +48,12 @@ CONFIGS = {
 
 CONFIGS.update(tv.CONFIGS)
 CONFIGS.update(vx.CONFIGS)
+CONFIGS.update(lz.CONFIGS)
 
 
 def forward(w, cfg, tokens, **kw):
     """The oracle's logits of a whole sequence."""
-    oracle = {"Lotozen": hybrid_oracle, "Tevirax": tevirax_oracle, "Vusalix": vusalix_oracle}[cfg["architecture"]]
+    oracle = {"Lotozen": hybrid_oracle, "Tevirax": tevirax_oracle, "Vusalix": vusalix_oracle, "Loluzen": loluzen_oracle}[cfg["architecture"]]
     return oracle.decoder_forward(w, cfg, tokens, **kw)
 
 
@@ -62,6 +63,8 @@ def weights(cfg, seed=0):
         return tv.weights(cfg, seed)
     if cfg["architecture"] == "Vusalix":
         return vx.weights(cfg, seed)
+    if cfg["architecture"] == "Loluzen":
+        return lz.weights(cfg, seed)
     g = torch.Generator().manual_seed(seed)
     w = {}
 
