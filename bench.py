@@ -10,7 +10,7 @@ head_dim 256 and 64; dense prefill of 64 x 512 and 4 x 8192 tokens; one chunk
 behind 200 000 cached keys at head_dim 128 and 256) under ``secondary``.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--no-secondary]
-                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen|tevirax|vusalix]
+                    [--workload c4|c2|c5|c1|c3|c3-d256|c3-d64|c3-d96|long-d128|long-d256|dense-64x512|dense-4x8192|engine|lotozen|tevirax|vusalix|loluzen]
     python bench.py --traffic-from-pmc NAME KERNEL FETCH.csv WRITE.csv   # refresh profiles/traffic.json
 """
 
@@ -102,7 +102,7 @@ def parse_args():
     ap.add_argument("--warmup", type=int, default=10)
     ap.add_argument("--workload", default="c4", choices=["c1", "c2", "c3", "c3-d256", "c3-d64", "c3-d96", "long-d128", "long-d256", "dense-64x512",
                                                          "dense-4x8192", "c4", "c5", "engine", "lotozen",
-                                                         "tevirax", "vusalix"])
+                                                         "tevirax", "vusalix", "loluzen"])
     ap.add_argument("--preheat-s", type=float, default=0.5,
                     help="seconds of untimed steps before the warmup steps: an idle GPU sits at its lowest clocks "
                          "and takes a few hundred milliseconds of work to leave them")
@@ -1399,6 +1399,179 @@ def bench_vusalix(args, dev) -> int:
     return 0
 
 
+# width; attention and talking-attention query heads, kv heads (of 128 x 128); HGRN2 heads (of 128 x 128); feed-forward without a
+# gate: one and a half times the inner width of a gated one is the same work
+LOLUZEN_SHAPES = {
+    "w2048": dict(width=2048, heads=16, kv_heads=4, r_heads=16, ff=8448),
+    "w4096": dict(width=4096, heads=32, kv_heads=8, r_heads=32, ff=21504),
+}
+
+
+def loluzen_model(p, dev, num_blocks, slots, max_positions):
+    """Parallel and attention layers in turn, three of five running twice, which makes eight runs; random weights."""
+    from research_amd.inference import HipPagedAttentionBackend, HybridConfig, HybridDecoder
+    from research_amd.inference.hybrid import LayerSpec, Loop
+    from research_amd.inference.mixers import AttentionSpec, Hgrn2Mixer, Hgrn2Spec, LlamaScaling, MLPSpec, ParallelSpec, TalkingAttention, TalkingSpec
+
+    att = AttentionSpec(heads=p["heads"], kv_heads=p["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, window=None, taps=4, rot_dims=64,
+                        rot_base=10000.0, rot_llama=LlamaScaling(8.0, 8192, 1.0, 4.0), qk_weights=True)
+    par = ParallelSpec(TalkingSpec(p["heads"], p["kv_heads"], 128, 128, 128 ** -0.5), Hgrn2Spec(p["r_heads"], 128, 128), 0.5, 0.5, norms=True)
+    ff = MLPSpec(p["ff"], "relu2")
+    cfg = HybridConfig(vocab_size=HYBRID_VOCAB, width=p["width"], norm_eps=1e-6, norm="rms", both_norms=True, norm_offset=1.0, residual_mult=0.5,
+                       loop=Loop(1, 4, 2), layers=tuple(LayerSpec(att if i % 2 else par, ff) for i in range(5)))
+    if len(cfg.runs()) != HYBRID_LAYERS:
+        raise AssertionError("as many runs as the other model has layers")
+    backend = HipPagedAttentionBackend(cfg.cache_config(num_blocks, 16, slots, torch.bfloat16, "cuda"))
+    model = HybridDecoder(cfg, backend, max_positions)
+    with torch.no_grad():
+        for q in model.parameters():
+            q.normal_(0.0, q.shape[-1] ** -0.5)
+        for m in model.modules():
+            if isinstance(m, TalkingAttention):
+                m.bias_size.uniform_(0.05, 1.5)
+                m.bias_rate.uniform_(0.05, 0.6)
+                m.talk.copy_((m.talk + torch.eye(p["heads"], device=dev)).to(torch.bfloat16))
+            if isinstance(m, Hgrn2Mixer):
+                m.lower.uniform_(0.0, 0.9)
+                m.f_bias.uniform_(-1.0, 6.0)
+    return model.eval()
+
+
+def loluzen_kernels(p, dev, steps):
+    """Every kernel of the design's blocks at the layer's shapes, against its roofline, with the like kernel of the Lotozen
+    block.  Bytes and FLOPs are the algorithmic ones: mixed heads add a product of their weights with the matrix."""
+    from research_amd import ops
+
+    bf, f32 = torch.bfloat16, torch.float32
+    rnd = lambda *s, dtype=bf: torch.randn(*s, device=dev, dtype=torch.float32).to(dtype)
+    i32 = lambda a: torch.as_tensor(np.ascontiguousarray(a), dtype=torch.int32).to(dev)
+    rows_out, add = kernel_table(steps)
+    width, heads, kv, rh, ff, d = p["width"], p["heads"], p["kv_heads"], p["r_heads"], p["ff"], 128
+    for phase, (batch, length) in (("prefill", HYBRID_PREFILL), ("decode", HYBRID_DECODE)):
+        dec = phase == "decode"
+        n = batch if dec else batch * length
+        per = length // 16 + (1 if dec else 0)
+        tables = np.random.default_rng(5).permutation(batch * per).reshape(batch, per).astype(np.int32)
+        ctx = np.full(batch, length + 1 if dec else length)
+        pos = np.full((batch, 1), length) if dec else np.tile(np.arange(length), (batch, 1))
+        slots = torch.from_numpy((np.take_along_axis(tables, pos // 16, 1).astype(np.int64) * 16 + pos % 16).reshape(-1)).to(dev)
+        bt, lens, sslots = i32(tables), i32(ctx), i32(np.arange(batch))
+        if dec:
+            por = ops.Portions(lens, sslots)
+        else:
+            first = np.arange(0, length, ops.QKV_TILE_ROWS)
+            tiles = np.stack([np.repeat(np.arange(batch), len(first)), np.tile(first, batch)], 1)
+            por = ops.Portions(lens, sslots, i32(ctx), i32(np.arange(batch) * length), i32(tiles), length)
+        # residual sums
+        x, y, z, w = rnd(n, width, dtype=f32), rnd(n, width), rnd(n, width), rnd(width, dtype=f32)
+        kw = dict(y_weight=w, y_eps=1e-6, norm="rms", weight=w, eps=1e-6)
+        add(phase, "residual + normed sum of two normed branches + norm", lambda: ops.residual_norm(x, bf, y=y, y2=(z, w, w), **kw),
+            "residual + RMS-normed branch + layer norm", n * width * 14.0)
+        add(phase, "residual + normed branch with bias + norm", lambda: ops.residual_norm(x, bf, y=y, y_bias=w, **kw),
+            "residual + RMS-normed branch + layer norm", n * width * 12.0)
+        table, ids = rnd(HYBRID_VOCAB, width), torch.randint(0, HYBRID_VOCAB, (n,), device=dev)
+        add(phase, "the same + embedding", lambda: ops.residual_norm(x, bf, y=y, y_bias=w, ids=ids, table=table, ids_add=True, **kw),
+            "residual + RMS-normed branch + layer norm", n * width * 14.0)
+        add(phase, "like: residual + RMS-normed branch + layer norm",
+            lambda: ops.residual_norm(x, bf, y=y, y_weight=w, y_eps=1e-6, norm="layer", weight=w, bias=w, eps=1e-6), "", n * width * 12.0)
+        del x, y, z, table
+        u, b = rnd(n, ff), rnd(ff, dtype=f32)
+        add(phase, "bias + square of relu", lambda: ops.bias_act(u, b, "relu2"), "silu(gate) * up", n * ff * 4.0)
+        add(phase, "like: silu(gate) * up", lambda: ops.glu(u[:, : ff // 2], u[:, ff // 2:], "silu"), "", n * ff * 3.0)
+        del u
+        # attention
+        chans = (heads + 2 * kv) * d
+        u = rnd(n, chans + heads)
+        total = batch * per * 16
+        kc, vc = rnd(total, kv, d), rnd(total, kv, d)
+        conv, cstate, bias = rnd(4, chans, dtype=f32), torch.zeros(batch, 3, chans, dtype=bf, device=dev), rnd(chans, dtype=f32)
+        rope, qn = rnd(length + 1, d // 4, 2, dtype=f32), rnd(d, dtype=f32)
+        q = torch.empty(n, heads, d, dtype=bf, device=dev)
+        lam, vf = rnd(1, dtype=f32), rnd(n, kv * d)
+        conv_bytes = n * 4.0 * chans + (batch * 12.0 * chans if dec else 0.0) + chans * 16.0
+        add(phase, "conv + q/k norm + rotation + append", lambda: ops.qkv_conv_append(u, por, slots, kc, vc, heads, d, d, 1.0, 1e-6, False, rope, d // 2,
+            conv, cstate, q_out=q, q_norm=qn, k_norm=qn), "conv + rotation + unit norm + append", conv_bytes)
+        add(phase, "like: conv + rotation + unit norm + append", lambda: ops.qkv_conv_append(u, por, slots, kc, vc, heads, d, d, 1.0, 1e-6, True, rope,
+            d // 2, conv, cstate, "mix", vf, lam, q_out=q), "", conv_bytes + n * 2.0 * kv * d)
+        add(phase, "biases + append", lambda: ops.qkv_conv_append(u, por, slots, kc, vc, heads, d, d, 1.0, 0.0, False, None, 0, None, None, q_out=q,
+            bias=bias), "conv + rotation + unit norm + append", n * 4.0 * chans)
+        o = torch.empty_like(q)
+        talk = (torch.eye(heads, device=dev) + 0.2 * rnd(heads, heads, dtype=f32)).to(bf).float()
+        size, rate = 0.05 + torch.rand(heads, device=dev), 0.05 + 0.5 * torch.rand(heads, device=dev)
+        tw = torch.empty(ops.talking_workspace_bytes(n, por, heads, kv, d, per * 16), dtype=torch.uint8, device=dev)
+        mixed = lambda: ops.talking_attention(q, kc, vc, d, por, bt, 16, d ** -0.5, talk, o, size, rate, workspace=tw)
+        if dec:
+            ws = ops.decode_workspace(q, kc)
+            moved = 4.0 * kv * d * float(ctx.sum())
+            add(phase, "attention, mixed heads", mixed, "decode attention", moved)
+            add(phase, "like: decode attention", lambda: ops.decode(q, kc, vc, bt, lens, 16, 0.1, ws, out=o), "", moved)
+        else:
+            pairs = batch * length * (length + 1) / 2.0
+            add(phase, "attention, mixed heads", mixed, "prefill attention", flops=heads * pairs * (4.0 * d + 2.0 * heads))
+            need = ops.prefill_workspace_bytes(q, bt, length, 16, kv, 0)
+            ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+            add(phase, "like: prefill attention", lambda: ops.prefill_paged(q, kc, vc, bt, lens, por.q_lens, por.q_starts, length, 16, 0.1, out=o,
+                workspace=ws if need else None), "", flops=4.0 * d * heads * pairs)
+        add(phase, "head gate", lambda: ops.head_gate(o, u[:, chans: chans + heads], d), "the same kernel", n * heads * 2.0 * (2 * d + 1))
+        del u, kc, vc, q, o, vf, tw
+        # HGRN2
+        inner = rh * d
+        u = rnd(n, 4 * inner)
+        u[:, inner: 2 * inner] += 2.5
+        state = torch.zeros(batch, rh, d, d, device=dev)
+        lower, fb = 0.9 * torch.rand(inner, device=dev), rnd(inner, dtype=f32)
+        powers = torch.full((rh, 65), 0.97, device=dev) ** torch.arange(65, device=dev)
+        o = torch.empty(n, inner, dtype=bf, device=dev)
+        bytes_r = n * inner * 8.0 + batch * rh * d * d * 8.0
+
+        def hgrn2(portions, rows_bytes, name, like):
+            nb = portions.ctx_lens.numel()
+            need = 0 if dec else max(ops.channel_linear_workspace_bytes(nb, rh, d, d, portions.max_q_len), ops.lightning_workspace_bytes(nb, rh, d, d, portions.max_q_len))
+            ws = torch.empty(max(need, 16), dtype=torch.uint8, device=dev)
+            add(phase, name, lambda: ops.channel_linear(u[:, :inner], u[:, inner: 2 * inner], u[:, 2 * inner: 3 * inner], fb, lower, portions, state, rh,
+                d, d, o, q_act="silu", workspace=ws), like, rows_bytes)
+            add(phase, "like: " + like, lambda: ops.lightning(u, portions, state, powers, rh, d, d, o, workspace=ws), "", rows_bytes)
+
+        hgrn2(por, bytes_r, "HGRN2", "lightning attention")
+        if not dec:  # one long portion alone, in segments
+            por1 = ops.Portions(i32([n]), i32([0]), i32([n]), i32([0]), None, n)
+            hgrn2(por1, n * inner * 8.0 + rh * d * d * 8.0, f"HGRN2, one sequence of {n}", "lightning attention, one sequence")
+        nw = rnd(inner, dtype=f32)
+        add(phase, "RMS norm per head", lambda: ops.rms_gate(o, None, nw, 1e-6, groups=rh, order=None), "RMS norm + sigmoid gate", n * inner * 4.0)
+        add(phase, "like: RMS norm + sigmoid gate", lambda: ops.rms_gate(o, u[:, 3 * inner:], nw, 1e-6), "", n * inner * 6.0)
+        del u, state, o
+        torch.cuda.empty_cache()
+    return rows_out
+
+
+def bench_loluzen(args, dev) -> int:
+    """Prefill and decode throughput of Loluzen-shaped models with random weights beside Lotozen-shaped ones of the same width,
+    heads, depth and feed-forward work, and the design's kernels against their rooflines.  Not the headline workload."""
+    sizes = {}
+    steps, warmup = min(args.steps, 20), min(args.warmup, 3)
+    for name, p in LOLUZEN_SHAPES.items():
+        batch, ctx_len = HYBRID_DECODE
+        blocks = batch * (ctx_len // 16 + 1)
+        model = loluzen_model(p, dev, blocks, batch, ctx_len + 16)
+        entry = {"shape": p, "loluzen": hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)}
+        del model
+        torch.cuda.empty_cache()
+        model = hybrid_model(HYBRID_SHAPES[name], dev, blocks, batch, ctx_len + 16)
+        entry["lotozen"] = hybrid_throughput(model, dev, True, steps, warmup, args.preheat_s)
+        del model
+        torch.cuda.empty_cache()
+        entry["kernels"] = loluzen_kernels(p, dev, steps)
+        sizes[name] = entry
+        print(f"[{name}] done", file=sys.stderr, flush=True)
+    main_size = sizes["w4096"]["loluzen"]
+    print(json.dumps({
+        "metric": "Loluzen prefill tokens/s", "value": main_size["prefill_tokens_per_s"], "unit": "tokens/s", "n_gpus": 1,
+        "steps": steps, "warmup": warmup, "ms_per_step": main_size["prefill_ms"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "loluzen", "layers": HYBRID_LAYERS, "prefill": HYBRID_PREFILL, "decode": HYBRID_DECODE}, "sizes": sizes}))
+    return 0
+
+
 def secondary(args, dev) -> dict:
     """Short runs of the configurations that are not the headline: what the step costs, the dominant kernel
     against its roofline and a few seconds of the CPU restatement, per workload."""
@@ -1446,6 +1619,8 @@ def main() -> int:
         return bench_tevirax(args, dev)
     if args.workload == "vusalix":
         return bench_vusalix(args, dev)
+    if args.workload == "loluzen":
+        return bench_loluzen(args, dev)
     if args.workload in PREFILL_HEAD_SHAPES:
         result = bench_prefill_head(args, dev, args.workload)
     elif args.workload in PREFILL_LONG_SHAPES:
