@@ -8,7 +8,7 @@
 //   1. S^T = K Q^T leaves a lane four keys of one row per head; the weights go to LDS, all heads of a (key, row) pair side by
 //      side, as two bf16 terms;
 //   2. T times these, the pairs of four keys per wave, and back to LDS as weights of (head, row), keys side by side;
-//   3. O^T += V^T W^T per head, V by transposing reads from the wave's own part of LDS (which is the weights' of step 1).
+//   3. O^T += V^T W^T per head, V by transposing reads from the wave's own part of LDS, 64 columns at a time.
 // Distance biases of a head are one logarithm per lane and tile, spread by LDS.
 #include "linear_tiles.h"
 #include "prefill_mfma.h"
@@ -133,97 +133,98 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
 }
 
 // ------------------------------------------------------------------ mixed weights times values
-constexpr int kTmRows = 16, kTmKeys = 32, kTmWaves = 8, kTmThreads = 64 * kTmWaves;
+constexpr int kTmRows = 16, kTmKeys = 32, kTmWaves = 8, kTmThreads = 64 * kTmWaves, kTmCols = 64;
 
-// D: keys and values padded to 64 or 128; HW: heads per wave, 2 or 4.
-template <int D, int HW> struct TmTile {
-    static constexpr int heads = kTmWaves * HW, vPitch = D + 8;
-    static constexpr int pair = 4 * heads;                                      // bytes of a (key, row) pair: both terms of all heads
-    static constexpr int pBytes = kTmKeys * kTmRows * pair, vBytes = kTmKeys * vPitch * 2;
-    static constexpr int first = pBytes > kTmWaves * vBytes ? pBytes : kTmWaves * vBytes, wBytes = heads * kTmRows * kTmKeys * 2;
-    static constexpr size_t bytes = (size_t)first + wBytes + kTmWaves * HW * 64 * 4;
+// HW: heads per wave, 2 or 4.  Weights, mixed weights, a wave's value columns (64 at a time), biases, T
+template <int HW> struct TmTile {
+    static constexpr int heads = kTmWaves * HW, vPitch = kTmCols + 8;
+    static constexpr int pair = 4 * heads;  // bytes of a (key, row) pair: both terms of all heads
+    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = heads * kTmRows * kTmKeys * 2, vBytes = kTmKeys * vPitch * 2;
+    static constexpr int biasFloats = HW * 64, tElems = heads * 32;  // (one term of T)
+    static constexpr size_t bytes = (size_t)pBytes + wBytes + kTmWaves * vBytes + kTmWaves * biasFloats * 4 + 2 * tElems * 2;
 };
 
-template <int D, int HW> __global__ __launch_bounds__(kTmThreads, 1) void talk_mix_kernel(const TalkArgs a) {
-    using L = TmTile<D, HW>;
-    constexpr int HP = L::heads, KS = D / 32, ET = D / 16, NV = kTmKeys * D / 8 / 64, MT = HP / 16;
+// D: keys and values padded to 64 or 128; FULL: they fill it.  SAME: a wave's heads share a kv head.
+template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmThreads) void talk_mix_kernel(const TalkArgs a) {
+    using L = TmTile<HW>;
+    constexpr int HP = L::heads, KS = D / 32, MT = HP / 16, NV = kTmKeys * kTmCols / 8 / 64, CT = kTmCols / 16, NC = D / kTmCols;
     extern __shared__ __align__(16) char tm_lds[];
-    char *w_s = tm_lds + L::first;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
-    float *biases = reinterpret_cast<float *>(w_s + L::wBytes) + wave * HW * 64;
-    __bf16 *v_s = reinterpret_cast<__bf16 *>(tm_lds + wave * L::vBytes);
+    char *w_s = tm_lds + L::pBytes;
+    __bf16 *v_s = reinterpret_cast<__bf16 *>(w_s + L::wBytes + wave * L::vBytes);
+    float *biases = reinterpret_cast<float *>(w_s + L::wBytes + kTmWaves * L::vBytes) + wave * L::biasFloats;
+    __bf16 *t_s = reinterpret_cast<__bf16 *>(w_s + L::wBytes + kTmWaves * (L::vBytes + L::biasFloats * 4));
     const int b = blockIdx.x;
     ScoredPortion p;
     if (!scored_portion(a, b, p)) return;
     const int row0 = (int)(gridDim.y - 1 - blockIdx.y) * kTmRows;  // (the rows with the most keys first)
     if (row0 >= p.n) return;
     const int row = row0 + l16, pos = row < p.n ? p.pos0 + row : -1, first_pos = p.pos0 + row0, end = p.pos0 + min(row0 + kTmRows, p.n);
-    const int64_t mem_row = p.row0 + min(row, p.n - 1);
     const float plain = a.scale * kScoredLog2e;
     const int head0 = wave * HW, n_heads = max(0, min(HW, a.heads - head0));  // of this wave
+    // T in the pairs' k order (terms of 32 heads, or both of 16): row = out head, 16 mt + l16; the second term of T meets the
+    // first of the weights only
+    bool exact = true;
+    for (int i = tid; i < L::tElems; i += kTmThreads) {
+        const int out = i / 32, in = i % 32 % HP;
+        const float x = out < a.heads && in < a.heads ? a.talk[(int64_t)out * a.heads + in] : 0.f;
+        const __bf16 hi = (__bf16)x, lo = (__bf16)(x - (float)hi);
+        exact = exact && (float)lo == 0.f;
+        t_s[i] = hi;
+        t_s[L::tElems + i] = HP == 16 && i % 32 >= 16 ? (__bf16)0.f : lo;
+    }
+    const bool t_rest = __syncthreads_or(!exact);  // (a matrix stored in 16 bits has no second term)
     bf8 q[HW][KS];
     float lse[HW];
+    {
+        const int64_t mem_row = p.row0 + min(row, p.n - 1);
 #pragma unroll
-    for (int i = 0; i < HW; ++i) {
-        const int h = min(head0 + i, a.heads - 1);
-        const uint16_t *src = reinterpret_cast<const uint16_t *>(a.q1) + mem_row * a.q1_row + h * a.q1_head;
+        for (int i = 0; i < HW; ++i) {
+            const int h = min(head0 + i, a.heads - 1);
+            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.q1) + mem_row * a.q1_row + h * a.q1_head;
 #pragma unroll
-        for (int k = 0; k < KS; ++k) q[i][k] = __builtin_bit_cast(bf8, scored_load16(src + 32 * k + 8 * g, 32 * k + 8 * g < a.n1));
-        lse[i] = a.lse[mem_row * a.heads + h];
-    }
-    // T: out head 16 mt + l16, in heads as the pairs' k order: first and second terms of 32 (or twice 16) heads
-    bf8 t_hi[MT], t_lo[MT];
-    bool exact = true;
-#pragma unroll
-    for (int mt = 0; mt < MT; ++mt) {
-        LaSplit sp;
-        const int out = 16 * mt + l16;
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            float x[2];
-#pragma unroll
-            for (int e = 0; e < 2; ++e) {
-                const int in = (8 * g + 2 * j + e) % HP;
-                x[e] = out < a.heads && in < a.heads ? a.talk[(int64_t)out * a.heads + in] : 0.f;
-            }
-            la_split2(x[0], x[1], sp.hi[j], sp.lo[j]);
-            exact = exact && sp.lo[j] == 0;
-            if (HP == 16 && g >= 2) sp.lo[j] = 0;  // (the second term of T meets the first of the weights only)
+            for (int k = 0; k < KS; ++k) q[i][k] = __builtin_bit_cast(bf8, scored_load16(src + 32 * k + 8 * g, 32 * k + 8 * g < a.n1));
+            lse[i] = a.lse[mem_row * a.heads + h];
         }
-        t_hi[mt] = sp.high();
-        t_lo[mt] = sp.low();
     }
-    const bool t_rest = __ballot(!exact) != 0;
-    f4 o[HW][ET];
+    f4 o[HW][NC][CT];
 #pragma unroll
     for (int i = 0; i < HW; ++i)
 #pragma unroll
-        for (int t = 0; t < ET; ++t) o[i][t] = f4{0.f, 0.f, 0.f, 0.f};
+        for (int c = 0; c < NC; ++c)
+#pragma unroll
+            for (int t = 0; t < CT; ++t) o[i][c][t] = f4{0.f, 0.f, 0.f, 0.f};
 
     const int32_t *table = a.bt + b * a.bt_stride;
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim, v_tok = (int64_t)a.hkv * a.v_dim;
     const int vreal = (a.vdim + 7) / 8 * 8;
-    auto slots_of = [&](int k0) { return scored_slot_of(a, scored_block_id(a, table, min(k0 + (lane & 31), end - 1)), k0 + (lane & 31), end); };
-    scored_u4 kr[2][KS], vr[NV];
-    auto fetch_k = [&](int kb, int kv, int slots) {  // keys 16 kb + l16
-        const int s = __shfl(slots, 16 * kb + l16, 64);
-        const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)max(s, 0) * k_tok + kv * a.k_dim + 8 * g;
-#pragma unroll
-        for (int k = 0; k < KS; ++k) kr[kb][k] = scored_load16(src + 32 * k, s >= 0 && 32 * k + 8 * g < a.n1);
+    // pool row of key k0 + lane % 32 (past the last key: the last one's, which nothing weighs)
+    auto slots_of = [&](int k0) {
+        const int key = min(k0 + (lane & 31), end - 1);
+        return scored_slot_of(a, scored_block_id(a, table, key), key, end);
     };
-    auto fetch_v = [&](int kv, int slots) {
+    scored_u4 kr[2][KS], vr[NV];
+    auto fetch_k = [&](int kv, int slots) {  // keys 16 kb + l16
+#pragma unroll
+        for (int kb = 0; kb < 2; ++kb) {
+            const int s = __shfl(slots, 16 * kb + l16, 64);
+            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)max(s, 0) * k_tok + kv * a.k_dim + 8 * g;
+#pragma unroll
+            for (int k = 0; k < KS; ++k) kr[kb][k] = FULL ? *reinterpret_cast<const scored_u4 *>(src + 32 * k) : scored_load16(src + 32 * k, 32 * k + 8 * g < a.n1);
+        }
+    };
+    auto fetch_v = [&](int kv, int slots, int c) {  // columns 64 c ..
+        const int e = kTmCols * c + lane % 8 * 8;
 #pragma unroll
         for (int n = 0; n < NV; ++n) {
-            const int c = lane + 64 * n, s = __shfl(slots, c / (D / 8), 64), e = c % (D / 8) * 8;
-            vr[n] = scored_load16(reinterpret_cast<const uint16_t *>(a.v) + (int64_t)max(s, 0) * v_tok + kv * a.v_dim + e, s >= 0 && e < vreal);
+            const int s = __shfl(slots, 8 * n + lane / 8, 64);
+            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.v) + (int64_t)max(s, 0) * v_tok + kv * a.v_dim + e;
+            vr[n] = FULL ? *reinterpret_cast<const scored_u4 *>(src) : scored_load16(src, e < vreal);
         }
     };
     auto put_v = [&]() {
 #pragma unroll
-        for (int n = 0; n < NV; ++n) {
-            const int c = lane + 64 * n;
-            *reinterpret_cast<scored_u4 *>(v_s + c / (D / 8) * L::vPitch + c % (D / 8) * 8) = vr[n];
-        }
+        for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + (8 * n + lane / 8) * L::vPitch + lane % 8 * 8) = vr[n];
     };
     // 16-byte pieces of a pair's row and of a (head, row)'s keys at places that spread over the banks
     auto pair_at = [&](int key, int piece) {
@@ -231,141 +232,168 @@ template <int D, int HW> __global__ __launch_bounds__(kTmThreads, 1) void talk_m
         return tm_lds + (key * kTmRows + l16) * L::pair + 16 * at;
     };
     auto weights_at = [&](int head, int piece) { return w_s + (head * kTmRows + l16) * (kTmKeys * 2) + 16 * (piece ^ ((l16 >> 2) & 3)); };
+    auto kv_of = [&](int i) { return min(head0 + i, a.heads - 1) / a.n_rep; };
 
-    const int kv0 = min(head0, a.heads - 1) / a.n_rep;
+    const int kv0 = kv_of(0);
     int slots = slots_of(0);
-    if (n_heads > 0) {
-        fetch_k(0, kv0, slots);
-        fetch_k(1, kv0, slots);
-    }
+    if (n_heads > 0) fetch_k(kv0, slots);
     for (int k0 = 0; k0 < end; k0 += kTmKeys) {
-        // ---- scores and weights ----
-        if (n_heads > 0) {
-            if (a.size) {  // distances first_pos + r - k of 16 rows and 32 keys, from their smallest
+        // ---- scores and weights of keys 16 kb + 4 g + j of row l16 ----
+        if (a.size) {  // distances first_pos + r - k of 16 rows and 32 keys, from their smallest
 #pragma unroll
-                for (int i = 0; i < HW; ++i) {
-                    const int h = min(head0 + i, a.heads - 1);
-                    biases[i * 64 + lane] = talk_bias(a.size[h], a.rate[h], max(first_pos - (k0 + 31) + lane, 0));
-                }
-                tp_own_lds();
+            for (int i = 0; i < HW; ++i) {
+                const int h = min(head0 + i, a.heads - 1);
+                biases[i * 64 + lane] = talk_bias(a.size[h], a.rate[h], max(first_pos - (k0 + 31) + lane, 0));
             }
-            float w[2][HW][4];  // keys 16 kb + 4 g + j of row l16
+            tp_own_lds();
+        }
+        auto weights = [&](int i, int kb, f4 s, float *w) {
+            const float *bp = biases + i * 64 + l16 + 31 - 16 * kb - 4 * g;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const float x = a.size ? fmaf(s[j], plain, bp[-j]) : s[j] * plain;
+                w[j] = i < n_heads && k0 + 16 * kb + 4 * g + j <= pos ? __builtin_amdgcn_exp2f(x - lse[i]) : 0.f;
+            }
+        };
+        auto put = [&](int kb, float (*w)[4]) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int key = 16 * kb + 4 * g + j;
+                if constexpr (HW == 4) {
+                    uint2 hi, lo;
+                    la_split2(w[0][j], w[1][j], hi.x, lo.x);
+                    la_split2(w[2][j], w[3][j], hi.y, lo.y);
+                    *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * (wave & 1)) = hi;
+                    *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * (wave & 1)) = lo;
+                } else {
+                    uint32_t hi, lo;
+                    la_split2(w[0][j], w[1][j], hi, lo);
+                    *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * (wave & 3)) = hi;
+                    *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * (wave & 3)) = lo;
+                }
+            }
+        };
+        if constexpr (SAME) {
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb) {
+                float w[HW][4];
+                f4 s[HW];
+#pragma unroll
+                for (int i = 0; i < HW; ++i) s[i] = f4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int k = 0; k < KS; ++k)
+#pragma unroll
+                    for (int i = 0; i < HW; ++i) s[i] = la_mfma(__builtin_bit_cast(bf8, kr[kb][k]), q[i][k], s[i]);
+#pragma unroll
+                for (int i = 0; i < HW; ++i) weights(i, kb, s[i], w[i]);
+                put(kb, w);
+                __builtin_amdgcn_sched_barrier(0);
+            }
+        } else {
+            float w[2][HW][4];
             int kv = kv0;
 #pragma unroll
             for (int i = 0; i < HW; ++i) {
-                if (i < n_heads) {
-                    const int own = (head0 + i) / a.n_rep;
-                    if (own != kv) {
-                        kv = own;
-                        fetch_k(0, kv, slots);
-                        fetch_k(1, kv, slots);
-                    }
-                }
+                if (kv_of(i) != kv) fetch_k(kv = kv_of(i), slots);
 #pragma unroll
                 for (int kb = 0; kb < 2; ++kb) {
                     f4 s = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
                     for (int k = 0; k < KS; ++k) s = la_mfma(__builtin_bit_cast(bf8, kr[kb][k]), q[i][k], s);
-                    const float *bp = biases + i * 64 + l16 + 31 - 16 * kb - 4 * g;
-#pragma unroll
-                    for (int j = 0; j < 4; ++j) {
-                        const float x = a.size ? fmaf(s[j], plain, bp[-j]) : s[j] * plain;
-                        w[kb][i][j] = i < n_heads && k0 + 16 * kb + 4 * g + j <= pos ? __builtin_amdgcn_exp2f(x - lse[i]) : 0.f;
-                    }
+                    weights(i, kb, s, w[kb][i]);
                 }
             }
-            fetch_v(kv0, slots);
-#pragma unroll
-            for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-                for (int j = 0; j < 4; ++j) {
-                    const int key = 16 * kb + 4 * g + j;
-                    if constexpr (HW == 4) {
-                        uint2 hi, lo;
-                        la_split2(w[kb][0][j], w[kb][1][j], hi.x, lo.x);
-                        la_split2(w[kb][2][j], w[kb][3][j], hi.y, lo.y);
-                        *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * (wave & 1)) = hi;
-                        *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * (wave & 1)) = lo;
-                    } else {
-                        uint32_t hi, lo;
-                        la_split2(w[kb][0][j], w[kb][1][j], hi, lo);
-                        *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * (wave & 3)) = hi;
-                        *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * (wave & 3)) = lo;
-                    }
-                }
-        } else {  // (no heads: zeros in their place)
-#pragma unroll
-            for (int kb = 0; kb < 2; ++kb)
-#pragma unroll
-                for (int j = 0; j < 4; ++j) {
-                    const int key = 16 * kb + 4 * g + j;
-                    if constexpr (HW == 4) {
-                        *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * (wave & 1)) = make_uint2(0, 0);
-                        *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * (wave & 1)) = make_uint2(0, 0);
-                    } else {
-                        *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * (wave & 3)) = 0;
-                        *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * (wave & 3)) = 0;
-                    }
-                }
+            put(0, w[0]);
+            put(1, w[1]);
         }
+        fetch_v(kv0, slots, 0);
         __syncthreads();
         // ---- mixed: keys 4 wave .. 4 wave + 3 of row l16, out heads 16 mt + 4 g + i ----
-        {
-            f4 x[4][MT];
 #pragma unroll
-            for (int k = 0; k < 4; ++k) {
-                const bf8 one = la_read8(reinterpret_cast<const __bf16 *>(pair_at(4 * wave + k, g)));
+        for (int half = 0; half < 2; ++half) {
+            f4 x[2][MT];
 #pragma unroll
-                for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(t_hi[mt], one, f4{0.f, 0.f, 0.f, 0.f});
+            for (int k = 0; k < 2; ++k) {
+                const int key = 4 * wave + 2 * half + k;
+                const bf8 one = la_read8(reinterpret_cast<const __bf16 *>(pair_at(key, g)));
+#pragma unroll
+                for (int mt = 0; mt < MT; ++mt)
+                    x[k][mt] = la_mfma(la_read8(t_s + (16 * mt + l16) * 32 + 8 * g), one, f4{0.f, 0.f, 0.f, 0.f});
                 if constexpr (HP == 32) {
-                    const bf8 two = la_read8(reinterpret_cast<const __bf16 *>(pair_at(4 * wave + k, 4 + g)));
+                    const bf8 two = la_read8(reinterpret_cast<const __bf16 *>(pair_at(key, 4 + g)));
 #pragma unroll
-                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(t_hi[mt], two, x[k][mt]);
+                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(la_read8(t_s + (16 * mt + l16) * 32 + 8 * g), two, x[k][mt]);
                 }
                 if (t_rest) {
 #pragma unroll
-                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(t_lo[mt], one, x[k][mt]);
+                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(la_read8(t_s + L::tElems + (16 * mt + l16) * 32 + 8 * g), one, x[k][mt]);
                 }
             }
 #pragma unroll
             for (int mt = 0; mt < MT; ++mt)
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
-                    *reinterpret_cast<uint2 *>(weights_at(16 * mt + 4 * g + i, wave >> 1) + 8 * (wave & 1)) =
-                        make_uint2(row_pack_bf16(x[0][mt][i], x[1][mt][i]), row_pack_bf16(x[2][mt][i], x[3][mt][i]));
+                    *reinterpret_cast<uint32_t *>(weights_at(16 * mt + 4 * g + i, wave >> 1) + 8 * (wave & 1) + 4 * half) = row_pack_bf16(x[0][mt][i], x[1][mt][i]);
+            __builtin_amdgcn_sched_barrier(0);
         }
+        // ---- values: 64 columns at a time ----
+        const int now = slots;
+        put_v();
+        if (NC > 1) fetch_v(kv0, now, NC - 1);
         __syncthreads();
-        // ---- values ----
-        if (n_heads > 0) {
-            put_v();
-            const int old = slots;
-            if (k0 + kTmKeys < end) {
-                slots = slots_of(k0 + kTmKeys);
-                fetch_k(0, kv0, slots);
-                fetch_k(1, kv0, slots);
-            }
-            tp_own_lds();
-            int kv = kv0;
+        auto weights_of = [&](int i) { return la_read8(reinterpret_cast<const __bf16 *>(weights_at(head0 + i, g))); };
+        auto values = [&](int t) {
+            const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::vPitch + 16 * t + 4 * (l16 & 3);
+            return la_join(la_read_tr(va), la_read_tr(va + 4 * L::vPitch));
+        };
+        if constexpr (SAME) {
+            bf8 x[HW];
 #pragma unroll
-            for (int i = 0; i < HW; ++i) {
-                if (i >= n_heads) continue;
-                const int own = (head0 + i) / a.n_rep;
-                if (own != kv) {
-                    kv = own;
-                    fetch_v(kv, old);
+            for (int i = 0; i < HW; ++i) x[i] = weights_of(i);
+#pragma unroll
+            for (int c = 0; c < NC; ++c) {
+                if (c > 0) {
                     tp_own_lds();
                     put_v();
                     tp_own_lds();
                 }
-                const bf8 x = la_read8(reinterpret_cast<const __bf16 *>(weights_at(head0 + i, g)));
-#pragma unroll
-                for (int t = 0; t < ET; ++t) {
-                    const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::vPitch + 16 * t + 4 * (l16 & 3);
-                    o[i][t] = la_mfma(la_join(la_read_tr(va), la_read_tr(va + 4 * L::vPitch)), x, o[i][t]);
+                if (c == NC - 1 && k0 + kTmKeys < end) {
+                    slots = slots_of(k0 + kTmKeys);
+                    if (n_heads > 0) fetch_k(kv0, slots);
                 }
+#pragma unroll
+                for (int t = 0; t < CT; ++t) {
+                    const bf8 v = values(t);
+#pragma unroll
+                    for (int i = 0; i < HW; ++i) o[i][c][t] = la_mfma(v, x[i], o[i][c][t]);
+                }
+                __builtin_amdgcn_sched_barrier(0);
+            }
+        } else {
+            int have = kv0, part = 0;  // what v_s holds
+            bool waiting = NC > 1;     // its last columns are in registers
+#pragma unroll
+            for (int i = 0; i < HW; ++i)
+#pragma unroll
+                for (int c = 0; c < NC; ++c) {
+                    if (have != kv_of(i) || part != c) {
+                        if (!(waiting && kv_of(i) == kv0 && c == NC - 1)) fetch_v(kv_of(i), now, c);
+                        waiting = false;
+                        have = kv_of(i);
+                        part = c;
+                        tp_own_lds();
+                        put_v();
+                        tp_own_lds();
+                    }
+                    const bf8 x = weights_of(i);
+#pragma unroll
+                    for (int t = 0; t < CT; ++t) o[i][c][t] = la_mfma(values(t), x, o[i][c][t]);
+                }
+            if (k0 + kTmKeys < end) {
+                slots = slots_of(k0 + kTmKeys);
+                fetch_k(kv0, slots);
             }
         }
-        __syncthreads();
     }
     if (row >= p.n) return;
 #pragma unroll
@@ -373,27 +401,35 @@ template <int D, int HW> __global__ __launch_bounds__(kTmThreads, 1) void talk_m
         if (i >= n_heads) continue;
         pa_bf16 *out = reinterpret_cast<pa_bf16 *>(a.out) + ((p.row0 + row) * a.heads + head0 + i) * a.vdim;
 #pragma unroll
-        for (int t = 0; t < ET; ++t) {
-            const int d = 16 * t + 4 * g;
-            if (d >= a.vdim) continue;
-            if (a.vdim % 4 == 0) {
-                *reinterpret_cast<uint2 *>(out + d) = make_uint2(row_pack_bf16(o[i][t][0], o[i][t][1]), row_pack_bf16(o[i][t][2], o[i][t][3]));
-            } else {
+        for (int c = 0; c < NC; ++c)
 #pragma unroll
-                for (int e = 0; e < 4; ++e)
-                    if (d + e < a.vdim) pa_scalar<pa_bf16>::store(out + d + e, o[i][t][e]);
+            for (int t = 0; t < CT; ++t) {
+                const f4 x = o[i][c][t];
+                const int d = kTmCols * c + 16 * t + 4 * g;
+                if (d >= a.vdim) continue;
+                if (FULL || a.vdim % 4 == 0) {
+                    *reinterpret_cast<uint2 *>(out + d) = make_uint2(row_pack_bf16(x[0], x[1]), row_pack_bf16(x[2], x[3]));
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (d + e < a.vdim) pa_scalar<pa_bf16>::store(out + d + e, x[e]);
+                }
             }
-        }
     }
 }
 
-template <int D, int HW> int launch_mix(const TalkArgs &a, hipStream_t s) {
-    constexpr size_t lds = TmTile<D, HW>::bytes;
+template <int D, int HW, bool FULL, bool SAME> int launch_mix(const TalkArgs &a, hipStream_t s) {
+    constexpr size_t lds = TmTile<HW>::bytes;
     static_assert(lds <= 160 * 1024, "LDS of one compute unit");
-    if (int rc = la_big_lds(talk_mix_kernel<D, HW>, lds, "pa_talking_attention")) return rc;
-    talk_mix_kernel<D, HW><<<dim3((unsigned)a.batch, (unsigned)((a.max_q_len + kTmRows - 1) / kTmRows)), dim3(kTmThreads), lds, s>>>(a);
+    if (int rc = la_big_lds(talk_mix_kernel<D, HW, FULL, SAME>, lds, "pa_talking_attention")) return rc;
+    talk_mix_kernel<D, HW, FULL, SAME><<<dim3((unsigned)a.batch, (unsigned)((a.max_q_len + kTmRows - 1) / kTmRows)), dim3(kTmThreads), lds, s>>>(a);
     PA_CHECK_LAUNCH("pa_talking_attention (portions)");
     return PA_OK;
+}
+template <int D, int HW> int launch_mix_size(const TalkArgs &a, hipStream_t s) {
+    const bool full = a.n1 == D && a.vdim == D, same = a.n_rep % HW == 0;
+    if (!same) return launch_mix<D, HW, false, false>(a, s);
+    return full ? launch_mix<D, HW, true, true>(a, s) : launch_mix<D, HW, false, true>(a, s);
 }
 
 }  // namespace
@@ -411,8 +447,8 @@ bool pa_talking_prefill_launch(const TalkArgs &a, int dtype, hipStream_t s, int 
         if (a.n1 <= 64) talk_sums_kernel<64><<<grid, dim3(256), 0, s>>>(a);
         else talk_sums_kernel<128><<<grid, dim3(256), 0, s>>>(a);
         PA_CHECK_LAUNCH("pa_talking_attention (sums)");
-        if (a.heads <= 16) return most <= 64 ? launch_mix<64, 2>(a, s) : launch_mix<128, 2>(a, s);
-        return most <= 64 ? launch_mix<64, 4>(a, s) : launch_mix<128, 4>(a, s);
+        if (a.heads <= 16) return most <= 64 ? launch_mix_size<64, 2>(a, s) : launch_mix_size<128, 2>(a, s);
+        return most <= 64 ? launch_mix_size<64, 4>(a, s) : launch_mix_size<128, 4>(a, s);
     }();
     return true;
 }
