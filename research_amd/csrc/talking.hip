@@ -149,6 +149,7 @@ extern "C" int pa_talking_attention(const void *q, int64_t q_row, int64_t q_head
     a.ctx_lens = ctx_lens; a.q_lens = q_lens; a.q_starts = q_starts; a.n_rows = n_rows; a.batch = batch;
     a.max_q_len = q_lens ? max_q_len : 1; a.heads = num_q_heads; a.hkv = num_kv_heads; a.n_rep = num_q_heads / num_kv_heads;
     a.scale = scale; a.out = out; a.splits = 1;
+    a.bs_shift = (block_size & (block_size - 1)) == 0 ? __builtin_ctz((unsigned)block_size) : -1;
     a.size = bias_size; a.rate = bias_rate; a.talk = talk; a.lse = (float *)workspace;
     hipStream_t s = (hipStream_t)stream;
     int rc = PA_OK;

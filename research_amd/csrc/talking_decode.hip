@@ -45,7 +45,7 @@ template <int KC> __global__ __launch_bounds__(256) void talk_scores_kernel(cons
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim;
     scored_u4 x[2][KC / 32];
     auto fetch = [&](scored_u4 *to, int key) {
-        const int slot = scored_slot_of(a, scored_block_id(a, table, min(key, p.end - 1)), key, p.end);
+        const int slot = talk_slot_of(a, talk_block_id(a, table, min(key, p.end - 1)), key, p.end);
         const uint16_t *src = kp + (int64_t)max(slot, 0) * k_tok;
 #pragma unroll
         for (int kk = 0; kk < KC / 32; ++kk) to[kk] = scored_load16(src + 32 * kk, slot >= 0 && 32 * kk + 8 * g < a.n1);
@@ -160,9 +160,9 @@ template <int VC, int HP> __global__ __launch_bounds__(256) void talk_values_ker
     const float *src = a.scores + (int64_t)b * a.heads * a.keys_cap;
     scored_u4 vr[kVL];
     f4 sr[kPL];
-    auto id_of = [&](int k0) { return scored_block_id(a, table, min(k0 + lane, p.end - 1)); };
+    auto id_of = [&](int k0) { return talk_block_id(a, table, min(k0 + lane, p.end - 1)); };
     auto fetch = [&](int id, int k0) {
-        const int slots = scored_slot_of(a, id, k0 + lane, p.end);
+        const int slots = talk_slot_of(a, id, k0 + lane, p.end);
 #pragma unroll
         for (int n = 0; n < kVL; ++n) {
             const int c = tid + 256 * n, s = __shfl(slots, c / (VC / 8), 64), e = c % (VC / 8) * 8;

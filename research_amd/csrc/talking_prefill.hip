@@ -3,13 +3,14 @@
 //
 // The first kernel leaves every row's and head's sum: a wave owns 32 rows of one head, a workgroup four (row block, head) pairs
 // of one kv head, which share tiles of 64 keys in LDS (as in scored_prefill.hip, without values).  The second one makes the
-// scores again, for all heads at once: a workgroup owns 16 rows, its eight waves have their own heads, queries and value
-// accumulators in registers.  Per tile of 32 keys
+// scores again, for all heads at once: a workgroup owns 16 rows and 16 out heads, its eight waves have their own heads' queries
+// and two out heads' accumulators in registers.  Per tile of 32 keys
 //   1. S^T = K Q^T leaves a lane four keys of one row per head; the weights go to LDS, all heads of a (key, row) pair side by
 //      side, as two bf16 terms;
-//   2. T times these, the pairs of four keys per wave, and back to LDS as weights of (head, row), keys side by side;
-//   3. O^T += V^T W^T per head, V by transposing reads from the wave's own part of LDS, 64 columns at a time.
-// Distance biases of a head are one logarithm per lane and tile, spread by LDS.
+//   2. T times these, the pairs of four keys per wave, and back to LDS as weights of (out head, row), keys side by side;
+//   3. O^T += V^T W^T per out head, V by transposing reads from the wave's own part of LDS.
+// The next tile's keys and values are on their way in registers.  Distance biases of a head are one logarithm per lane and
+// tile, spread by LDS.
 #include "linear_tiles.h"
 #include "prefill_mfma.h"
 #include "talking.h"
@@ -43,7 +44,7 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
     const int task = group * 4 + wave, last_task = min(n_tasks, group * 4 + 4) - 1;
     const bool live = task < n_tasks;
     const int row0 = (live ? task / a.n_rep : 0) * 32, h = kvh * a.n_rep + (live ? task % a.n_rep : 0);
-    const int row = row0 + col, pos = p.pos0 + min(row, p.n - 1), wave_hi = p.pos0 + min(row0 + 32, p.n);
+    const int row = row0 + col, wave_hi = p.pos0 + min(row0 + 32, p.n);
     const int wg_hi = p.pos0 + min(last_task / a.n_rep * 32 + 32, p.n);
     const float plain = a.scale * kScoredLog2e, size = a.size ? a.size[h] : 0.f, rate = a.rate ? a.rate[h] : 0.f;
     X8 q[KS];
@@ -59,10 +60,10 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
     const int32_t *table = a.bt + b * a.bt_stride;
     const uint16_t *kp = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)kvh * a.k_dim;
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim;
-    auto id_of = [&](int k0) { return scored_block_id(a, table, min(k0 + lane, wg_hi - 1)); };
+    auto id_of = [&](int k0) { return talk_block_id(a, table, min(k0 + lane, wg_hi - 1)); };
     scored_u4 kr[NK];
     auto fetch = [&](int id, int k0) {
-        const int slots = scored_slot_of(a, id, k0 + lane, wg_hi);
+        const int slots = talk_slot_of(a, id, k0 + lane, wg_hi);
 #pragma unroll
         for (int n = 0; n < NK; ++n) {
             const int c = tid + 256 * n, s = __shfl(slots, c / (DK / 8), 64), e = c % (DK / 8) * 8;
@@ -82,10 +83,10 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
             fetch(id, k0 + kTsKeys);
             id = id_of(k0 + 2 * kTsKeys);
         }
-        if (live && k0 < wave_hi && a.size) {  // distances p.pos0 + row0 + i - k of i < 32 and each half's 32 keys, from their smallest
+        if (live && k0 < wave_hi) {  // distances p.pos0 + row0 + i - k of i < 32 and each half's 32 keys, from their smallest
 #pragma unroll
             for (int sub = 0; sub < 2; ++sub)
-                biases[wave][sub][lane] = talk_bias(size, rate, max(p.pos0 + row0 - (k0 + 32 * sub + 31) + lane, 0));
+                biases[wave][sub][lane] = talk_masked_bias(size, rate, p.pos0 + row0 - (k0 + 32 * sub + 31) + lane);
             tp_own_lds();
         }
 #pragma unroll
@@ -99,19 +100,9 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
             for (int k = 0; k < KS; ++k)
                 s = M::mma(__builtin_bit_cast(X8, *reinterpret_cast<const uint4 *>(ks + (32 * sub + col) * kPitch + 16 * k + 8 * half)), q[k], s);
             // element i: key kb + 8 (i / 4) + 4 half + i % 4
-            if (a.size) {
-                const float *bp = biases[wave][sub] + col + 31 - 4 * half;
+            const float *bp = biases[wave][sub] + col + 31 - 4 * half;
 #pragma unroll
-                for (int i = 0; i < 16; ++i) s[i] = fmaf(s[i], plain, bp[-(8 * (i >> 2) + (i & 3))]);
-            } else {
-#pragma unroll
-                for (int i = 0; i < 16; ++i) s[i] *= plain;
-            }
-            if (kb + 31 > p.pos0 + row0) {
-                const int hi = pos - kb - 4 * half;
-#pragma unroll
-                for (int i = 0; i < 16; ++i) s[i] = 8 * (i >> 2) + (i & 3) <= hi ? s[i] : kScoredNone;
-            }
+            for (int i = 0; i < 16; ++i) s[i] = fmaf(s[i], plain, bp[-(8 * (i >> 2) + (i & 3))]);
             float top = fmaxf(s[0], s[1]);
 #pragma unroll
             for (int i = 2; i < 16; ++i) top = fmaxf(top, s[i]);
@@ -133,49 +124,61 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
 }
 
 // ------------------------------------------------------------------ mixed weights times values
-constexpr int kTmRows = 16, kTmKeys = 32, kTmWaves = 8, kTmThreads = 64 * kTmWaves, kTmCols = 64;
+constexpr int kTmRows = 16, kTmKeys = 32, kTmWaves = 8, kTmThreads = 64 * kTmWaves;
+constexpr int kTmOut = 2 * kTmWaves;  // out heads of a workgroup, two per wave
 
-// HW: heads per wave, 2 or 4.  Weights, mixed weights, a wave's value columns (64 at a time), biases, T
-template <int HW> struct TmTile {
-    static constexpr int heads = kTmWaves * HW, vPitch = kTmCols + 8;
+// HW: heads per wave, 2 or 4.  Weights, mixed weights, every wave's values and biases
+template <int D, int HW> struct TmTile {
+    static constexpr int heads = kTmWaves * HW, vPitch = D + 8;
     static constexpr int pair = 4 * heads;  // bytes of a (key, row) pair: both terms of all heads
-    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = heads * kTmRows * kTmKeys * 2, vBytes = kTmKeys * vPitch * 2;
-    static constexpr int biasFloats = HW * 64, tElems = heads * 32;  // (one term of T)
-    static constexpr size_t bytes = (size_t)pBytes + wBytes + kTmWaves * vBytes + kTmWaves * biasFloats * 4 + 2 * tElems * 2;
+    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = kTmOut * kTmRows * kTmKeys * 2, vBytes = kTmKeys * vPitch * 2;
+    static constexpr int biasFloats = HW * 48;
+    static constexpr size_t bytes = (size_t)pBytes + wBytes + kTmWaves * vBytes + kTmWaves * biasFloats * 4;
 };
 
-// D: keys and values padded to 64 or 128; FULL: they fill it.  SAME: a wave's heads share a kv head.
+// D: keys and values padded to 64 or 128; FULL: they fill it.  SAME: a wave's heads share a kv head, and so do its out heads.
 template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmThreads) void talk_mix_kernel(const TalkArgs a) {
-    using L = TmTile<HW>;
-    constexpr int HP = L::heads, KS = D / 32, MT = HP / 16, NV = kTmKeys * kTmCols / 8 / 64, CT = kTmCols / 16, NC = D / kTmCols;
+    using L = TmTile<D, HW>;
+    constexpr int HP = L::heads, KS = D / 32, NV = kTmKeys * D / 8 / 64, ET = D / 16;
     extern __shared__ __align__(16) char tm_lds[];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     char *w_s = tm_lds + L::pBytes;
     __bf16 *v_s = reinterpret_cast<__bf16 *>(w_s + L::wBytes + wave * L::vBytes);
     float *biases = reinterpret_cast<float *>(w_s + L::wBytes + kTmWaves * L::vBytes) + wave * L::biasFloats;
-    __bf16 *t_s = reinterpret_cast<__bf16 *>(w_s + L::wBytes + kTmWaves * (L::vBytes + L::biasFloats * 4));
     const int b = blockIdx.x;
     ScoredPortion p;
     if (!scored_portion(a, b, p)) return;
     const int row0 = (int)(gridDim.y - 1 - blockIdx.y) * kTmRows;  // (the rows with the most keys first)
     if (row0 >= p.n) return;
-    const int row = row0 + l16, pos = row < p.n ? p.pos0 + row : -1, first_pos = p.pos0 + row0, end = p.pos0 + min(row0 + kTmRows, p.n);
+    const int row = row0 + l16, first_pos = p.pos0 + row0, end = p.pos0 + min(row0 + kTmRows, p.n);
     const float plain = a.scale * kScoredLog2e;
-    const int head0 = wave * HW, n_heads = max(0, min(HW, a.heads - head0));  // of this wave
-    // T in the pairs' k order (terms of 32 heads, or both of 16): row = out head, 16 mt + l16; the second term of T meets the
-    // first of the weights only
-    bool exact = true;
-    for (int i = tid; i < L::tElems; i += kTmThreads) {
-        const int out = i / 32, in = i % 32 % HP;
-        const float x = out < a.heads && in < a.heads ? a.talk[(int64_t)out * a.heads + in] : 0.f;
-        const __bf16 hi = (__bf16)x, lo = (__bf16)(x - (float)hi);
-        exact = exact && (float)lo == 0.f;
-        t_s[i] = hi;
-        t_s[L::tElems + i] = HP == 16 && i % 32 >= 16 ? (__bf16)0.f : lo;
+    const int head0 = wave * HW, out0 = blockIdx.z * kTmOut, own0 = out0 + 2 * wave;  // the wave's heads and out heads
+    auto kv_of = [&](int h) { return min(h, a.heads - 1) / a.n_rep; };
+    // T in the pairs' k order (terms of 32 heads, or both of 16): out head out0 + l16; the second term of T meets the first of
+    // the weights only
+    bf8 t_hi, t_lo;
+    bool t_rest;  // (a matrix stored in 16 bits has no second term)
+    {
+        LaSplit sp;
+        bool exact = true;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            float x[2];
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                const int out = out0 + l16, in = (8 * g + 2 * j + e) % HP;
+                x[e] = out < a.heads && in < a.heads ? a.talk[(int64_t)out * a.heads + in] : 0.f;
+            }
+            la_split2(x[0], x[1], sp.hi[j], sp.lo[j]);
+            exact = exact && sp.lo[j] == 0;
+            if (HP == 16 && g >= 2) sp.lo[j] = 0;
+        }
+        t_hi = sp.high();
+        t_lo = sp.low();
+        t_rest = __ballot(!exact) != 0;
     }
-    const bool t_rest = __syncthreads_or(!exact);  // (a matrix stored in 16 bits has no second term)
     bf8 q[HW][KS];
-    float lse[HW];
+    float lse[HW], size[HW], rate[HW];
     {
         const int64_t mem_row = p.row0 + min(row, p.n - 1);
 #pragma unroll
@@ -184,47 +187,46 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
             const uint16_t *src = reinterpret_cast<const uint16_t *>(a.q1) + mem_row * a.q1_row + h * a.q1_head;
 #pragma unroll
             for (int k = 0; k < KS; ++k) q[i][k] = __builtin_bit_cast(bf8, scored_load16(src + 32 * k + 8 * g, 32 * k + 8 * g < a.n1));
-            lse[i] = a.lse[mem_row * a.heads + h];
+            lse[i] = row < p.n && head0 + i < a.heads ? a.lse[mem_row * a.heads + h] : -kScoredNone;  // (no head, no row: no weight)
+            size[i] = a.size ? a.size[h] : 0.f;
+            rate[i] = a.rate ? a.rate[h] : 0.f;
         }
     }
-    f4 o[HW][NC][CT];
+    f4 o[2][ET];
 #pragma unroll
-    for (int i = 0; i < HW; ++i)
+    for (int i = 0; i < 2; ++i)
 #pragma unroll
-        for (int c = 0; c < NC; ++c)
-#pragma unroll
-            for (int t = 0; t < CT; ++t) o[i][c][t] = f4{0.f, 0.f, 0.f, 0.f};
+        for (int t = 0; t < ET; ++t) o[i][t] = f4{0.f, 0.f, 0.f, 0.f};
 
     const int32_t *table = a.bt + b * a.bt_stride;
-    const int64_t k_tok = (int64_t)a.hkv * a.k_dim, v_tok = (int64_t)a.hkv * a.v_dim;
+    const uint32_t k_tok = (uint32_t)(a.hkv * a.k_dim), v_tok = (uint32_t)(a.hkv * a.v_dim);
     const int vreal = (a.vdim + 7) / 8 * 8;
-    // pool row of key k0 + lane % 32 (past the last key: the last one's, which nothing weighs)
-    auto slots_of = [&](int k0) {
-        const int key = min(k0 + (lane & 31), end - 1);
-        return scored_slot_of(a, scored_block_id(a, table, key), key, end);
-    };
+    // block and pool row of key k0 + lane % 32 (past the last key: the last one's, which nothing weighs)
+    auto key_of = [&](int k0) { return min(k0 + (lane & 31), end - 1); };
+    auto id_of = [&](int k0) { return talk_block_id(a, table, key_of(k0)); };
+    auto slot_of = [&](int id, int k0) { return max(talk_slot_of(a, id, key_of(k0), end), 0); };
     scored_u4 kr[2][KS], vr[NV];
     auto fetch_k = [&](int kv, int slots) {  // keys 16 kb + l16
 #pragma unroll
         for (int kb = 0; kb < 2; ++kb) {
-            const int s = __shfl(slots, 16 * kb + l16, 64);
-            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)max(s, 0) * k_tok + kv * a.k_dim + 8 * g;
+            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (uint64_t)(uint32_t)__shfl(slots, 16 * kb + l16, 64) * k_tok + kv * a.k_dim + 8 * g;
 #pragma unroll
             for (int k = 0; k < KS; ++k) kr[kb][k] = FULL ? *reinterpret_cast<const scored_u4 *>(src + 32 * k) : scored_load16(src + 32 * k, 32 * k + 8 * g < a.n1);
         }
     };
-    auto fetch_v = [&](int kv, int slots, int c) {  // columns 64 c ..
-        const int e = kTmCols * c + lane % 8 * 8;
+    auto fetch_v = [&](int kv, int slots) {
+        constexpr int per = D / 8;
+        const int e = lane % per * 8;
 #pragma unroll
         for (int n = 0; n < NV; ++n) {
-            const int s = __shfl(slots, 8 * n + lane / 8, 64);
-            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.v) + (int64_t)max(s, 0) * v_tok + kv * a.v_dim + e;
+            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.v) + (uint64_t)(uint32_t)__shfl(slots, (64 * n + lane) / per, 64) * v_tok + kv * a.v_dim + e;
             vr[n] = FULL ? *reinterpret_cast<const scored_u4 *>(src) : scored_load16(src, e < vreal);
         }
     };
     auto put_v = [&]() {
+        constexpr int per = D / 8;
 #pragma unroll
-        for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + (8 * n + lane / 8) * L::vPitch + lane % 8 * 8) = vr[n];
+        for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + (64 * n + lane) / per * L::vPitch + lane % per * 8) = vr[n];
     };
     // 16-byte pieces of a pair's row and of a (head, row)'s keys at places that spread over the banks
     auto pair_at = [&](int key, int piece) {
@@ -232,28 +234,23 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
         return tm_lds + (key * kTmRows + l16) * L::pair + 16 * at;
     };
     auto weights_at = [&](int head, int piece) { return w_s + (head * kTmRows + l16) * (kTmKeys * 2) + 16 * (piece ^ ((l16 >> 2) & 3)); };
-    auto kv_of = [&](int i) { return min(head0 + i, a.heads - 1) / a.n_rep; };
 
-    const int kv0 = kv_of(0);
-    int slots = slots_of(0);
-    if (n_heads > 0) fetch_k(kv0, slots);
+    int slots = slot_of(id_of(0), 0), id = id_of(kTmKeys);
+    fetch_k(kv_of(head0), slots);
+    fetch_v(kv_of(own0), slots);
     for (int k0 = 0; k0 < end; k0 += kTmKeys) {
         // ---- scores and weights of keys 16 kb + 4 g + j of row l16 ----
-        if (a.size) {  // distances first_pos + r - k of 16 rows and 32 keys, from their smallest
+        // (distances first_pos + r - k of 16 rows and 32 keys, from their smallest; a key behind its row gets no weight)
 #pragma unroll
-            for (int i = 0; i < HW; ++i) {
-                const int h = min(head0 + i, a.heads - 1);
-                biases[i * 64 + lane] = talk_bias(a.size[h], a.rate[h], max(first_pos - (k0 + 31) + lane, 0));
-            }
-            tp_own_lds();
+        for (int i = 0; i < HW; ++i) {
+            const float x = talk_masked_bias(size[i], rate[i], first_pos - (k0 + 31) + lane);
+            if (lane < 48) biases[i * 48 + lane] = x;
         }
+        tp_own_lds();
         auto weights = [&](int i, int kb, f4 s, float *w) {
-            const float *bp = biases + i * 64 + l16 + 31 - 16 * kb - 4 * g;
+            const float *bp = biases + i * 48 + l16 + 31 - 16 * kb - 4 * g;
 #pragma unroll
-            for (int j = 0; j < 4; ++j) {
-                const float x = a.size ? fmaf(s[j], plain, bp[-j]) : s[j] * plain;
-                w[j] = i < n_heads && k0 + 16 * kb + 4 * g + j <= pos ? __builtin_amdgcn_exp2f(x - lse[i]) : 0.f;
-            }
+            for (int j = 0; j < 4; ++j) w[j] = __builtin_amdgcn_exp2f(fmaf(s[j], plain, bp[-j]) - lse[i]);
         };
         auto put = [&](int kb, float (*w)[4]) {
 #pragma unroll
@@ -287,14 +284,14 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
 #pragma unroll
                 for (int i = 0; i < HW; ++i) weights(i, kb, s[i], w[i]);
                 put(kb, w);
-                __builtin_amdgcn_sched_barrier(0);
+                if (HW == 4) __builtin_amdgcn_sched_barrier(0);
             }
         } else {
             float w[2][HW][4];
-            int kv = kv0;
+            int kv = kv_of(head0);
 #pragma unroll
             for (int i = 0; i < HW; ++i) {
-                if (kv_of(i) != kv) fetch_k(kv = kv_of(i), slots);
+                if (kv_of(head0 + i) != kv) fetch_k(kv = kv_of(head0 + i), slots);
 #pragma unroll
                 for (int kb = 0; kb < 2; ++kb) {
                     f4 s = f4{0.f, 0.f, 0.f, 0.f};
@@ -306,123 +303,95 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
             put(0, w[0]);
             put(1, w[1]);
         }
-        fetch_v(kv0, slots, 0);
+        const int now = slots;
+        // (always, so that waits can be counted: past the last key these are the last key's again)
+        slots = slot_of(id, k0 + kTmKeys);
+        id = id_of(k0 + 2 * kTmKeys);
+        fetch_k(kv_of(head0), slots);
+        __builtin_amdgcn_sched_barrier(0);
         __syncthreads();
-        // ---- mixed: keys 4 wave .. 4 wave + 3 of row l16, out heads 16 mt + 4 g + i ----
+        // ---- mixed: keys 4 wave .. 4 wave + 3 of row l16, out heads 4 g + i ----
+        {
+            f4 x[4];
+            bf8 one[4];
 #pragma unroll
-        for (int half = 0; half < 2; ++half) {
-            f4 x[2][MT];
+            for (int k = 0; k < 4; ++k) one[k] = la_read8(reinterpret_cast<const __bf16 *>(pair_at(4 * wave + k, g)));
 #pragma unroll
-            for (int k = 0; k < 2; ++k) {
-                const int key = 4 * wave + 2 * half + k;
-                const bf8 one = la_read8(reinterpret_cast<const __bf16 *>(pair_at(key, g)));
+            for (int k = 0; k < 4; ++k) x[k] = la_mfma(t_hi, one[k], f4{0.f, 0.f, 0.f, 0.f});
+            if (t_rest) {
 #pragma unroll
-                for (int mt = 0; mt < MT; ++mt)
-                    x[k][mt] = la_mfma(la_read8(t_s + (16 * mt + l16) * 32 + 8 * g), one, f4{0.f, 0.f, 0.f, 0.f});
-                if constexpr (HP == 32) {
-                    const bf8 two = la_read8(reinterpret_cast<const __bf16 *>(pair_at(key, 4 + g)));
+                for (int k = 0; k < 4; ++k) x[k] = la_mfma(t_lo, one[k], x[k]);
+            }
+            if constexpr (HP == 32) {
 #pragma unroll
-                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(la_read8(t_s + (16 * mt + l16) * 32 + 8 * g), two, x[k][mt]);
-                }
-                if (t_rest) {
+                for (int k = 0; k < 4; ++k) one[k] = la_read8(reinterpret_cast<const __bf16 *>(pair_at(4 * wave + k, 4 + g)));
 #pragma unroll
-                    for (int mt = 0; mt < MT; ++mt) x[k][mt] = la_mfma(la_read8(t_s + L::tElems + (16 * mt + l16) * 32 + 8 * g), one, x[k][mt]);
-                }
+                for (int k = 0; k < 4; ++k) x[k] = la_mfma(t_hi, one[k], x[k]);
             }
 #pragma unroll
-            for (int mt = 0; mt < MT; ++mt)
-#pragma unroll
-                for (int i = 0; i < 4; ++i)
-                    *reinterpret_cast<uint32_t *>(weights_at(16 * mt + 4 * g + i, wave >> 1) + 8 * (wave & 1) + 4 * half) = row_pack_bf16(x[0][mt][i], x[1][mt][i]);
-            __builtin_amdgcn_sched_barrier(0);
+            for (int i = 0; i < 4; ++i)
+                *reinterpret_cast<uint2 *>(weights_at(4 * g + i, wave >> 1) + 8 * (wave & 1)) =
+                    make_uint2(row_pack_bf16(x[0][i], x[1][i]), row_pack_bf16(x[2][i], x[3][i]));
         }
-        // ---- values: 64 columns at a time ----
-        const int now = slots;
         put_v();
-        if (NC > 1) fetch_v(kv0, now, NC - 1);
+        fetch_v(kv_of(own0), slots);
+        __builtin_amdgcn_sched_barrier(0);
         __syncthreads();
-        auto weights_of = [&](int i) { return la_read8(reinterpret_cast<const __bf16 *>(weights_at(head0 + i, g))); };
+        // ---- values ----
+        bf8 x[2];
+#pragma unroll
+        for (int i = 0; i < 2; ++i) x[i] = la_read8(reinterpret_cast<const __bf16 *>(weights_at(2 * wave + i, g)));
         auto values = [&](int t) {
             const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::vPitch + 16 * t + 4 * (l16 & 3);
             return la_join(la_read_tr(va), la_read_tr(va + 4 * L::vPitch));
         };
-        if constexpr (SAME) {
-            bf8 x[HW];
+        if (SAME || kv_of(own0 + 1) == kv_of(own0)) {
 #pragma unroll
-            for (int i = 0; i < HW; ++i) x[i] = weights_of(i);
+            for (int t = 0; t < ET; ++t) {
+                const bf8 v = values(t);
 #pragma unroll
-            for (int c = 0; c < NC; ++c) {
-                if (c > 0) {
-                    tp_own_lds();
-                    put_v();
-                    tp_own_lds();
-                }
-                if (c == NC - 1 && k0 + kTmKeys < end) {
-                    slots = slots_of(k0 + kTmKeys);
-                    if (n_heads > 0) fetch_k(kv0, slots);
-                }
-#pragma unroll
-                for (int t = 0; t < CT; ++t) {
-                    const bf8 v = values(t);
-#pragma unroll
-                    for (int i = 0; i < HW; ++i) o[i][c][t] = la_mfma(v, x[i], o[i][c][t]);
-                }
-                __builtin_amdgcn_sched_barrier(0);
+                for (int i = 0; i < 2; ++i) o[i][t] = la_mfma(v, x[i], o[i][t]);
             }
         } else {
-            int have = kv0, part = 0;  // what v_s holds
-            bool waiting = NC > 1;     // its last columns are in registers
 #pragma unroll
-            for (int i = 0; i < HW; ++i)
+            for (int t = 0; t < ET; ++t) o[0][t] = la_mfma(values(t), x[0], o[0][t]);
+            fetch_v(kv_of(own0 + 1), now);
+            tp_own_lds();
+            put_v();
+            tp_own_lds();
 #pragma unroll
-                for (int c = 0; c < NC; ++c) {
-                    if (have != kv_of(i) || part != c) {
-                        if (!(waiting && kv_of(i) == kv0 && c == NC - 1)) fetch_v(kv_of(i), now, c);
-                        waiting = false;
-                        have = kv_of(i);
-                        part = c;
-                        tp_own_lds();
-                        put_v();
-                        tp_own_lds();
-                    }
-                    const bf8 x = weights_of(i);
-#pragma unroll
-                    for (int t = 0; t < CT; ++t) o[i][c][t] = la_mfma(values(t), x, o[i][c][t]);
-                }
-            if (k0 + kTmKeys < end) {
-                slots = slots_of(k0 + kTmKeys);
-                fetch_k(kv0, slots);
-            }
+            for (int t = 0; t < ET; ++t) o[1][t] = la_mfma(values(t), x[1], o[1][t]);
+            fetch_v(kv_of(own0), slots);
         }
+        __builtin_amdgcn_sched_barrier(0);
     }
     if (row >= p.n) return;
 #pragma unroll
-    for (int i = 0; i < HW; ++i) {
-        if (i >= n_heads) continue;
-        pa_bf16 *out = reinterpret_cast<pa_bf16 *>(a.out) + ((p.row0 + row) * a.heads + head0 + i) * a.vdim;
+    for (int i = 0; i < 2; ++i) {
+        if (own0 + i >= a.heads) continue;
+        pa_bf16 *out = reinterpret_cast<pa_bf16 *>(a.out) + ((p.row0 + row) * a.heads + own0 + i) * a.vdim;
 #pragma unroll
-        for (int c = 0; c < NC; ++c)
+        for (int t = 0; t < ET; ++t) {
+            const f4 x = o[i][t];
+            const int d = 16 * t + 4 * g;
+            if (d >= a.vdim) continue;
+            if (FULL || a.vdim % 4 == 0) {
+                *reinterpret_cast<uint2 *>(out + d) = make_uint2(row_pack_bf16(x[0], x[1]), row_pack_bf16(x[2], x[3]));
+            } else {
 #pragma unroll
-            for (int t = 0; t < CT; ++t) {
-                const f4 x = o[i][c][t];
-                const int d = kTmCols * c + 16 * t + 4 * g;
-                if (d >= a.vdim) continue;
-                if (FULL || a.vdim % 4 == 0) {
-                    *reinterpret_cast<uint2 *>(out + d) = make_uint2(row_pack_bf16(x[0], x[1]), row_pack_bf16(x[2], x[3]));
-                } else {
-#pragma unroll
-                    for (int e = 0; e < 4; ++e)
-                        if (d + e < a.vdim) pa_scalar<pa_bf16>::store(out + d + e, x[e]);
-                }
+                for (int e = 0; e < 4; ++e)
+                    if (d + e < a.vdim) pa_scalar<pa_bf16>::store(out + d + e, x[e]);
             }
+        }
     }
 }
 
 template <int D, int HW, bool FULL, bool SAME> int launch_mix(const TalkArgs &a, hipStream_t s) {
-    constexpr size_t lds = TmTile<HW>::bytes;
+    constexpr size_t lds = TmTile<D, HW>::bytes;
     static_assert(lds <= 160 * 1024, "LDS of one compute unit");
     if (int rc = la_big_lds(talk_mix_kernel<D, HW, FULL, SAME>, lds, "pa_talking_attention")) return rc;
-    talk_mix_kernel<D, HW, FULL, SAME><<<dim3((unsigned)a.batch, (unsigned)((a.max_q_len + kTmRows - 1) / kTmRows)), dim3(kTmThreads), lds, s>>>(a);
+    const dim3 grid((unsigned)a.batch, (unsigned)((a.max_q_len + kTmRows - 1) / kTmRows), (unsigned)((a.heads + kTmOut - 1) / kTmOut));
+    talk_mix_kernel<D, HW, FULL, SAME><<<grid, dim3(kTmThreads), lds, s>>>(a);
     PA_CHECK_LAUNCH("pa_talking_attention (portions)");
     return PA_OK;
 }
