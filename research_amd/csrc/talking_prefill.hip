@@ -127,24 +127,30 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
 constexpr int kTmRows = 16, kTmKeys = 32, kTmWaves = 8, kTmThreads = 64 * kTmWaves;
 constexpr int kTmOut = 2 * kTmWaves;  // out heads of a workgroup, two per wave
 
-// HW: heads per wave, 2 or 4.  Weights, mixed weights, every wave's values and biases
-template <int D, int HW> struct TmTile {
-    static constexpr int heads = kTmWaves * HW, vPitch = D + 8;
+// HW: heads per wave, 2 or 4.  NG: kv heads of the out heads, whose values are staged by the whole workgroup (0: each wave
+// stages its own).  With two heads per wave the keys of up to NG kv heads are staged as well.
+template <int D, int HW, int NG> struct TmTile {
+    static constexpr int heads = kTmWaves * HW, pitch = D + 8;
+    static constexpr bool keys = NG > 0 && HW == 2;
     static constexpr int pair = 4 * heads;  // bytes of a (key, row) pair: both terms of all heads
-    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = kTmOut * kTmRows * kTmKeys * 2, vBytes = kTmKeys * vPitch * 2;
+    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = kTmOut * kTmRows * kTmKeys * 2, tileBytes = kTmKeys * pitch * 2;
+    static constexpr int vBytes = (NG ? NG : kTmWaves) * tileBytes, kBytes = keys ? NG * tileBytes : 0;
     static constexpr int biasFloats = HW * 48;
-    static constexpr size_t bytes = (size_t)pBytes + wBytes + kTmWaves * vBytes + kTmWaves * biasFloats * 4;
+    static constexpr size_t bytes = (size_t)pBytes + wBytes + vBytes + kBytes + kTmWaves * biasFloats * 4;
 };
 
-// D: keys and values padded to 64 or 128; FULL: they fill it.  SAME: a wave's heads share a kv head, and so do its out heads.
-template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmThreads) void talk_mix_kernel(const TalkArgs a) {
-    using L = TmTile<D, HW>;
-    constexpr int HP = L::heads, KS = D / 32, NV = kTmKeys * D / 8 / 64, ET = D / 16;
+// D: keys and values padded to 64 or 128; FULL: they fill it.  NG > 0: a wave's heads share a kv head, and so do its out heads.
+template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThreads) void talk_mix_kernel(const TalkArgs a) {
+    using L = TmTile<D, HW, NG>;
+    constexpr bool SAME = NG > 0;
+    constexpr int HP = L::heads, KS = D / 32, ET = D / 16;
+    constexpr int kPer = D / 8, kTile = kTmKeys * kPer;                     // 16-byte pieces of a row, of a kv head's tile
+    constexpr int NV = SAME ? NG * kTile / kTmThreads : kTile / 64, NK = L::keys ? NV : 2 * KS;
     extern __shared__ __align__(16) char tm_lds[];
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l16 = lane & 15, g = lane >> 4;
     char *w_s = tm_lds + L::pBytes;
-    __bf16 *v_s = reinterpret_cast<__bf16 *>(w_s + L::wBytes + wave * L::vBytes);
-    float *biases = reinterpret_cast<float *>(w_s + L::wBytes + kTmWaves * L::vBytes) + wave * L::biasFloats;
+    __bf16 *v_all = reinterpret_cast<__bf16 *>(w_s + L::wBytes), *k_s = v_all + L::vBytes / 2;
+    float *biases = reinterpret_cast<float *>(w_s + L::wBytes + L::vBytes + L::kBytes) + wave * L::biasFloats;
     const int b = blockIdx.x;
     ScoredPortion p;
     if (!scored_portion(a, b, p)) return;
@@ -201,32 +207,70 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
     const int32_t *table = a.bt + b * a.bt_stride;
     const uint32_t k_tok = (uint32_t)(a.hkv * a.k_dim), v_tok = (uint32_t)(a.hkv * a.v_dim);
     const int vreal = (a.vdim + 7) / 8 * 8;
-    // block and pool row of key k0 + lane % 32 (past the last key: the last one's, which nothing weighs)
-    auto key_of = [&](int k0) { return min(k0 + (lane & 31), end - 1); };
+    // the kv heads that are staged: from the first of the out heads, from the first of all
+    const int v_kv0 = kv_of(out0);
+    __bf16 *v_s = v_all + (SAME ? kv_of(own0) - v_kv0 : wave) * (L::tileBytes / 2);
+    // Block and pool row of the key that this thread stages (values staged by all: the piece of a tile; else key lane % 32); past
+    // the last key: the last one's, which nothing weighs.
+    const int my_row = SAME ? tid % kTile / kPer : lane & 31;
+    auto key_of = [&](int k0) { return min(k0 + my_row, end - 1); };
     auto id_of = [&](int k0) { return talk_block_id(a, table, key_of(k0)); };
     auto slot_of = [&](int id, int k0) { return max(talk_slot_of(a, id, key_of(k0), end), 0); };
-    scored_u4 kr[2][KS], vr[NV];
-    auto fetch_k = [&](int kv, int slots) {  // keys 16 kb + l16
-#pragma unroll
-        for (int kb = 0; kb < 2; ++kb) {
-            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (uint64_t)(uint32_t)__shfl(slots, 16 * kb + l16, 64) * k_tok + kv * a.k_dim + 8 * g;
-#pragma unroll
-            for (int k = 0; k < KS; ++k) kr[kb][k] = FULL ? *reinterpret_cast<const scored_u4 *>(src + 32 * k) : scored_load16(src + 32 * k, 32 * k + 8 * g < a.n1);
-        }
-    };
-    auto fetch_v = [&](int kv, int slots) {
-        constexpr int per = D / 8;
-        const int e = lane % per * 8;
+    scored_u4 kr[NK], vr[NV];
+    // staged by the workgroup: piece tid + 512 n is of kv head (tid + 512 n) / kTile, the thread's own row
+    auto stage_from = [&](const void *pool, int slot, uint32_t tok, int head_dim, int kv_first, int real, scored_u4 *to) {
+        const uint16_t *src = reinterpret_cast<const uint16_t *>(pool) + (uint64_t)(uint32_t)slot * tok + tid % kPer * 8;
 #pragma unroll
         for (int n = 0; n < NV; ++n) {
-            const uint16_t *src = reinterpret_cast<const uint16_t *>(a.v) + (uint64_t)(uint32_t)__shfl(slots, (64 * n + lane) / per, 64) * v_tok + kv * a.v_dim + e;
-            vr[n] = FULL ? *reinterpret_cast<const scored_u4 *>(src) : scored_load16(src, e < vreal);
+            const uint16_t *at = src + min(kv_first + (tid + kTmThreads * n) / kTile, a.hkv - 1) * head_dim;
+            to[n] = FULL ? *reinterpret_cast<const scored_u4 *>(at) : scored_load16(at, tid % kPer * 8 < real);
         }
     };
-    auto put_v = [&]() {
-        constexpr int per = D / 8;
+    auto stage_to = [&](__bf16 *tiles, const scored_u4 *from) {
 #pragma unroll
-        for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + (64 * n + lane) / per * L::vPitch + lane % per * 8) = vr[n];
+        for (int n = 0; n < NV; ++n)
+            *reinterpret_cast<scored_u4 *>(tiles + (tid + kTmThreads * n) / kTile * (L::tileBytes / 2) + my_row * L::pitch + tid % kPer * 8) = from[n];
+    };
+    // straight to operands: keys 16 kb + l16 of one kv head (slots: of key lane % 32)
+    auto direct_k = [&](int kv, int slots) {
+        if constexpr (!L::keys) {
+#pragma unroll
+            for (int kb = 0; kb < 2; ++kb) {
+                const uint16_t *src = reinterpret_cast<const uint16_t *>(a.k) + (uint64_t)(uint32_t)__shfl(slots, 16 * kb + l16, 64) * k_tok + kv * a.k_dim + 8 * g;
+#pragma unroll
+                for (int k = 0; k < KS; ++k) kr[kb * KS + k] = FULL ? *reinterpret_cast<const scored_u4 *>(src + 32 * k) : scored_load16(src + 32 * k, 32 * k + 8 * g < a.n1);
+            }
+        }
+    };
+    auto fetch_k = [&](int slots, int near) {  // (near: the slots of keys lane % 32)
+        if constexpr (L::keys) stage_from(a.k, slots, k_tok, a.k_dim, 0, a.n1, kr);
+        else direct_k(kv_of(head0), near);
+    };
+    auto own_v = [&](int kv, int slots) {
+        if constexpr (!SAME) {
+#pragma unroll
+            for (int n = 0; n < NV; ++n) {
+                const uint16_t *src = reinterpret_cast<const uint16_t *>(a.v) + (uint64_t)(uint32_t)__shfl(slots, (64 * n + lane) / kPer, 64) * v_tok + kv * a.v_dim + lane % kPer * 8;
+                vr[n] = scored_load16(src, lane % kPer * 8 < vreal);
+            }
+        }
+    };
+    auto fetch_v = [&](int slots) {
+        if constexpr (SAME) stage_from(a.v, slots, v_tok, a.v_dim, v_kv0, vreal, vr);
+        else own_v(kv_of(own0), slots);
+    };
+    auto put_v = [&]() {
+        if constexpr (SAME) {
+            stage_to(v_all, vr);
+        } else {
+#pragma unroll
+            for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + (64 * n + lane) / kPer * L::pitch + lane % kPer * 8) = vr[n];
+        }
+    };
+    // keys by key lane % 32, where they go straight to operands beside values staged by all
+    auto near_id = [&](int k0) { return SAME && !L::keys ? talk_block_id(a, table, min(k0 + (lane & 31), end - 1)) : 0; };
+    auto near_slot = [&](int id, int k0, int slots) {
+        return SAME && !L::keys ? max(talk_slot_of(a, id, min(k0 + (lane & 31), end - 1), end), 0) : slots;
     };
     // 16-byte pieces of a pair's row and of a (head, row)'s keys at places that spread over the banks
     auto pair_at = [&](int key, int piece) {
@@ -235,9 +279,13 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
     };
     auto weights_at = [&](int head, int piece) { return w_s + (head * kTmRows + l16) * (kTmKeys * 2) + 16 * (piece ^ ((l16 >> 2) & 3)); };
 
-    int slots = slot_of(id_of(0), 0), id = id_of(kTmKeys);
-    fetch_k(kv_of(head0), slots);
-    fetch_v(kv_of(own0), slots);
+    int slots = slot_of(id_of(0), 0), id = id_of(kTmKeys), id_near = near_id(kTmKeys);
+    fetch_k(slots, near_slot(near_id(0), 0, slots));
+    fetch_v(slots);
+    if constexpr (L::keys) {
+        stage_to(k_s, kr);
+        __syncthreads();
+    }
     for (int k0 = 0; k0 < end; k0 += kTmKeys) {
         // ---- scores and weights of keys 16 kb + 4 g + j of row l16 ----
         // (distances first_pos + r - k of 16 rows and 32 keys, from their smallest; a key behind its row gets no weight)
@@ -278,9 +326,13 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
 #pragma unroll
                 for (int i = 0; i < HW; ++i) s[i] = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int k = 0; k < KS; ++k)
+                for (int k = 0; k < KS; ++k) {
+                    bf8 key;
+                    if constexpr (L::keys) key = la_read8(k_s + kv_of(head0) * (L::tileBytes / 2) + (16 * kb + l16) * L::pitch + 32 * k + 8 * g);
+                    else key = __builtin_bit_cast(bf8, kr[kb * KS + k]);
 #pragma unroll
-                    for (int i = 0; i < HW; ++i) s[i] = la_mfma(__builtin_bit_cast(bf8, kr[kb][k]), q[i][k], s[i]);
+                    for (int i = 0; i < HW; ++i) s[i] = la_mfma(key, q[i][k], s[i]);
+                }
 #pragma unroll
                 for (int i = 0; i < HW; ++i) weights(i, kb, s[i], w[i]);
                 put(kb, w);
@@ -291,12 +343,12 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
             int kv = kv_of(head0);
 #pragma unroll
             for (int i = 0; i < HW; ++i) {
-                if (kv_of(head0 + i) != kv) fetch_k(kv = kv_of(head0 + i), slots);
+                if (kv_of(head0 + i) != kv) direct_k(kv = kv_of(head0 + i), slots);
 #pragma unroll
                 for (int kb = 0; kb < 2; ++kb) {
                     f4 s = f4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                    for (int k = 0; k < KS; ++k) s = la_mfma(__builtin_bit_cast(bf8, kr[kb][k]), q[i][k], s);
+                    for (int k = 0; k < KS; ++k) s = la_mfma(__builtin_bit_cast(bf8, kr[kb * KS + k]), q[i][k], s);
                     weights(i, kb, s, w[kb][i]);
                 }
             }
@@ -307,7 +359,9 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
         // (always, so that waits can be counted: past the last key these are the last key's again)
         slots = slot_of(id, k0 + kTmKeys);
         id = id_of(k0 + 2 * kTmKeys);
-        fetch_k(kv_of(head0), slots);
+        const int near = near_slot(id_near, k0 + kTmKeys, slots);
+        id_near = near_id(k0 + 2 * kTmKeys);
+        fetch_k(slots, near);
         __builtin_amdgcn_sched_barrier(0);
         __syncthreads();
         // ---- mixed: keys 4 wave .. 4 wave + 3 of row l16, out heads 4 g + i ----
@@ -334,7 +388,8 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
                     make_uint2(row_pack_bf16(x[0][i], x[1][i]), row_pack_bf16(x[2][i], x[3][i]));
         }
         put_v();
-        fetch_v(kv_of(own0), slots);
+        if constexpr (L::keys) stage_to(k_s, kr);
+        fetch_v(slots);
         __builtin_amdgcn_sched_barrier(0);
         __syncthreads();
         // ---- values ----
@@ -342,8 +397,8 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
 #pragma unroll
         for (int i = 0; i < 2; ++i) x[i] = la_read8(reinterpret_cast<const __bf16 *>(weights_at(2 * wave + i, g)));
         auto values = [&](int t) {
-            const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::vPitch + 16 * t + 4 * (l16 & 3);
-            return la_join(la_read_tr(va), la_read_tr(va + 4 * L::vPitch));
+            const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::pitch + 16 * t + 4 * (l16 & 3);
+            return la_join(la_read_tr(va), la_read_tr(va + 4 * L::pitch));
         };
         if (SAME || kv_of(own0 + 1) == kv_of(own0)) {
 #pragma unroll
@@ -355,13 +410,13 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
         } else {
 #pragma unroll
             for (int t = 0; t < ET; ++t) o[0][t] = la_mfma(values(t), x[0], o[0][t]);
-            fetch_v(kv_of(own0 + 1), now);
+            own_v(kv_of(own0 + 1), now);
             tp_own_lds();
             put_v();
             tp_own_lds();
 #pragma unroll
             for (int t = 0; t < ET; ++t) o[1][t] = la_mfma(values(t), x[1], o[1][t]);
-            fetch_v(kv_of(own0), slots);
+            own_v(kv_of(own0), slots);
         }
         __builtin_amdgcn_sched_barrier(0);
     }
@@ -386,19 +441,20 @@ template <int D, int HW, bool FULL, bool SAME> __global__ __launch_bounds__(kTmT
     }
 }
 
-template <int D, int HW, bool FULL, bool SAME> int launch_mix(const TalkArgs &a, hipStream_t s) {
-    constexpr size_t lds = TmTile<D, HW>::bytes;
+template <int D, int HW, bool FULL, int NG> int launch_mix(const TalkArgs &a, hipStream_t s) {
+    constexpr size_t lds = TmTile<D, HW, NG>::bytes;
     static_assert(lds <= 160 * 1024, "LDS of one compute unit");
-    if (int rc = la_big_lds(talk_mix_kernel<D, HW, FULL, SAME>, lds, "pa_talking_attention")) return rc;
+    if (int rc = la_big_lds(talk_mix_kernel<D, HW, FULL, NG>, lds, "pa_talking_attention")) return rc;
     const dim3 grid((unsigned)a.batch, (unsigned)((a.max_q_len + kTmRows - 1) / kTmRows), (unsigned)((a.heads + kTmOut - 1) / kTmOut));
-    talk_mix_kernel<D, HW, FULL, SAME><<<grid, dim3(kTmThreads), lds, s>>>(a);
+    talk_mix_kernel<D, HW, FULL, NG><<<grid, dim3(kTmThreads), lds, s>>>(a);
     PA_CHECK_LAUNCH("pa_talking_attention (portions)");
     return PA_OK;
 }
 template <int D, int HW> int launch_mix_size(const TalkArgs &a, hipStream_t s) {
-    const bool full = a.n1 == D && a.vdim == D, same = a.n_rep % HW == 0;
-    if (!same) return launch_mix<D, HW, false, false>(a, s);
-    return full ? launch_mix<D, HW, true, true>(a, s) : launch_mix<D, HW, false, true>(a, s);
+    // kv heads beside each other that 16 out heads use at most (all of them, with two heads per wave)
+    const int use = HW == 2 ? a.hkv : a.n_rep % kTmOut == 0 ? 1 : kTmOut % a.n_rep == 0 ? kTmOut / a.n_rep : (kTmOut - 2) / a.n_rep + 2;
+    if (a.n_rep % HW != 0 || use > 4) return launch_mix<D, HW, false, 0>(a, s);
+    return a.n1 == D && a.vdim == D ? launch_mix<D, HW, true, 4>(a, s) : launch_mix<D, HW, false, 4>(a, s);
 }
 
 }  // namespace
