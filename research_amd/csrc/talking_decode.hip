@@ -103,7 +103,7 @@ template <int KC> __global__ __launch_bounds__(256) void talk_scores_kernel(cons
 
 // HP: heads padded to 32, 64 or 128 (the rows of P).
 template <int VC, int HP> struct TdTile {
-    static constexpr int vPitch = VC + 8, pPitch = kTdKeys + 8, vElems = kTdKeys * vPitch, pElems = HP * pPitch;
+    static constexpr int vPitch = VC + 16, pPitch = kTdKeys + 8, vElems = kTdKeys * vPitch, pElems = HP * pPitch;
     static constexpr size_t bytes = (size_t)(vElems + 2 * pElems) * 2 + HP * 4;
 };
 
@@ -314,7 +314,7 @@ bool pa_talking_decode_launch(const TalkArgs &in, int dtype, void *workspace, si
     TalkArgs a = in;
     const uintptr_t at = (uintptr_t)a.q1 | (uintptr_t)a.k | (uintptr_t)a.v | (uintptr_t)a.out;
     if (dtype != PA_BF16 || a.q_lens || (at & 15u) != 0 || a.n1 % 8 != 0 || a.k_dim % 8 != 0 || a.v_dim % 8 != 0 || a.q1_row % 8 != 0 ||
-        a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff || a.bt_stride == 0)
+        a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff || a.bt_stride == 0 || !(a.scale > 0.f))
         return false;
     const int64_t max_keys = a.bt_stride * a.bs;
     a.splits = td_splits(a.batch, a.heads, a.hkv, max_keys);

@@ -56,7 +56,12 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
             q[k] = __builtin_bit_cast(X8, d < a.n1 ? *reinterpret_cast<const uint4 *>(src + d) : make_uint4(0, 0, 0, 0));
         }
     }
-    float m = kScoredNone, l = 0.f;
+    // the row's reference m, which the products start from (as -m / plain), and the sum of 2^(score - m)
+    float m = 0.f, l = 0.f;
+    const float unplain = 1.f / plain;
+    f32x16 start;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) start[i] = 0.f;
     const int32_t *table = a.bt + b * a.bt_stride;
     const uint16_t *kp = reinterpret_cast<const uint16_t *>(a.k) + (int64_t)kvh * a.k_dim;
     const int64_t k_tok = (int64_t)a.hkv * a.k_dim;
@@ -93,9 +98,7 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
         for (int sub = 0; sub < 2; ++sub) {
             const int kb = k0 + 32 * sub;  // (uniform per wave)
             if (!live || kb >= wave_hi) continue;
-            f32x16 s;
-#pragma unroll
-            for (int i = 0; i < 16; ++i) s[i] = 0.f;
+            f32x16 s = start;
 #pragma unroll
             for (int k = 0; k < KS; ++k)
                 s = M::mma(__builtin_bit_cast(X8, *reinterpret_cast<const uint4 *>(ks + (32 * sub + col) * kPitch + 16 * k + 8 * half)), q[k], s);
@@ -106,17 +109,24 @@ template <int DK> __global__ __launch_bounds__(256, 2) void talk_sums_kernel(con
             float top = fmaxf(s[0], s[1]);
 #pragma unroll
             for (int i = 2; i < 16; ++i) top = fmaxf(top, s[i]);
-            if (__ballot(top > m + kTpSlack) != 0) {  // (every lane has a maximum of its own)
-                const float next = fmaxf(m, top);
-                l *= __builtin_amdgcn_exp2f(m - next);
-                m = next;
+            // (every lane has a reference of its own; it follows when a score is far above it, or the first ones all far below)
+            if (__ballot(top > kTpSlack || (l == 0.f && top > 0.5f * kScoredNone && top < -kTpSlack)) != 0) {
+                const float by = top > kTpSlack || (l == 0.f && top > 0.5f * kScoredNone) ? top : 0.f;
+                l *= __builtin_amdgcn_exp2f(-by);
+                m += by;
+#pragma unroll
+                for (int i = 0; i < 16; ++i) {
+                    s[i] -= by;
+                    start[i] = -m * unplain;
+                }
             }
 #pragma unroll
-            for (int i = 0; i < 16; i += 2) l += __builtin_amdgcn_exp2f(s[i] - m) + __builtin_amdgcn_exp2f(s[i + 1] - m);
+            for (int i = 0; i < 16; i += 2) l += __builtin_amdgcn_exp2f(s[i]) + __builtin_amdgcn_exp2f(s[i + 1]);
         }
         __syncthreads();
     }
-    // (a lane that saw no key has m = kScoredNone and counted its masked ones as 1: they vanish here)
+    // (a lane that saw no key has nothing to say)
+    if (l == 0.f) m = kScoredNone;
     const float other = __shfl_xor(m, 32, 64), top = fmaxf(m, other);
     l *= __builtin_amdgcn_exp2f(m - top);
     l += __shfl_xor(l, 32, 64);
@@ -130,11 +140,13 @@ constexpr int kTmOut = 2 * kTmWaves;  // out heads of a workgroup, two per wave
 // HW: heads per wave, 2 or 4.  NG: kv heads of the out heads, whose values are staged by the whole workgroup (0: each wave
 // stages its own).  With two heads per wave the keys of up to NG kv heads are staged as well.
 template <int D, int HW, int NG> struct TmTile {
-    static constexpr int heads = kTmWaves * HW, pitch = D + 8;
+    static constexpr int heads = kTmWaves * HW, kPitch = D + 8, vPitch = NG ? D + 16 : D + 8;
     static constexpr bool keys = NG > 0 && HW == 2;
     static constexpr int pair = 4 * heads;  // bytes of a (key, row) pair: both terms of all heads
-    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = kTmOut * kTmRows * kTmKeys * 2, tileBytes = kTmKeys * pitch * 2;
-    static constexpr int vBytes = (NG ? NG : kTmWaves) * tileBytes, kBytes = keys ? NG * tileBytes : 0;
+    static constexpr int pBytes = kTmKeys * kTmRows * pair, wBytes = kTmOut * kTmRows * kTmKeys * 2, kTile = kTmKeys * kPitch, vTile = kTmKeys * vPitch + (NG ? 3 * 64 : 0);
+    // (a transposing read takes four rows of four sets eight apart)
+    static constexpr __device__ int vRow(int row) { return row * vPitch + (NG ? row / 8 * 64 : 0); }
+    static constexpr int vBytes = (NG ? NG : kTmWaves) * vTile * 2, kBytes = keys ? NG * kTile * 2 : 0;
     static constexpr int biasFloats = HW * 48;
     static constexpr size_t bytes = (size_t)pBytes + wBytes + vBytes + kBytes + kTmWaves * biasFloats * 4;
 };
@@ -172,7 +184,8 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
             float x[2];
 #pragma unroll
             for (int e = 0; e < 2; ++e) {
-                const int out = out0 + l16, in = (8 * g + 2 * j + e) % HP;
+                const int turned = HW == 4 ? j ^ (2 * (wave & 1)) : j ^ (wave & 3);  // (as the weights of this wave's keys lie)
+                const int out = out0 + l16, in = (8 * g + 2 * turned + e) % HP;
                 x[e] = out < a.heads && in < a.heads ? a.talk[(int64_t)out * a.heads + in] : 0.f;
             }
             la_split2(x[0], x[1], sp.hi[j], sp.lo[j]);
@@ -185,6 +198,7 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
     }
     bf8 q[HW][KS];
     float lse[HW], size[HW], rate[HW];
+    f4 start[HW];  // two heads per wave: the products start from -lse
     {
         const int64_t mem_row = p.row0 + min(row, p.n - 1);
 #pragma unroll
@@ -196,6 +210,8 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
             lse[i] = row < p.n && head0 + i < a.heads ? a.lse[mem_row * a.heads + h] : -kScoredNone;  // (no head, no row: no weight)
             size[i] = a.size ? a.size[h] : 0.f;
             rate[i] = a.rate ? a.rate[h] : 0.f;
+            const float from = HW == 2 ? -lse[i] / plain : 0.f;
+            start[i] = f4{from, from, from, from};
         }
     }
     f4 o[2][ET];
@@ -209,7 +225,7 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
     const int vreal = (a.vdim + 7) / 8 * 8;
     // the kv heads that are staged: from the first of the out heads, from the first of all
     const int v_kv0 = kv_of(out0);
-    __bf16 *v_s = v_all + (SAME ? kv_of(own0) - v_kv0 : wave) * (L::tileBytes / 2);
+    __bf16 *v_s = v_all + (SAME ? kv_of(own0) - v_kv0 : wave) * L::vTile;
     // Block and pool row of the key that this thread stages (values staged by all: the piece of a tile; else key lane % 32); past
     // the last key: the last one's, which nothing weighs.
     const int my_row = SAME ? tid % kTile / kPer : lane & 31;
@@ -226,10 +242,9 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
             to[n] = FULL ? *reinterpret_cast<const scored_u4 *>(at) : scored_load16(at, tid % kPer * 8 < real);
         }
     };
-    auto stage_to = [&](__bf16 *tiles, const scored_u4 *from) {
+    auto stage_to = [&](__bf16 *tiles, int tile, int row_at, const scored_u4 *from) {
 #pragma unroll
-        for (int n = 0; n < NV; ++n)
-            *reinterpret_cast<scored_u4 *>(tiles + (tid + kTmThreads * n) / kTile * (L::tileBytes / 2) + my_row * L::pitch + tid % kPer * 8) = from[n];
+        for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(tiles + (tid + kTmThreads * n) / kTile * tile + row_at + tid % kPer * 8) = from[n];
     };
     // straight to operands: keys 16 kb + l16 of one kv head (slots: of key lane % 32)
     auto direct_k = [&](int kv, int slots) {
@@ -261,10 +276,10 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
     };
     auto put_v = [&]() {
         if constexpr (SAME) {
-            stage_to(v_all, vr);
+            stage_to(v_all, L::vTile, L::vRow(my_row), vr);
         } else {
 #pragma unroll
-            for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + (64 * n + lane) / kPer * L::pitch + lane % kPer * 8) = vr[n];
+            for (int n = 0; n < NV; ++n) *reinterpret_cast<scored_u4 *>(v_s + L::vRow((64 * n + lane) / kPer) + lane % kPer * 8) = vr[n];
         }
     };
     // keys by key lane % 32, where they go straight to operands beside values staged by all
@@ -272,7 +287,8 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
     auto near_slot = [&](int id, int k0, int slots) {
         return SAME && !L::keys ? max(talk_slot_of(a, id, min(k0 + (lane & 31), end - 1), end), 0) : slots;
     };
-    // 16-byte pieces of a pair's row and of a (head, row)'s keys at places that spread over the banks
+    // 16-byte pieces of a pair's row and of a (head, row)'s keys at places that spread over the banks; inside a piece the place
+    // of a wave's weights also turns with key / 4, and that of its keys with head / 4
     auto pair_at = [&](int key, int piece) {
         const int at = HP == 32 ? piece ^ ((l16 >> 1) & 7) : piece ^ ((l16 >> 2) & 3);
         return tm_lds + (key * kTmRows + l16) * L::pair + 16 * at;
@@ -283,7 +299,7 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
     fetch_k(slots, near_slot(near_id(0), 0, slots));
     fetch_v(slots);
     if constexpr (L::keys) {
-        stage_to(k_s, kr);
+        stage_to(k_s, L::kTile, my_row * L::kPitch, kr);
         __syncthreads();
     }
     for (int k0 = 0; k0 < end; k0 += kTmKeys) {
@@ -298,7 +314,7 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
         auto weights = [&](int i, int kb, f4 s, float *w) {
             const float *bp = biases + i * 48 + l16 + 31 - 16 * kb - 4 * g;
 #pragma unroll
-            for (int j = 0; j < 4; ++j) w[j] = __builtin_amdgcn_exp2f(fmaf(s[j], plain, bp[-j]) - lse[i]);
+            for (int j = 0; j < 4; ++j) w[j] = __builtin_amdgcn_exp2f(fmaf(s[j], plain, bp[-j]) - (HW == 2 ? 0.f : lse[i]));
         };
         auto put = [&](int kb, float (*w)[4]) {
 #pragma unroll
@@ -308,13 +324,13 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
                     uint2 hi, lo;
                     la_split2(w[0][j], w[1][j], hi.x, lo.x);
                     la_split2(w[2][j], w[3][j], hi.y, lo.y);
-                    *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * (wave & 1)) = hi;
-                    *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * (wave & 1)) = lo;
+                    *reinterpret_cast<uint2 *>(pair_at(key, wave >> 1) + 8 * ((wave ^ g) & 1)) = hi;
+                    *reinterpret_cast<uint2 *>(pair_at(key, 4 + (wave >> 1)) + 8 * ((wave ^ g) & 1)) = lo;
                 } else {
                     uint32_t hi, lo;
                     la_split2(w[0][j], w[1][j], hi, lo);
-                    *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * (wave & 3)) = hi;
-                    *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * (wave & 3)) = lo;
+                    *reinterpret_cast<uint32_t *>(pair_at(key, wave >> 2) + 4 * ((wave & 3) ^ g)) = hi;
+                    *reinterpret_cast<uint32_t *>(pair_at(key, 2 + (wave >> 2)) + 4 * ((wave & 3) ^ g)) = lo;
                 }
             }
         };
@@ -324,11 +340,11 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
                 float w[HW][4];
                 f4 s[HW];
 #pragma unroll
-                for (int i = 0; i < HW; ++i) s[i] = f4{0.f, 0.f, 0.f, 0.f};
+                for (int i = 0; i < HW; ++i) s[i] = start[i];
 #pragma unroll
                 for (int k = 0; k < KS; ++k) {
                     bf8 key;
-                    if constexpr (L::keys) key = la_read8(k_s + kv_of(head0) * (L::tileBytes / 2) + (16 * kb + l16) * L::pitch + 32 * k + 8 * g);
+                    if constexpr (L::keys) key = la_read8(k_s + kv_of(head0) * L::kTile + (16 * kb + l16) * L::kPitch + 32 * k + 8 * g);
                     else key = __builtin_bit_cast(bf8, kr[kb * KS + k]);
 #pragma unroll
                     for (int i = 0; i < HW; ++i) s[i] = la_mfma(key, q[i][k], s[i]);
@@ -346,7 +362,7 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
                 if (kv_of(head0 + i) != kv) direct_k(kv = kv_of(head0 + i), slots);
 #pragma unroll
                 for (int kb = 0; kb < 2; ++kb) {
-                    f4 s = f4{0.f, 0.f, 0.f, 0.f};
+                    f4 s = start[i];
 #pragma unroll
                     for (int k = 0; k < KS; ++k) s = la_mfma(__builtin_bit_cast(bf8, kr[kb * KS + k]), q[i][k], s);
                     weights(i, kb, s, w[kb][i]);
@@ -384,11 +400,11 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
             }
 #pragma unroll
             for (int i = 0; i < 4; ++i)
-                *reinterpret_cast<uint2 *>(weights_at(4 * g + i, wave >> 1) + 8 * (wave & 1)) =
+                *reinterpret_cast<uint2 *>(weights_at(4 * g + i, wave >> 1) + 8 * ((wave ^ g) & 1)) =
                     make_uint2(row_pack_bf16(x[0][i], x[1][i]), row_pack_bf16(x[2][i], x[3][i]));
         }
         put_v();
-        if constexpr (L::keys) stage_to(k_s, kr);
+        if constexpr (L::keys) stage_to(k_s, L::kTile, my_row * L::kPitch, kr);
         fetch_v(slots);
         __builtin_amdgcn_sched_barrier(0);
         __syncthreads();
@@ -396,9 +412,10 @@ template <int D, int HW, bool FULL, int NG> __global__ __launch_bounds__(kTmThre
         bf8 x[2];
 #pragma unroll
         for (int i = 0; i < 2; ++i) x[i] = la_read8(reinterpret_cast<const __bf16 *>(weights_at(2 * wave + i, g)));
+        const int turn = (wave >> 1 & 1) * 4 * L::vPitch;  // (which four keys come first)
         auto values = [&](int t) {
-            const __bf16 *va = v_s + (8 * g + (l16 >> 2)) * L::pitch + 16 * t + 4 * (l16 & 3);
-            return la_join(la_read_tr(va), la_read_tr(va + 4 * L::pitch));
+            const __bf16 *va = v_s + L::vRow(8 * g + (l16 >> 2)) + 16 * t + 4 * (l16 & 3);
+            return la_join(la_read_tr(va + turn), la_read_tr(va + 4 * L::vPitch - turn));
         };
         if (SAME || kv_of(own0 + 1) == kv_of(own0)) {
 #pragma unroll
@@ -463,7 +480,7 @@ bool pa_talking_prefill_launch(const TalkArgs &a, int dtype, hipStream_t s, int 
     const int most = a.n1 > a.vdim ? a.n1 : a.vdim;
     const uintptr_t at = (uintptr_t)a.q1 | (uintptr_t)a.k | (uintptr_t)a.v | (uintptr_t)a.out;
     if (dtype != PA_BF16 || !a.q_lens || most > 128 || a.heads > 32 || (at & 15u) != 0 || a.n1 % 8 != 0 || a.k_dim % 8 != 0 ||
-        a.v_dim % 8 != 0 || a.q1_row % 8 != 0 || a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff || a.bt_stride == 0)
+        a.v_dim % 8 != 0 || a.q1_row % 8 != 0 || a.q1_head % 8 != 0 || a.num_blocks * a.bs >= 0x7fffffff || a.bt_stride == 0 || !(a.scale > 0.f))
         return false;
     rc = [&]() -> int {
         const int groups = ((a.max_q_len + 31) / 32 * a.n_rep + 3) / 4;
