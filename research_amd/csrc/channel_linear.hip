@@ -149,7 +149,9 @@ template <int KD, int NW, bool STATES> struct ClTile {
 
 // Scores of one block token by token, a wave: a lane follows its channels' k_s f_(s+1) .. f_t for all s in `follow` (16 rows
 // of KD floats, the block's part of the K / P tiles: rows 0 .. 7 and 8 .. 15 apart).  Returns scores s = 4 g + i of row l16.
-template <int KD> __device__ __noinline__ f4 cl_slow_scores(const ClArgs &a, const uint16_t *uq, const uint16_t *uz, int h, int n_rows, float *lo8, float *hi8) {
+// (Out of line, and its arguments one by one: it is rarely called, and must not put the kernel's into memory.)
+template <int KD> __device__ __noinline__ f4 cl_slow_scores(const uint16_t *uq, int64_t ldq, const uint16_t *uz, int64_t ldz, const float *bias,
+                                                            const float *lower, int dim, int silu, int n_rows, float *lo8, float *hi8) {
     const int lane = threadIdx.x & 63, l16 = lane & 15, g = lane >> 4;
     f4 out = f4{0.f, 0.f, 0.f, 0.f};
     auto at = [&](int s) { return (s < 8 ? lo8 : hi8) + (s & 7) * KD; };
@@ -157,11 +159,10 @@ template <int KD> __device__ __noinline__ f4 cl_slow_scores(const ClArgs &a, con
         float part[kClBlock];
 #pragma unroll
         for (int s = 0; s < kClBlock; ++s) part[s] = 0.f;
-        for (int d = lane; d < a.dim; d += 64) {
-            const int c = h * a.dim + d;
-            float q = pa_scalar<pa_bf16>::load(reinterpret_cast<const pa_bf16 *>(uq) + t * a.ldq + d), f, k;
-            if (a.silu) q = row_silu<pa_bf16>(q);
-            cl_gate<pa_bf16>(pa_scalar<pa_bf16>::load(reinterpret_cast<const pa_bf16 *>(uz) + t * a.ldz + d) + (a.bias ? a.bias[c] : 0.f), a.lower[c], f, k);
+        for (int d = lane; d < dim; d += 64) {
+            float q = pa_scalar<pa_bf16>::load(reinterpret_cast<const pa_bf16 *>(uq) + t * ldq + d), f, k;
+            if (silu) q = row_silu<pa_bf16>(q);
+            cl_gate<pa_bf16>(pa_scalar<pa_bf16>::load(reinterpret_cast<const pa_bf16 *>(uz) + t * ldz + d) + (bias ? bias[d] : 0.f), lower[d], f, k);
 #pragma unroll
             for (int s = 0; s < kClBlock; ++s) {
                 if (s > t) continue;
@@ -368,7 +369,8 @@ __global__ __launch_bounds__(64 * NW, 1) void channel_chunk_kernel(const ClArgs 
                     }
                 } else {
                     const int n = nv - first;
-                    sc = cl_slow_scores<KD>(a, uq + (r0 + first) * a.ldq, uz + (r0 + first) * a.ldz, h, n < 0 ? 0 : n > kClBlock ? kClBlock : n,
+                    sc = cl_slow_scores<KD>(uq + (r0 + first) * a.ldq, a.ldq, uz + (r0 + first) * a.ldz, a.ldz, a.bias ? a.bias + h * a.dim : nullptr,
+                                            a.lower + h * a.dim, a.dim, a.silu, n < 0 ? 0 : n > kClBlock ? kClBlock : n,
                                             reinterpret_cast<float *>(i_hi + first * kPitch), reinterpret_cast<float *>(i_lo + first * kPitch));
                 }
 #pragma unroll
