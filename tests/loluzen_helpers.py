@@ -40,13 +40,13 @@ def config(width, vocab, layers, loop=None, mult=1.0, embed=1.0, eps=1e-5):
 # name -> config; sizes that differ from each other everywhere, including ones that are not multiples of 8
 CONFIGS = {
     "llz-plain": config(96, 101, [parallel((4, 2, 32, 24), (3, 16, 40), 56), attention(4, 2, 24, 40, 3, rot(500.0, 16, 3.0)),
-                                  parallel((4, 2, 32, 24), (3, 16, 40), None)], loop=(0, 2, 3), mult=0.6, embed=5.0),
+                                  parallel((4, 2, 32, 24), (3, 16, 40), None)], loop=(0, 2, 3), mult=1.2, embed=0.6),
     "llz-odd": config(76, 131, [attention(3, 1, 20, 36, 1, None, 52), parallel((6, 3, 20, 28), (5, 18, 22), 44),
                                 attention(5, 5, 26, 10, 5, rot(40.0, 10, 8.0, 0.5, 2.0, 30), None), parallel((5, 1, 13, 44), (2, 44, 12), 30)],
                       loop=(3, 4, 2), mult=1.3, embed=0.5, eps=1e-3),
     "llz-wide": config(128, 64, [parallel((20, 4, 72, 136), (2, 136, 144), 72), attention(2, 1, 136, 72, 2, rot(1000.0, 136))], mult=0.9),
     "llz-heads": config(64, 50, [parallel((24, 8, 64, 32), (4, 64, 64), 48), parallel((34, 34, 8, 16), (1, 8, 72), 24), attention(8, 2, 16, 8, 4, rot(90.0, 2))],
-                        loop=(1, 3, 2), mult=0.7, embed=12.0),
+                        loop=(1, 3, 2), mult=0.7, embed=1.5),
 }
 
 

@@ -379,3 +379,43 @@ def test_argument_checks_of_the_latent_scored_delta_and_stream_kernels():
            (dict(dt=_lib.PA_F16), -2, "dtype")])
     assert lib.pa_scored_workspace_bytes(0, 4, 2, 32, 32, 0, 100, 0) == 0
     assert lib.pa_delta_workspace_bytes(2, 3, 64, 64, 65) == 2 * 3 * 2 * (4 * 64 * 64 * 2 + 1024)
+
+
+def test_entry_points_of_mixed_heads_and_channel_gates_check_their_arguments():
+    f32, bf16 = _lib.PA_F32, _lib.PA_BF16
+    rc, msg = _status("pa_bias_act", FAKE, 60, None, FAKE, 4, 64, _lib.PA_ACT_RELU2, f32, None)
+    assert rc == -1 and "x_stride" in msg
+    rc, msg = _status("pa_bias_act", FAKE, 64, None, FAKE, 4, 64, 4, f32, None)
+    assert rc == -1 and "act" in msg
+    assert _status("pa_bias_act", None, 64, None, None, 0, 64, _lib.PA_ACT_NONE, bf16, None)[0] == 0
+    rc, msg = _status("pa_glu", FAKE, 64, FAKE, 64, None, 0, FAKE, 4, 64, _lib.PA_ACT_RELU2, f32, None)
+    assert rc == -1 and "act" in msg
+    rc, msg = _status("pa_rms_gate", FAKE, None, 0, FAKE, 1e-6, FAKE, 64, 4, 64, 1, 0, f32, None)
+    assert rc == -1 and "NULL" in msg
+
+    lib = _lib.load()
+    names = ("q", "qr", "qh", "dim", "k", "kd", "v", "vd", "vdim", "bt", "bts", "bs", "nb", "cl", "ql", "qs", "n", "batch", "mq", "h", "hkv", "scale", "size",
+             "rate", "talk", "out", "dt", "ws", "wb", "s")
+    talk = lambda **kw: [{**dict(q=FAKE, qr=128, qh=32, dim=32, k=FAKE, kd=32, v=FAKE, vd=32, vdim=24, bt=FAKE, bts=4, bs=16, nb=8, cl=FAKE, ql=FAKE,
+                                 qs=FAKE, n=4, batch=2, mq=2, h=4, hkv=2, scale=0.1, size=FAKE, rate=FAKE, talk=FAKE, out=FAKE, dt=bf16, ws=FAKE,
+                                 wb=1 << 20, s=None), **kw}[k] for k in names]
+    for kw, status, text in ((dict(hkv=3), -1, "multiple"), (dict(dim=33), -1, "fit the pool"), (dict(vdim=33), -1, "fit the pool"), (dict(ql=None), -1, "together"),
+                             (dict(rate=None), -1, "together"), (dict(bs=0), -1, "block_size"), (dict(dt=_lib.PA_F16), -2, "dtype"),
+                             (dict(dim=264, kd=264), -2, "above 256"), (dict(h=130, hkv=1), -2, "above 128"), (dict(talk=None), -1, "NULL"),
+                             (dict(ws=None), -3, "workspace"), (dict(wb=16), -3, "workspace"), (dict(ql=None, qs=None, batch=5), -1, "below batch")):
+        rc, msg = _status("pa_talking_attention", *talk(**kw))
+        assert rc == status and text in msg, (kw, msg)
+    assert _status("pa_talking_attention", *talk(n=0, q=None))[0] == 0
+    assert lib.pa_talking_workspace_bytes(5, 2, 4, 2, 24, 1000, 0) == 256 and lib.pa_talking_workspace_bytes(5, 2, 0, 2, 24, 1000, 0) == 0
+
+    names = ("q", "lq", "act", "f", "lf", "fb", "lo", "v", "lv", "n", "st", "sr", "cl", "ql", "qs", "ss", "batch", "mq", "out", "h", "dim", "vdim", "dt", "ws",
+             "wb", "s")
+    chan = lambda **kw: [{**dict(q=FAKE, lq=64, act=_lib.PA_ACT_SILU, f=FAKE, lf=64, fb=None, lo=FAKE, v=FAKE, lv=96, n=4, st=FAKE, sr=2, cl=FAKE, ql=FAKE,
+                                 qs=FAKE, ss=FAKE, batch=2, mq=2, out=FAKE, h=4, dim=16, vdim=24, dt=bf16, ws=None, wb=0, s=None), **kw}[k] for k in names]
+    for kw, status, text in ((dict(act=_lib.PA_ACT_GELU_TANH), -1, "q_act"), (dict(lq=63), -1, "stride"), (dict(lf=63), -1, "stride"), (dict(lv=95), -1, "stride"),
+                             (dict(dim=264, lq=2000, lf=2000), -2, "above 256"), (dict(lo=None), -1, "NULL"), (dict(qs=None), -1, "together"),
+                             (dict(ql=None, qs=None, batch=5), -1, "below batch"), (dict(dt=_lib.PA_F16), -2, "dtype"), (dict(vdim=0), -1, "positive")):
+        rc, msg = _status("pa_channel_linear", *chan(**kw))
+        assert rc == status and text in msg, (kw, msg)
+    assert _status("pa_channel_linear", *chan(n=0, q=None))[0] == 0
+    assert lib.pa_channel_linear_workspace_bytes(2, 0, 16, 24, 8) == 0 and "workspace_bytes" in _lib.last_error()
